@@ -6,7 +6,7 @@ compiled once, here, with ``hipcc --offload-arch=gfx950``.
 
 Layout:
   csrc/kernels/*.hip   device code, no torch headers (fast to compile, seconds each)
-  csrc/bindings.cpp    TORCH_LIBRARY registration (torch headers, compiled once)
+  csrc/bindings*.cpp   TORCH_LIBRARY registration (torch headers, compiled once)
   csrc/runtime/*.cpp   native host runtime (paged-KV block manager, scheduler, IO)
 
 Run: ``python -m docqa_amd.ops.build`` (or ``__graft_entry__.build()``).
@@ -73,7 +73,10 @@ def _compile(src: Path, flags: list[str], kind: str) -> Path:
 def build(verbose: bool = True, jobs: int | None = None) -> Path:
     BUILD.mkdir(parents=True, exist_ok=True)
     incs, libdir, abi = _torch_paths()
-    common = ["-O3", "-fPIC", "-std=c++17", f"-I{CSRC / 'include'}", f"-D_GLIBCXX_USE_CXX11_ABI={abi}"]
+    # no packed-fp32 VALU forms (v_pk_*_f32): hipcc makes them from ordinary float code, and some
+    # of them have returned wrong results on this hardware without an error
+    common = ["-O3", "-fPIC", "-std=c++17", f"-I{CSRC / 'include'}", f"-D_GLIBCXX_USE_CXX11_ABI={abi}",
+              "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
     dev_flags = common + [f"--offload-arch={ARCH}", "-munsafe-fp-atomics"]
     host_flags = common + [
         "-x", "hip", f"--offload-arch={ARCH}",
@@ -83,12 +86,13 @@ def build(verbose: bool = True, jobs: int | None = None) -> Path:
     ]
     kernels = sorted((CSRC / "kernels").glob("*.hip"))
     runtime = sorted((CSRC / "runtime").glob("*.cpp"))
+    bindings = sorted(CSRC.glob("bindings*.cpp"))
     jobs = jobs or min(16, os.cpu_count() or 4)
     objs: list[Path] = []
     with cf.ThreadPoolExecutor(max_workers=jobs) as ex:
         futs = [ex.submit(_compile, k, dev_flags, "dev") for k in kernels]
         futs += [ex.submit(_compile, r, host_flags, "rt") for r in runtime]
-        futs.append(ex.submit(_compile, CSRC / "bindings.cpp", host_flags, "bind"))
+        futs += [ex.submit(_compile, b, host_flags, "bind") for b in bindings]
         for f in futs:
             objs.append(f.result())
     link_key = hashlib.sha1("".join(sorted(o.name for o in objs)).encode()).hexdigest()[:16]
