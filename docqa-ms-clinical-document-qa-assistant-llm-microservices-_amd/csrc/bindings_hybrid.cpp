@@ -1,0 +1,297 @@
+// bindings_hybrid.cpp -- torch operators of the hybrid recurrent / windowed-attention decoder
+// kernels (docqa_hybrid.h).  Every shape the kernels index by is checked here against the
+// tensors' sizes before a launch.
+#include <tuple>
+
+#include "docqa_bind.h"
+#include "docqa_hybrid.h"
+
+namespace {
+
+using at::Tensor;
+using OptT = c10::optional<Tensor>;
+
+#define CHECK_F32(t) TORCH_CHECK((t).scalar_type() == at::kFloat, #t " must be float32")
+#define CHECK_ACT(t)                                                                                  \
+  TORCH_CHECK((t).is_cuda() && ((t).scalar_type() == at::kFloat || (t).scalar_type() == at::kBFloat16), \
+              #t " must be a bf16 or fp32 GPU tensor")
+
+bool is_f32(const Tensor& t) { return t.scalar_type() == at::kFloat; }
+
+// P [M, N] (a product) or [S, M, N] (split-K slabs), contiguous
+struct Slabs {
+  int S, M, N;
+  size_t slab;
+};
+Slabs slabs_of(const Tensor& P) {
+  CHECK_ACT(P); CHECK_CONTIG(P);
+  TORCH_CHECK(P.dim() == 2 || P.dim() == 3, "P must be [M, N] or [S, M, N]");
+  const int d = P.dim() - 2;
+  const int S = d ? P.size(0) : 1;
+  TORCH_CHECK(S >= 1, "P needs at least one slab");
+  return {S, (int)P.size(d), (int)P.size(d + 1), (size_t)P.size(d) * P.size(d + 1)};
+}
+void check_vec(const Tensor& t, int64_t n, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.is_contiguous() && t.numel() == n, name,
+              ": fp32 vector of ", n, " expected");
+}
+void check_i32(const Tensor& t, int64_t n, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kInt && t.is_contiguous() && t.numel() >= n, name,
+              ": int32 vector of >= ", n, " expected");
+}
+// a [rows, cols] view whose rows are contiguous
+void check_rows(const Tensor& t, int64_t rows, int64_t cols, const Tensor& like, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == like.scalar_type() && t.dim() == 2 && t.size(0) == rows &&
+                  t.size(1) >= cols && t.stride(1) == 1 && (rows <= 1 || t.stride(0) >= cols),
+              name, ": rows [", rows, ", >= ", cols, "] of the activations' dtype expected");
+}
+
+Tensor sandwich_rmsnorm(const Tensor& P, Tensor residual, const Tensor& w_post, const OptT& add, const Tensor& w_next,
+                        double eps, bool out_f32) {
+  const Slabs p = slabs_of(P);
+  CHECK_GPU(residual); CHECK_F32(residual); CHECK_CONTIG(residual);
+  TORCH_CHECK(residual.dim() == 2 && residual.size(0) == p.M && residual.size(1) == p.N, "residual shape mismatch");
+  check_vec(w_post, p.N, "w_post");
+  check_vec(w_next, p.N, "w_next");
+  const float* ap = nullptr;
+  if (add.has_value()) {
+    check_vec(*add, residual.numel(), "add");
+    ap = add->data_ptr<float>();
+  }
+  c10::DeviceGuard g(P.device());
+  auto out = at::empty({p.M, p.N}, P.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
+  CHECK_ALIGN16(P); CHECK_ALIGN16(residual); CHECK_ALIGN16(w_post); CHECK_ALIGN16(w_next);
+  CHECK_RC(docqa_sandwich_rmsnorm(P.data_ptr(), is_f32(P), p.S, residual.data_ptr<float>(), w_post.data_ptr<float>(),
+                                  ap, w_next.data_ptr<float>(), out.data_ptr(), out_f32, p.M, p.N, (float)eps,
+                                  stream()),
+           "sandwich_rmsnorm");
+  return out;
+}
+
+std::tuple<Tensor, Tensor, Tensor> embed_scale_rmsnorm(const Tensor& ids, const Tensor& table, double scale,
+                                                       const Tensor& w, double eps, bool keep) {
+  CHECK_ACT(table); CHECK_CONTIG(table); CHECK_ALIGN16(table);
+  TORCH_CHECK(table.dim() == 2, "table must be [vocab, width]");
+  const int T = ids.numel(), H = table.size(1);
+  check_i32(ids, T, "ids");
+  check_vec(w, H, "w");
+  CHECK_ALIGN16(w);
+  c10::DeviceGuard g(table.device());
+  auto f32 = table.options().dtype(at::kFloat);
+  auto res = at::empty({T, H}, f32);
+  auto emb = keep ? at::empty({T, H}, f32) : at::empty({0}, f32);
+  auto out = at::empty({T, H}, table.options());
+  CHECK_RC(docqa_embed_scale_rmsnorm(ids.data_ptr<int>(), table.data_ptr(), is_f32(table), (float)scale,
+                                     w.data_ptr<float>(), res.data_ptr<float>(),
+                                     keep ? emb.data_ptr<float>() : nullptr, out.data_ptr(), T, H,
+                                     (int)table.size(0), (float)eps, stream()),
+           "embed_scale_rmsnorm");
+  return {res, emb, out};
+}
+
+Tensor squared_relu(const Tensor& P, bool out_f32) {
+  const Slabs p = slabs_of(P);
+  CHECK_ALIGN16(P);
+  c10::DeviceGuard g(P.device());
+  auto out = at::empty({p.M, p.N}, P.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
+  CHECK_RC(docqa_squared_relu(P.data_ptr(), is_f32(P), p.S, p.slab, out.data_ptr(), out_f32, stream()),
+           "squared_relu");
+  return out;
+}
+
+Tensor qk_norm_store(const Tensor& P, const Tensor& w, const Tensor& slots, Tensor k_cache, Tensor k_scale, int64_t H,
+                     double eps) {
+  const Slabs p = slabs_of(P);
+  CHECK_ACT(k_cache); CHECK_CONTIG(k_cache); CHECK_CONTIG(k_scale); CHECK_F32(k_scale);
+  TORCH_CHECK(k_cache.dim() == 4, "k_cache must be [blocks, kv heads, block, dim]");
+  const int G = k_cache.size(1), BS = k_cache.size(2), D = k_cache.size(3);
+  TORCH_CHECK(p.N >= (H + G) * D, "qk_norm_store: projection width");
+  TORCH_CHECK(k_scale.numel() == k_cache.numel() / D, "k_scale must be [blocks, kv heads, block]");
+  check_vec(w, D, "w");
+  check_i32(slots, p.M, "slots");
+  c10::DeviceGuard g(P.device());
+  CHECK_ALIGN16(P); CHECK_ALIGN16(k_cache); CHECK_ALIGN16(w);
+  auto q = at::empty({p.M, H * D}, k_cache.options());
+  CHECK_RC(docqa_qk_norm_store(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, w.data_ptr<float>(), slots.data_ptr<int>(),
+                               q.data_ptr(), k_cache.data_ptr(), k_scale.data_ptr<float>(), is_f32(k_cache), p.M,
+                               (int)H, G, D, BS, (float)eps, stream()),
+           "qk_norm_store");
+  return q;
+}
+
+// cu: [B + 1] query offsets with ctx the first positions (prefill), or null: one query token a
+// row with ctx the context lengths (decode)
+Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, const OptT& k_scale,
+                   const Tensor& block_tables, const OptT& cu, const Tensor& ctx, int64_t max_q, double scale,
+                   int64_t window, const OptT& sink) {
+  CHECK_ACT(q); CHECK_CONTIG(q); CHECK_CONTIG(k_cache);
+  TORCH_CHECK(k_cache.dim() == 4 && k_cache.scalar_type() == q.scalar_type(), "k_cache dtype / shape");
+  const int G = k_cache.size(1), BS = k_cache.size(2), D = k_cache.size(3);
+  TORCH_CHECK(q.dim() == 2 && q.size(1) % D == 0, "q must be [rows, H * dim]");
+  const int H = q.size(1) / D, B = block_tables.size(0);
+  CHECK_GPU(block_tables); CHECK_I32(block_tables); CHECK_CONTIG(block_tables);
+  TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(1) >= 1, "block_tables must be [B, blocks]");
+  check_i32(ctx, B, "ctx");
+  if (cu.has_value()) check_i32(*cu, B + 1, "cu");
+  else TORCH_CHECK(q.size(0) == B && max_q == 1, "decode: one query row a sequence");
+  TORCH_CHECK(k_cache.numel() / D < (1ll << 31), "cache rows must fit 31 bits");
+  if (v_cache.has_value())
+    TORCH_CHECK(v_cache->sizes() == k_cache.sizes() && v_cache->scalar_type() == q.scalar_type() &&
+                    v_cache->is_contiguous(), "v_cache must match k_cache");
+  if (k_scale.has_value()) check_vec(*k_scale, k_cache.numel() / D, "k_scale");
+  if (sink.has_value()) check_vec(*sink, H, "sink");
+  c10::DeviceGuard g(q.device());
+  CHECK_ALIGN16(q); CHECK_ALIGN16(k_cache);
+  auto out = at::empty_like(q);
+  CHECK_RC(docqa_window_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.has_value() ? v_cache->data_ptr() : k_cache.data_ptr(),
+                             k_scale.has_value() ? k_scale->data_ptr<float>() : nullptr, block_tables.data_ptr<int>(),
+                             (int)block_tables.size(1), cu.has_value() ? cu->data_ptr<int>() : nullptr,
+                             ctx.data_ptr<int>(), sink.has_value() ? sink->data_ptr<float>() : nullptr,
+                             out.data_ptr(), is_f32(q), B, (int)max_q, H, G, D, BS, (float)scale, (int)window,
+                             stream()),
+           "window_attn");
+  return out;
+}
+
+void check_conv(const Tensor& w, const Tensor& bias, const Tensor& state, int C, int& taps) {
+  TORCH_CHECK(w.dim() == 2 && w.size(1) == C, "conv weight must be [taps, channels]");
+  taps = w.size(0);
+  check_vec(w, (int64_t)taps * C, "conv weight");
+  check_vec(bias, C, "conv bias");
+  CHECK_CONTIG(state);
+  TORCH_CHECK(state.dim() == 3 && state.size(1) == taps - 1 && state.size(2) == C, "conv state must be [slots, taps - 1, channels]");
+}
+
+// x: [tokens, >= C] rows (the first C columns are convolved); advances the sequences' state
+Tensor causal_conv(const Tensor& x, const Tensor& w, const Tensor& bias, Tensor state, const Tensor& slots,
+                   const Tensor& cu, const Tensor& ctx, int64_t max_len) {
+  CHECK_ACT(x);
+  const int C = w.size(1), T = x.size(0), B = cu.numel() - 1;
+  int taps;
+  check_conv(w, bias, state, C, taps);
+  check_rows(x, T, C, x, "x");
+  TORCH_CHECK(state.scalar_type() == x.scalar_type(), "conv state dtype");
+  check_i32(slots, B, "slots"); check_i32(cu, B + 1, "cu"); check_i32(ctx, B, "ctx");
+  c10::DeviceGuard g(x.device());
+  auto y = at::empty({T, C}, x.options());
+  CHECK_RC(docqa_causal_conv(x.data_ptr(), (int)x.stride(0), w.data_ptr<float>(), bias.data_ptr<float>(),
+                             state.data_ptr(), slots.data_ptr<int>(), cu.data_ptr<int>(), ctx.data_ptr<int>(),
+                             y.data_ptr(), is_f32(x), B, (int)max_len, C, taps, stream()),
+           "causal_conv");
+  return y;
+}
+
+// P: [x: C | z: C] input projection of one token a row -> (silu(conv x), z)
+std::tuple<Tensor, Tensor> conv_step(const Tensor& P, const Tensor& w, const Tensor& bias, Tensor state,
+                                     const Tensor& slots, const Tensor& positions) {
+  const Slabs p = slabs_of(P);
+  const int C = w.size(1);
+  int taps;
+  check_conv(w, bias, state, C, taps);
+  CHECK_ACT(state);
+  TORCH_CHECK(p.N == 2 * C, "conv_step: P must be [.., 2 C] wide");
+  TORCH_CHECK(is_f32(P) || !is_f32(state), "conv_step: fp32 state needs fp32 projections");
+  check_i32(slots, p.M, "slots"); check_i32(positions, p.M, "positions");
+  c10::DeviceGuard g(P.device());
+  auto y = at::empty({p.M, C}, state.options()), z = at::empty({p.M, C}, state.options());
+  CHECK_RC(docqa_conv_step(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, w.data_ptr<float>(), bias.data_ptr<float>(),
+                           state.data_ptr(), slots.data_ptr<int>(), positions.data_ptr<int>(), y.data_ptr(),
+                           z.data_ptr(), is_f32(state), p.M, C, taps, stream()),
+           "conv_step");
+  return {y, z};
+}
+
+int check_scan(const Tensor& x, const Tensor& dt, const Tensor& bc, const Tensor& z, const Tensor& A2, const Tensor& D,
+               const Tensor& dt_b, const Tensor& state, int64_t N, int64_t b_off, int64_t c_off) {
+  CHECK_ACT(x); CHECK_CONTIG(x); CHECK_CONTIG(dt);
+  TORCH_CHECK(x.dim() == 2, "x must be [tokens, channels]");
+  const int T = x.size(0), C = x.size(1);
+  TORCH_CHECK(dt.sizes() == x.sizes() && dt.scalar_type() == x.scalar_type(), "dt must match x");
+  TORCH_CHECK(A2.dim() == 2 && A2.size(0) == C && A2.size(1) >= N && A2.size(1) % 4 == 0, "A2 must be [channels, N padded to 4]");
+  const int Np = A2.size(1);
+  check_vec(A2, (int64_t)C * Np, "A2");
+  check_vec(D, C, "D"); check_vec(dt_b, C, "dt_b");
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == at::kFloat && state.is_contiguous() && state.dim() == 3 &&
+                  state.size(1) == C && state.size(2) == Np, "scan state must be fp32 [slots, channels, Np]");
+  TORCH_CHECK(b_off >= 0 && c_off >= 0, "B / C offsets");
+  check_rows(bc, T, std::max(b_off, c_off) + N, x, "bc");
+  check_rows(z, T, C, x, "z");
+  CHECK_ALIGN16(A2); CHECK_ALIGN16(state);
+  return Np;
+}
+
+Tensor selective_scan(const Tensor& x, const Tensor& dt, const Tensor& bc, int64_t b_off, int64_t c_off, int64_t N,
+                      const Tensor& z, const Tensor& A2, const Tensor& D, const Tensor& dt_b, Tensor state,
+                      const Tensor& slots, const Tensor& cu, const Tensor& ctx, int64_t max_len, int64_t chunk) {
+  const int Np = check_scan(x, dt, bc, z, A2, D, dt_b, state, N, b_off, c_off);
+  const int B = cu.numel() - 1, C = x.size(1);
+  check_i32(slots, B, "slots"); check_i32(cu, B + 1, "cu"); check_i32(ctx, B, "ctx");
+  TORCH_CHECK(chunk >= 1 && max_len >= 0, "chunk");
+  const int nchunk = (int)((max_len + chunk - 1) / chunk);
+  TORCH_CHECK(nchunk <= 65535 && B <= 65535, "scan grid");
+  c10::DeviceGuard g(x.device());
+  auto y = at::empty_like(x);
+  Tensor cs, sum;
+  if (nchunk > 1) {
+    cs = at::empty({B, nchunk, C, Np}, state.options());
+    sum = at::empty({B, nchunk, C}, state.options());
+  }
+  CHECK_RC(docqa_selective_scan(x.data_ptr(), dt.data_ptr(), bc.data_ptr(), (int)bc.stride(0), (int)b_off, (int)c_off,
+                                z.data_ptr(), (int)z.stride(0), A2.data_ptr<float>(), D.data_ptr<float>(),
+                                dt_b.data_ptr<float>(), state.data_ptr<float>(), slots.data_ptr<int>(),
+                                cu.data_ptr<int>(), ctx.data_ptr<int>(), y.data_ptr(),
+                                nchunk > 1 ? cs.data_ptr<float>() : nullptr, nchunk > 1 ? sum.data_ptr<float>() : nullptr,
+                                is_f32(x), B, C, (int)N, Np, (int)chunk, nchunk, stream()),
+           "selective_scan");
+  return y;
+}
+
+Tensor selective_step(const Tensor& x, const Tensor& dt, const Tensor& bc, int64_t b_off, int64_t c_off, int64_t N,
+                      const Tensor& z, const Tensor& A2, const Tensor& D, const Tensor& dt_b, Tensor state,
+                      const Tensor& slots, const Tensor& positions) {
+  const int Np = check_scan(x, dt, bc, z, A2, D, dt_b, state, N, b_off, c_off);
+  const int B = x.size(0), C = x.size(1);
+  check_i32(slots, B, "slots"); check_i32(positions, B, "positions");
+  c10::DeviceGuard g(x.device());
+  auto y = at::empty_like(x);
+  CHECK_RC(docqa_selective_step(x.data_ptr(), dt.data_ptr(), bc.data_ptr(), (int)bc.stride(0), (int)b_off, (int)c_off,
+                                z.data_ptr(), (int)z.stride(0), A2.data_ptr<float>(), D.data_ptr<float>(),
+                                dt_b.data_ptr<float>(), state.data_ptr<float>(), slots.data_ptr<int>(),
+                                positions.data_ptr<int>(), y.data_ptr(), is_f32(x), B, C, (int)N, Np, stream()),
+           "selective_step");
+  return y;
+}
+
+}  // namespace
+
+TORCH_LIBRARY_FRAGMENT(docqa, m) {
+  m.def("sandwich_rmsnorm(Tensor P, Tensor(a!) residual, Tensor w_post, Tensor? add, Tensor w_next, float eps, "
+        "bool out_f32) -> Tensor");
+  m.def("embed_scale_rmsnorm(Tensor ids, Tensor table, float scale, Tensor w, float eps, bool keep) "
+        "-> (Tensor, Tensor, Tensor)");
+  m.def("squared_relu(Tensor P, bool out_f32) -> Tensor");
+  m.def("qk_norm_store(Tensor P, Tensor w, Tensor slots, Tensor(a!) k_cache, Tensor(b!) k_scale, int H, float eps) "
+        "-> Tensor");
+  m.def("window_attn(Tensor q, Tensor k_cache, Tensor? v_cache, Tensor? k_scale, Tensor block_tables, Tensor? cu, "
+        "Tensor ctx, int max_q, float scale, int window, Tensor? sink) -> Tensor");
+  m.def("causal_conv(Tensor x, Tensor w, Tensor bias, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, "
+        "int max_len) -> Tensor");
+  m.def("conv_step(Tensor P, Tensor w, Tensor bias, Tensor(a!) state, Tensor slots, Tensor positions) "
+        "-> (Tensor, Tensor)");
+  m.def("selective_scan(Tensor x, Tensor dt, Tensor bc, int b_off, int c_off, int N, Tensor z, Tensor A2, Tensor D, "
+        "Tensor dt_b, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, int max_len, int chunk) -> Tensor");
+  m.def("selective_step(Tensor x, Tensor dt, Tensor bc, int b_off, int c_off, int N, Tensor z, Tensor A2, Tensor D, "
+        "Tensor dt_b, Tensor(a!) state, Tensor slots, Tensor positions) -> Tensor");
+}
+
+TORCH_LIBRARY_IMPL(docqa, CUDA, m) {
+  m.impl("sandwich_rmsnorm", &sandwich_rmsnorm);
+  m.impl("embed_scale_rmsnorm", &embed_scale_rmsnorm);
+  m.impl("squared_relu", &squared_relu);
+  m.impl("qk_norm_store", &qk_norm_store);
+  m.impl("window_attn", &window_attn);
+  m.impl("causal_conv", &causal_conv);
+  m.impl("conv_step", &conv_step);
+  m.impl("selective_scan", &selective_scan);
+  m.impl("selective_step", &selective_step);
+}

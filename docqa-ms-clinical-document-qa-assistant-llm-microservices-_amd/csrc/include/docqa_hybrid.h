@@ -1,0 +1,38 @@
+// docqa_hybrid.h -- host launchers of the kernels behind hybrid recurrent / windowed-attention
+// decoders (sandwich_norm.hip, attn_window.hip, ssm.hip, act.hip squared ReLU).  Same rules as
+// docqa_kernels.h: 0 on success, negative for an unsupported shape, else a hipError_t; nothing
+// is allocated and nothing synchronises.  "f32" flags pick fp32 over bf16 storage; P operands
+// are S split-K slabs (S = 1: the product itself).
+#pragma once
+#include <hip/hip_runtime.h>
+#include <stddef.h>
+#include <stdint.h>
+
+int docqa_sandwich_rmsnorm(const void* P, int p_f32, int S, float* res, const float* w_post, const float* add,
+                           const float* w_next, void* out, int out_f32, int rows, int H, float eps, hipStream_t s);
+int docqa_embed_scale_rmsnorm(const int* ids, const void* table, int f32, float scale, const float* w, float* res,
+                              float* emb, void* out, int rows, int H, int vocab, float eps, hipStream_t s);
+int docqa_squared_relu(const void* P, int p_f32, int S, size_t n, void* out, int out_f32, hipStream_t s);
+
+int docqa_qk_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* wq, const int* slots,
+                        void* q, void* kc, float* ks, int f32, int tokens, int H, int G, int D, int BS, float eps,
+                        hipStream_t s);
+// cu null: decode (one query token a row, ctx = context length including it)
+int docqa_window_attn(const void* q, const void* kc, const void* vc, const float* k_scale, const int* block_tables,
+                      int maxb, const int* cu, const int* ctx, const float* sink, void* out, int f32, int B,
+                      int max_q, int H, int G, int D, int BS, float scale, int window, hipStream_t s);
+
+int docqa_causal_conv(const void* x, int ldx, const float* w, const float* b, void* state, const int* slots,
+                      const int* cu, const int* ctx, void* y, int f32, int B, int max_len, int C, int taps,
+                      hipStream_t s);
+int docqa_conv_step(const void* P, int p_f32, int S, size_t slab, int ld, const float* w, const float* b, void* state,
+                    const int* slots, const int* positions, void* y, void* z, int f32, int B, int C, int taps,
+                    hipStream_t s);
+int docqa_selective_scan(const void* x, const void* dt, const void* bc, int ld_bc, int b_off, int c_off,
+                         const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
+                         const int* slots, const int* cu, const int* ctx, void* y, float* cstate, float* csum,
+                         int f32, int B, int C, int N, int Np, int chunk, int nchunk, hipStream_t s);
+int docqa_selective_step(const void* x, const void* dt, const void* bc, int ld_bc, int b_off, int c_off,
+                         const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
+                         const int* slots, const int* positions, void* y, int f32, int B, int C, int N, int Np,
+                         hipStream_t s);

@@ -8,6 +8,7 @@
 // All are 16-byte vectorised and grid-strided (cdna_hip_programming.md Guideline 13,
 // Guideline 11 grid sizing: <= 2048 blocks, grid-stride the rest).
 #include "docqa_common.h"
+#include "docqa_elem.h"
 
 using namespace docqa;
 
@@ -203,4 +204,45 @@ int docqa_bias_act(const void* x, const void* bias, const void* res, void* out, 
   }
   DOCQA_CHECK_LAUNCH();
   return 0;
+}
+
+// squared ReLU of a projection given as S split-K slabs (or its one [n] product), fp32 or
+// bf16 in, fp32 or bf16 out: out = max(sum_s P[s], 0)^2
+template <int V, typename PT, typename OT>
+__global__ __launch_bounds__(256) void squared_relu_kernel(const PT* __restrict__ P, int S, size_t n,
+                                                           OT* __restrict__ out) {
+  const size_t step = (size_t)gridDim.x * 256 * V;
+  for (size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * V; i < n; i += step) {
+    float f[V];
+    ld_slabs<V>(P + i, S, n, f);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      const float r = fmaxf(f[j], 0.f);
+      f[j] = r * r;
+    }
+    stv<V>(out + i, f);
+  }
+}
+
+template <typename PT, typename OT>
+static int launch_squared_relu(const PT* P, int S, size_t n, OT* out, hipStream_t s) {
+  if (n % 8 == 0) {
+    const size_t g = (n / 8 + 255) / 256;
+    squared_relu_kernel<8, PT, OT><<<(int)(g < 4096 ? g : 4096), 256, 0, s>>>(P, S, n, out);
+  } else {
+    const size_t g = (n + 255) / 256;
+    squared_relu_kernel<1, PT, OT><<<(int)(g < 4096 ? g : 4096), 256, 0, s>>>(P, S, n, out);
+  }
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+int docqa_squared_relu(const void* P, int p_f32, int S, size_t n, void* out, int out_f32, hipStream_t s) {
+  if (n == 0) return 0;
+  if (S < 1) return -1;
+  if (p_f32)
+    return out_f32 ? launch_squared_relu((const float*)P, S, n, (float*)out, s)
+                   : launch_squared_relu((const float*)P, S, n, (uint16_t*)out, s);
+  return out_f32 ? launch_squared_relu((const uint16_t*)P, S, n, (float*)out, s)
+                 : launch_squared_relu((const uint16_t*)P, S, n, (uint16_t*)out, s);
 }

@@ -1,0 +1,509 @@
+// ssm.hip -- recurrent mixers: a short causal convolution per channel and the selective scan
+// (Mamba, Gu & Dao 2023), each as a prefill kernel over packed sequences and a decode step.
+//
+//   conv:  y[t, c] = silu(b[c] + sum_k w[k, c] x[t - (taps - 1) + k, c])
+//   scan:  dt = softplus(dt_pre + dt_b);  S[c, n] <- 2^(dt A2[c, n]) S[c, n] + dt x B[n]
+//          y = (sum_n S[c, n] C[n] + D x) silu(z)           A2 = -exp(A_log) log2(e)
+//
+// Per sequence the state pool holds (slot = one live request):
+//   conv state [slots, taps - 1, C]  the last inputs, oldest first, in the compute dtype
+//   scan state [slots, C, Np]        fp32, Np = N rounded up to 4 (padding stays zero)
+// A sequence whose first token is position 0 starts from zero whatever its slot held, so a
+// slot needs no clearing when it changes hands.
+//
+// MI355X mapping of the scan: one lane owns a channel with all its states in registers
+// (LPC lanes a channel when there are more than 32 states), so the recurrence never leaves
+// the lane; B / C of 16 tokens at a time are widened into LDS once a workgroup and broadcast;
+// x, dt and z are loaded 8 tokens ahead.  A long prompt
+// is cut into chunks that run side by side -- chunk states from zero, a carry pass over the
+// chunks, then the scan proper from each chunk's true entry state -- because one sequence's
+// channels alone (8192 = 128 waves) leave most of the 1024 SIMDs idle.
+#include "docqa_common.h"
+#include "docqa_elem.h"
+
+using namespace docqa;
+
+namespace {
+constexpr int TB = 16;   // tokens whose B / C are staged in LDS at a time
+constexpr int UB = 8;    // tokens whose x / dt / z are loaded ahead of their use
+
+// ------------------------------------------------------------------ convolution, prefill
+// thread: V channels x TT consecutive tokens, a window of the last K inputs in registers
+template <typename T, int V, int K>
+__global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ x, int ldx,
+                                                          const float* __restrict__ w, const float* __restrict__ bias,
+                                                          const T* __restrict__ state, const int* __restrict__ slots,
+                                                          const int* __restrict__ cu, const int* __restrict__ ctx,
+                                                          T* __restrict__ y, int C, int taps) {
+  constexpr int TT = 8;
+  const int b = blockIdx.z, q0 = cu[b], L = cu[b + 1] - q0;
+  const int t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * TT;
+  const int c0 = (blockIdx.x * 64 + (threadIdx.x & 63)) * V;
+  if (t0 >= L || c0 >= C) return;
+  const int nt = K > 0 ? K : taps;
+  const bool carry = ctx[b] > 0 && slots[b] >= 0;
+  const T* st = carry ? state + (size_t)slots[b] * (nt - 1) * C + c0 : nullptr;
+  float bv[V];
+  ldv<V>(bias + c0, bv);
+  auto input = [&](int t, float* f) {       // input at token t of this portion (t < 0: carried)
+    if (t >= 0) {
+      ldv<V>(x + (size_t)(q0 + t) * ldx + c0, f);
+    } else if (carry) {
+      ldv<V>(st + (size_t)(nt - 1 + t) * C, f);
+    } else {
+#pragma unroll
+      for (int j = 0; j < V; ++j) f[j] = 0.f;
+    }
+  };
+  if constexpr (K > 0) {
+    float wv[K][V], win[K][V];
+#pragma unroll
+    for (int k = 0; k < K; ++k) ldv<V>(w + (size_t)k * C + c0, wv[k]);
+#pragma unroll
+    for (int k = 0; k < K - 1; ++k) input(t0 - (K - 1) + k, win[k]);
+#pragma unroll
+    for (int i = 0; i < TT; ++i) {
+      if (t0 + i >= L) break;
+      input(t0 + i, win[K - 1]);
+      float o[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        float s = bv[j];
+#pragma unroll
+        for (int k = 0; k < K; ++k) s += wv[k][j] * win[k][j];
+        o[j] = silu_exact(s);
+      }
+      stv<V>(y + (size_t)(q0 + t0 + i) * C + c0, o);
+#pragma unroll
+      for (int k = 0; k < K - 1; ++k)
+#pragma unroll
+        for (int j = 0; j < V; ++j) win[k][j] = win[k + 1][j];
+    }
+  } else {
+    for (int i = 0; i < TT && t0 + i < L; ++i) {
+      float s[V], f[V], wk[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) s[j] = bv[j];
+      for (int k = 0; k < nt; ++k) {
+        input(t0 + i - (nt - 1) + k, f);
+        ldv<V>(w + (size_t)k * C + c0, wk);
+#pragma unroll
+        for (int j = 0; j < V; ++j) s[j] += wk[j] * f[j];
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) s[j] = silu_exact(s[j]);
+      stv<V>(y + (size_t)(q0 + t0 + i) * C + c0, s);
+    }
+  }
+}
+
+// the last taps - 1 inputs of every sequence into its state rows.  Row r takes the input of
+// portion token L - (taps - 1) + r, or old row r + L (> r, so ascending r reads before it
+// writes), or zero ahead of the sequence.
+template <typename T>
+__global__ __launch_bounds__(256) void conv_tail_kernel(const T* __restrict__ x, int ldx, T* __restrict__ state,
+                                                        const int* __restrict__ slots, const int* __restrict__ cu,
+                                                        const int* __restrict__ ctx, int C, int taps) {
+  const int b = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
+  const int q0 = cu[b], L = cu[b + 1] - q0, slot = slots[b];
+  if (c >= C || slot < 0 || L <= 0) return;
+  T* st = state + (size_t)slot * (taps - 1) * C + c;
+  for (int r = 0; r < taps - 1; ++r) {
+    const int t = L - (taps - 1) + r;
+    T v = 0;
+    if (t >= 0) v = x[(size_t)(q0 + t) * ldx + c];
+    else if (ctx[b] > 0) v = st[(size_t)(r + L) * C];
+    st[(size_t)r * C] = v;
+  }
+}
+
+// ------------------------------------------------------------------ convolution, decode
+// one new token a row; P [S, B, ld]: the input projection [x: C | z: C] as split-K slabs (or
+// its product).  Writes silu(conv) and, when z_out, the summed gate; advances the state.
+template <typename PT, typename T, int V, int K>
+__global__ __launch_bounds__(256) void conv_step_kernel(const PT* __restrict__ P, int S, size_t slab, int ld,
+                                                        const float* __restrict__ w, const float* __restrict__ bias,
+                                                        T* __restrict__ state, const int* __restrict__ slots,
+                                                        const int* __restrict__ positions, T* __restrict__ y,
+                                                        T* __restrict__ z_out, int C, int taps) {
+  const int b = blockIdx.y, c0 = (blockIdx.x * 256 + threadIdx.x) * V;
+  const int nt = K > 0 ? K : taps;
+  if (c0 >= (z_out ? 2 * C : C)) return;
+  const PT* p = P + (size_t)b * ld + c0;
+  float xn[V];
+  ld_slabs<V>(p, S, slab, xn);
+  if (c0 >= C) {
+    stv<V>(z_out + (size_t)b * C + (c0 - C), xn);
+    return;
+  }
+  const int slot = slots[b];
+  const bool carry = slot >= 0 && positions[b] > 0;
+  T* st = state + (size_t)max(slot, 0) * (nt - 1) * C + c0;
+  float s[V], wk[V];
+  ldv<V>(bias + c0, s);
+#pragma unroll
+  for (int j = 0; j < V; ++j) xn[j] = rnd((const T*)nullptr, xn[j]);
+  ldv<V>(w + (size_t)(nt - 1) * C + c0, wk);
+#pragma unroll
+  for (int j = 0; j < V; ++j) s[j] += wk[j] * xn[j];
+  if constexpr (K > 0) {
+    float h[K][V];
+#pragma unroll
+    for (int k = 0; k < K - 1; ++k) {
+      if (carry) {
+        ldv<V>(st + (size_t)k * C, h[k]);
+      } else {
+#pragma unroll
+        for (int j = 0; j < V; ++j) h[k][j] = 0.f;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) h[K - 1][j] = xn[j];
+#pragma unroll
+    for (int k = 0; k < K - 1; ++k) {
+      ldv<V>(w + (size_t)k * C + c0, wk);
+#pragma unroll
+      for (int j = 0; j < V; ++j) s[j] += wk[j] * h[k][j];
+      if (slot >= 0) stv<V>(st + (size_t)k * C, h[k + 1]);
+    }
+  } else {
+    for (int k = 0; k < nt - 1; ++k) {
+      float h[V], nx[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) h[j] = 0.f, nx[j] = k == nt - 2 ? xn[j] : 0.f;
+      if (carry) {
+        ldv<V>(st + (size_t)k * C, h);
+        if (k < nt - 2) ldv<V>(st + (size_t)(k + 1) * C, nx);
+      }
+      ldv<V>(w + (size_t)k * C + c0, wk);
+#pragma unroll
+      for (int j = 0; j < V; ++j) s[j] += wk[j] * h[j];
+      if (slot >= 0) stv<V>(st + (size_t)k * C, nx);
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j) s[j] = silu_exact(s[j]);
+  stv<V>(y + (size_t)b * C + c0, s);
+}
+
+// ------------------------------------------------------------------ selective scan, prefill
+struct ScanArgs {
+  const void* x;       // [tokens, C] convolved input
+  const void* dt;      // [tokens, C] step projection ahead of bias and softplus
+  const void* bc;      // [tokens, ld_bc] B at bc_off, C at bc_off + c_off
+  const void* z;       // [tokens, ld_z] gate
+  void* y;             // [tokens, C]
+  int ld_bc, b_off, c_off, ld_z;
+  const float* A2;     // [C, Np]
+  const float* D;      // [C]
+  const float* dt_b;   // [C]
+  float* state;        // [slots, C, Np]
+  const int* slots;
+  const int* cu;
+  const int* ctx;
+  float* cstate;       // [B, nchunk, C, Np] chunk states (chunked prompts)
+  float* csum;         // [B, nchunk, C] sum of dt of each chunk
+  int C, N, Np, chunk, nchunk;
+};
+
+// LOCAL: the chunk's state from zero and its sum of dt (all chunks but a sequence's last).
+// Otherwise the scan proper, entering from the carried state (chunk 0) or the carry pass.
+template <typename T, int NS, int LPC, bool LOCAL>
+__global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs a) {
+  constexpr int NSP = NS * LPC, CB = 256 / LPC;
+  __shared__ __attribute__((aligned(16))) float sbc[2][TB][2 * NSP];
+  const int b = blockIdx.z, ck = blockIdx.y;
+  const int q0 = a.cu[b], L = a.cu[b + 1] - q0;
+  const int t_beg = ck * a.chunk, t_end = min(L, t_beg + a.chunk);
+  if (t_beg >= L || (LOCAL && t_end >= L)) return;
+  const int tid = threadIdx.x;
+  const int c = blockIdx.x * CB + tid / LPC, l = tid % LPC;
+  const bool ok = c < a.C;
+  const int cc = ok ? c : a.C - 1;
+  const int slot = a.slots[b];
+  const T *x = (const T*)a.x + cc, *dt = (const T*)a.dt + cc, *bc = (const T*)a.bc, *z = (const T*)a.z + cc;
+
+  float A[NS], S[NS];
+#pragma unroll
+  for (int i = 0; i < NS; ++i) {
+    const int n = l * NS + i;
+    A[i] = n < a.N ? a.A2[(size_t)cc * a.Np + n] : 0.f;
+    S[i] = 0.f;
+  }
+  if constexpr (!LOCAL) {
+    const float* s0 = nullptr;
+    if (ck > 0) s0 = a.cstate + (((size_t)b * a.nchunk + ck) * a.C + cc) * a.Np;
+    else if (a.ctx[b] > 0 && slot >= 0) s0 = a.state + ((size_t)slot * a.C + cc) * a.Np;
+    if (s0) {
+#pragma unroll
+      for (int i = 0; i < NS; ++i)
+        if (l * NS + i < a.N) S[i] = s0[l * NS + i];
+    }
+  }
+  const float Dc = a.D[cc], db = a.dt_b[cc];
+  float sum = 0.f;
+
+  auto stage = [&](int t0, int buf) {
+    for (int e = tid; e < TB * 2 * NSP; e += 256) {
+      const int t = e / (2 * NSP), j = e % (2 * NSP), n = j < NSP ? j : j - NSP;
+      float v = 0.f;
+      if (t0 + t < t_end && n < a.N)
+        v = ld1(bc + (size_t)(q0 + t0 + t) * a.ld_bc + (j < NSP ? a.b_off : a.c_off) + n);
+      sbc[buf][t][j] = v;
+    }
+  };
+  // x, dt, z of UB tokens from t (clamped: a token past the end is computed with dt = 0, which
+  // leaves the state alone, and stores nothing)
+  float xn[UB], dn[UB], zn[UB];
+  auto fetch = [&](int t0) {
+#pragma unroll
+    for (int i = 0; i < UB; ++i) {
+      const int t = min(t0 + i, t_end - 1);
+      xn[i] = ld1(x + (size_t)(q0 + t) * a.C);
+      dn[i] = ld1(dt + (size_t)(q0 + t) * a.C);
+      if constexpr (!LOCAL) zn[i] = ld1(z + (size_t)(q0 + t) * a.ld_z);
+    }
+  };
+  stage(t_beg, 0);
+  fetch(t_beg);
+  int buf = 0;
+  for (int t0 = t_beg; t0 < t_end; t0 += TB, buf ^= 1) {
+    __syncthreads();
+    if (t0 + TB < t_end) stage(t0 + TB, buf ^ 1);
+#pragma unroll 1
+    for (int u = 0; u < TB; u += UB) {
+      float xv[UB], dv[UB], zv[UB];
+#pragma unroll
+      for (int i = 0; i < UB; ++i) {
+        xv[i] = xn[i];
+        dv[i] = t0 + u + i < t_end ? softplus_f(dn[i] + db) : 0.f;
+        if constexpr (!LOCAL) zv[i] = silu_exact(zn[i]);
+      }
+      fetch(t0 + u + UB);
+#pragma unroll
+      for (int i = 0; i < UB; ++i) {
+        const float d = dv[i], dx = d * xv[i];
+        const float* Bt = &sbc[buf][u + i][l * NS];
+        const float* Ct = &sbc[buf][u + i][NSP + l * NS];
+        float y = 0.f;
+#pragma unroll
+        for (int n = 0; n < NS; ++n) {
+          S[n] = exp2f(d * A[n]) * S[n] + dx * Bt[n];
+          if constexpr (!LOCAL) y += S[n] * Ct[n];
+        }
+        if constexpr (LOCAL) {
+          sum += d;
+        } else {
+#pragma unroll
+          for (int o = 1; o < LPC; o <<= 1) y += __shfl_xor(y, o, 64);
+          if (l == 0 && ok && t0 + u + i < t_end)
+            st1((T*)a.y + (size_t)(q0 + t0 + u + i) * a.C + c, (y + Dc * xv[i]) * zv[i]);
+        }
+      }
+    }
+  }
+  if (!ok) return;
+  if constexpr (LOCAL) {
+    float* o = a.cstate + (((size_t)b * a.nchunk + ck + 1) * a.C + c) * a.Np;   // enters chunk ck + 1
+#pragma unroll
+    for (int i = 0; i < NS; ++i)
+      if (l * NS + i < a.N) o[l * NS + i] = S[i];
+    if (l == 0) a.csum[((size_t)b * a.nchunk + ck + 1) * a.C + c] = sum;
+  } else if (t_end == L && slot >= 0) {
+    float* o = a.state + ((size_t)slot * a.C + c) * a.Np;
+#pragma unroll
+    for (int i = 0; i < NS; ++i)
+      if (l * NS + i < a.N) o[l * NS + i] = S[i];
+  }
+}
+
+// chunk k's entry state: decay over chunk k - 1 times its own entry state, plus the local one
+__global__ __launch_bounds__(256) void scan_carry_kernel(ScanArgs a) {
+  const int b = blockIdx.y, L = a.cu[b + 1] - a.cu[b];
+  const int e = blockIdx.x * 256 + threadIdx.x;
+  const int c = e / a.Np, n = e % a.Np;
+  if (c >= a.C || n >= a.N || L <= a.chunk) return;
+  const float A = a.A2[e];
+  const int slot = a.slots[b];
+  float s = (a.ctx[b] > 0 && slot >= 0) ? a.state[(size_t)slot * a.C * a.Np + e] : 0.f;
+  for (int k = 1; k * a.chunk < L; ++k) {
+    const size_t o = ((size_t)b * a.nchunk + k) * a.C;
+    s = exp2f(A * a.csum[o + c]) * s + a.cstate[o * a.Np + e];
+    a.cstate[o * a.Np + e] = s;
+  }
+}
+
+// ------------------------------------------------------------------ selective scan, decode
+// one token a row: a lane holds 4 states of a channel (16-byte state accesses), RB rows a
+// workgroup so that A is read once for all of them
+template <typename T, int RB>
+__global__ __launch_bounds__(256) void selective_step_kernel(ScanArgs a, const int* __restrict__ positions, int B,
+                                                             int lq) {
+  const int tid = threadIdx.x;
+  const int c = blockIdx.x * (256 / lq) + tid / lq, g = tid % lq, n0 = g * 4;
+  const bool okc = c < a.C, ok = okc && n0 < a.Np;
+  const int cc = okc ? c : a.C - 1;
+  float4 A = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (ok) A = *reinterpret_cast<const float4*>(a.A2 + (size_t)c * a.Np + n0);
+  const float Dc = a.D[cc], db = a.dt_b[cc];
+  const int r0 = blockIdx.y * RB;
+  float4 S[RB];
+  int slot[RB];
+#pragma unroll
+  for (int i = 0; i < RB; ++i) {
+    const int r = min(r0 + i, B - 1);
+    slot[i] = a.slots[r];
+    S[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (ok && slot[i] >= 0 && positions[r] > 0)
+      S[i] = *reinterpret_cast<const float4*>(a.state + ((size_t)slot[i] * a.C + c) * a.Np + n0);
+  }
+#pragma unroll
+  for (int i = 0; i < RB; ++i) {
+    const int r = r0 + i;
+    if (r >= B) break;
+    const float x = ld1((const T*)a.x + (size_t)r * a.C + cc);
+    const float d = softplus_f(ld1((const T*)a.dt + (size_t)r * a.C + cc) + db), dx = d * x;
+    const T* bc = (const T*)a.bc + (size_t)r * a.ld_bc;
+    float bv[4], cv[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      bv[j] = n0 + j < a.N ? ld1(bc + a.b_off + n0 + j) : 0.f;
+      cv[j] = n0 + j < a.N ? ld1(bc + a.c_off + n0 + j) : 0.f;
+    }
+    float4 s = S[i];
+    s.x = exp2f(d * A.x) * s.x + dx * bv[0];
+    s.y = exp2f(d * A.y) * s.y + dx * bv[1];
+    s.z = exp2f(d * A.z) * s.z + dx * bv[2];
+    s.w = exp2f(d * A.w) * s.w + dx * bv[3];
+    float y = (s.x * cv[0] + s.y * cv[1]) + (s.z * cv[2] + s.w * cv[3]);
+    for (int o = 1; o < lq; o <<= 1) y += __shfl_xor(y, o, 64);
+    if (ok && slot[i] >= 0) *reinterpret_cast<float4*>(a.state + ((size_t)slot[i] * a.C + c) * a.Np + n0) = s;
+    if (okc && g == 0)
+      st1((T*)a.y + (size_t)r * a.C + c, (y + Dc * x) * silu_exact(ld1((const T*)a.z + (size_t)r * a.ld_z + c)));
+  }
+}
+
+template <typename T, int V>
+int launch_conv(const void* x, int ldx, const float* w, const float* b, void* state, const int* slots, const int* cu,
+                const int* ctx, void* y, int B, int max_len, int C, int taps, hipStream_t s) {
+  dim3 grid((C + 64 * V - 1) / (64 * V), (max_len + 31) / 32, B);
+#define GO(K) causal_conv_kernel<T, V, K><<<grid, 256, 0, s>>>((const T*)x, ldx, w, b, (const T*)state, slots, cu, ctx, (T*)y, C, taps)
+  switch (taps) {
+    case 2: GO(2); break;
+    case 3: GO(3); break;
+    case 4: GO(4); break;
+    default: GO(0); break;
+  }
+#undef GO
+  DOCQA_CHECK_LAUNCH();
+  if (taps > 1) {
+    conv_tail_kernel<T><<<dim3((C + 255) / 256, B), 256, 0, s>>>((const T*)x, ldx, (T*)state, slots, cu, ctx, C, taps);
+    DOCQA_CHECK_LAUNCH();
+  }
+  return 0;
+}
+
+template <typename PT, typename T, int V>
+int launch_conv_step(const void* P, int S, size_t slab, int ld, const float* w, const float* b, void* state,
+                     const int* slots, const int* pos, void* y, void* z, int B, int C, int taps, hipStream_t s) {
+  const int n = (z ? 2 * C : C) / V;
+  dim3 grid((n + 255) / 256, B);
+#define GO(K) conv_step_kernel<PT, T, V, K><<<grid, 256, 0, s>>>((const PT*)P, S, slab, ld, w, b, (T*)state, slots, pos, (T*)y, (T*)z, C, taps)
+  switch (taps) {
+    case 2: GO(2); break;
+    case 3: GO(3); break;
+    case 4: GO(4); break;
+    default: GO(0); break;
+  }
+#undef GO
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+template <typename T, int NS, int LPC>
+int launch_scan(const ScanArgs& a, int B, hipStream_t s) {
+  dim3 grid((a.C + 256 / LPC - 1) / (256 / LPC), a.nchunk, B);
+  if (a.nchunk > 1) {
+    selective_scan_kernel<T, NS, LPC, true><<<grid, 256, 0, s>>>(a);
+    DOCQA_CHECK_LAUNCH();
+    scan_carry_kernel<<<dim3((a.C * a.Np + 255) / 256, B), 256, 0, s>>>(a);
+    DOCQA_CHECK_LAUNCH();
+  }
+  selective_scan_kernel<T, NS, LPC, false><<<grid, 256, 0, s>>>(a);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+template <typename T>
+int dispatch_scan(const ScanArgs& a, int B, hipStream_t s) {
+  if (a.N <= 8) return launch_scan<T, 8, 1>(a, B, s);
+  if (a.N <= 16) return launch_scan<T, 16, 1>(a, B, s);
+  if (a.N <= 24) return launch_scan<T, 24, 1>(a, B, s);
+  if (a.N <= 32) return launch_scan<T, 32, 1>(a, B, s);
+  if (a.N <= 64) return launch_scan<T, 32, 2>(a, B, s);
+  if (a.N <= 128) return launch_scan<T, 32, 4>(a, B, s);
+  if (a.N <= 256) return launch_scan<T, 32, 8>(a, B, s);
+  return -1;
+}
+}  // namespace
+
+int docqa_causal_conv(const void* x, int ldx, const float* w, const float* b, void* state, const int* slots,
+                      const int* cu, const int* ctx, void* y, int f32, int B, int max_len, int C, int taps,
+                      hipStream_t s) {
+  if (B == 0 || max_len == 0) return 0;
+  if (taps < 1 || C < 1 || ldx < C) return -1;
+  const bool vec = C % 8 == 0 && ldx % 8 == 0 && docqa_aligned16(x) && docqa_aligned16(state) && docqa_aligned16(y);
+  if (f32)
+    return vec ? launch_conv<float, 4>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, s)
+               : launch_conv<float, 1>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, s);
+  return vec ? launch_conv<uint16_t, 8>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, s)
+             : launch_conv<uint16_t, 1>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, s);
+}
+
+int docqa_conv_step(const void* P, int p_f32, int S, size_t slab, int ld, const float* w, const float* b, void* state,
+                    const int* slots, const int* positions, void* y, void* z, int f32, int B, int C, int taps,
+                    hipStream_t s) {
+  if (B == 0) return 0;
+  if (taps < 1 || C < 1 || S < 1 || ld < (z ? 2 * C : C) || (f32 && !p_f32)) return -1;
+  const bool vec = C % 4 == 0 && ld % 4 == 0 && docqa_aligned16(P) && docqa_aligned16(state) && docqa_aligned16(y);
+#define ARGS P, S, slab, ld, w, b, state, slots, positions, y, z, B, C, taps, s
+  if (f32) return vec ? launch_conv_step<float, float, 4>(ARGS) : launch_conv_step<float, float, 1>(ARGS);
+  if (p_f32) return vec ? launch_conv_step<float, uint16_t, 4>(ARGS) : launch_conv_step<float, uint16_t, 1>(ARGS);
+  return vec ? launch_conv_step<uint16_t, uint16_t, 4>(ARGS) : launch_conv_step<uint16_t, uint16_t, 1>(ARGS);
+#undef ARGS
+}
+
+int docqa_selective_scan(const void* x, const void* dt, const void* bc, int ld_bc, int b_off, int c_off,
+                         const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
+                         const int* slots, const int* cu, const int* ctx, void* y, float* cstate, float* csum,
+                         int f32, int B, int C, int N, int Np, int chunk, int nchunk, hipStream_t s) {
+  if (B == 0 || nchunk == 0) return 0;
+  if (N < 1 || Np < N || Np % 4 || chunk < 1 || (nchunk > 1 && (!cstate || !csum))) return -1;
+  const ScanArgs a{x, dt, bc, z, y, ld_bc, b_off, c_off, ld_z, A2, D, dt_b, state, slots, cu, ctx, cstate, csum,
+                   C, N, Np, chunk, nchunk};
+  return f32 ? dispatch_scan<float>(a, B, s) : dispatch_scan<uint16_t>(a, B, s);
+}
+
+int docqa_selective_step(const void* x, const void* dt, const void* bc, int ld_bc, int b_off, int c_off,
+                         const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
+                         const int* slots, const int* positions, void* y, int f32, int B, int C, int N, int Np,
+                         hipStream_t s) {
+  if (B == 0) return 0;
+  if (N < 1 || Np < N || Np % 4 || Np > 256) return -1;
+  const ScanArgs a{x, dt, bc, z, y, ld_bc, b_off, c_off, ld_z, A2, D, dt_b, state, slots, nullptr, nullptr, nullptr,
+                   nullptr, C, N, Np, 0, 0};
+  int lq = 1;
+  while (lq * 4 < Np) lq *= 2;
+  const int gx = (C + 256 / lq - 1) / (256 / lq);
+#define GO(T, R) selective_step_kernel<T, R><<<dim3(gx, (B + R - 1) / R), 256, 0, s>>>(a, positions, B, lq)
+  if (f32) {
+    if (B >= 8) GO(float, 4);
+    else GO(float, 1);
+  } else {
+    if (B >= 8) GO(uint16_t, 4);
+    else GO(uint16_t, 1);
+  }
+#undef GO
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}

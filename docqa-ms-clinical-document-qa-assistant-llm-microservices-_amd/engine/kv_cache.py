@@ -8,10 +8,37 @@ whole 256-B rows.
 Block bookkeeping is done by the native allocator in ``csrc/runtime/block_manager.cpp``
 when the extension is loaded (O(1) alloc/free, refcounts for shared prompt prefixes)
 and by the pure-Python :class:`PyBlockAllocator` otherwise.
+
+A layer may instead keep one tensor that serves as K and V (:class:`KVSpec` ``shared``), and
+recurrent layers keep per-request state in slots (:class:`StatePool`).
 """
 from __future__ import annotations
 
+import threading
+from dataclasses import dataclass
+
 import torch
+
+
+@dataclass(frozen=True)
+class KVSpec:
+    """One layer's paged cache.  ``shared``: the key rows are the values too -- one tensor,
+    with an fp32 scale per row in place of V (ops.qk_norm_store)."""
+    kv_heads: int
+    head_dim: int
+    shared: bool = False
+
+    def bytes_per_token(self, dtype_bytes: int) -> int:
+        row = self.head_dim * dtype_bytes
+        return self.kv_heads * (row + 4 if self.shared else 2 * row)
+
+
+@dataclass(frozen=True)
+class StateSpec:
+    """One layer's recurrent state: the per-slot shapes of its tensors, each in the compute
+    dtype or, where ``fp32`` says so, in fp32."""
+    shapes: tuple
+    fp32: tuple
 
 
 class PyBlockAllocator:
@@ -60,18 +87,23 @@ def make_allocator(num_blocks: int, block_size: int = 64):
 
 class KVCache:
     def __init__(self, layers: int, num_blocks: int, kv_heads: int, head_dim: int,
-                 block_size: int = 64, device="cuda", dtype=torch.bfloat16):
+                 block_size: int = 64, device="cuda", dtype=torch.bfloat16, specs: list | None = None):
+        """``specs``: a :class:`KVSpec` per layer (default: ``layers`` equal K / V pairs)."""
         if block_size & (block_size - 1):
             raise ValueError("block_size must be a power of two")
         self.block_size = block_size
         self.num_blocks = num_blocks
-        shape = (num_blocks, kv_heads, block_size, head_dim)
+        specs = specs if specs is not None else [KVSpec(kv_heads, head_dim)] * layers
         # zeroed, not empty: the decode kernels stream whole 32-token tiles and mask the
         # positions past a sequence's end with p = 0, but 0 x NaN is NaN -- a never-written
         # slot holding a NaN bit pattern (whatever an earlier tensor of the process left
         # there) would poison the row.  Stale finite K/V of a reused block is harmless.
-        self.caches = [(torch.zeros(shape, device=device, dtype=dtype),
-                        torch.zeros(shape, device=device, dtype=dtype)) for _ in range(layers)]
+        self.caches = []
+        for sp in specs:
+            shape = (num_blocks, sp.kv_heads, block_size, sp.head_dim)
+            k = torch.zeros(shape, device=device, dtype=dtype)
+            self.caches.append((k, torch.zeros(shape[:3], device=device, dtype=torch.float32) if sp.shared
+                                else torch.zeros_like(k)))
         self.allocator = make_allocator(num_blocks, block_size)
 
     @staticmethod
@@ -86,6 +118,35 @@ class KVCache:
 
     def blocks_for(self, tokens: int) -> int:
         return (tokens + self.block_size - 1) // self.block_size
+
+
+class StatePool:
+    """Recurrent state of the live requests: per layer the tensors of its :class:`StateSpec`
+    with a leading slot dimension, and a free list of slots.  A slot is handed on as it is:
+    the kernels start a sequence at position 0 from zero (csrc/kernels/ssm.hip)."""
+
+    def __init__(self, specs: list, slots: int, device="cuda", dtype=torch.bfloat16):
+        self.slots = slots
+        self.states = [tuple(torch.zeros((slots, *sh), device=device, dtype=torch.float32 if f else dtype)
+                             for sh, f in zip(sp.shapes, sp.fp32)) for sp in specs]
+        self._free = list(range(slots - 1, -1, -1))
+        self._lock = threading.Lock()
+
+    def num_free(self) -> int:
+        return len(self._free)
+
+    def alloc(self, n: int = 1) -> list[int]:
+        with self._lock:
+            if n > len(self._free):
+                raise MemoryError(f"state slots exhausted: need {n}, {len(self._free)} free")
+            return [self._free.pop() for _ in range(n)]
+
+    def free(self, slots: list[int]) -> None:
+        with self._lock:
+            for s in slots:
+                if s in self._free:
+                    raise RuntimeError(f"double free of state slot {s}")
+                self._free.append(s)
 
 
 def chain_keys(tokens, block_size: int, nblocks: int) -> list[int]:

@@ -29,8 +29,9 @@ import torch
 from .. import ops
 from ..parallel import comm
 from ..utils import tracing
-from ..models.llama import AttnMeta, LlamaModel
-from .kv_cache import KVCache, TailCache, chain_keys
+from ..models.decoder import Decoder
+from ..models.llama import AttnMeta
+from .kv_cache import KVCache, StatePool, TailCache, chain_keys
 
 _PREFILL_LOG = os.environ.get("DOCQA_PREFILL_LOG") == "1"   # one JSON line per prefill chunk
 _PREFILL_DUMP = os.environ.get("DOCQA_PREFILL_DUMP", "")       # dir: save paged-prefill shapes for replay
@@ -62,6 +63,7 @@ class Reservation:
     n: int
     copies: list = field(default_factory=list)
     keys: list | None = None   # per prompt: chained block keys (kv_cache.chain_keys)
+    slots: list = field(default_factory=list)   # per prompt: its recurrent-state slot
 
 
 @dataclass
@@ -223,6 +225,8 @@ class _DecodeGraph:
         self.context_lens = torch.zeros(bp, dtype=torch.int32, device=dev)
         self.valid = torch.zeros(bp, dtype=torch.int32, device=dev)
         self.block_tables = torch.zeros(bp, eng.max_blocks_per_seq, dtype=torch.int32, device=dev)
+        # recurrent-state slot of each row, -1: a padded row (reads and leaves no state)
+        self.state_slots = torch.full((bp,), -1, dtype=torch.int32, device=dev)
         self.inv_temp = torch.ones(bp, dtype=torch.float32, device=dev)
         self.top_k = torch.zeros(bp, dtype=torch.int32, device=dev)
         self.top_p = torch.ones(bp, dtype=torch.float32, device=dev)
@@ -253,7 +257,7 @@ class _DecodeGraph:
         can change bucket between steps without copying state."""
         g = cls.__new__(cls)
         g.bp = bp
-        for name in ("tokens", "positions", "context_lens", "valid", "block_tables", "inv_temp",
+        for name in ("tokens", "positions", "context_lens", "valid", "block_tables", "state_slots", "inv_temp",
                      "top_k", "top_p", "out"):
             setattr(g, name, getattr(master, name)[:bp])
         g.shared_table, g.shared_len = master.shared_table, master.shared_len
@@ -268,14 +272,16 @@ class _DecodeGraph:
 
 
 class LLMEngine:
-    def __init__(self, model: LlamaModel, max_batch: int = 64, max_context: int = 2048,
+    def __init__(self, model: Decoder, max_batch: int = 64, max_context: int = 2048,
                  block_size: int = 64, num_blocks: int | None = None, use_graphs: bool = True,
                  max_prefill_tokens: int = 65536, prefix_cache: bool = True,
-                 kv_mem_fraction: float | None = None):
+                 kv_mem_fraction: float | None = None, state_slots: int | None = None):
         """``num_blocks``: KV pool size; default ``max_batch`` full-context sequences, or --
         with ``kv_mem_fraction`` (env DOCQA_KV_MEM_FRACTION) on a GPU -- that fraction of the
         HBM still free after the weights, minus the prefill activation headroom (the block
-        prefix cache keeps every block the running batches do not need)."""
+        prefix cache keeps every block the running batches do not need).  ``state_slots``:
+        recurrent-state slots (models that declare state; default two full batches, as
+        pipelined callers reserve the next batch while one runs)."""
         self.model = model
         self.cfg = model.cfg
         self.device = model.device
@@ -296,6 +302,9 @@ class LLMEngine:
                 cap = car.max_elems // model.cfg.hidden // block_size * block_size
                 max_prefill_tokens = max(block_size, min(max_prefill_tokens, cap))
         self.max_prefill_tokens = max_prefill_tokens
+        specs = model.state_specs()
+        self.state = (StatePool(specs, state_slots or 2 * max_batch, self.device, model.dtype)
+                      if specs else None)
         if num_blocks is None:
             num_blocks = max_batch * self.max_blocks_per_seq + 1
             if kv_mem_fraction is None and os.environ.get("DOCQA_KV_MEM_FRACTION"):
@@ -315,19 +324,20 @@ class LLMEngine:
                     raise MemoryError(f"KV pool: {fb} blocks fit in {kv_mem_fraction:.2f} of the free HBM, "
                                       f"one {self.max_context}-token sequence needs {self.max_blocks_per_seq + 1}")
         num_blocks = self._agree_across_tp(model, num_blocks)
-        self.kv = KVCache(self.cfg.layers, num_blocks, model.hkv, self.cfg.head_dim, block_size,
-                          self.device, model.dtype)
+        self.kv = KVCache(0, num_blocks, 0, 0, block_size, self.device, model.dtype, specs=model.kv_specs())
+        self.caches = model.bind_caches(self.kv, self.state)     # forward's per-layer operands
         self.use_graphs = use_graphs and self.device.type == "cuda"
         # TunableOp search for the decode buckets' library GEMMs (only the LM head below the
         # mid-M rows is left on hipBLASLt): off by default -- ~28 s of service start-up for no
         # measurable step time (docs/CONFIG.md)
         self.tune_decode_gemms = os.environ.get("DOCQA_TUNE_DECODE", "0") == "1"
         # reuse KV blocks of shared prompt prefixes (the fixed RAG instruction template)
-        self.prefix_cache = prefix_cache and os.environ.get("DOCQA_PREFIX_CACHE", "1") == "1"
+        # (a model with recurrent state leaves part of a prompt outside its K/V blocks)
+        self.prefix_cache = prefix_cache and model.prefix_reuse and os.environ.get("DOCQA_PREFIX_CACHE", "1") == "1"
         # cascade decode attention (csrc/include/docqa_cascade.h): when every sequence of a
         # batch starts with the same cached prompt-prefix blocks (the RAG instruction
         # template), that prefix is attended once per step for the whole batch
-        self.cascade = os.environ.get("DOCQA_CASCADE", "1") == "1"
+        self.cascade = model.prefix_reuse and os.environ.get("DOCQA_CASCADE", "1") == "1"
         self.cascade_min_tokens = int(os.environ.get("DOCQA_CASCADE_MIN_TOKENS", "128"))
         self.cascade_min_batch = int(os.environ.get("DOCQA_CASCADE_MIN_BATCH", "4"))
         # LPT dispatch of the decode-attention workgroups (mixed context lengths cost ~15 %
@@ -363,20 +373,46 @@ class LLMEngine:
         return num_blocks
 
     def _blocks_from_free_memory(self, model, block_size: int, fraction: float) -> int:
-        cfg = model.cfg
         free, _ = torch.cuda.mem_get_info(self.device)
         el = torch.finfo(model.dtype).bits // 8
-        block_bytes = cfg.layers * 2 * model.hkv * block_size * cfg.head_dim * el
-        # prefill activations at the token budget (hidden-sized buffers, QKV, the gate|up
-        # product / SwiGLU output) twice over, + 6 GB for graph pools, workspaces and the index
-        per_tok = (6 * cfg.hidden + (model.hq + 2 * model.hkv) * cfg.head_dim + 3 * model.inter) * el
+        block_bytes = max(1, block_size * sum(sp.bytes_per_token(el) for sp in model.kv_specs()))
+        # prefill activations at the token budget twice over, + 6 GB for graph pools, workspaces
+        # and the index
+        per_tok = model.activation_elems() * el
         headroom = 2 * self.max_prefill_tokens * per_tok + (6 << 30)
         budget = int(free * fraction) - headroom
         return max(0, budget // block_bytes)
 
     # ------------------------------------------------------------------ prefill
+    def prefill_batch(self, prompts: list[list[int]], tables: list[list[int]], start: list[int],
+                      slots: list[int] | None = None) -> tuple[torch.Tensor, AttnMeta, np.ndarray]:
+        """Packed tokens [start[i], len) of each prompt, their attention metadata and
+        cu_seqlens (host): one prefill forward's inputs.  ``slots``: state slots."""
+        dev = self.device
+        ids, pos, sm, cu = _prefill_inputs(prompts, tables, start, self.block_size)
+
+        def up(a):
+            return torch.as_tensor(a, dtype=torch.int32).to(dev, non_blocking=True)
+
+        meta = AttnMeta(prefill=True, positions=up(pos), slot_mapping=up(sm), cu_seqlens=up(cu),
+                        max_len=max(len(p) - c for p, c in zip(prompts, start)))
+        if any(start) or self.model.paged_prefill:
+            self.page_prefill(meta, tables, start)
+        if self.state is not None:
+            meta.state_slots = up(slots)
+        return up(ids), meta, cu
+
+    def page_prefill(self, meta: AttnMeta, tables: list[list[int]], start: list[int]) -> None:
+        """Block tables and prefix lengths of a prefill that attends through the paged cache."""
+        bt = torch.zeros(len(tables), max(len(tb) for tb in tables), dtype=torch.int32)
+        for r, tb in enumerate(tables):
+            bt[r, :len(tb)] = torch.tensor(tb, dtype=torch.int32)
+        meta.block_tables = bt.to(self.device, non_blocking=True)
+        meta.prefix_lens = torch.tensor(start, dtype=torch.int32).to(self.device, non_blocking=True)
+
     def _prefill(self, prompts: list[list[int]], tables: list[list[int]],
-                 cached: list[int] | None = None, greedy: bool = False) -> torch.Tensor:
+                 cached: list[int] | None = None, greedy: bool = False,
+                 slots: list[int] | None = None) -> torch.Tensor:
         """Prefill prompt tokens [cached[i], len) of each prompt (the first cached[i]
         tokens are prefix-cache hits already in the paged KV cache).  Returns the last
         position's logits per prompt, or (``greedy``) its greedy token id (the LM head's
@@ -391,7 +427,7 @@ class LLMEngine:
         for k, (p, tb) in enumerate(zip(prompts, tables)):
             while len(p) - cached[k] > budget:
                 end = cached[k] + budget
-                self._prefill([p[:end]], [tb], [cached[k]])
+                self._prefill([p[:end]], [tb], [cached[k]], slots=slots[k:k + 1] if slots else None)
                 cached[k] = end
         firsts = []
         i = 0
@@ -400,21 +436,8 @@ class LLMEngine:
             while j < len(prompts) and (j == i or tok + len(prompts[j]) - cached[j] <= self.max_prefill_tokens):
                 tok += len(prompts[j]) - cached[j]
                 j += 1
-            ids, pos, slots, cu = _prefill_inputs(prompts[i:j], tables[i:j], cached[i:j], BS)
-            t_ids = torch.from_numpy(ids).to(dev, non_blocking=True)
-            meta = AttnMeta(
-                prefill=True,
-                positions=torch.from_numpy(pos).to(dev, non_blocking=True),
-                slot_mapping=torch.from_numpy(slots).to(dev, non_blocking=True),
-                cu_seqlens=torch.from_numpy(cu).to(dev, non_blocking=True),
-                max_len=max(len(p) - c for p, c in zip(prompts[i:j], cached[i:j])))
-            if any(cached[i:j]):
-                maxb = max(len(tb) for tb in tables[i:j])
-                bt = torch.zeros(j - i, maxb, dtype=torch.int32)
-                for r, tb in enumerate(tables[i:j]):
-                    bt[r, :len(tb)] = torch.tensor(tb, dtype=torch.int32)
-                meta.block_tables = bt.to(dev, non_blocking=True)
-                meta.prefix_lens = torch.tensor(cached[i:j], dtype=torch.int32).to(dev, non_blocking=True)
+            t_ids, meta, cu = self.prefill_batch(prompts[i:j], tables[i:j], cached[i:j],
+                                                 slots[i:j] if slots else None)
             last = torch.from_numpy(cu[1:].astype(np.int64) - 1).to(dev, non_blocking=True)
             if _PREFILL_DUMP and meta.block_tables is not None:
                 os.makedirs(_PREFILL_DUMP, exist_ok=True)
@@ -426,7 +449,7 @@ class LLMEngine:
                 print(json.dumps({"prefill_chunk": j - i, "new_sum": sum(new), "new_max": max(new),
                                   "cached_mean": sum(cached[i:j]) / (j - i), "cached_max": max(cached[i:j]),
                                   "cached_min": min(cached[i:j])}), flush=True)
-            firsts.append(self.model.forward(t_ids, meta, self.kv.caches, logits_index=last, greedy_ids=greedy))
+            firsts.append(self.model.forward(t_ids, meta, self.caches, logits_index=last, greedy_ids=greedy))
             i = j
         return torch.cat(firsts, 0)
 
@@ -435,10 +458,36 @@ class LLMEngine:
         meta = self._decode_meta(g)
         if g.greedy:
             # greedy: the LM head's argmax is fused into its GEMM (no [B, vocab] logits)
-            nxt = self.model.forward(g.tokens, meta, self.kv.caches, greedy_ids=True)
+            nxt = self.model.forward(g.tokens, meta, self.caches, greedy_ids=True)
         else:
-            nxt = self._select(self.model.forward(g.tokens, meta, self.kv.caches), g)
+            nxt = self._select(self.model.forward(g.tokens, meta, self.caches), g)
         ops.decode_advance(nxt.long().contiguous(), g.out, g.tokens, g.positions, g.context_lens, g.valid)
+
+    def load_rows(self, g: _DecodeGraph, tokens: list[int] | None, positions: list[int], tables: list[list[int]],
+                  slots: list[int]) -> None:
+        """Upload the decode state of bucket ``g``: rows [0, len(positions)) at the given write
+        positions with their block tables and state slots, the rest padded.  ``tokens``
+        None: the caller sets ``g.tokens`` itself."""
+        B = len(positions)
+
+        def rows(vals, fill=0):
+            t = torch.full((g.bp,), fill, dtype=torch.int32)
+            t[:B] = torch.as_tensor(vals, dtype=torch.int32)
+            return t
+
+        bt = torch.zeros(g.bp, self.max_blocks_per_seq, dtype=torch.int32)
+        for i, tb in enumerate(tables):
+            bt[i, :len(tb)] = torch.tensor(tb, dtype=torch.int32)
+        _upload(g.block_tables, bt)
+        if slots:
+            _upload(g.state_slots, rows(slots, -1))
+        vl = rows([1] * B)
+        _upload(g.valid, vl)
+        pos = rows(positions)
+        _upload(g.positions, pos)
+        _upload(g.context_lens, pos + vl)
+        if tokens is not None:
+            _upload(g.tokens, rows(tokens))
 
     def _decode_meta(self, g: _DecodeGraph) -> AttnMeta:
         """Attention metadata of one decode step of bucket ``g`` (slots of the new tokens,
@@ -446,7 +495,8 @@ class LLMEngine:
         slots = ops.decode_slots(g.block_tables, g.positions, g.valid, self.block_size)
         meta = AttnMeta(prefill=False, positions=g.positions, slot_mapping=slots,
                         block_tables=g.block_tables, context_lens=g.context_lens,
-                        max_context=self.max_context, seq_order=g.order if self.lpt else None)
+                        max_context=self.max_context, seq_order=g.order if self.lpt else None,
+                        state_slots=g.state_slots if self.state is not None else None)
         if g.cascade:
             meta.shared_table, meta.shared_len = g.shared_table, g.shared_len
             meta.cascade_chunks = self._cascade_chunks(g.bp)
@@ -642,7 +692,9 @@ class LLMEngine:
             rot = int(os.environ.get("DOCQA_TUNE_ROTATE_MB", "512"))
             if rot > 0 and hasattr(tunable, "set_rotating_buffer_size"):
                 tunable.set_rotating_buffer_size(rot)
-        saved = [t.clone() for t in (g.tokens, g.positions, g.context_lens)]
+        saved = [t.clone() for t in (g.tokens, g.positions, g.context_lens, g.state_slots)]
+        # the warm-up step must not advance any recurrent state (K/V writes are idempotent)
+        g.state_slots.fill_(-1)
         try:
             s = torch.cuda.Stream()
             s.wait_stream(torch.cuda.current_stream())
@@ -667,7 +719,7 @@ class LLMEngine:
         finally:
             if tune and tunable is not None:
                 tunable.enable(False)
-        for t, v in zip((g.tokens, g.positions, g.context_lens), saved):
+        for t, v in zip((g.tokens, g.positions, g.context_lens, g.state_slots), saved):
             t.copy_(v)
         g.graph = graph
 
@@ -727,6 +779,8 @@ class LLMEngine:
         gen = params.max_new_tokens if gen is None else gen
         need = [self.kv.blocks_for(n + gen) for n in lens]
         r = Reservation([], [], params.max_new_tokens, len(prompts))
+        if self.state is not None:
+            r.slots = self.state.alloc(len(prompts))
         if not self._use_pc:
             try:
                 for n in need:
@@ -739,9 +793,9 @@ class LLMEngine:
         # one native call for the batch: longest cached full-block prefix of every prompt
         # (chained keys computed here, reused by the token-granular cache and registration)
         r.keys = [chain_keys(p, BS, (len(p) + BS - 1) // BS) for p in prompts]
-        hits, r.tables = self._retry(lambda: alloc.match_alloc_batch(
-            [k[1:len(p) // BS + 1] for k, p in zip(r.keys, prompts)], lens, need))
         try:
+            hits, r.tables = self._retry(lambda: alloc.match_alloc_batch(
+                [k[1:len(p) // BS + 1] for k, p in zip(r.keys, prompts)], lens, need))
             for i, p in enumerate(prompts):
                 k, c = hits[i], hits[i] * BS
                 if self.tail is not None and k < len(r.tables[i]):
@@ -769,6 +823,9 @@ class LLMEngine:
         for tb in r.tables:
             self.kv.allocator.free(tb)
         r.tables = []
+        if r.slots:
+            self.state.free(r.slots)
+            r.slots = []
         if r.copies:
             self.tail.unpin([src for src, _, _ in r.copies])
             r.copies = []
@@ -838,7 +895,7 @@ class LLMEngine:
                 ev[0].record()
             self.queue_prefix_copies(r)
             with tracing.span("engine.prefill", seqs=B, tokens=sum(lens) - sum(cached)):
-                logits = self._prefill(prompts, tables, cached, greedy=greedy)
+                logits = self._prefill(prompts, tables, cached, greedy=greedy, slots=r.slots)
             if use_pc:
                 with tracing.span("engine.register", seqs=B):
                     self.register_prefixes(prompts, tables, r.keys)
@@ -856,18 +913,7 @@ class LLMEngine:
                 st[:nshared] = torch.tensor(tables[0][:nshared], dtype=torch.int32)
                 _upload(g.shared_table, st)
                 g.shared_len.fill_(nshared * self.block_size)
-            # state for the first decode step
-            bt = torch.zeros(g.bp, self.max_blocks_per_seq, dtype=torch.int32)
-            for i, tb in enumerate(tables):
-                bt[i, :len(tb)] = torch.tensor(tb, dtype=torch.int32)
-            _upload(g.block_tables, bt)
-            vl = torch.zeros(g.bp, dtype=torch.int32)
-            vl[:B] = 1
-            _upload(g.valid, vl)
-            pos = torch.zeros(g.bp, dtype=torch.int32)
-            pos[:B] = torch.tensor(lens, dtype=torch.int32)
-            _upload(g.positions, pos)
-            _upload(g.context_lens, pos + vl)
+            self.load_rows(g, None, lens, tables, r.slots)      # state for the first decode step
             self.set_order(g, lens)
             if grouped and g.groups_fit:
                 self.set_groups(g, tables, [n + params.max_new_tokens for n in lens], nshared)

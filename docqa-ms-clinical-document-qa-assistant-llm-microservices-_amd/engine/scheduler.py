@@ -61,7 +61,7 @@ from .. import ops
 from ..parallel import comm
 from ..parallel.custom_ar import CollectiveError
 from ..utils import tracing
-from .llm_engine import LLMEngine, SamplingParams, _bucket, _DecodeGraph, _prefill_inputs
+from .llm_engine import LLMEngine, SamplingParams, _bucket, _DecodeGraph
 
 
 @dataclass
@@ -85,6 +85,7 @@ class Request:
     pos: int = 0
     preemptions: int = 0
     filled: int = 0      # mixed steps: prompt tokens already in the KV cache
+    slots: list[int] = field(default_factory=list)   # its recurrent-state slot, if the model has state
 
 
 class Lockstep:
@@ -275,8 +276,7 @@ class ContinuousEngine:
             if id(r) in seen:                # a completing prompt already placed in a slot
                 continue
             seen.add(id(r))
-            self.eng.kv.allocator.free(r.blocks)
-            r.blocks = []
+            self._free(r)
             if not r.future.done():
                 r.future.set_exception(e)
         self.running = []
@@ -284,6 +284,15 @@ class ContinuousEngine:
         self._version += 1
         self._master.valid.zero_()
         self._master.context_lens.zero_()
+        self._master.state_slots.fill_(-1)
+
+    def _free(self, r: Request) -> None:
+        """Give back a request's KV blocks and state slot."""
+        self.eng.kv.allocator.free(r.blocks)
+        r.blocks = []
+        if r.slots:
+            self.eng.state.free(r.slots)
+            r.slots = []
 
     # ------------------------------------------------------------------ one iteration
     @torch.inference_mode()
@@ -384,7 +393,8 @@ class ContinuousEngine:
                     self.kv_blocked += 1
                     break                        # retry after running requests retire
                 r.blocks, r.cached, r.res = res.tables[0], res.cached[0], res
-                res.tables = []                  # owned by the request from here on
+                r.slots = res.slots
+                res.tables, res.slots = [], []   # owned by the request from here on
                 admitted.append(self.waiting.popleft())
                 budget += len(r.prompt) - r.cached
                 if budget >= eng.max_prefill_tokens:
@@ -431,7 +441,7 @@ class ContinuousEngine:
         adm = self._take_waiting()
         if not adm:
             return
-        eng, alloc = self.eng, self.eng.kv.allocator
+        eng = self.eng
         t0 = time.perf_counter()
         try:
             with tracing.span("sched.admit", seqs=len(adm), tokens=sum(len(r.prompt) - r.cached for r in adm)):
@@ -439,20 +449,20 @@ class ContinuousEngine:
                     eng.queue_prefix_copies(r.res)
                 greedy = all(r.params.temperature <= 0 for r in adm)
                 out = eng._prefill([r.prompt for r in adm], [r.blocks for r in adm], [r.cached for r in adm],
-                                   greedy=greedy)
+                                   greedy=greedy, slots=[s for r in adm for s in r.slots])
                 err = comm.collective_error_snapshot()
                 first = out.tolist() if greedy else self._sample_rows(out, [r.params for r in adm])
                 comm.raise_on_collective_error(err)
         except CollectiveError:
             for r in adm:
                 eng.release(r.res)
-                alloc.free(r.blocks)
+                self._free(r)
                 r.future.set_exception(RuntimeError("TP collective failed during prefill"))
             raise
         except Exception as e:  # noqa: BLE001
             for r in adm:
                 eng.release(r.res)
-                alloc.free(r.blocks)
+                self._free(r)
                 r.future.set_exception(e)
             return
         eng.register_prefixes([r.prompt for r in adm], [r.blocks for r in adm], [r.res.keys[0] if r.res.keys else None
@@ -548,24 +558,16 @@ class ContinuousEngine:
                                [len(r.prompt) + r.params.max_new_tokens for r in self.running], self._nshared,
                                key=(self._version, self._nshared), ids=[r.rid for r in self.running])
             dmeta = eng._decode_meta(g)
-        from ..models.llama import AttnMeta
-
-        ids, pos, slots, cu = _prefill_inputs([r.prompt[:e] for r, _, e in pieces], [r.blocks for r, _, _ in pieces],
-                                              [s_ for _, s_, _ in pieces], BS)
-        maxb = max(len(r.blocks) for r, _, _ in pieces)
-        btab = torch.zeros(len(pieces), maxb, dtype=torch.int32)
-        for i, (r, _, _) in enumerate(pieces):
-            btab[i, :len(r.blocks)] = torch.tensor(r.blocks, dtype=torch.int32)
-        pmeta = AttnMeta(prefill=True, positions=torch.from_numpy(pos).to(dev), slot_mapping=torch.from_numpy(slots).to(dev),
-                         cu_seqlens=torch.from_numpy(cu).to(dev), max_len=max(e - s_ for _, s_, e in pieces),
-                         block_tables=btab.to(dev),
-                         prefix_lens=torch.tensor([s_ for _, s_, _ in pieces], dtype=torch.int32).to(dev))
+        chunk_ids, pmeta, cu = eng.prefill_batch([r.prompt[:e] for r, _, e in pieces], [r.blocks for r, _, _ in pieces],
+                                                 [s_ for _, s_, _ in pieces],
+                                                 [s_ for r, _, _ in pieces for s_ in r.slots])
+        if pmeta.block_tables is None:       # every piece starts its prompt: forward_mixed reads the cache anyway
+            eng.page_prefill(pmeta, [r.blocks for r, _, _ in pieces], [0] * len(pieces))
         done = [i for i, (r, _, e) in enumerate(pieces) if e == len(r.prompt)]
         rows = list(range(bp)) + [bp + int(cu[i + 1]) - 1 for i in done]
-        chunk_ids = torch.from_numpy(ids).to(dev)
         input_ids = torch.cat([g.tokens, chunk_ids]) if bp else chunk_ids
         with tracing.span("sched.mixed", running=n, bucket=bp, chunk_tokens=int(cu[-1]), completes=len(done)):
-            nxt = eng.model.forward_mixed(input_ids, bp, dmeta, pmeta, eng.kv.caches,
+            nxt = eng.model.forward_mixed(input_ids, bp, dmeta, pmeta, eng.caches,
                                           torch.tensor(rows, dtype=torch.long).to(dev))
             if bp:
                 ops.decode_advance(nxt[:bp].long().contiguous(), g.out, g.tokens, g.positions, g.context_lens,
@@ -672,6 +674,9 @@ class ContinuousEngine:
         m.tokens[sl].copy_(tok.to(dev, non_blocking=True))
         m.positions[sl].copy_(pos.to(dev, non_blocking=True))
         m.context_lens[sl].copy_((pos + 1).to(dev, non_blocking=True))
+        if self.eng.state is not None:
+            ss = torch.tensor([s for r in reqs for s in r.slots], dtype=torch.int32)
+            m.state_slots[sl].copy_(ss.to(dev, non_blocking=True))
         m.valid[sl].fill_(1)
         m.inv_temp[sl].copy_(it.to(dev, non_blocking=True))
         m.top_k[sl].copy_(tk.to(dev, non_blocking=True))
@@ -746,8 +751,8 @@ class ContinuousEngine:
             # have produced no token yet -- re-queue the latest of them first (the
             # last running row used to fail while prefilling prompts held the blocks it needed)
             v = max(self.prefilling, key=lambda r: (r.t_arrival, r.rid))
-            self.eng.kv.allocator.free(v.blocks)
-            v.blocks, v.res, v.cached, v.filled = [], None, 0, 0
+            self._free(v)
+            v.res, v.cached, v.filled = None, 0, 0
             self.prefilling = [r for r in self.prefilling if r is not v]
             v.preemptions += 1
             self.preempted += 1
@@ -759,16 +764,15 @@ class ContinuousEngine:
         v = max(self.running, key=lambda r: (r.t_arrival, r.rid))   # the latest arrival
         if len(self.running) == 1 and v.pos // self.eng.block_size >= len(v.blocks):
             # alone and still out of blocks: it can never finish in this pool
-            self.eng.kv.allocator.free(v.blocks)
-            v.blocks = []
+            self._free(v)
             v.done = True
             if not v.future.done():
                 v.future.set_exception(MemoryError("KV cache exhausted by a single request"))
             self._compact([])
             self._update_shared()
             return
-        self.eng.kv.allocator.free(v.blocks)
-        v.blocks, v.res, v.cached = [], None, 0
+        self._free(v)
+        v.res, v.cached = None, 0
         keep = [i for i, r in enumerate(self.running) if r is not v]
         self._compact(keep)
         v.prompt = v.prompt[:v.orig_len] + list(v.out)
@@ -881,8 +885,7 @@ class ContinuousEngine:
     def _retire(self, r: Request) -> None:
         self.completed += 1
         self.completed_short += len(r.out) < r.params.max_new_tokens
-        self.eng.kv.allocator.free(r.blocks)
-        r.blocks = []
+        self._free(r)
         if not r.future.done():
             r.future.set_result(list(r.out))
 
@@ -891,7 +894,7 @@ class ContinuousEngine:
         m, n, k = self._master, len(self.running), len(keep)
         if keep != list(range(k)):
             idx = torch.tensor(keep, dtype=torch.long, device=m.tokens.device)
-            for name in ("tokens", "positions", "context_lens", "valid", "block_tables", "inv_temp",
+            for name in ("tokens", "positions", "context_lens", "valid", "block_tables", "state_slots", "inv_temp",
                          "top_k", "top_p"):
                 t = getattr(m, name)
                 t[:k] = t[idx]
@@ -899,6 +902,7 @@ class ContinuousEngine:
         m.context_lens[k:n].zero_()
         m.positions[k:n].zero_()
         m.tokens[k:n].zero_()
+        m.state_slots[k:n].fill_(-1)
         self.running = [self.running[i] for i in keep]
         self._version += 1
 

@@ -1,4 +1,4 @@
-"""Hugging Face checkpoint IO for the generator and the encoders.
+"""Checkpoint IO and the registry of generator families.
 
 The reference downloads its weights through its runtimes (MiniLM from the HF hub inside
 sentence-transformers, semantic-indexer/indexer.py:21; Mistral pulled by Ollama,
@@ -15,13 +15,16 @@ from __future__ import annotations
 
 import json
 import os
-from collections.abc import Mapping
+from collections.abc import Callable, Mapping
+from dataclasses import dataclass
 from pathlib import Path
 
 import torch
 
 from ..ops import reference as ref
 from .bert import BertConfig, BertEncoder, BertTokenClassifier
+from . import saritar
+from .hybrid import HybridModel
 from .llama import LlamaConfig, LlamaModel
 
 
@@ -136,24 +139,93 @@ def save_llama(model: LlamaModel, path) -> None:
               str(p / "model.safetensors"))
 
 
-def resolve_llama_config(name_or_path) -> LlamaConfig:
+def load_saritar(path, device="cuda", dtype=torch.bfloat16) -> HybridModel:
+    """Saritar checkpoint directory (config.json + model.safetensors) -> :class:`HybridModel`."""
+    p = Path(path)
+    cfg = saritar.config_from_json(_config_json(p), name=p.name)
+    return HybridModel(cfg, device=device, dtype=dtype, weights=LazySafetensors(p))
+
+
+def save_saritar(cfg, weights: Mapping, path) -> None:
+    """Write a Saritar checkpoint: ``weights`` by :meth:`HybridConfig.tensor_shapes` name, in bf16."""
+    from safetensors.torch import save_file
+
+    p = Path(path)
+    p.mkdir(parents=True, exist_ok=True)
+    (p / "config.json").write_text(json.dumps(saritar.config_to_json(cfg), indent=1))
+    save_file({k: weights[k].detach().to(torch.bfloat16).cpu().contiguous() for k in cfg.tensor_shapes()},
+              str(p / "model.safetensors"))
+
+
+# ------------------------------------------------------------------ generator registry
+def _config_json(p: Path) -> dict:
+    return json.loads((p / "config.json").read_text())
+
+
+@dataclass(frozen=True)
+class DecoderFamily:
+    """A generator design: which config.json and preset names are its own, and how its
+    configuration and model come about."""
+    name: str
+    owns_json: Callable[[dict], bool]
+    owns_preset: Callable[[str], bool]
+    config_from_json: Callable
+    preset: Callable
+    load: Callable                  # (dir, device, dtype) -> model
+    build: Callable                 # (config, device, dtype, seed) -> randomly initialised model
+    gpu_dtypes: tuple               # dtypes its GPU kernels run in
+
+
+FAMILIES = (
+    DecoderFamily("saritar", lambda js: js.get("architecture") == saritar.ARCHITECTURE,
+                  lambda n: n.startswith("saritar"), saritar.config_from_json, saritar.preset, load_saritar,
+                  lambda cfg, device, dtype, seed: HybridModel(cfg, device=device, dtype=dtype, seed=seed),
+                  (torch.bfloat16, torch.float32)),
+    DecoderFamily("llama", lambda js: "architecture" not in js, lambda n: True, llama_config_from_hf,
+                  LlamaConfig.preset, load_llama,
+                  lambda cfg, device, dtype, seed: LlamaModel(cfg, device=device, dtype=dtype, seed=seed),
+                  (torch.bfloat16,)),
+)
+
+
+def decoder_family(name_or_path) -> DecoderFamily:
+    """The family of a checkpoint directory (by its config.json) or of a preset name."""
+    if is_checkpoint(name_or_path):
+        js = _config_json(Path(str(name_or_path)))
+        for f in FAMILIES:
+            if f.owns_json(js):
+                return f
+        raise NotImplementedError(f"architecture {js.get('architecture')!r} is not supported "
+                                  f"(families: {', '.join(f.name for f in FAMILIES)})")
+    return next(f for f in FAMILIES if f.owns_preset(str(name_or_path)))
+
+
+def resolve_decoder_config(name_or_path):
+    f = decoder_family(name_or_path)
     if is_checkpoint(name_or_path):
         p = Path(str(name_or_path))
-        return llama_config_from_hf(json.loads((p / "config.json").read_text()), name=p.name)
-    return LlamaConfig.preset(str(name_or_path))
+        return f.config_from_json(_config_json(p), name=p.name)
+    return f.preset(str(name_or_path))
 
 
-def resolve_llama(name_or_path, device="cuda", seed: int = 0) -> LlamaModel:
-    """A checkpoint directory -> its weights; a preset name -> random-init weights.
+def resolve_decoder(name_or_path, device="cuda", seed: int = 0, dtype: torch.dtype | None = None):
+    """A checkpoint directory -> its weights; a preset name -> random-init weights, of
+    whichever family it belongs to.  ``dtype``: default ``DOCQA_LLM_DTYPE``.
     ``DOCQA_LLM_DTYPE`` (bfloat16 | float32; default bfloat16): the weight / KV dtype --
     float32 for CPU rehearsals that compare TP = N against TP = 1 token for token (bf16
     rounds each TP split's sums differently, which flips near-tied greedy picks of a
     random-init model)."""
-    dtype = {"bfloat16": torch.bfloat16, "bf16": torch.bfloat16, "float32": torch.float32,
-             "fp32": torch.float32}[os.environ.get("DOCQA_LLM_DTYPE", "bfloat16")]
+    if dtype is None:
+        dtype = {"bfloat16": torch.bfloat16, "bf16": torch.bfloat16, "float32": torch.float32,
+                 "fp32": torch.float32}[os.environ.get("DOCQA_LLM_DTYPE", "bfloat16")]
+    f = decoder_family(name_or_path)
     if is_checkpoint(name_or_path):
-        return load_llama(name_or_path, device=device, dtype=dtype)
-    return LlamaModel(LlamaConfig.preset(str(name_or_path)), device=device, dtype=dtype, seed=seed)
+        return f.load(name_or_path, device=device, dtype=dtype)
+    return f.build(f.preset(str(name_or_path)), device, dtype, seed)
+
+
+# earlier names of the two entry points
+resolve_llama_config, resolve_llama = resolve_decoder_config, resolve_decoder
 
 
 # --------------------------------------------------------------------------- BERT
@@ -254,6 +326,7 @@ def tokenizer_json(name_or_path) -> str | None:
     return None
 
 
-__all__ = ["LazySafetensors", "is_checkpoint", "load_llama", "save_llama", "resolve_llama",
-           "resolve_llama_config", "load_bert_encoder", "load_bert_token_classifier", "resolve_bert",
+__all__ = ["LazySafetensors", "is_checkpoint", "load_llama", "save_llama", "load_saritar", "save_saritar",
+           "DecoderFamily", "FAMILIES", "decoder_family", "resolve_decoder", "resolve_decoder_config",
+           "resolve_llama", "resolve_llama_config", "load_bert_encoder", "load_bert_token_classifier", "resolve_bert",
            "resolve_bert_config", "tokenizer_json", "use_checkpoint_tokenizers", "llama_config_from_hf", "bert_config_from_hf"]

@@ -1,0 +1,388 @@
+"""Decoders whose layers mix windowed attention with recurrent (selective-scan) mixers, with
+an fp32 residual stream and a norm before and after every sublayer.
+
+A model is a list of layers (:class:`LayerSpec`: a mixer and an optional feed-forward), some
+of which may run several passes over the same weights (``loop``).  Every RUN of a layer has
+its own cache or state, so the engine sees as many caches as runs.
+
+MI355X layout:
+  * one sandwich_norm.hip launch stands between any two projections: it sums the split-K
+    slabs of the last one, normalises that output, updates the fp32 residual (and adds the
+    embedding ahead of a loop's next pass) and emits the next projection's input;
+  * attention keeps the key rows as projected, once, as key and value, with the row's inverse
+    RMS beside it (ops.qk_norm_store) -- half the cache bytes of a K / V pair;
+  * a recurrent layer runs in_proj -> conv -> x_proj -> dt_proj -> scan + gate -> out_proj,
+    conv and scan over packed sequences in prefill and one fused step each in decode, the
+    state in per-request slots (engine/kv_cache.py StatePool);
+  * projections run on the same GEMM plans as the Llama decoder (ops.project / ops.linear):
+    weights are padded with zero rows at load where that reaches a kernel's granule.
+
+bf16 runs matrix products and activations in bf16; the residual, norms, attention scores,
+decays, step sizes and states are fp32.  float32 runs everything in fp32.
+"""
+from __future__ import annotations
+
+import math
+import zlib
+from dataclasses import dataclass, field
+
+import torch
+
+from .. import ops
+from ..engine.kv_cache import KVSpec, StateSpec
+from ..parallel import comm
+from .decoder import Decoder
+from .llama import AttnMeta
+
+
+@dataclass(frozen=True)
+class WindowAttentionSpec:
+    """Causal attention over the last ``window`` tokens; no rotation; head-wise q / k norms;
+    the key projection is the value; a learned sink per query head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    window: int
+
+
+@dataclass(frozen=True)
+class SelectiveScanSpec:
+    """Mamba mixer: ``inner`` channels, ``state`` states each, ``dt_rank`` of the step
+    projection, ``conv`` taps of the short causal convolution."""
+    inner: int
+    state: int
+    dt_rank: int
+    conv: int
+
+
+@dataclass(frozen=True)
+class LayerSpec:
+    mixer: WindowAttentionSpec | SelectiveScanSpec
+    ff: int = 0                     # squared-ReLU feed-forward width, 0: none
+
+
+@dataclass
+class HybridConfig:
+    name: str
+    vocab_size: int
+    hidden: int
+    layer_specs: list
+    embed_scale: float = 1.0
+    rms_eps: float = 1e-5
+    loop: tuple | None = None       # (start, stop, times)
+    max_position: int = 1 << 20     # no position enters the weights
+    bos_token_id: int = -1          # no special tokens of its own
+    eos_token_id: int = -1
+    runs: list = field(init=False)  # (layer, embedding added ahead of it)
+
+    def __post_init__(self):
+        n = len(self.layer_specs)
+        lo, hi, times = self.loop or (0, 0, 1)
+        if not (0 <= lo <= hi <= n and times >= 1):
+            raise ValueError(f"loop {self.loop} does not fit {n} layers")
+        body = list(range(lo, hi))
+        self.runs = [(i, False) for i in range(lo)]
+        for p in range(times if body else 0):
+            self.runs += [(i, p > 0 and i == lo) for i in body]
+        self.runs += [(i, False) for i in range(hi, n)]
+        for sp in self.layer_specs:
+            m = sp.mixer
+            if isinstance(m, WindowAttentionSpec) and (m.heads % m.kv_heads or m.window < 1 or m.dim > 512):
+                raise ValueError(f"unsupported attention sizes {m}")
+            if isinstance(m, SelectiveScanSpec) and (m.state > 256 or m.conv < 1):
+                raise ValueError(f"unsupported scan sizes {m}")
+
+    @property
+    def layers(self) -> int:
+        return len(self.layer_specs)
+
+    def tensor_shapes(self) -> dict:
+        """Every weight's name and shape (linear weights [out, in])."""
+        W, V = self.hidden, self.vocab_size
+        out = {"embed": (V, W)}
+        for i, sp in enumerate(self.layer_specs):
+            p, m = f"l{i}.", sp.mixer
+            out[p + "norm1"] = out[p + "norm1b"] = (W,)
+            if isinstance(m, WindowAttentionSpec):
+                hd = m.heads * m.dim
+                out.update({p + "mix.q": (hd, W), p + "mix.k": (m.kv_heads * m.dim, W), p + "mix.q.norm": (m.dim,),
+                            p + "mix.k.norm": (m.dim,), p + "mix.sink": (m.heads,), p + "mix.o": (W, hd)})
+            else:
+                C, N, R = m.inner, m.state, m.dt_rank
+                out.update({p + "mix.in": (2 * C, W), p + "mix.conv": (C, m.conv), p + "mix.conv.b": (C,),
+                            p + "mix.x": (R + 2 * N, C), p + "mix.dt": (C, R), p + "mix.dt.b": (C,),
+                            p + "mix.A_log": (C, N), p + "mix.D": (C,), p + "mix.o": (W, C)})
+            if sp.ff:
+                out.update({p + "norm2": (W,), p + "norm2b": (W,), p + "mlp.up": (sp.ff, W), p + "mlp.down": (W, sp.ff)})
+        out.update({"final.norm": (W,), "head": (V, W)})
+        return out
+
+    def num_params(self) -> int:
+        return sum(math.prod(s) for s in self.tensor_shapes().values())
+
+
+def _pad_up(n: int, m: int) -> int:
+    return -(-n // m) * m
+
+
+@dataclass
+class _Part:
+    """Rows [lo, hi) of a forward that attend / scan together: one token a row (decode) or
+    packed sequences (prefill)."""
+    lo: int
+    hi: int
+    meta: AttnMeta
+
+    @property
+    def decode(self) -> bool:
+        return not self.meta.prefill
+
+
+def _split(t: torch.Tensor, part: _Part, parts: list) -> torch.Tensor:
+    return t if len(parts) == 1 else t[part.lo:part.hi]
+
+
+def _join(ts: list) -> torch.Tensor:
+    return ts[0] if len(ts) == 1 else torch.cat(ts)
+
+
+class WindowAttention:
+    def __init__(self, sp: WindowAttentionSpec, get, eps: float, dtype):
+        self.sp, self.eps = sp, eps
+        self.qk = torch.cat([get("q"), get("k")]).to(dtype).contiguous()
+        self.o = get("o").to(dtype).contiguous()
+        # the cached key is the projection itself: both norm weights go to the query side
+        self.qk_norm = (get("q.norm").float() * get("k.norm").float()).contiguous()
+        self.sink = get("sink").float().contiguous()
+
+    def cache_spec(self):
+        return KVSpec(self.sp.kv_heads, self.sp.dim, shared=True)
+
+    def activation_elems(self) -> int:
+        return (3 * self.sp.heads + self.sp.kv_heads) * self.sp.dim
+
+    def run(self, x, parts, slot_mapping, cache, decode):
+        sp = self.sp
+        kc, ks = cache
+        q = ops.qk_norm_store(ops.project(x, self.qk, decode), self.qk_norm, slot_mapping, kc, ks, sp.heads, self.eps)
+        out = []
+        for p in parts:
+            m = p.meta
+            kw = dict(window=sp.window, sink=self.sink, k_scale=ks)
+            if p.decode:
+                out.append(ops.window_attn(_split(q, p, parts), kc, m.block_tables, m.context_lens, sp.scale, **kw))
+            else:
+                out.append(ops.window_attn(_split(q, p, parts), kc, m.block_tables, m.prefix_lens, sp.scale,
+                                           cu=m.cu_seqlens, max_q=m.max_len, **kw))
+        return ops.project(_join(out), self.o, decode)
+
+
+class SelectiveScan:
+    def __init__(self, sp: SelectiveScanSpec, get, eps: float, dtype):
+        self.sp, self.dtype = sp, dtype
+        C, N, R = sp.inner, sp.state, sp.dt_rank
+        self.w_in = get("in").to(dtype).contiguous()
+        self.conv_w = get("conv").float().t().contiguous()        # [taps, C]
+        self.conv_b = get("conv.b").float().contiguous()
+        # [dt | B | C] rows, each section and the whole padded with zero rows to the GEMM granules
+        self.rp, self.np = _pad_up(R, 64), _pad_up(N, 8)
+        wx = get("x")
+        rows = self.rp + 2 * self.np
+        pad = wx.new_zeros(_pad_up(rows, 128 if rows <= 256 else 256), C)
+        pad[:R] = wx[:R]
+        pad[self.rp:self.rp + N] = wx[R:R + N]
+        pad[self.rp + self.np:self.rp + self.np + N] = wx[R + N:]
+        self.w_x = pad.to(dtype).contiguous()
+        wd = get("dt")
+        self.w_dt = torch.cat([wd, wd.new_zeros(C, self.rp - R)], 1).to(dtype).contiguous()
+        self.dt_b = get("dt.b").float().contiguous()
+        a = -torch.exp(get("A_log").float()) * math.log2(math.e)
+        self.A2 = torch.cat([a, a.new_zeros(C, _pad_up(N, 4) - N)], 1).contiguous()
+        self.D = get("D").float().contiguous()
+        self.w_o = get("o").to(dtype).contiguous()
+
+    def cache_spec(self):
+        return StateSpec(((self.sp.conv - 1, self.sp.inner), tuple(self.A2.shape)), (False, True))
+
+    def activation_elems(self) -> int:
+        return 5 * self.sp.inner + self.w_x.shape[0]
+
+    def run(self, x, parts, slot_mapping, cache, decode):
+        C, N = self.sp.inner, self.sp.state
+        conv_state, scan_state = cache
+        xz = ops.project(x, self.w_in, True) if decode and len(parts) == 1 else ops.linear(x, self.w_in, decode)
+        xc, zs = [], []
+        for p in parts:
+            m = p.meta
+            if p.decode:
+                y, z = ops.conv_step(_split(xz, p, parts), self.conv_w, self.conv_b, conv_state, m.state_slots,
+                                     m.positions)
+            else:
+                r = _split(xz, p, parts)
+                y, z = ops.causal_conv(r, self.conv_w, self.conv_b, conv_state, m.state_slots, m.cu_seqlens,
+                                       m.prefix_lens, m.max_len), r[:, C:]
+            xc.append(y)
+            zs.append(z)
+        xa = _join(xc)
+        pr = ops.linear(xa, self.w_x, decode)
+        dt = ops.linear(pr[:, :self.rp].contiguous(), self.w_dt, decode)
+        out = []
+        for p, y, z in zip(parts, xc, zs):
+            m = p.meta
+            args = (y, _split(dt, p, parts), _split(pr, p, parts), self.rp, self.rp + self.np, N, z, self.A2, self.D,
+                    self.dt_b, scan_state, m.state_slots)
+            if p.decode:
+                out.append(ops.selective_step(*args, m.positions))
+            else:
+                out.append(ops.selective_scan(*args, m.cu_seqlens, m.prefix_lens, m.max_len))
+        return ops.project(_join(out), self.w_o, decode)
+
+
+class SquaredReluMLP:
+    def __init__(self, get, dtype):
+        self.dtype = dtype
+        self.up = get("up").to(dtype).contiguous()
+        self.down = get("down").to(dtype).contiguous()
+
+    def run(self, x, decode):
+        return ops.project(ops.squared_relu(ops.project(x, self.up, decode), self.dtype), self.down, decode)
+
+
+class HybridModel(Decoder):
+    prefix_reuse = False      # a prompt's recurrent state is not in its K/V blocks
+    paged_prefill = True
+
+    def __init__(self, cfg: HybridConfig, device="cuda", dtype=torch.bfloat16, seed: int = 0, weights=None):
+        """``weights``: mapping of :meth:`HybridConfig.tensor_shapes` names to tensors, read one
+        at a time; None: random ones."""
+        if comm.state().tp_size > 1:
+            raise NotImplementedError("hybrid decoders run at TP = 1 (replicate them per GPU)")
+        self.cfg, self.device, self.dtype = cfg, torch.device(device), dtype
+        self.tp, self.tp_rank = 1, 0
+        self.vocab_shard = self.vocab_valid = cfg.vocab_size
+        self.vocab_start = 0
+        att = [s.mixer for s in cfg.layer_specs if isinstance(s.mixer, WindowAttentionSpec)]
+        self.hq, self.hkv = (att[0].heads, att[0].kv_heads) if att else (1, 1)
+        self.tap = None           # a list: receives the residual stream after every run
+        self._load(weights if weights is not None else _RandomWeights(cfg, self.device, seed))
+
+    def _load(self, weights) -> None:
+        cfg, dt = self.cfg, self.dtype
+        shapes = cfg.tensor_shapes()
+
+        def get(name):
+            t = weights[name]
+            if tuple(t.shape) != shapes[name]:
+                raise ValueError(f"{name}: shape {tuple(t.shape)}, expected {shapes[name]}")
+            return t.to(self.device)
+
+        def norm(name):
+            return get(name).float().contiguous()
+
+        self.embed = get("embed").to(dt).contiguous()
+        self.lm_head = get("head").to(dt).contiguous()
+        self.final_norm = norm("final.norm")
+        self.layers = []
+        for i, sp in enumerate(cfg.layer_specs):
+            p = f"l{i}."
+            cls = WindowAttention if isinstance(sp.mixer, WindowAttentionSpec) else SelectiveScan
+            L = {"mixer": cls(sp.mixer, lambda n: get(p + "mix." + n), cfg.rms_eps, dt),
+                 "norm1": norm(p + "norm1"), "norm1b": norm(p + "norm1b"), "mlp": None}
+            if sp.ff:
+                L.update(mlp=SquaredReluMLP(lambda n: get(p + "mlp." + n), dt), norm2=norm(p + "norm2"),
+                         norm2b=norm(p + "norm2b"))
+            self.layers.append(L)
+
+    # ------------------------------------------------------------------ caches
+    def _run_specs(self) -> list:
+        return [self.layers[i]["mixer"].cache_spec() for i, _ in self.cfg.runs]
+
+    def kv_specs(self) -> list:
+        return [s for s in self._run_specs() if isinstance(s, KVSpec)]
+
+    def state_specs(self) -> list:
+        return [s for s in self._run_specs() if isinstance(s, StateSpec)]
+
+    def bind_caches(self, kv, state) -> list:
+        k, s = iter(kv.caches), iter(state.states if state is not None else [])
+        return [next(k) if isinstance(sp, KVSpec) else next(s) for sp in self._run_specs()]
+
+    def activation_elems(self) -> int:
+        ff = max([s.ff for s in self.cfg.layer_specs] + [0])
+        return 8 * self.cfg.hidden + max(max(L["mixer"].activation_elems() for L in self.layers), 3 * ff)
+
+    def weight_bytes(self) -> int:
+        return self.cfg.num_params() * self.embed.element_size()
+
+    # ------------------------------------------------------------------ forward
+    def forward(self, input_ids, meta: AttnMeta, caches: list, logits_index=None, greedy_ids: bool = False):
+        """Same contract as :meth:`LlamaModel.forward`; prefill metadata always carries block
+        tables, prefix lengths and state slots."""
+        x = self._hidden(input_ids, [_Part(0, input_ids.shape[0], meta)], meta.slot_mapping, caches)
+        return self._head(x, logits_index, greedy_ids)
+
+    def forward_mixed(self, input_ids, n_dec: int, dmeta: AttnMeta, pmeta: AttnMeta, caches: list, logits_index,
+                      return_logits: bool = False):
+        """Same contract as :meth:`LlamaModel.forward_mixed`: rows [0, n_dec) decode, the rest
+        prompt portions; projections run over all rows at once."""
+        T = input_ids.shape[0]
+        parts = ([_Part(0, n_dec, dmeta)] if n_dec else []) + ([_Part(n_dec, T, pmeta)] if T > n_dec else [])
+        slots = _join([p.meta.slot_mapping for p in parts])
+        return self._head(self._hidden(input_ids, parts, slots, caches), logits_index, not return_logits)
+
+    def _hidden(self, input_ids, parts, slot_mapping, caches):
+        cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
+        decode = all(p.decode for p in parts)
+        runs = cfg.runs
+        loops = any(again for _, again in runs)
+        first = self.layers[runs[0][0]]["norm1"] if runs else self.final_norm
+        res, emb, x = ops.embed_scale_rmsnorm(input_ids, self.embed, cfg.embed_scale, first, eps, keep=loops)
+        for r, (i, _) in enumerate(runs):
+            L = self.layers[i]
+            last = r + 1 == len(runs)
+            nxt = self.final_norm if last else self.layers[runs[r + 1][0]]["norm1"]
+            add = emb if not last and runs[r + 1][1] else None
+            y = L["mixer"].run(x, parts, slot_mapping, caches[r], decode)
+            if L["mlp"] is not None:
+                x = ops.sandwich_rmsnorm(y, res, L["norm1b"], L["norm2"], eps, out_dtype=dt)
+                y = L["mlp"].run(x, decode)
+            x = ops.sandwich_rmsnorm(y, res, L["norm1b" if L["mlp"] is None else "norm2b"], nxt, eps, add=add,
+                                     out_dtype=dt)
+            if self.tap is not None:
+                self.tap.append(res - add if add is not None else res.clone())
+        return x
+
+    def _head(self, x, logits_index, greedy_ids):
+        if logits_index is not None:
+            x = x.index_select(0, logits_index)
+        if greedy_ids:
+            return self.greedy_ids(x)
+        return ops.lm_head_logits(x.contiguous(), self.lm_head)
+
+
+class _RandomWeights:
+    """Random weights by tensor name: unit-variance projections, a decay spectrum and step
+    sizes in the range of trained selective-scan models."""
+
+    def __init__(self, cfg: HybridConfig, device, seed: int):
+        self.shapes, self.device, self.seed = cfg.tensor_shapes(), device, seed
+
+    def __getitem__(self, name: str) -> torch.Tensor:
+        shape = self.shapes[name]
+        g = torch.Generator(device=self.device)
+        g.manual_seed((self.seed * 1_000_003 + zlib.crc32(name.encode())) & 0x7FFFFFFFFFFF)
+        kind = name.rsplit(".", 1)[-1]
+        if name.endswith("norm") or kind.startswith("norm"):
+            return torch.ones(shape, device=self.device)
+        if kind == "A_log":
+            return torch.log(torch.arange(1, shape[1] + 1, device=self.device).float()).expand(shape).contiguous()
+        if kind == "D":
+            return torch.ones(shape, device=self.device)
+        if name.endswith("dt.b"):
+            u = torch.rand(shape, device=self.device, generator=g)
+            dt = torch.exp(u * (math.log(0.1) - math.log(1e-3)) + math.log(1e-3))
+            return dt + torch.log(-torch.expm1(-dt))          # softplus^-1
+        std = 1.0 if len(shape) == 1 else (0.02 if name == "embed" else shape[-1] ** -0.5)
+        t = torch.empty(shape, device=self.device, dtype=torch.bfloat16 if len(shape) == 2 else torch.float32)
+        return t.normal_(0.0, std, generator=g)

@@ -34,7 +34,9 @@ import torch
 import torch.nn.functional as F
 
 from .. import ops
+from ..engine.kv_cache import KVSpec
 from ..parallel import comm
+from .decoder import Decoder
 
 # cascade decode over a library-GEMM QKV: DOCQA_CASCADE_ROPE=1 fuses RoPE + the new
 # token's cache write into the cascade kernels (ops.paged_decode_cascade_rope).  Off by
@@ -141,9 +143,11 @@ class AttnMeta:
     decode_defer: bool = False
     # ... a split plan whose items start at block 0 (the groups attend the shared prefix)
     decode_inline: bool = False
+    # state slot of each sequence (prefill) / row (decode, -1: padded) of a recurrent model
+    state_slots: torch.Tensor | None = None
 
 
-class LlamaModel:
+class LlamaModel(Decoder):
     def __init__(self, cfg: LlamaConfig, device="cuda", dtype=torch.bfloat16, seed: int = 0,
                  init: bool = True):
         self.cfg = cfg
@@ -285,6 +289,14 @@ class LlamaModel:
         for L in self.layers:
             n += sum(t.numel() for t in L.values())
         return n * self.embed.element_size()
+
+    def kv_specs(self) -> list:
+        return [KVSpec(self.hkv, self.cfg.head_dim)] * self.cfg.layers
+
+    def activation_elems(self) -> int:
+        # hidden-sized buffers, QKV, the gate|up product / SwiGLU output
+        cfg = self.cfg
+        return 6 * cfg.hidden + (self.hq + 2 * self.hkv) * cfg.head_dim + 3 * self.inter
 
     # ------------------------------------------------------------------ forward
     def forward(self, input_ids: torch.Tensor, meta: AttnMeta, kv_caches: list,
@@ -608,40 +620,3 @@ class LlamaModel:
             raise RuntimeError(f"decode ticket buffer holds {self._tick.numel()} words, a {B}-row bucket "
                                f"needs {need}: raise the first bucket size (buffers are never regrown)")
         return self._tick
-
-    def greedy_ids(self, x: torch.Tensor) -> torch.Tensor:
-        """Greedy token ids int64 [R] of the final normed hidden rows ``x``: the LM-head GEMM
-        with its argmax fused (mgemm.hip EPI_ARGMAX, no [R, vocab] logits) where the shape
-        allows, the vocab-parallel pick resolved by one packed-key MAX all-reduce at TP > 1."""
-        R = x.shape[0]
-        N, K = self.lm_head.shape
-        fused = ops.lm_head_argmax_ok(R, N, K) or (self.tp > 1 and 0 < R <= ops.MID_M_MAX
-                                                   and ops.lm_head_argmax_shape_ok(N, K))
-        if self.tp == 1:
-            if fused:
-                return ops.lm_head_argmax(x, self.lm_head, self.cfg.vocab_size)
-            return self.greedy(ops.lm_head_logits(x, self.lm_head))
-        if fused and self.vocab_valid > 0:
-            ids, vals = ops.lm_head_argmax(x, self.lm_head, self.vocab_valid, with_values=True)
-        else:
-            logits = ops.lm_head_logits(x, self.lm_head)[:, : max(1, self.vocab_valid)]
-            ids = ops.argmax(logits)
-            vals = logits.gather(1, ids[:, None])[:, 0].float()
-        if self.vocab_valid == 0:
-            vals = torch.full_like(vals, float("-inf"))
-        return comm.tp_argmax(vals, ids + self.vocab_start)
-
-    def greedy(self, logits: torch.Tensor) -> torch.Tensor:
-        """argmax over the (possibly vocab-parallel) logits -> int64 [R]."""
-        if self.tp == 1:
-            return ops.argmax(logits)
-        valid = logits[:, : max(1, self.vocab_valid)]
-        idx = ops.argmax(valid)
-        val = valid.gather(1, idx[:, None])[:, 0].float()
-        if self.vocab_valid == 0:
-            val = torch.full_like(val, float("-inf"))
-        return comm.tp_argmax(val, idx + self.vocab_start)
-
-    def full_logits(self, logits: torch.Tensor) -> torch.Tensor:
-        full = comm.tp_all_gather_last(logits)
-        return full[:, : self.cfg.vocab_size]

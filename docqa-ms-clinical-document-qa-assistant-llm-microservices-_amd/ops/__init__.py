@@ -52,6 +52,11 @@ def load_native(build_if_missing: bool = False) -> bool:
         return _loaded
 
 
+def native_error() -> str | None:
+    """Why the last :func:`load_native` failed."""
+    return _load_error
+
+
 def native_loaded() -> bool:
     return _loaded
 
@@ -578,7 +583,7 @@ def lm_head_logits(x, w):
     kernel with 256-wide tiles up to 512, the prefill kernels
     beyond -- no library GEMM.  Greedy rows never get here: their
     argmax is fused into the GEMM (:func:`lm_head_argmax`)."""
-    if _gpu(x):
+    if _gpu(x) and x.dtype == torch.bfloat16:
         N, K = w.shape
         M = x.numel() // K
         if 0 < M <= 192 and N % 64 == 0 and K % 512 == 0:
@@ -1182,6 +1187,138 @@ def flash_prefill_paged(qkv, cu_seqlens, max_len, Hq, Hkv, D, scale, k_cache, v_
                                              v_cache, block_tables, ctx_start)
     return ref.flash_prefill_paged(qkv, cu_seqlens, max_len, Hq, Hkv, D, scale, k_cache, v_cache,
                                    block_tables, ctx_start)
+
+
+# ----------------------------------------------------------------------------- hybrid decoders
+# Building blocks of decoders with an fp32 residual stream, norms around every sublayer,
+# windowed attention and recurrent mixers (models/hybrid.py); bf16 or fp32 activations.  A
+# projection feeding one of them is its product [M, N] or its split-K slabs [S, M, N].
+def embed_scale_rmsnorm(ids, table, scale: float, w, eps: float, keep: bool = False):
+    """(h, copy of h or None, x): h = table[ids] * scale in fp32 (the residual stream),
+    x = rmsnorm(h) * w in the table's dtype."""
+    if _gpu(table):
+        h, e, x = _native().embed_scale_rmsnorm(ids.contiguous(), table, float(scale), w, float(eps), keep)
+        return h, (e if keep else None), x
+    return ref.embed_scale_rmsnorm(ids, table, scale, w, eps, keep)
+
+
+def sandwich_rmsnorm(P, residual, w_post, w_next, eps: float, add=None, out_dtype=torch.bfloat16):
+    """residual (fp32, in place) += rmsnorm(P) * w_post (+ ``add``); returns
+    rmsnorm(residual) * w_next in ``out_dtype``."""
+    if _gpu(P):
+        return _native().sandwich_rmsnorm(P.contiguous(), residual, w_post, add, w_next, float(eps),
+                                          out_dtype == torch.float32)
+    return ref.sandwich_rmsnorm(P, residual, w_post, w_next, eps, add, out_dtype)
+
+
+def squared_relu(P, out_dtype=torch.bfloat16):
+    """max(P, 0)^2 of a projection."""
+    if _gpu(P):
+        return _native().squared_relu(P.contiguous(), out_dtype == torch.float32)
+    return ref.squared_relu(P, out_dtype)
+
+
+def qk_norm_store(P, w, slots, k_cache, k_scale, H: int, eps: float):
+    """Queries rms(q) * w per head [M, H * D] from a [q | k] projection; the key rows go to
+    the paged cache as projected, with their inverse root mean square in ``k_scale``.  A
+    key norm's weight is folded into ``w`` by the caller: q_n . k_n = k_scale (q' . k)."""
+    if _gpu(P):
+        return _native().qk_norm_store(P.contiguous(), w, slots, k_cache, k_scale, int(H), float(eps))
+    return ref.qk_norm_store(P, w, slots, k_cache, k_scale, H, eps)
+
+
+def window_attn(q, k_cache, block_tables, ctx, scale: float, window: int = 0, sink=None, k_scale=None, v_cache=None,
+                cu=None, max_q: int = 1):
+    """Causal attention over the last ``window`` tokens (0: all) of the paged cache, scores
+    times ``k_scale`` per cached key, ``sink`` [H] in the denominator, ``v_cache`` None: the
+    keys are the values.  With ``cu`` [B + 1]: packed query tokens, ``ctx`` the position of
+    each sequence's first; without: one query token a row, ``ctx`` the context lengths."""
+    if _gpu(q):
+        return _native().window_attn(q.contiguous(), k_cache, v_cache, k_scale, block_tables, cu, ctx, int(max_q),
+                                     float(scale), int(window), sink)
+    return ref.window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink)
+
+
+def causal_conv(x, w, bias, state, slots, cu, ctx, max_len: int):
+    """silu(causal convolution) of the first C columns of packed rows ``x``; ``w`` [taps, C]
+    (last row: the current token).  ``state`` [slots, taps - 1, C]: the inputs ahead of each
+    sequence's portion (``ctx`` > 0), replaced by its last ones."""
+    if _gpu(x):
+        return _native().causal_conv(x, w, bias, state, slots, cu, ctx, int(max_len))
+    return ref.causal_conv(x, w, bias, state, slots, cu, ctx)
+
+
+def conv_step(P, w, bias, state, slots, positions):
+    """One token a row: (silu(conv) [B, C], gate [B, C]) of an [x | z] projection; advances
+    ``state`` (rows with slot -1 leave none)."""
+    if _gpu(P):
+        return _native().conv_step(P.contiguous(), w, bias, state, slots, positions)
+    return ref.conv_step(P, w, bias, state, slots, positions)
+
+
+def scan_chunk(tokens: int, max_len: int, channels: int) -> int:
+    """Tokens per chunk of the prefill scan: chunks until the launch has ~2048 waves (64
+    channels each), never under 64 tokens -- a chunked prompt's decays are computed twice,
+    so a batch that fills the chip by itself is not cut."""
+    waves = max(1, (channels + 63) // 64)
+    n = max(1, min(2048 * max_len // max(1, waves * tokens), (max_len + 63) // 64))
+    return max(64, -(-max_len // n) if max_len else 64)
+
+
+def selective_scan(x, dt, bc, b_off: int, c_off: int, N: int, z, A2, D, dt_b, state, slots, cu, ctx, max_len: int,
+                   chunk: int = 0):
+    """Gated selective scan of packed sequences (csrc/kernels/ssm.hip): ``x`` [T, C] the
+    convolved input, ``dt`` [T, C] ahead of bias and softplus, B / C at columns ``b_off`` /
+    ``c_off`` of ``bc``, ``A2`` = -exp(A_log) log2(e) [C, Np].  Advances ``state``."""
+    if _gpu(x):
+        chunk = chunk or scan_chunk(x.shape[0], max_len, x.shape[1])
+        return _native().selective_scan(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, cu, ctx,
+                                        int(max_len), int(chunk))
+    return ref.selective_scan(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, cu, ctx)
+
+
+def selective_step(x, dt, bc, b_off: int, c_off: int, N: int, z, A2, D, dt_b, state, slots, positions):
+    """:func:`selective_scan` of one token a row."""
+    if _gpu(x):
+        return _native().selective_step(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions)
+    return ref.selective_step(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions)
+
+
+def linear(x, w, decode: bool = False):
+    """x @ w^T in x's dtype: bf16 on the decode / prefill GEMMs above, fp32 (and the CPU) by
+    the library product."""
+    if _gpu(x) and x.dtype == torch.bfloat16:
+        return decode_linear(x, w) if decode else prefill_linear(x, w)
+    return torch.nn.functional.linear(x, w)
+
+
+def project(x, w, decode: bool = False):
+    """x @ w^T for a consumer that sums split-K slabs: the slabs [S, M, N] of whichever
+    bf16 GEMM :func:`gemv_plan` / :func:`mid_plan` / :func:`decode_plan` (decode) or
+    :func:`prefill_plan` / :func:`prefill_split_plan` picks, else the product [M, N]."""
+    if not (_gpu(x) and x.dtype == torch.bfloat16):
+        return torch.nn.functional.linear(x, w)
+    N, K = w.shape
+    M = x.numel() // K
+    if decode or M <= MID_M_MAX:
+        S, R = gemv_plan(M, N, K)
+        if S:
+            return gemv_partial(x, w, S, R)
+        S, c = mid_plan(M, N, K)
+        if S:
+            return mgemm_partial(x, w, S, c, bf16=SLAB_BF16 and S > 1)
+        S, t = decode_plan(M, N, K)
+        if S:
+            return dgemm_partial(x, w, S, t)
+    else:
+        S, c = prefill_plan(M, N, K)
+        if S >= 2:
+            return mgemm_partial(x, w, S, c, bf16=SLAB_BF16)
+        if not S:
+            S = prefill_split_plan(M, N, K)
+            if S:
+                return pgemm_partial(x, w, S)
+    return linear(x, w, decode)
 
 
 # ----------------------------------------------------------------------------- search

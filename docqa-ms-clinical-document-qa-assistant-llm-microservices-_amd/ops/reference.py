@@ -339,3 +339,124 @@ def coarse_probes(xq, centroids, cnorm, nprobe: int):
     d = cnorm.float()[None, :] - 2.0 * (xq.float() @ centroids.float().t())
     order = torch.sort(d, dim=1, stable=True).indices
     return order[:, :nprobe].contiguous()
+
+
+# --------------------------------------------------- hybrid decoders (fp32 residual stream)
+def _slab_sum(P):
+    """The fp32 product of split-K slabs [S, M, N], or of the product [M, N] itself."""
+    return P.float().sum(0) if P.dim() == 3 else P.float()
+
+
+def _rms(x, eps):
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def sandwich_rmsnorm(P, residual, w_post, w_next, eps, add=None, out_dtype=None):
+    residual.add_(_rms(_slab_sum(P), eps) * w_post)
+    if add is not None:
+        residual.add_(add)
+    return (_rms(residual, eps) * w_next).to(out_dtype or residual.dtype)
+
+
+def embed_scale_rmsnorm(ids, table, scale, w, eps, keep):
+    h = table[ids.long()].float() * scale
+    return h, (h.clone() if keep else None), (_rms(h, eps) * w).to(table.dtype)
+
+
+def squared_relu(P, out_dtype):
+    return _slab_sum(P).clamp(min=0).square().to(out_dtype)
+
+
+def qk_norm_store(P, w, slots, k_cache, k_scale, H, eps):
+    x = _slab_sum(P)
+    T = x.shape[0]
+    NB, G, BS, D = k_cache.shape
+    q = (_rms(x[:, :H * D].view(T, H, D), eps) * w).to(k_cache.dtype).reshape(T, H * D)
+    k = x[:, H * D:(H + G) * D].reshape(T, G, D).to(k_cache.dtype)
+    sm = slots.long()
+    ok = sm >= 0
+    blk, off = sm[ok] // BS, sm[ok] % BS
+    k_cache[blk, :, off] = k[ok]
+    k_scale.view(NB, G, BS)[blk, :, off] = torch.rsqrt(k[ok].float().pow(2).mean(-1) + eps)
+    return q
+
+
+def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink):
+    NB, G, BS, D = k_cache.shape
+    H = q.shape[1] // D
+    v_cache = k_cache if v_cache is None else v_cache
+    out = torch.zeros_like(q)
+    for b in range(block_tables.shape[0]):
+        q0, L, p0 = (b, 1, int(ctx[b]) - 1) if cu is None else (int(cu[b]), int(cu[b + 1] - cu[b]), int(ctx[b]))
+        if L <= 0 or p0 < 0:
+            continue
+        n = p0 + L
+        lo = max(0, p0 - window + 1) if window > 0 else 0
+        pos = torch.arange(lo, n, device=q.device)
+        blk, off = block_tables[b, (pos // BS)].long(), pos % BS
+        k = k_cache[blk, :, off].float().transpose(0, 1)                # [G, keys, D]
+        v = v_cache[blk, :, off].float().transpose(0, 1)
+        qb = q[q0:q0 + L].view(L, G, H // G, D).float().permute(1, 2, 0, 3)
+        s = torch.einsum("ghld,gkd->ghlk", qb, k) * scale
+        if k_scale is not None:
+            s = s * k_scale.view(NB, G, BS)[blk, :, off].t()[:, None, None, :]
+        i = torch.arange(p0, n, device=q.device)[:, None]
+        dead = pos[None, :] > i
+        if window > 0:
+            dead = dead | (pos[None, :] <= i - window)
+        s = s.masked_fill(dead, -math.inf)
+        if sink is not None:
+            s = torch.cat([s, sink.float().view(G, H // G, 1, 1).expand(G, H // G, L, 1)], -1)
+        p = torch.softmax(s, -1)[..., :n - lo]
+        o = torch.einsum("ghlk,gkd->ghld", p, v)
+        out[q0:q0 + L] = o.permute(2, 0, 1, 3).reshape(L, H * D).to(q.dtype)
+    return out
+
+
+def causal_conv(x, w, bias, state, slots, cu, ctx):
+    taps, C = w.shape
+    y = torch.empty(x.shape[0], C, dtype=x.dtype, device=x.device)
+    for b in range(cu.numel() - 1):
+        q0, q1, slot = int(cu[b]), int(cu[b + 1]), int(slots[b])
+        if q1 <= q0:
+            continue
+        head = (state[slot] if slot >= 0 and int(ctx[b]) > 0
+                else torch.zeros(taps - 1, C, dtype=x.dtype, device=x.device))
+        seq = torch.cat([head, x[q0:q1, :C]])
+        acc = bias.expand(q1 - q0, C).clone()
+        for k in range(taps):
+            acc += w[k] * seq[k:k + q1 - q0].float()
+        y[q0:q1] = F.silu(acc).to(x.dtype)
+        if slot >= 0 and taps > 1:
+            state[slot] = seq[-(taps - 1):]
+    return y
+
+
+def conv_step(P, w, bias, state, slots, positions):
+    C = w.shape[1]
+    B = P.shape[-2]
+    xz = _slab_sum(P).to(state.dtype)
+    cu = torch.arange(B + 1, dtype=torch.int32)
+    return causal_conv(xz[:, :C], w, bias, state, slots, cu, positions), xz[:, C:].contiguous()
+
+
+def selective_scan(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, cu, ctx):
+    C, Np = A2.shape
+    y = torch.empty_like(x)
+    d = F.softplus(dt.float() + dt_b)
+    xf = x.float()
+    Bv, Cv = F.pad(bc[:, b_off:b_off + N].float(), (0, Np - N)), F.pad(bc[:, c_off:c_off + N].float(), (0, Np - N))
+    for b in range(cu.numel() - 1):
+        q0, q1, slot = int(cu[b]), int(cu[b + 1]), int(slots[b])
+        S = (state[slot].clone() if slot >= 0 and int(ctx[b]) > 0 else torch.zeros(C, Np, device=x.device))
+        for t in range(q0, q1):
+            S = torch.exp2(d[t][:, None] * A2) * S + (d[t] * xf[t])[:, None] * Bv[t]
+            y[t] = ((S @ Cv[t] + D * xf[t]) * F.silu(z[t, :C].float())).to(x.dtype)
+        if slot >= 0 and q1 > q0:
+            state[slot] = S
+    return y
+
+
+def selective_step(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions):
+    cu = torch.arange(x.shape[0] + 1, dtype=torch.int32)
+    return selective_scan(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, cu, positions)

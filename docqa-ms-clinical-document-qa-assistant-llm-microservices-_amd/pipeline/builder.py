@@ -38,7 +38,7 @@ def build_stack(sc: StackConfig, device="cuda", log=print) -> tuple[RAGPipeline,
     s = comm.state()
     # names are presets (random-init weights) or Hugging Face checkpoint directories
     ck.use_checkpoint_tokenizers(sc.llm, sc.embed)
-    llm_cfg = ck.resolve_llama_config(sc.llm)
+    llm_cfg = ck.resolve_decoder_config(sc.llm)
     enc_tok = WordPieceTokenizer()
     chat_tok = ChatTokenizer(model_vocab=llm_cfg.vocab_size)
     encoder = ck.resolve_bert(sc.embed, device=device, seed=sc.seed)
@@ -59,7 +59,7 @@ def build_stack(sc: StackConfig, device="cuda", log=print) -> tuple[RAGPipeline,
         torch.cuda.synchronize()
     info["index_build_s"] = time.perf_counter() - t0
     info["index_vectors"] = n
-    model = ck.resolve_llama(sc.llm, device=device, seed=sc.seed)
+    model = ck.resolve_decoder(sc.llm, device=device, seed=sc.seed)
     engine = LLMEngine(model, max_batch=sc.max_batch, max_context=sc.max_context,
                        use_graphs=sc.use_graphs, kv_mem_fraction=sc.kv_mem_fraction)
     info["kv_blocks"] = engine.kv.allocator.num_blocks if hasattr(engine.kv.allocator, "num_blocks") else None

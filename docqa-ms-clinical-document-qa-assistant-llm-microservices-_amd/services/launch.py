@@ -157,7 +157,7 @@ def run_parallel(a, opts: "StackOptions") -> None:
 
         signal.signal(signal.SIGINT, signal.SIG_IGN)
         ck.use_checkpoint_tokenizers(opts.llm, opts.embed)
-        model = ck.resolve_llama(opts.llm, device=opts.device)
+        model = ck.resolve_decoder(opts.llm, device=opts.device)
         ctx = min(opts.max_context or st.max_context, model.cfg.max_position)
         eng = LLMEngine(model, max_batch=opts.max_batch, max_context=ctx, use_graphs=opts.use_graphs,
                         kv_mem_fraction=opts.kv_mem_fraction)

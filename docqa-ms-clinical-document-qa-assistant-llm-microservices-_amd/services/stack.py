@@ -106,7 +106,7 @@ class DocQAStack:
         self.db = docs_db.DocsDB(self.st.database_url) if svc & {"ingest", "indexer"} else None
         ck.use_checkpoint_tokenizers(opts.llm, opts.embed)
         self.enc_tok = WordPieceTokenizer()
-        llm_cfg = ck.resolve_llama_config(opts.llm)
+        llm_cfg = ck.resolve_decoder_config(opts.llm)
         self.chat_tok = ChatTokenizer(model_vocab=llm_cfg.vocab_size)
         self.encoder = ck.resolve_bert(opts.embed, device=dev) if svc & {"indexer", "qa"} else None
         self.deid = self.indexer = self.follower = self.engine = self.pipeline = None
@@ -142,7 +142,7 @@ class DocQAStack:
                 self.follower = IndexFollower(self.st.index_dir, self.st.index_file, self.st.metadata_file,
                                               d=self.encoder.cfg.hidden, device=dev, settings=self.st).start()
                 index, metadata = self.follower.index, self.follower.metadata
-            self.model = ck.resolve_llama(opts.llm, device=dev)
+            self.model = ck.resolve_decoder(opts.llm, device=dev)
             ctx = min(opts.max_context or self.st.max_context, self.model.cfg.max_position)
             self.engine = LLMEngine(self.model, max_batch=opts.max_batch, max_context=ctx,
                                     use_graphs=opts.use_graphs, kv_mem_fraction=opts.kv_mem_fraction)
