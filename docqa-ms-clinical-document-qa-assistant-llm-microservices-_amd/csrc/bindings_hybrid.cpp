@@ -141,7 +141,7 @@ Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, 
   if (k_scale.has_value()) check_vec(*k_scale, k_cache.numel() / D, "k_scale");
   if (sink.has_value()) check_vec(*sink, H, "sink");
   c10::DeviceGuard g(q.device());
-  CHECK_ALIGN16(q); CHECK_ALIGN16(k_cache);
+  CHECK_ALIGN16(k_cache);     // cached rows are read in 16-byte pieces, q row by row
   auto out = at::empty_like(q);
   CHECK_RC(docqa_window_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.has_value() ? v_cache->data_ptr() : k_cache.data_ptr(),
                              k_scale.has_value() ? k_scale->data_ptr<float>() : nullptr, block_tables.data_ptr<int>(),

@@ -133,7 +133,8 @@ __device__ __forceinline__ void better(float& bv, int& bi, float v, int i) {
   if (v > bv || (v == bv && i < bi)) { bv = v; bi = i; }
 }
 
-template <bool BF16>
+// VEC: rows and base are 16-byte aligned (any V: the last chunk's rest is read one by one)
+template <bool BF16, bool VEC>
 __global__ __launch_bounds__(256) void argmax_pass1(const void* __restrict__ logits, int V,
                                                     int ld, int splits, float* __restrict__ pv,
                                                     int* __restrict__ pi) {
@@ -142,9 +143,14 @@ __global__ __launch_bounds__(256) void argmax_pass1(const void* __restrict__ log
   const int lo = sp * chunk, hi = min(V, lo + chunk);
   float bv = -FLT_MAX;
   int bi = 0x7fffffff;
-  if constexpr (BF16) {
+  if constexpr (!VEC) {
+    const size_t r0 = (size_t)row * ld;
+    for (int i = lo + threadIdx.x; i < hi; i += 256)
+      better(bv, bi, BF16 ? bf2f(reinterpret_cast<const uint16_t*>(logits)[r0 + i])
+                          : reinterpret_cast<const float*>(logits)[r0 + i], i);
+  } else if constexpr (BF16) {
     const uint16_t* r = reinterpret_cast<const uint16_t*>(logits) + (size_t)row * ld;
-    // vector body (ld and lo are multiples of 8 when V % 8 == 0)
+    // vector body (ld and lo are multiples of 8)
     int i = lo + threadIdx.x * 8;
     for (; i + 8 <= hi; i += 256 * 8) {
       float f[8];
@@ -348,12 +354,12 @@ int docqa_bert_embed_ln(const int* ids, const int* pos, const int* tt, const voi
 int docqa_argmax(const void* logits, int rows, int V, int ld, int is_bf16, float* ws_v, int* ws_i,
                  int splits, int64_t* out, hipStream_t s) {
   if (rows == 0) return 0;
-  if (is_bf16 && (V % 8 != 0 || ld % 8 != 0)) return -1;
-  if (!is_bf16 && (ld % 4 != 0)) return -1;
-  if (!docqa_aligned16(logits)) return -1;
+  const bool vec = ld % (is_bf16 ? 8 : 4) == 0 && docqa_aligned16(logits);
   dim3 g1(splits, rows);
-  if (is_bf16) argmax_pass1<true><<<g1, 256, 0, s>>>(logits, V, ld, splits, ws_v, ws_i);
-  else argmax_pass1<false><<<g1, 256, 0, s>>>(logits, V, ld, splits, ws_v, ws_i);
+  if (is_bf16 && vec) argmax_pass1<true, true><<<g1, 256, 0, s>>>(logits, V, ld, splits, ws_v, ws_i);
+  else if (is_bf16) argmax_pass1<true, false><<<g1, 256, 0, s>>>(logits, V, ld, splits, ws_v, ws_i);
+  else if (vec) argmax_pass1<false, true><<<g1, 256, 0, s>>>(logits, V, ld, splits, ws_v, ws_i);
+  else argmax_pass1<false, false><<<g1, 256, 0, s>>>(logits, V, ld, splits, ws_v, ws_i);
   argmax_pass2<<<rows, 64, 0, s>>>(ws_v, ws_i, splits, out);
   DOCQA_CHECK_LAUNCH();
   return 0;
