@@ -99,6 +99,34 @@ Tensor squared_relu(const Tensor& P, bool out_f32) {
   return out;
 }
 
+// squared ReLU of x . w^T on the decode GEMMs: skinny up to 192 rows, the mid-M kernel beyond
+Tensor decode_relu2(const Tensor& x, const Tensor& w) {
+  CHECK_GPU(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_CONTIG(x); CHECK_CONTIG(w); CHECK_ALIGN16(x); CHECK_ALIGN16(w);
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1), "decode_relu2: shapes");
+  const int M = x.size(0), N = w.size(0), K = x.size(1);
+  c10::DeviceGuard g(x.device());
+  auto out = at::empty({M, N}, x.options());
+  CHECK_RC(M <= 192 && N % 64 == 0 && K % 512 == 0
+               ? docqa_dgemm_relu2(x.data_ptr(), w.data_ptr(), out.data_ptr(), M, N, K, stream())
+               : docqa_mgemm_relu2(x.data_ptr(), w.data_ptr(), out.data_ptr(), M, N, K, stream()),
+           "decode_relu2");
+  return out;
+}
+
+// columns [0, n0) and [n0, n0 + n1) of a projection (product or slabs) as two tensors
+std::tuple<Tensor, Tensor> slab_columns(const Tensor& P, int64_t n0, int64_t n1, bool out_f32) {
+  const Slabs p = slabs_of(P);
+  CHECK_ALIGN16(P);
+  TORCH_CHECK(n0 >= 0 && n1 >= 0 && n0 % 4 == 0 && n1 % 4 == 0 && p.N % 4 == 0 && n0 + n1 <= p.N, "slab_columns: columns");
+  c10::DeviceGuard g(P.device());
+  auto opt = P.options().dtype(out_f32 ? at::kFloat : at::kBFloat16);
+  auto a = at::empty({p.M, n0}, opt), b = at::empty({p.M, n1}, opt);
+  CHECK_RC(docqa_slab_columns(P.data_ptr(), is_f32(P), p.S, p.M, p.N, a.data_ptr(), (int)n0, b.data_ptr(), (int)n1,
+                              out_f32, stream()),
+           "slab_columns");
+  return {a, b};
+}
+
 Tensor qk_norm_store(const Tensor& P, const Tensor& w, const Tensor& slots, Tensor k_cache, Tensor k_scale, int64_t H,
                      double eps) {
   const Slabs p = slabs_of(P);
@@ -269,6 +297,8 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
         "bool out_f32) -> Tensor");
   m.def("embed_scale_rmsnorm(Tensor ids, Tensor table, float scale, Tensor w, float eps, bool keep) "
         "-> (Tensor, Tensor, Tensor)");
+  m.def("decode_relu2(Tensor x, Tensor w) -> Tensor");
+  m.def("slab_columns(Tensor P, int n0, int n1, bool out_f32) -> (Tensor, Tensor)");
   m.def("squared_relu(Tensor P, bool out_f32) -> Tensor");
   m.def("qk_norm_store(Tensor P, Tensor w, Tensor slots, Tensor(a!) k_cache, Tensor(b!) k_scale, int H, float eps) "
         "-> Tensor");
@@ -287,6 +317,8 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
 TORCH_LIBRARY_IMPL(docqa, CUDA, m) {
   m.impl("sandwich_rmsnorm", &sandwich_rmsnorm);
   m.impl("embed_scale_rmsnorm", &embed_scale_rmsnorm);
+  m.impl("decode_relu2", &decode_relu2);
+  m.impl("slab_columns", &slab_columns);
   m.impl("squared_relu", &squared_relu);
   m.impl("qk_norm_store", &qk_norm_store);
   m.impl("window_attn", &window_attn);

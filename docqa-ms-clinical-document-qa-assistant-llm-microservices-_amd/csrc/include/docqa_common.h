@@ -46,6 +46,12 @@ __device__ __forceinline__ uint4 pack8(const float* f) {
   return v;
 }
 
+// squared ReLU (GEMM epilogues and act.hip)
+__device__ __forceinline__ float relu2(float v) {
+  const float r = fmaxf(v, 0.f);
+  return r * r;
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);

@@ -12,6 +12,12 @@ int docqa_sandwich_rmsnorm(const void* P, int p_f32, int S, float* res, const fl
                            const float* w_next, void* out, int out_f32, int rows, int H, float eps, hipStream_t s);
 int docqa_embed_scale_rmsnorm(const int* ids, const void* table, int f32, float scale, const float* w, float* res,
                               float* emb, void* out, int rows, int H, int vocab, float eps, hipStream_t s);
+// Y [M, N] = squared ReLU of X [M, K] . W [N, K]^T, bf16 (dgemm.hip: M <= 192, N % 64, K % 512;
+// mgemm.hip: N % 128, K % 128)
+int docqa_dgemm_relu2(const void* X, const void* W, void* Y, int M, int N, int K, hipStream_t s);
+int docqa_mgemm_relu2(const void* X, const void* W, void* Y, int M, int N, int K, hipStream_t s);
+int docqa_slab_columns(const void* P, int p_f32, int S, int T, int ld, void* out0, int n0, void* out1, int n1,
+                       int out_f32, hipStream_t s);
 int docqa_squared_relu(const void* P, int p_f32, int S, size_t n, void* out, int out_f32, hipStream_t s);
 
 int docqa_qk_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* wq, const int* slots,

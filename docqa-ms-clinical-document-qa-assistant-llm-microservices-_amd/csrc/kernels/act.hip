@@ -216,12 +216,46 @@ __global__ __launch_bounds__(256) void squared_relu_kernel(const PT* __restrict_
     float f[V];
     ld_slabs<V>(P + i, S, n, f);
 #pragma unroll
-    for (int j = 0; j < V; ++j) {
-      const float r = fmaxf(f[j], 0.f);
-      f[j] = r * r;
-    }
+    for (int j = 0; j < V; ++j) f[j] = relu2(f[j]);
     stv<V>(out + i, f);
   }
+}
+
+// columns [0, n0) and [n0, n0 + n1) of a projection given as S split-K slabs [S, T, ld] (or its
+// product), as two matrices of their own: out0 [T, n0], out1 [T, n1] (V | n0, n1, ld)
+template <int V, typename PT, typename OT>
+__global__ __launch_bounds__(256) void slab_columns_kernel(const PT* __restrict__ P, int S, size_t slab, int T, int ld,
+                                                           OT* __restrict__ out0, int n0, OT* __restrict__ out1,
+                                                           int n1) {
+  const int cpr = (n0 + n1) / V, total = T * cpr;
+  for (int i = blockIdx.x * 256 + threadIdx.x; i < total; i += gridDim.x * 256) {
+    const int t = i / cpr, c = (i - t * cpr) * V;
+    float f[V];
+    ld_slabs<V>(P + (size_t)t * ld + c, S, slab, f);
+    if (c < n0) stv<V>(out0 + (size_t)t * n0 + c, f);
+    else stv<V>(out1 + (size_t)t * n1 + (c - n0), f);
+  }
+}
+
+template <typename PT, typename OT>
+static int launch_slab_columns(const PT* P, int S, int T, int ld, OT* out0, int n0, OT* out1, int n1, hipStream_t s) {
+  const long long total = (long long)T * ((n0 + n1) / 4);
+  if (total >= (1ll << 31)) return -1;
+  const long long g = (total + 255) / 256;
+  slab_columns_kernel<4, PT, OT><<<(int)(g < 4096 ? g : 4096), 256, 0, s>>>(P, S, (size_t)T * ld, T, ld, out0, n0, out1, n1);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+int docqa_slab_columns(const void* P, int p_f32, int S, int T, int ld, void* out0, int n0, void* out1, int n1,
+                       int out_f32, hipStream_t s) {
+  if (T == 0) return 0;
+  if (S < 1 || n0 % 4 || n1 % 4 || ld % 4 || n0 + n1 > ld) return -1;
+  if (p_f32)
+    return out_f32 ? launch_slab_columns((const float*)P, S, T, ld, (float*)out0, n0, (float*)out1, n1, s)
+                   : launch_slab_columns((const float*)P, S, T, ld, (uint16_t*)out0, n0, (uint16_t*)out1, n1, s);
+  return out_f32 ? launch_slab_columns((const uint16_t*)P, S, T, ld, (float*)out0, n0, (float*)out1, n1, s)
+                 : launch_slab_columns((const uint16_t*)P, S, T, ld, (uint16_t*)out0, n0, (uint16_t*)out1, n1, s);
 }
 
 template <typename PT, typename OT>

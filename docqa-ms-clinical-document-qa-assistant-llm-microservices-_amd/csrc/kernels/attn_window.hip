@@ -9,7 +9,8 @@
 //   w the normalised key is never materialised: one cached row serves as key and as value,
 //   half the bytes of a K / V pair.
 // * window <= 0: no window; sink null: none; k_scale null: 1; V may be the K cache itself.
-// * prefill (several query tokens a sequence) and decode (one) share the kernels.
+// * prefill (several query tokens a sequence) and decode (one) share the kernels: bf16 heads of
+//   up to 256 elements run on MFMA, fp32 and odd head sizes on a wave-per-row kernel.
 #include "docqa_common.h"
 #include "docqa_elem.h"
 #include <float.h>
@@ -186,6 +187,330 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
   }
 }
 
+// ---- MFMA form (bf16, head sizes that are multiples of 8) ---------------------------------
+// Query rows are (token, head of the GQA group) pairs, so any group size fills the 16-row MFMA
+// tiles.  S^T = K Q^T on v_mfma_f32_16x16x32_bf16: a lane holds one query row's scores of
+// 4 keys per 16-key sub-tile, so the online softmax is in-lane plus two cross-group shuffles,
+// and the scores turned bf16 are the B operand of O^T += V^T P^T as they are (the key order of
+// a k-step is the accumulators': keys 4g..4g+3 of two sub-tiles for lane group g).  V^T comes
+// from the row-major tile by transposing LDS reads -- from the K tile itself when the keys are
+// the values.  Tile rows are padded by 16 bytes: conflict-free for both read patterns.
+//   SPLIT = false: 4 waves, each 16 QT rows of its own, one double-buffered K (V) tile for all;
+//   SPLIT = true (few rows, decode): NW waves take every NW-th key tile of the same rows, each
+//   with a private LDS tile, and merge at the end.
+typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
+
+template <int DP, int QT, int KB, int NW, bool SHARED, bool SPLIT>
+__global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_t* __restrict__ q,
+                                                                   const uint16_t* __restrict__ kc,
+                                                                   const uint16_t* __restrict__ vc,
+                                                                   uint16_t* __restrict__ out, WindowArgs a) {
+  constexpr int PITCH = DP + 8, NCH = DP / 8, NKT = KB / 16, NKS = DP / 32, NDT = DP / 16;
+  constexpr int TILES = SPLIT ? NW : 2, NT = SHARED ? 1 : 2;
+  constexpr int TILE = KB * PITCH;                                  // elements of one tile
+  constexpr int LOADERS = SPLIT ? 64 : 64 * NW;                     // threads staging one tile
+  constexpr int CPT = (KB * NCH + LOADERS - 1) / LOADERS;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  uint16_t* tiles = reinterpret_cast<uint16_t*>(smem);
+  float* scales = reinterpret_cast<float*>(tiles + TILES * NT * TILE);   // [TILES][KB]
+
+  const int kvh = blockIdx.x, b = blockIdx.y;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int fr = lane & 15, g4 = lane >> 4;
+  int q0 = 0, L = 0, p0 = 0;
+  const bool live = seq_range(a, b, q0, L, p0);
+  const int Gs = a.H / a.G, D = a.D;
+  constexpr int RW = 16 * QT;
+  const int tile_rows = SPLIT ? RW : RW * NW;
+  const int row0 = (gridDim.z - 1 - blockIdx.z) * tile_rows;         // longest windows first
+  if (!live) {                                                       // a padded decode row
+    if (!a.cu)
+      for (int e = tid; e < Gs * D; e += 64 * NW) out[((size_t)b * a.H + kvh * Gs) * D + e] = 0;
+    return;
+  }
+  const int rows = L * Gs;
+  if (row0 >= rows) return;
+  const int wrow = row0 + (SPLIT ? 0 : wave * RW);                   // first row of this wave
+  // positions the workgroup's rows / this wave's rows span
+  const int pos_lo = p0 + row0 / Gs, pos_hi = p0 + (min(row0 + tile_rows, rows) - 1) / Gs;
+  const int wpos_lo = p0 + min(wrow, rows - 1) / Gs, wpos_hi = p0 + (min(wrow + RW, rows) - 1) / Gs;
+  const bool wlive = wrow < rows;
+  const int key0 = a.window > 0 ? max(0, pos_lo - a.window + 1) : 0;
+  const int ntiles = (pos_hi - key0) / KB + 1;
+
+  bf16x8 qf[QT][NKS];
+  int pos[QT];
+  float m[QT], l[QT];
+  f32x4 o[QT][NDT];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    const int r = wrow + t * 16 + fr, rc = min(r, rows - 1);
+    const int tok = rc / Gs, h = kvh * Gs + rc % Gs;
+    pos[t] = p0 + tok;
+    const uint16_t* qp = q + ((size_t)(q0 + tok) * a.H + h) * D;
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks) {
+      const int c = ks * 32 + g4 * 8;
+      uint4 v = c < D ? *reinterpret_cast<const uint4*>(qp + c) : make_uint4(0, 0, 0, 0);
+      qf[t][ks] = *reinterpret_cast<bf16x8*>(&v);
+    }
+    // the sink: one more exponential in the denominator (in one wave only when they split)
+    const bool sk = a.sink && (!SPLIT || wave == 0);
+    m[t] = sk ? a.sink[h] * kLog2e : -1e30f;
+    l[t] = sk ? 1.f : 0.f;
+#pragma unroll
+    for (int i = 0; i < NDT; ++i) o[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  const float sl2 = a.scale * kLog2e;
+
+  const int ltid = SPLIT ? lane : tid;
+  uint4 rk[CPT], rv[SHARED ? 1 : CPT];
+  float rs_ = 1.f;
+  auto cache_row = [&](int key) {
+    const int blk = a.block_tables[(size_t)b * a.maxb + key / a.BS];
+    return ((size_t)blk * a.G + kvh) * a.BS + key % a.BS;
+  };
+  auto load = [&](int t) {
+    const int kb = key0 + t * KB;
+#pragma unroll
+    for (int i = 0; i < CPT; ++i) {
+      const int e = ltid + LOADERS * i, row = e / NCH, c = (e % NCH) * 8;
+      rk[i] = make_uint4(0, 0, 0, 0);
+      if constexpr (!SHARED) rv[i] = make_uint4(0, 0, 0, 0);
+      if (e < KB * NCH && kb + row <= pos_hi && c < D) {
+        const size_t off = cache_row(kb + row) * D + c;
+        rk[i] = *reinterpret_cast<const uint4*>(kc + off);
+        if constexpr (!SHARED) rv[i] = *reinterpret_cast<const uint4*>(vc + off);
+      }
+    }
+    if (ltid < KB) {
+      const int key = kb + ltid;
+      rs_ = (a.k_scale && key <= pos_hi) ? a.k_scale[cache_row(key)] * sl2 : sl2;
+    }
+  };
+  auto store = [&](int buf) {
+    uint16_t* k = tiles + buf * NT * TILE;
+#pragma unroll
+    for (int i = 0; i < CPT; ++i) {
+      const int e = ltid + LOADERS * i, row = e / NCH, c = (e % NCH) * 8;
+      if (e < KB * NCH) {
+        *reinterpret_cast<uint4*>(k + row * PITCH + c) = rk[i];
+        if constexpr (!SHARED) *reinterpret_cast<uint4*>(k + TILE + row * PITCH + c) = rv[i];
+      }
+    }
+    if (ltid < KB) scales[buf * KB + ltid] = rs_;
+  };
+  auto compute = [&](int t, int buf) {
+    const int kb = key0 + t * KB;
+    if (!wlive || kb > wpos_hi || (a.window > 0 && kb + KB - 1 <= wpos_lo - a.window)) return;
+    const bool whole = kb + KB - 1 <= wpos_lo && (a.window <= 0 || kb > wpos_hi - a.window);
+    const uint16_t* sk = tiles + buf * NT * TILE;
+    const uint16_t* sv = SHARED ? sk : sk + TILE;
+    const float* sc = scales + buf * KB;
+    f32x4 x[QT][NKT];
+#pragma unroll
+    for (int kt = 0; kt < NKT; ++kt) {
+#pragma unroll
+      for (int t2 = 0; t2 < QT; ++t2) x[t2][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < NKS; ++ks) {
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(sk + (kt * 16 + fr) * PITCH + ks * 32 + g4 * 8);
+#pragma unroll
+        for (int t2 = 0; t2 < QT; ++t2)
+          x[t2][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[t2][ks], x[t2][kt], 0, 0, 0);
+      }
+    }
+#pragma unroll
+    for (int t2 = 0; t2 < QT; ++t2) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int kt = 0; kt < NKT; ++kt) {
+        const float4 ks4 = *reinterpret_cast<const float4*>(sc + kt * 16 + g4 * 4);
+        const float kss[4] = {ks4.x, ks4.y, ks4.z, ks4.w};
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          float v = x[t2][kt][r] * kss[r];
+          if (!whole) {
+            const int key = kb + kt * 16 + g4 * 4 + r;
+            if (key > pos[t2] || (a.window > 0 && key <= pos[t2] - a.window)) v = -INFINITY;
+          }
+          x[t2][kt][r] = v;
+          mx = fmaxf(mx, v);
+        }
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m[t2], mx);
+      const float alpha = __builtin_amdgcn_exp2f(m[t2] - mn);
+      float rs = 0.f;
+#pragma unroll
+      for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float p = __builtin_amdgcn_exp2f(x[t2][kt][r] - mn);
+          x[t2][kt][r] = p;
+          rs += p;
+        }
+      rs += __shfl_xor(rs, 16, 64);
+      rs += __shfl_xor(rs, 32, 64);
+      l[t2] = l[t2] * alpha + rs;
+      m[t2] = mn;
+#pragma unroll
+      for (int i = 0; i < NDT; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[t2][i][r] *= alpha;
+    }
+    const int tq = fr >> 2, tp = fr & 3;
+#pragma unroll
+    for (int s = 0; s < NKT / 2; ++s) {
+      bf16x8 pb[QT];
+#pragma unroll
+      for (int t2 = 0; t2 < QT; ++t2)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          pb[t2][j] = (__bf16)x[t2][2 * s][j];
+          pb[t2][4 + j] = (__bf16)x[t2][2 * s + 1][j];
+        }
+      const uint16_t* vr = sv + (s * 32 + g4 * 4 + tq) * PITCH + 4 * tp;
+#pragma unroll
+      for (int i = 0; i < NDT; ++i) {
+        const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + i * 16));
+        const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 16 * PITCH + i * 16));
+        bf16x8 vf;
+        const __bf16* lp = reinterpret_cast<const __bf16*>(&lo);
+        const __bf16* hp = reinterpret_cast<const __bf16*>(&hi);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { vf[j] = lp[j]; vf[4 + j] = hp[j]; }
+#pragma unroll
+        for (int t2 = 0; t2 < QT; ++t2)
+          o[t2][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pb[t2], o[t2][i], 0, 0, 0);
+      }
+    }
+  };
+
+  if constexpr (!SPLIT) {
+    load(0);
+    store(0);
+    __syncthreads();
+    for (int t = 0; t < ntiles; ++t) {
+      if (t + 1 < ntiles) load(t + 1);
+      compute(t, t & 1);
+      if (t + 1 < ntiles) store((t + 1) & 1);    // last read one iteration (one barrier) ago
+      __syncthreads();
+    }
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+      const int r = wrow + t * 16 + fr;
+      if (r >= rows) continue;
+      uint16_t* op = out + ((size_t)(q0 + r / Gs) * a.H + kvh * Gs + r % Gs) * D;
+      const float inv = 1.f / l[t];
+#pragma unroll
+      for (int i = 0; i < NDT; ++i) {
+        const int c = i * 16 + g4 * 4;
+        if (c < D) {
+          uint2 v;
+          v.x = pack2(o[t][i][0] * inv, o[t][i][1] * inv);
+          v.y = pack2(o[t][i][2] * inv, o[t][i][3] * inv);
+          *reinterpret_cast<uint2*>(op + c) = v;
+        }
+      }
+    }
+  } else {
+    static_assert(QT == 1 || !SPLIT, "split rows: one 16-row tile");
+    if (wave < ntiles) load(wave);
+    for (int t = wave; t < ntiles; t += NW) {
+      wave_lds_sync();                           // this wave's reads of the tile are done
+      store(wave);
+      wave_lds_sync();
+      if (t + NW < ntiles) load(t + NW);
+      compute(t, wave);
+    }
+    __syncthreads();                             // tiles dead: partials [NW][16][DP] + (m, l)
+    constexpr int OP = DP + 4;
+    float* po = reinterpret_cast<float*>(smem);
+    float2* pml = reinterpret_cast<float2*>(po + NW * 16 * OP);
+#pragma unroll
+    for (int i = 0; i < NDT; ++i)
+      *reinterpret_cast<float4*>(po + (wave * 16 + fr) * OP + i * 16 + g4 * 4) =
+          make_float4(o[0][i][0], o[0][i][1], o[0][i][2], o[0][i][3]);
+    if (g4 == 0) pml[wave * 16 + fr] = make_float2(m[0], l[0]);
+    __syncthreads();
+    const int n = min(16, rows - row0);
+    for (int e = tid; e < n * (DP / 4); e += 64 * NW) {
+      const int r = e / (DP / 4), c = (e % (DP / 4)) * 4;
+      if (c >= D) continue;
+      float mm = -1e30f;
+#pragma unroll
+      for (int w = 0; w < NW; ++w) mm = fmaxf(mm, pml[w * 16 + r].x);
+      float ll = 0.f;
+      float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+      for (int w = 0; w < NW; ++w) {
+        const float2 ml = pml[w * 16 + r];
+        const float f = __builtin_amdgcn_exp2f(ml.x - mm);
+        const float4 p = *reinterpret_cast<const float4*>(po + (w * 16 + r) * OP + c);
+        ll += ml.y * f;
+        v.x += p.x * f; v.y += p.y * f; v.z += p.z * f; v.w += p.w * f;
+      }
+      const float inv = 1.f / ll;
+      uint2 w2;
+      w2.x = pack2(v.x * inv, v.y * inv);
+      w2.y = pack2(v.z * inv, v.w * inv);
+      const int row = row0 + r;
+      *reinterpret_cast<uint2*>(out + ((size_t)(q0 + row / Gs) * a.H + kvh * Gs + row % Gs) * D + c) = w2;
+    }
+  }
+}
+
+template <int DP, int QT, int KB, int NW, bool SHARED, bool SPLIT>
+int launch_mfma(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
+                hipStream_t s) {
+  constexpr int TILES = SPLIT ? NW : 2, NT = SHARED ? 1 : 2;
+  constexpr size_t tile_b = (size_t)TILES * NT * KB * (DP + 8) * 2 + (size_t)TILES * KB * 4;
+  constexpr size_t merge_b = SPLIT ? (size_t)NW * 16 * (DP + 4) * 4 + (size_t)NW * 16 * 8 : 0;
+  constexpr size_t lds = tile_b > merge_b ? tile_b : merge_b;
+  static_assert(lds <= 160 * 1024, "LDS");
+  const int tile_rows = 16 * QT * (SPLIT ? 1 : NW), Gs = a.H / a.G;
+  const long long nz = ((long long)max_q * Gs + tile_rows - 1) / tile_rows;
+  if (nz > 65535) return -1;
+  auto kern = window_attn_mfma_kernel<DP, QT, KB, NW, SHARED, SPLIT>;
+  if constexpr (lds > 64 * 1024) {
+    static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
+                                                    hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return (int)e;
+  }
+  kern<<<dim3(a.G, B, (int)nz), 64 * NW, lds, s>>>((const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc,
+                                                   (uint16_t*)out, a);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+// decode-like launches (the rows of one sequence fit one 16-row tile): waves split the keys;
+// 16 of them when there are too few workgroups to fill the chip
+template <int DP, bool SHARED>
+int dispatch_mfma(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
+                  hipStream_t s) {
+  constexpr int QT = DP <= 128 ? 2 : 1;
+  if (max_q * (a.H / a.G) <= 16) {
+    if constexpr (DP <= 128) {
+      if ((long long)B * a.G <= 128) return launch_mfma<DP, 1, 32, SHARED ? 16 : 8, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+    }
+    return launch_mfma<DP, 1, 32, 4, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+  }
+  return launch_mfma<DP, QT, 64, 4, SHARED, false>(q, kc, vc, out, a, B, max_q, s);
+}
+
+template <bool SHARED>
+int dispatch_dim(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
+                 hipStream_t s) {
+  if (a.D <= 32) return dispatch_mfma<32, SHARED>(q, kc, vc, out, a, B, max_q, s);
+  if (a.D <= 64) return dispatch_mfma<64, SHARED>(q, kc, vc, out, a, B, max_q, s);
+  if (a.D <= 96) return dispatch_mfma<96, SHARED>(q, kc, vc, out, a, B, max_q, s);
+  if (a.D <= 128) return dispatch_mfma<128, SHARED>(q, kc, vc, out, a, B, max_q, s);
+  if (a.D <= 192) return dispatch_mfma<192, SHARED>(q, kc, vc, out, a, B, max_q, s);
+  return dispatch_mfma<256, SHARED>(q, kc, vc, out, a, B, max_q, s);
+}
+
 template <typename PT, typename T>
 int qk_store(const PT* P, int S, size_t slab, int ld, const float* wq, const int* sm, T* q, T* kc, float* ks,
              int tokens, int H, int G, int D, int BS, float eps, hipStream_t s) {
@@ -226,6 +551,9 @@ int docqa_window_attn(const void* q, const void* kc, const void* vc, const float
   if (B == 0 || max_q == 0) return 0;
   if (H % G != 0 || D < 1 || D > 512 || (BS & (BS - 1)) != 0) return -1;
   const WindowArgs a{block_tables, maxb, cu, ctx, k_scale, sink, H, G, D, BS, scale, window};
+  if (!f32 && D % 8 == 0 && D <= 256 && docqa_aligned16(q) && docqa_aligned16(out))
+    return kc == vc ? dispatch_dim<true>(q, kc, vc, out, a, B, max_q, s)
+                    : dispatch_dim<false>(q, kc, vc, out, a, B, max_q, s);
   dim3 grid((max_q * H + 3) / 4, B);
 #define GO(T, N) window_attn_kernel<T, N><<<grid, 256, 0, s>>>((const T*)q, (const T*)kc, (const T*)vc, (T*)out, a)
   if (f32) {

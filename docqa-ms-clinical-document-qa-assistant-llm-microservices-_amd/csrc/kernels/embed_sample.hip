@@ -133,7 +133,7 @@ __device__ __forceinline__ void better(float& bv, int& bi, float v, int i) {
   if (v > bv || (v == bv && i < bi)) { bv = v; bi = i; }
 }
 
-// VEC: rows and base are 16-byte aligned (any V: the last chunk's rest is read one by one)
+// VEC: every row is 16-byte aligned (any V: the last chunk's rest is read one by one)
 template <bool BF16, bool VEC>
 __global__ __launch_bounds__(256) void argmax_pass1(const void* __restrict__ logits, int V,
                                                     int ld, int splits, float* __restrict__ pv,
@@ -354,7 +354,8 @@ int docqa_bert_embed_ln(const int* ids, const int* pos, const int* tt, const voi
 int docqa_argmax(const void* logits, int rows, int V, int ld, int is_bf16, float* ws_v, int* ws_i,
                  int splits, int64_t* out, hipStream_t s) {
   if (rows == 0) return 0;
-  const bool vec = ld % (is_bf16 ? 8 : 4) == 0 && docqa_aligned16(logits);
+  if (!docqa_aligned16(logits)) return -1;
+  const bool vec = ld % (is_bf16 ? 8 : 4) == 0;
   dim3 g1(splits, rows);
   if (is_bf16 && vec) argmax_pass1<true, true><<<g1, 256, 0, s>>>(logits, V, ld, splits, ws_v, ws_i);
   else if (is_bf16) argmax_pass1<true, false><<<g1, 256, 0, s>>>(logits, V, ld, splits, ws_v, ws_i);

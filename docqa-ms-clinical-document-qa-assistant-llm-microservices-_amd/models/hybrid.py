@@ -225,13 +225,13 @@ class SelectiveScan:
             xc.append(y)
             zs.append(z)
         xa = _join(xc)
-        pr = ops.linear(xa, self.w_x, decode)
-        dt = ops.linear(pr[:, :self.rp].contiguous(), self.w_dt, decode)
+        dt_in, bc = ops.slab_columns(ops.project(xa, self.w_x, decode), self.rp, 2 * self.np, self.dtype)
+        dt = ops.linear(dt_in, self.w_dt, decode)
         out = []
         for p, y, z in zip(parts, xc, zs):
             m = p.meta
-            args = (y, _split(dt, p, parts), _split(pr, p, parts), self.rp, self.rp + self.np, N, z, self.A2, self.D,
-                    self.dt_b, scan_state, m.state_slots)
+            args = (y, _split(dt, p, parts), _split(bc, p, parts), 0, self.np, N, z, self.A2, self.D, self.dt_b,
+                    scan_state, m.state_slots)
             if p.decode:
                 out.append(ops.selective_step(*args, m.positions))
             else:
@@ -241,12 +241,11 @@ class SelectiveScan:
 
 class SquaredReluMLP:
     def __init__(self, get, dtype):
-        self.dtype = dtype
         self.up = get("up").to(dtype).contiguous()
         self.down = get("down").to(dtype).contiguous()
 
     def run(self, x, decode):
-        return ops.project(ops.squared_relu(ops.project(x, self.up, decode), self.dtype), self.down, decode)
+        return ops.project(ops.relu2_linear(x, self.up, decode), self.down, decode)
 
 
 class HybridModel(Decoder):

@@ -1218,6 +1218,29 @@ def squared_relu(P, out_dtype=torch.bfloat16):
     return ref.squared_relu(P, out_dtype)
 
 
+def relu2_linear(x, w, decode: bool = False):
+    """max(x @ w^T, 0)^2, the activation in the GEMM's epilogue where a hand-written bf16 GEMM
+    takes the shape without splitting K (the decode kernels, the 256 x 256 prefill kernel)."""
+    if _gpu(x) and x.dtype == torch.bfloat16:
+        N, K = w.shape
+        M = x.numel() // K
+        if (decode or M <= MID_M_MAX) and M > 1:
+            if (M <= 128 and N % 64 == 0 and K % 512 == 0 and decode_plan(M, N, K)[0] == 1) or (
+                    129 <= M <= MID_M_MAX and mid_plan(M, N, K)[0] == 1):
+                return _native().decode_relu2(x.contiguous(), w)
+        elif M > MID_M_MAX and pgemm_ok(M, N, K) and not prefill_split_plan(M, N, K):
+            return _native().pgemm(x.contiguous(), w, 3)
+    return squared_relu(project(x, w, decode), x.dtype)
+
+
+def slab_columns(P, n0: int, n1: int, out_dtype=torch.bfloat16):
+    """Columns [0, n0) and [n0, n0 + n1) of a projection (product or slabs) as two matrices."""
+    if _gpu(P):
+        return _native().slab_columns(P.contiguous(), n0, n1, out_dtype == torch.float32)
+    x = ref._slab_sum(P).to(out_dtype)
+    return x[:, :n0].contiguous(), x[:, n0:n0 + n1].contiguous()
+
+
 def qk_norm_store(P, w, slots, k_cache, k_scale, H: int, eps: float):
     """Queries rms(q) * w per head [M, H * D] from a [q | k] projection; the key rows go to
     the paged cache as projected, with their inverse root mean square in ``k_scale``.  A

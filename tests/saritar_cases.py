@@ -126,6 +126,28 @@ def squared_relu_case(device):
         close(ops.squared_relu(p.to(device), BF16), want, BF16)
 
 
+def relu2_linear_case(device, shapes):
+    for M, N, K in shapes:
+        g = torch.Generator().manual_seed(M)
+        x, w = (torch.randn(n, K, generator=g).to(BF16) for n in (M, N))
+        want = O.squared_relu((x.to(device).float() @ w.to(device).float().T / K ** 0.5).cpu())
+        for decode in (True, False):
+            got = ops.relu2_linear(x.to(device), (w.float() / K ** 0.5).to(BF16).to(device), decode)
+            assert got.shape == (M, N) and got.dtype == BF16
+            close(got, want, BF16, (M, N, K, decode))
+
+
+def slab_columns_case(device):
+    P = torch.randn(3, 7, 40, generator=torch.Generator().manual_seed(3))
+    for p in (P, P[0].contiguous()):
+        want = p.sum(0) if p.dim() == 3 else p
+        for dt in (F32, BF16):
+            a, b = ops.slab_columns(p.to(device), 12, 20, dt)
+            assert a.is_contiguous() and b.is_contiguous() and a.dtype == b.dtype == dt
+            close(a, want[:, :12], dt)
+            close(b, want[:, 12:32], dt)
+
+
 # ------------------------------------------------------------------ attention
 def _paged(T, G, d, bs, device, dtype, seed):
     nb = (T + bs - 1) // bs + 3

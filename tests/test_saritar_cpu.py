@@ -28,6 +28,8 @@ def test_norms_and_activations():
     C.norm_case("cpu")
     C.embed_case("cpu")
     C.squared_relu_case("cpu")
+    C.slab_columns_case("cpu")
+    C.relu2_linear_case("cpu", [(3, 8, 16)])
 
 
 @pytest.mark.parametrize("case", ["window_edge_case", "sink_case", "general_attention_case", "batch_attention_case",

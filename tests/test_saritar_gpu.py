@@ -24,6 +24,10 @@ def test_norms_and_activations():
     C.norm_case("cuda")
     C.embed_case("cuda")
     C.squared_relu_case("cuda")
+    C.slab_columns_case("cuda")
+    # odd shapes, then each GEMM with the activation in its epilogue
+    C.relu2_linear_case("cuda", [(3, 40, 24), (1, 4096, 2048), (5, 12288, 512), (100, 12288, 512), (200, 14592, 256),
+                                 (600, 16384, 256)])
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
