@@ -163,7 +163,7 @@ def bench_kernels(size: str) -> list[dict]:
         # a state's step: multiply, exponential (2 lane-operations), two FMAs, multiply
         row("selective_scan", "prefill", M, lambda i: ops.selective_scan(x[i % nc], dt[i % nc], bc, 0, N, N,
                                                                          xz[i % nc][:, C:], A2, Dv, dtb, st, sl, cu, ctx, M),
-            M * C * 8, lane_ops=6.0 * M * C * N, like="flash_prefill")
+            M * C * 8, lane_ops=6.0 * M * C * N, like="flash_prefill_paged")
         del xz, x, dt
         nb = (M + BS - 1) // BS
         kc, ks = rnd(nb, G, BS, d), torch.ones(nb, G, BS, device=dev)
@@ -206,9 +206,10 @@ def bench_kernels(size: str) -> list[dict]:
         nc = copies(B * C * N * 4)
         sl, pos, ctx = i32(list(range(B))), i32([1024] * B), i32([1025] * B)
         st = [torch.zeros(B, C, N, device=dev) for _ in range(nc)]
-        x, dt, z, bc = rnd(B, C), rnd(B, C), rnd(B, C), rnd(B, 2 * N)
-        row("selective_step", "decode", B, lambda i: ops.selective_step(x, dt, bc, 0, N, N, z, A2, Dv, dtb, st[i % nc], sl, pos),
-            B * C * (N * 8 + 8), lane_ops=6.0 * B * C * N, like="paged_decode")
+        x, z, bc, dti, wdt = rnd(B, C), rnd(B, C), rnd(B, 2 * N), rnd(B, R), rnd(C, R)
+        row("selective_step+dt_proj", "decode", B, lambda i: ops.selective_step(x, (dti, wdt), bc, 0, N, N, z, A2, Dv, dtb,
+                                                                                st[i % nc], sl, pos),
+            B * C * (N * 8 + 6) + C * R * 2, lane_ops=6.0 * B * C * N, like="paged_decode")
         del st
         cst = torch.zeros(B, 3, C, device=dev, dtype=bf)
         P = rnd(B, 2 * C, dt=f32)[None] if B <= 192 else rnd(B, 2 * C)
@@ -240,7 +241,7 @@ def bench_kernels(size: str) -> list[dict]:
         row("rope_cache_splitk", "decode", B, lambda i: ops.rope_cache_splitk(qkv, pos, cs, slots, kc, kc2, H, G, d),
             B * (H + 2 * G) * d * 6)
         for name, n, k, like in (("in_proj", 2 * C, W, "qkv_proj"), ("out_proj", W, C, "qkv_proj"), ("qkv_proj", (H + 2 * G) * d, W, ""),
-                                 ("x_proj", 512 if R + 2 * N > 256 else 256, C, "qkv_proj"), ("dt_proj", C, R, "qkv_proj")):
+                                 ("x_proj", 512 if R + 2 * N > 256 else 256, C, "qkv_proj")):
             nc = copies(n * k * 2)
             ws, xx = [rnd(n, k) for _ in range(nc)], rnd(B, k)
             row(name, "decode", B, lambda i: ops.project(xx, ws[i % nc], True), n * k * 2.0, 2.0 * B * n * k, like=like)

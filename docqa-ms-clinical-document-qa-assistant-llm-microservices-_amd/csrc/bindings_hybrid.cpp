@@ -229,12 +229,13 @@ std::tuple<Tensor, Tensor> conv_step(const Tensor& P, const Tensor& w, const Ten
   return {y, z};
 }
 
-int check_scan(const Tensor& x, const Tensor& dt, const Tensor& bc, const Tensor& z, const Tensor& A2, const Tensor& D,
+int check_scan(const Tensor& x, const OptT& dt, const Tensor& bc, const Tensor& z, const Tensor& A2, const Tensor& D,
                const Tensor& dt_b, const Tensor& state, int64_t N, int64_t b_off, int64_t c_off) {
-  CHECK_ACT(x); CHECK_CONTIG(x); CHECK_CONTIG(dt);
+  CHECK_ACT(x); CHECK_CONTIG(x);
   TORCH_CHECK(x.dim() == 2, "x must be [tokens, channels]");
   const int T = x.size(0), C = x.size(1);
-  TORCH_CHECK(dt.sizes() == x.sizes() && dt.scalar_type() == x.scalar_type(), "dt must match x");
+  if (dt.has_value())
+    TORCH_CHECK(dt->is_contiguous() && dt->sizes() == x.sizes() && dt->scalar_type() == x.scalar_type(), "dt must match x");
   TORCH_CHECK(A2.dim() == 2 && A2.size(0) == C && A2.size(1) >= N && A2.size(1) % 4 == 0, "A2 must be [channels, N padded to 4]");
   const int Np = A2.size(1);
   check_vec(A2, (int64_t)C * Np, "A2");
@@ -274,18 +275,30 @@ Tensor selective_scan(const Tensor& x, const Tensor& dt, const Tensor& bc, int64
   return y;
 }
 
-Tensor selective_step(const Tensor& x, const Tensor& dt, const Tensor& bc, int64_t b_off, int64_t c_off, int64_t N,
-                      const Tensor& z, const Tensor& A2, const Tensor& D, const Tensor& dt_b, Tensor state,
-                      const Tensor& slots, const Tensor& positions) {
+// dt: the step projection [B, C], or (dt_in [B, R], w_dt [C, R]) to run it inside the launch
+Tensor selective_step(const Tensor& x, const OptT& dt, const OptT& dt_in, const OptT& w_dt, const Tensor& bc,
+                      int64_t b_off, int64_t c_off, int64_t N, const Tensor& z, const Tensor& A2, const Tensor& D,
+                      const Tensor& dt_b, Tensor state, const Tensor& slots, const Tensor& positions) {
   const int Np = check_scan(x, dt, bc, z, A2, D, dt_b, state, N, b_off, c_off);
   const int B = x.size(0), C = x.size(1);
   check_i32(slots, B, "slots"); check_i32(positions, B, "positions");
+  TORCH_CHECK(dt.has_value() != w_dt.has_value() && dt_in.has_value() == w_dt.has_value(), "dt, or dt_in and w_dt");
+  int R = 0;
+  if (w_dt.has_value()) {
+    CHECK_BF16(*w_dt); CHECK_BF16(*dt_in); CHECK_BF16(x); CHECK_CONTIG(*w_dt); CHECK_CONTIG(*dt_in);
+    CHECK_GPU(*w_dt); CHECK_GPU(*dt_in);
+    R = w_dt->size(1);
+    TORCH_CHECK(w_dt->dim() == 2 && w_dt->size(0) == C && dt_in->dim() == 2 && dt_in->size(0) == B && dt_in->size(1) == R,
+                "w_dt [C, R], dt_in [B, R]");
+  }
   c10::DeviceGuard g(x.device());
   auto y = at::empty_like(x);
-  CHECK_RC(docqa_selective_step(x.data_ptr(), dt.data_ptr(), bc.data_ptr(), (int)bc.stride(0), (int)b_off, (int)c_off,
-                                z.data_ptr(), (int)z.stride(0), A2.data_ptr<float>(), D.data_ptr<float>(),
-                                dt_b.data_ptr<float>(), state.data_ptr<float>(), slots.data_ptr<int>(),
-                                positions.data_ptr<int>(), y.data_ptr(), is_f32(x), B, C, (int)N, Np, stream()),
+  CHECK_RC(docqa_selective_step(x.data_ptr(), dt.has_value() ? dt->data_ptr() : nullptr,
+                                w_dt.has_value() ? dt_in->data_ptr() : nullptr, w_dt.has_value() ? w_dt->data_ptr() : nullptr,
+                                R, bc.data_ptr(), (int)bc.stride(0), (int)b_off, (int)c_off, z.data_ptr(),
+                                (int)z.stride(0), A2.data_ptr<float>(), D.data_ptr<float>(), dt_b.data_ptr<float>(),
+                                state.data_ptr<float>(), slots.data_ptr<int>(), positions.data_ptr<int>(), y.data_ptr(),
+                                is_f32(x), B, C, (int)N, Np, stream()),
            "selective_step");
   return y;
 }
@@ -310,7 +323,7 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
         "-> (Tensor, Tensor)");
   m.def("selective_scan(Tensor x, Tensor dt, Tensor bc, int b_off, int c_off, int N, Tensor z, Tensor A2, Tensor D, "
         "Tensor dt_b, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, int max_len, int chunk) -> Tensor");
-  m.def("selective_step(Tensor x, Tensor dt, Tensor bc, int b_off, int c_off, int N, Tensor z, Tensor A2, Tensor D, "
+  m.def("selective_step(Tensor x, Tensor? dt, Tensor? dt_in, Tensor? w_dt, Tensor bc, int b_off, int c_off, int N, Tensor z, Tensor A2, Tensor D, "
         "Tensor dt_b, Tensor(a!) state, Tensor slots, Tensor positions) -> Tensor");
 }
 

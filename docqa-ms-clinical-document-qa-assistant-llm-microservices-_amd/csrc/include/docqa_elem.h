@@ -95,8 +95,13 @@ __device__ __forceinline__ void ld_slabs(const PT* p, int S, size_t slab, float*
   }
 }
 
-__device__ __forceinline__ float silu_exact(float x) { return x / (1.f + __expf(-x)); }
-// log(1 + e^x): e^-|x| keeps it finite on both sides
-__device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(__expf(-fabsf(x))); }
+__device__ __forceinline__ float silu_fast(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
+// log(1 + e^x) = max(x, 0) + log1p(e), e = e^-|x|; log1p(e) = log(u) e / (u - 1) with u = 1 + e
+// rounded (Kahan's correction of the rounding in u), e itself once u rounds to 1
+__device__ __forceinline__ float softplus_f(float x) {
+  const float e = __expf(-fabsf(x)), u = 1.f + e, v = u - 1.f;
+  const float l = v > 0.f ? __logf(u) * e * __builtin_amdgcn_rcpf(v) : e;
+  return fmaxf(x, 0.f) + l;
+}
 
 }  // namespace docqa

@@ -38,7 +38,8 @@ int docqa_selective_scan(const void* x, const void* dt, const void* bc, int ld_b
                          const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
                          const int* slots, const int* cu, const int* ctx, void* y, float* cstate, float* csum,
                          int f32, int B, int C, int N, int Np, int chunk, int nchunk, hipStream_t s);
-int docqa_selective_step(const void* x, const void* dt, const void* bc, int ld_bc, int b_off, int c_off,
-                         const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
-                         const int* slots, const int* positions, void* y, int f32, int B, int C, int N, int Np,
-                         hipStream_t s);
+// w_dt (bf16 [C, R], R % 32): the step projection of dt_in [B, R] inside the launch, else dt [B, C]
+int docqa_selective_step(const void* x, const void* dt, const void* dt_in, const void* w_dt, int R, const void* bc,
+                         int ld_bc, int b_off, int c_off, const void* z, int ld_z, const float* A2, const float* D,
+                         const float* dt_b, float* state, const int* slots, const int* positions, void* y, int f32,
+                         int B, int C, int N, int Np, hipStream_t s);

@@ -20,22 +20,24 @@ using namespace docqa;
 namespace {
 constexpr float kLog2e = 1.4426950408889634f;
 
-// one wave per (token, head); heads [0, H) are queries, [H, H + G) keys
-template <int V, int NI, typename PT, typename T>
+// LPH lanes per (token, head), V elements a lane at a time; heads [0, H) are queries,
+// [H, H + G) keys
+template <int V, int NI, int LPH, typename PT, typename T>
 __global__ __launch_bounds__(256) void qk_norm_store_kernel(const PT* __restrict__ P, int S, size_t slab, int ld,
                                                             const float* __restrict__ wq,
                                                             const int* __restrict__ slot_mapping, T* __restrict__ q,
                                                             T* __restrict__ kc, float* __restrict__ ks, int tokens,
-                                                            int H, int G, int D, int BS, float eps) {
-  const int u = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  const int t = u / (H + G), h = u % (H + G);
-  if (t >= tokens) return;
+                                                            int H, int G, int D, int log2BS, float eps) {
+  const int heads = H + G;
+  const unsigned u = blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
+  const int lane = threadIdx.x % LPH, t = u / heads, h = u - t * heads;
+  if (t >= tokens) return;                 // whole lane groups
   const PT* p = P + (size_t)t * ld + (size_t)h * D;
   float x[NI][V];
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
-    const int c = (lane + 64 * i) * V;
+    const int c = (lane + LPH * i) * V;
     if (c < D) {
       ld_slabs<V>(p + c, S, slab, x[i]);
 #pragma unroll
@@ -45,12 +47,12 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(const PT* __restrict
       }
     }
   }
-  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)D + eps);
+  const float inv = 1.f / sqrtf(group_sum<LPH>(ss) / (float)D + eps);
   if (h < H) {
     T* o = q + ((size_t)t * H + h) * D;
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      const int c = (lane + 64 * i) * V;
+      const int c = (lane + LPH * i) * V;
       if (c < D) {
         float w[V];
         ldv<V>(wq + c, w);
@@ -62,10 +64,10 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(const PT* __restrict
   } else {
     const int slot = slot_mapping[t];
     if (slot < 0) return;
-    const size_t row = ((size_t)(slot / BS) * G + (h - H)) * BS + slot % BS;
+    const size_t row = ((((size_t)(slot >> log2BS)) * G + (h - H)) << log2BS) + (slot & ((1 << log2BS) - 1));
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      const int c = (lane + 64 * i) * V;
+      const int c = (lane + LPH * i) * V;
       if (c < D) stv<V>(kc + row * D + c, x[i]);
     }
     if (lane == 0) ks[row] = inv;
@@ -80,7 +82,7 @@ struct WindowArgs {
                           // context length including the new token
   const float* k_scale;   // [blocks, G, BS] or null
   const float* sink;      // [H] or null
-  int H, G, D, BS;
+  int H, G, D, BS, log2BS;
   float scale;
   int window;
 };
@@ -139,8 +141,8 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
     float s = -INFINITY;
     int row = 0;
     if (key <= pos) {
-      const int blk = a.block_tables[(size_t)b * a.maxb + key / a.BS];
-      row = (blk * a.G + g) * a.BS + key % a.BS;
+      const int blk = a.block_tables[(size_t)b * a.maxb + (key >> a.log2BS)];
+      row = ((blk * a.G + g) << a.log2BS) + (key & (a.BS - 1));
       const T* kp = kc + (size_t)row * D;
       float d0 = 0.f, d1 = 0.f;
       int c = 0;
@@ -267,8 +269,8 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_
   uint4 rk[CPT], rv[SHARED ? 1 : CPT];
   float rs_ = 1.f;
   auto cache_row = [&](int key) {
-    const int blk = a.block_tables[(size_t)b * a.maxb + key / a.BS];
-    return ((size_t)blk * a.G + kvh) * a.BS + key % a.BS;
+    const int blk = a.block_tables[(size_t)b * a.maxb + (key >> a.log2BS)];
+    return (size_t)((((blk * a.G + kvh) << a.log2BS)) + (key & (a.BS - 1)));
   };
   auto load = [&](int t) {
     const int kb = key0 + t * KB;
@@ -514,16 +516,20 @@ int dispatch_dim(const void* q, const void* kc, const void* vc, void* out, const
 template <typename PT, typename T>
 int qk_store(const PT* P, int S, size_t slab, int ld, const float* wq, const int* sm, T* q, T* kc, float* ks,
              int tokens, int H, int G, int D, int BS, float eps, hipStream_t s) {
-  const int grid = (int)(((long long)tokens * (H + G) + 3) / 4);
-#define GO(V, N) qk_norm_store_kernel<V, N, PT, T><<<grid, 256, 0, s>>>(P, S, slab, ld, wq, sm, q, kc, ks, tokens, H, G, D, BS, eps)
-  if (D % 2 == 0 && ld % 2 == 0) {
-    if (D <= 128) GO(2, 1);
-    else if (D <= 256) GO(2, 2);
-    else GO(2, 4);
+  int log2BS = 0;
+  while ((1 << log2BS) < BS) ++log2BS;
+#define GO(V, N, L)                                                                                        \
+  qk_norm_store_kernel<V, N, L, PT, T><<<(int)(((long long)tokens * (H + G) + 256 / L - 1) / (256 / L)), 256, 0, s>>>( \
+      P, S, slab, ld, wq, sm, q, kc, ks, tokens, H, G, D, log2BS, eps)
+  if (D % 8 == 0 && ld % 8 == 0) {
+    if (D <= 64) GO(8, 1, 8);
+    else if (D <= 128) GO(8, 1, 16);
+    else if (D <= 256) GO(8, 1, 32);
+    else GO(8, 1, 64);
   } else {
-    if (D <= 64) GO(1, 1);
-    else if (D <= 128) GO(1, 2);
-    else GO(1, 8);
+    if (D <= 64) GO(1, 1, 64);
+    else if (D <= 128) GO(1, 2, 64);
+    else GO(1, 8, 64);
   }
 #undef GO
   DOCQA_CHECK_LAUNCH();
@@ -535,7 +541,8 @@ int docqa_qk_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, co
                         void* q, void* kc, float* ks, int f32, int tokens, int H, int G, int D, int BS, float eps,
                         hipStream_t s) {
   if (tokens == 0) return 0;
-  if (S < 1 || D < 1 || D > 512 || H < 1 || G < 1 || ld < (H + G) * D) return -1;
+  if (S < 1 || D < 1 || D > 512 || H < 1 || G < 1 || ld < (H + G) * D || (BS & (BS - 1)) != 0) return -1;
+  if ((long long)tokens * (H + G) >= (1ll << 31)) return -1;
   if (f32) {
     if (!p_f32) return -1;
     return qk_store((const float*)P, S, slab, ld, wq, slots, (float*)q, (float*)kc, ks, tokens, H, G, D, BS, eps, s);
@@ -550,7 +557,9 @@ int docqa_window_attn(const void* q, const void* kc, const void* vc, const float
                       int max_q, int H, int G, int D, int BS, float scale, int window, hipStream_t s) {
   if (B == 0 || max_q == 0) return 0;
   if (H % G != 0 || D < 1 || D > 512 || (BS & (BS - 1)) != 0) return -1;
-  const WindowArgs a{block_tables, maxb, cu, ctx, k_scale, sink, H, G, D, BS, scale, window};
+  int log2BS = 0;
+  while ((1 << log2BS) < BS) ++log2BS;
+  const WindowArgs a{block_tables, maxb, cu, ctx, k_scale, sink, H, G, D, BS, log2BS, scale, window};
   if (!f32 && D % 8 == 0 && D <= 256 && docqa_aligned16(q) && docqa_aligned16(out))
     return kc == vc ? dispatch_dim<true>(q, kc, vc, out, a, B, max_q, s)
                     : dispatch_dim<false>(q, kc, vc, out, a, B, max_q, s);

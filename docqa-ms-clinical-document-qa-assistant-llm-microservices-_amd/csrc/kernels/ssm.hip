@@ -32,7 +32,7 @@ constexpr int UB = 8;    // tokens whose x / dt / z are loaded ahead of their us
 template <typename T, int V, int K>
 __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ x, int ldx,
                                                           const float* __restrict__ w, const float* __restrict__ bias,
-                                                          const T* __restrict__ state, const int* __restrict__ slots,
+                                                          T* __restrict__ state, const int* __restrict__ slots,
                                                           const int* __restrict__ cu, const int* __restrict__ ctx,
                                                           T* __restrict__ y, int C, int taps) {
   constexpr int TT = 8;
@@ -56,28 +56,22 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
     }
   };
   if constexpr (K > 0) {
-    float wv[K][V], win[K][V];
+    float wv[K][V], in[TT + K - 1][V];      // inputs t0 - (K - 1) .. t0 + TT - 1, all in flight at once
+#pragma unroll
+    for (int i = 0; i < TT + K - 1; ++i) input(min(t0 + i - (K - 1), L - 1), in[i]);
 #pragma unroll
     for (int k = 0; k < K; ++k) ldv<V>(w + (size_t)k * C + c0, wv[k]);
 #pragma unroll
-    for (int k = 0; k < K - 1; ++k) input(t0 - (K - 1) + k, win[k]);
-#pragma unroll
     for (int i = 0; i < TT; ++i) {
-      if (t0 + i >= L) break;
-      input(t0 + i, win[K - 1]);
       float o[V];
 #pragma unroll
       for (int j = 0; j < V; ++j) {
         float s = bv[j];
 #pragma unroll
-        for (int k = 0; k < K; ++k) s += wv[k][j] * win[k][j];
-        o[j] = silu_exact(s);
+        for (int k = 0; k < K; ++k) s += wv[k][j] * in[i + k][j];
+        o[j] = silu_fast(s);
       }
-      stv<V>(y + (size_t)(q0 + t0 + i) * C + c0, o);
-#pragma unroll
-      for (int k = 0; k < K - 1; ++k)
-#pragma unroll
-        for (int j = 0; j < V; ++j) win[k][j] = win[k + 1][j];
+      if (t0 + i < L) stv<V>(y + (size_t)(q0 + t0 + i) * C + c0, o);
     }
   } else {
     for (int i = 0; i < TT && t0 + i < L; ++i) {
@@ -91,29 +85,20 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
         for (int j = 0; j < V; ++j) s[j] += wk[j] * f[j];
       }
 #pragma unroll
-      for (int j = 0; j < V; ++j) s[j] = silu_exact(s[j]);
+      for (int j = 0; j < V; ++j) s[j] = silu_fast(s[j]);
       stv<V>(y + (size_t)(q0 + t0 + i) * C + c0, s);
     }
   }
-}
-
-// the last taps - 1 inputs of every sequence into its state rows.  Row r takes the input of
-// portion token L - (taps - 1) + r, or old row r + L (> r, so ascending r reads before it
-// writes), or zero ahead of the sequence.
-template <typename T>
-__global__ __launch_bounds__(256) void conv_tail_kernel(const T* __restrict__ x, int ldx, T* __restrict__ state,
-                                                        const int* __restrict__ slots, const int* __restrict__ cu,
-                                                        const int* __restrict__ ctx, int C, int taps) {
-  const int b = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
-  const int q0 = cu[b], L = cu[b + 1] - q0, slot = slots[b];
-  if (c >= C || slot < 0 || L <= 0) return;
-  T* st = state + (size_t)slot * (taps - 1) * C + c;
-  for (int r = 0; r < taps - 1; ++r) {
-    const int t = L - (taps - 1) + r;
-    T v = 0;
-    if (t >= 0) v = x[(size_t)(q0 + t) * ldx + c];
-    else if (ctx[b] > 0) v = st[(size_t)(r + L) * C];
-    st[(size_t)r * C] = v;
+  // The last taps - 1 inputs into the state, by the one thread that read it (t0 = 0): row r
+  // takes the input of portion token L - (taps - 1) + r, or old row r + L (> r, so ascending r
+  // reads before it writes), or zero ahead of the sequence.
+  if (t0 == 0 && slots[b] >= 0) {
+    T* so = state + (size_t)slots[b] * (nt - 1) * C + c0;
+    for (int r = 0; r < nt - 1; ++r) {
+      float f[V];
+      input(L - (nt - 1) + r, f);
+      stv<V>(so + (size_t)r * C, f);
+    }
   }
 }
 
@@ -182,7 +167,7 @@ __global__ __launch_bounds__(256) void conv_step_kernel(const PT* __restrict__ P
     }
   }
 #pragma unroll
-  for (int j = 0; j < V; ++j) s[j] = silu_exact(s[j]);
+  for (int j = 0; j < V; ++j) s[j] = silu_fast(s[j]);
   stv<V>(y + (size_t)b * C + c0, s);
 }
 
@@ -277,7 +262,7 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs a) {
       for (int i = 0; i < UB; ++i) {
         xv[i] = xn[i];
         dv[i] = t0 + u + i < t_end ? softplus_f(dn[i] + db) : 0.f;
-        if constexpr (!LOCAL) zv[i] = silu_exact(zn[i]);
+        if constexpr (!LOCAL) zv[i] = silu_fast(zn[i]);
       }
       fetch(t0 + u + UB);
 #pragma unroll
@@ -288,7 +273,7 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs a) {
         float y = 0.f;
 #pragma unroll
         for (int n = 0; n < NS; ++n) {
-          S[n] = exp2f(d * A[n]) * S[n] + dx * Bt[n];
+          S[n] = __builtin_amdgcn_exp2f(d * A[n]) * S[n] + dx * Bt[n];
           if constexpr (!LOCAL) y += S[n] * Ct[n];
         }
         if constexpr (LOCAL) {
@@ -328,58 +313,100 @@ __global__ __launch_bounds__(256) void scan_carry_kernel(ScanArgs a) {
   float s = (a.ctx[b] > 0 && slot >= 0) ? a.state[(size_t)slot * a.C * a.Np + e] : 0.f;
   for (int k = 1; k * a.chunk < L; ++k) {
     const size_t o = ((size_t)b * a.nchunk + k) * a.C;
-    s = exp2f(A * a.csum[o + c]) * s + a.cstate[o * a.Np + e];
+    s = __builtin_amdgcn_exp2f(A * a.csum[o + c]) * s + a.cstate[o * a.Np + e];
     a.cstate[o * a.Np + e] = s;
   }
 }
 
 // ------------------------------------------------------------------ selective scan, decode
-// one token a row: a lane holds 4 states of a channel (16-byte state accesses), RB rows a
-// workgroup so that A is read once for all of them
+// One token a row.  A lane holds 4 states of a channel (16-byte state accesses, the launch's
+// HBM traffic), a workgroup 256 / lq channels of RB rows, so A is read once for all of them;
+// every row's state is in flight before anything is computed.  The rows' step sizes, inputs,
+// gates, B and C go through LDS.  w_dt given: the step projection runs here too, on MFMA
+// (the RB rows against the workgroup's channels, K = R), instead of a GEMM launch of its own.
+struct StepDt {
+  const uint16_t* w;    // [C, R] bf16, R % 32 == 0; null: ScanArgs::dt holds the product
+  const uint16_t* in;   // [B, R]
+  int R;
+};
 template <typename T, int RB>
-__global__ __launch_bounds__(256) void selective_step_kernel(ScanArgs a, const int* __restrict__ positions, int B,
-                                                             int lq) {
-  const int tid = threadIdx.x;
-  const int c = blockIdx.x * (256 / lq) + tid / lq, g = tid % lq, n0 = g * 4;
-  const bool okc = c < a.C, ok = okc && n0 < a.Np;
-  const int cc = okc ? c : a.C - 1;
-  float4 A = make_float4(0.f, 0.f, 0.f, 0.f);
-  if (ok) A = *reinterpret_cast<const float4*>(a.A2 + (size_t)c * a.Np + n0);
-  const float Dc = a.D[cc], db = a.dt_b[cc];
+__global__ __launch_bounds__(256) void selective_step_kernel(ScanArgs a, StepDt sd, const int* __restrict__ positions,
+                                                             int B, int lq) {
+  __shared__ float sdt[RB][256], sx[RB][256], sg[RB][256];
+  __shared__ __attribute__((aligned(16))) float sb[RB][256], sc[RB][256];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int CB = 256 / lq;                              // channels of this workgroup
+  const int cb = blockIdx.x * CB, cl = tid / lq, c = cb + cl, g = tid % lq, n0 = g * 4;
   const int r0 = blockIdx.y * RB;
-  float4 S[RB];
+  const bool ok = c < a.C && n0 < a.Np;
+  float4 A = make_float4(0.f, 0.f, 0.f, 0.f), S[RB];
   int slot[RB];
 #pragma unroll
   for (int i = 0; i < RB; ++i) {
     const int r = min(r0 + i, B - 1);
-    slot[i] = a.slots[r];
+    slot[i] = r0 + i < B ? a.slots[r] : -1;
     S[i] = make_float4(0.f, 0.f, 0.f, 0.f);
     if (ok && slot[i] >= 0 && positions[r] > 0)
       S[i] = *reinterpret_cast<const float4*>(a.state + ((size_t)slot[i] * a.C + c) * a.Np + n0);
   }
+  if (ok) A = *reinterpret_cast<const float4*>(a.A2 + (size_t)c * a.Np + n0);
+  const float Dc = a.D[min(c, a.C - 1)];
+
+  for (int e = tid; e < RB * CB; e += 256) {
+    const int i = e / CB, j = e % CB, cc = min(cb + j, a.C - 1);
+    const size_t r = min(r0 + i, B - 1);
+    sx[i][j] = ld1((const T*)a.x + r * a.C + cc);
+    sg[i][j] = silu_fast(ld1((const T*)a.z + r * a.ld_z + cc));
+    if (!sd.w) sdt[i][j] = softplus_f(ld1((const T*)a.dt + r * a.C + cc) + a.dt_b[cc]);
+  }
+  for (int e = tid; e < RB * a.Np; e += 256) {
+    const int i = e / a.Np, n = e % a.Np;
+    const T* bc = (const T*)a.bc + (size_t)min(r0 + i, B - 1) * a.ld_bc;
+    sb[i][n] = n < a.N ? ld1(bc + a.b_off + n) : 0.f;
+    sc[i][n] = n < a.N ? ld1(bc + a.c_off + n) : 0.f;
+  }
+  if (sd.w) {
+    // 16-channel tiles: A rows = token rows, B rows = channels; D: lane & 15 the channel,
+    // 4 (lane >> 4) + r the row
+    const int fr = lane & 15, g4 = lane >> 4;
+    const uint16_t* ip = sd.in + (size_t)min(r0 + min(fr, RB - 1), B - 1) * sd.R + g4 * 8;
+    for (int t = wave; t < (CB + 15) / 16; t += 4) {
+      const int ch = min(cb + t * 16 + fr, a.C - 1);
+      const uint16_t* wp = sd.w + (size_t)ch * sd.R + g4 * 8;
+      f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+      for (int k = 0; k < sd.R; k += 32)
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(ip + k),
+                                                      *reinterpret_cast<const bf16x8*>(wp + k), acc, 0, 0, 0);
+      const float db = a.dt_b[ch];
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (g4 * 4 + r < RB && t * 16 + fr < CB) sdt[g4 * 4 + r][t * 16 + fr] = softplus_f(acc[r] + db);
+    }
+  }
+  __syncthreads();
 #pragma unroll
   for (int i = 0; i < RB; ++i) {
-    const int r = r0 + i;
-    if (r >= B) break;
-    const float x = ld1((const T*)a.x + (size_t)r * a.C + cc);
-    const float d = softplus_f(ld1((const T*)a.dt + (size_t)r * a.C + cc) + db), dx = d * x;
-    const T* bc = (const T*)a.bc + (size_t)r * a.ld_bc;
-    float bv[4], cv[4];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      bv[j] = n0 + j < a.N ? ld1(bc + a.b_off + n0 + j) : 0.f;
-      cv[j] = n0 + j < a.N ? ld1(bc + a.c_off + n0 + j) : 0.f;
-    }
+    const float d = sdt[i][cl], x = sx[i][cl], dx = d * x;
     float4 s = S[i];
-    s.x = exp2f(d * A.x) * s.x + dx * bv[0];
-    s.y = exp2f(d * A.y) * s.y + dx * bv[1];
-    s.z = exp2f(d * A.z) * s.z + dx * bv[2];
-    s.w = exp2f(d * A.w) * s.w + dx * bv[3];
-    float y = (s.x * cv[0] + s.y * cv[1]) + (s.z * cv[2] + s.w * cv[3]);
+    float y = 0.f;
+    if (ok) {
+      const float4 bv = *reinterpret_cast<const float4*>(&sb[i][n0]), cv = *reinterpret_cast<const float4*>(&sc[i][n0]);
+      s.x = __builtin_amdgcn_exp2f(d * A.x) * s.x + dx * bv.x;
+      s.y = __builtin_amdgcn_exp2f(d * A.y) * s.y + dx * bv.y;
+      s.z = __builtin_amdgcn_exp2f(d * A.z) * s.z + dx * bv.z;
+      s.w = __builtin_amdgcn_exp2f(d * A.w) * s.w + dx * bv.w;
+      y = (s.x * cv.x + s.y * cv.y) + (s.z * cv.z + s.w * cv.w);
+      if (slot[i] >= 0) *reinterpret_cast<float4*>(a.state + ((size_t)slot[i] * a.C + c) * a.Np + n0) = s;
+    }
     for (int o = 1; o < lq; o <<= 1) y += __shfl_xor(y, o, 64);
-    if (ok && slot[i] >= 0) *reinterpret_cast<float4*>(a.state + ((size_t)slot[i] * a.C + c) * a.Np + n0) = s;
-    if (okc && g == 0)
-      st1((T*)a.y + (size_t)r * a.C + c, (y + Dc * x) * silu_exact(ld1((const T*)a.z + (size_t)r * a.ld_z + c)));
+    // a channel's lanes are one wave's: they have all read sx[i][cl] above
+    if (g == 0) sx[i][cl] = (y + Dc * x) * sg[i][cl];
+  }
+  __syncthreads();
+  for (int e = tid; e < RB * CB; e += 256) {
+    const int i = e / CB, j = e % CB;
+    if (r0 + i < B && cb + j < a.C) st1((T*)a.y + (size_t)(r0 + i) * a.C + cb + j, sx[i][j]);
   }
 }
 
@@ -387,7 +414,7 @@ template <typename T, int V>
 int launch_conv(const void* x, int ldx, const float* w, const float* b, void* state, const int* slots, const int* cu,
                 const int* ctx, void* y, int B, int max_len, int C, int taps, hipStream_t s) {
   dim3 grid((C + 64 * V - 1) / (64 * V), (max_len + 31) / 32, B);
-#define GO(K) causal_conv_kernel<T, V, K><<<grid, 256, 0, s>>>((const T*)x, ldx, w, b, (const T*)state, slots, cu, ctx, (T*)y, C, taps)
+#define GO(K) causal_conv_kernel<T, V, K><<<grid, 256, 0, s>>>((const T*)x, ldx, w, b, (T*)state, slots, cu, ctx, (T*)y, C, taps)
   switch (taps) {
     case 2: GO(2); break;
     case 3: GO(3); break;
@@ -396,10 +423,6 @@ int launch_conv(const void* x, int ldx, const float* w, const float* b, void* st
   }
 #undef GO
   DOCQA_CHECK_LAUNCH();
-  if (taps > 1) {
-    conv_tail_kernel<T><<<dim3((C + 255) / 256, B), 256, 0, s>>>((const T*)x, ldx, (T*)state, slots, cu, ctx, C, taps);
-    DOCQA_CHECK_LAUNCH();
-  }
   return 0;
 }
 
@@ -484,24 +507,29 @@ int docqa_selective_scan(const void* x, const void* dt, const void* bc, int ld_b
   return f32 ? dispatch_scan<float>(a, B, s) : dispatch_scan<uint16_t>(a, B, s);
 }
 
-int docqa_selective_step(const void* x, const void* dt, const void* bc, int ld_bc, int b_off, int c_off,
-                         const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
-                         const int* slots, const int* positions, void* y, int f32, int B, int C, int N, int Np,
-                         hipStream_t s) {
+int docqa_selective_step(const void* x, const void* dt, const void* dt_in, const void* w_dt, int R, const void* bc,
+                         int ld_bc, int b_off, int c_off, const void* z, int ld_z, const float* A2, const float* D,
+                         const float* dt_b, float* state, const int* slots, const int* positions, void* y, int f32,
+                         int B, int C, int N, int Np, hipStream_t s) {
   if (B == 0) return 0;
   if (N < 1 || Np < N || Np % 4 || Np > 256) return -1;
+  if (w_dt ? (f32 || !dt_in || R < 32 || R % 32 || !docqa_aligned16(w_dt) || !docqa_aligned16(dt_in)) : !dt) return -1;
   const ScanArgs a{x, dt, bc, z, y, ld_bc, b_off, c_off, ld_z, A2, D, dt_b, state, slots, nullptr, nullptr, nullptr,
                    nullptr, C, N, Np, 0, 0};
+  const StepDt sd{(const uint16_t*)w_dt, (const uint16_t*)dt_in, R};
   int lq = 1;
   while (lq * 4 < Np) lq *= 2;
   const int gx = (C + 256 / lq - 1) / (256 / lq);
-#define GO(T, R) selective_step_kernel<T, R><<<dim3(gx, (B + R - 1) / R), 256, 0, s>>>(a, positions, B, lq)
+#define GO(T, RB) selective_step_kernel<T, RB><<<dim3(gx, (B + RB - 1) / RB), 256, 0, s>>>(a, sd, positions, B, lq)
   if (f32) {
-    if (B >= 8) GO(float, 4);
+    if (B >= 4) GO(float, 4);
     else GO(float, 1);
+  } else if (B >= 32) {
+    GO(uint16_t, 8);
+  } else if (B >= 4) {
+    GO(uint16_t, 4);
   } else {
-    if (B >= 8) GO(uint16_t, 4);
-    else GO(uint16_t, 1);
+    GO(uint16_t, 1);
   }
 #undef GO
   DOCQA_CHECK_LAUNCH();

@@ -12,8 +12,9 @@ MI355X layout:
   * attention keeps the key rows as projected, once, as key and value, with the row's inverse
     RMS beside it (ops.qk_norm_store) -- half the cache bytes of a K / V pair;
   * a recurrent layer runs in_proj -> conv -> x_proj -> dt_proj -> scan + gate -> out_proj,
-    conv and scan over packed sequences in prefill and one fused step each in decode, the
-    state in per-request slots (engine/kv_cache.py StatePool);
+    conv and scan over packed sequences in prefill; in decode the conv step reads the in_proj
+    slabs, and dt_proj, scan step and gate are one launch; the state is in per-request slots
+    (engine/kv_cache.py StatePool);
   * projections run on the same GEMM plans as the Llama decoder (ops.project / ops.linear):
     weights are padded with zero rows at load where that reaches a kernel's granule.
 
@@ -226,16 +227,15 @@ class SelectiveScan:
             zs.append(z)
         xa = _join(xc)
         dt_in, bc = ops.slab_columns(ops.project(xa, self.w_x, decode), self.rp, 2 * self.np, self.dtype)
-        dt = ops.linear(dt_in, self.w_dt, decode)
         out = []
         for p, y, z in zip(parts, xc, zs):
             m = p.meta
-            args = (y, _split(dt, p, parts), _split(bc, p, parts), 0, self.np, N, z, self.A2, self.D, self.dt_b,
-                    scan_state, m.state_slots)
-            if p.decode:
-                out.append(ops.selective_step(*args, m.positions))
+            r = _split(dt_in, p, parts)
+            args = (_split(bc, p, parts), 0, self.np, N, z, self.A2, self.D, self.dt_b, scan_state, m.state_slots)
+            if p.decode:       # the step projection runs inside the step
+                out.append(ops.selective_step(y, (r, self.w_dt), *args, m.positions))
             else:
-                out.append(ops.selective_scan(*args, m.cu_seqlens, m.prefix_lens, m.max_len))
+                out.append(ops.selective_scan(y, ops.linear(r, self.w_dt), *args, m.cu_seqlens, m.prefix_lens, m.max_len))
         return ops.project(_join(out), self.w_o, decode)
 
 

@@ -1301,9 +1301,14 @@ def selective_scan(x, dt, bc, b_off: int, c_off: int, N: int, z, A2, D, dt_b, st
 
 
 def selective_step(x, dt, bc, b_off: int, c_off: int, N: int, z, A2, D, dt_b, state, slots, positions):
-    """:func:`selective_scan` of one token a row."""
+    """:func:`selective_scan` of one token a row.  ``dt``: the step projection [B, C], or
+    (its input [B, R], its weight [C, R]) -- then bf16 rows run it on MFMA inside the launch."""
+    if isinstance(dt, tuple):
+        if _gpu(x) and x.dtype == torch.bfloat16 and dt[1].shape[1] % 32 == 0:
+            return _native().selective_step(x, None, *dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions)
+        dt = linear(*dt, True)
     if _gpu(x):
-        return _native().selective_step(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions)
+        return _native().selective_step(x, dt, None, None, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions)
     return ref.selective_step(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions)
 
 

@@ -368,6 +368,15 @@ def scan_batch_case(device, dtype):
     S, pos = S0.clone(), [4] * 10 + [0]
     a = (x[:B], dt[:B], bc[:B], 0, N, N, z[:B], *par)
     y = ops.selective_step(*a, S, i32(*slots), i32(*pos))
+    # the step projection inside the step, over more channels and ranks than one MFMA tile
+    R, w = 64, torch.randn(C, 64, generator=g).to(device, dtype) * 0.1
+    r = torch.randn(B, R, generator=g).to(device, dtype)
+    S2, S3 = S0.clone(), S0.clone()
+    wd = (r.float() @ w.float().T)
+    y2 = ops.selective_step(x[:B], (r, w), *a[2:], S2, i32(*slots), i32(*pos))
+    y3 = ops.selective_step(x[:B].float(), wd, *[t.float() if torch.is_tensor(t) else t for t in a[2:]], S3, i32(*slots), i32(*pos))
+    close(y2, y3.cpu(), dtype, "fused step projection")
+    close(S2, S3.cpu(), F32)
     for r in range(B):
         S1 = S0.clone()
         a1 = tuple(t[r:r + 1].contiguous() if torch.is_tensor(t) and t.dim() == 2 and t.shape[0] == B else t for t in a)
