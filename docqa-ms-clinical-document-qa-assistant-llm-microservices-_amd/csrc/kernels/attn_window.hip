@@ -14,11 +14,13 @@
 #include "docqa_common.h"
 #include "docqa_elem.h"
 #include <float.h>
+#include <type_traits>
 
 using namespace docqa;
 
 namespace {
 constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kMaxBT = 256;   // block ids of a row tile's keys staged in LDS (else read per tile)
 
 // LPH lanes per (token, head), V elements a lane at a time; heads [0, H) are queries,
 // [H, H + G) keys
@@ -203,7 +205,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
 typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
 
 template <int DP, int QT, int KB, int NW, bool SHARED, bool SPLIT>
-__global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_t* __restrict__ q,
+__global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_kernel(const uint16_t* __restrict__ q,
                                                                    const uint16_t* __restrict__ kc,
                                                                    const uint16_t* __restrict__ vc,
                                                                    uint16_t* __restrict__ out, WindowArgs a) {
@@ -215,6 +217,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_
   extern __shared__ __attribute__((aligned(16))) char smem[];
   uint16_t* tiles = reinterpret_cast<uint16_t*>(smem);
   float* scales = reinterpret_cast<float*>(tiles + TILES * NT * TILE);   // [TILES][KB]
+  __shared__ int s_bt[kMaxBT];              // block ids of the keys the rows see
 
   const int kvh = blockIdx.x, b = blockIdx.y;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -240,8 +243,15 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_
   const int key0 = a.window > 0 ? max(0, pos_lo - a.window + 1) : 0;
   const int ntiles = (pos_hi - key0) / KB + 1;
 
+  const int blk0 = key0 >> a.log2BS, nblk = (pos_hi >> a.log2BS) - blk0 + 1;
+  const bool bt_lds = nblk <= kMaxBT;
+  if (bt_lds) {
+    for (int i = tid; i < nblk; i += 64 * NW) s_bt[i] = a.block_tables[(size_t)b * a.maxb + blk0 + i];
+    __syncthreads();
+  }
+
   bf16x8 qf[QT][NKS];
-  int pos[QT];
+  int pos[QT], below[QT];                  // a row sees keys in (below, pos]
   float m[QT], l[QT];
   f32x4 o[QT][NDT];
 #pragma unroll
@@ -249,6 +259,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_
     const int r = wrow + t * 16 + fr, rc = min(r, rows - 1);
     const int tok = rc / Gs, h = kvh * Gs + rc % Gs;
     pos[t] = p0 + tok;
+    below[t] = a.window > 0 ? pos[t] - a.window : -1;
     const uint16_t* qp = q + ((size_t)(q0 + tok) * a.H + h) * D;
 #pragma unroll
     for (int ks = 0; ks < NKS; ++ks) {
@@ -269,7 +280,8 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_
   uint4 rk[CPT], rv[SHARED ? 1 : CPT];
   float rs_ = 1.f;
   auto cache_row = [&](int key) {
-    const int blk = a.block_tables[(size_t)b * a.maxb + (key >> a.log2BS)];
+    const int kblk = key >> a.log2BS;
+    const int blk = bt_lds ? s_bt[kblk - blk0] : a.block_tables[(size_t)b * a.maxb + kblk];
     return (size_t)((((blk * a.G + kvh) << a.log2BS)) + (key & (a.BS - 1)));
   };
   auto load = [&](int t) {
@@ -302,10 +314,9 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_
     }
     if (ltid < KB) scales[buf * KB + ltid] = rs_;
   };
-  auto compute = [&](int t, int buf) {
-    const int kb = key0 + t * KB;
-    if (!wlive || kb > wpos_hi || (a.window > 0 && kb + KB - 1 <= wpos_lo - a.window)) return;
-    const bool whole = kb + KB - 1 <= wpos_lo && (a.window <= 0 || kb > wpos_hi - a.window);
+  // one key tile against this wave's rows; `part`: some of its keys are hidden from some rows
+  auto compute_tile = [&](int kb, int buf, auto part) {
+    constexpr bool PART = decltype(part)::value;
     const uint16_t* sk = tiles + buf * NT * TILE;
     const uint16_t* sv = SHARED ? sk : sk + TILE;
     const float* sc = scales + buf * KB;
@@ -332,9 +343,9 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           float v = x[t2][kt][r] * kss[r];
-          if (!whole) {
+          if constexpr (PART) {
             const int key = kb + kt * 16 + g4 * 4 + r;
-            if (key > pos[t2] || (a.window > 0 && key <= pos[t2] - a.window)) v = -INFINITY;
+            v = ((key <= pos[t2]) & (key > below[t2])) ? v : -INFINITY;
           }
           x[t2][kt][r] = v;
           mx = fmaxf(mx, v);
@@ -388,6 +399,15 @@ __global__ __launch_bounds__(64 * NW) void window_attn_mfma_kernel(const uint16_
           o[t2][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pb[t2], o[t2][i], 0, 0, 0);
       }
     }
+  };
+
+  auto compute = [&](int t, int buf) {
+    const int kb = key0 + t * KB;
+    if (!wlive || kb > wpos_hi || (a.window > 0 && kb + KB - 1 <= wpos_lo - a.window)) return;
+    if (kb + KB - 1 <= wpos_lo && (a.window <= 0 || kb > wpos_hi - a.window))
+      compute_tile(kb, buf, std::false_type{});
+    else
+      compute_tile(kb, buf, std::true_type{});
   };
 
   if constexpr (!SPLIT) {
@@ -487,15 +507,19 @@ int launch_mfma(const void* q, const void* kc, const void* vc, void* out, const 
   return 0;
 }
 
-// decode-like launches (the rows of one sequence fit one 16-row tile): waves split the keys;
-// 16 of them when there are too few workgroups to fill the chip
+// decode-like launches (the rows of one sequence fit one 16-row tile): waves split the keys, as
+// many to a workgroup as give a CU 16 of them
 template <int DP, bool SHARED>
 int dispatch_mfma(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
                   hipStream_t s) {
   constexpr int QT = DP <= 128 ? 2 : 1;
   if (max_q * (a.H / a.G) <= 16) {
     if constexpr (DP <= 128) {
-      if ((long long)B * a.G <= 128) return launch_mfma<DP, 1, 32, SHARED ? 16 : 8, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+      const long long wgs = (long long)B * a.G;
+      if constexpr (SHARED) {
+        if (wgs <= 256) return launch_mfma<DP, 1, 32, 16, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+      }
+      if (wgs <= 512) return launch_mfma<DP, 1, 32, 8, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
     }
     return launch_mfma<DP, 1, 32, 4, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
   }

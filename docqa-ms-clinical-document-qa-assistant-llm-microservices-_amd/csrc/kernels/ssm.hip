@@ -11,7 +11,7 @@
 // A sequence whose first token is position 0 starts from zero whatever its slot held, so a
 // slot needs no clearing when it changes hands.
 //
-// MI355X mapping of the scan: one lane owns a channel with all its states in registers
+// MI355X mapping of the scan: one lane owns one or two channels with all their states in registers
 // (LPC lanes a channel when there are more than 32 states), so the recurrence never leaves
 // the lane; B / C of 16 tokens at a time are widened into LDS once a workgroup and broadcast;
 // x, dt and z are loaded 8 tokens ahead.  A long prompt
@@ -29,13 +29,12 @@ constexpr int UB = 8;    // tokens whose x / dt / z are loaded ahead of their us
 
 // ------------------------------------------------------------------ convolution, prefill
 // thread: V channels x TT consecutive tokens, a window of the last K inputs in registers
-template <typename T, int V, int K>
+template <typename T, int V, int K, int TT>
 __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ x, int ldx,
                                                           const float* __restrict__ w, const float* __restrict__ bias,
                                                           T* __restrict__ state, const int* __restrict__ slots,
                                                           const int* __restrict__ cu, const int* __restrict__ ctx,
                                                           T* __restrict__ y, int C, int taps) {
-  constexpr int TT = 8;
   const int b = blockIdx.z, q0 = cu[b], L = cu[b + 1] - q0;
   const int t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * TT;
   const int c0 = (blockIdx.x * 64 + (threadIdx.x & 63)) * V;
@@ -193,27 +192,34 @@ struct ScanArgs {
 
 // LOCAL: the chunk's state from zero and its sum of dt (all chunks but a sequence's last).
 // Otherwise the scan proper, entering from the carried state (chunk 0) or the carry pass.
-template <typename T, int NS, int LPC, bool LOCAL>
+// CPL: channels per lane -- two share a token's loads, address arithmetic and B / C reads.
+template <typename T, int NS, int LPC, int CPL, bool LOCAL>
 __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs a) {
-  constexpr int NSP = NS * LPC, CB = 256 / LPC;
+  constexpr int NSP = NS * LPC, CB = 256 / LPC * CPL;
   __shared__ __attribute__((aligned(16))) float sbc[2][TB][2 * NSP];
   const int b = blockIdx.z, ck = blockIdx.y;
   const int q0 = a.cu[b], L = a.cu[b + 1] - q0;
   const int t_beg = ck * a.chunk, t_end = min(L, t_beg + a.chunk);
   if (t_beg >= L || (LOCAL && t_end >= L)) return;
   const int tid = threadIdx.x;
-  const int c = blockIdx.x * CB + tid / LPC, l = tid % LPC;
+  const int c = blockIdx.x * CB + tid / LPC * CPL, l = tid % LPC;
   const bool ok = c < a.C;
-  const int cc = ok ? c : a.C - 1;
+  const int cc = ok ? c : a.C - CPL;
   const int slot = a.slots[b];
-  const T *x = (const T*)a.x + cc, *dt = (const T*)a.dt + cc, *bc = (const T*)a.bc, *z = (const T*)a.z + cc;
+  const T *X = (const T*)a.x, *DT = (const T*)a.dt, *bc = (const T*)a.bc, *Z = (const T*)a.z;
 
-  float A[NS], S[NS];
+  float A[CPL][NS], S[CPL][NS], Dc[CPL], db[CPL], sum[CPL];
 #pragma unroll
-  for (int i = 0; i < NS; ++i) {
-    const int n = l * NS + i;
-    A[i] = n < a.N ? a.A2[(size_t)cc * a.Np + n] : 0.f;
-    S[i] = 0.f;
+  for (int j = 0; j < CPL; ++j) {
+#pragma unroll
+    for (int i = 0; i < NS; ++i) {
+      const int n = l * NS + i;
+      A[j][i] = n < a.N ? a.A2[(size_t)(cc + j) * a.Np + n] : 0.f;
+      S[j][i] = 0.f;
+    }
+    Dc[j] = a.D[cc + j];
+    db[j] = a.dt_b[cc + j];
+    sum[j] = 0.f;
   }
   if constexpr (!LOCAL) {
     const float* s0 = nullptr;
@@ -221,12 +227,12 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs a) {
     else if (a.ctx[b] > 0 && slot >= 0) s0 = a.state + ((size_t)slot * a.C + cc) * a.Np;
     if (s0) {
 #pragma unroll
-      for (int i = 0; i < NS; ++i)
-        if (l * NS + i < a.N) S[i] = s0[l * NS + i];
+      for (int j = 0; j < CPL; ++j)
+#pragma unroll
+        for (int i = 0; i < NS; ++i)
+          if (l * NS + i < a.N) S[j][i] = s0[(size_t)j * a.Np + l * NS + i];
     }
   }
-  const float Dc = a.D[cc], db = a.dt_b[cc];
-  float sum = 0.f;
 
   auto stage = [&](int t0, int buf) {
     for (int e = tid; e < TB * 2 * NSP; e += 256) {
@@ -238,15 +244,15 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs a) {
     }
   };
   // x, dt, z of UB tokens from t (clamped: a token past the end is computed with dt = 0, which
-  // leaves the state alone, and stores nothing)
-  float xn[UB], dn[UB], zn[UB];
+  // leaves the state alone, and stores nothing); row pointers are uniform, lanes add a column
+  float xn[UB][CPL], dn[UB][CPL], zn[UB][CPL];
   auto fetch = [&](int t0) {
 #pragma unroll
     for (int i = 0; i < UB; ++i) {
-      const int t = min(t0 + i, t_end - 1);
-      xn[i] = ld1(x + (size_t)(q0 + t) * a.C);
-      dn[i] = ld1(dt + (size_t)(q0 + t) * a.C);
-      if constexpr (!LOCAL) zn[i] = ld1(z + (size_t)(q0 + t) * a.ld_z);
+      const size_t r = q0 + min(t0 + i, t_end - 1);
+      ldv<CPL>(X + r * a.C + (unsigned)cc, xn[i]);
+      ldv<CPL>(DT + r * a.C + (unsigned)cc, dn[i]);
+      if constexpr (!LOCAL) ldv<CPL>(Z + r * a.ld_z + (unsigned)cc, zn[i]);
     }
   };
   stage(t_beg, 0);
@@ -257,48 +263,56 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs a) {
     if (t0 + TB < t_end) stage(t0 + TB, buf ^ 1);
 #pragma unroll 1
     for (int u = 0; u < TB; u += UB) {
-      float xv[UB], dv[UB], zv[UB];
+      float xv[UB][CPL], dv[UB][CPL], zv[UB][CPL];
 #pragma unroll
-      for (int i = 0; i < UB; ++i) {
-        xv[i] = xn[i];
-        dv[i] = t0 + u + i < t_end ? softplus_f(dn[i] + db) : 0.f;
-        if constexpr (!LOCAL) zv[i] = silu_fast(zn[i]);
-      }
+      for (int i = 0; i < UB; ++i)
+#pragma unroll
+        for (int j = 0; j < CPL; ++j) {
+          xv[i][j] = xn[i][j];
+          dv[i][j] = t0 + u + i < t_end ? softplus_f(dn[i][j] + db[j]) : 0.f;
+          if constexpr (!LOCAL) zv[i][j] = silu_fast(zn[i][j]);
+        }
       fetch(t0 + u + UB);
 #pragma unroll
       for (int i = 0; i < UB; ++i) {
-        const float d = dv[i], dx = d * xv[i];
         const float* Bt = &sbc[buf][u + i][l * NS];
         const float* Ct = &sbc[buf][u + i][NSP + l * NS];
-        float y = 0.f;
+        float y[CPL];
 #pragma unroll
-        for (int n = 0; n < NS; ++n) {
-          S[n] = __builtin_amdgcn_exp2f(d * A[n]) * S[n] + dx * Bt[n];
-          if constexpr (!LOCAL) y += S[n] * Ct[n];
+        for (int j = 0; j < CPL; ++j) {
+          const float d = dv[i][j], dx = d * xv[i][j];
+          y[j] = 0.f;
+#pragma unroll
+          for (int n = 0; n < NS; ++n) {
+            S[j][n] = __builtin_amdgcn_exp2f(d * A[j][n]) * S[j][n] + dx * Bt[n];
+            if constexpr (!LOCAL) y[j] += S[j][n] * Ct[n];
+          }
+          sum[j] += d;
         }
-        if constexpr (LOCAL) {
-          sum += d;
-        } else {
+        if constexpr (!LOCAL) {
 #pragma unroll
-          for (int o = 1; o < LPC; o <<= 1) y += __shfl_xor(y, o, 64);
+          for (int j = 0; j < CPL; ++j) {
+#pragma unroll
+            for (int o = 1; o < LPC; o <<= 1) y[j] += __shfl_xor(y[j], o, 64);
+            y[j] = (y[j] + Dc[j] * xv[i][j]) * zv[i][j];
+          }
           if (l == 0 && ok && t0 + u + i < t_end)
-            st1((T*)a.y + (size_t)(q0 + t0 + u + i) * a.C + c, (y + Dc * xv[i]) * zv[i]);
+            stv<CPL>((T*)a.y + (size_t)(q0 + t0 + u + i) * a.C + (unsigned)c, y);
         }
       }
     }
   }
   if (!ok) return;
-  if constexpr (LOCAL) {
-    float* o = a.cstate + (((size_t)b * a.nchunk + ck + 1) * a.C + c) * a.Np;   // enters chunk ck + 1
+  float* o = nullptr;
+  if constexpr (LOCAL) o = a.cstate + (((size_t)b * a.nchunk + ck + 1) * a.C + c) * a.Np;   // enters chunk ck + 1
+  else if (t_end == L && slot >= 0) o = a.state + ((size_t)slot * a.C + c) * a.Np;
+  if (!o) return;
+#pragma unroll
+  for (int j = 0; j < CPL; ++j) {
 #pragma unroll
     for (int i = 0; i < NS; ++i)
-      if (l * NS + i < a.N) o[l * NS + i] = S[i];
-    if (l == 0) a.csum[((size_t)b * a.nchunk + ck + 1) * a.C + c] = sum;
-  } else if (t_end == L && slot >= 0) {
-    float* o = a.state + ((size_t)slot * a.C + c) * a.Np;
-#pragma unroll
-    for (int i = 0; i < NS; ++i)
-      if (l * NS + i < a.N) o[l * NS + i] = S[i];
+      if (l * NS + i < a.N) o[(size_t)j * a.Np + l * NS + i] = S[j][i];
+    if (LOCAL && l == 0) a.csum[((size_t)b * a.nchunk + ck + 1) * a.C + c + j] = sum[j];
   }
 }
 
@@ -413,8 +427,15 @@ __global__ __launch_bounds__(256) void selective_step_kernel(ScanArgs a, StepDt 
 template <typename T, int V>
 int launch_conv(const void* x, int ldx, const float* w, const float* b, void* state, const int* slots, const int* cu,
                 const int* ctx, void* y, int B, int max_len, int C, int taps, hipStream_t s) {
-  dim3 grid((C + 64 * V - 1) / (64 * V), (max_len + 31) / 32, B);
-#define GO(K) causal_conv_kernel<T, V, K><<<grid, 256, 0, s>>>((const T*)x, ldx, w, b, (T*)state, slots, cu, ctx, (T*)y, C, taps)
+  const int gx = (C + 64 * V - 1) / (64 * V);
+  // 8 tokens a thread; 2 where that leaves most of the chip without a workgroup
+  const bool few = (long long)gx * ((max_len + 31) / 32) * B < 1024;
+  dim3 grid(gx, few ? (max_len + 7) / 8 : (max_len + 31) / 32, B);
+#define GO(K)                                                                                              \
+  do {                                                                                                     \
+    if (few) causal_conv_kernel<T, V, K, 2><<<grid, 256, 0, s>>>((const T*)x, ldx, w, b, (T*)state, slots, cu, ctx, (T*)y, C, taps); \
+    else causal_conv_kernel<T, V, K, 8><<<grid, 256, 0, s>>>((const T*)x, ldx, w, b, (T*)state, slots, cu, ctx, (T*)y, C, taps);     \
+  } while (0)
   switch (taps) {
     case 2: GO(2); break;
     case 3: GO(3); break;
@@ -443,29 +464,32 @@ int launch_conv_step(const void* P, int S, size_t slab, int ld, const float* w, 
   return 0;
 }
 
-template <typename T, int NS, int LPC>
+template <typename T, int NS, int LPC, int CPL>
 int launch_scan(const ScanArgs& a, int B, hipStream_t s) {
-  dim3 grid((a.C + 256 / LPC - 1) / (256 / LPC), a.nchunk, B);
+  constexpr int CB = 256 / LPC * CPL;
+  dim3 grid((a.C + CB - 1) / CB, a.nchunk, B);
   if (a.nchunk > 1) {
-    selective_scan_kernel<T, NS, LPC, true><<<grid, 256, 0, s>>>(a);
+    selective_scan_kernel<T, NS, LPC, CPL, true><<<grid, 256, 0, s>>>(a);
     DOCQA_CHECK_LAUNCH();
     scan_carry_kernel<<<dim3((a.C * a.Np + 255) / 256, B), 256, 0, s>>>(a);
     DOCQA_CHECK_LAUNCH();
   }
-  selective_scan_kernel<T, NS, LPC, false><<<grid, 256, 0, s>>>(a);
+  selective_scan_kernel<T, NS, LPC, CPL, false><<<grid, 256, 0, s>>>(a);
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
 
 template <typename T>
 int dispatch_scan(const ScanArgs& a, int B, hipStream_t s) {
-  if (a.N <= 8) return launch_scan<T, 8, 1>(a, B, s);
-  if (a.N <= 16) return launch_scan<T, 16, 1>(a, B, s);
-  if (a.N <= 24) return launch_scan<T, 24, 1>(a, B, s);
-  if (a.N <= 32) return launch_scan<T, 32, 1>(a, B, s);
-  if (a.N <= 64) return launch_scan<T, 32, 2>(a, B, s);
-  if (a.N <= 128) return launch_scan<T, 32, 4>(a, B, s);
-  if (a.N <= 256) return launch_scan<T, 32, 8>(a, B, s);
+  const bool pair = a.C % 2 == 0 && a.ld_z % 2 == 0 && docqa_aligned16(a.x) && docqa_aligned16(a.dt) &&
+                    (reinterpret_cast<uintptr_t>(a.z) & 7) == 0 && docqa_aligned16(a.y);
+  if (a.N <= 8) return pair ? launch_scan<T, 8, 1, 2>(a, B, s) : launch_scan<T, 8, 1, 1>(a, B, s);
+  if (a.N <= 16) return pair ? launch_scan<T, 16, 1, 2>(a, B, s) : launch_scan<T, 16, 1, 1>(a, B, s);
+  if (a.N <= 24) return launch_scan<T, 24, 1, 1>(a, B, s);
+  if (a.N <= 32) return launch_scan<T, 32, 1, 1>(a, B, s);
+  if (a.N <= 64) return launch_scan<T, 32, 2, 1>(a, B, s);
+  if (a.N <= 128) return launch_scan<T, 32, 4, 1>(a, B, s);
+  if (a.N <= 256) return launch_scan<T, 32, 8, 1>(a, B, s);
   return -1;
 }
 }  // namespace
