@@ -316,14 +316,14 @@ class HybridModel(Decoder):
 
     # ------------------------------------------------------------------ forward
     def forward(self, input_ids, meta: AttnMeta, caches: list, logits_index=None, greedy_ids: bool = False):
-        """Same contract as :meth:`LlamaModel.forward`; prefill metadata always carries block
+        """Same arguments and result as :meth:`LlamaModel.forward`; prefill metadata always carries block
         tables, prefix lengths and state slots."""
         x = self._hidden(input_ids, [_Part(0, input_ids.shape[0], meta)], meta.slot_mapping, caches)
         return self._head(x, logits_index, greedy_ids)
 
     def forward_mixed(self, input_ids, n_dec: int, dmeta: AttnMeta, pmeta: AttnMeta, caches: list, logits_index,
                       return_logits: bool = False):
-        """Same contract as :meth:`LlamaModel.forward_mixed`: rows [0, n_dec) decode, the rest
+        """Same arguments and result as :meth:`LlamaModel.forward_mixed`: rows [0, n_dec) decode, the rest
         prompt portions; projections run over all rows at once."""
         T = input_ids.shape[0]
         parts = ([_Part(0, n_dec, dmeta)] if n_dec else []) + ([_Part(n_dec, T, pmeta)] if T > n_dec else [])
