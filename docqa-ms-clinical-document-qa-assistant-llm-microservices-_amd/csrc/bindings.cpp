@@ -969,7 +969,8 @@ at::Tensor pgemm(const at::Tensor& x, const at::Tensor& w, int64_t epi) {
   CHECK_ALIGN16(x); CHECK_ALIGN16(w);
   const int K = x.size(-1), N = w.size(0);
   TORCH_CHECK(w.size(1) == K, "pgemm: K mismatch");
-  TORCH_CHECK(epi == 0 || epi == 1 || epi == 3, "pgemm: epi must be 0 (bf16), 1 (SwiGLU) or 3 (squared ReLU)");
+  TORCH_CHECK(epi == 0 || epi == 1 || epi == 3 || epi == 4,
+              "pgemm: epi must be 0 (bf16), 1 (SwiGLU), 3 (squared ReLU) or 4 (tanh GELU)");
   const int M = x.numel() / K;
   TORCH_CHECK(M == 0 || docqa_pgemm_ok(M, N, K), "pgemm: unsupported shape M=", M, " N=", N, " K=", K,
               " (N % 256, K % 128, 32-bit row offsets)");

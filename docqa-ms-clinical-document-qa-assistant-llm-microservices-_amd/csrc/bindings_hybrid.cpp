@@ -89,27 +89,90 @@ std::tuple<Tensor, Tensor, Tensor> embed_scale_rmsnorm(const Tensor& ids, const 
   return {res, emb, out};
 }
 
-Tensor squared_relu(const Tensor& P, bool out_f32) {
+// residual += m (P + Q); the bf16 copy of it (empty when out_f32)
+Tensor add_scaled(const Tensor& P, const OptT& Q, Tensor residual, double m, bool out_f32) {
+  const Slabs p = slabs_of(P);
+  CHECK_GPU(residual); CHECK_F32(residual); CHECK_CONTIG(residual);
+  TORCH_CHECK(residual.dim() == 2 && residual.size(0) == p.M && residual.size(1) == p.N, "residual shape mismatch");
+  CHECK_ALIGN16(P); CHECK_ALIGN16(residual);
+  Slabs q{1, p.M, p.N, 0};
+  if (Q.has_value()) {
+    q = slabs_of(*Q);
+    TORCH_CHECK(q.M == p.M && q.N == p.N, "Q shape mismatch");
+    CHECK_ALIGN16(*Q);
+  }
+  c10::DeviceGuard g(P.device());
+  auto out = at::empty(out_f32 ? at::IntArrayRef({0}) : residual.sizes(), P.options().dtype(at::kBFloat16));
+  CHECK_RC(docqa_add_scaled(P.data_ptr(), is_f32(P), p.S, Q.has_value() ? Q->data_ptr() : nullptr,
+                            Q.has_value() && is_f32(*Q), q.S, residual.data_ptr<float>(), (float)m,
+                            out_f32 ? nullptr : out.data_ptr(), (size_t)p.M * p.N, stream()),
+           "add_scaled");
+  return out;
+}
+
+Tensor soft_cap(const Tensor& x, double cap) {
+  CHECK_ACT(x); CHECK_CONTIG(x);
+  TORCH_CHECK(cap > 0, "cap");
+  c10::DeviceGuard g(x.device());
+  auto out = at::empty(x.sizes(), x.options().dtype(at::kFloat));
+  CHECK_RC(docqa_soft_cap(x.data_ptr(), is_f32(x), out.data_ptr<float>(), x.numel(), (float)cap, stream()), "soft_cap");
+  return out;
+}
+
+void check_side(const Slabs& p, const Tensor& ids, const Tensor& table, int64_t col, int64_t n) {
+  CHECK_ACT(table); CHECK_CONTIG(table); CHECK_ALIGN16(table);
+  TORCH_CHECK(table.dim() == 2 && col >= 0 && n >= 0 && n <= p.N && col + n <= table.size(1), "side columns");
+  check_i32(ids, p.M, "ids");
+}
+
+Tensor side_gate(const Tensor& P, const Tensor& ids, const Tensor& table, int64_t col, int64_t n, bool out_f32) {
+  const Slabs p = slabs_of(P);
+  check_side(p, ids, table, col, n);
+  CHECK_ALIGN16(P);
+  TORCH_CHECK(out_f32 == is_f32(table), "side_gate: the output has the table's dtype");
+  c10::DeviceGuard g(P.device());
+  auto out = at::empty({p.M, p.N}, table.options());
+  CHECK_RC(docqa_side_gate(P.data_ptr(), is_f32(P), p.S, p.M, p.N, ids.data_ptr<int>(), table.data_ptr(), out_f32,
+                           (int)table.size(1), (int)table.size(0), (int)col, (int)n, out.data_ptr(), stream()),
+           "side_gate");
+  return out;
+}
+
+Tensor side_project(const Tensor& P, const Tensor& ids, const Tensor& table, int64_t col, int64_t n, const Tensor& w) {
+  const Slabs p = slabs_of(P);
+  check_side(p, ids, table, col, n);
+  CHECK_BF16(table); CHECK_BF16(w); CHECK_GPU(w); CHECK_CONTIG(w);
+  TORCH_CHECK(w.dim() == 2 && w.size(1) == p.N, "side_project: w must be [width, N]");
+  c10::DeviceGuard g(P.device());
+  auto out = at::empty({p.M, w.size(0)}, table.options());
+  CHECK_RC(docqa_side_project(P.data_ptr(), is_f32(P), p.S, p.M, p.N, ids.data_ptr<int>(), table.data_ptr(),
+                              (int)table.size(1), (int)table.size(0), (int)col, (int)n, w.data_ptr(), (int)w.size(0),
+                              out.data_ptr(), stream()),
+           "side_project");
+  return out;
+}
+
+Tensor slab_activation(const Tensor& P, int64_t act, bool out_f32) {
   const Slabs p = slabs_of(P);
   CHECK_ALIGN16(P);
   c10::DeviceGuard g(P.device());
   auto out = at::empty({p.M, p.N}, P.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
-  CHECK_RC(docqa_squared_relu(P.data_ptr(), is_f32(P), p.S, p.slab, out.data_ptr(), out_f32, stream()),
-           "squared_relu");
+  CHECK_RC(docqa_slab_activation(P.data_ptr(), is_f32(P), p.S, p.slab, (int)act, out.data_ptr(), out_f32, stream()),
+           "slab_activation");
   return out;
 }
 
-// squared ReLU of x . w^T on the decode GEMMs: skinny up to 192 rows, the mid-M kernel beyond
-Tensor decode_relu2(const Tensor& x, const Tensor& w) {
+// act(x . w^T) on the decode GEMMs: skinny up to 192 rows, the mid-M kernel beyond
+Tensor decode_act(const Tensor& x, const Tensor& w, int64_t act) {
   CHECK_GPU(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_CONTIG(x); CHECK_CONTIG(w); CHECK_ALIGN16(x); CHECK_ALIGN16(w);
-  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1), "decode_relu2: shapes");
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1), "decode_act: shapes");
   const int M = x.size(0), N = w.size(0), K = x.size(1);
   c10::DeviceGuard g(x.device());
   auto out = at::empty({M, N}, x.options());
   CHECK_RC(M <= 192 && N % 64 == 0 && K % 512 == 0
-               ? docqa_dgemm_relu2(x.data_ptr(), w.data_ptr(), out.data_ptr(), M, N, K, stream())
-               : docqa_mgemm_relu2(x.data_ptr(), w.data_ptr(), out.data_ptr(), M, N, K, stream()),
-           "decode_relu2");
+               ? docqa_dgemm_act(x.data_ptr(), w.data_ptr(), out.data_ptr(), (int)act, M, N, K, stream())
+               : docqa_mgemm_act(x.data_ptr(), w.data_ptr(), out.data_ptr(), (int)act, M, N, K, stream()),
+           "decode_act");
   return out;
 }
 
@@ -151,12 +214,13 @@ Tensor qk_norm_store(const Tensor& P, const Tensor& w, const Tensor& slots, Tens
 // row with ctx the context lengths (decode)
 Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, const OptT& k_scale,
                    const Tensor& block_tables, const OptT& cu, const Tensor& ctx, int64_t max_q, double scale,
-                   int64_t window, const OptT& sink) {
+                   int64_t window, const OptT& sink, int64_t v_dim) {
   CHECK_ACT(q); CHECK_CONTIG(q); CHECK_CONTIG(k_cache);
   TORCH_CHECK(k_cache.dim() == 4 && k_cache.scalar_type() == q.scalar_type(), "k_cache dtype / shape");
   const int G = k_cache.size(1), BS = k_cache.size(2), D = k_cache.size(3);
   TORCH_CHECK(q.dim() == 2 && q.size(1) % D == 0, "q must be [rows, H * dim]");
-  const int H = q.size(1) / D, B = block_tables.size(0);
+  const int H = q.size(1) / D, B = block_tables.size(0), DV = v_dim ? v_dim : D;
+  TORCH_CHECK(DV >= 1 && DV <= D && (DV == D || !v_cache.has_value()), "v_dim: part of the shared row");
   CHECK_GPU(block_tables); CHECK_I32(block_tables); CHECK_CONTIG(block_tables);
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(1) >= 1, "block_tables must be [B, blocks]");
   check_i32(ctx, B, "ctx");
@@ -170,29 +234,117 @@ Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, 
   if (sink.has_value()) check_vec(*sink, H, "sink");
   c10::DeviceGuard g(q.device());
   CHECK_ALIGN16(k_cache);     // cached rows are read in 16-byte pieces, q row by row
-  auto out = at::empty_like(q);
+  auto out = at::empty({q.size(0), (int64_t)H * DV}, q.options());
   CHECK_RC(docqa_window_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.has_value() ? v_cache->data_ptr() : k_cache.data_ptr(),
                              k_scale.has_value() ? k_scale->data_ptr<float>() : nullptr, block_tables.data_ptr<int>(),
                              (int)block_tables.size(1), cu.has_value() ? cu->data_ptr<int>() : nullptr,
                              ctx.data_ptr<int>(), sink.has_value() ? sink->data_ptr<float>() : nullptr,
-                             out.data_ptr(), is_f32(q), B, (int)max_q, H, G, D, BS, (float)scale, (int)window,
+                             out.data_ptr(), is_f32(q), B, (int)max_q, H, G, D, DV, BS, (float)scale, (int)window,
                              stream()),
            "window_attn");
   return out;
 }
 
-void check_conv(const Tensor& w, const Tensor& bias, const Tensor& state, int C, int& taps) {
+Tensor packed_window_attn(const Tensor& q, const Tensor& kv, const Tensor& kr, int64_t H, int64_t dim, int64_t vdim,
+                          const Tensor& cu, const Tensor& cu_k, int64_t max_q, double scale, int64_t window,
+                          const OptT& sink) {
+  CHECK_GPU(q); CHECK_BF16(q); CHECK_BF16(kv); CHECK_BF16(kr); CHECK_CONTIG(q); CHECK_CONTIG(kv); CHECK_CONTIG(kr);
+  CHECK_GPU(kv); CHECK_GPU(kr);
+  TORCH_CHECK(q.dim() == 2 && kv.dim() == 2 && kr.dim() == 2 && kr.size(0) == kv.size(0) && H >= 1, "packed_window_attn: shapes");
+  const int64_t r8 = kr.size(1), d8 = (dim + 7) / 8 * 8;
+  TORCH_CHECK(q.size(1) == H * (d8 + r8), "packed_window_attn: query width");
+  const int B = cu.numel() - 1;
+  check_i32(cu, B + 1, "cu"); check_i32(cu_k, B + 1, "cu_k");
+  if (sink.has_value()) check_vec(*sink, H, "sink");
+  c10::DeviceGuard g(q.device());
+  auto out = at::empty({q.size(0), H * vdim}, q.options());
+  CHECK_RC(docqa_packed_window_attn(q.data_ptr(), kv.data_ptr(), kr.data_ptr(), cu.data_ptr<int>(), cu_k.data_ptr<int>(),
+                                    sink.has_value() ? sink->data_ptr<float>() : nullptr, out.data_ptr(), B, (int)max_q,
+                                    (int)H, (int)d8, (int)r8, (int)vdim, (int)kv.size(1), (float)scale, (int)window,
+                                    stream()),
+           "packed_window_attn");
+  return out;
+}
+
+Tensor rope_table(const Tensor& positions, const Tensor& freq) {
+  const int T = positions.numel(), half = freq.numel();
+  check_i32(positions, T, "positions");
+  TORCH_CHECK(freq.is_cuda() && freq.scalar_type() == at::kDouble && freq.is_contiguous(), "freq: fp64 vector expected");
+  c10::DeviceGuard g(positions.device());
+  auto out = at::empty({T, 2 * half}, positions.options().dtype(at::kFloat));
+  CHECK_RC(docqa_rope_table(positions.data_ptr<int>(), freq.data_ptr<double>(), out.data_ptr<float>(), T, half, stream()),
+           "rope_table");
+  return out;
+}
+
+// P: [q: H (dim + r) | latent: rank | r] (c_norm) or the query heads only -> rotated query heads
+Tensor latent_store(const Tensor& P, const Tensor& cs, const Tensor& slots, Tensor cache, const OptT& c_norm, int64_t H,
+                    int64_t dim, int64_t rank, double eps) {
+  const Slabs p = slabs_of(P);
+  CHECK_ACT(cache); CHECK_CONTIG(cache); CHECK_ALIGN16(cache); CHECK_ALIGN16(P); CHECK_ALIGN16(cs);
+  TORCH_CHECK(cs.dim() == 2, "cs must be [tokens, r]");
+  const int64_t r = cs.size(1), d8 = (dim + 7) / 8 * 8, r8 = (r + 7) / 8 * 8;
+  check_vec(cs, p.M * r, "cs");
+  check_i32(slots, p.M, "slots");
+  TORCH_CHECK(cache.dim() == 4 && cache.size(1) == 1 && cache.size(3) == (rank + 7) / 8 * 8 + r8,
+              "cache must be [blocks, 1, block, latent + rotated part]");
+  TORCH_CHECK(p.N >= H * (dim + r) + (c_norm.has_value() ? rank + r : 0), "latent_store: projection width");
+  if (c_norm.has_value()) {
+    check_vec(*c_norm, rank, "c_norm");
+    CHECK_ALIGN16(*c_norm);
+  }
+  c10::DeviceGuard g(P.device());
+  auto q = at::empty({p.M, H * (d8 + r8)}, cache.options());
+  CHECK_RC(docqa_latent_store(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, cs.data_ptr<float>(), slots.data_ptr<int>(),
+                              c_norm.has_value() ? c_norm->data_ptr<float>() : nullptr, q.data_ptr(), cache.data_ptr(),
+                              is_f32(cache), p.M, (int)H, (int)dim, (int)r, (int)rank, (int)cache.size(2), (float)eps,
+                              stream()),
+           "latent_store");
+  return q;
+}
+
+Tensor head_project(const Tensor& x, const Tensor& w, int64_t carry) {
+  CHECK_GPU(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_GPU(w); CHECK_CONTIG(x); CHECK_CONTIG(w);
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && carry >= 0 && x.size(1) == w.size(0) * (w.size(2) + carry), "head_project: shapes");
+  c10::DeviceGuard g(x.device());
+  auto y = at::empty({x.size(0), w.size(0) * (w.size(1) + carry)}, x.options());
+  CHECK_RC(docqa_head_project(x.data_ptr(), w.data_ptr(), y.data_ptr(), (int)x.size(0), (int)w.size(0), (int)w.size(2),
+                              (int)w.size(1), (int)carry, stream()),
+           "head_project");
+  return y;
+}
+
+std::tuple<Tensor, Tensor> latent_gather(const Tensor& cache, const Tensor& block_tables, const Tensor& first,
+                                         const Tensor& cu_k, int64_t total, int64_t rank) {
+  CHECK_GPU(cache); CHECK_BF16(cache); CHECK_CONTIG(cache); CHECK_ALIGN16(cache);
+  TORCH_CHECK(cache.dim() == 4 && cache.size(1) == 1 && rank >= 8 && rank < cache.size(3), "latent_gather: cache");
+  const int B = block_tables.size(0);
+  CHECK_GPU(block_tables); CHECK_I32(block_tables); CHECK_CONTIG(block_tables);
+  check_i32(first, B, "first"); check_i32(cu_k, B + 1, "cu_k");
+  c10::DeviceGuard g(cache.device());
+  const int64_t r8 = cache.size(3) - rank;
+  auto c = at::empty({total, rank}, cache.options()), kr = at::empty({total, r8}, cache.options());
+  // a sequence's keys are at most the table's blocks, and at most all of them
+  const int64_t most = std::min<int64_t>(total, block_tables.size(1) * cache.size(2));
+  CHECK_RC(docqa_latent_gather(cache.data_ptr(), block_tables.data_ptr<int>(), (int)block_tables.size(1),
+                               first.data_ptr<int>(), cu_k.data_ptr<int>(), c.data_ptr(), kr.data_ptr(), B, (int)most,
+                               (int)rank, (int)r8, (int)cache.size(2), stream()),
+           "latent_gather");
+  return {c, kr};
+}
+
+void check_conv(const Tensor& w, const OptT& bias, const Tensor& state, int C, int& taps) {
   TORCH_CHECK(w.dim() == 2 && w.size(1) == C, "conv weight must be [taps, channels]");
   taps = w.size(0);
   check_vec(w, (int64_t)taps * C, "conv weight");
-  check_vec(bias, C, "conv bias");
+  if (bias.has_value()) check_vec(*bias, C, "conv bias");
   CHECK_CONTIG(state);
   TORCH_CHECK(state.dim() == 3 && state.size(1) == taps - 1 && state.size(2) == C, "conv state must be [slots, taps - 1, channels]");
 }
 
 // x: [tokens, >= C] rows (the first C columns are convolved); advances the sequences' state
-Tensor causal_conv(const Tensor& x, const Tensor& w, const Tensor& bias, Tensor state, const Tensor& slots,
-                   const Tensor& cu, const Tensor& ctx, int64_t max_len) {
+Tensor causal_conv(const Tensor& x, const Tensor& w, const OptT& bias, Tensor state, const Tensor& slots,
+                   const Tensor& cu, const Tensor& ctx, int64_t max_len, bool silu) {
   CHECK_ACT(x);
   const int C = w.size(1), T = x.size(0), B = cu.numel() - 1;
   int taps;
@@ -202,29 +354,31 @@ Tensor causal_conv(const Tensor& x, const Tensor& w, const Tensor& bias, Tensor 
   check_i32(slots, B, "slots"); check_i32(cu, B + 1, "cu"); check_i32(ctx, B, "ctx");
   c10::DeviceGuard g(x.device());
   auto y = at::empty({T, C}, x.options());
-  CHECK_RC(docqa_causal_conv(x.data_ptr(), (int)x.stride(0), w.data_ptr<float>(), bias.data_ptr<float>(),
-                             state.data_ptr(), slots.data_ptr<int>(), cu.data_ptr<int>(), ctx.data_ptr<int>(),
-                             y.data_ptr(), is_f32(x), B, (int)max_len, C, taps, stream()),
+  CHECK_RC(docqa_causal_conv(x.data_ptr(), (int)x.stride(0), w.data_ptr<float>(),
+                             bias.has_value() ? bias->data_ptr<float>() : nullptr, state.data_ptr(), slots.data_ptr<int>(), cu.data_ptr<int>(), ctx.data_ptr<int>(),
+                             y.data_ptr(), is_f32(x), B, (int)max_len, C, taps, silu, stream()),
            "causal_conv");
   return y;
 }
 
-// P: [x: C | z: C] input projection of one token a row -> (silu(conv x), z)
-std::tuple<Tensor, Tensor> conv_step(const Tensor& P, const Tensor& w, const Tensor& bias, Tensor state,
-                                     const Tensor& slots, const Tensor& positions) {
+// P: [x: C | z: C] input projection of one token a row -> (conv x, z); [x: C] -> (conv x, empty)
+std::tuple<Tensor, Tensor> conv_step(const Tensor& P, const Tensor& w, const OptT& bias, Tensor state,
+                                     const Tensor& slots, const Tensor& positions, bool silu) {
   const Slabs p = slabs_of(P);
   const int C = w.size(1);
   int taps;
   check_conv(w, bias, state, C, taps);
   CHECK_ACT(state);
-  TORCH_CHECK(p.N == 2 * C, "conv_step: P must be [.., 2 C] wide");
+  TORCH_CHECK(p.N == 2 * C || p.N == C, "conv_step: P must be [.., C] or [.., 2 C] wide");
+  const bool gated = p.N == 2 * C;
   TORCH_CHECK(is_f32(P) || !is_f32(state), "conv_step: fp32 state needs fp32 projections");
   check_i32(slots, p.M, "slots"); check_i32(positions, p.M, "positions");
   c10::DeviceGuard g(P.device());
-  auto y = at::empty({p.M, C}, state.options()), z = at::empty({p.M, C}, state.options());
-  CHECK_RC(docqa_conv_step(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, w.data_ptr<float>(), bias.data_ptr<float>(),
+  auto y = at::empty({p.M, C}, state.options()), z = at::empty({gated ? p.M : 0, C}, state.options());
+  CHECK_RC(docqa_conv_step(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, w.data_ptr<float>(),
+                           bias.has_value() ? bias->data_ptr<float>() : nullptr,
                            state.data_ptr(), slots.data_ptr<int>(), positions.data_ptr<int>(), y.data_ptr(),
-                           z.data_ptr(), is_f32(state), p.M, C, taps, stream()),
+                           gated ? z.data_ptr() : nullptr, is_f32(state), p.M, C, taps, silu, stream()),
            "conv_step");
   return {y, z};
 }
@@ -310,16 +464,28 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
         "bool out_f32) -> Tensor");
   m.def("embed_scale_rmsnorm(Tensor ids, Tensor table, float scale, Tensor w, float eps, bool keep) "
         "-> (Tensor, Tensor, Tensor)");
-  m.def("decode_relu2(Tensor x, Tensor w) -> Tensor");
+  m.def("decode_act(Tensor x, Tensor w, int act) -> Tensor");
+  m.def("add_scaled(Tensor P, Tensor? Q, Tensor(a!) residual, float m, bool out_f32) -> Tensor");
+  m.def("soft_cap(Tensor x, float cap) -> Tensor");
+  m.def("side_gate(Tensor P, Tensor ids, Tensor table, int col, int n, bool out_f32) -> Tensor");
+  m.def("side_project(Tensor P, Tensor ids, Tensor table, int col, int n, Tensor w) -> Tensor");
+  m.def("packed_window_attn(Tensor q, Tensor kv, Tensor kr, int H, int dim, int vdim, Tensor cu, Tensor cu_k, int max_q, "
+        "float scale, int window, Tensor? sink) -> Tensor");
+  m.def("rope_table(Tensor positions, Tensor freq) -> Tensor");
+  m.def("latent_store(Tensor P, Tensor cs, Tensor slots, Tensor(a!) cache, Tensor? c_norm, int H, int dim, int rank, "
+        "float eps) -> Tensor");
+  m.def("head_project(Tensor x, Tensor w, int carry) -> Tensor");
+  m.def("latent_gather(Tensor cache, Tensor block_tables, Tensor first, Tensor cu_k, int total, int rank) "
+        "-> (Tensor, Tensor)");
   m.def("slab_columns(Tensor P, int n0, int n1, bool out_f32) -> (Tensor, Tensor)");
-  m.def("squared_relu(Tensor P, bool out_f32) -> Tensor");
+  m.def("slab_activation(Tensor P, int act, bool out_f32) -> Tensor");
   m.def("qk_norm_store(Tensor P, Tensor w, Tensor slots, Tensor(a!) k_cache, Tensor(b!) k_scale, int H, float eps) "
         "-> Tensor");
   m.def("window_attn(Tensor q, Tensor k_cache, Tensor? v_cache, Tensor? k_scale, Tensor block_tables, Tensor? cu, "
-        "Tensor ctx, int max_q, float scale, int window, Tensor? sink) -> Tensor");
-  m.def("causal_conv(Tensor x, Tensor w, Tensor bias, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, "
-        "int max_len) -> Tensor");
-  m.def("conv_step(Tensor P, Tensor w, Tensor bias, Tensor(a!) state, Tensor slots, Tensor positions) "
+        "Tensor ctx, int max_q, float scale, int window, Tensor? sink, int v_dim) -> Tensor");
+  m.def("causal_conv(Tensor x, Tensor w, Tensor? bias, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, "
+        "int max_len, bool silu) -> Tensor");
+  m.def("conv_step(Tensor P, Tensor w, Tensor? bias, Tensor(a!) state, Tensor slots, Tensor positions, bool silu) "
         "-> (Tensor, Tensor)");
   m.def("selective_scan(Tensor x, Tensor dt, Tensor bc, int b_off, int c_off, int N, Tensor z, Tensor A2, Tensor D, "
         "Tensor dt_b, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, int max_len, int chunk) -> Tensor");
@@ -330,9 +496,18 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
 TORCH_LIBRARY_IMPL(docqa, CUDA, m) {
   m.impl("sandwich_rmsnorm", &sandwich_rmsnorm);
   m.impl("embed_scale_rmsnorm", &embed_scale_rmsnorm);
-  m.impl("decode_relu2", &decode_relu2);
+  m.impl("decode_act", &decode_act);
+  m.impl("add_scaled", &add_scaled);
+  m.impl("soft_cap", &soft_cap);
+  m.impl("side_gate", &side_gate);
+  m.impl("side_project", &side_project);
+  m.impl("packed_window_attn", &packed_window_attn);
+  m.impl("rope_table", &rope_table);
+  m.impl("latent_store", &latent_store);
+  m.impl("head_project", &head_project);
+  m.impl("latent_gather", &latent_gather);
   m.impl("slab_columns", &slab_columns);
-  m.impl("squared_relu", &squared_relu);
+  m.impl("slab_activation", &slab_activation);
   m.impl("qk_norm_store", &qk_norm_store);
   m.impl("window_attn", &window_attn);
   m.impl("causal_conv", &causal_conv);

@@ -52,6 +52,18 @@ __device__ __forceinline__ float relu2(float v) {
   return r * r;
 }
 
+// tanh form of GELU: 0.5 v (1 + tanh u) = v / (1 + e^-2u), u = sqrt(2 / pi) (v + 0.044715 v^3)
+__device__ __forceinline__ float gelu_tanh(float v) {
+  const float u = 0.7978845608028654f * (v + 0.044715f * v * v * v);
+  return v / (1.f + __expf(-2.f * u));
+}
+// the feed-forward activations a GEMM epilogue can apply
+enum { ACT_RELU2 = 0, ACT_GELU_TANH = 1 };
+template <int ACT>
+__device__ __forceinline__ float act_f(float v) {
+  return ACT == ACT_RELU2 ? relu2(v) : gelu_tanh(v);
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);

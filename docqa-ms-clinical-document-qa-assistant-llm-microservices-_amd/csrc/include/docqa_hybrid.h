@@ -1,5 +1,6 @@
-// docqa_hybrid.h -- host launchers of the kernels behind hybrid recurrent / windowed-attention
-// decoders (sandwich_norm.hip, attn_window.hip, ssm.hip, act.hip squared ReLU).  Same rules as
+// docqa_hybrid.h -- host launchers of the kernels behind hybrid recurrent / windowed- and latent-
+// attention decoders (sandwich_norm.hip, attn_window.hip, attn_latent.hip, side_input.hip, ssm.hip,
+// act.hip).  Same rules as
 // docqa_kernels.h: 0 on success, negative for an unsupported shape, else a hipError_t; nothing
 // is allocated and nothing synchronises.  "f32" flags pick fp32 over bf16 storage; P operands
 // are S split-K slabs (S = 1: the product itself).
@@ -12,28 +13,50 @@ int docqa_sandwich_rmsnorm(const void* P, int p_f32, int S, float* res, const fl
                            const float* w_next, void* out, int out_f32, int rows, int H, float eps, hipStream_t s);
 int docqa_embed_scale_rmsnorm(const int* ids, const void* table, int f32, float scale, const float* w, float* res,
                               float* emb, void* out, int rows, int H, int vocab, float eps, hipStream_t s);
-// Y [M, N] = squared ReLU of X [M, K] . W [N, K]^T, bf16 (dgemm.hip: M <= 192, N % 64, K % 512;
-// mgemm.hip: N % 128, K % 128)
-int docqa_dgemm_relu2(const void* X, const void* W, void* Y, int M, int N, int K, hipStream_t s);
-int docqa_mgemm_relu2(const void* X, const void* W, void* Y, int M, int N, int K, hipStream_t s);
+// res [n] += m (P + Q) (Q null: P alone), each with its own slab count; out null or bf16 [n]: a copy of res
+int docqa_add_scaled(const void* P, int p_f32, int SP, const void* Q, int q_f32, int SQ, float* res, float m, void* out,
+                     size_t n, hipStream_t s);
+// Y [M, N] = act(X [M, K] . W [N, K]^T), bf16, act: docqa_common.h ACT_* (dgemm.hip: M <= 192, N % 64,
+// K % 512; mgemm.hip: N % 128, K % 128)
+int docqa_dgemm_act(const void* X, const void* W, void* Y, int act, int M, int N, int K, hipStream_t s);
+int docqa_mgemm_act(const void* X, const void* W, void* Y, int act, int M, int N, int K, hipStream_t s);
 int docqa_slab_columns(const void* P, int p_f32, int S, int T, int ld, void* out0, int n0, void* out1, int n1,
                        int out_f32, hipStream_t s);
-int docqa_squared_relu(const void* P, int p_f32, int S, size_t n, void* out, int out_f32, hipStream_t s);
+int docqa_slab_activation(const void* P, int p_f32, int S, size_t n, int act, void* out, int out_f32, hipStream_t s);
+int docqa_soft_cap(const void* x, int f32, float* out, size_t n, float cap, hipStream_t s);
+// g [M, N] = gelu_tanh(P) * table[ids][col + c] (c < n, else 0); side_project: y [M, W] = g . w [W, N]^T (bf16)
+int docqa_side_gate(const void* P, int p_f32, int S, int M, int N, const int* ids, const void* table, int f32, int ld,
+                    int vocab, int col, int n, void* out, hipStream_t s);
+int docqa_side_project(const void* P, int p_f32, int S, int M, int N, const int* ids, const void* table, int ld,
+                       int vocab, int col, int n, const void* w, int W, void* out, hipStream_t s);
 
 int docqa_qk_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* wq, const int* slots,
                         void* q, void* kc, float* ks, int f32, int tokens, int H, int G, int D, int BS, float eps,
                         hipStream_t s);
-// cu null: decode (one query token a row, ctx = context length including it)
+// cu null: decode (one query token a row, ctx = context length including it); DV: value elements of a row
 int docqa_window_attn(const void* q, const void* kc, const void* vc, const float* k_scale, const int* block_tables,
                       int maxb, const int* cu, const int* ctx, const float* sink, void* out, int f32, int B,
-                      int max_q, int H, int G, int D, int BS, float scale, int window, hipStream_t s);
+                      int max_q, int H, int G, int D, int DV, int BS, float scale, int window, hipStream_t s);
+// kv [keys, ld] rows [H x d8 keys | H x v8 values], kr [keys, r8]; bf16
+int docqa_packed_window_attn(const void* q, const void* kv, const void* kr, const int* cu, const int* cu_k,
+                             const float* sink, void* out, int B, int max_q, int H, int d8, int r8, int vdim, int ld,
+                             float scale, int window, hipStream_t s);
+
+int docqa_rope_table(const int* positions, const double* freq, float* out, int T, int half, hipStream_t s);
+// c_norm null: the projection holds query heads only
+int docqa_latent_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* cs, const int* slots,
+                       const float* c_norm, void* q, void* cache, int f32, int T, int H, int d, int r, int R, int BS,
+                       float eps, hipStream_t s);
+int docqa_head_project(const void* x, const void* w, void* y, int T, int H, int K, int N, int E, hipStream_t s);
+int docqa_latent_gather(const void* cache, const int* block_tables, int maxb, const int* first, const int* cu_k, void* c,
+                        void* kr, int B, int max_keys, int R8, int r8, int BS, hipStream_t s);
 
 int docqa_causal_conv(const void* x, int ldx, const float* w, const float* b, void* state, const int* slots,
                       const int* cu, const int* ctx, void* y, int f32, int B, int max_len, int C, int taps,
-                      hipStream_t s);
+                      int silu, hipStream_t s);
 int docqa_conv_step(const void* P, int p_f32, int S, size_t slab, int ld, const float* w, const float* b, void* state,
                     const int* slots, const int* positions, void* y, void* z, int f32, int B, int C, int taps,
-                    hipStream_t s);
+                    int silu, hipStream_t s);
 int docqa_selective_scan(const void* x, const void* dt, const void* bc, int ld_bc, int b_off, int c_off,
                          const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
                          const int* slots, const int* cu, const int* ctx, void* y, float* cstate, float* csum,

@@ -206,19 +206,28 @@ int docqa_bias_act(const void* x, const void* bias, const void* res, void* out, 
   return 0;
 }
 
-// squared ReLU of a projection given as S split-K slabs (or its one [n] product), fp32 or
-// bf16 in, fp32 or bf16 out: out = max(sum_s P[s], 0)^2
-template <int V, typename PT, typename OT>
-__global__ __launch_bounds__(256) void squared_relu_kernel(const PT* __restrict__ P, int S, size_t n,
+// activation of a projection given as S split-K slabs (or its one [n] product), fp32 or
+// bf16 in, fp32 or bf16 out: out = act(sum_s P[s])
+template <int ACT, int V, typename PT, typename OT>
+__global__ __launch_bounds__(256) void slab_activation_kernel(const PT* __restrict__ P, int S, size_t n,
                                                            OT* __restrict__ out) {
   const size_t step = (size_t)gridDim.x * 256 * V;
   for (size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * V; i < n; i += step) {
     float f[V];
     ld_slabs<V>(P + i, S, n, f);
 #pragma unroll
-    for (int j = 0; j < V; ++j) f[j] = relu2(f[j]);
+    for (int j = 0; j < V; ++j) f[j] = act_f<ACT>(f[j]);
     stv<V>(out + i, f);
   }
+}
+
+// cap tanh(x / cap), fp32 out
+template <typename T>
+__global__ __launch_bounds__(256) void soft_cap_kernel(const T* __restrict__ x, float* __restrict__ out, size_t n,
+                                                       float cap) {
+  const float inv = 1.f / cap;
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256)
+    out[i] = cap * tanhf(ld1(x + i) * inv);
 }
 
 // columns [0, n0) and [n0, n0 + n1) of a projection given as S split-K slabs [S, T, ld] (or its
@@ -258,25 +267,42 @@ int docqa_slab_columns(const void* P, int p_f32, int S, int T, int ld, void* out
                  : launch_slab_columns((const uint16_t*)P, S, T, ld, (uint16_t*)out0, n0, (uint16_t*)out1, n1, s);
 }
 
-template <typename PT, typename OT>
-static int launch_squared_relu(const PT* P, int S, size_t n, OT* out, hipStream_t s) {
+template <int ACT, typename PT, typename OT>
+static int launch_activation(const PT* P, int S, size_t n, OT* out, hipStream_t s) {
   if (n % 8 == 0) {
     const size_t g = (n / 8 + 255) / 256;
-    squared_relu_kernel<8, PT, OT><<<(int)(g < 4096 ? g : 4096), 256, 0, s>>>(P, S, n, out);
+    slab_activation_kernel<ACT, 8, PT, OT><<<(int)(g < 4096 ? g : 4096), 256, 0, s>>>(P, S, n, out);
   } else {
     const size_t g = (n + 255) / 256;
-    squared_relu_kernel<1, PT, OT><<<(int)(g < 4096 ? g : 4096), 256, 0, s>>>(P, S, n, out);
+    slab_activation_kernel<ACT, 1, PT, OT><<<(int)(g < 4096 ? g : 4096), 256, 0, s>>>(P, S, n, out);
   }
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
 
-int docqa_squared_relu(const void* P, int p_f32, int S, size_t n, void* out, int out_f32, hipStream_t s) {
+template <int ACT>
+static int activation_types(const void* P, int p_f32, int S, size_t n, void* out, int out_f32, hipStream_t s) {
+  if (p_f32)
+    return out_f32 ? launch_activation<ACT>((const float*)P, S, n, (float*)out, s)
+                   : launch_activation<ACT>((const float*)P, S, n, (uint16_t*)out, s);
+  return out_f32 ? launch_activation<ACT>((const uint16_t*)P, S, n, (float*)out, s)
+                 : launch_activation<ACT>((const uint16_t*)P, S, n, (uint16_t*)out, s);
+}
+
+int docqa_slab_activation(const void* P, int p_f32, int S, size_t n, int act, void* out, int out_f32, hipStream_t s) {
   if (n == 0) return 0;
   if (S < 1) return -1;
-  if (p_f32)
-    return out_f32 ? launch_squared_relu((const float*)P, S, n, (float*)out, s)
-                   : launch_squared_relu((const float*)P, S, n, (uint16_t*)out, s);
-  return out_f32 ? launch_squared_relu((const uint16_t*)P, S, n, (float*)out, s)
-                 : launch_squared_relu((const uint16_t*)P, S, n, (uint16_t*)out, s);
+  if (act == ACT_RELU2) return activation_types<ACT_RELU2>(P, p_f32, S, n, out, out_f32, s);
+  if (act == ACT_GELU_TANH) return activation_types<ACT_GELU_TANH>(P, p_f32, S, n, out, out_f32, s);
+  return -1;
+}
+
+int docqa_soft_cap(const void* x, int f32, float* out, size_t n, float cap, hipStream_t s) {
+  if (n == 0) return 0;
+  const size_t g = (n + 255) / 256;
+  const int grid = (int)(g < 8192 ? g : 8192);
+  if (f32) soft_cap_kernel<<<grid, 256, 0, s>>>((const float*)x, out, n, cap);
+  else soft_cap_kernel<<<grid, 256, 0, s>>>((const uint16_t*)x, out, n, cap);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
 }

@@ -8,7 +8,10 @@
 //   inverse root mean square beside them (k_scale).  With the key norm's weight folded into
 //   w the normalised key is never materialised: one cached row serves as key and as value,
 //   half the bytes of a K / V pair.
-// * window <= 0: no window; sink null: none; k_scale null: 1; V may be the K cache itself.
+// * window <= 0: no window; sink null: none; k_scale null: 1; V may be the K cache itself, or the
+//   first DV elements of its rows (latent attention; its MFMA form is attn_latent.hip).
+// * packed keys (latent attention over prompts): per-head keys and values of the visible rows in
+//   one matrix, a key part all heads share in another, instead of the paged cache.
 // * prefill (several query tokens a sequence) and decode (one) share the kernels: bf16 heads of
 //   up to 256 elements run on MFMA, fp32 and odd head sizes on a wave-per-row kernel.
 #include "docqa_common.h"
@@ -87,6 +90,12 @@ struct WindowArgs {
   int H, G, D, BS, log2BS;
   float scale;
   int window;
+  int DV;                 // value elements of a row (D, or fewer)
+  // packed keys: row j of sequence b at cu_k[b] + j holds [H x kd | H x vd ..] (ld elements), the
+  // other D - kd key elements at kr; the last query token is at the last key
+  const int* cu_k;
+  const uint16_t* kr;
+  int ld, kd, vd;
 };
 
 // LDS written by some lanes of a wave and read by others: in order in hardware, so only the
@@ -107,13 +116,21 @@ __device__ __forceinline__ bool seq_range(const WindowArgs& a, int b, int& q0, i
   return L > 0 && p0 >= 0;
 }
 
+// the same over packed keys: positions count from the sequence's first visible key
+__device__ __forceinline__ bool packed_range(const WindowArgs& a, int b, int& q0, int& L, int& p0) {
+  q0 = a.cu[b];
+  L = a.cu[b + 1] - q0;
+  p0 = a.cu_k[b + 1] - a.cu_k[b] - L;
+  return L > 0 && p0 >= 0;
+}
+
 // Any head size and element type: one wave per (token, head).  64 keys at a time, one per
 // lane for the scores, then the lanes run over the value's elements.
 template <typename T, int NI>
 __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ q, const T* __restrict__ kc,
                                                           const T* __restrict__ vc, T* __restrict__ out,
                                                           WindowArgs a) {
-  __shared__ float sq[4][512];
+  extern __shared__ __attribute__((aligned(16))) float sq_all[];      // [4][D]
   __shared__ float sp[4][64];
   __shared__ int srow[4][64];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -122,15 +139,16 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
   int q0 = 0, L = 0, p0 = 0;
   const bool live = seq_range(a, b, q0, L, p0);
   if (tok >= (a.cu ? L : 1)) return;       // whole waves; no workgroup barrier below
-  const int D = a.D;
-  T* o = out + ((size_t)(q0 + tok) * a.H + h) * D;
+  const int D = a.D, DV = a.DV;
+  T* o = out + ((size_t)(q0 + tok) * a.H + h) * DV;
   if (!live) {                             // a padded decode row
-    for (int c = lane; c < D; c += 64) st1(o + c, 0.f);
+    for (int c = lane; c < DV; c += 64) st1(o + c, 0.f);
     return;
   }
+  float* sq = sq_all + wave * D;
   const int g = h / (a.H / a.G), pos = p0 + tok;
   const T* qp = q + ((size_t)(q0 + tok) * a.H + h) * D;
-  for (int c = lane; c < D; c += 64) sq[wave][c] = ld1(qp + c);
+  for (int c = lane; c < D; c += 64) sq[c] = ld1(qp + c);
   wave_lds_sync();
   const int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
   float m = a.sink ? a.sink[h] * kLog2e : -INFINITY, l = a.sink ? 1.f : 0.f;
@@ -154,12 +172,12 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
           ldv<8>(kp + c, f);
 #pragma unroll
           for (int j = 0; j < 4; ++j) {
-            d0 += f[j] * sq[wave][c + j];
-            d1 += f[4 + j] * sq[wave][c + 4 + j];
+            d0 += f[j] * sq[c + j];
+            d1 += f[4 + j] * sq[c + 4 + j];
           }
         }
       } else {
-        for (; c < D; ++c) d0 += ld1(kp + c) * sq[wave][c];
+        for (; c < D; ++c) d0 += ld1(kp + c) * sq[c];
       }
       s = (d0 + d1) * sl2 * (a.k_scale ? a.k_scale[row] : 1.f);
     }
@@ -175,7 +193,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const int c = lane + 64 * i;
-      if (c < D) {
+      if (c < DV) {
         float v = acc[i] * alpha;
         for (int j = 0; j < n; ++j) v += sp[wave][j] * ld1(vc + (size_t)srow[wave][j] * D + c);
         acc[i] = v;
@@ -187,7 +205,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int c = lane + 64 * i;
-    if (c < D) st1(o + c, acc[i] * inv);
+    if (c < DV) st1(o + c, acc[i] * inv);
   }
 }
 
@@ -204,33 +222,36 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
 //   with a private LDS tile, and merge at the end.
 typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
 
-template <int DP, int QT, int KB, int NW, bool SHARED, bool SPLIT>
+// PACKED: keys and values from packed matrices (WindowArgs::cu_k) instead of the paged cache.
+template <int DP, int DPV, int QT, int KB, int NW, bool SHARED, bool SPLIT, bool PACKED = false>
 __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_kernel(const uint16_t* __restrict__ q,
                                                                    const uint16_t* __restrict__ kc,
                                                                    const uint16_t* __restrict__ vc,
                                                                    uint16_t* __restrict__ out, WindowArgs a) {
-  constexpr int PITCH = DP + 8, NCH = DP / 8, NKT = KB / 16, NKS = DP / 32, NDT = DP / 16;
-  constexpr int TILES = SPLIT ? NW : 2, NT = SHARED ? 1 : 2;
-  constexpr int TILE = KB * PITCH;                                  // elements of one tile
+  static_assert(!SHARED || DP == DPV, "shared rows");
+  constexpr int PITCH = DP + 8, PITCHV = DPV + 8, NCH = DP / 8, NCV = DPV / 8, NKT = KB / 16, NKS = DP / 32,
+                NDT = DPV / 16;
+  constexpr int TILES = SPLIT ? NW : 2;
+  constexpr int KTILE = KB * PITCH, TILE = KTILE + (SHARED ? 0 : KB * PITCHV);    // elements of one buffer
   constexpr int LOADERS = SPLIT ? 64 : 64 * NW;                     // threads staging one tile
-  constexpr int CPT = (KB * NCH + LOADERS - 1) / LOADERS;
+  constexpr int CPT = (KB * NCH + LOADERS - 1) / LOADERS, CPV = (KB * NCV + LOADERS - 1) / LOADERS;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   uint16_t* tiles = reinterpret_cast<uint16_t*>(smem);
-  float* scales = reinterpret_cast<float*>(tiles + TILES * NT * TILE);   // [TILES][KB]
+  float* scales = reinterpret_cast<float*>(tiles + TILES * TILE);   // [TILES][KB]
   __shared__ int s_bt[kMaxBT];              // block ids of the keys the rows see
 
   const int kvh = blockIdx.x, b = blockIdx.y;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int fr = lane & 15, g4 = lane >> 4;
   int q0 = 0, L = 0, p0 = 0;
-  const bool live = seq_range(a, b, q0, L, p0);
-  const int Gs = a.H / a.G, D = a.D;
+  const bool live = PACKED ? packed_range(a, b, q0, L, p0) : seq_range(a, b, q0, L, p0);
+  const int Gs = PACKED ? 1 : a.H / a.G, D = a.D, DV = a.DV;
   constexpr int RW = 16 * QT;
   const int tile_rows = SPLIT ? RW : RW * NW;
   const int row0 = (gridDim.z - 1 - blockIdx.z) * tile_rows;         // longest windows first
   if (!live) {                                                       // a padded decode row
     if (!a.cu)
-      for (int e = tid; e < Gs * D; e += 64 * NW) out[((size_t)b * a.H + kvh * Gs) * D + e] = 0;
+      for (int e = tid; e < Gs * DV; e += 64 * NW) out[((size_t)b * a.H + kvh * Gs) * DV + e] = 0;
     return;
   }
   const int rows = L * Gs;
@@ -245,7 +266,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
 
   const int blk0 = key0 >> a.log2BS, nblk = (pos_hi >> a.log2BS) - blk0 + 1;
   const bool bt_lds = nblk <= kMaxBT;
-  if (bt_lds) {
+  const int kbase = PACKED ? a.cu_k[b] : 0;
+  if (!PACKED && bt_lds) {
     for (int i = tid; i < nblk; i += 64 * NW) s_bt[i] = a.block_tables[(size_t)b * a.maxb + blk0 + i];
     __syncthreads();
   }
@@ -277,7 +299,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
   const float sl2 = a.scale * kLog2e;
 
   const int ltid = SPLIT ? lane : tid;
-  uint4 rk[CPT], rv[SHARED ? 1 : CPT];
+  uint4 rk[CPT], rv[SHARED ? 1 : CPV];
   float rs_ = 1.f;
   auto cache_row = [&](int key) {
     const int kblk = key >> a.log2BS;
@@ -290,11 +312,27 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
     for (int i = 0; i < CPT; ++i) {
       const int e = ltid + LOADERS * i, row = e / NCH, c = (e % NCH) * 8;
       rk[i] = make_uint4(0, 0, 0, 0);
-      if constexpr (!SHARED) rv[i] = make_uint4(0, 0, 0, 0);
       if (e < KB * NCH && kb + row <= pos_hi && c < D) {
-        const size_t off = cache_row(kb + row) * D + c;
-        rk[i] = *reinterpret_cast<const uint4*>(kc + off);
-        if constexpr (!SHARED) rv[i] = *reinterpret_cast<const uint4*>(vc + off);
+        if constexpr (PACKED) {
+          const size_t j = kbase + kb + row;
+          rk[i] = *reinterpret_cast<const uint4*>(c < a.kd ? kc + j * a.ld + kvh * a.kd + c
+                                                           : a.kr + j * (D - a.kd) + (c - a.kd));
+        } else {
+          rk[i] = *reinterpret_cast<const uint4*>(kc + cache_row(kb + row) * D + c);
+        }
+      }
+    }
+    if constexpr (!SHARED) {
+#pragma unroll
+      for (int i = 0; i < CPV; ++i) {
+        const int e = ltid + LOADERS * i, row = e / NCV, c = (e % NCV) * 8;
+        rv[i] = make_uint4(0, 0, 0, 0);
+        if (e < KB * NCV && kb + row <= pos_hi && c < (PACKED ? a.vd : D)) {
+          if constexpr (PACKED)
+            rv[i] = *reinterpret_cast<const uint4*>(vc + (size_t)(kbase + kb + row) * a.ld + kvh * a.vd + c);
+          else
+            rv[i] = *reinterpret_cast<const uint4*>(vc + cache_row(kb + row) * D + c);
+        }
       }
     }
     if (ltid < KB) {
@@ -303,13 +341,19 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
     }
   };
   auto store = [&](int buf) {
-    uint16_t* k = tiles + buf * NT * TILE;
+    uint16_t* k = tiles + buf * TILE;
 #pragma unroll
     for (int i = 0; i < CPT; ++i) {
       const int e = ltid + LOADERS * i, row = e / NCH, c = (e % NCH) * 8;
       if (e < KB * NCH) {
         *reinterpret_cast<uint4*>(k + row * PITCH + c) = rk[i];
-        if constexpr (!SHARED) *reinterpret_cast<uint4*>(k + TILE + row * PITCH + c) = rv[i];
+      }
+    }
+    if constexpr (!SHARED) {
+#pragma unroll
+      for (int i = 0; i < CPV; ++i) {
+        const int e = ltid + LOADERS * i, row = e / NCV, c = (e % NCV) * 8;
+        if (e < KB * NCV) *reinterpret_cast<uint4*>(k + KTILE + row * PITCHV + c) = rv[i];
       }
     }
     if (ltid < KB) scales[buf * KB + ltid] = rs_;
@@ -317,8 +361,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
   // one key tile against this wave's rows; `part`: some of its keys are hidden from some rows
   auto compute_tile = [&](int kb, int buf, auto part) {
     constexpr bool PART = decltype(part)::value;
-    const uint16_t* sk = tiles + buf * NT * TILE;
-    const uint16_t* sv = SHARED ? sk : sk + TILE;
+    const uint16_t* sk = tiles + buf * TILE;
+    const uint16_t* sv = SHARED ? sk : sk + KTILE;
     const float* sc = scales + buf * KB;
     f32x4 x[QT][NKT];
 #pragma unroll
@@ -384,11 +428,11 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
           pb[t2][j] = (__bf16)x[t2][2 * s][j];
           pb[t2][4 + j] = (__bf16)x[t2][2 * s + 1][j];
         }
-      const uint16_t* vr = sv + (s * 32 + g4 * 4 + tq) * PITCH + 4 * tp;
+      const uint16_t* vr = sv + (s * 32 + g4 * 4 + tq) * PITCHV + 4 * tp;
 #pragma unroll
       for (int i = 0; i < NDT; ++i) {
         const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + i * 16));
-        const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 16 * PITCH + i * 16));
+        const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 16 * PITCHV + i * 16));
         bf16x8 vf;
         const __bf16* lp = reinterpret_cast<const __bf16*>(&lo);
         const __bf16* hp = reinterpret_cast<const __bf16*>(&hi);
@@ -424,12 +468,12 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
     for (int t = 0; t < QT; ++t) {
       const int r = wrow + t * 16 + fr;
       if (r >= rows) continue;
-      uint16_t* op = out + ((size_t)(q0 + r / Gs) * a.H + kvh * Gs + r % Gs) * D;
+      uint16_t* op = out + ((size_t)(q0 + r / Gs) * a.H + kvh * Gs + r % Gs) * DV;
       const float inv = 1.f / l[t];
 #pragma unroll
       for (int i = 0; i < NDT; ++i) {
         const int c = i * 16 + g4 * 4;
-        if (c < D) {
+        if (c < DV) {
           uint2 v;
           v.x = pack2(o[t][i][0] * inv, o[t][i][1] * inv);
           v.y = pack2(o[t][i][2] * inv, o[t][i][3] * inv);
@@ -484,24 +528,24 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
   }
 }
 
-template <int DP, int QT, int KB, int NW, bool SHARED, bool SPLIT>
+template <int DP, int DPV, int QT, int KB, int NW, bool SHARED, bool SPLIT, bool PACKED = false>
 int launch_mfma(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
                 hipStream_t s) {
-  constexpr int TILES = SPLIT ? NW : 2, NT = SHARED ? 1 : 2;
-  constexpr size_t tile_b = (size_t)TILES * NT * KB * (DP + 8) * 2 + (size_t)TILES * KB * 4;
+  constexpr int TILES = SPLIT ? NW : 2;
+  constexpr size_t tile_b = (size_t)TILES * KB * (DP + 8 + (SHARED ? 0 : DPV + 8)) * 2 + (size_t)TILES * KB * 4;
   constexpr size_t merge_b = SPLIT ? (size_t)NW * 16 * (DP + 4) * 4 + (size_t)NW * 16 * 8 : 0;
   constexpr size_t lds = tile_b > merge_b ? tile_b : merge_b;
   static_assert(lds <= 160 * 1024, "LDS");
-  const int tile_rows = 16 * QT * (SPLIT ? 1 : NW), Gs = a.H / a.G;
+  const int tile_rows = 16 * QT * (SPLIT ? 1 : NW), Gs = PACKED ? 1 : a.H / a.G;
   const long long nz = ((long long)max_q * Gs + tile_rows - 1) / tile_rows;
   if (nz > 65535) return -1;
-  auto kern = window_attn_mfma_kernel<DP, QT, KB, NW, SHARED, SPLIT>;
+  auto kern = window_attn_mfma_kernel<DP, DPV, QT, KB, NW, SHARED, SPLIT, PACKED>;
   if constexpr (lds > 64 * 1024) {
     static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
                                                     hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return (int)e;
   }
-  kern<<<dim3(a.G, B, (int)nz), 64 * NW, lds, s>>>((const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc,
+  kern<<<dim3(PACKED ? a.H : a.G, B, (int)nz), 64 * NW, lds, s>>>((const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc,
                                                    (uint16_t*)out, a);
   DOCQA_CHECK_LAUNCH();
   return 0;
@@ -517,13 +561,13 @@ int dispatch_mfma(const void* q, const void* kc, const void* vc, void* out, cons
     if constexpr (DP <= 128) {
       const long long wgs = (long long)B * a.G;
       if constexpr (SHARED) {
-        if (wgs <= 256) return launch_mfma<DP, 1, 32, 16, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+        if (wgs <= 256) return launch_mfma<DP, DP, 1, 32, 16, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
       }
-      if (wgs <= 512) return launch_mfma<DP, 1, 32, 8, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+      if (wgs <= 512) return launch_mfma<DP, DP, 1, 32, 8, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
     }
-    return launch_mfma<DP, 1, 32, 4, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+    return launch_mfma<DP, DP, 1, 32, 4, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
   }
-  return launch_mfma<DP, QT, 64, 4, SHARED, false>(q, kc, vc, out, a, B, max_q, s);
+  return launch_mfma<DP, DP, QT, 64, 4, SHARED, false>(q, kc, vc, out, a, B, max_q, s);
 }
 
 template <bool SHARED>
@@ -578,29 +622,52 @@ int docqa_qk_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, co
 
 int docqa_window_attn(const void* q, const void* kc, const void* vc, const float* k_scale, const int* block_tables,
                       int maxb, const int* cu, const int* ctx, const float* sink, void* out, int f32, int B,
-                      int max_q, int H, int G, int D, int BS, float scale, int window, hipStream_t s) {
+                      int max_q, int H, int G, int D, int DV, int BS, float scale, int window, hipStream_t s) {
   if (B == 0 || max_q == 0) return 0;
-  if (H % G != 0 || D < 1 || D > 512 || (BS & (BS - 1)) != 0) return -1;
+  if (H % G != 0 || D < 1 || D > 2560 || DV < 1 || DV > D || DV > 2048 || (BS & (BS - 1)) != 0) return -1;
   int log2BS = 0;
   while ((1 << log2BS) < BS) ++log2BS;
-  const WindowArgs a{block_tables, maxb, cu, ctx, k_scale, sink, H, G, D, BS, log2BS, scale, window};
-  if (!f32 && D % 8 == 0 && D <= 256 && docqa_aligned16(q) && docqa_aligned16(out))
+  const WindowArgs a{block_tables, maxb, cu, ctx, k_scale, sink, H, G, D, BS, log2BS, scale, window, DV,
+                     nullptr, nullptr, 0, 0, 0};
+  if (!f32 && D % 8 == 0 && D <= 256 && DV == D && docqa_aligned16(q) && docqa_aligned16(out))
     return kc == vc ? dispatch_dim<true>(q, kc, vc, out, a, B, max_q, s)
                     : dispatch_dim<false>(q, kc, vc, out, a, B, max_q, s);
   dim3 grid((max_q * H + 3) / 4, B);
-#define GO(T, N) window_attn_kernel<T, N><<<grid, 256, 0, s>>>((const T*)q, (const T*)kc, (const T*)vc, (T*)out, a)
+#define GO(T, N) window_attn_kernel<T, N><<<grid, 256, (size_t)D * 16, s>>>((const T*)q, (const T*)kc, (const T*)vc, (T*)out, a)
   if (f32) {
-    if (D <= 64) GO(float, 1);
-    else if (D <= 128) GO(float, 2);
-    else if (D <= 256) GO(float, 4);
-    else GO(float, 8);
+    if (DV <= 64) GO(float, 1);
+    else if (DV <= 128) GO(float, 2);
+    else if (DV <= 256) GO(float, 4);
+    else if (DV <= 512) GO(float, 8);
+    else GO(float, 32);
   } else {
-    if (D <= 64) GO(uint16_t, 1);
-    else if (D <= 128) GO(uint16_t, 2);
-    else if (D <= 256) GO(uint16_t, 4);
-    else GO(uint16_t, 8);
+    if (DV <= 64) GO(uint16_t, 1);
+    else if (DV <= 128) GO(uint16_t, 2);
+    else if (DV <= 256) GO(uint16_t, 4);
+    else if (DV <= 512) GO(uint16_t, 8);
+    else GO(uint16_t, 32);
   }
 #undef GO
   DOCQA_CHECK_LAUNCH();
   return 0;
+}
+
+int docqa_packed_window_attn(const void* q, const void* kv, const void* kr, const int* cu, const int* cu_k,
+                             const float* sink, void* out, int B, int max_q, int H, int d8, int r8, int vdim, int ld,
+                             float scale, int window, hipStream_t s) {
+  if (B == 0 || max_q == 0) return 0;
+  const int D = d8 + r8, v8 = (vdim + 7) / 8 * 8;
+  if (H < 1 || d8 < 8 || d8 % 8 || r8 < 0 || r8 % 8 || D > 256 || vdim < 4 || vdim % 4 || vdim > 256) return -1;
+  if (ld % 8 || ld < H * (d8 + v8) || B > 65535) return -1;
+  if (!docqa_aligned16(q) || !docqa_aligned16(kv) || !docqa_aligned16(kr) || !docqa_aligned16(out)) return -1;
+  const WindowArgs a{nullptr, 0, cu, nullptr, nullptr, sink, H, H, D, 64, 6, scale, window, vdim,
+                     cu_k, (const uint16_t*)kr, ld, d8, v8};
+  const uint16_t* v = (const uint16_t*)kv + (size_t)H * d8;
+#define GO(DP, DPV, QT, KB) return launch_mfma<DP, DPV, QT, KB, 4, false, false, true>(q, kv, v, out, a, B, max_q, s)
+  if (D <= 64 && vdim <= 64) GO(64, 64, 2, 64);
+  if (D <= 96 && vdim <= 64) GO(96, 64, 2, 64);
+  if (D <= 128 && vdim <= 128) GO(128, 128, 2, 64);
+  if (D <= 192 && vdim <= 128) GO(192, 128, 2, 32);
+  GO(256, 256, 1, 32);
+#undef GO
 }

@@ -40,7 +40,7 @@ using namespace docqa;
 namespace {
 constexpr int BN = 64, BKD = 128, NS = 4, MR = 192;   // NS: default ring slots, K granule 4 stages
 constexpr int KSTEPS = BKD / 32;               // 16x16x32 k-steps per stage
-enum { EPI_BF16 = 0, EPI_PARTIAL = 1, EPI_GLU = 2, EPI_ARGMAX = 3, EPI_RELU2 = 4 };
+enum { EPI_BF16 = 0, EPI_PARTIAL = 1, EPI_GLU = 2, EPI_ARGMAX = 3, EPI_RELU2 = 4, EPI_GELU = 5 };
 typedef __attribute__((address_space(3))) void lds_void;
 
 // The ring's DMA / X loads are inline asm (docqa_asm.h): the counted waits below are the
@@ -373,7 +373,7 @@ __global__ __launch_bounds__(256) void dgemm_kernel(const uint16_t* __restrict__
     if constexpr (NORM)
       __hip_atomic_store(P + ((size_t)slice * M + row) * N + col, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     else if constexpr (EPI == EPI_PARTIAL) P[((size_t)slice * M + row) * N + col] = v;
-    else Y[(size_t)row * N + col] = f2bf(EPI == EPI_RELU2 ? relu2(v) : v);
+    else Y[(size_t)row * N + col] = f2bf(EPI == EPI_RELU2 ? relu2(v) : EPI == EPI_GELU ? gelu_tanh(v) : v);
   };
   // SwiGLU pair: gate value at an 8-block's low half, up value 8 columns later
   auto store_glu = [&](int row, int col, float g, float u) {
@@ -587,12 +587,18 @@ int docqa_dgemm(const void* X, const void* W, void* Y, float* partial, int M, in
   return 0;
 }
 
-// Y [M, N] = squared ReLU of X . W^T (S = 1)
-int docqa_dgemm_relu2(const void* X, const void* W, void* Y, int M, int N, int K, hipStream_t s) {
+// Y [M, N] = act(X . W^T) (S = 1)
+int docqa_dgemm_act(const void* X, const void* W, void* Y, int act, int M, int N, int K, hipStream_t s) {
   if (M == 0) return 0;
   if (!shape_ok(M, N, K, 1, BN)) return -1;
-  launch_mt<EPI_RELU2, 4>((M + 15) / 16, dim3(N / BN, 1), s, (const uint16_t*)X, (const uint16_t*)W, (uint16_t*)Y,
-                          nullptr, M, N, K, K);
+  if (act == ACT_RELU2)
+    launch_mt<EPI_RELU2, 4>((M + 15) / 16, dim3(N / BN, 1), s, (const uint16_t*)X, (const uint16_t*)W, (uint16_t*)Y,
+                            nullptr, M, N, K, K);
+  else if (act == ACT_GELU_TANH)
+    launch_mt<EPI_GELU, 4>((M + 15) / 16, dim3(N / BN, 1), s, (const uint16_t*)X, (const uint16_t*)W, (uint16_t*)Y,
+                           nullptr, M, N, K, K);
+  else
+    return -1;
   DOCQA_CHECK_LAUNCH();
   return 0;
 }

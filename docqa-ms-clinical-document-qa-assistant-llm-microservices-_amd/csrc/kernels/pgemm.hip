@@ -1,7 +1,7 @@
 // pgemm.hip -- prefill GEMM for the Llama generator (large M: packed prompt tokens)
 //   C[M, N] = A[M, K] . W[N, K]^T           (bf16 in, fp32 accumulate, bf16 out)
 //   C[M, N/2] = silu(gate) * up             (EPI_GLU: W = the 8-interleaved gate|up rows)
-//   C[M, N] = max(A . W^T, 0)^2             (EPI_RELU2)
+//   C[M, N] = act(A . W^T)                  (EPI_RELU2, EPI_GELU)
 // Replaces hipBLASLt for the prefill QKV / O / gate|up (+ fused SwiGLU) / down projections
 // (llm-qa/main.py:117 -> prefill inside Ollama in the reference).
 //
@@ -48,7 +48,7 @@ constexpr int BUF_B = 4 * HALF_B;        // bytes of one K-tile buffer (64 KiB)
 constexpr int SCR_PITCH = 72;            // epilogue scratch row pitch (bf16), 144 B
 constexpr int LDS_B = (2 * BUF_B > 8 * 128 * SCR_PITCH * 2) ? 2 * BUF_B : 8 * 128 * SCR_PITCH * 2;
 enum { HA0 = 0, HA1 = 1, HB0 = 2, HB1 = 3 };
-enum { EPI_BF16 = 0, EPI_GLU = 1, EPI_PARTIAL = 2, EPI_RELU2 = 3 };
+enum { EPI_BF16 = 0, EPI_GLU = 1, EPI_PARTIAL = 2, EPI_RELU2 = 3, EPI_GELU = 4 };
 
 // byte offset of logical 16-B chunk `ch` of `row` inside a [128][64] bf16 half-tile
 __device__ __forceinline__ uint32_t swz(int row, int ch) {
@@ -242,7 +242,7 @@ __device__ __forceinline__ void pgemm_store(char* smem, f32x4 (&acc)[2][4][2][2]
 
   // ---- epilogue: the wave's 128 x 64 tile -> bf16 scratch [128][SCR_PITCH] -> row stores
   uint16_t* scr = reinterpret_cast<uint16_t*>(smem) + wave * 128 * SCR_PITCH;
-  if constexpr (EPI == EPI_BF16 || EPI == EPI_RELU2) {
+  if constexpr (EPI == EPI_BF16 || EPI == EPI_RELU2 || EPI == EPI_GELU) {
 #pragma unroll
     for (int mh = 0; mh < 2; ++mh)
 #pragma unroll
@@ -254,7 +254,9 @@ __device__ __forceinline__ void pgemm_store(char* smem, f32x4 (&acc)[2][4][2][2]
 #pragma unroll
             for (int r = 0; r < 4; ++r)
               scr[(mh * 64 + i * 16 + fk * 4 + r) * SCR_PITCH + nh * 32 + j * 16 + fr] =
-                  f2bf(EPI == EPI_RELU2 ? relu2(acc[mh][i][nh][j][r]) : acc[mh][i][nh][j][r]);
+                  f2bf(EPI == EPI_RELU2   ? relu2(acc[mh][i][nh][j][r])
+                       : EPI == EPI_GELU ? gelu_tanh(acc[mh][i][nh][j][r])
+                                         : acc[mh][i][nh][j][r]);
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     // 8 lanes per 128-B row segment, 8 rows per sweep
 #pragma unroll 4
@@ -369,13 +371,13 @@ bool docqa_pgemm_ok(int M, int N, int K) {
 }
 
 // epi 0: C [M, N] bf16; epi 1: C [M, N / 2] = silu(gate) * up (8-interleaved gate|up W);
-// epi 3: C [M, N] = squared ReLU; epi 2: P [S, M, N] fp32 split-K slabs (S >= 1 slices of K / S)
+// epi 3 / 4: C [M, N] = squared ReLU / tanh GELU; epi 2: P [S, M, N] fp32 split-K slabs (S >= 1 slices of K / S)
 int docqa_pgemm(const void* A, const void* W, void* C, float* P, int M, int N, int K, int S, int epi,
                 hipStream_t s) {
   if (M == 0) return 0;
   if (!docqa_pgemm_ok(M, N, K) || S < 1 || K % (S * 2 * BK) != 0) return -1;
   if (epi == EPI_PARTIAL ? P == nullptr : (C == nullptr || S != 1)) return -1;
-  if (epi != EPI_BF16 && epi != EPI_GLU && epi != EPI_PARTIAL && epi != EPI_RELU2) return -1;
+  if (epi != EPI_BF16 && epi != EPI_GLU && epi != EPI_PARTIAL && epi != EPI_RELU2 && epi != EPI_GELU) return -1;
   if (!docqa_aligned16(A) || !docqa_aligned16(W) || !docqa_aligned16(epi == EPI_PARTIAL ? (void*)P : C)) return -1;
   const int ntm = (M + BM - 1) / BM, ntn = N / BN;
   const uint16_t *a = (const uint16_t*)A, *w = (const uint16_t*)W;
@@ -385,6 +387,8 @@ int docqa_pgemm(const void* A, const void* W, void* C, float* P, int M, int N, i
     pgemm_kernel<EPI_BF16><<<grid, 512, 0, s>>>(a, w, c, P, M, N, K, ntm, ntn, S, Ks);
   else if (epi == EPI_RELU2)
     pgemm_kernel<EPI_RELU2><<<grid, 512, 0, s>>>(a, w, c, P, M, N, K, ntm, ntn, S, Ks);
+  else if (epi == EPI_GELU)
+    pgemm_kernel<EPI_GELU><<<grid, 512, 0, s>>>(a, w, c, P, M, N, K, ntm, ntn, S, Ks);
   else if (epi == EPI_GLU)
     pgemm_kernel<EPI_GLU><<<grid, 512, 0, s>>>(a, w, c, P, M, N, K, ntm, ntn, S, Ks);
   else

@@ -114,6 +114,42 @@ __global__ __launch_bounds__(256) void embed_scale_rmsnorm_kernel(const int* __r
   }
 }
 
+// res += m (P + Q) of two projections (Q null: one), each a product or split-K slabs, and a copy
+// in the compute dtype: the stream update between sublayers without a norm of their own
+template <int V, typename PT, typename QT>
+__global__ __launch_bounds__(256) void add_scaled_kernel(const PT* __restrict__ P, int SP, const QT* __restrict__ Q,
+                                                         int SQ, float* __restrict__ res, float m,
+                                                         uint16_t* __restrict__ out, size_t n) {
+  const size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * V;
+  if (i >= n) return;
+  float x[V], y[V];
+  ldv<V>(res + i, x);
+  ld_slabs<V>(P + i, SP, n, y);
+  if (Q) {
+    float z[V];
+    ld_slabs<V>(Q + i, SQ, n, z);
+#pragma unroll
+    for (int j = 0; j < V; ++j) y[j] += z[j];
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j) x[j] += m * y[j];
+  stv<V>(res + i, x);
+  if (out) stv<V>(out + i, x);
+}
+
+template <typename PT, typename QT>
+int launch_add_scaled(const void* P, int SP, const void* Q, int SQ, float* res, float m, void* out, size_t n,
+                      hipStream_t s) {
+  if (n % 4 == 0)
+    add_scaled_kernel<4, PT, QT><<<(unsigned)((n / 4 + 255) / 256), 256, 0, s>>>((const PT*)P, SP, (const QT*)Q, SQ, res,
+                                                                                 m, (uint16_t*)out, n);
+  else
+    add_scaled_kernel<1, PT, QT><<<(unsigned)((n + 255) / 256), 256, 0, s>>>((const PT*)P, SP, (const QT*)Q, SQ, res, m,
+                                                                             (uint16_t*)out, n);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
 template <int V, typename PT, typename OT>
 int launch_sandwich(const PT* P, int S, float* res, const float* w_post, const float* add, const float* w_next,
                     OT* out, int rows, int H, float eps, hipStream_t s) {
@@ -175,4 +211,15 @@ int docqa_embed_scale_rmsnorm(const int* ids, const void* table, int f32, float 
   return H % 4 == 0
              ? launch_embed<4>(ids, (const uint16_t*)table, scale, w, res, emb, (uint16_t*)out, rows, H, vocab, eps, s)
              : launch_embed<1>(ids, (const uint16_t*)table, scale, w, res, emb, (uint16_t*)out, rows, H, vocab, eps, s);
+}
+
+int docqa_add_scaled(const void* P, int p_f32, int SP, const void* Q, int q_f32, int SQ, float* res, float m, void* out,
+                     size_t n, hipStream_t s) {
+  if (n == 0) return 0;
+  if (SP < 1 || (Q && SQ < 1) || n >= ((size_t)1 << 38)) return -1;
+  if (p_f32)
+    return q_f32 ? launch_add_scaled<float, float>(P, SP, Q, SQ, res, m, out, n, s)
+                 : launch_add_scaled<float, uint16_t>(P, SP, Q, SQ, res, m, out, n, s);
+  return q_f32 ? launch_add_scaled<uint16_t, float>(P, SP, Q, SQ, res, m, out, n, s)
+               : launch_add_scaled<uint16_t, uint16_t>(P, SP, Q, SQ, res, m, out, n, s);
 }

@@ -1,7 +1,7 @@
 // ssm.hip -- recurrent mixers: a short causal convolution per channel and the selective scan
 // (Mamba, Gu & Dao 2023), each as a prefill kernel over packed sequences and a decode step.
 //
-//   conv:  y[t, c] = silu(b[c] + sum_k w[k, c] x[t - (taps - 1) + k, c])
+//   conv:  y[t, c] = act(b[c] + sum_k w[k, c] x[t - (taps - 1) + k, c]), act silu or none
 //   scan:  dt = softplus(dt_pre + dt_b);  S[c, n] <- 2^(dt A2[c, n]) S[c, n] + dt x B[n]
 //          y = (sum_n S[c, n] C[n] + D x) silu(z)           A2 = -exp(A_log) log2(e)
 //
@@ -34,16 +34,22 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
                                                           const float* __restrict__ w, const float* __restrict__ bias,
                                                           T* __restrict__ state, const int* __restrict__ slots,
                                                           const int* __restrict__ cu, const int* __restrict__ ctx,
-                                                          T* __restrict__ y, int C, int taps) {
+                                                          T* __restrict__ y, int C, int taps, int silu) {
   const int b = blockIdx.z, q0 = cu[b], L = cu[b + 1] - q0;
-  const int t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * TT;
+  const int nt = K > 0 ? K : taps;
+  // a thread's tokens: at least the carried inputs, so the thread of token 0 alone reads (and
+  // then replaces) a sequence's state
+  static_assert(K <= 0 || TT >= K - 1, "tokens per thread");
+  const int tt = K > 0 ? TT : max(TT, nt - 1);
+  const int t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * tt;
   const int c0 = (blockIdx.x * 64 + (threadIdx.x & 63)) * V;
   if (t0 >= L || c0 >= C) return;
-  const int nt = K > 0 ? K : taps;
   const bool carry = ctx[b] > 0 && slots[b] >= 0;
   const T* st = carry ? state + (size_t)slots[b] * (nt - 1) * C + c0 : nullptr;
   float bv[V];
-  ldv<V>(bias + c0, bv);
+#pragma unroll
+  for (int j = 0; j < V; ++j) bv[j] = 0.f;
+  if (bias) ldv<V>(bias + c0, bv);
   auto input = [&](int t, float* f) {       // input at token t of this portion (t < 0: carried)
     if (t >= 0) {
       ldv<V>(x + (size_t)(q0 + t) * ldx + c0, f);
@@ -68,12 +74,12 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
         float s = bv[j];
 #pragma unroll
         for (int k = 0; k < K; ++k) s += wv[k][j] * in[i + k][j];
-        o[j] = silu_fast(s);
+        o[j] = silu ? silu_fast(s) : s;
       }
       if (t0 + i < L) stv<V>(y + (size_t)(q0 + t0 + i) * C + c0, o);
     }
   } else {
-    for (int i = 0; i < TT && t0 + i < L; ++i) {
+    for (int i = 0; i < tt && t0 + i < L; ++i) {
       float s[V], f[V], wk[V];
 #pragma unroll
       for (int j = 0; j < V; ++j) s[j] = bv[j];
@@ -84,7 +90,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
         for (int j = 0; j < V; ++j) s[j] += wk[j] * f[j];
       }
 #pragma unroll
-      for (int j = 0; j < V; ++j) s[j] = silu_fast(s[j]);
+      for (int j = 0; j < V; ++j) s[j] = silu ? silu_fast(s[j]) : s[j];
       stv<V>(y + (size_t)(q0 + t0 + i) * C + c0, s);
     }
   }
@@ -109,7 +115,7 @@ __global__ __launch_bounds__(256) void conv_step_kernel(const PT* __restrict__ P
                                                         const float* __restrict__ w, const float* __restrict__ bias,
                                                         T* __restrict__ state, const int* __restrict__ slots,
                                                         const int* __restrict__ positions, T* __restrict__ y,
-                                                        T* __restrict__ z_out, int C, int taps) {
+                                                        T* __restrict__ z_out, int C, int taps, int silu) {
   const int b = blockIdx.y, c0 = (blockIdx.x * 256 + threadIdx.x) * V;
   const int nt = K > 0 ? K : taps;
   if (c0 >= (z_out ? 2 * C : C)) return;
@@ -124,7 +130,9 @@ __global__ __launch_bounds__(256) void conv_step_kernel(const PT* __restrict__ P
   const bool carry = slot >= 0 && positions[b] > 0;
   T* st = state + (size_t)max(slot, 0) * (nt - 1) * C + c0;
   float s[V], wk[V];
-  ldv<V>(bias + c0, s);
+#pragma unroll
+  for (int j = 0; j < V; ++j) s[j] = 0.f;
+  if (bias) ldv<V>(bias + c0, s);
 #pragma unroll
   for (int j = 0; j < V; ++j) xn[j] = rnd((const T*)nullptr, xn[j]);
   ldv<V>(w + (size_t)(nt - 1) * C + c0, wk);
@@ -166,7 +174,7 @@ __global__ __launch_bounds__(256) void conv_step_kernel(const PT* __restrict__ P
     }
   }
 #pragma unroll
-  for (int j = 0; j < V; ++j) s[j] = silu_fast(s[j]);
+  for (int j = 0; j < V; ++j) s[j] = silu ? silu_fast(s[j]) : s[j];
   stv<V>(y + (size_t)b * C + c0, s);
 }
 
@@ -426,15 +434,18 @@ __global__ __launch_bounds__(256) void selective_step_kernel(ScanArgs a, StepDt 
 
 template <typename T, int V>
 int launch_conv(const void* x, int ldx, const float* w, const float* b, void* state, const int* slots, const int* cu,
-                const int* ctx, void* y, int B, int max_len, int C, int taps, hipStream_t s) {
+                const int* ctx, void* y, int B, int max_len, int C, int taps, int silu, hipStream_t s) {
   const int gx = (C + 64 * V - 1) / (64 * V);
-  // 8 tokens a thread; 2 where that leaves most of the chip without a workgroup
+  // 8 tokens a thread; fewer where that leaves most of the chip without a workgroup
   const bool few = (long long)gx * ((max_len + 31) / 32) * B < 1024;
-  dim3 grid(gx, few ? (max_len + 7) / 8 : (max_len + 31) / 32, B);
-#define GO(K)                                                                                              \
-  do {                                                                                                     \
-    if (few) causal_conv_kernel<T, V, K, 2><<<grid, 256, 0, s>>>((const T*)x, ldx, w, b, (T*)state, slots, cu, ctx, (T*)y, C, taps); \
-    else causal_conv_kernel<T, V, K, 8><<<grid, 256, 0, s>>>((const T*)x, ldx, w, b, (T*)state, slots, cu, ctx, (T*)y, C, taps);     \
+#define LAUNCH(K, TT, tt)                                                                                   \
+  causal_conv_kernel<T, V, K, TT><<<dim3(gx, (max_len + 4 * (tt)-1) / (4 * (tt)), B), 256, 0, s>>>(         \
+      (const T*)x, ldx, w, b, (T*)state, slots, cu, ctx, (T*)y, C, taps, silu)
+#define GO(K)                                        \
+  do {                                               \
+    constexpr int TF = K == 4 ? 3 : 2;               \
+    if (few) LAUNCH(K, TF, K > 0 ? TF : (TF > taps - 1 ? TF : taps - 1)); \
+    else LAUNCH(K, 8, K > 0 ? 8 : (8 > taps - 1 ? 8 : taps - 1));        \
   } while (0)
   switch (taps) {
     case 2: GO(2); break;
@@ -443,16 +454,17 @@ int launch_conv(const void* x, int ldx, const float* w, const float* b, void* st
     default: GO(0); break;
   }
 #undef GO
+#undef LAUNCH
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
 
 template <typename PT, typename T, int V>
 int launch_conv_step(const void* P, int S, size_t slab, int ld, const float* w, const float* b, void* state,
-                     const int* slots, const int* pos, void* y, void* z, int B, int C, int taps, hipStream_t s) {
+                     const int* slots, const int* pos, void* y, void* z, int B, int C, int taps, int silu, hipStream_t s) {
   const int n = (z ? 2 * C : C) / V;
   dim3 grid((n + 255) / 256, B);
-#define GO(K) conv_step_kernel<PT, T, V, K><<<grid, 256, 0, s>>>((const PT*)P, S, slab, ld, w, b, (T*)state, slots, pos, (T*)y, (T*)z, C, taps)
+#define GO(K) conv_step_kernel<PT, T, V, K><<<grid, 256, 0, s>>>((const PT*)P, S, slab, ld, w, b, (T*)state, slots, pos, (T*)y, (T*)z, C, taps, silu)
   switch (taps) {
     case 2: GO(2); break;
     case 3: GO(3); break;
@@ -496,24 +508,24 @@ int dispatch_scan(const ScanArgs& a, int B, hipStream_t s) {
 
 int docqa_causal_conv(const void* x, int ldx, const float* w, const float* b, void* state, const int* slots,
                       const int* cu, const int* ctx, void* y, int f32, int B, int max_len, int C, int taps,
-                      hipStream_t s) {
+                      int silu, hipStream_t s) {
   if (B == 0 || max_len == 0) return 0;
   if (taps < 1 || C < 1 || ldx < C) return -1;
   const bool vec = C % 8 == 0 && ldx % 8 == 0 && docqa_aligned16(x) && docqa_aligned16(state) && docqa_aligned16(y);
   if (f32)
-    return vec ? launch_conv<float, 4>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, s)
-               : launch_conv<float, 1>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, s);
-  return vec ? launch_conv<uint16_t, 8>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, s)
-             : launch_conv<uint16_t, 1>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, s);
+    return vec ? launch_conv<float, 4>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, silu, s)
+               : launch_conv<float, 1>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, silu, s);
+  return vec ? launch_conv<uint16_t, 8>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, silu, s)
+             : launch_conv<uint16_t, 1>(x, ldx, w, b, state, slots, cu, ctx, y, B, max_len, C, taps, silu, s);
 }
 
 int docqa_conv_step(const void* P, int p_f32, int S, size_t slab, int ld, const float* w, const float* b, void* state,
                     const int* slots, const int* positions, void* y, void* z, int f32, int B, int C, int taps,
-                    hipStream_t s) {
+                    int silu, hipStream_t s) {
   if (B == 0) return 0;
   if (taps < 1 || C < 1 || S < 1 || ld < (z ? 2 * C : C) || (f32 && !p_f32)) return -1;
   const bool vec = C % 4 == 0 && ld % 4 == 0 && docqa_aligned16(P) && docqa_aligned16(state) && docqa_aligned16(y);
-#define ARGS P, S, slab, ld, w, b, state, slots, positions, y, z, B, C, taps, s
+#define ARGS P, S, slab, ld, w, b, state, slots, positions, y, z, B, C, taps, silu, s
   if (f32) return vec ? launch_conv_step<float, float, 4>(ARGS) : launch_conv_step<float, float, 1>(ARGS);
   if (p_f32) return vec ? launch_conv_step<float, uint16_t, 4>(ARGS) : launch_conv_step<float, uint16_t, 1>(ARGS);
   return vec ? launch_conv_step<uint16_t, uint16_t, 4>(ARGS) : launch_conv_step<uint16_t, uint16_t, 1>(ARGS);

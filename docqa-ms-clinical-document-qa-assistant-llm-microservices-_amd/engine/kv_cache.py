@@ -9,8 +9,8 @@ Block bookkeeping is done by the native allocator in ``csrc/runtime/block_manage
 when the extension is loaded (O(1) alloc/free, refcounts for shared prompt prefixes)
 and by the pure-Python :class:`PyBlockAllocator` otherwise.
 
-A layer may instead keep one tensor that serves as K and V (:class:`KVSpec` ``shared``), and
-recurrent layers keep per-request state in slots (:class:`StatePool`).
+A layer may instead keep one tensor that serves as K and V (:class:`KVSpec` ``shared``,
+``latent``), also for later layers that read it, and recurrent layers keep per-request state in slots (:class:`StatePool`).
 """
 from __future__ import annotations
 
@@ -23,14 +23,16 @@ import torch
 @dataclass(frozen=True)
 class KVSpec:
     """One layer's paged cache.  ``shared``: the key rows are the values too -- one tensor,
-    with an fp32 scale per row in place of V (ops.qk_norm_store)."""
+    with an fp32 scale per row in place of V (ops.qk_norm_store); ``latent``: one tensor of
+    rows that keys and values are made from (ops.latent_store), no V."""
     kv_heads: int
     head_dim: int
     shared: bool = False
+    latent: bool = False
 
     def bytes_per_token(self, dtype_bytes: int) -> int:
         row = self.head_dim * dtype_bytes
-        return self.kv_heads * (row + 4 if self.shared else 2 * row)
+        return self.kv_heads * (row if self.latent else row + 4 if self.shared else 2 * row)
 
 
 @dataclass(frozen=True)
@@ -102,7 +104,8 @@ class KVCache:
         for sp in specs:
             shape = (num_blocks, sp.kv_heads, block_size, sp.head_dim)
             k = torch.zeros(shape, device=device, dtype=dtype)
-            self.caches.append((k, torch.zeros(shape[:3], device=device, dtype=torch.float32) if sp.shared
+            self.caches.append((k, None if sp.latent
+                                else torch.zeros(shape[:3], device=device, dtype=torch.float32) if sp.shared
                                 else torch.zeros_like(k)))
         self.allocator = make_allocator(num_blocks, block_size)
 

@@ -395,7 +395,8 @@ class LLMEngine:
             return torch.as_tensor(a, dtype=torch.int32).to(dev, non_blocking=True)
 
         meta = AttnMeta(prefill=True, positions=up(pos), slot_mapping=up(sm), cu_seqlens=up(cu),
-                        max_len=max(len(p) - c for p, c in zip(prompts, start)))
+                        max_len=max(len(p) - c for p, c in zip(prompts, start)),
+                        spans=[(c, len(p)) for p, c in zip(prompts, start)])
         if any(start) or self.model.paged_prefill:
             self.page_prefill(meta, tables, start)
         if self.state is not None:

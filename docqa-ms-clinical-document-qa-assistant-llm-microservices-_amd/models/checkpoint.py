@@ -23,7 +23,7 @@ import torch
 
 from ..ops import reference as ref
 from .bert import BertConfig, BertEncoder, BertTokenClassifier
-from . import saritar
+from . import dolodra, saritar
 from .hybrid import HybridModel
 from .llama import LlamaConfig, LlamaModel
 
@@ -139,20 +139,38 @@ def save_llama(model: LlamaModel, path) -> None:
               str(p / "model.safetensors"))
 
 
+def _load_hybrid(design, path, device="cuda", dtype=torch.bfloat16) -> HybridModel:
+    p = Path(path)
+    cfg = design.config_from_json(_config_json(p), name=p.name)
+    return HybridModel(cfg, device=device, dtype=dtype, weights=LazySafetensors(p))
+
+
 def load_saritar(path, device="cuda", dtype=torch.bfloat16) -> HybridModel:
     """Saritar checkpoint directory (config.json + model.safetensors) -> :class:`HybridModel`."""
-    p = Path(path)
-    cfg = saritar.config_from_json(_config_json(p), name=p.name)
-    return HybridModel(cfg, device=device, dtype=dtype, weights=LazySafetensors(p))
+    return _load_hybrid(saritar, path, device, dtype)
+
+
+def load_dolodra(path, device="cuda", dtype=torch.bfloat16) -> HybridModel:
+    """Dolodra checkpoint directory (config.json + model.safetensors) -> :class:`HybridModel`."""
+    return _load_hybrid(dolodra, path, device, dtype)
 
 
 def save_saritar(cfg, weights: Mapping, path) -> None:
     """Write a Saritar checkpoint: ``weights`` by :meth:`HybridConfig.tensor_shapes` name, in bf16."""
+    _save_hybrid(saritar, cfg, weights, path)
+
+
+def save_dolodra(cfg, weights: Mapping, path) -> None:
+    """Write a Dolodra checkpoint: ``weights`` by :meth:`HybridConfig.tensor_shapes` name, in bf16."""
+    _save_hybrid(dolodra, cfg, weights, path)
+
+
+def _save_hybrid(design, cfg, weights: Mapping, path) -> None:
     from safetensors.torch import save_file
 
     p = Path(path)
     p.mkdir(parents=True, exist_ok=True)
-    (p / "config.json").write_text(json.dumps(saritar.config_to_json(cfg), indent=1))
+    (p / "config.json").write_text(json.dumps(design.config_to_json(cfg), indent=1))
     save_file({k: weights[k].detach().to(torch.bfloat16).cpu().contiguous() for k in cfg.tensor_shapes()},
               str(p / "model.safetensors"))
 
@@ -179,6 +197,10 @@ class DecoderFamily:
 FAMILIES = (
     DecoderFamily("saritar", lambda js: js.get("architecture") == saritar.ARCHITECTURE,
                   lambda n: n.startswith("saritar"), saritar.config_from_json, saritar.preset, load_saritar,
+                  lambda cfg, device, dtype, seed: HybridModel(cfg, device=device, dtype=dtype, seed=seed),
+                  (torch.bfloat16, torch.float32)),
+    DecoderFamily("dolodra", lambda js: js.get("architecture") == dolodra.ARCHITECTURE,
+                  lambda n: n.startswith("dolodra"), dolodra.config_from_json, dolodra.preset, load_dolodra,
                   lambda cfg, device, dtype, seed: HybridModel(cfg, device=device, dtype=dtype, seed=seed),
                   (torch.bfloat16, torch.float32)),
     DecoderFamily("llama", lambda js: "architecture" not in js, lambda n: True, llama_config_from_hf,
@@ -327,6 +349,7 @@ def tokenizer_json(name_or_path) -> str | None:
 
 
 __all__ = ["LazySafetensors", "is_checkpoint", "load_llama", "save_llama", "load_saritar", "save_saritar",
+           "load_dolodra", "save_dolodra",
            "DecoderFamily", "FAMILIES", "decoder_family", "resolve_decoder", "resolve_decoder_config",
            "resolve_llama", "resolve_llama_config", "load_bert_encoder", "load_bert_token_classifier", "resolve_bert",
            "resolve_bert_config", "tokenizer_json", "use_checkpoint_tokenizers", "llama_config_from_hf", "bert_config_from_hf"]

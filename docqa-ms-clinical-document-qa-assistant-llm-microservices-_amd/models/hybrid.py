@@ -1,9 +1,13 @@
-"""Decoders whose layers mix windowed attention with recurrent (selective-scan) mixers, with
-an fp32 residual stream and a norm before and after every sublayer.
+"""Decoders made of windowed attention, latent attention and recurrent (selective-scan)
+mixers, with an fp32 residual stream.
 
-A model is a list of layers (:class:`LayerSpec`: a mixer and an optional feed-forward), some
-of which may run several passes over the same weights (``loop``).  Every RUN of a layer has
-its own cache or state, so the engine sees as many caches as runs.
+A model is a list of layers (:class:`LayerSpec`: a mixer and an optional feed-forward) in one
+of two forms: a norm before and after every sublayer, one after the other, or -- with a
+:class:`ParallelForm` -- one norm whose output both sublayers read, a convolution over time
+ahead of the mixer and a second input from the token's side embedding.  Layers may run
+several passes over the same weights (``loop``).  Every RUN of a layer has its own cache or
+state, so the engine sees as many caches as runs; a latent-attention layer may read the cache
+of an earlier one (``kv_from``) instead.
 
 MI355X layout:
   * one sandwich_norm.hip launch stands between any two projections: it sums the split-K
@@ -15,6 +19,12 @@ MI355X layout:
     conv and scan over packed sequences in prefill; in decode the conv step reads the in_proj
     slabs, and dt_proj, scan step and gate are one launch; the state is in per-request slots
     (engine/kv_cache.py StatePool);
+  * latent attention caches one row a token for all heads and attends in one of two forms:
+    with the key / value projections absorbed into the query and the output (decode, short
+    portions: the cached row is key and value), or with keys and values of the visible rows
+    made once by a GEMM (prompts);
+  * the parallel form's stream update, side input, next norm and (decode) convolution step are
+    two launches around the side input's two small projections;
   * projections run on the same GEMM plans as the Llama decoder (ops.project / ops.linear):
     weights are padded with zero rows at load where that reaches a kernel's granule.
 
@@ -58,9 +68,36 @@ class SelectiveScanSpec:
 
 
 @dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Causal attention over the last ``window`` tokens whose per-head keys (``dim``) and values
+    (``vdim``) are linear in one normed latent of ``kv_rank`` a token, with ``rot_dim`` more
+    query / key dimensions rotated by position (key part shared by the heads) and a learned
+    sink per head.  ``kv_from``: reads the latents of that layer's cache."""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    window: int
+    rope_base: float
+    kv_from: int | None = None
+
+
+@dataclass(frozen=True)
+class ParallelForm:
+    """Layers x <- x + mult (mixer(h + conv(h)) + ff(h)), h = norm1(x), then
+    x <- x + mult rms(proj(gelu(gate x) * e)) * norm with e the layer's part of the token's
+    side embedding.  ``conv`` taps, ``side`` elements of e."""
+    mult: float
+    conv: int
+    side: int
+
+
+@dataclass(frozen=True)
 class LayerSpec:
-    mixer: WindowAttentionSpec | SelectiveScanSpec
-    ff: int = 0                     # squared-ReLU feed-forward width, 0: none
+    mixer: WindowAttentionSpec | SelectiveScanSpec | LatentAttentionSpec
+    ff: int = 0                     # feed-forward width, 0: none
 
 
 @dataclass
@@ -72,6 +109,10 @@ class HybridConfig:
     embed_scale: float = 1.0
     rms_eps: float = 1e-5
     loop: tuple | None = None       # (start, stop, times)
+    parallel: ParallelForm | None = None    # None: norms around every sublayer
+    act: str = ops.ACT_RELU2        # of the feed-forward
+    norm_offset: float = 0.0        # added to the stored weights of the layers' and final norms
+    logit_softcap: float | None = None
     max_position: int = 1 << 20     # no position enters the weights
     bos_token_id: int = -1          # no special tokens of its own
     eos_token_id: int = -1
@@ -87,8 +128,23 @@ class HybridConfig:
         for p in range(times if body else 0):
             self.runs += [(i, p > 0 and i == lo) for i in body]
         self.runs += [(i, False) for i in range(hi, n)]
-        for sp in self.layer_specs:
+        if self.parallel is not None:
+            if self.loop is not None or not all(isinstance(s.mixer, LatentAttentionSpec) for s in self.layer_specs):
+                raise ValueError("parallel layers: latent attention, no loop")
+            if self.parallel.conv < 1 or self.parallel.side < 1:
+                raise ValueError(f"unsupported sizes {self.parallel}")
+        for i, sp in enumerate(self.layer_specs):
             m = sp.mixer
+            if isinstance(m, LatentAttentionSpec):
+                if m.rot_dim % 2 or m.window < 1 or m.kv_rank > 2048 or min(m.heads, m.dim, m.vdim, m.kv_rank, m.rot_dim) < 1:
+                    raise ValueError(f"unsupported attention sizes {m}")
+                if m.kv_from is not None:
+                    src = self.layer_specs[m.kv_from].mixer if 0 <= m.kv_from < i else None
+                    if not isinstance(src, LatentAttentionSpec) or src.kv_from is not None or (
+                            (src.kv_rank, src.rot_dim, src.rope_base) != (m.kv_rank, m.rot_dim, m.rope_base)):
+                        raise ValueError(f"layer {i}: kv_from {m.kv_from} is no earlier layer with such latents of its own")
+                elif self.parallel is None:
+                    raise ValueError("latent attention runs in parallel layers")
             if isinstance(m, WindowAttentionSpec) and (m.heads % m.kv_heads or m.window < 1 or m.dim > 512):
                 raise ValueError(f"unsupported attention sizes {m}")
             if isinstance(m, SelectiveScanSpec) and (m.state > 256 or m.conv < 1):
@@ -101,11 +157,24 @@ class HybridConfig:
     def tensor_shapes(self) -> dict:
         """Every weight's name and shape (linear weights [out, in])."""
         W, V = self.hidden, self.vocab_size
-        out = {"embed": (V, W)}
+        out, par = {"embed": (V, W)}, self.parallel
+        if par is not None:
+            out["side.embed"] = (V, self.layers * par.side)
         for i, sp in enumerate(self.layer_specs):
             p, m = f"l{i}.", sp.mixer
-            out[p + "norm1"] = out[p + "norm1b"] = (W,)
-            if isinstance(m, WindowAttentionSpec):
+            out[p + "norm1"] = (W,)
+            if par is None:
+                out[p + "norm1b"] = (W,)
+            else:
+                out.update({p + "canon1": (W, par.conv), p + "side.gate": (par.side, W), p + "side.proj": (W, par.side),
+                            p + "side.norm": (W,)})
+            if isinstance(m, LatentAttentionSpec):
+                H, R = m.heads, m.kv_rank
+                out.update({p + "mix.q": (H * (m.dim + m.rot_dim), W), p + "mix.uk": (H * m.dim, R),
+                            p + "mix.uv": (H * m.vdim, R), p + "mix.sink": (H,), p + "mix.o": (W, H * m.vdim)})
+                if m.kv_from is None:
+                    out.update({p + "mix.dkv": (R + m.rot_dim, W), p + "mix.dkv.norm": (R,)})
+            elif isinstance(m, WindowAttentionSpec):
                 hd = m.heads * m.dim
                 out.update({p + "mix.q": (hd, W), p + "mix.k": (m.kv_heads * m.dim, W), p + "mix.q.norm": (m.dim,),
                             p + "mix.k.norm": (m.dim,), p + "mix.sink": (m.heads,), p + "mix.o": (W, hd)})
@@ -115,7 +184,9 @@ class HybridConfig:
                             p + "mix.x": (R + 2 * N, C), p + "mix.dt": (C, R), p + "mix.dt.b": (C,),
                             p + "mix.A_log": (C, N), p + "mix.D": (C,), p + "mix.o": (W, C)})
             if sp.ff:
-                out.update({p + "norm2": (W,), p + "norm2b": (W,), p + "mlp.up": (sp.ff, W), p + "mlp.down": (W, sp.ff)})
+                out.update({p + "mlp.up": (sp.ff, W), p + "mlp.down": (W, sp.ff)})
+                if par is None:
+                    out.update({p + "norm2": (W,), p + "norm2b": (W,)})
         out.update({"final.norm": (W,), "head": (V, W)})
         return out
 
@@ -138,6 +209,35 @@ class _Part:
     @property
     def decode(self) -> bool:
         return not self.meta.prefill
+
+
+class _Keys:
+    """The visible keys of a prompt batch under one window: every sequence's [first, end) rows,
+    packed (``cu``), and how many there are."""
+
+    def __init__(self, spans: list, window: int, device):
+        lo = [max(0, a - window + 1) for a, _ in spans]
+        cu = [0]
+        for k, (_, e) in zip(lo, spans):
+            cu.append(cu[-1] + e - k)
+        t = torch.tensor(lo + cu, dtype=torch.int32)
+        t = (t.pin_memory() if device.type == "cuda" else t).to(device, non_blocking=True)
+        self.first, self.cu, self.total = t[:len(lo)], t[len(lo):], cu[-1]
+        self.tokens = sum(e - a for a, e in spans)
+
+        def seen(n):           # (query, key) pairs of positions below n
+            k = min(n, window)
+            return k * (k + 1) // 2 + (n - k) * window
+
+        self.pairs = sum(seen(e) - seen(a) for a, e in spans)
+
+
+@dataclass
+class _Forward:
+    """What the layers of one forward share: rotation tables by (base, dims), the visible keys of
+    prompts by window."""
+    rope: dict
+    keys: dict
 
 
 def _split(t: torch.Tensor, part: _Part, parts: list) -> torch.Tensor:
@@ -239,13 +339,122 @@ class SelectiveScan:
         return ops.project(_join(out), self.w_o, decode)
 
 
-class SquaredReluMLP:
-    def __init__(self, get, dtype):
+class LatentAttention:
+    def __init__(self, sp: LatentAttentionSpec, get, eps: float, dtype):
+        self.sp, self.eps, self.dtype = sp, eps, dtype
+        H, d, vd, R = sp.heads, sp.dim, sp.vdim, sp.kv_rank
+        self.d8, self.r8, self.R8, self.v8 = (_pad_up(n, 8) for n in (d, sp.rot_dim, R, vd))
+        rows = [get("q")] + ([get("dkv")] if sp.kv_from is None else [])
+        n = sum(t.shape[0] for t in rows)
+        rows.append(rows[0].new_zeros(_pad_up(n, 256 if n >= 1024 else 64) - n, rows[0].shape[1]))
+        self.w_in = torch.cat(rows).to(dtype).contiguous()          # q | latent | key part
+        self.c_norm = get("dkv.norm").float().contiguous() if sp.kv_from is None else None
+        uk, uv = get("uk").view(H, d, R), get("uv").view(H, vd, R)
+        pad = torch.nn.functional.pad
+        # absorbed: query heads into the latent space, attended latents to values
+        self.w_qc = pad(uk.transpose(1, 2), (0, self.d8 - d, 0, self.R8 - R)).to(dtype).contiguous()   # [H, R8, d8]
+        self.w_cv = pad(uv, (0, self.R8 - R)).to(dtype).contiguous()                                   # [H, vd, R8]
+        # expanded: every head's keys, then values
+        self.w_kv = None
+        if ops.packed_attn_ok(dtype, self.d8, self.r8, vd):
+            kv = torch.cat([pad(uk, (0, self.R8 - R, 0, self.d8 - d)).reshape(H * self.d8, self.R8),
+                            pad(uv, (0, self.R8 - R, 0, self.v8 - vd)).reshape(H * self.v8, self.R8)])
+            n = kv.shape[0]
+            self.w_kv = pad(kv, (0, 0, 0, _pad_up(n, 256 if n >= 1024 else 64) - n)).to(dtype).contiguous()
+        self.sink = get("sink").float().contiguous()
+        self.o = get("o").to(dtype).contiguous()
+        self.rope_key = (sp.rope_base, sp.rot_dim)
+
+    def cache_spec(self):
+        """Its own rows, or (``kv_from``) the index of the run whose rows it reads."""
+        return KVSpec(1, self.R8 + self.r8, latent=True) if self.sp.kv_from is None else self.sp.kv_from
+
+    def activation_elems(self) -> int:
+        H = self.sp.heads
+        return self.w_in.shape[0] + H * (self.d8 + self.r8 + self.sp.vdim) + 2 * H * (self.d8 + self.v8)
+
+    def _expanded(self, keys: _Keys | None) -> bool:
+        """Whether making keys and values of the visible rows costs less than attending in the
+        latent space (multiply-adds a head; the absorbed projections are one product a query)."""
+        if keys is None or self.w_kv is None:
+            return False
+        kv = self.d8 + self.v8
+        return (keys.total * self.R8 * kv + keys.pairs * (kv + self.r8)
+                < keys.tokens * self.R8 * kv + keys.pairs * (2 * self.R8 + self.r8))
+
+    def run(self, x, parts, slot_mapping, cache, decode, fw: _Forward):
+        sp = self.sp
+        q = ops.latent_store(ops.project(x, self.w_in, decode), fw.rope[self.rope_key], slot_mapping, cache, self.c_norm,
+                             sp.heads, sp.dim, sp.kv_rank, self.eps, self.dtype)
+        out = []
+        for p in parts:
+            m, qp = p.meta, _split(q, p, parts)
+            keys = None if p.decode else fw.keys.get(sp.window)
+            if self._expanded(keys):
+                c, kr = ops.latent_gather(cache, m.block_tables, keys.first, keys.cu, keys.total, self.R8)
+                out.append(ops.packed_window_attn(qp, ops.linear(c, self.w_kv), kr, sp.heads, sp.dim, sp.vdim, m.cu_seqlens,
+                                                  keys.cu, m.max_len, sp.scale, window=sp.window, sink=self.sink))
+                continue
+            qc = ops.head_project(qp, self.w_qc, self.r8)
+            kw = dict(window=sp.window, sink=self.sink, v_dim=self.R8)
+            if p.decode:
+                a = ops.window_attn(qc, cache, m.block_tables, m.context_lens, sp.scale, **kw)
+            else:
+                a = ops.window_attn(qc, cache, m.block_tables, m.prefix_lens, sp.scale, cu=m.cu_seqlens,
+                                    max_q=m.max_len, **kw)
+            out.append(ops.head_project(a, self.w_cv))
+        return ops.project(_join(out), self.o, decode)
+
+
+class MLP:
+    """down(act(up x))."""
+
+    def __init__(self, get, dtype, act: str):
         self.up = get("up").to(dtype).contiguous()
         self.down = get("down").to(dtype).contiguous()
+        self.act = act
 
     def run(self, x, decode):
-        return ops.project(ops.relu2_linear(x, self.up, decode), self.down, decode)
+        return ops.project(ops.act_linear(x, self.up, self.act, decode), self.down, decode)
+
+
+class InputConv:
+    """h + conv(h): the causal convolution per channel ahead of a mixer, the identity in its
+    last tap."""
+
+    def __init__(self, w):
+        w = w.float().t().contiguous()                              # [taps, W]
+        w[-1] += 1.0
+        self.w = w
+
+    def cache_spec(self):
+        return StateSpec((((self.w.shape[0] - 1), self.w.shape[1]),), (False,))
+
+    def run(self, h, parts, state):
+        out = []
+        for p in parts:
+            m, x = p.meta, _split(h, p, parts)
+            if p.decode:
+                out.append(ops.conv_step(x, self.w, None, state, m.state_slots, m.positions, silu=False)[0])
+            else:
+                out.append(ops.causal_conv(x, self.w, None, state, m.state_slots, m.cu_seqlens, m.prefix_lens, m.max_len,
+                                           silu=False))
+        return _join(out)
+
+
+class SideInput:
+    """proj(gelu(gate x) * e), e = columns [col, col + n) of the token's side embedding."""
+
+    def __init__(self, get, dtype, col: int):
+        gate, proj = get("gate"), get("proj")
+        n = gate.shape[0]
+        pad = _pad_up(n, 256 if n > 128 else 64) - n                # zero rows: a zero gate
+        self.gate = torch.cat([gate, gate.new_zeros(pad, gate.shape[1])]).to(dtype).contiguous()
+        self.proj = torch.cat([proj, proj.new_zeros(proj.shape[0], pad)], 1).to(dtype).contiguous()
+        self.col, self.n = col, n
+
+    def run(self, x, ids, table, decode):
+        return ops.side_project(ops.project(x, self.gate, decode), ids, table, self.col, self.n, self.proj, decode)
 
 
 class HybridModel(Decoder):
@@ -261,8 +470,8 @@ class HybridModel(Decoder):
         self.tp, self.tp_rank = 1, 0
         self.vocab_shard = self.vocab_valid = cfg.vocab_size
         self.vocab_start = 0
-        att = [s.mixer for s in cfg.layer_specs if isinstance(s.mixer, WindowAttentionSpec)]
-        self.hq, self.hkv = (att[0].heads, att[0].kv_heads) if att else (1, 1)
+        att = [s.mixer for s in cfg.layer_specs if not isinstance(s.mixer, SelectiveScanSpec)]
+        self.hq, self.hkv = (att[0].heads, getattr(att[0], "kv_heads", 1)) if att else (1, 1)
         self.tap = None           # a list: receives the residual stream after every run
         self._load(weights if weights is not None else _RandomWeights(cfg, self.device, seed))
 
@@ -276,36 +485,60 @@ class HybridModel(Decoder):
                 raise ValueError(f"{name}: shape {tuple(t.shape)}, expected {shapes[name]}")
             return t.to(self.device)
 
-        def norm(name):
+        def vec(name):
             return get(name).float().contiguous()
 
+        def norm(name):
+            return vec(name) + cfg.norm_offset if cfg.norm_offset else vec(name)
+
+        par = cfg.parallel
         self.embed = get("embed").to(dt).contiguous()
         self.lm_head = get("head").to(dt).contiguous()
         self.final_norm = norm("final.norm")
         self.layers = []
         for i, sp in enumerate(cfg.layer_specs):
             p = f"l{i}."
-            cls = WindowAttention if isinstance(sp.mixer, WindowAttentionSpec) else SelectiveScan
-            L = {"mixer": cls(sp.mixer, lambda n: get(p + "mix." + n), cfg.rms_eps, dt),
-                 "norm1": norm(p + "norm1"), "norm1b": norm(p + "norm1b"), "mlp": None}
+            L = {"mixer": _MIXERS[type(sp.mixer)](sp.mixer, lambda n: get(p + "mix." + n), cfg.rms_eps, dt),
+                 "norm1": norm(p + "norm1"), "mlp": None}
             if sp.ff:
-                L.update(mlp=SquaredReluMLP(lambda n: get(p + "mlp." + n), dt), norm2=norm(p + "norm2"),
-                         norm2b=norm(p + "norm2b"))
+                L["mlp"] = MLP(lambda n: get(p + "mlp." + n), dt, cfg.act)
+            if par is not None:
+                L.update(conv=InputConv(get(p + "canon1")), side_norm=vec(p + "side.norm") * par.mult,
+                         side=SideInput(lambda n: get(p + "side." + n), dt, i * par.side))
+            else:
+                L["norm1b"] = norm(p + "norm1b")
+                if sp.ff:
+                    L.update(norm2=norm(p + "norm2"), norm2b=norm(p + "norm2b"))
             self.layers.append(L)
+        if par is not None:
+            self.side_embed = get("side.embed").to(dt).contiguous()
+            self.rope_freq = {(b, r): b ** (-torch.arange(0, r, 2, dtype=torch.float64) / r) for b, r in
+                              {L["mixer"].rope_key for L in self.layers}}
+            self.rope_freq = {k: v.to(self.device) for k, v in self.rope_freq.items()}
+            self.windows = sorted({s.mixer.window for s, L in zip(cfg.layer_specs, self.layers)
+                                   if L["mixer"].w_kv is not None})
 
     # ------------------------------------------------------------------ caches
     def _run_specs(self) -> list:
-        return [self.layers[i]["mixer"].cache_spec() for i, _ in self.cfg.runs]
+        """Per run: what its mixer keeps (or, an integer, whose cache it reads), what its input
+        convolution keeps."""
+        return [[self.layers[i][k].cache_spec() for k in ("mixer", "conv") if k in self.layers[i]]
+                for i, _ in self.cfg.runs]
 
     def kv_specs(self) -> list:
-        return [s for s in self._run_specs() if isinstance(s, KVSpec)]
+        return [s for run in self._run_specs() for s in run if isinstance(s, KVSpec)]
 
     def state_specs(self) -> list:
-        return [s for s in self._run_specs() if isinstance(s, StateSpec)]
+        return [s for run in self._run_specs() for s in run if isinstance(s, StateSpec)]
 
     def bind_caches(self, kv, state) -> list:
+        """Per run its mixer's tensors; in the parallel form (latent rows, convolution inputs)."""
         k, s = iter(kv.caches), iter(state.states if state is not None else [])
-        return [next(k) if isinstance(sp, KVSpec) else next(s) for sp in self._run_specs()]
+        out = []
+        for run in self._run_specs():
+            own = [next(k) if isinstance(sp, KVSpec) else next(s) if isinstance(sp, StateSpec) else out[sp] for sp in run]
+            out.append(own[0] if len(own) == 1 else (own[0][0], own[1][0]))
+        return out
 
     def activation_elems(self) -> int:
         ff = max([s.ff for s in self.cfg.layer_specs] + [0])
@@ -331,6 +564,8 @@ class HybridModel(Decoder):
         return self._head(self._hidden(input_ids, parts, slots, caches), logits_index, not return_logits)
 
     def _hidden(self, input_ids, parts, slot_mapping, caches):
+        if self.cfg.parallel is not None:
+            return self._hidden_parallel(input_ids, parts, slot_mapping, caches)
         cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
         decode = all(p.decode for p in parts)
         runs = cfg.runs
@@ -352,12 +587,38 @@ class HybridModel(Decoder):
                 self.tap.append(res - add if add is not None else res.clone())
         return x
 
+    def _hidden_parallel(self, input_ids, parts, slot_mapping, caches):
+        cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
+        decode = all(p.decode for p in parts)
+        fw = _Forward({}, {})
+        for p in parts:
+            if not p.decode and p.meta.spans is not None:
+                fw.keys = {w: _Keys(p.meta.spans, w, self.device) for w in self.windows}
+        pos = _join([p.meta.positions for p in parts])
+        fw.rope = {k: ops.rope_table(pos, f) for k, f in self.rope_freq.items()}
+        first = self.layers[0]["norm1"] if self.layers else self.final_norm
+        res, _, h = ops.embed_scale_rmsnorm(input_ids, self.embed, cfg.embed_scale, first, eps)
+        for i, (L, (cache, conv_state)) in enumerate(zip(self.layers, caches)):
+            nxt = self.layers[i + 1]["norm1"] if i + 1 < len(self.layers) else self.final_norm
+            y = L["mixer"].run(L["conv"].run(h, parts, conv_state), parts, slot_mapping, cache, decode, fw)
+            f = L["mlp"].run(h, decode) if L["mlp"] is not None else None
+            xs = ops.add_scaled(y, f, res, cfg.parallel.mult, dt)
+            y = L["side"].run(xs, input_ids, self.side_embed, decode)
+            h = ops.sandwich_rmsnorm(y, res, L["side_norm"], nxt, eps, out_dtype=dt)
+            if self.tap is not None:
+                self.tap.append(res.clone())
+        return h
+
     def _head(self, x, logits_index, greedy_ids):
         if logits_index is not None:
             x = x.index_select(0, logits_index)
         if greedy_ids:
-            return self.greedy_ids(x)
-        return ops.lm_head_logits(x.contiguous(), self.lm_head)
+            return self.greedy_ids(x)          # (a soft cap keeps the order of the logits)
+        logits = ops.lm_head_logits(x.contiguous(), self.lm_head)
+        return logits if self.cfg.logit_softcap is None else ops.soft_cap(logits, self.cfg.logit_softcap)
+
+
+_MIXERS = {WindowAttentionSpec: WindowAttention, SelectiveScanSpec: SelectiveScan, LatentAttentionSpec: LatentAttention}
 
 
 class _RandomWeights:
@@ -365,7 +626,7 @@ class _RandomWeights:
     sizes in the range of trained selective-scan models."""
 
     def __init__(self, cfg: HybridConfig, device, seed: int):
-        self.shapes, self.device, self.seed = cfg.tensor_shapes(), device, seed
+        self.shapes, self.device, self.seed, self.offset = cfg.tensor_shapes(), device, seed, cfg.norm_offset
 
     def __getitem__(self, name: str) -> torch.Tensor:
         shape = self.shapes[name]
@@ -373,7 +634,8 @@ class _RandomWeights:
         g.manual_seed((self.seed * 1_000_003 + zlib.crc32(name.encode())) & 0x7FFFFFFFFFFF)
         kind = name.rsplit(".", 1)[-1]
         if name.endswith("norm") or kind.startswith("norm"):
-            return torch.ones(shape, device=self.device)
+            stored_off = self.offset if kind.startswith("norm1") or name == "final.norm" else 0.0
+            return torch.full(shape, 1.0 - stored_off, device=self.device)
         if kind == "A_log":
             return torch.log(torch.arange(1, shape[1] + 1, device=self.device).float()).expand(shape).contiguous()
         if kind == "D":

@@ -145,6 +145,8 @@ class AttnMeta:
     decode_inline: bool = False
     # state slot of each sequence (prefill) / row (decode, -1: padded) of a recurrent model
     state_slots: torch.Tensor | None = None
+    # (prefill) host copy of each sequence's [first, end) positions in this forward
+    spans: list | None = None
 
 
 class LlamaModel(Decoder):

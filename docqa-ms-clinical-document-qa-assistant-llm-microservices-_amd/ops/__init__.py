@@ -1211,15 +1211,24 @@ def sandwich_rmsnorm(P, residual, w_post, w_next, eps: float, add=None, out_dtyp
     return ref.sandwich_rmsnorm(P, residual, w_post, w_next, eps, add, out_dtype)
 
 
+ACT_RELU2, ACT_GELU_TANH = "relu2", "gelu_tanh"
+_ACT_CODE = {ACT_RELU2: 0, ACT_GELU_TANH: 1}
+
+
+def activation(P, act: str, out_dtype=torch.bfloat16):
+    """``act`` of a projection: max(P, 0)^2 ("relu2") or the tanh form of GELU ("gelu_tanh")."""
+    if _gpu(P):
+        return _native().slab_activation(P.contiguous(), _ACT_CODE[act], out_dtype == torch.float32)
+    return ref.activation(P, act, out_dtype)
+
+
 def squared_relu(P, out_dtype=torch.bfloat16):
     """max(P, 0)^2 of a projection."""
-    if _gpu(P):
-        return _native().squared_relu(P.contiguous(), out_dtype == torch.float32)
-    return ref.squared_relu(P, out_dtype)
+    return activation(P, ACT_RELU2, out_dtype)
 
 
-def relu2_linear(x, w, decode: bool = False):
-    """max(x @ w^T, 0)^2, the activation in the GEMM's epilogue where a hand-written bf16 GEMM
+def act_linear(x, w, act: str, decode: bool = False):
+    """act(x @ w^T), the activation in the GEMM's epilogue where a hand-written bf16 GEMM
     takes the shape without splitting K (the decode kernels, the 256 x 256 prefill kernel)."""
     if _gpu(x) and x.dtype == torch.bfloat16:
         N, K = w.shape
@@ -1227,10 +1236,48 @@ def relu2_linear(x, w, decode: bool = False):
         if (decode or M <= MID_M_MAX) and M > 1:
             if (M <= 128 and N % 64 == 0 and K % 512 == 0 and decode_plan(M, N, K)[0] == 1) or (
                     129 <= M <= MID_M_MAX and mid_plan(M, N, K)[0] == 1):
-                return _native().decode_relu2(x.contiguous(), w)
+                return _native().decode_act(x.contiguous(), w, _ACT_CODE[act])
         elif M > MID_M_MAX and pgemm_ok(M, N, K) and not prefill_split_plan(M, N, K):
-            return _native().pgemm(x.contiguous(), w, 3)
-    return squared_relu(project(x, w, decode), x.dtype)
+            return _native().pgemm(x.contiguous(), w, 3 + _ACT_CODE[act])
+    return activation(project(x, w, decode), act, x.dtype)
+
+
+def relu2_linear(x, w, decode: bool = False):
+    """max(x @ w^T, 0)^2."""
+    return act_linear(x, w, ACT_RELU2, decode)
+
+
+def add_scaled(P, Q, residual, m: float, out_dtype=torch.bfloat16):
+    """residual (fp32, in place) += m (P + Q) of one or two projections (``Q`` None: one);
+    returns it in ``out_dtype`` (fp32: itself)."""
+    if _gpu(P):
+        out = _native().add_scaled(P.contiguous(), None if Q is None else Q.contiguous(), residual, float(m),
+                                   out_dtype == torch.float32)
+        return residual if out_dtype == torch.float32 else out
+    return ref.add_scaled(P, Q, residual, m, out_dtype)
+
+
+def side_gate(P, ids, table, col: int, n: int, out_dtype=torch.bfloat16):
+    """gelu_tanh(P) times columns [col, col + n) of ``table[ids]``; columns of ``P`` past n (a
+    padded projection) give zero."""
+    if _gpu(P):
+        return _native().side_gate(P.contiguous(), ids, table, int(col), int(n), out_dtype == torch.float32)
+    return ref.side_gate(P, ids, table, col, n, out_dtype)
+
+
+def side_project(P, ids, table, col: int, n: int, w, decode: bool = False):
+    """:func:`side_gate` of the gate projection ``P``, projected by ``w``: one launch for bf16
+    decode rows, where a row's gate is cheap to build in every workgroup."""
+    if _gpu(P) and w.dtype == torch.bfloat16 and P.shape[-2] <= MID_M_MAX and w.shape[1] <= 1024:
+        return _native().side_project(P.contiguous(), ids, table, int(col), int(n), w)
+    return project(side_gate(P, ids, table, col, n, w.dtype), w, decode)
+
+
+def soft_cap(x, cap: float):
+    """cap tanh(x / cap) in fp32."""
+    if _gpu(x):
+        return _native().soft_cap(x.contiguous(), float(cap))
+    return ref.soft_cap(x, cap)
 
 
 def slab_columns(P, n0: int, n1: int, out_dtype=torch.bfloat16):
@@ -1251,32 +1298,86 @@ def qk_norm_store(P, w, slots, k_cache, k_scale, H: int, eps: float):
 
 
 def window_attn(q, k_cache, block_tables, ctx, scale: float, window: int = 0, sink=None, k_scale=None, v_cache=None,
-                cu=None, max_q: int = 1):
+                cu=None, max_q: int = 1, v_dim: int = 0):
     """Causal attention over the last ``window`` tokens (0: all) of the paged cache, scores
     times ``k_scale`` per cached key, ``sink`` [H] in the denominator, ``v_cache`` None: the
-    keys are the values.  With ``cu`` [B + 1]: packed query tokens, ``ctx`` the position of
-    each sequence's first; without: one query token a row, ``ctx`` the context lengths."""
+    keys are the values -- their first ``v_dim`` elements (0: all of them).  With ``cu``
+    [B + 1]: packed query tokens, ``ctx`` the position of each sequence's first; without: one
+    query token a row, ``ctx`` the context lengths."""
     if _gpu(q):
         return _native().window_attn(q.contiguous(), k_cache, v_cache, k_scale, block_tables, cu, ctx, int(max_q),
-                                     float(scale), int(window), sink)
-    return ref.window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink)
+                                     float(scale), int(window), sink, int(v_dim))
+    return ref.window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink, v_dim)
 
 
-def causal_conv(x, w, bias, state, slots, cu, ctx, max_len: int):
-    """silu(causal convolution) of the first C columns of packed rows ``x``; ``w`` [taps, C]
-    (last row: the current token).  ``state`` [slots, taps - 1, C]: the inputs ahead of each
-    sequence's portion (``ctx`` > 0), replaced by its last ones."""
-    if _gpu(x):
-        return _native().causal_conv(x, w, bias, state, slots, cu, ctx, int(max_len))
-    return ref.causal_conv(x, w, bias, state, slots, cu, ctx)
+# Latent attention (csrc/kernels/attn_latent.hip).  A cached row is [latent: R | rotated key
+# part: r], each padded with zeros to 8 elements (R8, r8); a query head is [unrotated: d |
+# rotated: r], padded alike (d8, r8).
+def rope_table(positions, inv_freq):
+    """fp32 [cos | sin] rows of the angles position * inv_freq (``inv_freq`` fp64 [r / 2])."""
+    if _gpu(positions):
+        return _native().rope_table(positions, inv_freq)
+    return ref.rope_table(positions, inv_freq)
 
 
-def conv_step(P, w, bias, state, slots, positions):
-    """One token a row: (silu(conv) [B, C], gate [B, C]) of an [x | z] projection; advances
-    ``state`` (rows with slot -1 leave none)."""
+def latent_store(P, cs, slots, cache, c_norm, H: int, dim: int, rank: int, eps: float, dtype):
+    """Of a projection [q: H (dim + r) | latent: rank | key part: r]: the query heads, rotated by
+    the rows ``cs`` of :func:`rope_table` [T, H (d8 + r8)]; the cache row -- normed latent times
+    ``c_norm``, rotated key part -- into ``cache`` (``c_norm`` None: the projection is q only)."""
     if _gpu(P):
-        return _native().conv_step(P.contiguous(), w, bias, state, slots, positions)
-    return ref.conv_step(P, w, bias, state, slots, positions)
+        return _native().latent_store(P.contiguous(), cs, slots, cache, c_norm, int(H), int(dim), int(rank), float(eps))
+    return ref.latent_store(P, cs, slots, cache, c_norm, H, dim, rank, eps, dtype)
+
+
+def head_project(x, w, carry: int = 0):
+    """Per head: x [T, H (K + carry)] rows' first K elements times ``w`` [H, N, K]^T, followed by
+    the other ``carry`` as they are: [T, H (N + carry)]."""
+    if _gpu(x) and x.dtype == torch.bfloat16:
+        return _native().head_project(x.contiguous(), w, int(carry))
+    return ref.head_project(x, w, carry)
+
+
+def latent_gather(cache, block_tables, first, cu_k, total: int, rank: int):
+    """Cached rows of positions [first[b], first[b] + n_b), n_b = cu_k[b + 1] - cu_k[b], of every
+    sequence, packed: (latents [total, rank], key parts [total, r8]); ``rank`` = R8."""
+    if _gpu(cache):
+        return _native().latent_gather(cache, block_tables, first, cu_k, int(total), int(rank))
+    return ref.latent_gather(cache, block_tables, first, cu_k, total, rank)
+
+
+def packed_window_attn(q, kv, kr, H: int, dim: int, vdim: int, cu, cu_k, max_q: int, scale: float, window: int = 0,
+                       sink=None):
+    """Causal attention of packed queries [T, H (d8 + r8)] over packed keys and values: ``kv``
+    [keys, >= H d8 + H v8] per-head keys then values, ``kr`` [keys, r8] the key part all heads
+    share.  Sequence b's keys end at its last query token.  [T, H vdim]."""
+    if _gpu(q):
+        return _native().packed_window_attn(q.contiguous(), kv, kr, int(H), int(dim), int(vdim), cu, cu_k, int(max_q),
+                                            float(scale), int(window), sink)
+    return ref.packed_window_attn(q, kv, kr, H, dim, vdim, cu, cu_k, scale, window, sink)
+
+
+def packed_attn_ok(dtype, dim: int, rot: int, vdim: int) -> bool:
+    """Head sizes the packed kernel takes (MFMA, bf16)."""
+    return dtype == torch.bfloat16 and dim + rot <= 256 and vdim <= 256 and vdim % 4 == 0
+
+
+def causal_conv(x, w, bias, state, slots, cu, ctx, max_len: int, silu: bool = True):
+    """Causal convolution of the first C columns of packed rows ``x`` (silu of it, unless not);
+    ``w`` [taps, C] (last row: the current token), ``bias`` [C] or None.  ``state`` [slots,
+    taps - 1, C]: the inputs ahead of each sequence's portion (``ctx`` > 0), replaced by its
+    last ones."""
+    if _gpu(x):
+        return _native().causal_conv(x, w, bias, state, slots, cu, ctx, int(max_len), silu)
+    return ref.causal_conv(x, w, bias, state, slots, cu, ctx, silu)
+
+
+def conv_step(P, w, bias, state, slots, positions, silu: bool = True):
+    """One token a row: (conv [B, C], gate [B, C]) of an [x | z] projection -- (conv, None) of an
+    [x] one; advances ``state`` (rows with slot -1 leave none)."""
+    if _gpu(P):
+        y, z = _native().conv_step(P.contiguous(), w, bias, state, slots, positions, silu)
+        return y, (z if z.numel() else None)
+    return ref.conv_step(P, w, bias, state, slots, positions, silu)
 
 
 def scan_chunk(tokens: int, max_len: int, channels: int) -> int:

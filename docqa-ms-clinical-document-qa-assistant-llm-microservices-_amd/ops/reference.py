@@ -363,8 +363,67 @@ def embed_scale_rmsnorm(ids, table, scale, w, eps, keep):
     return h, (h.clone() if keep else None), (_rms(h, eps) * w).to(table.dtype)
 
 
-def squared_relu(P, out_dtype):
-    return _slab_sum(P).clamp(min=0).square().to(out_dtype)
+def activation(P, act, out_dtype):
+    x = _slab_sum(P)
+    return (F.gelu(x, approximate="tanh") if act == "gelu_tanh" else x.clamp(min=0).square()).to(out_dtype)
+
+
+def add_scaled(P, Q, residual, m, out_dtype):
+    y = _slab_sum(P)
+    residual.add_((y if Q is None else y + _slab_sum(Q)) * m)
+    return residual.to(out_dtype)
+
+
+def side_gate(P, ids, table, col, n, out_dtype):
+    x = _slab_sum(P)
+    e = torch.zeros_like(x)
+    e[:, :n] = table[ids.long(), col:col + n].float()
+    return (F.gelu(x, approximate="tanh") * e).to(out_dtype)
+
+
+def soft_cap(x, cap):
+    return cap * torch.tanh(x.float() / cap)
+
+
+def rope_table(positions, inv_freq):
+    a = positions.double()[:, None] * inv_freq
+    return torch.cat([a.cos(), a.sin()], -1).float()
+
+
+def _rotate(x, cs):
+    """x [T, ..., r] by the [cos | sin] rows cs [T, r], dimension i paired with i + r / 2."""
+    h = x.shape[-1] // 2
+    cs = cs.view(cs.shape[0], *[1] * (x.dim() - 2), 2 * h)
+    u, v, c, s = x[..., :h], x[..., h:], cs[..., :h], cs[..., h:]
+    return torch.cat([u * c - v * s, v * c + u * s], -1)
+
+
+def latent_store(P, cs, slots, cache, c_norm, H, dim, rank, eps, dtype):
+    x = _slab_sum(P)
+    T, r = cs.shape
+    d8, r8 = -(-dim // 8) * 8, -(-r // 8) * 8
+    q = torch.zeros(T, H, d8 + r8, dtype=dtype, device=x.device)
+    xq = x[:, :H * (dim + r)].view(T, H, dim + r)
+    q[..., :dim] = xq[..., :dim].to(dtype)
+    q[..., d8:d8 + r] = _rotate(xq[..., dim:], cs).to(dtype)
+    if c_norm is not None:
+        BS, D = cache.shape[2:]
+        xk = x[:, H * (dim + r):H * (dim + r) + rank + r]
+        row = torch.zeros(T, D, dtype=cache.dtype, device=x.device)
+        row[:, :rank] = (_rms(xk[:, :rank], eps) * c_norm).to(cache.dtype)
+        row[:, D - r8:D - r8 + r] = _rotate(xk[:, rank:], cs).to(cache.dtype)
+        sm = slots.long()
+        ok = sm >= 0
+        cache[sm[ok] // BS, 0, sm[ok] % BS] = row[ok]
+    return q.view(T, H * (d8 + r8))
+
+
+def head_project(x, w, carry):
+    H, N, K = w.shape
+    T = x.shape[0]
+    xh = x.view(T, H, -1)
+    y = torch.matmul(xh[..., :K].float().transpose(0, 1), w.float().transpose(1, 2)).transpose(0, 1).to(x.dtype)
+    return torch.cat([y, xh[..., K:K + carry]], -1).reshape(T, H * (N + carry)) if carry else y.reshape(T, H * N)
 
 
 def qk_norm_store(P, w, slots, k_cache, k_scale, H, eps):
@@ -381,11 +440,12 @@ def qk_norm_store(P, w, slots, k_cache, k_scale, H, eps):
     return q
 
 
-def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink):
+def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink, v_dim):
     NB, G, BS, D = k_cache.shape
     H = q.shape[1] // D
     v_cache = k_cache if v_cache is None else v_cache
-    out = torch.zeros_like(q)
+    v_dim = v_dim or D
+    out = q.new_zeros(q.shape[0], H * v_dim)
     for b in range(block_tables.shape[0]):
         q0, L, p0 = (b, 1, int(ctx[b]) - 1) if cu is None else (int(cu[b]), int(cu[b + 1] - cu[b]), int(ctx[b]))
         if L <= 0 or p0 < 0:
@@ -395,7 +455,7 @@ def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, wind
         pos = torch.arange(lo, n, device=q.device)
         blk, off = block_tables[b, (pos // BS)].long(), pos % BS
         k = k_cache[blk, :, off].float().transpose(0, 1)                # [G, keys, D]
-        v = v_cache[blk, :, off].float().transpose(0, 1)
+        v = v_cache[blk, :, off, :v_dim].float().transpose(0, 1)
         qb = q[q0:q0 + L].view(L, G, H // G, D).float().permute(1, 2, 0, 3)
         s = torch.einsum("ghld,gkd->ghlk", qb, k) * scale
         if k_scale is not None:
@@ -409,11 +469,43 @@ def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, wind
             s = torch.cat([s, sink.float().view(G, H // G, 1, 1).expand(G, H // G, L, 1)], -1)
         p = torch.softmax(s, -1)[..., :n - lo]
         o = torch.einsum("ghlk,gkd->ghld", p, v)
-        out[q0:q0 + L] = o.permute(2, 0, 1, 3).reshape(L, H * D).to(q.dtype)
+        out[q0:q0 + L] = o.permute(2, 0, 1, 3).reshape(L, H * v_dim).to(q.dtype)
     return out
 
 
-def causal_conv(x, w, bias, state, slots, cu, ctx):
+def latent_gather(cache, block_tables, first, cu_k, total, rank):
+    BS, D = cache.shape[2:]
+    out = cache.new_zeros(total, D)
+    for b in range(block_tables.shape[0]):
+        k0, n = int(first[b]), int(cu_k[b + 1] - cu_k[b])
+        pos = torch.arange(k0, k0 + n, device=cache.device)
+        out[int(cu_k[b]):int(cu_k[b + 1])] = cache[block_tables[b, pos // BS].long(), 0, pos % BS]
+    return out[:, :rank].contiguous(), out[:, rank:].contiguous()
+
+
+def packed_window_attn(q, kv, kr, H, dim, vdim, cu, cu_k, scale, window, sink):
+    r8 = kr.shape[1]
+    d8, v8 = -(-dim // 8) * 8, -(-vdim // 8) * 8
+    out = q.new_zeros(q.shape[0], H * vdim)
+    for b in range(cu.numel() - 1):
+        q0, L, k0, n = int(cu[b]), int(cu[b + 1] - cu[b]), int(cu_k[b]), int(cu_k[b + 1] - cu_k[b])
+        if L <= 0:
+            continue
+        qb = q[q0:q0 + L].view(L, H, d8 + r8).float()
+        k = kv[k0:k0 + n, :H * d8].view(n, H, d8).float()
+        v = kv[k0:k0 + n, H * d8:H * (d8 + v8)].view(n, H, v8).float()
+        s = torch.einsum("lhd,khd->hlk", qb[..., :d8], k) + torch.einsum("lhr,kr->hlk", qb[..., d8:], kr[k0:k0 + n].float())
+        i, j = torch.arange(n - L, n, device=q.device)[:, None], torch.arange(n, device=q.device)[None]
+        dead = (j > i) | (j <= i - window) if window > 0 else j > i
+        s = (s * scale).masked_fill(dead, -math.inf)
+        if sink is not None:
+            s = torch.cat([s, sink.float().view(H, 1, 1).expand(H, L, 1)], -1)
+        p = torch.softmax(s, -1)[..., :n]
+        out[q0:q0 + L] = torch.einsum("hlk,khd->lhd", p, v)[..., :vdim].reshape(L, H * vdim).to(q.dtype)
+    return out
+
+
+def causal_conv(x, w, bias, state, slots, cu, ctx, silu=True):
     taps, C = w.shape
     y = torch.empty(x.shape[0], C, dtype=x.dtype, device=x.device)
     for b in range(cu.numel() - 1):
@@ -423,21 +515,22 @@ def causal_conv(x, w, bias, state, slots, cu, ctx):
         head = (state[slot] if slot >= 0 and int(ctx[b]) > 0
                 else torch.zeros(taps - 1, C, dtype=x.dtype, device=x.device))
         seq = torch.cat([head, x[q0:q1, :C]])
-        acc = bias.expand(q1 - q0, C).clone()
+        acc = (w.new_zeros(C) if bias is None else bias).expand(q1 - q0, C).clone()
         for k in range(taps):
             acc += w[k] * seq[k:k + q1 - q0].float()
-        y[q0:q1] = F.silu(acc).to(x.dtype)
+        y[q0:q1] = (F.silu(acc) if silu else acc).to(x.dtype)
         if slot >= 0 and taps > 1:
             state[slot] = seq[-(taps - 1):]
     return y
 
 
-def conv_step(P, w, bias, state, slots, positions):
+def conv_step(P, w, bias, state, slots, positions, silu=True):
     C = w.shape[1]
     B = P.shape[-2]
     xz = _slab_sum(P).to(state.dtype)
     cu = torch.arange(B + 1, dtype=torch.int32)
-    return causal_conv(xz[:, :C], w, bias, state, slots, cu, positions), xz[:, C:].contiguous()
+    y = causal_conv(xz[:, :C], w, bias, state, slots, cu, positions, silu)
+    return y, (xz[:, C:].contiguous() if xz.shape[1] > C else None)
 
 
 def selective_scan(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, cu, ctx):
