@@ -235,6 +235,25 @@ Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, 
   c10::DeviceGuard g(q.device());
   CHECK_ALIGN16(k_cache);     // cached rows are read in 16-byte pieces, q row by row
   auto out = at::empty({q.size(0), (int64_t)H * DV}, q.options());
+  if (!is_f32(q) && G == 1 && DV < D && !v_cache.has_value() && !k_scale.has_value() && docqa_latent_attn_ok(D, DV)) {
+    CHECK_ALIGN16(q);
+    const int64_t table = block_tables.size(1) * (int64_t)BS;
+    const int keys = (int)(window > 0 ? std::min<int64_t>(window + max_q - 1, table) : table);
+    const int ns = docqa_latent_splits(B, (int)max_q, H, DV, keys);
+    Tensor part, ml;
+    if (ns > 1) {
+      auto f32 = q.options().dtype(at::kFloat);
+      part = at::empty({ns, q.size(0), (int64_t)H * DV}, f32);
+      ml = at::empty({ns, q.size(0), H, 2}, f32);
+    }
+    CHECK_RC(docqa_latent_attn(q.data_ptr(), k_cache.data_ptr(), block_tables.data_ptr<int>(), (int)block_tables.size(1),
+                               cu.has_value() ? cu->data_ptr<int>() : nullptr, ctx.data_ptr<int>(),
+                               sink.has_value() ? sink->data_ptr<float>() : nullptr, out.data_ptr(),
+                               ns > 1 ? part.data_ptr<float>() : nullptr, ns > 1 ? ml.data_ptr() : nullptr, ns, B,
+                               (int)max_q, (int)q.size(0), H, D, DV, BS, (float)scale, (int)window, stream()),
+             "latent_attn");
+    return out;
+  }
   CHECK_RC(docqa_window_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.has_value() ? v_cache->data_ptr() : k_cache.data_ptr(),
                              k_scale.has_value() ? k_scale->data_ptr<float>() : nullptr, block_tables.data_ptr<int>(),
                              (int)block_tables.size(1), cu.has_value() ? cu->data_ptr<int>() : nullptr,

@@ -48,6 +48,13 @@ int docqa_latent_store(const void* P, int p_f32, int S, size_t slab, int ld, con
                        const float* c_norm, void* q, void* cache, int f32, int T, int H, int d, int r, int R, int BS,
                        float eps, hipStream_t s);
 int docqa_head_project(const void* x, const void* w, void* y, int T, int H, int K, int N, int E, hipStream_t s);
+// attention in the latent space, bf16, one KV head, values = the first DV elements of a row (sizes:
+// latent_attn_ok).  nsplit > 1 (latent_splits): part fp32 [nsplit, tokens H, DV], ml float2 [nsplit, tokens H]
+int docqa_latent_attn_ok(int D, int DV);
+int docqa_latent_splits(int B, int max_q, int H, int DV, int max_keys);
+int docqa_latent_attn(const void* q, const void* kc, const int* block_tables, int maxb, const int* cu, const int* ctx,
+                      const float* sink, void* out, float* part, void* ml, int nsplit, int B, int max_q, int tokens, int H,
+                      int D, int DV, int BS, float scale, int window, hipStream_t s);
 int docqa_latent_gather(const void* cache, const int* block_tables, int maxb, const int* first, const int* cu_k, void* c,
                         void* kr, int B, int max_keys, int R8, int r8, int BS, hipStream_t s);
 

@@ -229,6 +229,309 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(const uint16_t* __re
   else *reinterpret_cast<uint4*>(kr + dst * r8 + (e - R8)) = v;
 }
 
+// ------------------------------------------------------------------ attention, latent space
+typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
+constexpr int KB = 64;        // keys of a tile: 16 per wave of S^T
+constexpr int kMaxBT = 256;   // block ids staged in LDS (else read per tile)
+
+struct LatentArgs {
+  const uint16_t* q;      // [tokens, H, D]
+  const uint16_t* kc;     // paged rows [slots, D]
+  uint16_t* out;          // [tokens, H, DV]
+  const int* bt;
+  int maxb;
+  const int* cu;          // null: decode
+  const int* ctx;
+  const float* sink;
+  float* part;            // [nsplit, tokens H, DV] unnormalised outputs, null: one split
+  float2* ml;             // [nsplit, tokens H] (row maximum, row sum)
+  int tokens, H, D, DV, log2BS, nsplit, window;
+  float scale;
+};
+
+// grid (row tiles, sequences, key splits)
+template <int DPV, int DPK, int QT, int NW>
+__global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
+  constexpr int PITCH = DPK + 8, NCH = DPK / 8, NKS = DPK / 32, RW = 16 * QT, PP = KB + 8;
+  constexpr int CPT = (KB * NCH + 64 * NW - 1) / (64 * NW);
+  constexpr int QTW = QT / (NW / 4);           // row tiles whose scores this wave makes
+  constexpr int NDT = DPV / 16 / NW;           // 16-column tiles of its slice of the output
+  static_assert(NW % 4 == 0 && QTW >= 1 && NDT >= 1, "wave roles");
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  uint16_t* tiles = reinterpret_cast<uint16_t*>(smem);                  // [2][KB][PITCH]
+  uint16_t* sp = tiles + 2 * KB * PITCH;                                // [RW][PP]
+  float* smax = reinterpret_cast<float*>(sp + RW * PP);                 // [4][RW]
+  __shared__ int s_bt[kMaxBT];
+
+  const int b = blockIdx.y, split = blockIdx.z;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
+  int q0, L, p0;
+  if (a.cu) {
+    q0 = a.cu[b];
+    L = a.cu[b + 1] - q0;
+    p0 = a.ctx[b];
+  } else {
+    q0 = b;
+    L = 1;
+    p0 = a.ctx[b] - 1;
+  }
+  const int row0 = (gridDim.x - 1 - blockIdx.x) * RW, rows = L * a.H;   // longest windows first
+  if (row0 >= rows) return;
+  const size_t grow0 = (size_t)q0 * a.H;                                // first row of the sequence
+  const size_t all = (size_t)a.tokens * a.H;
+  const int nrow = min(RW, rows - row0);
+  if (p0 < 0) {                                                         // a padded decode row
+    if (a.nsplit == 1) {
+      for (int e = tid; e < nrow * a.DV; e += 64 * NW) a.out[(grow0 + row0) * a.DV + e] = 0;
+    } else {
+      for (int r = tid; r < nrow; r += 64 * NW) a.ml[split * all + grow0 + row0 + r] = make_float2(-1e30f, 0.f);
+    }
+    return;
+  }
+  const int pos_lo = p0 + row0 / a.H, pos_hi = p0 + (row0 + nrow - 1) / a.H;
+  const int key0 = a.window > 0 ? max(0, pos_lo - a.window + 1) : 0;
+  const int ntiles = (pos_hi - key0) / KB + 1, per = (ntiles + a.nsplit - 1) / a.nsplit;
+  const int t0 = split * per, t1 = min(ntiles, t0 + per);
+  if (t0 >= t1) {                                                       // more splits than tiles
+    for (int r = tid; r < nrow; r += 64 * NW) a.ml[split * all + grow0 + row0 + r] = make_float2(-1e30f, 0.f);
+    return;
+  }
+  const int first = key0 + t0 * KB, last = min(pos_hi, key0 + t1 * KB - 1);
+  const int blk0 = first >> a.log2BS, nblk = (last >> a.log2BS) - blk0 + 1;
+  const bool bt_lds = nblk <= kMaxBT;
+  if (bt_lds) {
+    for (int i = tid; i < nblk; i += 64 * NW) s_bt[i] = a.bt[(size_t)b * a.maxb + blk0 + i];
+    __syncthreads();
+  }
+
+  uint4 rk[CPT];
+  auto load = [&](int t) {
+    const int kb = key0 + t * KB;
+#pragma unroll
+    for (int i = 0; i < CPT; ++i) {
+      const int e = tid + 64 * NW * i, row = e / NCH, c = (e % NCH) * 8, key = kb + row;
+      rk[i] = make_uint4(0, 0, 0, 0);
+      if (e < KB * NCH && key <= last && c < a.D) {
+        const int kblk = key >> a.log2BS;
+        const int blk = bt_lds ? s_bt[kblk - blk0] : a.bt[(size_t)b * a.maxb + kblk];
+        rk[i] = *reinterpret_cast<const uint4*>(a.kc + (((size_t)blk << a.log2BS) + (key & ((1 << a.log2BS) - 1))) * a.D + c);
+      }
+    }
+  };
+  auto store = [&](int buf) {
+    uint16_t* k = tiles + buf * KB * PITCH;
+#pragma unroll
+    for (int i = 0; i < CPT; ++i) {
+      const int e = tid + 64 * NW * i, row = e / NCH, c = (e % NCH) * 8;
+      if (e < KB * NCH) *reinterpret_cast<uint4*>(k + row * PITCH + c) = rk[i];
+    }
+  };
+  load(t0);
+
+  const int ksub = wave & 3, rg = (wave >> 2) * QTW;     // this wave's keys of a tile / first row tile
+  bf16x8 qf[QTW][NKS];
+  int pos[QTW], below[QTW];                              // a row sees keys in (below, pos]
+#pragma unroll
+  for (int t = 0; t < QTW; ++t) {
+    const int r = min(row0 + (rg + t) * 16 + fr, rows - 1);
+    pos[t] = p0 + r / a.H;
+    below[t] = a.window > 0 ? pos[t] - a.window : -1;
+    const uint16_t* qp = a.q + (grow0 + r) * a.D;
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks) {
+      const int c = ks * 32 + g4 * 8;
+      uint4 v = c < a.D ? *reinterpret_cast<const uint4*>(qp + c) : make_uint4(0, 0, 0, 0);
+      qf[t][ks] = *reinterpret_cast<bf16x8*>(&v);
+    }
+  }
+  // the sink is the sum's first term: the maximum starts there in every wave, the sum in one
+  float m[QT], l[QTW];
+  f32x4 o[QT][NDT];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    const int r = min(row0 + t * 16 + fr, rows - 1);
+    m[t] = a.sink && split == 0 ? a.sink[r % a.H] * kLog2e : -1e30f;
+#pragma unroll
+    for (int i = 0; i < NDT; ++i) o[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+#pragma unroll
+  for (int t = 0; t < QTW; ++t) l[t] = a.sink && split == 0 && ksub == 0 && g4 == 0 ? 1.f : 0.f;
+  const float sl2 = a.scale * kLog2e;
+  const int tq = fr >> 2, tp = fr & 3;
+
+  store(0);
+  __syncthreads();
+  for (int t = t0; t < t1; ++t) {
+    const int buf = (t - t0) & 1, kb = key0 + t * KB;
+    if (t + 1 < t1) load(t + 1);
+    const uint16_t* sk = tiles + buf * KB * PITCH;
+    f32x4 x[QTW];
+#pragma unroll
+    for (int i = 0; i < QTW; ++i) x[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks) {
+      const bf16x8 kf = *reinterpret_cast<const bf16x8*>(sk + (ksub * 16 + fr) * PITCH + ks * 32 + g4 * 8);
+#pragma unroll
+      for (int i = 0; i < QTW; ++i) x[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][ks], x[i], 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < QTW; ++i) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = kb + ksub * 16 + g4 * 4 + r;
+        const float v = ((key <= pos[i]) & (key > below[i])) ? x[i][r] * sl2 : -INFINITY;
+        x[i][r] = v;
+        mx = fmaxf(mx, v);
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      if (g4 == 0) smax[ksub * RW + (rg + i) * 16 + fr] = mx;
+    }
+    __syncthreads();                                     // maxima; every wave is past the last tile
+    float alpha[QT];
+#pragma unroll
+    for (int i = 0; i < QT; ++i) {
+      float mn = m[i];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) mn = fmaxf(mn, smax[k * RW + i * 16 + fr]);
+      alpha[i] = __builtin_amdgcn_exp2f(m[i] - mn);
+      m[i] = mn;
+    }
+#pragma unroll
+    for (int i = 0; i < QTW; ++i) {
+      const float mn = NW == 4 ? m[i] : (rg == 0 ? m[i] : m[(QTW + i) % QT]);
+      const float al = NW == 4 ? alpha[i] : (rg == 0 ? alpha[i] : alpha[(QTW + i) % QT]);
+      float p[4], rs = 0.f;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        p[r] = __builtin_amdgcn_exp2f(x[i][r] - mn);
+        rs += p[r];
+      }
+      l[i] = l[i] * al + rs;
+      stv<4>(sp + ((rg + i) * 16 + fr) * PP + ksub * 16 + g4 * 4, p);
+    }
+    if (t + 1 < t1) store(buf ^ 1);
+    __syncthreads();                                     // scores, next tile
+#pragma unroll
+    for (int i = 0; i < QT; ++i)
+#pragma unroll
+      for (int n = 0; n < NDT; ++n)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[i][n][r] *= alpha[i];
+#pragma unroll
+    for (int s = 0; s < KB / 32; ++s) {
+      bf16x8 pb[QT];
+#pragma unroll
+      for (int i = 0; i < QT; ++i) {
+        const uint16_t* pr = sp + (i * 16 + fr) * PP + s * 32 + g4 * 4;
+        uint2 lo = *reinterpret_cast<const uint2*>(pr), hi = *reinterpret_cast<const uint2*>(pr + 16);
+        uint4 v = make_uint4(lo.x, lo.y, hi.x, hi.y);
+        pb[i] = *reinterpret_cast<bf16x8*>(&v);
+      }
+      const uint16_t* vr = sk + (s * 32 + g4 * 4 + tq) * PITCH + wave * NDT * 16 + 4 * tp;
+#pragma unroll
+      for (int n = 0; n < NDT; ++n) {
+        const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + n * 16));
+        const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_i16x4*)(vr + 16 * PITCH + n * 16));
+        bf16x8 vf;
+        const __bf16* lp = reinterpret_cast<const __bf16*>(&lo);
+        const __bf16* hp = reinterpret_cast<const __bf16*>(&hi);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { vf[j] = lp[j]; vf[4 + j] = hp[j]; }
+#pragma unroll
+        for (int i = 0; i < QT; ++i) o[i][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pb[i], o[i][n], 0, 0, 0);
+      }
+    }
+  }
+  // row sums: over a wave's key groups, then over the four key waves of the row
+#pragma unroll
+  for (int i = 0; i < QTW; ++i) {
+    l[i] += __shfl_xor(l[i], 16, 64);
+    l[i] += __shfl_xor(l[i], 32, 64);
+    if (g4 == 0) smax[ksub * RW + (rg + i) * 16 + fr] = l[i];
+  }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < QT; ++i) {
+    const int r = i * 16 + fr;
+    if (r >= nrow) continue;
+    const float sum = (smax[r] + smax[RW + r]) + (smax[2 * RW + r] + smax[3 * RW + r]);
+    const size_t row = grow0 + row0 + r;
+    const float inv = 1.f / sum;
+    if (a.nsplit > 1 && wave == 0 && g4 == 0) a.ml[split * all + row] = make_float2(m[i], sum);
+#pragma unroll
+    for (int n = 0; n < NDT; ++n) {
+      const int c = wave * NDT * 16 + n * 16 + g4 * 4;
+      if (c >= a.DV) continue;
+      if (a.nsplit > 1) {
+        *reinterpret_cast<float4*>(a.part + (split * all + row) * a.DV + c) =
+            make_float4(o[i][n][0], o[i][n][1], o[i][n][2], o[i][n][3]);
+      } else {
+        const float f[4] = {o[i][n][0] * inv, o[i][n][1] * inv, o[i][n][2] * inv, o[i][n][3] * inv};
+        stv<4>(a.out + row * a.DV + c, f);
+      }
+    }
+  }
+}
+
+// out [rows, DV] from the splits' partials: sum_s e^(m_s - m) part_s / sum_s e^(m_s - m) l_s
+__global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part, const float2* __restrict__ ml,
+                                                           int nsplit, size_t rows, int DV, uint16_t* __restrict__ out) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  const size_t row = i / (DV / 4);
+  if (row >= rows) return;
+  const int c = (int)(i - row * (DV / 4)) * 4;
+  float m = -1e30f, l = 0.f, f[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int s = 0; s < nsplit; ++s) m = fmaxf(m, ml[s * rows + row].x);
+  for (int s = 0; s < nsplit; ++s) {
+    const float2 v = ml[s * rows + row];
+    if (v.y <= 0.f) continue;                            // nothing seen: the partial was not written
+    const float w = __builtin_amdgcn_exp2f(v.x - m);
+    const float4 p = *reinterpret_cast<const float4*>(part + (s * rows + row) * DV + c);
+    l += w * v.y;
+    f[0] += w * p.x; f[1] += w * p.y; f[2] += w * p.z; f[3] += w * p.w;
+  }
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) f[j] *= inv;
+  stv<4>(out + row * DV + c, f);
+}
+
+template <int DPV, int QT, int NW>
+int launch_latent(const LatentArgs& a, int B, int max_q, hipStream_t s) {
+  constexpr int DPK = DPV + 64, RW = 16 * QT;
+  constexpr size_t lds = (size_t)2 * KB * (DPK + 8) * 2 + (size_t)RW * (KB + 8) * 2 + (size_t)4 * RW * 4;
+  static_assert(lds + kMaxBT * 4 <= 160 * 1024, "LDS");
+  const long long nz = ((long long)max_q * a.H + RW - 1) / RW;
+  if (nz >= (1ll << 31) || B > 65535) return -1;
+  auto kern = latent_attn_kernel<DPV, DPK, QT, NW>;
+  if constexpr (lds > 64 * 1024) {
+    static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
+                                                    hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return (int)e;
+  }
+  kern<<<dim3((unsigned)nz, B, a.nsplit), 64 * NW, lds, s>>>(a);
+  DOCQA_CHECK_LAUNCH();
+  if (a.nsplit > 1) {
+    const size_t rows = (size_t)a.tokens * a.H, n = rows * (a.DV / 4);
+    latent_merge_kernel<<<(unsigned)((n + 255) / 256), 256, 0, s>>>(a.part, a.ml, a.nsplit, rows, a.DV, a.out);
+    DOCQA_CHECK_LAUNCH();
+  }
+  return 0;
+}
+
+// row tiles of a workgroup by the rows a sequence has
+template <int DPV>
+int dispatch_latent(const LatentArgs& a, int B, int max_q, hipStream_t s) {
+  const long long rows = (long long)max_q * a.H;
+  constexpr int NW = DPV >= 128 ? 8 : 4;
+  if (rows <= 16) return launch_latent<DPV, 1, 4>(a, B, max_q, s);
+  if (DPV > 256 || rows <= 32) return launch_latent<DPV, 2, NW>(a, B, max_q, s);
+  if constexpr (DPV <= 256) return launch_latent<DPV, 4, NW>(a, B, max_q, s);
+  return -1;
+}
+
 template <typename PT, typename T>
 int store_types(const void* P, void* q, void* cache, int T_, const StoreArgs& a, hipStream_t s) {
   const bool v4 = a.d % 8 == 0 && a.r % 8 == 0 && a.R % 8 == 0 && a.ld % 4 == 0;
@@ -306,4 +609,32 @@ int docqa_latent_gather(const void* cache, const int* block_tables, int maxb, co
       (const uint16_t*)cache, block_tables, maxb, first, cu_k, (uint16_t*)c, (uint16_t*)kr, R8, r8, log2_of(BS));
   DOCQA_CHECK_LAUNCH();
   return 0;
+}
+
+int docqa_latent_attn_ok(int D, int DV) { return D % 8 == 0 && DV % 8 == 0 && DV <= 512 && D > DV && D <= (DV <= 64 ? 128 : DV <= 128 ? 192 : DV <= 256 ? 320 : 576); }
+
+// Key splits: enough workgroups for every CU, at least two tiles each
+int docqa_latent_splits(int B, int max_q, int H, int DV, int max_keys) {
+  const long long rows = (long long)max_q * H;
+  const int rw = rows <= 16 ? 16 : (DV > 256 || rows <= 32) ? 32 : 64;
+  const long long wgs = (long long)B * ((rows + rw - 1) / rw);
+  const int tiles = (max_keys + KB - 1) / KB + 1;
+  const long long n = wgs > 0 ? 256 / wgs : 1;
+  const int most = tiles / 2 < 16 ? tiles / 2 : 16;
+  return n < 1 || most < 1 ? 1 : (int)(n < most ? n : most);
+}
+
+int docqa_latent_attn(const void* q, const void* kc, const int* block_tables, int maxb, const int* cu, const int* ctx,
+                      const float* sink, void* out, float* part, void* ml, int nsplit, int B, int max_q, int tokens, int H,
+                      int D, int DV, int BS, float scale, int window, hipStream_t s) {
+  if (B == 0 || max_q == 0 || tokens == 0) return 0;
+  if (!docqa_latent_attn_ok(D, DV) || H < 1 || (BS & (BS - 1)) != 0 || nsplit < 1 || nsplit > 65535) return -1;
+  if (nsplit > 1 && (!part || !ml)) return -1;
+  if (!docqa_aligned16(q) || !docqa_aligned16(kc) || !docqa_aligned16(out)) return -1;
+  const LatentArgs a{(const uint16_t*)q, (const uint16_t*)kc, (uint16_t*)out, block_tables, maxb, cu, ctx, sink, part,
+                     (float2*)ml, tokens, H, D, DV, log2_of(BS), nsplit, window, scale};
+  if (DV <= 64) return dispatch_latent<64>(a, B, max_q, s);
+  if (DV <= 128) return dispatch_latent<128>(a, B, max_q, s);
+  if (DV <= 256) return dispatch_latent<256>(a, B, max_q, s);
+  return dispatch_latent<512>(a, B, max_q, s);
 }

@@ -423,9 +423,8 @@ class InputConv:
     last tap."""
 
     def __init__(self, w):
-        w = w.float().t().contiguous()                              # [taps, W]
-        w[-1] += 1.0
-        self.w = w
+        self.w = w.float().t().clone(memory_format=torch.contiguous_format)      # [taps, W]
+        self.w[-1] += 1.0
 
     def cache_spec(self):
         return StateSpec((((self.w.shape[0] - 1), self.w.shape[1]),), (False,))
