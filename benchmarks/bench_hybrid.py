@@ -49,12 +49,17 @@ def _engine(model, batch: int, context: int):
                      max_prefill_tokens=1 << 20)
 
 
-def bench_model(kind: str, size: str, warmup: int, steps: int) -> list[dict]:
-    from docqa_amd.engine.llm_engine import SamplingParams
+def build_model(kind: str, size: str):
     from docqa_amd.models.hybrid import HybridModel
     from docqa_amd.models.llama import LlamaModel
 
-    model = (HybridModel(hybrid_config(size)) if kind == "saritar" else LlamaModel(llama_config(size)))
+    return HybridModel(hybrid_config(size)) if kind == "saritar" else LlamaModel(llama_config(size))
+
+
+def bench_model(kind: str, size: str, warmup: int, steps: int, build=build_model) -> list[dict]:
+    from docqa_amd.engine.llm_engine import SamplingParams
+
+    model = build(kind, size)
     params = model.cfg.num_params()
     rows = []
     g = torch.Generator().manual_seed(1)
@@ -256,7 +261,11 @@ def bench_kernels(size: str) -> list[dict]:
             (lambda i: ops.mgemm_glu(xx, ws[i % nc], cfg[1])) if cfg[0] else (lambda i: ops.glu_linear(xx, ws[i % nc])))
         row("glu", "decode", B, glu, 2.0 * F * W * 2, 4.0 * B * F * W)
         del ws
-    # distance from the bound beside the like kernel's
+    return beside_like(out)
+
+
+def beside_like(out: list[dict]) -> list[dict]:
+    """Each kernel's distance from its bound over that of the like kernel (``vs_like``)."""
     at = {(r["kernel"], r["phase"], r["rows"]): r["times_bound"] for r in out}
     for r in out:
         like = at.get((r["like"], r["phase"], r["rows"]))
@@ -265,7 +274,8 @@ def bench_kernels(size: str) -> list[dict]:
     return out
 
 
-def main(args) -> None:
+def main(args, name: str = "saritar", build=build_model, kernels=bench_kernels) -> None:
+    """Every row of design ``name`` and of the Llama beside it, as JSON lines."""
     from docqa_amd import ops
 
     assert ops.load_native(), ops.native_error()
@@ -274,15 +284,15 @@ def main(args) -> None:
     for size in args.arch_sizes.split(","):
         if args.arch_part in ("all", "models"):
             rows = []
-            for kind in ("saritar", "llama"):
-                for r in bench_model(kind, size, args.warmup, args.steps):
+            for kind in (name, "llama"):
+                for r in bench_model(kind, size, args.warmup, args.steps, build):
                     rows.append(r)
                     print(json.dumps(r), flush=True)
             half = len(rows) // 2
             for a, b in zip(rows[:half], rows[half:]):
                 print(json.dumps({"size": size, "phase": a["phase"], "batch": a["batch"], "tokens": a.get("tokens", a["batch"]),
-                                  "saritar_over_llama": round(a["tokens_per_s"] / b["tokens_per_s"], 2)}), flush=True)
+                                  f"{name}_over_llama": round(a["tokens_per_s"] / b["tokens_per_s"], 2)}), flush=True)
         if args.arch_part in ("all", "kernels"):
-            for r in bench_kernels(size):
+            for r in kernels(size):
                 print(json.dumps(r), flush=True)
     print(json.dumps({"seconds": round(time.time() - t0, 1)}), flush=True)

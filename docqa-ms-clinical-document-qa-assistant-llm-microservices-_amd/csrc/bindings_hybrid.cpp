@@ -162,14 +162,16 @@ Tensor slab_activation(const Tensor& P, int64_t act, bool out_f32) {
   return out;
 }
 
-// act(x . w^T) on the decode GEMMs: skinny up to 192 rows, the mid-M kernel beyond
+// act(x . w^T) on the decode GEMMs: the GEMV for one row, skinny up to 192, the mid-M kernel beyond
 Tensor decode_act(const Tensor& x, const Tensor& w, int64_t act) {
   CHECK_GPU(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_CONTIG(x); CHECK_CONTIG(w); CHECK_ALIGN16(x); CHECK_ALIGN16(w);
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1), "decode_act: shapes");
   const int M = x.size(0), N = w.size(0), K = x.size(1);
   c10::DeviceGuard g(x.device());
   auto out = at::empty({M, N}, x.options());
-  CHECK_RC(M <= 192 && N % 64 == 0 && K % 512 == 0
+  CHECK_RC(M == 1 && N % 8 == 0 && (K == 2048 || K == 4096)
+               ? docqa_gemv_act(x.data_ptr(), w.data_ptr(), out.data_ptr(), (int)act, N, K, stream())
+           : M <= 192 && N % 64 == 0 && K % 512 == 0
                ? docqa_dgemm_act(x.data_ptr(), w.data_ptr(), out.data_ptr(), (int)act, M, N, K, stream())
                : docqa_mgemm_act(x.data_ptr(), w.data_ptr(), out.data_ptr(), (int)act, M, N, K, stream()),
            "decode_act");
@@ -235,25 +237,6 @@ Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, 
   c10::DeviceGuard g(q.device());
   CHECK_ALIGN16(k_cache);     // cached rows are read in 16-byte pieces, q row by row
   auto out = at::empty({q.size(0), (int64_t)H * DV}, q.options());
-  if (!is_f32(q) && G == 1 && DV < D && !v_cache.has_value() && !k_scale.has_value() && docqa_latent_attn_ok(D, DV)) {
-    CHECK_ALIGN16(q);
-    const int64_t table = block_tables.size(1) * (int64_t)BS;
-    const int keys = (int)(window > 0 ? std::min<int64_t>(window + max_q - 1, table) : table);
-    const int ns = docqa_latent_splits(B, (int)max_q, H, DV, keys);
-    Tensor part, ml;
-    if (ns > 1) {
-      auto f32 = q.options().dtype(at::kFloat);
-      part = at::empty({ns, q.size(0), (int64_t)H * DV}, f32);
-      ml = at::empty({ns, q.size(0), H, 2}, f32);
-    }
-    CHECK_RC(docqa_latent_attn(q.data_ptr(), k_cache.data_ptr(), block_tables.data_ptr<int>(), (int)block_tables.size(1),
-                               cu.has_value() ? cu->data_ptr<int>() : nullptr, ctx.data_ptr<int>(),
-                               sink.has_value() ? sink->data_ptr<float>() : nullptr, out.data_ptr(),
-                               ns > 1 ? part.data_ptr<float>() : nullptr, ns > 1 ? ml.data_ptr() : nullptr, ns, B,
-                               (int)max_q, (int)q.size(0), H, D, DV, BS, (float)scale, (int)window, stream()),
-             "latent_attn");
-    return out;
-  }
   CHECK_RC(docqa_window_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.has_value() ? v_cache->data_ptr() : k_cache.data_ptr(),
                              k_scale.has_value() ? k_scale->data_ptr<float>() : nullptr, block_tables.data_ptr<int>(),
                              (int)block_tables.size(1), cu.has_value() ? cu->data_ptr<int>() : nullptr,
@@ -262,6 +245,44 @@ Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, 
                              stream()),
            "window_attn");
   return out;
+}
+
+// window_attn in the latent space (one KV head, values = the first K elements of a cached row, K =
+// w.size(2)) followed by head_project with w [H, N, K]; bf16, sizes by docqa_latent_attn_ok
+Tensor latent_attn(const Tensor& q, const Tensor& cache, const Tensor& block_tables, const OptT& cu, const Tensor& ctx,
+                   int64_t max_q, double scale, int64_t window, const OptT& sink, const Tensor& w) {
+  CHECK_GPU(q); CHECK_BF16(q); CHECK_CONTIG(q); CHECK_GPU(cache); CHECK_BF16(cache); CHECK_CONTIG(cache);
+  CHECK_GPU(w); CHECK_BF16(w); CHECK_CONTIG(w);
+  TORCH_CHECK(cache.dim() == 4 && cache.size(1) == 1 && w.dim() == 3, "latent_attn: cache [blocks, 1, block, D], w [H, N, K]");
+  const int BS = cache.size(2), D = cache.size(3), H = w.size(0), N = w.size(1), DV = w.size(2);
+  TORCH_CHECK(q.dim() == 2 && q.size(1) == (int64_t)H * D && docqa_latent_attn_ok(D, DV), "latent_attn: sizes");
+  const int T = q.size(0), B = block_tables.size(0);
+  CHECK_GPU(block_tables); CHECK_I32(block_tables); CHECK_CONTIG(block_tables);
+  TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(1) >= 1, "block_tables must be [B, blocks]");
+  check_i32(ctx, B, "ctx");
+  if (cu.has_value()) check_i32(*cu, B + 1, "cu");
+  else TORCH_CHECK(T == B && max_q == 1, "decode: one query row a sequence");
+  TORCH_CHECK(cache.numel() / D < (1ll << 31), "cache rows must fit 31 bits");
+  if (sink.has_value()) check_vec(*sink, H, "sink");
+  CHECK_ALIGN16(cache); CHECK_ALIGN16(q); CHECK_ALIGN16(w);
+  c10::DeviceGuard g(q.device());
+  const int64_t table = block_tables.size(1) * (int64_t)BS;
+  const int keys = (int)(window > 0 ? std::min<int64_t>(window + max_q - 1, table) : table);
+  const int ns = docqa_latent_splits(B, (int)max_q, H, DV, keys);
+  auto f32 = q.options().dtype(at::kFloat);
+  auto x = at::empty({ns > 1 ? 0 : T, (int64_t)H * DV}, q.options());
+  auto part = at::empty({ns > 1 ? ns : 0, T, (int64_t)H * DV}, q.options()), ml = at::empty({ns > 1 ? ns : 0, T, H, 2}, f32);
+  void* pp = ns > 1 ? part.data_ptr() : nullptr;
+  void* mp = ns > 1 ? ml.data_ptr() : nullptr;
+  CHECK_RC(docqa_latent_attn(q.data_ptr(), cache.data_ptr(), block_tables.data_ptr<int>(), (int)block_tables.size(1),
+                             cu.has_value() ? cu->data_ptr<int>() : nullptr, ctx.data_ptr<int>(),
+                             sink.has_value() ? sink->data_ptr<float>() : nullptr, x.data_ptr(), pp, mp, ns, B,
+                             (int)max_q, T, H, D, DV, BS, (float)scale, (int)window, stream()),
+           "latent_attn");
+  auto y = at::empty({T, (int64_t)H * N}, q.options());
+  CHECK_RC(docqa_head_project(x.data_ptr(), pp, mp, ns, w.data_ptr(), y.data_ptr(), T, H, DV, N, 0, stream()),
+           "latent_attn values");
+  return y;
 }
 
 Tensor packed_window_attn(const Tensor& q, const Tensor& kv, const Tensor& kr, int64_t H, int64_t dim, int64_t vdim,
@@ -327,7 +348,7 @@ Tensor head_project(const Tensor& x, const Tensor& w, int64_t carry) {
   TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && carry >= 0 && x.size(1) == w.size(0) * (w.size(2) + carry), "head_project: shapes");
   c10::DeviceGuard g(x.device());
   auto y = at::empty({x.size(0), w.size(0) * (w.size(1) + carry)}, x.options());
-  CHECK_RC(docqa_head_project(x.data_ptr(), w.data_ptr(), y.data_ptr(), (int)x.size(0), (int)w.size(0), (int)w.size(2),
+  CHECK_RC(docqa_head_project(x.data_ptr(), nullptr, nullptr, 1, w.data_ptr(), y.data_ptr(), (int)x.size(0), (int)w.size(0), (int)w.size(2),
                               (int)w.size(1), (int)carry, stream()),
            "head_project");
   return y;
@@ -378,6 +399,30 @@ Tensor causal_conv(const Tensor& x, const Tensor& w, const OptT& bias, Tensor st
                              y.data_ptr(), is_f32(x), B, (int)max_len, C, taps, silu, stream()),
            "causal_conv");
   return y;
+}
+
+// sandwich_rmsnorm of one token a row and its input convolution: (h, h + conv(h)) in the state's dtype
+std::tuple<Tensor, Tensor> sandwich_rmsnorm_conv(const Tensor& P, Tensor residual, const Tensor& w_post,
+                                                 const Tensor& w_next, const Tensor& cw, Tensor state,
+                                                 const Tensor& slots, const Tensor& positions, double eps) {
+  const Slabs p = slabs_of(P);
+  CHECK_GPU(residual); CHECK_F32(residual); CHECK_CONTIG(residual);
+  TORCH_CHECK(residual.dim() == 2 && residual.size(0) == p.M && residual.size(1) == p.N, "residual shape mismatch");
+  check_vec(w_post, p.N, "w_post");
+  check_vec(w_next, p.N, "w_next");
+  int taps;
+  check_conv(cw, c10::nullopt, state, p.N, taps);
+  CHECK_ACT(state);
+  check_i32(slots, p.M, "slots"); check_i32(positions, p.M, "positions");
+  CHECK_ALIGN16(P); CHECK_ALIGN16(residual); CHECK_ALIGN16(w_post); CHECK_ALIGN16(w_next); CHECK_ALIGN16(cw); CHECK_ALIGN16(state);
+  c10::DeviceGuard g(P.device());
+  auto h = at::empty({p.M, p.N}, state.options()), hc = at::empty({p.M, p.N}, state.options());
+  CHECK_RC(docqa_sandwich_rmsnorm_conv(P.data_ptr(), is_f32(P), p.S, residual.data_ptr<float>(), w_post.data_ptr<float>(),
+                                       w_next.data_ptr<float>(), cw.data_ptr<float>(), taps, state.data_ptr(),
+                                       slots.data_ptr<int>(), positions.data_ptr<int>(), h.data_ptr(), hc.data_ptr(),
+                                       is_f32(state), p.M, p.N, (float)eps, stream()),
+           "sandwich_rmsnorm_conv");
+  return {h, hc};
 }
 
 // P: [x: C | z: C] input projection of one token a row -> (conv x, z); [x: C] -> (conv x, empty)
@@ -488,6 +533,10 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
   m.def("soft_cap(Tensor x, float cap) -> Tensor");
   m.def("side_gate(Tensor P, Tensor ids, Tensor table, int col, int n, bool out_f32) -> Tensor");
   m.def("side_project(Tensor P, Tensor ids, Tensor table, int col, int n, Tensor w) -> Tensor");
+  m.def("latent_attn(Tensor q, Tensor cache, Tensor block_tables, Tensor? cu, Tensor ctx, int max_q, float scale, "
+        "int window, Tensor? sink, Tensor w) -> Tensor");
+  m.def("sandwich_rmsnorm_conv(Tensor P, Tensor(a!) residual, Tensor w_post, Tensor w_next, Tensor cw, "
+        "Tensor(b!) state, Tensor slots, Tensor positions, float eps) -> (Tensor, Tensor)");
   m.def("packed_window_attn(Tensor q, Tensor kv, Tensor kr, int H, int dim, int vdim, Tensor cu, Tensor cu_k, int max_q, "
         "float scale, int window, Tensor? sink) -> Tensor");
   m.def("rope_table(Tensor positions, Tensor freq) -> Tensor");
@@ -520,6 +569,8 @@ TORCH_LIBRARY_IMPL(docqa, CUDA, m) {
   m.impl("soft_cap", &soft_cap);
   m.impl("side_gate", &side_gate);
   m.impl("side_project", &side_project);
+  m.impl("latent_attn", &latent_attn);
+  m.impl("sandwich_rmsnorm_conv", &sandwich_rmsnorm_conv);
   m.impl("packed_window_attn", &packed_window_attn);
   m.impl("rope_table", &rope_table);
   m.impl("latent_store", &latent_store);

@@ -13,11 +13,17 @@ int docqa_sandwich_rmsnorm(const void* P, int p_f32, int S, float* res, const fl
                            const float* w_next, void* out, int out_f32, int rows, int H, float eps, hipStream_t s);
 int docqa_embed_scale_rmsnorm(const int* ids, const void* table, int f32, float scale, const float* w, float* res,
                               float* emb, void* out, int rows, int H, int vocab, float eps, hipStream_t s);
+// sandwich_rmsnorm of one token a row, and h + conv(h): w [taps, H] with the identity in its last tap,
+// state [slots, taps - 1, H] of out's type; out2 [rows, H]
+int docqa_sandwich_rmsnorm_conv(const void* P, int p_f32, int S, float* res, const float* w_post, const float* w_next,
+                                const float* cw, int taps, void* state, const int* slots, const int* positions, void* out,
+                                void* out2, int out_f32, int rows, int H, float eps, hipStream_t s);
 // res [n] += m (P + Q) (Q null: P alone), each with its own slab count; out null or bf16 [n]: a copy of res
 int docqa_add_scaled(const void* P, int p_f32, int SP, const void* Q, int q_f32, int SQ, float* res, float m, void* out,
                      size_t n, hipStream_t s);
 // Y [M, N] = act(X [M, K] . W [N, K]^T), bf16, act: docqa_common.h ACT_* (dgemm.hip: M <= 192, N % 64,
 // K % 512; mgemm.hip: N % 128, K % 128)
+int docqa_gemv_act(const void* X, const void* W, void* Y, int act, int N, int K, hipStream_t s);   // M = 1
 int docqa_dgemm_act(const void* X, const void* W, void* Y, int act, int M, int N, int K, hipStream_t s);
 int docqa_mgemm_act(const void* X, const void* W, void* Y, int act, int M, int N, int K, hipStream_t s);
 int docqa_slab_columns(const void* P, int p_f32, int S, int T, int ld, void* out0, int n0, void* out1, int n1,
@@ -47,13 +53,16 @@ int docqa_rope_table(const int* positions, const double* freq, float* out, int T
 int docqa_latent_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* cs, const int* slots,
                        const float* c_norm, void* q, void* cache, int f32, int T, int H, int d, int r, int R, int BS,
                        float eps, hipStream_t s);
-int docqa_head_project(const void* x, const void* w, void* y, int T, int H, int K, int N, int E, hipStream_t s);
+// part null: rows x; else the rows are docqa_latent_attn's nsplit partials (E = 0)
+int docqa_head_project(const void* x, const void* part, const void* ml, int nsplit, const void* w, void* y, int T, int H,
+                       int K, int N, int E, hipStream_t s);
 // attention in the latent space, bf16, one KV head, values = the first DV elements of a row (sizes:
-// latent_attn_ok).  nsplit > 1 (latent_splits): part fp32 [nsplit, tokens H, DV], ml float2 [nsplit, tokens H]
+// latent_attn_ok).  nsplit > 1 (latent_splits): partials for docqa_head_project instead of out -- part
+// bf16 [nsplit, tokens H, DV] each split's output, ml float2 [nsplit, tokens H] (maximum, sum)
 int docqa_latent_attn_ok(int D, int DV);
 int docqa_latent_splits(int B, int max_q, int H, int DV, int max_keys);
 int docqa_latent_attn(const void* q, const void* kc, const int* block_tables, int maxb, const int* cu, const int* ctx,
-                      const float* sink, void* out, float* part, void* ml, int nsplit, int B, int max_q, int tokens, int H,
+                      const float* sink, void* out, void* part, void* ml, int nsplit, int B, int max_q, int tokens, int H,
                       int D, int DV, int BS, float scale, int window, hipStream_t s);
 int docqa_latent_gather(const void* cache, const int* block_tables, int maxb, const int* first, const int* cu_k, void* c,
                         void* kr, int B, int max_keys, int R8, int r8, int BS, hipStream_t s);

@@ -18,7 +18,7 @@
 // bf16 scores through LDS, and take a slice of the latent's columns each for O^T += V^T P^T (V^T by
 // transposing LDS reads of the same tile).  So a tile is read twice per workgroup however many rows
 // it serves, and a wave's accumulators are a slice of a row, not the 512-wide row itself.  Few
-// sequences: the keys are split over workgroups (partials in fp32, merged by latent_merge).
+// sequences: the keys are split over workgroups; the value projection sums the splits' outputs.
 #include "docqa_common.h"
 #include "docqa_elem.h"
 #include "docqa_hybrid.h"
@@ -34,6 +34,10 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
   __syncthreads();
   return red[0] + red[1] + red[2] + red[3];
 }
+
+// LDS-only workgroup barrier: __syncthreads() also drains the global loads in flight, and the
+// next tiles' are meant to stay there
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
 __global__ __launch_bounds__(256) void rope_table_kernel(const int* __restrict__ pos, const double* __restrict__ freq,
                                                          float* __restrict__ out, int T, int half) {
@@ -135,23 +139,65 @@ __global__ __launch_bounds__(256) void latent_store_kernel(const PT* __restrict_
 
 // ------------------------------------------------------------------ per-head products
 // y[t, h, :N] = x[t, h, :K] . w[h]^T; y[t, h, N : N + E] = x[t, h, K : K + E].  One workgroup:
-// 16 MT rows of one head, 128 outputs; x rows staged in LDS, w straight to registers.
-template <int MT>
+// 16 MT rows of one head, 64 NJ outputs; x rows staged in LDS, w straight to registers.  MERGE: the
+// rows are attended latents as key splits' outputs, x = sum_s w_s part_s, w_s = e^(m_s - m) l_s / sum.
+constexpr int kMaxSplit = 32;
+
+template <int MT, int NJ, bool MERGE>
 __global__ __launch_bounds__(256) void head_project_kernel(const uint16_t* __restrict__ x,
+                                                           const uint16_t* __restrict__ part,
+                                                           const float2* __restrict__ ml, int nsplit,
                                                            const uint16_t* __restrict__ w, uint16_t* __restrict__ y,
                                                            int T, int H, int K, int N, int E) {
   extern __shared__ __attribute__((aligned(16))) uint16_t sx[];       // [16 MT][pitch]
+  __shared__ float sw[MERGE ? 16 * MT : 1][kMaxSplit];                // a row's weight of each split
   const int kp = (K + 31) / 32 * 32, pitch = kp + 8;
   const int h = blockIdx.x, m0 = blockIdx.y * 16 * MT, tid = threadIdx.x;
   const int ldx = H * (K + E), ldy = H * (N + E);
   const uint16_t* xh = x + (size_t)h * (K + E);
   uint16_t* yh = y + (size_t)h * (N + E);
   const int per = kp / 8;
-  for (int i = tid; i < 16 * MT * per; i += 256) {
-    const int r = i / per, c = (i - r * per) * 8;
-    uint4 v = make_uint4(0, 0, 0, 0);
-    if (m0 + r < T && c < K) v = *reinterpret_cast<const uint4*>(xh + (size_t)(m0 + r) * ldx + c);
-    *reinterpret_cast<uint4*>(sx + r * pitch + c) = v;
+  if constexpr (MERGE) {
+    const size_t all = (size_t)T * H;
+    for (int i = tid; i < 16 * MT; i += 256) {
+      const size_t row = (size_t)min(m0 + i, T - 1) * H + h;
+      float m = -1e30f, l = 0.f;
+#pragma unroll 8
+      for (int s = 0; s < nsplit; ++s) m = fmaxf(m, ml[s * all + row].x);
+#pragma unroll 8
+      for (int s = 0; s < nsplit; ++s) {
+        const float2 v = ml[s * all + row];
+        const float e = v.y > 0.f ? __builtin_amdgcn_exp2f(v.x - m) * v.y : 0.f;     // 0: nothing seen, nothing written
+        sw[i][s] = e;
+        l += e;
+      }
+      const float inv = l > 0.f ? 1.f / l : 0.f;
+      for (int s = 0; s < nsplit; ++s) sw[i][s] *= inv;
+    }
+    __syncthreads();
+    for (int i = tid; i < 16 * MT * per; i += 256) {
+      const int r = i / per, c = (i - r * per) * 8;
+      float f[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (m0 + r < T && c < K) {
+        const uint16_t* p = part + ((size_t)(m0 + r) * H + h) * K + c;
+#pragma unroll 4
+        for (int s = 0; s < nsplit; ++s) {
+          const float e = sw[r][s];
+          float g[8];
+          ldv<8>(p + s * all * K, g);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) f[j] += e > 0.f ? e * g[j] : 0.f;        // (not written: any bits)
+        }
+      }
+      stv<8>(sx + r * pitch + c, f);
+    }
+  } else {
+    for (int i = tid; i < 16 * MT * per; i += 256) {
+      const int r = i / per, c = (i - r * per) * 8;
+      uint4 v = make_uint4(0, 0, 0, 0);
+      if (m0 + r < T && c < K) v = *reinterpret_cast<const uint4*>(xh + (size_t)(m0 + r) * ldx + c);
+      *reinterpret_cast<uint4*>(sx + r * pitch + c) = v;
+    }
   }
   if (blockIdx.z == 0 && E > 0) {
     const int pe = E / 8;
@@ -164,20 +210,20 @@ __global__ __launch_bounds__(256) void head_project_kernel(const uint16_t* __res
   }
   __syncthreads();
   const int lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
-  const int n0 = blockIdx.z * 128 + wave * 32;                        // this wave's outputs n0 .. n0 + 31
+  const int n0 = (blockIdx.z * 4 + wave) * 16 * NJ;                   // this wave's first output
   if (n0 >= N) return;
-  f32x4 acc[MT][2];
+  f32x4 acc[MT][NJ];
 #pragma unroll
   for (int i = 0; i < MT; ++i)
 #pragma unroll
-    for (int j = 0; j < 2; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int j = 0; j < NJ; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   const uint16_t* wh = w + (size_t)h * N * K;
-#pragma unroll 4
+#pragma unroll 8
   for (int k = 0; k < kp; k += 32) {
     const int kk = k + g4 * 8;
-    bf16x8 wf[2], xf[MT];
+    bf16x8 wf[NJ], xf[MT];
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
+    for (int j = 0; j < NJ; ++j) {
       const int n = n0 + 16 * j + fr;
       uint4 v = make_uint4(0, 0, 0, 0);
       if (n < N && kk < K) v = *reinterpret_cast<const uint4*>(wh + (size_t)n * K + kk);
@@ -188,14 +234,14 @@ __global__ __launch_bounds__(256) void head_project_kernel(const uint16_t* __res
 #pragma unroll
     for (int i = 0; i < MT; ++i)
 #pragma unroll
-      for (int j = 0; j < 2; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[j], xf[i], acc[i][j], 0, 0, 0);
+      for (int j = 0; j < NJ; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[j], xf[i], acc[i][j], 0, 0, 0);
   }
 #pragma unroll
   for (int i = 0; i < MT; ++i) {
     const int row = m0 + i * 16 + fr;
     if (row >= T) continue;
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
+    for (int j = 0; j < NJ; ++j) {
       const int n = n0 + 16 * j + g4 * 4;
       uint16_t* op = yh + (size_t)row * ldy + n;
       if (N % 4 == 0) {
@@ -232,7 +278,7 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(const uint16_t* __re
 // ------------------------------------------------------------------ attention, latent space
 typedef __attribute__((address_space(3))) i16x4 lds_i16x4;
 constexpr int KB = 64;        // keys of a tile: 16 per wave of S^T
-constexpr int kMaxBT = 256;   // block ids staged in LDS (else read per tile)
+constexpr int kMaxBT = 256;   // block ids staged in LDS at a time
 
 struct LatentArgs {
   const uint16_t* q;      // [tokens, H, D]
@@ -243,7 +289,7 @@ struct LatentArgs {
   const int* cu;          // null: decode
   const int* ctx;
   const float* sink;
-  float* part;            // [nsplit, tokens H, DV] unnormalised outputs, null: one split
+  uint16_t* part;         // [nsplit, tokens H, DV] each split's output, null: one split
   float2* ml;             // [nsplit, tokens H] (row maximum, row sum)
   int tokens, H, D, DV, log2BS, nsplit, window;
   float scale;
@@ -253,10 +299,10 @@ struct LatentArgs {
 template <int DPV, int DPK, int QT, int NW>
 __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
   constexpr int PITCH = DPK + 8, NCH = DPK / 8, NKS = DPK / 32, RW = 16 * QT, PP = KB + 8;
-  constexpr int CPT = (KB * NCH + 64 * NW - 1) / (64 * NW);
+  constexpr int CPT = NCH / NW;                // 16-byte pieces of a tile a thread stages
   constexpr int QTW = QT / (NW / 4);           // row tiles whose scores this wave makes
   constexpr int NDT = DPV / 16 / NW;           // 16-column tiles of its slice of the output
-  static_assert(NW % 4 == 0 && QTW >= 1 && NDT >= 1, "wave roles");
+  static_assert(NW % 4 == 0 && QTW >= 1 && NDT >= 1 && NCH % NW == 0, "wave roles");
   extern __shared__ __attribute__((aligned(16))) char smem[];
   uint16_t* tiles = reinterpret_cast<uint16_t*>(smem);                  // [2][KB][PITCH]
   uint16_t* sp = tiles + 2 * KB * PITCH;                                // [RW][PP]
@@ -296,26 +342,31 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
     for (int r = tid; r < nrow; r += 64 * NW) a.ml[split * all + grow0 + row0 + r] = make_float2(-1e30f, 0.f);
     return;
   }
-  const int first = key0 + t0 * KB, last = min(pos_hi, key0 + t1 * KB - 1);
-  const int blk0 = first >> a.log2BS, nblk = (last >> a.log2BS) - blk0 + 1;
-  const bool bt_lds = nblk <= kMaxBT;
-  if (bt_lds) {
-    for (int i = tid; i < nblk; i += 64 * NW) s_bt[i] = a.bt[(size_t)b * a.maxb + blk0 + i];
+  const int last = min(pos_hi, key0 + t1 * KB - 1);
+  int blk0 = (key0 + t0 * KB) >> a.log2BS;               // first staged block id
+  auto stage_blocks = [&]() {
+    const int n = min(kMaxBT, (last >> a.log2BS) - blk0 + 1);
+    for (int i = tid; i < n; i += 64 * NW) s_bt[i] = a.bt[(size_t)b * a.maxb + blk0 + i];
     __syncthreads();
-  }
+  };
+  stage_blocks();
 
-  uint4 rk[CPT];
+  // Every load of a tile issues without a branch: keys past the end repeat the last one (their
+  // scores are masked), columns past the row repeat its first (the query is zero there, the
+  // output is dropped).
+  u32x4 rk[CPT];
   auto load = [&](int t) {
     const int kb = key0 + t * KB;
+    if ((min(kb + KB - 1, last) >> a.log2BS) - blk0 >= kMaxBT) {       // the whole workgroup
+      lds_barrier();
+      blk0 = kb >> a.log2BS;
+      stage_blocks();
+    }
 #pragma unroll
     for (int i = 0; i < CPT; ++i) {
-      const int e = tid + 64 * NW * i, row = e / NCH, c = (e % NCH) * 8, key = kb + row;
-      rk[i] = make_uint4(0, 0, 0, 0);
-      if (e < KB * NCH && key <= last && c < a.D) {
-        const int kblk = key >> a.log2BS;
-        const int blk = bt_lds ? s_bt[kblk - blk0] : a.bt[(size_t)b * a.maxb + kblk];
-        rk[i] = *reinterpret_cast<const uint4*>(a.kc + (((size_t)blk << a.log2BS) + (key & ((1 << a.log2BS) - 1))) * a.D + c);
-      }
+      const int e = tid + 64 * NW * i, c0 = (e % NCH) * 8, c = c0 < a.D ? c0 : 0, key = min(kb + e / NCH, last);
+      const int blk = s_bt[(key >> a.log2BS) - blk0];
+      rk[i] = *reinterpret_cast<const u32x4*>(a.kc + (((size_t)blk << a.log2BS) + (key & ((1 << a.log2BS) - 1))) * a.D + c);
     }
   };
   auto store = [&](int buf) {
@@ -323,7 +374,7 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
 #pragma unroll
     for (int i = 0; i < CPT; ++i) {
       const int e = tid + 64 * NW * i, row = e / NCH, c = (e % NCH) * 8;
-      if (e < KB * NCH) *reinterpret_cast<uint4*>(k + row * PITCH + c) = rk[i];
+      *reinterpret_cast<u32x4*>(k + row * PITCH + c) = rk[i];
     }
   };
   load(t0);
@@ -340,7 +391,8 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
 #pragma unroll
     for (int ks = 0; ks < NKS; ++ks) {
       const int c = ks * 32 + g4 * 8;
-      uint4 v = c < a.D ? *reinterpret_cast<const uint4*>(qp + c) : make_uint4(0, 0, 0, 0);
+      uint4 v = *reinterpret_cast<const uint4*>(qp + (c < a.D ? c : 0));
+      if (c >= a.D) v = make_uint4(0, 0, 0, 0);
       qf[t][ks] = *reinterpret_cast<bf16x8*>(&v);
     }
   }
@@ -360,10 +412,10 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
   const int tq = fr >> 2, tp = fr & 3;
 
   store(0);
-  __syncthreads();
+  load(min(t0 + 1, t1 - 1));                             // in flight for a whole tile's work
+  lds_barrier();
   for (int t = t0; t < t1; ++t) {
     const int buf = (t - t0) & 1, kb = key0 + t * KB;
-    if (t + 1 < t1) load(t + 1);
     const uint16_t* sk = tiles + buf * KB * PITCH;
     f32x4 x[QTW];
 #pragma unroll
@@ -388,7 +440,7 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
       if (g4 == 0) smax[ksub * RW + (rg + i) * 16 + fr] = mx;
     }
-    __syncthreads();                                     // maxima; every wave is past the last tile
+    lds_barrier();                                       // maxima; every wave is past the last tile
     float alpha[QT];
 #pragma unroll
     for (int i = 0; i < QT; ++i) {
@@ -412,7 +464,8 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
       stv<4>(sp + ((rg + i) * 16 + fr) * PP + ksub * 16 + g4 * 4, p);
     }
     if (t + 1 < t1) store(buf ^ 1);
-    __syncthreads();                                     // scores, next tile
+    if (t + 2 < t1) load(t + 2);
+    lds_barrier();                                       // scores, next tile
 #pragma unroll
     for (int i = 0; i < QT; ++i)
 #pragma unroll
@@ -458,44 +511,16 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
     if (r >= nrow) continue;
     const float sum = (smax[r] + smax[RW + r]) + (smax[2 * RW + r] + smax[3 * RW + r]);
     const size_t row = grow0 + row0 + r;
-    const float inv = 1.f / sum;
+    const float inv = sum > 0.f ? 1.f / sum : 0.f;
     if (a.nsplit > 1 && wave == 0 && g4 == 0) a.ml[split * all + row] = make_float2(m[i], sum);
 #pragma unroll
     for (int n = 0; n < NDT; ++n) {
       const int c = wave * NDT * 16 + n * 16 + g4 * 4;
       if (c >= a.DV) continue;
-      if (a.nsplit > 1) {
-        *reinterpret_cast<float4*>(a.part + (split * all + row) * a.DV + c) =
-            make_float4(o[i][n][0], o[i][n][1], o[i][n][2], o[i][n][3]);
-      } else {
-        const float f[4] = {o[i][n][0] * inv, o[i][n][1] * inv, o[i][n][2] * inv, o[i][n][3] * inv};
-        stv<4>(a.out + row * a.DV + c, f);
-      }
+      const float f[4] = {o[i][n][0] * inv, o[i][n][1] * inv, o[i][n][2] * inv, o[i][n][3] * inv};
+      stv<4>(a.nsplit > 1 ? a.part + (split * all + row) * a.DV + c : a.out + row * a.DV + c, f);
     }
   }
-}
-
-// out [rows, DV] from the splits' partials: sum_s e^(m_s - m) part_s / sum_s e^(m_s - m) l_s
-__global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part, const float2* __restrict__ ml,
-                                                           int nsplit, size_t rows, int DV, uint16_t* __restrict__ out) {
-  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
-  const size_t row = i / (DV / 4);
-  if (row >= rows) return;
-  const int c = (int)(i - row * (DV / 4)) * 4;
-  float m = -1e30f, l = 0.f, f[4] = {0.f, 0.f, 0.f, 0.f};
-  for (int s = 0; s < nsplit; ++s) m = fmaxf(m, ml[s * rows + row].x);
-  for (int s = 0; s < nsplit; ++s) {
-    const float2 v = ml[s * rows + row];
-    if (v.y <= 0.f) continue;                            // nothing seen: the partial was not written
-    const float w = __builtin_amdgcn_exp2f(v.x - m);
-    const float4 p = *reinterpret_cast<const float4*>(part + (s * rows + row) * DV + c);
-    l += w * v.y;
-    f[0] += w * p.x; f[1] += w * p.y; f[2] += w * p.z; f[3] += w * p.w;
-  }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
-#pragma unroll
-  for (int j = 0; j < 4; ++j) f[j] *= inv;
-  stv<4>(out + row * DV + c, f);
 }
 
 template <int DPV, int QT, int NW>
@@ -513,11 +538,6 @@ int launch_latent(const LatentArgs& a, int B, int max_q, hipStream_t s) {
   }
   kern<<<dim3((unsigned)nz, B, a.nsplit), 64 * NW, lds, s>>>(a);
   DOCQA_CHECK_LAUNCH();
-  if (a.nsplit > 1) {
-    const size_t rows = (size_t)a.tokens * a.H, n = rows * (a.DV / 4);
-    latent_merge_kernel<<<(unsigned)((n + 255) / 256), 256, 0, s>>>(a.part, a.ml, a.nsplit, rows, a.DV, a.out);
-    DOCQA_CHECK_LAUNCH();
-  }
   return 0;
 }
 
@@ -535,11 +555,14 @@ int dispatch_latent(const LatentArgs& a, int B, int max_q, hipStream_t s) {
 template <typename PT, typename T>
 int store_types(const void* P, void* q, void* cache, int T_, const StoreArgs& a, hipStream_t s) {
   const bool v4 = a.d % 8 == 0 && a.r % 8 == 0 && a.R % 8 == 0 && a.ld % 4 == 0;
-  const int V = v4 ? 4 : 1;
+  // many tokens: 16-byte pieces of bf16 rows
+  const bool v8 = v4 && T_ >= 256 && sizeof(T) == 2 && a.r % 16 == 0 && a.ld % 8 == 0;
+  const int V = v8 ? 8 : v4 ? 4 : 1;
   const int per = a.d / V + a.r / 2 / V + (v4 ? 0 : a.d8 - a.d + a.r8 - a.r);
   const int ny = (a.H * per + 255) / 256;
   dim3 grid(T_, ny + (a.wn ? 1 : 0));
-  if (v4) latent_store_kernel<4, 2, PT, T><<<grid, 256, 0, s>>>((const PT*)P, (T*)q, (T*)cache, ny, a);
+  if (v8) latent_store_kernel<8, 1, PT, T><<<grid, 256, 0, s>>>((const PT*)P, (T*)q, (T*)cache, ny, a);
+  else if (v4) latent_store_kernel<4, 2, PT, T><<<grid, 256, 0, s>>>((const PT*)P, (T*)q, (T*)cache, ny, a);
   else latent_store_kernel<1, 8, PT, T><<<grid, 256, 0, s>>>((const PT*)P, (T*)q, (T*)cache, ny, a);
   DOCQA_CHECK_LAUNCH();
   return 0;
@@ -574,27 +597,36 @@ int docqa_latent_store(const void* P, int p_f32, int S, size_t slab, int ld, con
                : store_types<uint16_t, uint16_t>(P, q, cache, T, a, s);
 }
 
-int docqa_head_project(const void* x, const void* w, void* y, int T, int H, int K, int N, int E, hipStream_t s) {
+int docqa_head_project(const void* x, const void* part, const void* ml, int nsplit, const void* w, void* y, int T, int H,
+                       int K, int N, int E, hipStream_t s) {
   if (T == 0) return 0;
   if (H < 1 || K < 8 || K % 8 || K > 2048 || N < 1 || E < 0 || E % 8 || (E > 0 && N % 8)) return -1;
-  if (!docqa_aligned16(x) || !docqa_aligned16(w) || !docqa_aligned16(y)) return -1;
+  if (!docqa_aligned16(w) || !docqa_aligned16(y) || !docqa_aligned16(part ? part : x)) return -1;
+  if (part && (!ml || nsplit < 1 || nsplit > kMaxSplit || E > 0)) return -1;
   const int pitch = (K + 31) / 32 * 32 + 8;
-#define GO(MT)                                                                                                        \
+#define LAUNCH(MT, NJ, MERGE)                                                                                         \
   do {                                                                                                                \
     const size_t lds = (size_t)16 * MT * pitch * 2;                                                                   \
-    auto kern = head_project_kernel<MT>;                                                                              \
-    if (lds > 64 * 1024) {                                                                                            \
+    auto kern = head_project_kernel<MT, NJ, MERGE>;                                                                   \
+    if (lds > 56 * 1024) {                                                                                            \
       static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern),                            \
                                                       hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 1024);         \
       if (e != hipSuccess) return (int)e;                                                                             \
     }                                                                                                                 \
-    kern<<<dim3(H, (T + 16 * MT - 1) / (16 * MT), (N + 127) / 128), 256, lds, s>>>((const uint16_t*)x,                \
-        (const uint16_t*)w, (uint16_t*)y, T, H, K, N, E);                                                             \
+    kern<<<dim3(H, (T + 16 * MT - 1) / (16 * MT), (N + 64 * NJ - 1) / (64 * NJ)), 256, lds, s>>>(                     \
+        (const uint16_t*)x, (const uint16_t*)part, (const float2*)ml, nsplit, (const uint16_t*)w, (uint16_t*)y, T, H, K, N, E);        \
   } while (0)
-  if (T > 32 && K <= 256) GO(4);
-  else if (T > 16 && K <= 1024) GO(2);
-  else GO(1);
+#define GO(MT, NJ)                       \
+  do {                                   \
+    if (part) LAUNCH(MT, NJ, true);      \
+    else LAUNCH(MT, NJ, false);          \
+  } while (0)
+  if (T > 64 && K <= 256) GO(4, 2);
+  else if (T > 64 && K <= 1024) GO(2, 2);
+  else if (T > 16 && part && N > 64) GO(1, 2);           // one workgroup sums a row's splits
+  else GO(1, 1);
 #undef GO
+#undef LAUNCH
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
@@ -613,25 +645,26 @@ int docqa_latent_gather(const void* cache, const int* block_tables, int maxb, co
 
 int docqa_latent_attn_ok(int D, int DV) { return D % 8 == 0 && DV % 8 == 0 && DV <= 512 && D > DV && D <= (DV <= 64 ? 128 : DV <= 128 ? 192 : DV <= 256 ? 320 : 576); }
 
-// Key splits: enough workgroups for every CU, at least two tiles each
+// Key splits: enough workgroups for every CU; two tiles each unless there are few sequences
 int docqa_latent_splits(int B, int max_q, int H, int DV, int max_keys) {
   const long long rows = (long long)max_q * H;
   const int rw = rows <= 16 ? 16 : (DV > 256 || rows <= 32) ? 32 : 64;
   const long long wgs = (long long)B * ((rows + rw - 1) / rw);
   const int tiles = (max_keys + KB - 1) / KB + 1;
   const long long n = wgs > 0 ? 256 / wgs : 1;
-  const int most = tiles / 2 < 16 ? tiles / 2 : 16;
+  int most = n >= 8 ? tiles : tiles / 2;
+  if (most > kMaxSplit) most = kMaxSplit;
   return n < 1 || most < 1 ? 1 : (int)(n < most ? n : most);
 }
 
 int docqa_latent_attn(const void* q, const void* kc, const int* block_tables, int maxb, const int* cu, const int* ctx,
-                      const float* sink, void* out, float* part, void* ml, int nsplit, int B, int max_q, int tokens, int H,
+                      const float* sink, void* out, void* part, void* ml, int nsplit, int B, int max_q, int tokens, int H,
                       int D, int DV, int BS, float scale, int window, hipStream_t s) {
   if (B == 0 || max_q == 0 || tokens == 0) return 0;
   if (!docqa_latent_attn_ok(D, DV) || H < 1 || (BS & (BS - 1)) != 0 || nsplit < 1 || nsplit > 65535) return -1;
   if (nsplit > 1 && (!part || !ml)) return -1;
   if (!docqa_aligned16(q) || !docqa_aligned16(kc) || !docqa_aligned16(out)) return -1;
-  const LatentArgs a{(const uint16_t*)q, (const uint16_t*)kc, (uint16_t*)out, block_tables, maxb, cu, ctx, sink, part,
+  const LatentArgs a{(const uint16_t*)q, (const uint16_t*)kc, (uint16_t*)out, block_tables, maxb, cu, ctx, sink, (uint16_t*)part,
                      (float2*)ml, tokens, H, D, DV, log2_of(BS), nsplit, window, scale};
   if (DV <= 64) return dispatch_latent<64>(a, B, max_q, s);
   if (DV <= 128) return dispatch_latent<128>(a, B, max_q, s);

@@ -229,6 +229,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
                                                                    const uint16_t* __restrict__ vc,
                                                                    uint16_t* __restrict__ out, WindowArgs a) {
   static_assert(!SHARED || DP == DPV, "shared rows");
+  static_assert(!PACKED || ((KB * DP / 8) % (64 * NW) == 0 && (KB * DPV / 8) % (64 * NW) == 0), "packed loads");
   constexpr int PITCH = DP + 8, PITCHV = DPV + 8, NCH = DP / 8, NCV = DPV / 8, NKT = KB / 16, NKS = DP / 32,
                 NDT = DPV / 16;
   constexpr int TILES = SPLIT ? NW : 2;
@@ -299,7 +300,24 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
   const float sl2 = a.scale * kLog2e;
 
   const int ltid = SPLIT ? lane : tid;
-  uint4 rk[CPT], rv[SHARED ? 1 : CPV];
+  // packed: every thread's pieces of a tile start at fixed pointers, a row apart by a fixed stride, and
+  // load without a branch: keys past the end repeat the last one (masked), columns past a row its first
+  const uint16_t *kp[PACKED ? CPT : 1], *vp[PACKED ? CPV : 1];
+  size_t kst[PACKED ? CPT : 1];
+  if constexpr (PACKED) {
+#pragma unroll
+    for (int i = 0; i < CPT; ++i) {
+      const int c0 = ((ltid + LOADERS * i) % NCH) * 8, c = c0 < D ? c0 : 0;
+      kp[i] = c < a.kd ? kc + (size_t)kvh * a.kd + c : a.kr + (c - a.kd);
+      kst[i] = c < a.kd ? a.ld : D - a.kd;
+    }
+#pragma unroll
+    for (int i = 0; i < CPV; ++i) {
+      const int c = ((ltid + LOADERS * i) % NCV) * 8;
+      vp[i] = vc + (size_t)kvh * a.vd + (c < a.vd ? c : 0);
+    }
+  }
+  u32x4 rk[CPT], rv[SHARED ? 1 : CPV];
   float rs_ = 1.f;
   auto cache_row = [&](int key) {
     const int kblk = key >> a.log2BS;
@@ -311,27 +329,24 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
 #pragma unroll
     for (int i = 0; i < CPT; ++i) {
       const int e = ltid + LOADERS * i, row = e / NCH, c = (e % NCH) * 8;
-      rk[i] = make_uint4(0, 0, 0, 0);
-      if (e < KB * NCH && kb + row <= pos_hi && c < D) {
-        if constexpr (PACKED) {
-          const size_t j = kbase + kb + row;
-          rk[i] = *reinterpret_cast<const uint4*>(c < a.kd ? kc + j * a.ld + kvh * a.kd + c
-                                                           : a.kr + j * (D - a.kd) + (c - a.kd));
-        } else {
-          rk[i] = *reinterpret_cast<const uint4*>(kc + cache_row(kb + row) * D + c);
-        }
+      if constexpr (PACKED) {
+        rk[i] = *reinterpret_cast<const u32x4*>(kp[i] + (kbase + min(kb + row, pos_hi)) * kst[i]);
+      } else {
+        rk[i] = u32x4{0, 0, 0, 0};
+        if (e < KB * NCH && kb + row <= pos_hi && c < D)
+          rk[i] = *reinterpret_cast<const u32x4*>(kc + cache_row(kb + row) * D + c);
       }
     }
     if constexpr (!SHARED) {
 #pragma unroll
       for (int i = 0; i < CPV; ++i) {
         const int e = ltid + LOADERS * i, row = e / NCV, c = (e % NCV) * 8;
-        rv[i] = make_uint4(0, 0, 0, 0);
-        if (e < KB * NCV && kb + row <= pos_hi && c < (PACKED ? a.vd : D)) {
-          if constexpr (PACKED)
-            rv[i] = *reinterpret_cast<const uint4*>(vc + (size_t)(kbase + kb + row) * a.ld + kvh * a.vd + c);
-          else
-            rv[i] = *reinterpret_cast<const uint4*>(vc + cache_row(kb + row) * D + c);
+        if constexpr (PACKED) {
+          rv[i] = *reinterpret_cast<const u32x4*>(vp[i] + (size_t)(kbase + min(kb + row, pos_hi)) * a.ld);
+        } else {
+          rv[i] = u32x4{0, 0, 0, 0};
+          if (e < KB * NCV && kb + row <= pos_hi && c < D)
+            rv[i] = *reinterpret_cast<const u32x4*>(vc + cache_row(kb + row) * D + c);
         }
       }
     }
@@ -346,14 +361,14 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
     for (int i = 0; i < CPT; ++i) {
       const int e = ltid + LOADERS * i, row = e / NCH, c = (e % NCH) * 8;
       if (e < KB * NCH) {
-        *reinterpret_cast<uint4*>(k + row * PITCH + c) = rk[i];
+        *reinterpret_cast<u32x4*>(k + row * PITCH + c) = rk[i];
       }
     }
     if constexpr (!SHARED) {
 #pragma unroll
       for (int i = 0; i < CPV; ++i) {
         const int e = ltid + LOADERS * i, row = e / NCV, c = (e % NCV) * 8;
-        if (e < KB * NCV) *reinterpret_cast<uint4*>(k + KTILE + row * PITCHV + c) = rv[i];
+        if (e < KB * NCV) *reinterpret_cast<u32x4*>(k + KTILE + row * PITCHV + c) = rv[i];
       }
     }
     if (ltid < KB) scales[buf * KB + ltid] = rs_;
@@ -663,11 +678,19 @@ int docqa_packed_window_attn(const void* q, const void* kv, const void* kr, cons
   const WindowArgs a{nullptr, 0, cu, nullptr, nullptr, sink, H, H, D, 64, 6, scale, window, vdim,
                      cu_k, (const uint16_t*)kr, ld, d8, v8};
   const uint16_t* v = (const uint16_t*)kv + (size_t)H * d8;
-#define GO(DP, DPV, QT, KB) return launch_mfma<DP, DPV, QT, KB, 4, false, false, true>(q, kv, v, out, a, B, max_q, s)
-  if (D <= 64 && vdim <= 64) GO(64, 64, 2, 64);
-  if (D <= 96 && vdim <= 64) GO(96, 64, 2, 64);
-  if (D <= 128 && vdim <= 128) GO(128, 128, 2, 64);
-  if (D <= 192 && vdim <= 128) GO(192, 128, 2, 32);
-  GO(256, 256, 1, 32);
+  // 128 query rows a workgroup, 64 where that leaves CUs without one
+  const bool few = (long long)B * H * ((max_q + 127) / 128) < 384;
+#define RUN(DP, DPV, QT, KB) return launch_mfma<DP, DPV, QT, KB, 4, false, false, true>(q, kv, v, out, a, B, max_q, s)
+#define GO(DP, DPV, KB)               \
+  do {                                \
+    if (few) RUN(DP, DPV, 1, KB);     \
+    RUN(DP, DPV, 2, KB);              \
+  } while (0)
+  if (D <= 64 && vdim <= 64) GO(64, 64, 64);
+  if (D <= 96 && vdim <= 64) GO(96, 64, 64);
+  if (D <= 128 && vdim <= 128) GO(128, 128, 64);
+  if (D <= 192 && vdim <= 128) GO(192, 128, 32);
+  RUN(256, 256, 1, 32);
 #undef GO
+#undef RUN
 }

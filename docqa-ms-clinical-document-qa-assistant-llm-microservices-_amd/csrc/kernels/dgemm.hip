@@ -730,6 +730,7 @@ int docqa_dgemm_argmax(const void* X, const void* W, int64_t* out, float* outv, 
 // row; the 4 waves split K and meet in LDS.  Workgroup = R output rows x one K slice.
 //   * EPI_PARTIAL: fp32 slab P[slice][n] for the split-K consumers (same layout as dgemm);
 //   * EPI_GLU: R = 16 rows = one 8-interleaved gate|up group -> 8 SwiGLU outputs, bf16;
+//   * EPI_RELU2, EPI_GELU: the activation of R outputs, bf16;
 //   * XN: the input row is built in LDS from the previous projection's slabs (XNormIn),
 //     its loads queued behind the weight loads (the stream is already in flight).
 // Shapes: N % R == 0, Ks = K / S with Ks % 2048 == 0 (C = Ks / 2048 chunks per lane), and
@@ -747,7 +748,8 @@ __global__ __launch_bounds__(256) void gemv_kernel(const uint16_t* __restrict__ 
                                                    uint16_t* __restrict__ Y, float* __restrict__ P, int N, int K,
                                                    int Ks, XNormIn xn, int* __restrict__ pi = nullptr,
                                                    int n_valid = 0) {
-  static_assert(EPI == EPI_PARTIAL || (EPI == EPI_GLU && R == 16) || (EPI == EPI_ARGMAX && R == 16),
+  constexpr bool ACT = EPI == EPI_RELU2 || EPI == EPI_GELU;
+  static_assert(EPI == EPI_PARTIAL || ACT || (EPI == EPI_GLU && R == 16) || (EPI == EPI_ARGMAX && R == 16),
                 "GLU: one 16-row gate|up group; ARGMAX: 16 logits per workgroup");
   static_assert(R * C <= 32, "loads in flight per lane must fit the vmcnt counter");
   __shared__ __attribute__((aligned(16))) uint16_t sx[XN ? kXnMaxK : 8];
@@ -809,6 +811,10 @@ __global__ __launch_bounds__(256) void gemv_kernel(const uint16_t* __restrict__ 
   __syncthreads();
   if constexpr (EPI == EPI_PARTIAL) {
     if (tid < R) P[(size_t)slice * N + n0 + tid] = red[0][tid] + red[1][tid] + red[2][tid] + red[3][tid];
+  } else if constexpr (ACT) {
+    if (tid < R)
+      Y[n0 + tid] = f2bf(act_f<EPI == EPI_RELU2 ? ACT_RELU2 : ACT_GELU_TANH>(red[0][tid] + red[1][tid] + red[2][tid] +
+                                                                             red[3][tid]));
   } else if constexpr (EPI == EPI_ARGMAX) {
     // LM head + greedy pick: the 16 logits (bf16-rounded, as the unfused logits) -> one
     // (value, id) partial per workgroup at P / pi [blockIdx.x] for argmax_merge_kernel
@@ -896,6 +902,26 @@ int docqa_gemv(const void* X, const void* W, void* Y, float* P, int N, int K, in
     rc = xnm ? launch_gemv<EPI_PARTIAL, true>(R, C, grid, s, x, w, nullptr, P, N, K, Ks, xn)
              : launch_gemv<EPI_PARTIAL, false>(R, C, grid, s, x, w, nullptr, P, N, K, Ks, xn);
   if (rc) return rc;
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+// Y [1, N] = act(X . W^T) of one row (K = 2048 or 4096)
+int docqa_gemv_act(const void* X, const void* W, void* Y, int act, int N, int K, hipStream_t s) {
+  if (N % 8 || (K != 2048 && K != 4096)) return -1;
+  const XNormIn xn{};
+  const uint16_t *x = (const uint16_t*)X, *w = (const uint16_t*)W;
+#define GO(E, C) gemv_kernel<8, C, E, false, true><<<N / 8, 256, 0, s>>>(x, w, (uint16_t*)Y, nullptr, N, K, K, xn)
+  if (act == ACT_RELU2) {
+    if (K == 2048) GO(EPI_RELU2, 1);
+    else GO(EPI_RELU2, 2);
+  } else if (act == ACT_GELU_TANH) {
+    if (K == 2048) GO(EPI_GELU, 1);
+    else GO(EPI_GELU, 2);
+  } else {
+    return -1;
+  }
+#undef GO
   DOCQA_CHECK_LAUNCH();
   return 0;
 }

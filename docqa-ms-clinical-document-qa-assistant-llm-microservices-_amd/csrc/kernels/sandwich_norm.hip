@@ -8,6 +8,7 @@
 // read and written once.
 #include "docqa_common.h"
 #include "docqa_elem.h"
+#include <type_traits>
 
 using namespace docqa;
 
@@ -19,17 +20,47 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
   return red[0] + red[1] + red[2] + red[3];
 }
 
-template <int NV, int V, typename PT, typename OT>
+// one new token a row, an input convolution behind the norm: out2 = h + conv(h), the identity in
+// w's last tap; state holds the last taps - 1 rows h of each slot (slot -1: none, position 0: zeros)
+template <typename OT>
+struct ConvArgs {
+  const float* w;         // [taps, H]
+  int taps;
+  OT* state;              // [slots, taps - 1, H]
+  const int* slots;
+  const int* positions;
+  OT* out2;
+};
+
+// CONV: 0 none, taps of 2 to 4 with the state's rows loaded ahead of the reductions, -1 any taps
+template <int NV, int V, typename PT, typename OT, int CONV = 0>
 __global__ __launch_bounds__(256) void sandwich_rmsnorm_kernel(const PT* __restrict__ P, int S, size_t slab,
                                                                float* __restrict__ res,
                                                                const float* __restrict__ w_post,
                                                                const float* __restrict__ add,
                                                                const float* __restrict__ w_next,
-                                                               OT* __restrict__ out, int H, float eps) {
+                                                               OT* __restrict__ out, int H, float eps,
+                                                               ConvArgs<OT> cv) {
   __shared__ float red[2][4];
   const size_t row = blockIdx.x;
   const int tid = threadIdx.x, n = H / V;
   float y[NV][V], x[NV][V];
+  constexpr int NS = CONV > 0 ? CONV - 1 : 1;
+  float st[CONV > 0 ? NV : 1][NS][V];                    // the slot's rows (zeros at position 0)
+  if constexpr (CONV > 0) {
+    const int slot = cv.slots[row];
+    const bool carry = slot >= 0 && cv.positions[row] > 0;
+    const OT* sp = cv.state + (size_t)max(slot, 0) * NS * H;
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+#pragma unroll
+      for (int k = 0; k < NS; ++k) {
+        const int c = min(tid + 256 * i, n - 1);
+        ldv<V>(sp + (size_t)k * H + c * V, st[i][k]);
+#pragma unroll
+        for (int j = 0; j < V; ++j) st[i][k][j] = carry ? st[i][k][j] : 0.f;
+      }
+  }
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
@@ -69,6 +100,50 @@ __global__ __launch_bounds__(256) void sandwich_rmsnorm_kernel(const PT* __restr
 #pragma unroll
       for (int j = 0; j < V; ++j) o[j] = x[i][j] * ix * g[j];
       stv<V>(out + row * H + c * V, o);
+      if constexpr (CONV > 0) {
+        float s[V], wk[V];
+        ldv<V>(cv.w + (size_t)NS * H + c * V, wk);
+#pragma unroll
+        for (int j = 0; j < V; ++j) {
+          o[j] = rnd((const OT*)nullptr, o[j]);
+          s[j] = wk[j] * o[j];
+        }
+        const int slot = cv.slots[row];
+#pragma unroll
+        for (int k = 0; k < NS; ++k) {
+          ldv<V>(cv.w + (size_t)k * H + c * V, wk);
+#pragma unroll
+          for (int j = 0; j < V; ++j) s[j] += wk[j] * st[i][k][j];
+          if (slot >= 0)
+            stv<V>(cv.state + ((size_t)slot * NS + k) * H + c * V, k + 1 < NS ? st[i][k + 1 < NS ? k + 1 : 0] : o);
+        }
+        stv<V>(cv.out2 + row * H + c * V, s);
+      } else if constexpr (CONV < 0) {
+        const int slot = cv.slots[row], last = cv.taps - 1;
+        const bool carry = slot >= 0 && cv.positions[row] > 0;
+        OT* st = cv.state + (size_t)max(slot, 0) * last * H + c * V;
+        float s[V], wk[V];
+        ldv<V>(cv.w + (size_t)last * H + c * V, wk);
+#pragma unroll
+        for (int j = 0; j < V; ++j) {
+          o[j] = rnd((const OT*)nullptr, o[j]);
+          s[j] = wk[j] * o[j];
+        }
+        for (int k = 0; k < last; ++k) {               // row k <- row k + 1, the last <- h
+          float f[V], nx[V];
+#pragma unroll
+          for (int j = 0; j < V; ++j) f[j] = 0.f, nx[j] = k + 1 == last ? o[j] : 0.f;
+          if (carry) {
+            ldv<V>(st + (size_t)k * H, f);
+            if (k + 1 < last) ldv<V>(st + (size_t)(k + 1) * H, nx);
+          }
+          ldv<V>(cv.w + (size_t)k * H + c * V, wk);
+#pragma unroll
+          for (int j = 0; j < V; ++j) s[j] += wk[j] * f[j];
+          if (slot >= 0) stv<V>(st + (size_t)k * H, nx);
+        }
+        stv<V>(cv.out2 + row * H + c * V, s);
+      }
     }
   }
 }
@@ -152,10 +227,20 @@ int launch_add_scaled(const void* P, int SP, const void* Q, int SQ, float* res, 
 
 template <int V, typename PT, typename OT>
 int launch_sandwich(const PT* P, int S, float* res, const float* w_post, const float* add, const float* w_next,
-                    OT* out, int rows, int H, float eps, hipStream_t s) {
+                    OT* out, int rows, int H, float eps, const std::common_type_t<ConvArgs<OT>>* cv, hipStream_t s) {
   const size_t slab = (size_t)rows * H;
   const int nv = (H / V + 255) / 256;
-#define GO(N) sandwich_rmsnorm_kernel<N, V, PT, OT><<<rows, 256, 0, s>>>(P, S, slab, res, w_post, add, w_next, out, H, eps)
+  const ConvArgs<OT> none{};
+#define LAUNCH(N, C) sandwich_rmsnorm_kernel<N, V, PT, OT, (C)><<<rows, 256, 0, s>>>(P, S, slab, res, w_post, add, w_next, out, H, eps, cv ? *cv : none)
+#define GO(N)                                                      \
+  do {                                                             \
+    const int taps = cv ? cv->taps : 0;                            \
+    if (!cv) LAUNCH(N, 0);                                         \
+    else if (V > 1 && N <= 8 && taps == 2) LAUNCH(N, V > 1 && N <= 8 ? 2 : -1); \
+    else if (V > 1 && N <= 8 && taps == 3) LAUNCH(N, V > 1 && N <= 8 ? 3 : -1); \
+    else if (V > 1 && N <= 8 && taps == 4) LAUNCH(N, V > 1 && N <= 8 ? 4 : -1); \
+    else LAUNCH(N, -1);                                            \
+  } while (0)
   if (nv <= 1) GO(1);
   else if (nv <= 2) GO(2);
   else if (nv <= 4) GO(4);
@@ -163,6 +248,7 @@ int launch_sandwich(const PT* P, int S, float* res, const float* w_post, const f
   else if (nv <= 16) GO(16);
   else return -1;
 #undef GO
+#undef LAUNCH
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
@@ -171,10 +257,19 @@ template <typename PT>
 int sandwich_out(const PT* P, int S, float* res, const float* w_post, const float* add, const float* w_next,
                  void* out, int out_f32, int rows, int H, float eps, hipStream_t s) {
   if (out_f32)
-    return H % 4 == 0 ? launch_sandwich<4>(P, S, res, w_post, add, w_next, (float*)out, rows, H, eps, s)
-                      : launch_sandwich<1>(P, S, res, w_post, add, w_next, (float*)out, rows, H, eps, s);
-  return H % 4 == 0 ? launch_sandwich<4>(P, S, res, w_post, add, w_next, (uint16_t*)out, rows, H, eps, s)
-                    : launch_sandwich<1>(P, S, res, w_post, add, w_next, (uint16_t*)out, rows, H, eps, s);
+    return H % 4 == 0 ? launch_sandwich<4>(P, S, res, w_post, add, w_next, (float*)out, rows, H, eps, nullptr, s)
+                      : launch_sandwich<1>(P, S, res, w_post, add, w_next, (float*)out, rows, H, eps, nullptr, s);
+  return H % 4 == 0 ? launch_sandwich<4>(P, S, res, w_post, add, w_next, (uint16_t*)out, rows, H, eps, nullptr, s)
+                    : launch_sandwich<1>(P, S, res, w_post, add, w_next, (uint16_t*)out, rows, H, eps, nullptr, s);
+}
+
+template <typename PT, typename OT>
+int sandwich_conv(const PT* P, int S, float* res, const float* w_post, const float* w_next, const float* cw, int taps,
+                  void* state, const int* slots, const int* positions, void* out, void* out2, int rows, int H, float eps,
+                  hipStream_t s) {
+  const ConvArgs<OT> cv{cw, taps, (OT*)state, slots, positions, (OT*)out2};
+  return H % 4 == 0 ? launch_sandwich<4>(P, S, res, w_post, (const float*)nullptr, w_next, (OT*)out, rows, H, eps, &cv, s)
+                    : launch_sandwich<1>(P, S, res, w_post, (const float*)nullptr, w_next, (OT*)out, rows, H, eps, &cv, s);
 }
 
 template <int V, typename T>
@@ -222,4 +317,15 @@ int docqa_add_scaled(const void* P, int p_f32, int SP, const void* Q, int q_f32,
                  : launch_add_scaled<float, uint16_t>(P, SP, Q, SQ, res, m, out, n, s);
   return q_f32 ? launch_add_scaled<uint16_t, float>(P, SP, Q, SQ, res, m, out, n, s)
                : launch_add_scaled<uint16_t, uint16_t>(P, SP, Q, SQ, res, m, out, n, s);
+}
+
+int docqa_sandwich_rmsnorm_conv(const void* P, int p_f32, int S, float* res, const float* w_post, const float* w_next,
+                                const float* cw, int taps, void* state, const int* slots, const int* positions, void* out,
+                                void* out2, int out_f32, int rows, int H, float eps, hipStream_t s) {
+  if (rows == 0) return 0;
+  if (S < 1 || H < 1 || taps < 1 || (out_f32 && !p_f32)) return -1;
+#define ARGS S, res, w_post, w_next, cw, taps, state, slots, positions, out, out2, rows, H, eps, s
+  if (out_f32) return sandwich_conv<float, float>((const float*)P, ARGS);
+  return p_f32 ? sandwich_conv<float, uint16_t>((const float*)P, ARGS) : sandwich_conv<uint16_t, uint16_t>((const uint16_t*)P, ARGS);
+#undef ARGS
 }

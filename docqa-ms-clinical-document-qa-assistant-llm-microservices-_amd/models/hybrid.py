@@ -34,6 +34,7 @@ decays, step sizes and states are fp32.  float32 runs everything in fp32.
 from __future__ import annotations
 
 import math
+import os
 import zlib
 from dataclasses import dataclass, field
 
@@ -192,6 +193,10 @@ class HybridConfig:
 
     def num_params(self) -> int:
         return sum(math.prod(s) for s in self.tensor_shapes().values())
+
+
+# decode rows up to which a captured step runs a parallel layer's sublayers as two graph branches
+FORK_MAX_ROWS = int(os.environ.get("DOCQA_FORK_MAX_ROWS", "64"))
 
 
 def _pad_up(n: int, m: int) -> int:
@@ -396,13 +401,13 @@ class LatentAttention:
                                                   keys.cu, m.max_len, sp.scale, window=sp.window, sink=self.sink))
                 continue
             qc = ops.head_project(qp, self.w_qc, self.r8)
-            kw = dict(window=sp.window, sink=self.sink, v_dim=self.R8)
+            kw = dict(window=sp.window, sink=self.sink)
             if p.decode:
-                a = ops.window_attn(qc, cache, m.block_tables, m.context_lens, sp.scale, **kw)
+                a = ops.latent_attn(qc, cache, m.block_tables, m.context_lens, sp.scale, self.w_cv, **kw)
             else:
-                a = ops.window_attn(qc, cache, m.block_tables, m.prefix_lens, sp.scale, cu=m.cu_seqlens,
+                a = ops.latent_attn(qc, cache, m.block_tables, m.prefix_lens, sp.scale, self.w_cv, cu=m.cu_seqlens,
                                     max_q=m.max_len, **kw)
-            out.append(ops.head_project(a, self.w_cv))
+            out.append(a)
         return ops.project(_join(out), self.o, decode)
 
 
@@ -471,6 +476,7 @@ class HybridModel(Decoder):
         self.vocab_start = 0
         att = [s.mixer for s in cfg.layer_specs if not isinstance(s.mixer, SelectiveScanSpec)]
         self.hq, self.hkv = (att[0].heads, getattr(att[0], "kv_heads", 1)) if att else (1, 1)
+        self._side_stream = None  # second branch of captured decode steps
         self.tap = None           # a list: receives the residual stream after every run
         self._load(weights if weights is not None else _RandomWeights(cfg, self.device, seed))
 
@@ -597,16 +603,46 @@ class HybridModel(Decoder):
         fw.rope = {k: ops.rope_table(pos, f) for k, f in self.rope_freq.items()}
         first = self.layers[0]["norm1"] if self.layers else self.final_norm
         res, _, h = ops.embed_scale_rmsnorm(input_ids, self.embed, cfg.embed_scale, first, eps)
-        for i, (L, (cache, conv_state)) in enumerate(zip(self.layers, caches)):
-            nxt = self.layers[i + 1]["norm1"] if i + 1 < len(self.layers) else self.final_norm
-            y = L["mixer"].run(L["conv"].run(h, parts, conv_state), parts, slot_mapping, cache, decode, fw)
-            f = L["mlp"].run(h, decode) if L["mlp"] is not None else None
+        hm = self.layers[0]["conv"].run(h, parts, caches[0][1]) if self.layers else h
+        for i, L in enumerate(self.layers):
+            y, f = self._sublayers(L, h, hm, parts, slot_mapping, caches[i][0], decode, fw)
             xs = ops.add_scaled(y, f, res, cfg.parallel.mult, dt)
             y = L["side"].run(xs, input_ids, self.side_embed, decode)
-            h = ops.sandwich_rmsnorm(y, res, L["side_norm"], nxt, eps, out_dtype=dt)
+            if i + 1 == len(self.layers):
+                h = ops.sandwich_rmsnorm(y, res, L["side_norm"], self.final_norm, eps, out_dtype=dt)
+            else:
+                nxt, state = self.layers[i + 1], caches[i + 1][1]
+                if decode:
+                    m = parts[0].meta
+                    h, hm = ops.sandwich_rmsnorm_conv(y, res, L["side_norm"], nxt["norm1"], eps, nxt["conv"].w, state,
+                                                      m.state_slots, m.positions)
+                else:
+                    h = ops.sandwich_rmsnorm(y, res, L["side_norm"], nxt["norm1"], eps, out_dtype=dt)
+                    hm = nxt["conv"].run(h, parts, state)
             if self.tap is not None:
                 self.tap.append(res.clone())
         return h
+
+    def _sublayers(self, L, h, hm, parts, slot_mapping, cache, decode, fw):
+        """The layer's mixer and feed-forward (or None).  In a captured decode step they are two
+        branches of the graph: the mixer's chain of small launches runs beside the feed-forward's
+        two weight-streaming ones."""
+        if L["mlp"] is None:
+            return L["mixer"].run(hm, parts, slot_mapping, cache, decode, fw), None
+        fork = (decode and h.is_cuda and h.shape[0] <= FORK_MAX_ROWS and torch.cuda.is_current_stream_capturing())
+        if not fork:
+            return L["mixer"].run(hm, parts, slot_mapping, cache, decode, fw), L["mlp"].run(h, decode)
+        if self._side_stream is None:
+            self._side_stream = torch.cuda.Stream(self.device)
+        main = torch.cuda.current_stream()
+        # h outlives the join below and f is consumed after it, so neither is handed out again while
+        # the other stream may still use it
+        self._side_stream.wait_stream(main)
+        with torch.cuda.stream(self._side_stream):
+            f = L["mlp"].run(h, decode)
+        y = L["mixer"].run(hm, parts, slot_mapping, cache, decode, fw)
+        main.wait_stream(self._side_stream)
+        return y, f
 
     def _head(self, x, logits_index, greedy_ids):
         if logits_index is not None:

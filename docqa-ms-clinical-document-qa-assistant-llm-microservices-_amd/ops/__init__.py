@@ -1222,9 +1222,23 @@ def activation(P, act: str, out_dtype=torch.bfloat16):
     return ref.activation(P, act, out_dtype)
 
 
+def sandwich_rmsnorm_conv(P, residual, w_post, w_next, eps: float, conv_w, state, slots, positions):
+    """:func:`sandwich_rmsnorm` of one token a row with the input convolution of the next layer
+    behind it: (h, h + conv(h)) in ``state``'s dtype, ``conv_w`` [taps, W] with the identity in
+    its last tap; advances ``state`` (rows with slot -1 leave none)."""
+    if _gpu(P):
+        return _native().sandwich_rmsnorm_conv(P.contiguous(), residual, w_post, w_next, conv_w, state, slots, positions,
+                                               float(eps))
+    h = ref.sandwich_rmsnorm(P, residual, w_post, w_next, eps, None, state.dtype)
+    return h, ref.conv_step(h, conv_w, None, state, slots, positions, False)[0]
+
+
 def squared_relu(P, out_dtype=torch.bfloat16):
     """max(P, 0)^2 of a projection."""
     return activation(P, ACT_RELU2, out_dtype)
+
+
+_PGEMM_ACT_TILES = int(os.environ.get("DOCQA_PGEMM_ACT_TILES", "96"))
 
 
 def act_linear(x, w, act: str, decode: bool = False):
@@ -1233,6 +1247,10 @@ def act_linear(x, w, act: str, decode: bool = False):
     if _gpu(x) and x.dtype == torch.bfloat16:
         N, K = w.shape
         M = x.numel() // K
+        if not decode and 256 < M <= MID_M_MAX and pgemm_ok(M, N, K) and ((M + 255) // 256) * (N // 256) >= _PGEMM_ACT_TILES:
+            return _native().pgemm(x.contiguous(), w, 3 + _ACT_CODE[act])
+        if M == 1 and gemv_plan(M, N, K)[0] == 1 and K <= 4096:
+            return _native().decode_act(x.contiguous(), w, _ACT_CODE[act])
         if (decode or M <= MID_M_MAX) and M > 1:
             if (M <= 128 and N % 64 == 0 and K % 512 == 0 and decode_plan(M, N, K)[0] == 1) or (
                     129 <= M <= MID_M_MAX and mid_plan(M, N, K)[0] == 1):
@@ -1266,11 +1284,20 @@ def side_gate(P, ids, table, col: int, n: int, out_dtype=torch.bfloat16):
 
 
 def side_project(P, ids, table, col: int, n: int, w, decode: bool = False):
-    """:func:`side_gate` of the gate projection ``P``, projected by ``w``: one launch for bf16
-    decode rows, where a row's gate is cheap to build in every workgroup."""
-    if _gpu(P) and w.dtype == torch.bfloat16 and P.shape[-2] <= MID_M_MAX and w.shape[1] <= 1024:
-        return _native().side_project(P.contiguous(), ids, table, int(col), int(n), w)
+    """:func:`side_gate` of the gate projection ``P``, projected by ``w``: one launch for a few
+    bf16 rows, where every workgroup builds their gate itself; else two."""
+    if _gpu(P) and w.dtype == torch.bfloat16 and w.shape[1] <= 1024:
+        if P.shape[-2] <= SIDE_FUSED_MAX:
+            return _native().side_project(P.contiguous(), ids, table, int(col), int(n), w)
+        g = side_gate(P, ids, table, col, n, w.dtype)
+        if P.shape[-2] <= SIDE_HEAD_MAX:
+            return head_project(g, w[None])
+        return project(g, w, decode)
     return project(side_gate(P, ids, table, col, n, w.dtype), w, decode)
+
+
+SIDE_FUSED_MAX = int(os.environ.get("DOCQA_SIDE_FUSED_MAX", "16"))
+SIDE_HEAD_MAX = int(os.environ.get("DOCQA_SIDE_HEAD_MAX", "512"))
 
 
 def soft_cap(x, cap: float):
@@ -1335,6 +1362,22 @@ def head_project(x, w, carry: int = 0):
     if _gpu(x) and x.dtype == torch.bfloat16:
         return _native().head_project(x.contiguous(), w, int(carry))
     return ref.head_project(x, w, carry)
+
+
+_LATENT_ROW = {64: 128, 128: 192, 256: 320, 512: 576}      # latent columns -> row elements, attn_latent.hip
+
+
+def latent_attn(q, cache, block_tables, ctx, scale: float, w, window: int = 0, sink=None, cu=None, max_q: int = 1):
+    """Attention in the latent space and the projection of what it attends: :func:`window_attn` of
+    queries [T, H (R8 + r8)] over the cached rows, whose first R8 elements are the values, then
+    :func:`head_project` with ``w`` [H, vdim, R8].  bf16 rows run on MFMA, the keys split over
+    workgroups where sequences are few and summed by the projection."""
+    K, D = w.shape[2], cache.shape[3]
+    if _gpu(q) and q.dtype == torch.bfloat16 and D <= next((_LATENT_ROW[n] for n in _LATENT_ROW if K <= n), 0):
+        return _native().latent_attn(q.contiguous(), cache, block_tables, cu, ctx, int(max_q), float(scale), int(window),
+                                     sink, w)
+    return head_project(window_attn(q, cache, block_tables, ctx, scale, window=window, sink=sink, cu=cu, max_q=max_q,
+                                    v_dim=K), w)
 
 
 def latent_gather(cache, block_tables, first, cu_k, total: int, rank: int):
@@ -1432,6 +1475,10 @@ def project(x, w, decode: bool = False):
         return torch.nn.functional.linear(x, w)
     N, K = w.shape
     M = x.numel() // K
+    if not decode and K >= 8192:
+        S = down_small_split(M, N, K)
+        if S:
+            return pgemm_partial(x, w, S)
     if decode or M <= MID_M_MAX:
         S, R = gemv_plan(M, N, K)
         if S:

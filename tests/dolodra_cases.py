@@ -128,6 +128,33 @@ def side_case(device, dtype):
             close(ops.side_project(p, *a, w.to(device), True), gate @ w[:, :n].float().T, dtype, (M, n, N, W, col))
 
 
+def norm_conv_case(device, dtype):
+    """The stream update, the next norm and its input convolution of one token a row, against the
+    three apart, over several steps and with rows that have no slot."""
+    for W, taps, S in ((40, 4, 1), (30, 2, 3), (48, 1, 2), (1000, 7, 1)):
+        g = torch.Generator().manual_seed(W)
+        eps, slots, T = 1e-4, [2, -1, 0], 9
+        wp, wn, cw = torch.randn(W, generator=g), torch.randn(W, generator=g), torch.randn(W, taps, generator=g)
+        P = torch.randn(T, S, 3, W, generator=g)
+        P = P.to(dtype).float() if S == 1 else P
+        x = torch.randn(T, 3, W, generator=g)
+        conv = cw.t().clone(memory_format=torch.contiguous_format)
+        conv[-1] += 1.0
+        state = torch.full((3, taps - 1, W), 9.0, dtype=dtype, device=device)
+        want_res = x + O.rms(P.sum(1), eps) * wp
+        want_h = O.rms(want_res, eps) * wn
+        for t in range(T):
+            r = x[t].clone().to(device)
+            h, hc = ops.sandwich_rmsnorm_conv(P[t].to(device) if S > 1 else P[t, 0].to(device, dtype), r, wp.to(device),
+                                              wn.to(device), eps, conv.to(device), state, i32(device, *slots),
+                                              i32(device, t, t, t))
+            close(r, want_res[t])
+            close(h, want_h[t], dtype)
+            for b in (0, 2):
+                close(hc[b:b + 1], O.conv_input(want_h[:t + 1, b], cw)[t:], dtype, (W, taps, t))
+        assert (state[1] == 9).all()
+
+
 def input_conv_case(device, dtype):
     """h + conv(h) in portions of several sizes, single tokens in both forms; a slot that another
     sequence used; and sequences side by side."""
@@ -225,13 +252,13 @@ class Latent:
                 out.append(ops.packed_window_attn(q, ops.linear(c, self.w_kv), kr, self.H, self.d, self.vd, i32(dev, 0, n),
                                                   i32(dev, 0, t0 + n - k0), n, self.scale, window=self.window, sink=sink))
             else:
-                kw = dict(window=self.window, sink=sink, v_dim=self.R8)
+                kw = dict(window=self.window, sink=sink)
                 q = ops.head_project(q, self.w_qc, self.r8)
                 if n == 1 and t0 > 0:
-                    a = ops.window_attn(q, cache, bt, i32(dev, t0 + 1), self.scale, **kw)
+                    out.append(ops.latent_attn(q, cache, bt, i32(dev, t0 + 1), self.scale, self.w_cv, **kw))
                 else:
-                    a = ops.window_attn(q, cache, bt, i32(dev, t0), self.scale, cu=i32(dev, 0, n), max_q=n, **kw)
-                out.append(ops.head_project(a, self.w_cv))
+                    out.append(ops.latent_attn(q, cache, bt, i32(dev, t0), self.scale, self.w_cv, cu=i32(dev, 0, n),
+                                               max_q=n, **kw))
             t0 += n
         assert t0 == T
         return torch.cat(out)
@@ -323,17 +350,21 @@ def batch_latent_case(device, dtype):
     cu = [0]
     for n in lens:
         cu.append(cu[-1] + n)
-    kw = dict(window=window, sink=sink, v_dim=R8)
-    both = ops.window_attn(q, cache, bt, i32(device, *ctx0), 0.1, cu=i32(device, *cu), max_q=max(lens), **kw)
-    assert both.shape == (sum(lens), H * R8)
+    kw = dict(window=window, sink=sink)
+    wv = (torch.randn(H, vd, R8, generator=g) * R8 ** -0.5).to(device, dtype)
+    both = ops.latent_attn(q, cache, bt, i32(device, *ctx0), 0.1, wv, cu=i32(device, *cu), max_q=max(lens), **kw)
+    assert both.shape == (sum(lens), H * vd)
+    plain = ops.head_project(ops.window_attn(q, cache, bt, i32(device, *ctx0), 0.1, cu=i32(device, *cu), max_q=max(lens),
+                                             v_dim=R8, **kw), wv)
+    close(both, plain.cpu(), dtype)
     for b, n in enumerate(lens):
-        one = ops.window_attn(q[cu[b]:cu[b + 1]], cache, bt[b:b + 1].contiguous(), i32(device, ctx0[b]), 0.1,
+        one = ops.latent_attn(q[cu[b]:cu[b + 1]], cache, bt[b:b + 1].contiguous(), i32(device, ctx0[b]), 0.1, wv,
                               cu=i32(device, 0, n), max_q=n, **kw)
         close(both[cu[b]:cu[b + 1]], one.cpu(), dtype)
-    dec = ops.window_attn(q[:4].contiguous(), cache, bt, i32(device, 21, 0, 80, 1), 0.1, **kw)
-    assert torch.equal(dec[1].float().cpu(), torch.zeros(H * R8))           # a padded row
+    dec = ops.latent_attn(q[:4].contiguous(), cache, bt, i32(device, 21, 0, 80, 1), 0.1, wv, **kw)
+    assert torch.equal(dec[1].float().cpu(), torch.zeros(H * vd))           # a padded row
     for b, n in ((0, 21), (2, 80), (3, 1)):
-        one = ops.window_attn(q[b:b + 1].contiguous(), cache, bt[b:b + 1].contiguous(), i32(device, n), 0.1, **kw)
+        one = ops.latent_attn(q[b:b + 1].contiguous(), cache, bt[b:b + 1].contiguous(), i32(device, n), 0.1, wv, **kw)
         close(dec[b:b + 1], one.cpu(), dtype)
     if len(forms(device, dtype)) == 1:
         return

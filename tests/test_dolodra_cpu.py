@@ -31,7 +31,7 @@ def test_stream_and_activations():
     C.rope_case("cpu")
 
 
-@pytest.mark.parametrize("case", ["side_case", "input_conv_case", "window_edge_case", "sink_case", "batch_latent_case",
+@pytest.mark.parametrize("case", ["side_case", "norm_conv_case", "input_conv_case", "window_edge_case", "sink_case", "batch_latent_case",
                                   "latent_odd_case", "head_project_case"])
 def test_mechanisms(case):
     getattr(C, case)("cpu", F32)

@@ -29,7 +29,7 @@ def test_stream_and_activations():
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("case", ["side_case", "input_conv_case", "head_project_case", "latent_case", "latent_odd_case",
+@pytest.mark.parametrize("case", ["side_case", "norm_conv_case", "input_conv_case", "head_project_case", "latent_case", "latent_odd_case",
                                   "window_edge_case", "sink_case", "batch_latent_case"])
 def test_mechanisms(case, dtype):
     getattr(C, case)("cuda", dtype)
