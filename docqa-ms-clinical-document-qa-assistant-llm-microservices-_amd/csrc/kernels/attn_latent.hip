@@ -159,20 +159,15 @@ __global__ __launch_bounds__(256) void head_project_kernel(const uint16_t* __res
   const int per = kp / 8;
   if constexpr (MERGE) {
     const size_t all = (size_t)T * H;
-    for (int i = tid; i < 16 * MT; i += 256) {
+    static_assert(kMaxSplit == 32, "a row's splits in 32 lanes");
+    for (int i = tid >> 5; i < 16 * MT; i += 8) {
       const size_t row = (size_t)min(m0 + i, T - 1) * H + h;
-      float m = -1e30f, l = 0.f;
-#pragma unroll 8
-      for (int s = 0; s < nsplit; ++s) m = fmaxf(m, ml[s * all + row].x);
-#pragma unroll 8
-      for (int s = 0; s < nsplit; ++s) {
-        const float2 v = ml[s * all + row];
-        const float e = v.y > 0.f ? __builtin_amdgcn_exp2f(v.x - m) * v.y : 0.f;     // 0: nothing seen, nothing written
-        sw[i][s] = e;
-        l += e;
-      }
-      const float inv = l > 0.f ? 1.f / l : 0.f;
-      for (int s = 0; s < nsplit; ++s) sw[i][s] *= inv;
+      const int s = tid & 31;
+      const float2 v = s < nsplit ? ml[s * all + row] : make_float2(-1e30f, 0.f);
+      const float m = group_max<32>(v.x);
+      const float e = v.y > 0.f ? __builtin_amdgcn_exp2f(v.x - m) * v.y : 0.f;       // 0: nothing seen, nothing written
+      const float l = group_sum<32>(e);
+      sw[i][s] = l > 0.f ? e / l : 0.f;
     }
     __syncthreads();
     for (int i = tid; i < 16 * MT * per; i += 256) {
@@ -180,13 +175,16 @@ __global__ __launch_bounds__(256) void head_project_kernel(const uint16_t* __res
       float f[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
       if (m0 + r < T && c < K) {
         const uint16_t* p = part + ((size_t)(m0 + r) * H + h) * K + c;
-#pragma unroll 4
-        for (int s = 0; s < nsplit; ++s) {
-          const float e = sw[r][s];
-          float g[8];
-          ldv<8>(p + s * all * K, g);
+        for (int s0 = 0; s0 < nsplit; s0 += 4) {         // four at a time: past the last, weight 0
+          float g[4][8];
 #pragma unroll
-          for (int j = 0; j < 8; ++j) f[j] += e > 0.f ? e * g[j] : 0.f;        // (not written: any bits)
+          for (int u = 0; u < 4; ++u) ldv<8>(p + min(s0 + u, nsplit - 1) * all * K, g[u]);
+#pragma unroll
+          for (int u = 0; u < 4; ++u) {
+            const float e = sw[r][s0 + u];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) f[j] += e > 0.f ? e * g[u][j] : 0.f;   // (not written: any bits)
+          }
         }
       }
       stv<8>(sx + r * pitch + c, f);
@@ -298,11 +296,14 @@ struct LatentArgs {
 // grid (row tiles, sequences, key splits)
 template <int DPV, int DPK, int QT, int NW>
 __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
-  constexpr int PITCH = DPK + 8, NCH = DPK / 8, NKS = DPK / 32, RW = 16 * QT, PP = KB + 8;
-  constexpr int CPT = NCH / NW;                // 16-byte pieces of a tile a thread stages
+  constexpr int PITCH = DPK + 8, NKS = DPK / 32, RW = 16 * QT, PP = KB + 8;
+  // a tile's 16-byte pieces: the first DPV columns a wave takes RPI rows at a time, the other 64
+  // eight rows at a time
+  static_assert(DPK == DPV + 64, "row layout");
+  constexpr int LPR = DPV / 8, RPI = 64 / LPR, NL = KB / RPI / NW, NE = KB / 8 / NW;
   constexpr int QTW = QT / (NW / 4);           // row tiles whose scores this wave makes
   constexpr int NDT = DPV / 16 / NW;           // 16-column tiles of its slice of the output
-  static_assert(NW % 4 == 0 && QTW >= 1 && NDT >= 1 && NCH % NW == 0, "wave roles");
+  static_assert(NW % 4 == 0 && QTW >= 1 && NDT >= 1 && LPR <= 64 && NL >= 1 && NE >= 1, "wave roles");
   extern __shared__ __attribute__((aligned(16))) char smem[];
   uint16_t* tiles = reinterpret_cast<uint16_t*>(smem);                  // [2][KB][PITCH]
   uint16_t* sp = tiles + 2 * KB * PITCH;                                // [RW][PP]
@@ -310,7 +311,8 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
   __shared__ int s_bt[kMaxBT];
 
   const int b = blockIdx.y, split = blockIdx.z;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
+  const int tid = threadIdx.x, lane = tid & 63, fr = lane & 15, g4 = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   int q0, L, p0;
   if (a.cu) {
     q0 = a.cu[b];
@@ -354,8 +356,13 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
   // Every load of a tile issues without a branch: keys past the end repeat the last one (their
   // scores are masked), columns past the row repeat its first (the query is zero there, the
   // output is dropped).
-  u32x4 rk[CPT];
-  auto load = [&](int t) {
+  const int lrow = lane / LPR, c0 = (lane % LPR) * 8, cl = c0 < a.D ? c0 : 0;       // first columns
+  const int erow = lane >> 3, e0 = DPV + (lane & 7) * 8, ce = e0 < a.D ? e0 : 0;    // the others
+  auto cached = [&](int key) {                           // element offset of a key's row
+    const int blk = s_bt[(key >> a.log2BS) - blk0];
+    return (((size_t)blk << a.log2BS) + (key & ((1 << a.log2BS) - 1))) * a.D;
+  };
+  auto load = [&](int t, u32x4 (&rk)[NL + NE]) {
     const int kb = key0 + t * KB;
     if ((min(kb + KB - 1, last) >> a.log2BS) - blk0 >= kMaxBT) {       // the whole workgroup
       lds_barrier();
@@ -363,21 +370,50 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
       stage_blocks();
     }
 #pragma unroll
-    for (int i = 0; i < CPT; ++i) {
-      const int e = tid + 64 * NW * i, c0 = (e % NCH) * 8, c = c0 < a.D ? c0 : 0, key = min(kb + e / NCH, last);
-      const int blk = s_bt[(key >> a.log2BS) - blk0];
-      rk[i] = *reinterpret_cast<const u32x4*>(a.kc + (((size_t)blk << a.log2BS) + (key & ((1 << a.log2BS) - 1))) * a.D + c);
-    }
+    for (int i = 0; i < NL; ++i)
+      rk[i] = *reinterpret_cast<const u32x4*>(a.kc + cached(min(kb + (i * NW + wave) * RPI + lrow, last)) + cl);
+#pragma unroll
+    for (int i = 0; i < NE; ++i)
+      rk[NL + i] = *reinterpret_cast<const u32x4*>(a.kc + cached(min(kb + (i * NW + wave) * 8 + erow, last)) + ce);
   };
-  auto store = [&](int buf) {
+  auto store = [&](int buf, const u32x4 (&rk)[NL + NE]) {
     uint16_t* k = tiles + buf * KB * PITCH;
 #pragma unroll
-    for (int i = 0; i < CPT; ++i) {
-      const int e = tid + 64 * NW * i, row = e / NCH, c = (e % NCH) * 8;
-      *reinterpret_cast<u32x4*>(k + row * PITCH + c) = rk[i];
-    }
+    for (int i = 0; i < NL; ++i)
+      *reinterpret_cast<u32x4*>(k + ((i * NW + wave) * RPI + lrow) * PITCH + c0) = rk[i];
+#pragma unroll
+    for (int i = 0; i < NE; ++i)
+      *reinterpret_cast<u32x4*>(k + ((i * NW + wave) * 8 + erow) * PITCH + e0) = rk[NL + i];
   };
-  load(t0);
+  // the query rows come through LDS (a wave's fragments are 16 rows wide: read directly, every wave
+  // of a row tile would fetch 16 cache lines an instruction)
+  constexpr int QL = (RW + RPI * NW - 1) / (RPI * NW), QE = (RW + 8 * NW - 1) / (8 * NW);
+  u32x4 rq[QL + QE], rk[NL + NE], rk2[NL + NE];
+  const u32x4 zero = {0, 0, 0, 0};
+#pragma unroll
+  for (int i = 0; i < QL; ++i) {
+    const int r = min(row0 + (i * NW + wave) * RPI + lrow, rows - 1);
+    rq[i] = *reinterpret_cast<const u32x4*>(a.q + (grow0 + r) * a.D + cl);
+  }
+#pragma unroll
+  for (int i = 0; i < QE; ++i) {
+    const int r = min(row0 + (i * NW + wave) * 8 + erow, rows - 1);
+    rq[QL + i] = *reinterpret_cast<const u32x4*>(a.q + (grow0 + r) * a.D + ce);
+  }
+  load(t0, rk);
+  if (t0 + 1 < t1) load(t0 + 1, rk2);
+  uint16_t* sq = tiles + KB * PITCH;                     // [RW][PITCH], where tile t0 + 1 goes next
+#pragma unroll
+  for (int i = 0; i < QL; ++i) {
+    const int r = (i * NW + wave) * RPI + lrow;
+    if (r < RW) *reinterpret_cast<u32x4*>(sq + r * PITCH + c0) = c0 < a.D ? rq[i] : zero;
+  }
+#pragma unroll
+  for (int i = 0; i < QE; ++i) {
+    const int r = (i * NW + wave) * 8 + erow;
+    if (r < RW) *reinterpret_cast<u32x4*>(sq + r * PITCH + e0) = e0 < a.D ? rq[QL + i] : zero;
+  }
+  lds_barrier();
 
   const int ksub = wave & 3, rg = (wave >> 2) * QTW;     // this wave's keys of a tile / first row tile
   bf16x8 qf[QTW][NKS];
@@ -387,15 +423,11 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
     const int r = min(row0 + (rg + t) * 16 + fr, rows - 1);
     pos[t] = p0 + r / a.H;
     below[t] = a.window > 0 ? pos[t] - a.window : -1;
-    const uint16_t* qp = a.q + (grow0 + r) * a.D;
 #pragma unroll
-    for (int ks = 0; ks < NKS; ++ks) {
-      const int c = ks * 32 + g4 * 8;
-      uint4 v = *reinterpret_cast<const uint4*>(qp + (c < a.D ? c : 0));
-      if (c >= a.D) v = make_uint4(0, 0, 0, 0);
-      qf[t][ks] = *reinterpret_cast<bf16x8*>(&v);
-    }
+    for (int ks = 0; ks < NKS; ++ks)
+      qf[t][ks] = *reinterpret_cast<const bf16x8*>(sq + ((rg + t) * 16 + fr) * PITCH + ks * 32 + g4 * 8);
   }
+  lds_barrier();
   // the sink is the sum's first term: the maximum starts there in every wave, the sum in one
   float m[QT], l[QTW];
   f32x4 o[QT][NDT];
@@ -411,8 +443,10 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
   const float sl2 = a.scale * kLog2e;
   const int tq = fr >> 2, tp = fr & 3;
 
-  store(0);
-  load(min(t0 + 1, t1 - 1));                             // in flight for a whole tile's work
+  store(0, rk);
+  if (t0 + 1 < t1) store(1, rk2);
+  u32x4 rn[NL + NE];                                     // the tile after next, in flight for a tile's work
+  if (t0 + 2 < t1) load(t0 + 2, rn);
   lds_barrier();
   for (int t = t0; t < t1; ++t) {
     const int buf = (t - t0) & 1, kb = key0 + t * KB;
@@ -463,8 +497,8 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_kernel(LatentArgs a) {
       l[i] = l[i] * al + rs;
       stv<4>(sp + ((rg + i) * 16 + fr) * PP + ksub * 16 + g4 * 4, p);
     }
-    if (t + 1 < t1) store(buf ^ 1);
-    if (t + 2 < t1) load(t + 2);
+    if (t > t0 && t + 1 < t1) store(buf ^ 1, rn);
+    if (t > t0 && t + 2 < t1) load(t + 2, rn);
     lds_barrier();                                       // scores, next tile
 #pragma unroll
     for (int i = 0; i < QT; ++i)
@@ -527,7 +561,7 @@ template <int DPV, int QT, int NW>
 int launch_latent(const LatentArgs& a, int B, int max_q, hipStream_t s) {
   constexpr int DPK = DPV + 64, RW = 16 * QT;
   constexpr size_t lds = (size_t)2 * KB * (DPK + 8) * 2 + (size_t)RW * (KB + 8) * 2 + (size_t)4 * RW * 4;
-  static_assert(lds + kMaxBT * 4 <= 160 * 1024, "LDS");
+  static_assert(lds + kMaxBT * 4 <= 160 * 1024 && RW <= KB, "LDS");
   const long long nz = ((long long)max_q * a.H + RW - 1) / RW;
   if (nz >= (1ll << 31) || B > 65535) return -1;
   auto kern = latent_attn_kernel<DPV, DPK, QT, NW>;

@@ -13,11 +13,16 @@
 using namespace docqa;
 
 namespace {
+// over a workgroup of NT threads
+template <int NT = 256>
 __device__ __forceinline__ float block_sum(float v, float* red) {
   v = wave_sum(v);
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
   __syncthreads();
-  return red[0] + red[1] + red[2] + red[3];
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < NT / 64; ++i) s += red[i];
+  return s;
 }
 
 // one new token a row, an input convolution behind the norm: out2 = h + conv(h), the identity in
@@ -33,15 +38,16 @@ struct ConvArgs {
 };
 
 // CONV: 0 none, taps of 2 to 4 with the state's rows loaded ahead of the reductions, -1 any taps
-template <int NV, int V, typename PT, typename OT, int CONV = 0>
-__global__ __launch_bounds__(256) void sandwich_rmsnorm_kernel(const PT* __restrict__ P, int S, size_t slab,
+// NT threads a row: 256, or 1024 where rows are few and wide
+template <int NT, int NV, int V, typename PT, typename OT, int CONV = 0>
+__global__ __launch_bounds__(NT) void sandwich_rmsnorm_kernel(const PT* __restrict__ P, int S, size_t slab,
                                                                float* __restrict__ res,
                                                                const float* __restrict__ w_post,
                                                                const float* __restrict__ add,
                                                                const float* __restrict__ w_next,
                                                                OT* __restrict__ out, int H, float eps,
                                                                ConvArgs<OT> cv) {
-  __shared__ float red[2][4];
+  __shared__ float red[2][NT / 64];
   const size_t row = blockIdx.x;
   const int tid = threadIdx.x, n = H / V;
   float y[NV][V], x[NV][V];
@@ -55,7 +61,7 @@ __global__ __launch_bounds__(256) void sandwich_rmsnorm_kernel(const PT* __restr
     for (int i = 0; i < NV; ++i)
 #pragma unroll
       for (int k = 0; k < NS; ++k) {
-        const int c = min(tid + 256 * i, n - 1);
+        const int c = min(tid + NT * i, n - 1);
         ldv<V>(sp + (size_t)k * H + c * V, st[i][k]);
 #pragma unroll
         for (int j = 0; j < V; ++j) st[i][k][j] = carry ? st[i][k][j] : 0.f;
@@ -64,7 +70,7 @@ __global__ __launch_bounds__(256) void sandwich_rmsnorm_kernel(const PT* __restr
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = tid + 256 * i;
+    const int c = tid + NT * i;
     if (c < n) {
       ld_slabs<V>(P + row * H + c * V, S, slab, y[i]);
       ldv<V>(res + row * H + c * V, x[i]);
@@ -72,11 +78,11 @@ __global__ __launch_bounds__(256) void sandwich_rmsnorm_kernel(const PT* __restr
       for (int j = 0; j < V; ++j) ss += y[i][j] * y[i][j];
     }
   }
-  const float iy = 1.f / sqrtf(block_sum(ss, red[0]) / (float)H + eps);
+  const float iy = 1.f / sqrtf(block_sum<NT>(ss, red[0]) / (float)H + eps);
   ss = 0.f;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = tid + 256 * i;
+    const int c = tid + NT * i;
     if (c < n) {
       float g[V], a[V];
       ldv<V>(w_post + c * V, g);
@@ -90,10 +96,10 @@ __global__ __launch_bounds__(256) void sandwich_rmsnorm_kernel(const PT* __restr
       stv<V>(res + row * H + c * V, x[i]);
     }
   }
-  const float ix = 1.f / sqrtf(block_sum(ss, red[1]) / (float)H + eps);
+  const float ix = 1.f / sqrtf(block_sum<NT>(ss, red[1]) / (float)H + eps);
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = tid + 256 * i;
+    const int c = tid + NT * i;
     if (c < n) {
       float g[V], o[V];
       ldv<V>(w_next + c * V, g);
@@ -231,7 +237,17 @@ int launch_sandwich(const PT* P, int S, float* res, const float* w_post, const f
   const size_t slab = (size_t)rows * H;
   const int nv = (H / V + 255) / 256;
   const ConvArgs<OT> none{};
-#define LAUNCH(N, C) sandwich_rmsnorm_kernel<N, V, PT, OT, (C)><<<rows, 256, 0, s>>>(P, S, slab, res, w_post, add, w_next, out, H, eps, cv ? *cv : none)
+#define LAUNCH(N, C)                                                                                                   \
+  do {                                                                                                                 \
+    if (V > 1 && rows <= 512 && N >= 4) {                                                                              \
+      constexpr int NW = N >= 4 ? N / 4 : 1;                                                                           \
+      sandwich_rmsnorm_kernel<1024, NW, V, PT, OT, (C)><<<rows, 1024, 0, s>>>(P, S, slab, res, w_post, add, w_next,    \
+                                                                              out, H, eps, cv ? *cv : none);           \
+    } else {                                                                                                           \
+      sandwich_rmsnorm_kernel<256, N, V, PT, OT, (C)><<<rows, 256, 0, s>>>(P, S, slab, res, w_post, add, w_next, out,  \
+                                                                           H, eps, cv ? *cv : none);                   \
+    }                                                                                                                  \
+  } while (0)
 #define GO(N)                                                      \
   do {                                                             \
     const int taps = cv ? cv->taps : 0;                            \

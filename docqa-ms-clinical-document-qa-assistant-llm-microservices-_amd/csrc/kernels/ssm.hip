@@ -41,7 +41,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
   // then replaces) a sequence's state
   static_assert(K <= 0 || TT >= K - 1, "tokens per thread");
   const int tt = K > 0 ? TT : max(TT, nt - 1);
-  const int t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * tt;
+  const int t0 = (blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6)) * tt;
   const int c0 = (blockIdx.x * 64 + (threadIdx.x & 63)) * V;
   if (t0 >= L || c0 >= C) return;
   const bool carry = ctx[b] > 0 && slots[b] >= 0;
@@ -62,8 +62,13 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
   };
   if constexpr (K > 0) {
     float wv[K][V], in[TT + K - 1][V];      // inputs t0 - (K - 1) .. t0 + TT - 1, all in flight at once
+    if (t0 >= K - 1) {                      // whole waves: nothing carried, no branch between the loads
 #pragma unroll
-    for (int i = 0; i < TT + K - 1; ++i) input(min(t0 + i - (K - 1), L - 1), in[i]);
+      for (int i = 0; i < TT + K - 1; ++i) ldv<V>(x + (size_t)(q0 + min(t0 + i - (K - 1), L - 1)) * ldx + c0, in[i]);
+    } else {
+#pragma unroll
+      for (int i = 0; i < TT + K - 1; ++i) input(min(t0 + i - (K - 1), L - 1), in[i]);
+    }
 #pragma unroll
     for (int k = 0; k < K; ++k) ldv<V>(w + (size_t)k * C + c0, wv[k]);
 #pragma unroll
@@ -437,7 +442,7 @@ int launch_conv(const void* x, int ldx, const float* w, const float* b, void* st
                 const int* ctx, void* y, int B, int max_len, int C, int taps, int silu, hipStream_t s) {
   const int gx = (C + 64 * V - 1) / (64 * V);
   // 8 tokens a thread; fewer where that leaves most of the chip without a workgroup
-  const bool few = (long long)gx * ((max_len + 31) / 32) * B < 1024;
+  const bool few = (long long)gx * ((max_len + 31) / 32) * B < 512;
 #define LAUNCH(K, TT, tt)                                                                                   \
   causal_conv_kernel<T, V, K, TT><<<dim3(gx, (max_len + 4 * (tt)-1) / (4 * (tt)), B), 256, 0, s>>>(         \
       (const T*)x, ldx, w, b, (T*)state, slots, cu, ctx, (T*)y, C, taps, silu)

@@ -195,8 +195,10 @@ class HybridConfig:
         return sum(math.prod(s) for s in self.tensor_shapes().values())
 
 
-# decode rows up to which a captured step runs a parallel layer's sublayers as two graph branches
-FORK_MAX_ROWS = int(os.environ.get("DOCQA_FORK_MAX_ROWS", "64"))
+# Feed-forward weights from which a captured decode step runs a parallel layer's sublayers as two
+# branches of the graph: 352 MB (width 4096, ff 21504) 1.07 -> 0.98 ms a step of 8 layers at batch 1,
+# 1.92 -> 1.69 at 64, 2.52 -> 2.47 at 256; 100 MB lose 6 % at batch 1 to 16
+FORK_MIN_BYTES = int(os.environ.get("DOCQA_FORK_MIN_MB", "192")) << 20
 
 
 def _pad_up(n: int, m: int) -> int:
@@ -418,6 +420,7 @@ class MLP:
         self.up = get("up").to(dtype).contiguous()
         self.down = get("down").to(dtype).contiguous()
         self.act = act
+        self.nbytes = 2 * self.up.numel() * self.up.element_size()
 
     def run(self, x, decode):
         return ops.project(ops.act_linear(x, self.up, self.act, decode), self.down, decode)
@@ -458,7 +461,7 @@ class SideInput:
         self.col, self.n = col, n
 
     def run(self, x, ids, table, decode):
-        return ops.side_project(ops.project(x, self.gate, decode), ids, table, self.col, self.n, self.proj, decode)
+        return ops.side_project(ops.narrow_project(x, self.gate, decode), ids, table, self.col, self.n, self.proj, decode)
 
 
 class HybridModel(Decoder):
@@ -629,7 +632,7 @@ class HybridModel(Decoder):
         two weight-streaming ones."""
         if L["mlp"] is None:
             return L["mixer"].run(hm, parts, slot_mapping, cache, decode, fw), None
-        fork = (decode and h.is_cuda and h.shape[0] <= FORK_MAX_ROWS and torch.cuda.is_current_stream_capturing())
+        fork = (decode and h.is_cuda and L["mlp"].nbytes >= FORK_MIN_BYTES and torch.cuda.is_current_stream_capturing())
         if not fork:
             return L["mixer"].run(hm, parts, slot_mapping, cache, decode, fw), L["mlp"].run(h, decode)
         if self._side_stream is None:

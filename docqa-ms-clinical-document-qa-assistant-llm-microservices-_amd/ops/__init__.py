@@ -1284,20 +1284,37 @@ def side_gate(P, ids, table, col: int, n: int, out_dtype=torch.bfloat16):
 
 
 def side_project(P, ids, table, col: int, n: int, w, decode: bool = False):
-    """:func:`side_gate` of the gate projection ``P``, projected by ``w``: one launch for a few
-    bf16 rows, where every workgroup builds their gate itself; else two."""
-    if _gpu(P) and w.dtype == torch.bfloat16 and w.shape[1] <= 1024:
-        if P.shape[-2] <= SIDE_FUSED_MAX:
+    """:func:`side_gate` of the gate projection ``P``, projected by ``w`` [W, N]: one launch for a
+    few bf16 rows, where every workgroup builds their gate itself; else two, the product on the
+    kernels that take its short K: :func:`head_project` up to 64 rows (3.5 us at W 4096, N 256),
+    the 128 x 128 GEMM beyond (512 rows 6.3 us; 4096 rows 17.5, the 256 x 256 one 16.9)."""
+    M, N = P.shape[-2], P.shape[-1]
+    if _gpu(P) and w.dtype == torch.bfloat16 and N <= 1024:
+        if M <= SIDE_FUSED_MAX:
             return _native().side_project(P.contiguous(), ids, table, int(col), int(n), w)
         g = side_gate(P, ids, table, col, n, w.dtype)
-        if P.shape[-2] <= SIDE_HEAD_MAX:
+        if M <= 64 or w.shape[0] % 128 or N % 64:
             return head_project(g, w[None])
-        return project(g, w, decode)
+        return _native().gemm(g, w, None, None, EPI_NONE)
     return project(side_gate(P, ids, table, col, n, w.dtype), w, decode)
 
 
-SIDE_FUSED_MAX = int(os.environ.get("DOCQA_SIDE_FUSED_MAX", "16"))
-SIDE_HEAD_MAX = int(os.environ.get("DOCQA_SIDE_HEAD_MAX", "512"))
+SIDE_FUSED_MAX = 8      # rows; at 8 the two launches take the same 6.3 us
+
+
+def narrow_project(x, w, decode: bool = False):
+    """:func:`project` for few outputs (N <= 512) of many rows: K split until the mid-M kernel's
+    256-row tiles fill the chip, bf16 slabs (N 256, K 4096: 4096 rows 15.8 us against 25.6 on
+    :func:`prefill_split_plan`, 2048 rows 10.4 / 23.2, 1024 rows 7.9 / 22.4)."""
+    N, K = w.shape
+    M = x.numel() // K
+    if _gpu(x) and x.dtype == torch.bfloat16 and not decode and M > MID_M_MAX and N % 128 == 0 and K % 128 == 0 and N <= 512:
+        mt, kb = (M + 255) // 256, K // 128
+        for width, cfg in ((64, 7), (128, 2)):
+            S = max((s for s in (2, 4, 8, 16) if kb % s == 0 and mt * (N // width) * s <= 256), default=1)
+            if S >= 4 or (cfg == 2 and S >= 2):
+                return mgemm_partial(x, w, S, cfg, bf16=True)
+    return project(x, w, decode)
 
 
 def soft_cap(x, cap: float):

@@ -77,8 +77,44 @@ def test_graph_replays_match_eager_steps(dtype):
     assert any(g.graph is not None for g in eng._graphs.values())
 
 
+def test_two_branch_steps_match(monkeypatch):
+    """A captured step whose layers run mixer and feed-forward as two graph branches, replayed with
+    eager work in between, gives the eager steps' tokens."""
+    from docqa_amd.models import hybrid
+
+    monkeypatch.setattr(hybrid, "FORK_MIN_BYTES", 0)
+    js, w, m = C.make("mixed", "cuda", torch.bfloat16, seed=41)
+    prompts = [C.toks(n, js["vocab"], n) for n in (9, 30, 17)]
+    sp = C.SamplingParams(max_new_tokens=25)
+    eager = C.engine(m, tokens=512, slots=4).generate(prompts, sp)
+    eng = C.engine(m, tokens=512, slots=4, use_graphs=True)
+    for _ in range(3):
+        assert eng.generate(prompts, sp) == eager
+        torch.cuda.synchronize()
+    assert m._side_stream is not None
+
+
 WIDE = C.conf(1024, 2048, [C.lat(16, 128, 64, 128, 512, 96, ff=4096), C.lat(32, 64, 64, 64, 512, 200, ff=2048, kv_from=0)],
               4, 256, 0.5, 30.0)
+
+
+def test_narrow_products():
+    """Few outputs of many rows (K split over bf16 slabs), and the short-K product behind the side
+    gate at the row counts where its kernel changes."""
+    from docqa_amd import ops
+
+    g = torch.Generator().manual_seed(1)
+    for M, N, K in ((600, 256, 512), (1024, 128, 4096), (2100, 256, 1024), (5000, 512, 256), (700, 64, 320)):
+        x, w = torch.randn(M, K, generator=g), torch.randn(N, K, generator=g) * K ** -0.5
+        P = ops.narrow_project(x.to("cuda", torch.bfloat16), w.to("cuda", torch.bfloat16))
+        C.close(P.float().sum(0) if P.dim() == 3 else P, x.to(torch.bfloat16).float() @ w.to(torch.bfloat16).float().T,
+                torch.bfloat16, (M, N, K))
+    for M in (8, 9, 64, 65, 300):
+        P, w = torch.randn(M, 64, generator=g), (torch.randn(256, 64, generator=g) / 8).to(torch.bfloat16)
+        table, ids = torch.randn(9, 100, generator=g).to(torch.bfloat16), torch.randint(0, 9, (M,), generator=g, dtype=torch.int32)
+        gate = C.O.gelu_tanh(P.to(torch.bfloat16).float()[:, :60]) * table[ids.long(), 40:].float()
+        y = ops.side_project(P.to("cuda", torch.bfloat16), ids.cuda(), table.cuda(), 40, 60, w.cuda(), True)
+        C.close(y, gate @ w[:, :60].float().T, torch.bfloat16, M)
 
 
 @pytest.mark.parametrize("rows", [1, 3, 40, 200])
