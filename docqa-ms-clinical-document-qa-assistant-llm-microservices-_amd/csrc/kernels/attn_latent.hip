@@ -657,7 +657,6 @@ int docqa_head_project(const void* x, const void* part, const void* ml, int nspl
   } while (0)
   if (T > 64 && K <= 256) GO(4, 2);
   else if (T > 64 && K <= 1024) GO(2, 2);
-  else if (T > 16 && part && N > 64) GO(1, 2);           // one workgroup sums a row's splits
   else GO(1, 1);
 #undef GO
 #undef LAUNCH

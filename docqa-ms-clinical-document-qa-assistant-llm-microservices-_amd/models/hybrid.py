@@ -137,7 +137,7 @@ class HybridConfig:
         for i, sp in enumerate(self.layer_specs):
             m = sp.mixer
             if isinstance(m, LatentAttentionSpec):
-                if m.rot_dim % 2 or m.window < 1 or m.kv_rank > 2048 or min(m.heads, m.dim, m.vdim, m.kv_rank, m.rot_dim) < 1:
+                if m.rot_dim % 2 or m.window < 1 or max(m.kv_rank, m.dim) > 2048 or min(m.heads, m.dim, m.vdim, m.kv_rank, m.rot_dim) < 1:
                     raise ValueError(f"unsupported attention sizes {m}")
                 if m.kv_from is not None:
                     src = self.layer_specs[m.kv_from].mixer if 0 <= m.kv_from < i else None

@@ -1238,7 +1238,9 @@ def squared_relu(P, out_dtype=torch.bfloat16):
     return activation(P, ACT_RELU2, out_dtype)
 
 
-_PGEMM_ACT_TILES = int(os.environ.get("DOCQA_PGEMM_ACT_TILES", "96"))
+# 256 x 256 tiles from which a 257..512-row prompt's activation runs in that GEMM's epilogue
+# (512 x 21504 x 4096: 95 us, the mid-M kernel 136)
+_PGEMM_ACT_TILES = 96
 
 
 def act_linear(x, w, act: str, decode: bool = False):
