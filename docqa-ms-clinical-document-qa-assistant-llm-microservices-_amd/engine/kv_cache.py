@@ -24,15 +24,18 @@ import torch
 class KVSpec:
     """One layer's paged cache.  ``shared``: the key rows are the values too -- one tensor,
     with an fp32 scale per row in place of V (ops.qk_norm_store); ``latent``: one tensor of
-    rows that keys and values are made from (ops.latent_store), no V."""
+    rows that keys and values are made from (ops.latent_store), no V; ``v_dim``: size of a value
+    row, if not the key's."""
     kv_heads: int
     head_dim: int
     shared: bool = False
     latent: bool = False
+    v_dim: int = 0
 
     def bytes_per_token(self, dtype_bytes: int) -> int:
         row = self.head_dim * dtype_bytes
-        return self.kv_heads * (row if self.latent else row + 4 if self.shared else 2 * row)
+        return self.kv_heads * (row if self.latent else row + 4 if self.shared
+                                else row + (self.v_dim or self.head_dim) * dtype_bytes)
 
 
 @dataclass(frozen=True)
@@ -106,7 +109,7 @@ class KVCache:
             k = torch.zeros(shape, device=device, dtype=dtype)
             self.caches.append((k, None if sp.latent
                                 else torch.zeros(shape[:3], device=device, dtype=torch.float32) if sp.shared
-                                else torch.zeros_like(k)))
+                                else torch.zeros((*shape[:3], sp.v_dim or sp.head_dim), device=device, dtype=dtype)))
         self.allocator = make_allocator(num_blocks, block_size)
 
     @staticmethod

@@ -1,10 +1,12 @@
-"""Decoders made of windowed attention, latent attention and recurrent (selective-scan)
+"""Decoders made of attention, latent attention and recurrent (selective-scan, linear-attention)
 mixers, with an fp32 residual stream.
 
 A model is a list of layers (:class:`LayerSpec`: a mixer and an optional feed-forward) in one
-of two forms: a norm before and after every sublayer, one after the other, or -- with a
-:class:`ParallelForm` -- one norm whose output both sublayers read, a convolution over time
-ahead of the mixer and a second input from the token's side embedding.  Layers may run
+of three forms: a norm before and after every sublayer, one after the other; with a
+:class:`ParallelForm` one norm whose output both sublayers read, a convolution over time
+ahead of the mixer and a second input from the token's side embedding; with a
+:class:`PostNormForm` sublayers that read the stream itself, their gated results added to it and
+the sum normed.  Layers may run
 several passes over the same weights (``loop``).  Every RUN of a layer has its own cache or
 state, so the engine sees as many caches as runs; a latent-attention layer may read the cache
 of an earlier one (``kv_from``) instead.
@@ -23,6 +25,14 @@ MI355X layout:
     with the key / value projections absorbed into the query and the output (decode, short
     portions: the cached row is key and value), or with keys and values of the visible rows
     made once by a GEMM (prompts);
+  * a linear-attention recurrence keeps one [key, value] matrix a head in fp32: decode is one launch
+    from the projection's slabs to the gated heads, prompts run in chunks on fp32 MFMA; a mixer of
+    two sides has one input projection, both sides write their part of one matrix, and one product
+    projects it;
+  * experts run as a grouped GEMM over (token, choice) rows sorted by expert (prompts), or one
+    weight-streaming launch per projection that finds its rows itself (decode);
+  * the post-norm form's gate rows are part of the sublayer's first projection, and one launch
+    gates, adds, norms and updates the residual;
   * the parallel form's stream update, side input, next norm and (decode) convolution step are
     two launches around the side input's two small projections;
   * projections run on the same GEMM plans as the Llama decoder (ops.project / ops.linear):
@@ -36,7 +46,7 @@ from __future__ import annotations
 import math
 import os
 import zlib
-from dataclasses import dataclass, field
+from dataclasses import dataclass, field, replace
 
 import torch
 
@@ -86,6 +96,106 @@ class LatentAttentionSpec:
 
 
 @dataclass(frozen=True)
+class Rotation:
+    """Rotary positions on a head's first ``dims`` dimensions, i paired with i + dims / 2.
+    ``scaling``: YaRN's (factor, original, fast, slow) -- frequencies that turn fewer than ``slow``
+    times in ``original`` tokens are divided by ``factor``, those beyond ``fast`` kept, a ramp
+    between."""
+    base: float
+    dims: int
+    scaling: tuple | None = None
+
+    def frequencies(self) -> tuple:
+        """(fp64 [dims / 2] angles per position, factor on cosines and sines)."""
+        r = self.dims
+        f = self.base ** (-torch.arange(0, r, 2, dtype=torch.float64) / r)
+        if self.scaling is None:
+            return f, 1.0
+        factor, original, fast, slow = self.scaling
+
+        def at(turns):
+            return r * math.log(original / (2 * math.pi * turns)) / (2 * math.log(self.base))
+
+        lo, hi = max(math.floor(at(fast)), 0), min(math.ceil(at(slow)), r - 1)
+        ramp = ((torch.arange(r // 2, dtype=torch.float64) - lo) / max(hi - lo, 1e-3)).clamp(0, 1)
+        return f / factor * ramp + f * (1 - ramp), 0.1 * math.log(factor) + 1
+
+
+@dataclass(frozen=True)
+class AttentionSpec:
+    """Causal attention with normed, rotated queries and keys (over the last ``window`` tokens, 0:
+    all), scores capped by ``softcap`` (0: not), biases on the projections where ``bias``."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot: Rotation
+    window: int = 0
+    softcap: float = 0.0
+    bias: bool = False
+
+
+@dataclass(frozen=True)
+class GatedLinearSpec:
+    """Gated linear attention: a decay sigmoid(z)^(1 / tau) per key channel, z a projection through
+    ``rank`` elements (0: as the checkpoint's tensor has it)."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    rank: int = 0
+
+
+@dataclass(frozen=True)
+class RetentionSpec:
+    """Linear attention with rotated queries and keys and a fixed decay per head."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+    rot: Rotation
+
+
+@dataclass(frozen=True)
+class GatedDeltaSpec:
+    """Gated delta rule: ``conv``-tap convolutions over q, k and v, unit q and k, the state's answer
+    to the key subtracted from the value before it is written; ``heads`` share ``kv_heads`` q / k."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+
+
+@dataclass(frozen=True)
+class TwoSidedSpec:
+    """left_scale attention + right_scale linear attention of the same input."""
+    left: AttentionSpec
+    right: GatedLinearSpec | RetentionSpec
+    left_scale: float
+    right_scale: float
+
+
+@dataclass(frozen=True)
+class MoESpec:
+    """``top`` of ``experts`` SwiGLU feed-forwards of ``ff`` by sigmoid score, each reading the input
+    times its score, and one of ``shared`` (0: none) for every token times a gate."""
+    experts: int
+    top: int
+    ff: int
+    shared: int = 0
+
+
+@dataclass(frozen=True)
+class PostNormForm:
+    """Layers x <- norm(alpha x + sigmoid(W x + b) * sublayer(x)), the norm over ``groups`` equal
+    parts of x."""
+    alpha: float
+    groups: int
+
+
+@dataclass(frozen=True)
 class ParallelForm:
     """Layers x <- x + mult (mixer(h + conv(h)) + ff(h)), h = norm1(x), then
     x <- x + mult rms(proj(gelu(gate x) * e)) * norm with e the layer's part of the token's
@@ -97,8 +207,9 @@ class ParallelForm:
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: WindowAttentionSpec | SelectiveScanSpec | LatentAttentionSpec
+    mixer: WindowAttentionSpec | SelectiveScanSpec | LatentAttentionSpec | TwoSidedSpec | GatedDeltaSpec
     ff: int = 0                     # feed-forward width, 0: none
+    moe: MoESpec | None = None      # or experts (post-norm form)
 
 
 @dataclass
@@ -110,7 +221,8 @@ class HybridConfig:
     embed_scale: float = 1.0
     rms_eps: float = 1e-5
     loop: tuple | None = None       # (start, stop, times)
-    parallel: ParallelForm | None = None    # None: norms around every sublayer
+    parallel: ParallelForm | None = None    # neither: norms around every sublayer
+    post: PostNormForm | None = None
     act: str = ops.ACT_RELU2        # of the feed-forward
     norm_offset: float = 0.0        # added to the stored weights of the layers' and final norms
     logit_softcap: float | None = None
@@ -134,8 +246,16 @@ class HybridConfig:
                 raise ValueError("parallel layers: latent attention, no loop")
             if self.parallel.conv < 1 or self.parallel.side < 1:
                 raise ValueError(f"unsupported sizes {self.parallel}")
+        if self.post is not None:
+            if self.loop is not None or self.parallel is not None or self.hidden % self.post.groups:
+                raise ValueError("post-norm layers: groups that divide the width, no loop")
         for i, sp in enumerate(self.layer_specs):
             m = sp.mixer
+            if (self.post is not None) != isinstance(m, (TwoSidedSpec, GatedDeltaSpec)) or (sp.moe and self.post is None) or (
+                    sp.ff and self.post is not None):
+                raise ValueError("two-sided and delta mixers and experts run in post-norm layers")
+            if self.post is not None:
+                _check_post(sp)
             if isinstance(m, LatentAttentionSpec):
                 if m.rot_dim % 2 or m.window < 1 or max(m.kv_rank, m.dim) > 2048 or min(m.heads, m.dim, m.vdim, m.kv_rank, m.rot_dim) < 1:
                     raise ValueError(f"unsupported attention sizes {m}")
@@ -159,6 +279,11 @@ class HybridConfig:
         """Every weight's name and shape (linear weights [out, in])."""
         W, V = self.hidden, self.vocab_size
         out, par = {"embed": (V, W)}, self.parallel
+        if self.post is not None:
+            for i, sp in enumerate(self.layer_specs):
+                out.update(_post_shapes(sp, W, f"l{i}."))
+            out.update({"final.norm": (W,), "head": (V, W)})
+            return out
         if par is not None:
             out["side.embed"] = (V, self.layers * par.side)
         for i, sp in enumerate(self.layer_specs):
@@ -192,7 +317,71 @@ class HybridConfig:
         return out
 
     def num_params(self) -> int:
+        """(a size that only the checkpoint knows counts as nothing)"""
         return sum(math.prod(s) for s in self.tensor_shapes().values())
+
+
+def _check_post(sp: LayerSpec) -> None:
+    m = sp.mixer
+    sides = [m.left, m.right] if isinstance(m, TwoSidedSpec) else [m]
+    for s in sides:
+        if min(s.heads, s.dim, s.vdim) < 1 or s.heads % getattr(s, "kv_heads", 1):
+            raise ValueError(f"unsupported sizes {s}")
+        rot = getattr(s, "rot", None)
+        if rot is not None and (rot.dims % 2 or not 2 <= rot.dims <= s.dim):
+            raise ValueError(f"unsupported rotation {rot} of heads of {s.dim}")
+        if isinstance(s, AttentionSpec):
+            if s.dim > 512 or s.vdim > 512 or s.window < 0 or s.softcap < 0:
+                raise ValueError(f"unsupported attention sizes {s}")
+        elif s.dim > 256 or s.vdim > 512:
+            raise ValueError(f"unsupported state sizes {s}")
+        if isinstance(s, RetentionSpec) and (len(s.decay) != s.heads or not all(0 < d <= 1 for d in s.decay)):
+            raise ValueError(f"one decay in (0, 1] per head expected: {s.decay}")
+        if isinstance(s, GatedDeltaSpec) and s.conv < 1:
+            raise ValueError(f"unsupported sizes {s}")
+        if isinstance(s, GatedLinearSpec) and s.tau <= 0:
+            raise ValueError(f"unsupported sizes {s}")
+    if sp.moe is not None and not (1 <= sp.moe.top <= min(sp.moe.experts, 16) and sp.moe.ff >= 1 and sp.moe.shared >= 0
+                                   and sp.moe.experts <= 512):
+        raise ValueError(f"unsupported experts {sp.moe}")
+
+
+def _post_shapes(sp: LayerSpec, W: int, p: str) -> dict:
+    out, m = {p + "norm1": (W,), p + "rg1": (W, W), p + "rg1.b": (W,)}, sp.mixer
+
+    def linear(x, s):
+        kv = getattr(s, "kv_heads", s.heads)
+        out.update({x + "q": (kv * s.dim, W), x + "k": (kv * s.dim, W), x + "v": (s.heads * s.vdim, W),
+                    x + "g": (s.heads * s.vdim, W), x + "o": (W, s.heads * s.vdim)})
+
+    if isinstance(m, GatedDeltaSpec):
+        x = p + "mix."
+        linear(x, m)
+        out.update({x + "q.conv": (m.kv_heads * m.dim, m.conv), x + "k.conv": (m.kv_heads * m.dim, m.conv),
+                    x + "v.conv": (m.heads * m.vdim, m.conv), x + "b": (m.heads, W), x + "a": (m.heads, W),
+                    x + "A_log": (m.heads,), x + "dt_bias": (m.heads,), x + "norm": (m.vdim,)})
+    else:
+        x, s = p + "mix.left.", m.left
+        sizes = {"q": s.heads * s.dim, "k": s.kv_heads * s.dim, "v": s.kv_heads * s.vdim}
+        out.update({x + n: (r, W) for n, r in sizes.items()})
+        if s.bias:
+            out.update({f"{x}{n}.b": (r,) for n, r in sizes.items()})
+        out.update({x + "q.norm": (s.dim,), x + "k.norm": (s.dim,), x + "o": (W, s.heads * s.vdim)})
+        x, s = p + "mix.right.", m.right
+        linear(x, s)
+        if isinstance(s, GatedLinearSpec):
+            n = s.heads * s.dim
+            out.update({x + "norm": (s.vdim,), x + "a1": (s.rank, W), x + "a2": (n, s.rank), x + "a2.b": (n,)})
+    if sp.moe is not None:
+        x, f = p + "mlp.", sp.moe
+        out.update({p + "norm2": (W,), p + "rg2": (W, W), p + "rg2.b": (W,), x + "router": (f.experts, W)})
+        sizes = {f"e{e}.": f.ff for e in range(f.experts)}
+        if f.shared:
+            sizes["shared."] = f.shared
+            out[x + "shared.sg"] = (1, W)
+        for n, ff in sizes.items():
+            out.update({x + n + "gate": (ff, W), x + n + "up": (ff, W), x + n + "down": (W, ff)})
+    return out
 
 
 # Feed-forward weights from which a captured decode step runs a parallel layer's sublayers as two
@@ -426,6 +615,208 @@ class MLP:
         return ops.project(ops.act_linear(x, self.up, self.act, decode), self.down, decode)
 
 
+def _joint(rows: list, dtype) -> torch.Tensor:
+    """One weight of several projections of the same input, padded with zero rows to the GEMM granules."""
+    n = sum(t.shape[0] for t in rows)
+    pad = rows[0].new_zeros(_pad_up(n, 256 if n >= 1024 else 64) - n, rows[0].shape[1])
+    return torch.cat([*rows, pad]).to(dtype).contiguous()
+
+
+def _in_project(x, w, parts: list, decode: bool):
+    """A projection whose consumers take slabs, if one part has all of its rows, else the product."""
+    return ops.project(x, w, decode) if len(parts) == 1 else ops.linear(x, w, decode)
+
+
+class Attention:
+    """The attention side of a mixer: rows [q | k | v] of its input projection."""
+
+    def __init__(self, sp: AttentionSpec, get, eps: float, dtype, out_scale: float):
+        self.sp, self.eps, self.out_scale = sp, eps, out_scale
+        self.rows = [get(n) for n in "qkv"]
+        self.n = sum(t.shape[0] for t in self.rows)
+        self.bias = torch.cat([get(n + ".b") for n in "qkv"]).float().contiguous() if sp.bias else None
+        self.q_norm, self.k_norm = (get(n + ".norm").float().contiguous() for n in "qk")
+        self.o = get("o")
+
+    def cache_spec(self):
+        return KVSpec(self.sp.kv_heads, self.sp.dim, v_dim=self.sp.vdim)
+
+    def run(self, P, parts, slot_mapping, cache, fw, out):
+        sp = self.sp
+        kc, vc = cache
+        q = ops.qkv_rope_store(P, self.bias, self.q_norm, self.k_norm, fw.rope[sp.rot], slot_mapping, kc, vc, sp.heads, self.eps)
+        for p in parts:
+            m = p.meta
+            kw = dict(window=sp.window, v_cache=vc, cap=sp.softcap, out_scale=self.out_scale, out=_split(out, p, parts))
+            if p.decode:
+                ops.window_attn(_split(q, p, parts), kc, m.block_tables, m.context_lens, sp.scale, **kw)
+            else:
+                ops.window_attn(_split(q, p, parts), kc, m.block_tables, m.prefix_lens, sp.scale, cu=m.cu_seqlens,
+                                max_q=m.max_len, **kw)
+
+
+class LinearAttention:
+    """A linear-attention recurrence: rows [q | k | v | g | a | b] of its input projection, from
+    column ``at`` on."""
+
+    def __init__(self, sp, get, eps: float, dtype, at: int = 0, out_scale: float = 1.0):
+        self.sp, self.rot = sp, None
+        kv = getattr(sp, "kv_heads", sp.heads)
+        names, kw, self.b_gate = ["q", "k", "v", "g"], {}, None
+        norm = torch.ones(sp.vdim, device=get("o").device)
+        if isinstance(sp, GatedLinearSpec):
+            kind, norm = "channel", get("norm").float()
+            names.append("a1")
+            self.w_gate, self.b_gate = get("a2").float().contiguous(), get("a2.b").float().contiguous()
+            kw = dict(q_scale=sp.dim ** -0.5, inv_tau=1.0 / sp.tau, rank=self.w_gate.shape[1])
+        elif isinstance(sp, RetentionSpec):
+            kind, self.rot = "fixed", sp.rot
+            self.w_gate = torch.tensor(sp.decay, dtype=torch.float64).log().float().to(norm.device)
+            kw = dict(k_scale=sp.dim ** -0.5)
+        else:
+            kind, norm = "delta", get("norm").float()
+            names += ["a", "b"]
+            self.w_gate, self.b_gate = (-torch.exp(get("A_log").float())).contiguous(), get("dt_bias").float().contiguous()
+            kw = dict(q_scale=sp.dim ** -0.5)
+        self.norm = (norm * out_scale).contiguous()
+        self.rows = [get(n) for n in names]
+        cols = [at]
+        for t in self.rows:
+            cols.append(cols[-1] + t.shape[0])
+        self.n = cols[-1] - at
+        self.mix = ops.LinearMix(kind, sp.heads, kv, sp.dim, sp.vdim, *cols[:4], a=cols[4], b=cols[5] if kind == "delta" else 0,
+                                 eps=eps, **kw)
+        self.o = get("o")
+
+    def state_shape(self) -> tuple:
+        return ops.linear_state_shape(self.sp.heads, self.sp.dim, self.sp.vdim)
+
+    def cache_spec(self):
+        return StateSpec((self.state_shape(),), (True,))
+
+    def run_part(self, X, Z, mix, p: _Part, state, cs, out):
+        m = p.meta
+        a = (X, Z, mix, self.w_gate, self.b_gate, cs, self.norm, state, m.state_slots)
+        if p.decode:
+            ops.linear_step(*a, m.positions, out)
+        else:
+            ops.linear_scan(*a, m.cu_seqlens, m.prefix_lens, m.max_len, out)
+
+    def run(self, P, parts, state, fw, out):
+        for p in parts:
+            x = _split(P, p, parts)
+            cs = _split(fw.rope[self.rot], p, parts) if self.rot is not None else None
+            self.run_part(x, x, self.mix, p, state[0], cs, _split(out, p, parts))
+
+
+class TwoSidedMixer:
+    """Attention and linear attention of the same input, scaled and added: one input projection of
+    both sides (and the ``tail`` rows), one product of both results."""
+
+    def __init__(self, sp: TwoSidedSpec, get, eps: float, dtype, tail):
+        self.left = Attention(sp.left, lambda n: get("left." + n), eps, dtype, sp.left_scale)
+        self.right = LinearAttention(sp.right, lambda n: get("right." + n), eps, dtype, self.left.n, sp.right_scale)
+        self.tail = self.left.n + self.right.n
+        self.w_in = _joint(self.left.rows + self.right.rows + [tail], dtype)
+        self.split = self.left.o.shape[1]
+        self.o = torch.cat([self.left.o, self.right.o], 1).to(dtype).contiguous()
+        self.left.rows = self.right.rows = self.left.o = self.right.o = None
+
+    def rotations(self) -> set:
+        return {r for r in (self.left.sp.rot, self.right.rot) if r is not None}
+
+    def cache_specs(self) -> list:
+        return [self.left.cache_spec(), self.right.cache_spec()]
+
+    def activation_elems(self) -> int:
+        lf, r = self.left.sp, self.right.sp
+        return self.w_in.shape[0] + 2 * self.o.shape[1] + lf.heads * lf.dim + 2 * r.heads * (4 * r.dim + 2 * r.vdim + 64)
+
+    def run(self, x, parts, slot_mapping, cache, decode, fw: _Forward):
+        P = _in_project(x, self.w_in, parts, decode)
+        out = x.new_empty(x.shape[0], self.o.shape[1])
+        self.left.run(P, parts, slot_mapping, cache[0], fw, out[:, :self.split])
+        self.right.run(P, parts, cache[1], fw, out[:, self.split:])
+        return ops.project(out, self.o, decode), P, self.tail
+
+
+class DeltaMixer:
+    """Gated delta rule behind short convolutions of q, k and v."""
+
+    def __init__(self, sp: GatedDeltaSpec, get, eps: float, dtype, tail):
+        self.sp = sp
+        self.lin = LinearAttention(sp, get, eps, dtype)
+        self.conv_w = torch.cat([get(n + ".conv") for n in "qkv"]).float().t().contiguous()      # [taps, C]
+        self.C = self.conv_w.shape[1]
+        self.tail = self.lin.n
+        self.rest = self.tail - self.C                     # gate, decay and step columns
+        m = self.lin.mix
+        self.step_mix = replace(m, g=m.g - self.C, a=m.a - self.C, b=m.b - self.C)
+        self.w_in = _joint(self.lin.rows + [tail], dtype)
+        self.o = self.lin.o.to(dtype).contiguous()
+        self.lin.rows = self.lin.o = None
+
+    def rotations(self) -> set:
+        return set()
+
+    def cache_specs(self) -> list:
+        return [StateSpec(((self.sp.conv - 1, self.C), self.lin.state_shape()), (False, True))]
+
+    def activation_elems(self) -> int:
+        sp = self.sp
+        return self.w_in.shape[0] + self.C + self.o.shape[1] + 2 * sp.heads * (4 * sp.dim + 3 * sp.vdim + 64)
+
+    def run(self, x, parts, slot_mapping, cache, decode, fw: _Forward):
+        conv_state, state = cache[0]
+        one = decode and len(parts) == 1
+        P = ops.project(x, self.w_in, True) if one else ops.linear(x, self.w_in, decode)
+        out = x.new_empty(x.shape[0], self.o.shape[1])
+        for p in parts:
+            m, r = p.meta, _split(P, p, parts)
+            if p.decode:
+                y, z = ops.conv_step(r, self.conv_w, None, conv_state, m.state_slots, m.positions, rest=self.rest)
+                mix = self.step_mix
+            else:
+                y, z = ops.causal_conv(r, self.conv_w, None, conv_state, m.state_slots, m.cu_seqlens, m.prefix_lens, m.max_len), r
+                mix = self.lin.mix
+            self.lin.run_part(y, z, mix, p, state, None, _split(out, p, parts))
+        return ops.project(out, self.o, decode), P, self.tail
+
+
+class Experts:
+    """Routed experts and a shared one.  The shared expert's gate and up rows and the ``tail`` rows
+    are one projection; routing is fp32."""
+
+    def __init__(self, sp: MoESpec, get, dtype, tail):
+        self.sp, self.dtype = sp, dtype
+        pad = torch.nn.functional.pad
+        F = _pad_up(sp.ff, 64)
+        self.up = torch.stack([torch.stack([pad(get(f"e{e}.{n}").to(dtype), (0, 0, 0, F - sp.ff)) for n in ("gate", "up")])
+                               for e in range(sp.experts)])                                     # [E, 2, F, W]
+        self.down = torch.stack([pad(get(f"e{e}.down").to(dtype), (0, F - sp.ff)) for e in range(sp.experts)])
+        router, rows = [get("router")], [tail]
+        self.shared = None
+        if sp.shared:
+            self.fs = _pad_up(sp.shared, 64)
+            rows = [pad(get("shared." + n), (0, 0, 0, self.fs - sp.shared)) for n in ("gate", "up")] + rows
+            self.shared = pad(get("shared.down").to(dtype), (0, self.fs - sp.shared)).contiguous()
+            router.append(get("shared.sg"))
+        self.router = torch.cat(router).to(dtype).contiguous()
+        self.tail = 2 * self.fs if sp.shared else 0
+        self.w_in = _joint(rows, dtype)
+
+    def activation_elems(self) -> int:
+        return self.w_in.shape[0] + self.sp.top * (self.up.shape[2] + self.up.shape[3]) + self.tail
+
+    def run(self, x, decode):
+        P = ops.project(x, self.w_in, decode)
+        ids, wts, sg = ops.moe_route(x, self.router, self.sp.experts, self.sp.top)
+        y = ops.moe_experts(x, ids, wts, self.up, self.down)
+        if self.shared is None:
+            return y, None, P, self.tail
+        return y, ops.project(ops.glu(P, 0, self.fs, sg, self.dtype), self.shared, decode), P, self.tail
+
+
 class InputConv:
     """h + conv(h): the causal convolution per channel ahead of a mixer, the identity in its
     last tap."""
@@ -477,7 +868,7 @@ class HybridModel(Decoder):
         self.tp, self.tp_rank = 1, 0
         self.vocab_shard = self.vocab_valid = cfg.vocab_size
         self.vocab_start = 0
-        att = [s.mixer for s in cfg.layer_specs if not isinstance(s.mixer, SelectiveScanSpec)]
+        att = [getattr(s.mixer, "left", s.mixer) for s in cfg.layer_specs if not isinstance(s.mixer, SelectiveScanSpec)]
         self.hq, self.hkv = (att[0].heads, getattr(att[0], "kv_heads", 1)) if att else (1, 1)
         self._side_stream = None  # second branch of captured decode steps
         self.tap = None           # a list: receives the residual stream after every run
@@ -489,7 +880,7 @@ class HybridModel(Decoder):
 
         def get(name):
             t = weights[name]
-            if tuple(t.shape) != shapes[name]:
+            if len(t.shape) != len(shapes[name]) or any(n not in (0, k) for n, k in zip(shapes[name], t.shape)):
                 raise ValueError(f"{name}: shape {tuple(t.shape)}, expected {shapes[name]}")
             return t.to(self.device)
 
@@ -503,7 +894,20 @@ class HybridModel(Decoder):
         self.embed = get("embed").to(dt).contiguous()
         self.lm_head = get("head").to(dt).contiguous()
         self.final_norm = norm("final.norm")
-        self.layers = []
+        self.layers, self.rope_freq = [], {}
+        if cfg.post is not None:
+            for i, sp in enumerate(cfg.layer_specs):
+                p = f"l{i}."
+                L = {"mixer": _MIXERS[type(sp.mixer)](sp.mixer, lambda n: get(p + "mix." + n), cfg.rms_eps, dt, get(p + "rg1")),
+                     "norm1": norm(p + "norm1"), "rg1_b": vec(p + "rg1.b"), "mlp": None}
+                if sp.moe is not None:
+                    L.update(mlp=Experts(sp.moe, lambda n: get(p + "mlp." + n), dt, get(p + "rg2")), norm2=norm(p + "norm2"),
+                             rg2_b=vec(p + "rg2.b"))
+                self.layers.append(L)
+            for rot in {r for L in self.layers for r in L["mixer"].rotations()}:
+                f, mult = rot.frequencies()
+                self.rope_freq[rot] = (f.to(self.device), mult)
+            return
         for i, sp in enumerate(cfg.layer_specs):
             p = f"l{i}."
             L = {"mixer": _MIXERS[type(sp.mixer)](sp.mixer, lambda n: get(p + "mix." + n), cfg.rms_eps, dt),
@@ -530,6 +934,8 @@ class HybridModel(Decoder):
     def _run_specs(self) -> list:
         """Per run: what its mixer keeps (or, an integer, whose cache it reads), what its input
         convolution keeps."""
+        if self.cfg.post is not None:
+            return [L["mixer"].cache_specs() for L in self.layers]
         return [[self.layers[i][k].cache_spec() for k in ("mixer", "conv") if k in self.layers[i]]
                 for i, _ in self.cfg.runs]
 
@@ -540,15 +946,22 @@ class HybridModel(Decoder):
         return [s for run in self._run_specs() for s in run if isinstance(s, StateSpec)]
 
     def bind_caches(self, kv, state) -> list:
-        """Per run its mixer's tensors; in the parallel form (latent rows, convolution inputs)."""
+        """Per run its mixer's tensors; in the parallel form (latent rows, convolution inputs), in the
+        post-norm form a tuple of tensors for each of its mixer's specs."""
         k, s = iter(kv.caches), iter(state.states if state is not None else [])
         out = []
         for run in self._run_specs():
             own = [next(k) if isinstance(sp, KVSpec) else next(s) if isinstance(sp, StateSpec) else out[sp] for sp in run]
+            if self.cfg.post is not None:
+                out.append(own)
+                continue
             out.append(own[0] if len(own) == 1 else (own[0][0], own[1][0]))
         return out
 
     def activation_elems(self) -> int:
+        if self.cfg.post is not None:
+            return 10 * self.cfg.hidden + max([max(L["mixer"].activation_elems(), L["mlp"].activation_elems() if L["mlp"] else 0)
+                                               for L in self.layers] + [0])
         ff = max([s.ff for s in self.cfg.layer_specs] + [0])
         return 8 * self.cfg.hidden + max(max(L["mixer"].activation_elems() for L in self.layers), 3 * ff)
 
@@ -574,6 +987,8 @@ class HybridModel(Decoder):
     def _hidden(self, input_ids, parts, slot_mapping, caches):
         if self.cfg.parallel is not None:
             return self._hidden_parallel(input_ids, parts, slot_mapping, caches)
+        if self.cfg.post is not None:
+            return self._hidden_post(input_ids, parts, slot_mapping, caches)
         cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
         decode = all(p.decode for p in parts)
         runs = cfg.runs
@@ -626,6 +1041,24 @@ class HybridModel(Decoder):
                 self.tap.append(res.clone())
         return h
 
+    def _hidden_post(self, input_ids, parts, slot_mapping, caches):
+        cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
+        alpha, groups = cfg.post.alpha, cfg.post.groups
+        decode = all(p.decode for p in parts)
+        pos = _join([p.meta.positions for p in parts])
+        fw = _Forward({r: ops.rope_table(pos, f, mult) for r, (f, mult) in self.rope_freq.items()}, {})
+        x = ops.embedding(input_ids, self.embed)
+        res = x.float()
+        for L, cache in zip(self.layers, caches):
+            y, P, col = L["mixer"].run(x, parts, slot_mapping, cache, decode, fw)
+            x = ops.post_norm(y, None, P, col, L["rg1_b"], res, alpha, L["norm1"], groups, eps, dt)
+            if L["mlp"] is not None:
+                y, z, P, col = L["mlp"].run(x, decode)
+                x = ops.post_norm(y, z, P, col, L["rg2_b"], res, alpha, L["norm2"], groups, eps, dt)
+            if self.tap is not None:
+                self.tap.append(res.clone())
+        return ops.post_norm(None, None, None, 0, None, res, 1.0, self.final_norm, groups, eps, dt)
+
     def _sublayers(self, L, h, hm, parts, slot_mapping, cache, decode, fw):
         """The layer's mixer and feed-forward (or None).  In a captured decode step they are two
         branches of the graph: the mixer's chain of small launches runs beside the feed-forward's
@@ -656,7 +1089,8 @@ class HybridModel(Decoder):
         return logits if self.cfg.logit_softcap is None else ops.soft_cap(logits, self.cfg.logit_softcap)
 
 
-_MIXERS = {WindowAttentionSpec: WindowAttention, SelectiveScanSpec: SelectiveScan, LatentAttentionSpec: LatentAttention}
+_MIXERS = {WindowAttentionSpec: WindowAttention, SelectiveScanSpec: SelectiveScan, LatentAttentionSpec: LatentAttention,
+           TwoSidedSpec: TwoSidedMixer, GatedDeltaSpec: DeltaMixer}
 
 
 class _RandomWeights:
@@ -674,11 +1108,13 @@ class _RandomWeights:
         if name.endswith("norm") or kind.startswith("norm"):
             stored_off = self.offset if kind.startswith("norm1") or name == "final.norm" else 0.0
             return torch.full(shape, 1.0 - stored_off, device=self.device)
+        if kind == "A_log" and len(shape) == 1:
+            return torch.empty(shape, device=self.device).uniform_(1.0, 16.0, generator=g).log()
         if kind == "A_log":
             return torch.log(torch.arange(1, shape[1] + 1, device=self.device).float()).expand(shape).contiguous()
         if kind == "D":
             return torch.ones(shape, device=self.device)
-        if name.endswith("dt.b"):
+        if name.endswith(("dt.b", "dt_bias")):
             u = torch.rand(shape, device=self.device, generator=g)
             dt = torch.exp(u * (math.log(0.1) - math.log(1e-3)) + math.log(1e-3))
             return dt + torch.log(-torch.expm1(-dt))          # softplus^-1

@@ -11,6 +11,7 @@ from __future__ import annotations
 
 import os
 import threading
+from dataclasses import dataclass
 from pathlib import Path
 
 import torch
@@ -1344,26 +1345,33 @@ def qk_norm_store(P, w, slots, k_cache, k_scale, H: int, eps: float):
 
 
 def window_attn(q, k_cache, block_tables, ctx, scale: float, window: int = 0, sink=None, k_scale=None, v_cache=None,
-                cu=None, max_q: int = 1, v_dim: int = 0):
+                cu=None, max_q: int = 1, v_dim: int = 0, cap: float = 0.0, out_scale: float = 1.0, out=None):
     """Causal attention over the last ``window`` tokens (0: all) of the paged cache, scores
     times ``k_scale`` per cached key, ``sink`` [H] in the denominator, ``v_cache`` None: the
-    keys are the values -- their first ``v_dim`` elements (0: all of them).  With ``cu``
+    keys are the values -- their first ``v_dim`` elements (0: all of them); ``v_cache`` rows may
+    be of another size than the keys.  ``cap``: scores become cap tanh(score / cap).  With ``cu``
     [B + 1]: packed query tokens, ``ctx`` the position of each sequence's first; without: one
-    query token a row, ``ctx`` the context lengths."""
+    query token a row, ``ctx`` the context lengths.  The result, times ``out_scale``, goes to
+    ``out`` (rows of a wider matrix) where given."""
     if _gpu(q):
-        return _native().window_attn(q.contiguous(), k_cache, v_cache, k_scale, block_tables, cu, ctx, int(max_q),
-                                     float(scale), int(window), sink, int(v_dim))
-    return ref.window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink, v_dim)
+        T, H = q.shape[0], q.shape[1] // k_cache.shape[3]
+        if out is None:
+            out = q.new_empty(T, H * (v_dim or (k_cache if v_cache is None else v_cache).shape[3]))
+        _native().window_attn(q.contiguous(), k_cache, v_cache, k_scale, block_tables, cu, ctx, int(max_q),
+                              float(scale), int(window), sink, int(v_dim), float(cap), float(out_scale), out)
+        return out
+    return ref.window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink, v_dim, cap, out_scale, out)
 
 
 # Latent attention (csrc/kernels/attn_latent.hip).  A cached row is [latent: R | rotated key
 # part: r], each padded with zeros to 8 elements (R8, r8); a query head is [unrotated: d |
 # rotated: r], padded alike (d8, r8).
-def rope_table(positions, inv_freq):
-    """fp32 [cos | sin] rows of the angles position * inv_freq (``inv_freq`` fp64 [r / 2])."""
+def rope_table(positions, inv_freq, mult: float = 1.0):
+    """fp32 [cos | sin] rows of the angles position * inv_freq (``inv_freq`` fp64 [r / 2]), times
+    ``mult``."""
     if _gpu(positions):
-        return _native().rope_table(positions, inv_freq)
-    return ref.rope_table(positions, inv_freq)
+        return _native().rope_table(positions, inv_freq, float(mult))
+    return ref.rope_table(positions, inv_freq, mult)
 
 
 def latent_store(P, cs, slots, cache, c_norm, H: int, dim: int, rank: int, eps: float, dtype):
@@ -1433,13 +1441,13 @@ def causal_conv(x, w, bias, state, slots, cu, ctx, max_len: int, silu: bool = Tr
     return ref.causal_conv(x, w, bias, state, slots, cu, ctx, silu)
 
 
-def conv_step(P, w, bias, state, slots, positions, silu: bool = True):
-    """One token a row: (conv [B, C], gate [B, C]) of an [x | z] projection -- (conv, None) of an
-    [x] one; advances ``state`` (rows with slot -1 leave none)."""
+def conv_step(P, w, bias, state, slots, positions, silu: bool = True, rest: int = -1):
+    """One token a row: (conv [B, C], z) of an [x: C | z] projection, z its next ``rest`` columns
+    (-1: all of them; none: None); advances ``state`` (rows with slot -1 leave none)."""
     if _gpu(P):
-        y, z = _native().conv_step(P.contiguous(), w, bias, state, slots, positions, silu)
+        y, z = _native().conv_step(P.contiguous(), w, bias, state, slots, positions, silu, int(rest))
         return y, (z if z.numel() else None)
-    return ref.conv_step(P, w, bias, state, slots, positions, silu)
+    return ref.conv_step(P, w, bias, state, slots, positions, silu, rest)
 
 
 def scan_chunk(tokens: int, max_len: int, channels: int) -> int:
@@ -1476,6 +1484,109 @@ def selective_step(x, dt, bc, b_off: int, c_off: int, N: int, z, A2, D, dt_b, st
     if _gpu(x):
         return _native().selective_step(x, dt, None, None, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions)
     return ref.selective_step(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions)
+
+
+# Attention with normed, rotated keys; linear attention (csrc/kernels/linear_attn.hip); experts
+# (csrc/kernels/moe.hip).
+def qkv_rope_store(P, bias, q_norm, k_norm, cs, slots, k_cache, v_cache, H: int, eps: float):
+    """Query heads [T, H * D] of a [q | k | v | ..] projection (plus ``bias``): RMS norm per head
+    (``q_norm`` [D] or None), then the first r dimensions rotated by the rows ``cs`` [T, r] of
+    :func:`rope_table`; keys alike and values go to the paged cache."""
+    if _gpu(P):
+        return _native().qkv_rope_store(P.contiguous(), bias, q_norm, k_norm, cs, slots, k_cache, v_cache, int(H), float(eps))
+    return ref.qkv_rope_store(P, bias, q_norm, k_norm, cs, slots, k_cache, v_cache, H, eps)
+
+
+@dataclass(frozen=True)
+class LinearMix:
+    """A linear-attention recurrence S <- decay S + k u^T, o = S^T q per head: where its operands
+    stand and what is done to them.  ``kind`` "channel": decays sigmoid(a . w + b)^inv_tau per key
+    channel; "fixed": a decay per head, q and k rotated; "delta": unit q and k, a decay per head
+    exp(w softplus(a + b)), u = sigmoid(beta) (v - (decay S)^T k).  Columns ``q`` ``k`` ``v`` of the
+    matrix X, ``g`` (the output gate), ``a`` and ``b`` of Z.  Each head's o is normed over ``vdim``
+    (``eps``), weighted, and multiplied by silu(g)."""
+    kind: str
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    q: int
+    k: int
+    v: int
+    g: int
+    a: int = 0
+    b: int = 0
+    rank: int = 0
+    q_scale: float = 1.0
+    k_scale: float = 1.0
+    inv_tau: float = 1.0
+    eps: float = 1e-5
+
+    def native(self):
+        return ([("channel", "fixed", "delta").index(self.kind), self.heads, self.kv_heads, self.dim, self.vdim, self.q, self.k,
+                 self.v, self.g, self.a, self.b, self.rank], [self.q_scale, self.k_scale, self.inv_tau, self.eps])
+
+
+def linear_state_shape(heads: int, dim: int, vdim: int) -> tuple:
+    """fp32 state of one request: [heads, dim, vdim padded to 4]."""
+    return heads, dim, -(-vdim // 4) * 4
+
+
+def linear_step(X, Z, m: LinearMix, w_gate, b_gate, cs, norm, state, slots, positions, out):
+    """One token a row through the recurrence: reads and advances ``state`` [slots, H, dim, vdim4]
+    (position 0 starts from zero; rows with slot -1 leave none), writes the gated heads to ``out``
+    [B, H * vdim].  X, Z: products or split-K slabs."""
+    if _gpu(X):
+        _native().linear_step(X.contiguous(), Z.contiguous(), *m.native(), w_gate, b_gate, cs, norm, state, slots, positions, out)
+        return out
+    return ref.linear_step(X, Z, m, w_gate, b_gate, cs, norm, state, slots, positions, out)
+
+
+def linear_scan(X, Z, m: LinearMix, w_gate, b_gate, cs, norm, state, slots, cu, ctx, max_len: int, out):
+    """:func:`linear_step` over packed sequences (``cu`` [B + 1]; ``ctx`` > 0: enters from ``state``)."""
+    if _gpu(X):
+        _native().linear_scan(X.contiguous(), Z.contiguous(), *m.native(), w_gate, b_gate, cs, norm, state, slots, cu, ctx,
+                              int(max_len), out)
+        return out
+    return ref.linear_scan(X, Z, m, w_gate, b_gate, cs, norm, state, slots, cu, ctx, out)
+
+
+def post_norm(P, Q, gate, col: int, gate_b, residual, alpha: float, w, groups: int, eps: float, out_dtype=torch.bfloat16):
+    """residual (fp32, in place) <- grouped RMS norm of alpha residual + sigmoid(gate + gate_b) (P + Q)
+    times ``w``; returns it in ``out_dtype``.  ``gate``: columns [col, col + W) of a projection; P, Q,
+    gate products or slabs, Q (or all three) None: left out."""
+    if _gpu(residual):
+        def c(t):
+            return None if t is None else t.contiguous()
+
+        out = _native().post_norm(c(P), c(Q), c(gate), int(col), gate_b, residual, float(alpha), w, int(groups), float(eps),
+                                  out_dtype == torch.float32)
+        return out if out_dtype != torch.float32 else residual
+    return ref.post_norm(P, Q, gate, col, gate_b, residual, alpha, w, groups, eps, out_dtype)
+
+
+def moe_route(x, w, experts: int, top: int):
+    """Scores sigmoid(x w^T) in fp32: (ids [T, top], scores [T, top]) of the largest of the first
+    ``experts``, and the other columns' scores [T, n - experts]."""
+    if _gpu(x):
+        return _native().moe_route(x.contiguous(), w, int(experts), int(top))
+    return ref.moe_route(x, w, experts, top)
+
+
+def glu(P, col: int, n: int, scale=None, out_dtype=torch.bfloat16):
+    """silu(gate) * up of columns [col, col + n), [col + n, col + 2 n) of a projection, rows times
+    ``scale`` [T]."""
+    if _gpu(P):
+        return _native().slab_glu(P.contiguous(), int(col), int(n), scale, out_dtype == torch.float32)
+    return ref.glu(P, col, n, scale, out_dtype)
+
+
+def moe_experts(x, ids, wts, up, down):
+    """Slabs [top, T, W]: slab k holds, for every token, expert ids[:, k]'s output for the input
+    wts[:, k] x; ``up`` [E, 2 (gate, up), F, K], ``down`` [E, W, F]."""
+    if _gpu(x):
+        return _native().moe_experts(x.contiguous(), ids, wts, up, down)
+    return ref.moe_experts(x, ids, wts, up, down)
 
 
 def linear(x, w, decode: bool = False):

@@ -385,9 +385,9 @@ def soft_cap(x, cap):
     return cap * torch.tanh(x.float() / cap)
 
 
-def rope_table(positions, inv_freq):
+def rope_table(positions, inv_freq, mult=1.0):
     a = positions.double()[:, None] * inv_freq
-    return torch.cat([a.cos(), a.sin()], -1).float()
+    return (torch.cat([a.cos(), a.sin()], -1) * mult).float()
 
 
 def _rotate(x, cs):
@@ -440,12 +440,13 @@ def qk_norm_store(P, w, slots, k_cache, k_scale, H, eps):
     return q
 
 
-def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink, v_dim):
+def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, window, sink, v_dim, cap=0.0, out_scale=1.0,
+                out=None):
     NB, G, BS, D = k_cache.shape
     H = q.shape[1] // D
     v_cache = k_cache if v_cache is None else v_cache
-    v_dim = v_dim or D
-    out = q.new_zeros(q.shape[0], H * v_dim)
+    v_dim = v_dim or v_cache.shape[3]
+    out = q.new_zeros(q.shape[0], H * v_dim) if out is None else out
     for b in range(block_tables.shape[0]):
         q0, L, p0 = (b, 1, int(ctx[b]) - 1) if cu is None else (int(cu[b]), int(cu[b + 1] - cu[b]), int(ctx[b]))
         if L <= 0 or p0 < 0:
@@ -460,6 +461,8 @@ def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, wind
         s = torch.einsum("ghld,gkd->ghlk", qb, k) * scale
         if k_scale is not None:
             s = s * k_scale.view(NB, G, BS)[blk, :, off].t()[:, None, None, :]
+        if cap:
+            s = cap * torch.tanh(s / cap)
         i = torch.arange(p0, n, device=q.device)[:, None]
         dead = pos[None, :] > i
         if window > 0:
@@ -469,7 +472,7 @@ def window_attn(q, k_cache, v_cache, k_scale, block_tables, cu, ctx, scale, wind
             s = torch.cat([s, sink.float().view(G, H // G, 1, 1).expand(G, H // G, L, 1)], -1)
         p = torch.softmax(s, -1)[..., :n - lo]
         o = torch.einsum("ghlk,gkd->ghld", p, v)
-        out[q0:q0 + L] = o.permute(2, 0, 1, 3).reshape(L, H * v_dim).to(q.dtype)
+        out[q0:q0 + L] = (o.permute(2, 0, 1, 3).reshape(L, H * v_dim) * out_scale).to(q.dtype)
     return out
 
 
@@ -524,10 +527,11 @@ def causal_conv(x, w, bias, state, slots, cu, ctx, silu=True):
     return y
 
 
-def conv_step(P, w, bias, state, slots, positions, silu=True):
+def conv_step(P, w, bias, state, slots, positions, silu=True, rest=-1):
     C = w.shape[1]
     B = P.shape[-2]
     xz = _slab_sum(P).to(state.dtype)
+    xz = xz if rest < 0 else xz[:, :C + rest]
     cu = torch.arange(B + 1, dtype=torch.int32)
     y = causal_conv(xz[:, :C], w, bias, state, slots, cu, positions, silu)
     return y, (xz[:, C:].contiguous() if xz.shape[1] > C else None)
@@ -553,3 +557,114 @@ def selective_scan(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, cu,
 def selective_step(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, positions):
     cu = torch.arange(x.shape[0] + 1, dtype=torch.int32)
     return selective_scan(x, dt, bc, b_off, c_off, N, z, A2, D, dt_b, state, slots, cu, positions)
+
+
+# ------------------------------------------- attention with rotated keys, linear attention
+def qkv_rope_store(P, bias, qw, kw, cs, slots, k_cache, v_cache, H, eps):
+    x = _slab_sum(P)
+    T = x.shape[0]
+    G, BS, D = k_cache.shape[1:]
+    DV = v_cache.shape[3]
+    n = (H + G) * D + G * DV
+    x = x[:, :n] + bias if bias is not None else x[:, :n]
+    q, k = x[:, :H * D].reshape(T, H, D), x[:, H * D:(H + G) * D].reshape(T, G, D)
+    r = cs.shape[1]
+
+    def head(y, w):
+        y = _rms(y, eps) * w if w is not None else y
+        return torch.cat([_rotate(y[..., :r], cs), y[..., r:]], -1).to(k_cache.dtype) if r else y.to(k_cache.dtype)
+
+    sm = slots.long()
+    ok = sm >= 0
+    blk, off = sm[ok] // BS, sm[ok] % BS
+    k_cache[blk, :, off] = head(k, kw)[ok]
+    v_cache[blk, :, off] = x[:, (H + G) * D:].reshape(T, G, DV).to(v_cache.dtype)[ok]
+    return head(q, qw).reshape(T, H * D)
+
+
+def _linear_inputs(X, Z, m, w_gate, b_gate, cs):
+    """fp32 (q, k [T, H, d], v, gate [T, H, vd], log decay [T, H, d or 1], beta [T, H] or None)."""
+    x, z = _slab_sum(X), _slab_sum(Z)
+    T, H, G, d, vd = x.shape[0], m.heads, m.kv_heads, m.dim, m.vdim
+
+    def cols(t, at, h, n):
+        return t[:, at:at + h * n].reshape(T, h, n)
+
+    q, k, v, g = cols(x, m.q, G, d), cols(x, m.k, G, d), cols(x, m.v, H, vd), cols(z, m.g, H, vd)
+    beta = None
+    if m.kind == "delta":
+        q, k = (t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6) for t in (q, k))
+        la = (w_gate * F.softplus(z[:, m.a:m.a + H] + b_gate))[..., None]
+        beta = torch.sigmoid(z[:, m.b:m.b + H])
+    elif m.kind == "channel":
+        la = (F.logsigmoid(z[:, m.a:m.a + m.rank] @ w_gate.t() + b_gate) * m.inv_tau).view(T, H, d)
+    else:
+        r = cs.shape[1]
+        q, k = (torch.cat([_rotate(t[..., :r], cs), t[..., r:]], -1) for t in (q, k))
+        la = w_gate.view(1, H, 1).expand(T, H, 1)
+    q, k = (t.repeat_interleave(H // G, 1) for t in (q * m.q_scale, k * m.k_scale))
+    return q, k, v, g, la, beta
+
+
+def linear_scan(X, Z, m, w_gate, b_gate, cs, norm, state, slots, cu, ctx, out):
+    q, k, v, g, la, beta = _linear_inputs(X, Z, m, w_gate, b_gate, cs)
+    H, d, vd = m.heads, m.dim, m.vdim
+    for b in range(cu.numel() - 1):
+        q0, q1, slot = int(cu[b]), int(cu[b + 1]), int(slots[b])
+        if q1 <= q0:
+            continue
+        S = (state[slot, ..., :vd].clone() if slot >= 0 and int(ctx[b]) > 0
+             else torch.zeros(H, d, vd, device=state.device))
+        for t in range(q0, q1):
+            S = torch.exp(la[t])[..., None] * S
+            u = v[t] if beta is None else beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
+            S = S + k[t][..., None] * u[:, None]
+            o = torch.einsum("hdv,hd->hv", S, q[t])
+            out[t] = (_rms(o, m.eps) * norm * F.silu(g[t])).reshape(-1).to(out.dtype)
+        if slot >= 0:
+            state[slot, ..., :vd] = S
+    return out
+
+
+def linear_step(X, Z, m, w_gate, b_gate, cs, norm, state, slots, positions, out):
+    n = X.shape[-2]
+    return linear_scan(X, Z, m, w_gate, b_gate, cs, norm, state, slots, torch.arange(n + 1, dtype=torch.int32), positions, out)
+
+
+# ------------------------------------------------------------ norms after the sum, experts
+def post_norm(P, Q, gate, col, gate_b, res, alpha, w, groups, eps, out_dtype):
+    x = alpha * res
+    if P is not None:
+        y = _slab_sum(P)
+        if Q is not None:
+            y = y + _slab_sum(Q)
+        x = x + torch.sigmoid(_slab_sum(gate)[:, col:col + res.shape[1]] + gate_b) * y
+    T, W = res.shape
+    res.copy_(_rms(x.view(T, groups, W // groups), eps).view(T, W) * w)
+    return res.to(out_dtype)
+
+
+def moe_route(x, w, experts, top):
+    z = x.float() @ w.float().t()
+    s = torch.sigmoid(z)
+    best = torch.topk(s[:, :experts], top, -1)
+    return best.indices.to(torch.int32), best.values, s[:, experts:].contiguous()
+
+
+def glu(P, col, n, scale, out_dtype):
+    x = _slab_sum(P)
+    y = F.silu(x[:, col:col + n]) * x[:, col + n:col + 2 * n]
+    return (y if scale is None else y * scale.view(-1, 1)).to(out_dtype)
+
+
+def moe_experts(x, ids, wts, up, down):
+    T, top = ids.shape
+    out = torch.zeros(top, T, down.shape[1], dtype=x.dtype, device=x.device)
+    for e in range(up.shape[0]):
+        t, k = (ids == e).nonzero(as_tuple=True)
+        if t.numel() == 0:
+            continue
+        s = wts[t, k][:, None]
+        a = (F.silu(s * (x[t].float() @ up[e, 0].float().t())) * (s * (x[t].float() @ up[e, 1].float().t()))).to(x.dtype)
+        out[k, t] = (a.float() @ down[e].float().t()).to(x.dtype)
+    return out
