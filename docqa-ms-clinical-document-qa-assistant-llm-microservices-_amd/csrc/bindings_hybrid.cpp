@@ -69,20 +69,22 @@ Tensor sandwich_rmsnorm(const Tensor& P, Tensor residual, const Tensor& w_post, 
 }
 
 std::tuple<Tensor, Tensor, Tensor> embed_scale_rmsnorm(const Tensor& ids, const Tensor& table, double scale,
-                                                       const Tensor& w, double eps, bool keep) {
+                                                       const OptT& w, double eps, bool keep) {
   CHECK_ACT(table); CHECK_CONTIG(table); CHECK_ALIGN16(table);
   TORCH_CHECK(table.dim() == 2, "table must be [vocab, width]");
   const int T = ids.numel(), H = table.size(1);
   check_i32(ids, T, "ids");
-  check_vec(w, H, "w");
-  CHECK_ALIGN16(w);
+  if (w.has_value()) {
+    check_vec(*w, H, "w");
+    CHECK_ALIGN16(*w);
+  }
   c10::DeviceGuard g(table.device());
   auto f32 = table.options().dtype(at::kFloat);
   auto res = at::empty({T, H}, f32);
   auto emb = keep ? at::empty({T, H}, f32) : at::empty({0}, f32);
   auto out = at::empty({T, H}, table.options());
   CHECK_RC(docqa_embed_scale_rmsnorm(ids.data_ptr<int>(), table.data_ptr(), is_f32(table), (float)scale,
-                                     w.data_ptr<float>(), res.data_ptr<float>(),
+                                     w.has_value() ? w->data_ptr<float>() : nullptr, res.data_ptr<float>(),
                                      keep ? emb.data_ptr<float>() : nullptr, out.data_ptr(), T, H,
                                      (int)table.size(0), (float)eps, stream()),
            "embed_scale_rmsnorm");
@@ -214,15 +216,16 @@ Tensor qk_norm_store(const Tensor& P, const Tensor& w, const Tensor& slots, Tens
 
 // cu: [B + 1] query offsets with ctx the first positions (prefill), or null: one query token a
 // row with ctx the context lengths (decode)
-Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, const OptT& k_scale,
-                   const Tensor& block_tables, const OptT& cu, const Tensor& ctx, int64_t max_q, double scale,
-                   int64_t window, const OptT& sink, int64_t v_dim) {
+void window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, const OptT& k_scale,
+                 const Tensor& block_tables, const OptT& cu, const Tensor& ctx, int64_t max_q, double scale,
+                 int64_t window, const OptT& sink, int64_t v_dim, double cap, double out_scale, Tensor out) {
   CHECK_ACT(q); CHECK_CONTIG(q); CHECK_CONTIG(k_cache);
   TORCH_CHECK(k_cache.dim() == 4 && k_cache.scalar_type() == q.scalar_type(), "k_cache dtype / shape");
   const int G = k_cache.size(1), BS = k_cache.size(2), D = k_cache.size(3);
   TORCH_CHECK(q.dim() == 2 && q.size(1) % D == 0, "q must be [rows, H * dim]");
-  const int H = q.size(1) / D, B = block_tables.size(0), DV = v_dim ? v_dim : D;
-  TORCH_CHECK(DV >= 1 && DV <= D && (DV == D || !v_cache.has_value()), "v_dim: part of the shared row");
+  const int H = q.size(1) / D, B = block_tables.size(0);
+  const int DV = v_cache.has_value() ? v_cache->size(3) : v_dim ? v_dim : D;
+  TORCH_CHECK(DV >= 1 && (v_cache.has_value() ? !v_dim || v_dim == DV : DV <= D), "v_dim: part of the shared row");
   CHECK_GPU(block_tables); CHECK_I32(block_tables); CHECK_CONTIG(block_tables);
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(1) >= 1, "block_tables must be [B, blocks]");
   check_i32(ctx, B, "ctx");
@@ -230,21 +233,50 @@ Tensor window_attn(const Tensor& q, const Tensor& k_cache, const OptT& v_cache, 
   else TORCH_CHECK(q.size(0) == B && max_q == 1, "decode: one query row a sequence");
   TORCH_CHECK(k_cache.numel() / D < (1ll << 31), "cache rows must fit 31 bits");
   if (v_cache.has_value())
-    TORCH_CHECK(v_cache->sizes() == k_cache.sizes() && v_cache->scalar_type() == q.scalar_type() &&
-                    v_cache->is_contiguous(), "v_cache must match k_cache");
+    TORCH_CHECK(v_cache->is_cuda() && v_cache->dim() == 4 && v_cache->sizes().slice(0, 3) == k_cache.sizes().slice(0, 3) &&
+                    v_cache->scalar_type() == q.scalar_type() && v_cache->is_contiguous() &&
+                    (reinterpret_cast<uintptr_t>(v_cache->data_ptr()) & 15u) == 0, "v_cache must match k_cache");
   if (k_scale.has_value()) check_vec(*k_scale, k_cache.numel() / D, "k_scale");
   if (sink.has_value()) check_vec(*sink, H, "sink");
   c10::DeviceGuard g(q.device());
   CHECK_ALIGN16(k_cache);     // cached rows are read in 16-byte pieces, q row by row
-  auto out = at::empty({q.size(0), (int64_t)H * DV}, q.options());
+  TORCH_CHECK(out.size(1) == (int64_t)H * DV, "window_attn: output width");
+  check_rows(out, q.size(0), (int64_t)H * DV, q, "out");
   CHECK_RC(docqa_window_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.has_value() ? v_cache->data_ptr() : k_cache.data_ptr(),
                              k_scale.has_value() ? k_scale->data_ptr<float>() : nullptr, block_tables.data_ptr<int>(),
                              (int)block_tables.size(1), cu.has_value() ? cu->data_ptr<int>() : nullptr,
                              ctx.data_ptr<int>(), sink.has_value() ? sink->data_ptr<float>() : nullptr,
-                             out.data_ptr(), is_f32(q), B, (int)max_q, H, G, D, DV, BS, (float)scale, (int)window,
-                             stream()),
+                             out.data_ptr(), (int)out.stride(0), is_f32(q), B, (int)max_q, H, G, D, DV, BS, (float)scale,
+                             (int)window, (float)cap, (float)out_scale, stream()),
            "window_attn");
-  return out;
+}
+
+Tensor qkv_rope_store(const Tensor& P, const OptT& bias, const OptT& qw, const OptT& kw, const Tensor& cs, const Tensor& slots,
+                      Tensor k_cache, Tensor v_cache, int64_t H, double eps) {
+  const Slabs p = slabs_of(P);
+  CHECK_ACT(k_cache); CHECK_CONTIG(k_cache); CHECK_CONTIG(v_cache); CHECK_ALIGN16(k_cache); CHECK_ALIGN16(v_cache);
+  CHECK_ALIGN16(P); CHECK_ALIGN16(cs);
+  TORCH_CHECK(k_cache.dim() == 4 && v_cache.dim() == 4 && v_cache.is_cuda() && v_cache.scalar_type() == k_cache.scalar_type() &&
+                  v_cache.sizes().slice(0, 3) == k_cache.sizes().slice(0, 3), "caches must be [blocks, kv heads, block, dim]");
+  const int G = k_cache.size(1), BS = k_cache.size(2), D = k_cache.size(3), DV = v_cache.size(3);
+  TORCH_CHECK(H >= 1 && p.N >= (H + G) * D + (int64_t)G * DV, "qkv_rope_store: projection width");
+  auto vec = [](const OptT& t, int64_t n, const char* name) -> const float* {
+    if (!t.has_value()) return nullptr;
+    check_vec(*t, n, name);
+    CHECK_ALIGN16(*t);
+    return t->data_ptr<float>();
+  };
+  TORCH_CHECK(cs.dim() == 2 && cs.size(1) <= D, "cs must be [tokens, r]");
+  check_vec(cs, (int64_t)p.M * cs.size(1), "cs");
+  check_i32(slots, p.M, "slots");
+  c10::DeviceGuard g(P.device());
+  auto q = at::empty({p.M, H * D}, k_cache.options());
+  CHECK_RC(docqa_qkv_rope_store(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, vec(bias, (H + G) * D + (int64_t)G * DV, "bias"),
+                                vec(qw, D, "q norm"), vec(kw, D, "k norm"), cs.data_ptr<float>(), (int)cs.size(1),
+                                slots.data_ptr<int>(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), is_f32(k_cache),
+                                p.M, (int)H, G, D, DV, BS, (float)eps, stream()),
+           "qkv_rope_store");
+  return q;
 }
 
 // window_attn in the latent space (one KV head, values = the first K elements of a cached row, K =
@@ -306,13 +338,13 @@ Tensor packed_window_attn(const Tensor& q, const Tensor& kv, const Tensor& kr, i
   return out;
 }
 
-Tensor rope_table(const Tensor& positions, const Tensor& freq) {
+Tensor rope_table(const Tensor& positions, const Tensor& freq, double mult) {
   const int T = positions.numel(), half = freq.numel();
   check_i32(positions, T, "positions");
   TORCH_CHECK(freq.is_cuda() && freq.scalar_type() == at::kDouble && freq.is_contiguous(), "freq: fp64 vector expected");
   c10::DeviceGuard g(positions.device());
   auto out = at::empty({T, 2 * half}, positions.options().dtype(at::kFloat));
-  CHECK_RC(docqa_rope_table(positions.data_ptr<int>(), freq.data_ptr<double>(), out.data_ptr<float>(), T, half, stream()),
+  CHECK_RC(docqa_rope_table(positions.data_ptr<int>(), freq.data_ptr<double>(), out.data_ptr<float>(), T, half, mult, stream()),
            "rope_table");
   return out;
 }
@@ -425,24 +457,24 @@ std::tuple<Tensor, Tensor> sandwich_rmsnorm_conv(const Tensor& P, Tensor residua
   return {h, hc};
 }
 
-// P: [x: C | z: C] input projection of one token a row -> (conv x, z); [x: C] -> (conv x, empty)
+// P: [x: C | z: rest | ..] input projection of one token a row -> (conv x, z); rest -1: all of the columns
 std::tuple<Tensor, Tensor> conv_step(const Tensor& P, const Tensor& w, const OptT& bias, Tensor state,
-                                     const Tensor& slots, const Tensor& positions, bool silu) {
+                                     const Tensor& slots, const Tensor& positions, bool silu, int64_t rest) {
   const Slabs p = slabs_of(P);
   const int C = w.size(1);
   int taps;
   check_conv(w, bias, state, C, taps);
   CHECK_ACT(state);
-  TORCH_CHECK(p.N == 2 * C || p.N == C, "conv_step: P must be [.., C] or [.., 2 C] wide");
-  const bool gated = p.N == 2 * C;
+  const int64_t nz = rest < 0 ? p.N - C : rest;
+  TORCH_CHECK(nz >= 0 && C + nz <= p.N, "conv_step: columns of P");
   TORCH_CHECK(is_f32(P) || !is_f32(state), "conv_step: fp32 state needs fp32 projections");
   check_i32(slots, p.M, "slots"); check_i32(positions, p.M, "positions");
   c10::DeviceGuard g(P.device());
-  auto y = at::empty({p.M, C}, state.options()), z = at::empty({gated ? p.M : 0, C}, state.options());
+  auto y = at::empty({p.M, C}, state.options()), z = at::empty({nz ? p.M : 0, nz}, state.options());
   CHECK_RC(docqa_conv_step(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, w.data_ptr<float>(),
                            bias.has_value() ? bias->data_ptr<float>() : nullptr,
                            state.data_ptr(), slots.data_ptr<int>(), positions.data_ptr<int>(), y.data_ptr(),
-                           gated ? z.data_ptr() : nullptr, is_f32(state), p.M, C, taps, silu, stream()),
+                           nz ? z.data_ptr() : nullptr, is_f32(state), p.M, C, (int)nz, taps, silu, stream()),
            "conv_step");
   return {y, z};
 }
@@ -521,12 +553,175 @@ Tensor selective_step(const Tensor& x, const OptT& dt, const OptT& dt_in, const 
   return y;
 }
 
+// the recurrence's operands: dims / consts are ops.LinearMix.native()
+DocqaLinear linear_args(const Tensor& X, const Tensor& Z, at::IntArrayRef d, at::ArrayRef<double> f, const Tensor& w_gate,
+                        const OptT& b_gate, const OptT& cs, const Tensor& norm, const Tensor& state, Tensor& out) {
+  const Slabs x = slabs_of(X), z = slabs_of(Z);
+  CHECK_ALIGN16(X); CHECK_ALIGN16(Z); CHECK_ALIGN16(state);
+  TORCH_CHECK(d.size() == 12 && f.size() == 4, "linear attention: arguments");
+  DocqaLinear a{};
+  int* di = &a.kind;
+  for (int i = 0; i < 12; ++i) {
+    TORCH_CHECK(d[i] >= 0 && d[i] < (1 << 24), "linear attention: sizes");
+    di[i] = (int)d[i];
+  }
+  a.X = X.data_ptr(); a.Z = Z.data_ptr();
+  a.xf32 = is_f32(X); a.Sx = x.S; a.ldx = x.N; a.xslab = x.slab;
+  a.zf32 = is_f32(Z); a.Sz = z.S; a.ldz = z.N; a.zslab = z.slab;
+  a.qs = (float)f[0]; a.ks = (float)f[1]; a.inv_tau = (float)f[2]; a.eps = (float)f[3];
+  TORCH_CHECK(a.kind <= LIN_DELTA && a.H >= 1 && a.G >= 1 && a.H % a.G == 0 && a.dk >= 1 && a.dk <= 256 && a.dv >= 1 && a.dv <= 512,
+              "linear attention: heads up to [256, 512]");
+  TORCH_CHECK(a.qo + a.G * a.dk <= x.N && a.ko + a.G * a.dk <= x.N && a.vo + a.H * a.dv <= x.N && a.go + a.H * a.dv <= z.N &&
+                  x.M == z.M, "linear attention: columns");
+  const int64_t n = (int64_t)a.H * a.dk;
+  if (a.kind == LIN_CHANNEL) {
+    TORCH_CHECK(a.rank >= 1 && a.rank <= 1024 && a.ao + a.rank <= z.N && b_gate.has_value(), "linear attention: decay projection");
+    check_vec(w_gate, n * a.rank, "w_gate");
+    check_vec(*b_gate, n, "b_gate");
+  } else {
+    check_vec(w_gate, a.H, "w_gate");
+    if (a.kind == LIN_DELTA) {
+      TORCH_CHECK(a.ao + a.H <= z.N && a.bo + a.H <= z.N && b_gate.has_value(), "linear attention: decay columns");
+      check_vec(*b_gate, a.H, "b_gate");
+    }
+  }
+  if (a.kind == LIN_FIXED) {
+    TORCH_CHECK(cs.has_value() && cs->dim() == 2 && cs->size(1) <= a.dk && cs->size(1) % 2 == 0, "linear attention: rotation rows");
+    a.r = cs->size(1);
+    check_vec(*cs, (int64_t)x.M * a.r, "cs");
+    a.cs = cs->data_ptr<float>();
+  }
+  a.w_gate = w_gate.data_ptr<float>();
+  a.b_gate = b_gate.has_value() ? b_gate->data_ptr<float>() : nullptr;
+  check_vec(norm, a.dv, "norm");
+  a.norm = norm.data_ptr<float>();
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == at::kFloat && state.is_contiguous() && state.dim() == 4 &&
+                  state.size(1) == a.H && state.size(2) == a.dk && state.size(3) == (a.dv + 3) / 4 * 4,
+              "linear attention: state must be fp32 [slots, H, dk, dv padded to 4]");
+  a.state = state.data_ptr<float>();
+  CHECK_ACT(out);
+  TORCH_CHECK(out.size(1) == (int64_t)a.H * a.dv, "linear attention: output width");
+  check_rows(out, x.M, (int64_t)a.H * a.dv, out, "out");
+  a.out = out.data_ptr(); a.of32 = is_f32(out); a.ldo = (int)out.stride(0);
+  return a;
+}
+
+void linear_step(const Tensor& X, const Tensor& Z, at::IntArrayRef dims, at::ArrayRef<double> consts, const Tensor& w_gate,
+                 const OptT& b_gate, const OptT& cs, const Tensor& norm, Tensor state, const Tensor& slots,
+                 const Tensor& positions, Tensor out) {
+  DocqaLinear a = linear_args(X, Z, dims, consts, w_gate, b_gate, cs, norm, state, out);
+  const int B = out.size(0);
+  check_i32(slots, B, "slots"); check_i32(positions, B, "positions");
+  a.slots = slots.data_ptr<int>();
+  c10::DeviceGuard g(X.device());
+  CHECK_RC(docqa_linear_step(a, positions.data_ptr<int>(), B, stream()), "linear_step");
+}
+
+void linear_scan(const Tensor& X, const Tensor& Z, at::IntArrayRef dims, at::ArrayRef<double> consts, const Tensor& w_gate,
+                 const OptT& b_gate, const OptT& cs, const Tensor& norm, Tensor state, const Tensor& slots, const Tensor& cu,
+                 const Tensor& ctx, int64_t max_len, Tensor out) {
+  DocqaLinear a = linear_args(X, Z, dims, consts, w_gate, b_gate, cs, norm, state, out);
+  const int T = out.size(0), B = cu.numel() - 1;
+  check_i32(slots, B, "slots"); check_i32(cu, B + 1, "cu"); check_i32(ctx, B, "ctx");
+  TORCH_CHECK(max_len >= 0 && max_len <= T && B <= 65535, "linear_scan: lengths");
+  a.slots = slots.data_ptr<int>();
+  c10::DeviceGuard g(X.device());
+  auto scratch = at::empty({(int64_t)docqa_linear_scratch(a.kind, T, B, a.H, a.dk, a.dv)}, X.options().dtype(at::kFloat));
+  CHECK_RC(docqa_linear_scan(a, cu.data_ptr<int>(), ctx.data_ptr<int>(), scratch.data_ptr<float>(), T, B, (int)max_len,
+                             stream()),
+           "linear_scan");
+}
+
+Tensor post_norm(const OptT& P, const OptT& Q, const OptT& gate, int64_t col, const OptT& gate_b, Tensor residual,
+                 double alpha, const Tensor& w, int64_t groups, double eps, bool out_f32) {
+  CHECK_GPU(residual); CHECK_F32(residual); CHECK_CONTIG(residual); CHECK_ALIGN16(residual);
+  TORCH_CHECK(residual.dim() == 2, "residual must be [rows, width]");
+  DocqaPostNorm a{};
+  a.rows = residual.size(0); a.W = residual.size(1); a.groups = (int)groups;
+  a.SP = a.SQ = a.SG = 1;
+  check_vec(w, a.W, "w");
+  CHECK_ALIGN16(w);
+  if (P.has_value()) {
+    const Slabs p = slabs_of(*P);
+    TORCH_CHECK(p.M == a.rows && p.N == a.W && gate.has_value() && gate_b.has_value(), "post_norm: P, gate");
+    CHECK_ALIGN16(*P);
+    const Slabs s = slabs_of(*gate);
+    TORCH_CHECK(s.M == a.rows && col >= 0 && col + a.W <= s.N, "post_norm: gate columns");
+    CHECK_ALIGN16(*gate);
+    check_vec(*gate_b, a.W, "gate_b");
+    CHECK_ALIGN16(*gate_b);
+    a.P = P->data_ptr(); a.pf32 = is_f32(*P); a.SP = p.S;
+    a.gate = gate->data_ptr(); a.gf32 = is_f32(*gate); a.SG = s.S; a.ldg = s.N; a.gslab = s.slab; a.col = (int)col;
+    a.gb = gate_b->data_ptr<float>();
+  }
+  if (Q.has_value()) {
+    const Slabs q = slabs_of(*Q);
+    TORCH_CHECK(P.has_value() && q.M == a.rows && q.N == a.W, "post_norm: Q");
+    CHECK_ALIGN16(*Q);
+    a.Q = Q->data_ptr(); a.qf32 = is_f32(*Q); a.SQ = q.S;
+  }
+  c10::DeviceGuard g(residual.device());
+  auto out = at::empty({out_f32 ? 0 : a.rows, a.W}, residual.options().dtype(at::kBFloat16));
+  a.res = residual.data_ptr<float>(); a.w = w.data_ptr<float>(); a.out = out_f32 ? nullptr : out.data_ptr();
+  a.alpha = (float)alpha; a.eps = (float)eps;
+  CHECK_RC(docqa_post_norm(a, stream()), "post_norm");
+  return out;
+}
+
+std::tuple<Tensor, Tensor, Tensor> moe_route(const Tensor& x, const Tensor& w, int64_t experts, int64_t top) {
+  CHECK_ACT(x); CHECK_CONTIG(x); CHECK_CONTIG(w); CHECK_GPU(w); CHECK_ALIGN16(x); CHECK_ALIGN16(w);
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1) && w.scalar_type() == x.scalar_type(), "moe_route: shapes");
+  const int64_t T = x.size(0), N = w.size(0);
+  TORCH_CHECK(top >= 1 && top <= experts && experts <= N, "moe_route: experts");
+  c10::DeviceGuard g(x.device());
+  auto f32 = x.options().dtype(at::kFloat);
+  auto ids = at::empty({T, top}, x.options().dtype(at::kInt)), wts = at::empty({T, top}, f32), rest = at::empty({T, N - experts}, f32);
+  CHECK_RC(docqa_moe_route(x.data_ptr(), w.data_ptr(), is_f32(x), ids.data_ptr<int>(), wts.data_ptr<float>(),
+                           rest.data_ptr<float>(), (int)T, (int)x.size(1), (int)N, (int)experts, (int)top, stream()),
+           "moe_route");
+  return {ids, wts, rest};
+}
+
+Tensor slab_glu(const Tensor& P, int64_t col, int64_t n, const OptT& scale, bool out_f32) {
+  const Slabs p = slabs_of(P);
+  CHECK_ALIGN16(P);
+  TORCH_CHECK(col >= 0 && n >= 1 && col + 2 * n <= p.N, "slab_glu: columns");
+  if (scale.has_value()) check_vec(*scale, p.M, "scale");
+  c10::DeviceGuard g(P.device());
+  auto out = at::empty({p.M, n}, P.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
+  CHECK_RC(docqa_slab_glu(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, (int)col, (int)n,
+                          scale.has_value() ? scale->data_ptr<float>() : nullptr, out.data_ptr(), out_f32, p.M, stream()),
+           "slab_glu");
+  return out;
+}
+
+Tensor moe_experts(const Tensor& x, const Tensor& ids, const Tensor& wts, const Tensor& up, const Tensor& down) {
+  CHECK_ACT(x); CHECK_CONTIG(x); CHECK_CONTIG(up); CHECK_CONTIG(down); CHECK_GPU(up); CHECK_GPU(down);
+  CHECK_ALIGN16(x); CHECK_ALIGN16(up); CHECK_ALIGN16(down);
+  TORCH_CHECK(x.dim() == 2 && up.dim() == 4 && up.size(1) == 2 && down.dim() == 3 && ids.dim() == 2 && ids.size(0) == x.size(0),
+              "moe_experts: shapes");
+  const int64_t T = x.size(0), K = x.size(1), E = up.size(0), F = up.size(2), W = down.size(1), top = ids.size(1);
+  TORCH_CHECK(up.size(3) == K && down.size(0) == E && down.size(2) == F && up.scalar_type() == x.scalar_type() &&
+                  down.scalar_type() == x.scalar_type(), "moe_experts: weights");
+  check_i32(ids, T * top, "ids");
+  check_vec(wts, T * top, "wts");
+  c10::DeviceGuard g(x.device());
+  auto act = at::empty({T * top, F}, x.options()), out = at::empty({top, T, W}, x.options());
+  const int n = docqa_moe_scratch(is_f32(x), (int)T, (int)top, (int)E, (int)K, (int)F, (int)W);
+  auto scratch = at::empty({n}, ids.options());
+  CHECK_RC(docqa_moe_experts(x.data_ptr(), ids.data_ptr<int>(), wts.data_ptr<float>(), up.data_ptr(), down.data_ptr(),
+                             act.data_ptr(), out.data_ptr(), n ? scratch.data_ptr<int>() : nullptr, is_f32(x), (int)T,
+                             (int)top, (int)E, (int)K, (int)F, (int)W, stream()),
+           "moe_experts");
+  return out;
+}
+
 }  // namespace
 
 TORCH_LIBRARY_FRAGMENT(docqa, m) {
   m.def("sandwich_rmsnorm(Tensor P, Tensor(a!) residual, Tensor w_post, Tensor? add, Tensor w_next, float eps, "
         "bool out_f32) -> Tensor");
-  m.def("embed_scale_rmsnorm(Tensor ids, Tensor table, float scale, Tensor w, float eps, bool keep) "
+  m.def("embed_scale_rmsnorm(Tensor ids, Tensor table, float scale, Tensor? w, float eps, bool keep) "
         "-> (Tensor, Tensor, Tensor)");
   m.def("decode_act(Tensor x, Tensor w, int act) -> Tensor");
   m.def("add_scaled(Tensor P, Tensor? Q, Tensor(a!) residual, float m, bool out_f32) -> Tensor");
@@ -539,7 +734,7 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
         "Tensor(b!) state, Tensor slots, Tensor positions, float eps) -> (Tensor, Tensor)");
   m.def("packed_window_attn(Tensor q, Tensor kv, Tensor kr, int H, int dim, int vdim, Tensor cu, Tensor cu_k, int max_q, "
         "float scale, int window, Tensor? sink) -> Tensor");
-  m.def("rope_table(Tensor positions, Tensor freq) -> Tensor");
+  m.def("rope_table(Tensor positions, Tensor freq, float mult) -> Tensor");
   m.def("latent_store(Tensor P, Tensor cs, Tensor slots, Tensor(a!) cache, Tensor? c_norm, int H, int dim, int rank, "
         "float eps) -> Tensor");
   m.def("head_project(Tensor x, Tensor w, int carry) -> Tensor");
@@ -550,11 +745,22 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
   m.def("qk_norm_store(Tensor P, Tensor w, Tensor slots, Tensor(a!) k_cache, Tensor(b!) k_scale, int H, float eps) "
         "-> Tensor");
   m.def("window_attn(Tensor q, Tensor k_cache, Tensor? v_cache, Tensor? k_scale, Tensor block_tables, Tensor? cu, "
-        "Tensor ctx, int max_q, float scale, int window, Tensor? sink, int v_dim) -> Tensor");
+        "Tensor ctx, int max_q, float scale, int window, Tensor? sink, int v_dim, float cap, float out_scale, Tensor(a!) out) -> ()");
+  m.def("qkv_rope_store(Tensor P, Tensor? bias, Tensor? qw, Tensor? kw, Tensor cs, Tensor slots, Tensor(a!) k_cache, "
+        "Tensor(b!) v_cache, int H, float eps) -> Tensor");
+  m.def("linear_step(Tensor X, Tensor Z, int[] dims, float[] consts, Tensor w_gate, Tensor? b_gate, Tensor? cs, Tensor norm, "
+        "Tensor(a!) state, Tensor slots, Tensor positions, Tensor(b!) out) -> ()");
+  m.def("linear_scan(Tensor X, Tensor Z, int[] dims, float[] consts, Tensor w_gate, Tensor? b_gate, Tensor? cs, Tensor norm, "
+        "Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, int max_len, Tensor(b!) out) -> ()");
+  m.def("post_norm(Tensor? P, Tensor? Q, Tensor? gate, int col, Tensor? gate_b, Tensor(a!) residual, float alpha, Tensor w, "
+        "int groups, float eps, bool out_f32) -> Tensor");
+  m.def("moe_route(Tensor x, Tensor w, int experts, int top) -> (Tensor, Tensor, Tensor)");
+  m.def("slab_glu(Tensor P, int col, int n, Tensor? scale, bool out_f32) -> Tensor");
+  m.def("moe_experts(Tensor x, Tensor ids, Tensor wts, Tensor up, Tensor down) -> Tensor");
   m.def("causal_conv(Tensor x, Tensor w, Tensor? bias, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, "
         "int max_len, bool silu) -> Tensor");
-  m.def("conv_step(Tensor P, Tensor w, Tensor? bias, Tensor(a!) state, Tensor slots, Tensor positions, bool silu) "
-        "-> (Tensor, Tensor)");
+  m.def("conv_step(Tensor P, Tensor w, Tensor? bias, Tensor(a!) state, Tensor slots, Tensor positions, bool silu, "
+        "int rest) -> (Tensor, Tensor)");
   m.def("selective_scan(Tensor x, Tensor dt, Tensor bc, int b_off, int c_off, int N, Tensor z, Tensor A2, Tensor D, "
         "Tensor dt_b, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, int max_len, int chunk) -> Tensor");
   m.def("selective_step(Tensor x, Tensor? dt, Tensor? dt_in, Tensor? w_dt, Tensor bc, int b_off, int c_off, int N, Tensor z, Tensor A2, Tensor D, "
@@ -580,6 +786,13 @@ TORCH_LIBRARY_IMPL(docqa, CUDA, m) {
   m.impl("slab_activation", &slab_activation);
   m.impl("qk_norm_store", &qk_norm_store);
   m.impl("window_attn", &window_attn);
+  m.impl("qkv_rope_store", &qkv_rope_store);
+  m.impl("linear_step", &linear_step);
+  m.impl("linear_scan", &linear_scan);
+  m.impl("post_norm", &post_norm);
+  m.impl("moe_route", &moe_route);
+  m.impl("slab_glu", &slab_glu);
+  m.impl("moe_experts", &moe_experts);
   m.impl("causal_conv", &causal_conv);
   m.impl("conv_step", &conv_step);
   m.impl("selective_scan", &selective_scan);

@@ -40,15 +40,21 @@ int docqa_qk_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, co
                         void* q, void* kc, float* ks, int f32, int tokens, int H, int G, int D, int BS, float eps,
                         hipStream_t s);
 // cu null: decode (one query token a row, ctx = context length including it); DV: value elements of a row
+// (vc == kc: the first DV of the key's D); ldo: elements of an output row; cap 0: scores as they are
 int docqa_window_attn(const void* q, const void* kc, const void* vc, const float* k_scale, const int* block_tables,
-                      int maxb, const int* cu, const int* ctx, const float* sink, void* out, int f32, int B,
-                      int max_q, int H, int G, int D, int DV, int BS, float scale, int window, hipStream_t s);
+                      int maxb, const int* cu, const int* ctx, const float* sink, void* out, int ldo, int f32, int B,
+                      int max_q, int H, int G, int D, int DV, int BS, float scale, int window, float cap, float out_scale,
+                      hipStream_t s);
+// P [T, ld]: [q: H D | k: G D | v: G DV | ..]; bias, norm weights qw / kw [D] may be null; cs [T, r]
+int docqa_qkv_rope_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* bias, const float* qw,
+                         const float* kw, const float* cs, int r, const int* slots, void* q, void* kc, void* vc, int f32,
+                         int tokens, int H, int G, int D, int DV, int BS, float eps, hipStream_t s);
 // kv [keys, ld] rows [H x d8 keys | H x v8 values], kr [keys, r8]; bf16
 int docqa_packed_window_attn(const void* q, const void* kv, const void* kr, const int* cu, const int* cu_k,
                              const float* sink, void* out, int B, int max_q, int H, int d8, int r8, int vdim, int ld,
                              float scale, int window, hipStream_t s);
 
-int docqa_rope_table(const int* positions, const double* freq, float* out, int T, int half, hipStream_t s);
+int docqa_rope_table(const int* positions, const double* freq, float* out, int T, int half, double mult, hipStream_t s);
 // c_norm null: the projection holds query heads only
 int docqa_latent_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* cs, const int* slots,
                        const float* c_norm, void* q, void* cache, int f32, int T, int H, int d, int r, int R, int BS,
@@ -71,7 +77,7 @@ int docqa_causal_conv(const void* x, int ldx, const float* w, const float* b, vo
                       const int* cu, const int* ctx, void* y, int f32, int B, int max_len, int C, int taps,
                       int silu, hipStream_t s);
 int docqa_conv_step(const void* P, int p_f32, int S, size_t slab, int ld, const float* w, const float* b, void* state,
-                    const int* slots, const int* positions, void* y, void* z, int f32, int B, int C, int taps,
+                    const int* slots, const int* positions, void* y, void* z, int f32, int B, int C, int NZ, int taps,
                     int silu, hipStream_t s);
 int docqa_selective_scan(const void* x, const void* dt, const void* bc, int ld_bc, int b_off, int c_off,
                          const void* z, int ld_z, const float* A2, const float* D, const float* dt_b, float* state,
@@ -82,3 +88,50 @@ int docqa_selective_step(const void* x, const void* dt, const void* dt_in, const
                          int ld_bc, int b_off, int c_off, const void* z, int ld_z, const float* A2, const float* D,
                          const float* dt_b, float* state, const int* slots, const int* positions, void* y, int f32,
                          int B, int C, int N, int Np, hipStream_t s);
+
+// ---- linear attention (linear_attn.hip)
+enum { LIN_CHANNEL = 0, LIN_FIXED = 1, LIN_DELTA = 2 };
+struct DocqaLinear {
+  const void *X, *Z;        // [tokens, ldx], [tokens, ldz]: products or slabs
+  int xf32, Sx, ldx, zf32, Sz, ldz;
+  size_t xslab, zslab;
+  int kind, H, G, dk, dv, qo, ko, vo, go, ao, bo, rank, r;   // column offsets; rotated dimensions
+  float qs, ks, inv_tau, eps;
+  const float *w_gate, *b_gate;   // channel: [H dk, rank], [H dk]; fixed: log decay [H], -; delta: -exp(A) [H], [H]
+  const float* cs;          // [tokens, r]
+  const float* norm;        // [dv]
+  float* state;             // [slots, H, dk, dvp], dvp = dv rounded up to 4
+  const int* slots;
+  void* out;                // [tokens, ldo]
+  int of32, ldo;
+};
+int docqa_linear_step(const DocqaLinear& a, const int* positions, int B, hipStream_t s);
+// chunk of a scan and the fp32 scratch (elements) it needs
+int docqa_linear_chunk(int dk);
+size_t docqa_linear_scratch(int kind, int tokens, int B, int H, int dk, int dv);
+int docqa_linear_scan(const DocqaLinear& a, const int* cu, const int* ctx, float* scratch, int tokens, int B, int max_len,
+                      hipStream_t s);
+
+// ---- norms after the sum (sandwich_norm.hip): res <- groupnorm(alpha res + sigmoid(gate[:, col:] + gb) (P + Q)) w
+struct DocqaPostNorm {
+  const void *P, *Q, *gate;       // null: left out (gate with P)
+  int pf32, SP, qf32, SQ, gf32, SG, ldg, col;
+  size_t gslab;
+  const float* gb;
+  float* res;
+  const float* w;
+  void* out;                      // null: none
+  int of32, rows, W, groups;
+  float alpha, eps;
+};
+int docqa_post_norm(const DocqaPostNorm& a, hipStream_t s);
+
+// ---- experts (moe.hip)
+int docqa_moe_route(const void* x, const void* w, int f32, int* ids, float* wts, float* rest, int T, int K, int N, int E,
+                    int top, hipStream_t s);
+int docqa_slab_glu(const void* P, int p_f32, int S, size_t slab, int ld, int col, int n, const float* scale, void* out,
+                   int out_f32, int T, hipStream_t s);
+// int32 scratch of a sorted launch; 0: the rows are found in the launch
+int docqa_moe_scratch(int f32, int T, int top, int E, int K, int F, int W);
+int docqa_moe_experts(const void* x, const int* ids, const float* wts, const void* up, const void* down, void* act,
+                      void* out, int* scratch, int f32, int T, int top, int E, int K, int F, int W, hipStream_t s);

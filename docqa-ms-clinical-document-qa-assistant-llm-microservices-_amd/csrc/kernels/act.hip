@@ -306,3 +306,45 @@ int docqa_soft_cap(const void* x, int f32, float* out, size_t n, float cap, hipS
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
+
+// silu(gate) * up of columns [col, col + n) and [col + n, col + 2 n), rows times scale [T]
+template <int V, typename PT, typename OT>
+__global__ __launch_bounds__(256) void slab_glu_kernel(const PT* __restrict__ P, int S, size_t slab, int ld, int col, int n,
+                                                       const float* __restrict__ scale, OT* __restrict__ out, int T) {
+  const int per = n / V;
+  const size_t total = (size_t)T * per;
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
+    const size_t t = i / per;
+    const int c = (int)(i - t * per) * V;
+    float g[V], u[V];
+    docqa::ld_slabs<V>(P + t * ld + col + c, S, slab, g);
+    docqa::ld_slabs<V>(P + t * ld + col + n + c, S, slab, u);
+    const float s = scale ? scale[t] : 1.f;
+#pragma unroll
+    for (int j = 0; j < V; ++j) g[j] = g[j] / (1.f + __expf(-g[j])) * u[j] * s;
+    docqa::stv<V>(out + t * n + c, g);
+  }
+}
+
+template <typename PT, typename OT>
+static int launch_slab_glu(const PT* P, int S, size_t slab, int ld, int col, int n, const float* scale, OT* out, int T,
+                           hipStream_t s) {
+  const bool vec = n % 4 == 0 && ld % 4 == 0 && col % 4 == 0;
+  const size_t g = ((size_t)T * n / (vec ? 4 : 1) + 255) / 256;
+  const int grid = (int)(g < 8192 ? (g ? g : 1) : 8192);
+  if (vec) slab_glu_kernel<4, PT, OT><<<grid, 256, 0, s>>>(P, S, slab, ld, col, n, scale, out, T);
+  else slab_glu_kernel<1, PT, OT><<<grid, 256, 0, s>>>(P, S, slab, ld, col, n, scale, out, T);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+int docqa_slab_glu(const void* P, int p_f32, int S, size_t slab, int ld, int col, int n, const float* scale, void* out,
+                   int out_f32, int T, hipStream_t s) {
+  if (T == 0) return 0;
+  if (S < 1 || n < 1 || col < 0 || col + 2 * n > ld) return -1;
+  if (p_f32)
+    return out_f32 ? launch_slab_glu((const float*)P, S, slab, ld, col, n, scale, (float*)out, T, s)
+                   : launch_slab_glu((const float*)P, S, slab, ld, col, n, scale, (uint16_t*)out, T, s);
+  return out_f32 ? launch_slab_glu((const uint16_t*)P, S, slab, ld, col, n, scale, (float*)out, T, s)
+                 : launch_slab_glu((const uint16_t*)P, S, slab, ld, col, n, scale, (uint16_t*)out, T, s);
+}

@@ -40,14 +40,14 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
 __global__ __launch_bounds__(256) void rope_table_kernel(const int* __restrict__ pos, const double* __restrict__ freq,
-                                                         float* __restrict__ out, int T, int half) {
+                                                         float* __restrict__ out, int T, int half, double mult) {
   const int i = blockIdx.x * 256 + threadIdx.x;
   if (i >= T * half) return;
   const int t = i / half, k = i - t * half;
   double s, c;
   sincos((double)pos[t] * freq[k], &s, &c);
-  out[(size_t)t * 2 * half + k] = (float)c;
-  out[(size_t)t * 2 * half + half + k] = (float)s;
+  out[(size_t)t * 2 * half + k] = (float)(c * mult);
+  out[(size_t)t * 2 * half + half + k] = (float)(s * mult);
 }
 
 struct StoreArgs {
@@ -609,10 +609,10 @@ int log2_of(int n) {
 }
 }  // namespace
 
-int docqa_rope_table(const int* positions, const double* freq, float* out, int T, int half, hipStream_t s) {
+int docqa_rope_table(const int* positions, const double* freq, float* out, int T, int half, double mult, hipStream_t s) {
   if (T == 0) return 0;
   if (half < 1 || (long long)T * half >= (1ll << 31)) return -1;
-  rope_table_kernel<<<(T * half + 255) / 256, 256, 0, s>>>(positions, freq, out, T, half);
+  rope_table_kernel<<<(T * half + 255) / 256, 256, 0, s>>>(positions, freq, out, T, half, mult);
   DOCQA_CHECK_LAUNCH();
   return 0;
 }

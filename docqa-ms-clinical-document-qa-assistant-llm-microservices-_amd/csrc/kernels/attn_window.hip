@@ -1,9 +1,11 @@
 // attn_window.hip -- causal attention over a sliding window with an optional per-head sink,
 // read from the paged cache; head-wise query / key RMS norm; keys shared as values.
 //
-//   s_j = scale * k_scale_j * (q . K_j)   for  pos - window < j <= pos
-//   out = sum_j exp(s_j) V_j / (sum_j exp(s_j) + exp(sink_h))
+//   s_j = cap(scale * k_scale_j * (q . K_j))   for  pos - window < j <= pos,  cap(s) = c tanh(s / c)
+//   out = out_scale * sum_j exp(s_j) V_j / (sum_j exp(s_j) + exp(sink_h))
 //
+// * qkv_rope_store: [q | k | v] projection -> query heads (bias, norm, rotation of the first r
+//   dimensions), keys alike and values into the paged cache; key and value rows may differ in size.
 // * qk_norm_store: q <- rms(q) * w over each head, K rows stored as projected with their
 //   inverse root mean square beside them (k_scale).  With the key norm's weight folded into
 //   w the normalised key is never materialised: one cached row serves as key and as value,
@@ -90,7 +92,11 @@ struct WindowArgs {
   int H, G, D, BS, log2BS;
   float scale;
   int window;
-  int DV;                 // value elements of a row (D, or fewer)
+  int DV;                 // value elements of a head
+  int ldv;                // elements of a cached value row (D where the keys are the values)
+  float cap;              // 0: none
+  float out_scale;
+  int ldo;                // elements of an output row
   // packed keys: row j of sequence b at cu_k[b] + j holds [H x kd | H x vd ..] (ld elements), the
   // other D - kd key elements at kr; the last query token is at the last key
   const int* cu_k;
@@ -140,7 +146,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
   const bool live = seq_range(a, b, q0, L, p0);
   if (tok >= (a.cu ? L : 1)) return;       // whole waves; no workgroup barrier below
   const int D = a.D, DV = a.DV;
-  T* o = out + ((size_t)(q0 + tok) * a.H + h) * DV;
+  T* o = out + (size_t)(q0 + tok) * a.ldo + h * DV;
   if (!live) {                             // a padded decode row
     for (int c = lane; c < DV; c += 64) st1(o + c, 0.f);
     return;
@@ -180,6 +186,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
         for (; c < D; ++c) d0 += ld1(kp + c) * sq[c];
       }
       s = (d0 + d1) * sl2 * (a.k_scale ? a.k_scale[row] : 1.f);
+      if (a.cap > 0.f) s = a.cap * kLog2e * tanhf(s / (a.cap * kLog2e));
     }
     const float mn = fmaxf(m, wave_max(s));
     const float alpha = exp2f(m - mn);
@@ -195,13 +202,13 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const T* __restrict__ 
       const int c = lane + 64 * i;
       if (c < DV) {
         float v = acc[i] * alpha;
-        for (int j = 0; j < n; ++j) v += sp[wave][j] * ld1(vc + (size_t)srow[wave][j] * D + c);
+        for (int j = 0; j < n; ++j) v += sp[wave][j] * ld1(vc + (size_t)srow[wave][j] * a.ldv + c);
         acc[i] = v;
       }
     }
     wave_lds_sync();
   }
-  const float inv = 1.f / l;
+  const float inv = a.out_scale / l;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int c = lane + 64 * i;
@@ -252,7 +259,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
   const int row0 = (gridDim.z - 1 - blockIdx.z) * tile_rows;         // longest windows first
   if (!live) {                                                       // a padded decode row
     if (!a.cu)
-      for (int e = tid; e < Gs * DV; e += 64 * NW) out[((size_t)b * a.H + kvh * Gs) * DV + e] = 0;
+      for (int e = tid; e < Gs * DV; e += 64 * NW) out[(size_t)b * a.ldo + kvh * Gs * DV + e] = 0;
     return;
   }
   const int rows = L * Gs;
@@ -345,8 +352,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
           rv[i] = *reinterpret_cast<const u32x4*>(vp[i] + (size_t)(kbase + min(kb + row, pos_hi)) * a.ld);
         } else {
           rv[i] = u32x4{0, 0, 0, 0};
-          if (e < KB * NCV && kb + row <= pos_hi && c < D)
-            rv[i] = *reinterpret_cast<const u32x4*>(vc + cache_row(kb + row) * D + c);
+          if (e < KB * NCV && kb + row <= pos_hi && c < DV)
+            rv[i] = *reinterpret_cast<const u32x4*>(vc + cache_row(kb + row) * DV + c);
         }
       }
     }
@@ -392,6 +399,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
           x[t2][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[t2][ks], x[t2][kt], 0, 0, 0);
       }
     }
+    const float cap2 = a.cap * kLog2e;
 #pragma unroll
     for (int t2 = 0; t2 < QT; ++t2) {
       float mx = -INFINITY;
@@ -402,6 +410,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           float v = x[t2][kt][r] * kss[r];
+          // cap tanh(v / cap), tanh y = 1 - 2 / (e^2y + 1)
+          if (cap2 > 0.f) v = cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v * (2.f * kLog2e / cap2)) + 1.f);
           if constexpr (PART) {
             const int key = kb + kt * 16 + g4 * 4 + r;
             v = ((key <= pos[t2]) & (key > below[t2])) ? v : -INFINITY;
@@ -483,8 +493,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
     for (int t = 0; t < QT; ++t) {
       const int r = wrow + t * 16 + fr;
       if (r >= rows) continue;
-      uint16_t* op = out + ((size_t)(q0 + r / Gs) * a.H + kvh * Gs + r % Gs) * DV;
-      const float inv = 1.f / l[t];
+      uint16_t* op = out + (size_t)(q0 + r / Gs) * a.ldo + (kvh * Gs + r % Gs) * DV;
+      const float inv = a.out_scale / l[t];
 #pragma unroll
       for (int i = 0; i < NDT; ++i) {
         const int c = i * 16 + g4 * 4;
@@ -506,8 +516,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
       if (t + NW < ntiles) load(t + NW);
       compute(t, wave);
     }
-    __syncthreads();                             // tiles dead: partials [NW][16][DP] + (m, l)
-    constexpr int OP = DP + 4;
+    __syncthreads();                             // tiles dead: partials [NW][16][DPV] + (m, l)
+    constexpr int OP = DPV + 4;
     float* po = reinterpret_cast<float*>(smem);
     float2* pml = reinterpret_cast<float2*>(po + NW * 16 * OP);
 #pragma unroll
@@ -517,9 +527,9 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
     if (g4 == 0) pml[wave * 16 + fr] = make_float2(m[0], l[0]);
     __syncthreads();
     const int n = min(16, rows - row0);
-    for (int e = tid; e < n * (DP / 4); e += 64 * NW) {
-      const int r = e / (DP / 4), c = (e % (DP / 4)) * 4;
-      if (c >= D) continue;
+    for (int e = tid; e < n * (DPV / 4); e += 64 * NW) {
+      const int r = e / (DPV / 4), c = (e % (DPV / 4)) * 4;
+      if (c >= DV) continue;
       float mm = -1e30f;
 #pragma unroll
       for (int w = 0; w < NW; ++w) mm = fmaxf(mm, pml[w * 16 + r].x);
@@ -533,12 +543,12 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
         ll += ml.y * f;
         v.x += p.x * f; v.y += p.y * f; v.z += p.z * f; v.w += p.w * f;
       }
-      const float inv = 1.f / ll;
+      const float inv = a.out_scale / ll;
       uint2 w2;
       w2.x = pack2(v.x * inv, v.y * inv);
       w2.y = pack2(v.z * inv, v.w * inv);
       const int row = row0 + r;
-      *reinterpret_cast<uint2*>(out + ((size_t)(q0 + row / Gs) * a.H + kvh * Gs + row % Gs) * D + c) = w2;
+      *reinterpret_cast<uint2*>(out + (size_t)(q0 + row / Gs) * a.ldo + (kvh * Gs + row % Gs) * DV + c) = w2;
     }
   }
 }
@@ -548,7 +558,7 @@ int launch_mfma(const void* q, const void* kc, const void* vc, void* out, const 
                 hipStream_t s) {
   constexpr int TILES = SPLIT ? NW : 2;
   constexpr size_t tile_b = (size_t)TILES * KB * (DP + 8 + (SHARED ? 0 : DPV + 8)) * 2 + (size_t)TILES * KB * 4;
-  constexpr size_t merge_b = SPLIT ? (size_t)NW * 16 * (DP + 4) * 4 + (size_t)NW * 16 * 8 : 0;
+  constexpr size_t merge_b = SPLIT ? (size_t)NW * 16 * (DPV + 4) * 4 + (size_t)NW * 16 * 8 : 0;
   constexpr size_t lds = tile_b > merge_b ? tile_b : merge_b;
   static_assert(lds <= 160 * 1024, "LDS");
   const int tile_rows = 16 * QT * (SPLIT ? 1 : NW), Gs = PACKED ? 1 : a.H / a.G;
@@ -568,32 +578,162 @@ int launch_mfma(const void* q, const void* kc, const void* vc, void* out, const 
 
 // decode-like launches (the rows of one sequence fit one 16-row tile): waves split the keys, as
 // many to a workgroup as give a CU 16 of them
-template <int DP, bool SHARED>
+template <int DP, int DPV, bool SHARED>
 int dispatch_mfma(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
                   hipStream_t s) {
-  constexpr int QT = DP <= 128 ? 2 : 1;
+  constexpr int QT = DP <= 128 && DPV <= 128 ? 2 : 1;
   if (max_q * (a.H / a.G) <= 16) {
-    if constexpr (DP <= 128) {
+    if constexpr (DP <= 128 && DPV <= 128) {
       const long long wgs = (long long)B * a.G;
       if constexpr (SHARED) {
-        if (wgs <= 256) return launch_mfma<DP, DP, 1, 32, 16, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+        if (wgs <= 256) return launch_mfma<DP, DPV, 1, 32, 16, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
       }
-      if (wgs <= 512) return launch_mfma<DP, DP, 1, 32, 8, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+      if (wgs <= 512) return launch_mfma<DP, DPV, 1, 32, 8, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
     }
-    return launch_mfma<DP, DP, 1, 32, 4, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
+    return launch_mfma<DP, DPV, 1, 32, 4, SHARED, true>(q, kc, vc, out, a, B, max_q, s);
   }
-  return launch_mfma<DP, DP, QT, 64, 4, SHARED, false>(q, kc, vc, out, a, B, max_q, s);
+  return launch_mfma<DP, DPV, QT, 64, 4, SHARED, false>(q, kc, vc, out, a, B, max_q, s);
 }
 
-template <bool SHARED>
-int dispatch_dim(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
-                 hipStream_t s) {
-  if (a.D <= 32) return dispatch_mfma<32, SHARED>(q, kc, vc, out, a, B, max_q, s);
-  if (a.D <= 64) return dispatch_mfma<64, SHARED>(q, kc, vc, out, a, B, max_q, s);
-  if (a.D <= 96) return dispatch_mfma<96, SHARED>(q, kc, vc, out, a, B, max_q, s);
-  if (a.D <= 128) return dispatch_mfma<128, SHARED>(q, kc, vc, out, a, B, max_q, s);
-  if (a.D <= 192) return dispatch_mfma<192, SHARED>(q, kc, vc, out, a, B, max_q, s);
-  return dispatch_mfma<256, SHARED>(q, kc, vc, out, a, B, max_q, s);
+int dispatch_shared(const void* q, const void* kc, void* out, const WindowArgs& a, int B, int max_q, hipStream_t s) {
+#define GO(N) return dispatch_mfma<N, N, true>(q, kc, kc, out, a, B, max_q, s)
+  if (a.D <= 32) GO(32);
+  if (a.D <= 64) GO(64);
+  if (a.D <= 96) GO(96);
+  if (a.D <= 128) GO(128);
+  if (a.D <= 192) GO(192);
+  GO(256);
+#undef GO
+}
+// key and value rows of their own
+template <int DP>
+int dispatch_values(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
+                    hipStream_t s) {
+  if (a.DV <= 64) return dispatch_mfma<DP, 64, false>(q, kc, vc, out, a, B, max_q, s);
+  if (a.DV <= 128) return dispatch_mfma<DP, 128, false>(q, kc, vc, out, a, B, max_q, s);
+  return dispatch_mfma<DP, 256, false>(q, kc, vc, out, a, B, max_q, s);
+}
+int dispatch_pair(const void* q, const void* kc, const void* vc, void* out, const WindowArgs& a, int B, int max_q,
+                  hipStream_t s) {
+  if (a.D <= 64) return dispatch_values<64>(q, kc, vc, out, a, B, max_q, s);
+  if (a.D <= 128) return dispatch_values<128>(q, kc, vc, out, a, B, max_q, s);
+  return dispatch_values<256>(q, kc, vc, out, a, B, max_q, s);
+}
+
+// heads of a [q: H D | k: G D | v: G DV] projection, LPH lanes each: bias, RMS norm and rotation of
+// query and key heads, V items of two kinds -- V pairs (i, i + r / 2) of the rotated dimensions, V
+// unrotated ones -- then the stores; value heads are copied
+struct QkvArgs {
+  int S, ld;
+  size_t slab;
+  const float* bias;      // [H D + G D + G DV] or null
+  const float *qw, *kw;   // [D] or null: no norm
+  const float* cs;        // [tokens, r]: cosines, sines
+  const int* slots;
+  int tokens, H, G, D, DV, r, log2BS;
+  float eps;
+};
+template <int V, int NI, int LPH, typename PT, typename T>
+__global__ __launch_bounds__(256) void qkv_rope_store_kernel(const PT* __restrict__ P, T* __restrict__ q,
+                                                             T* __restrict__ kc, T* __restrict__ vc, QkvArgs a) {
+  const int heads = a.H + 2 * a.G;
+  const unsigned u = blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
+  const int lane = threadIdx.x % LPH, t = u / heads, h = u - t * heads;
+  if (t >= a.tokens) return;                 // whole lane groups
+  const PT* row = P + (size_t)t * a.ld;
+  const int D = a.D, r2 = a.r / 2, slot = h < a.H ? 0 : a.slots[t];
+  if (slot < 0) return;
+  const int BS = 1 << a.log2BS;
+  auto cache_row = [&](int g) { return ((((size_t)(slot >> a.log2BS)) * a.G + g) << a.log2BS) + (slot & (BS - 1)); };
+  auto get = [&](int c, float* f) {
+    ld_slabs<V>(row + c, a.S, a.slab, f);
+    if (a.bias) {
+      float b[V];
+      ldv<V>(a.bias + c, b);
+#pragma unroll
+      for (int j = 0; j < V; ++j) f[j] += b[j];
+    }
+  };
+  if (h >= a.H + a.G) {
+    const int g = h - a.H - a.G, c0 = (a.H + a.G) * D + g * a.DV;
+    T* o = vc + cache_row(g) * a.DV;
+    for (int c = lane * V; c < a.DV; c += LPH * V) {
+      float f[V];
+      get(c0 + c, f);
+      stv<V>(o + c, f);
+    }
+    return;
+  }
+  const int items = (D - r2) / V, npair = r2 / V;
+  float x[NI][V], y[NI][V], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int e = lane + LPH * i;
+    if (e < items) {
+      const int c = e < npair ? e * V : e * V + r2;
+      get(h * D + c, x[i]);
+#pragma unroll
+      for (int j = 0; j < V; ++j) ss += x[i][j] * x[i][j];
+      if (e < npair) {
+        get(h * D + c + r2, y[i]);
+#pragma unroll
+        for (int j = 0; j < V; ++j) ss += y[i][j] * y[i][j];
+      }
+    }
+  }
+  const float* w = h < a.H ? a.qw : a.kw;
+  const float inv = w ? 1.f / sqrtf(group_sum<LPH>(ss) / (float)D + a.eps) : 1.f;
+  T* o = h < a.H ? q + ((size_t)t * a.H + h) * D : kc + cache_row(h - a.H) * D;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int e = lane + LPH * i;
+    if (e >= items) continue;
+    const int c = e < npair ? e * V : e * V + r2;
+    float f[V];
+    if (w) {
+      ldv<V>(w + c, f);
+#pragma unroll
+      for (int j = 0; j < V; ++j) x[i][j] *= inv * f[j];
+    }
+    if (e < npair) {
+      float co[V], si[V];
+      if (w) {
+        ldv<V>(w + c + r2, f);
+#pragma unroll
+        for (int j = 0; j < V; ++j) y[i][j] *= inv * f[j];
+      }
+      ldv<V>(a.cs + (size_t)t * a.r + c, co);
+      ldv<V>(a.cs + (size_t)t * a.r + r2 + c, si);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const float xu = x[i][j], xv = y[i][j];
+        x[i][j] = xu * co[j] - xv * si[j];
+        y[i][j] = xv * co[j] + xu * si[j];
+      }
+      stv<V>(o + c + r2, y[i]);
+    }
+    stv<V>(o + c, x[i]);
+  }
+}
+
+template <typename PT, typename T>
+int qkv_store(const PT* P, T* q, T* kc, T* vc, const QkvArgs& a, hipStream_t s) {
+  const long long units = (long long)a.tokens * (a.H + 2 * a.G);
+#define GO(V, N, L) qkv_rope_store_kernel<V, N, L, PT, T><<<(int)((units + 256 / L - 1) / (256 / L)), 256, 0, s>>>(P, q, kc, vc, a)
+  const int items = a.D - a.r / 2;
+  if (a.D % 4 == 0 && a.DV % 4 == 0 && a.r % 8 == 0 && a.ld % 4 == 0) {
+    if (items <= 32) GO(4, 1, 8);
+    else if (items <= 64) GO(4, 1, 16);
+    else if (items <= 128) GO(4, 1, 32);
+    else GO(4, 2, 64);
+  } else {
+    if (items <= 64) GO(1, 1, 64);
+    else if (items <= 128) GO(1, 2, 64);
+    else GO(1, 8, 64);
+  }
+#undef GO
+  DOCQA_CHECK_LAUNCH();
+  return 0;
 }
 
 template <typename PT, typename T>
@@ -635,18 +775,35 @@ int docqa_qk_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, co
   return qk_store((const uint16_t*)P, S, slab, ld, wq, slots, (uint16_t*)q, (uint16_t*)kc, ks, tokens, H, G, D, BS, eps, s);
 }
 
+int docqa_qkv_rope_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* bias, const float* qw,
+                         const float* kw, const float* cs, int r, const int* slots, void* q, void* kc, void* vc, int f32,
+                         int tokens, int H, int G, int D, int DV, int BS, float eps, hipStream_t s) {
+  if (tokens == 0) return 0;
+  if (S < 1 || D < 1 || D > 512 || DV < 1 || H < 1 || G < 1 || r < 0 || r % 2 || r > D || (BS & (BS - 1)) != 0) return -1;
+  if (ld < (H + G) * D + G * DV || (long long)tokens * (H + 2 * G) >= (1ll << 31) || (f32 && !p_f32)) return -1;
+  QkvArgs a{S, ld, slab, bias, qw, kw, cs, slots, tokens, H, G, D, DV, r, 0, eps};
+  while ((1 << a.log2BS) < BS) ++a.log2BS;
+  if (f32) return qkv_store((const float*)P, (float*)q, (float*)kc, (float*)vc, a, s);
+  if (p_f32) return qkv_store((const float*)P, (uint16_t*)q, (uint16_t*)kc, (uint16_t*)vc, a, s);
+  return qkv_store((const uint16_t*)P, (uint16_t*)q, (uint16_t*)kc, (uint16_t*)vc, a, s);
+}
+
 int docqa_window_attn(const void* q, const void* kc, const void* vc, const float* k_scale, const int* block_tables,
-                      int maxb, const int* cu, const int* ctx, const float* sink, void* out, int f32, int B,
-                      int max_q, int H, int G, int D, int DV, int BS, float scale, int window, hipStream_t s) {
+                      int maxb, const int* cu, const int* ctx, const float* sink, void* out, int ldo, int f32, int B,
+                      int max_q, int H, int G, int D, int DV, int BS, float scale, int window, float cap, float out_scale,
+                      hipStream_t s) {
   if (B == 0 || max_q == 0) return 0;
-  if (H % G != 0 || D < 1 || D > 2560 || DV < 1 || DV > D || DV > 2048 || (BS & (BS - 1)) != 0) return -1;
+  const bool shared = kc == vc;
+  if (H % G != 0 || D < 1 || D > 2560 || DV < 1 || (shared && DV > D) || DV > 2048 || (BS & (BS - 1)) != 0) return -1;
+  if (ldo < H * DV || cap < 0.f) return -1;
   int log2BS = 0;
   while ((1 << log2BS) < BS) ++log2BS;
   const WindowArgs a{block_tables, maxb, cu, ctx, k_scale, sink, H, G, D, BS, log2BS, scale, window, DV,
-                     nullptr, nullptr, 0, 0, 0};
-  if (!f32 && D % 8 == 0 && D <= 256 && DV == D && docqa_aligned16(q) && docqa_aligned16(out))
-    return kc == vc ? dispatch_dim<true>(q, kc, vc, out, a, B, max_q, s)
-                    : dispatch_dim<false>(q, kc, vc, out, a, B, max_q, s);
+                     shared ? D : DV, cap, out_scale, ldo, nullptr, nullptr, 0, 0, 0};
+  // rows are stored 8 bytes at a time
+  const bool stores = ldo % 4 == 0 && DV % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & 7) == 0;
+  if (!f32 && D % 8 == 0 && DV % 8 == 0 && D <= 256 && DV <= 256 && (!shared || DV == D) && docqa_aligned16(q) && stores)
+    return shared ? dispatch_shared(q, kc, out, a, B, max_q, s) : dispatch_pair(q, kc, vc, out, a, B, max_q, s);
   dim3 grid((max_q * H + 3) / 4, B);
 #define GO(T, N) window_attn_kernel<T, N><<<grid, 256, (size_t)D * 16, s>>>((const T*)q, (const T*)kc, (const T*)vc, (T*)out, a)
   if (f32) {
@@ -675,7 +832,7 @@ int docqa_packed_window_attn(const void* q, const void* kv, const void* kr, cons
   if (H < 1 || d8 < 8 || d8 % 8 || r8 < 0 || r8 % 8 || D > 256 || vdim < 4 || vdim % 4 || vdim > 256) return -1;
   if (ld % 8 || ld < H * (d8 + v8) || B > 65535) return -1;
   if (!docqa_aligned16(q) || !docqa_aligned16(kv) || !docqa_aligned16(kr) || !docqa_aligned16(out)) return -1;
-  const WindowArgs a{nullptr, 0, cu, nullptr, nullptr, sink, H, H, D, 64, 6, scale, window, vdim,
+  const WindowArgs a{nullptr, 0, cu, nullptr, nullptr, sink, H, H, D, 64, 6, scale, window, vdim, 0, 0.f, 1.f, H * vdim,
                      cu_k, (const uint16_t*)kr, ld, d8, v8};
   const uint16_t* v = (const uint16_t*)kv + (size_t)H * d8;
   // 128 query rows a workgroup, 64 where that leaves CUs without one

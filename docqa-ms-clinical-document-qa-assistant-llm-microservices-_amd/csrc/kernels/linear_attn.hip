@@ -1,0 +1,654 @@
+// linear_attn.hip -- linear-attention recurrences with one [dk, dv] matrix S a head:
+//   S_t = diag(a_t) S_{t-1} + k_t u_t^T,  o_t = S_t^T q_t,  y = rms(o) w silu(g)
+//   channel: a = sigmoid(z)^(1/tau) per key channel, z = w1 . w2 + b of a low-rank projection; u = v
+//   fixed:   a constant per head; q, k rotated by position; u = v
+//   delta:   a = exp(A softplus(z + b)) per head; unit q, k; u = sigmoid(beta) (v - (a S_{t-1})^T k)
+// The state pool holds [slots, H, dk, dvp] fp32 (dvp: dv rounded up to 4, padding zero).  A sequence
+// whose first token is position 0 starts from zero whatever its slot held.
+//
+// Everything between the projections and the gated heads is fp32, matrix products included
+// (v_mfma_f32_16x16x4_f32).
+//
+// step (one token a row): a workgroup a head; a wave holds 32 columns of S in registers (8 lanes of
+//   4 columns x 8 row groups), so the state is read and written once in 128-byte pieces.
+// scan (prompts), chunks of C tokens, b_t the log decays summed inside the chunk:
+//   prep   per (chunk, head), all side by side:  Q' = q e^{b_t},  K' = k e^{b_C - b_t} (transposed),
+//          A[t, s] = q_t . k_s e^{b_t - b_s} (s <= t); delta: M[t, s] = beta_t e^{b_t - b_s} k_t . k_s
+//          (s < t) and by forward substitution U = (1 + M)^-1 beta v, W = (1 + M)^-1 beta e^{b_t} k.
+//          No exponent is positive: where decays differ by channel, a 16 x 16 block of A below the
+//          diagonal takes both factors relative to the last token ahead of its rows, one on the
+//          diagonal is summed directly.
+//   chunk  per (sequence, head, dv tile), chunk after chunk, S in accumulators:
+//          u = v or U - W S;  o = Q' S + A u;  S = e^{b_C} S + K'^T u
+//   gate   y = rms(o) w silu(g) per (token, head)
+#include "docqa_common.h"
+#include "docqa_elem.h"
+#include "docqa_hybrid.h"
+
+using namespace docqa;
+
+namespace {
+// V columns of a product or of slabs, element type by a uniform flag
+template <int V>
+__device__ __forceinline__ void ldx(const void* p, int f32, int S, size_t slab, size_t off, float* f) {
+  if (f32) ld_slabs<V>((const float*)p + off, S, slab, f);
+  else ld_slabs<V>((const uint16_t*)p + off, S, slab, f);
+}
+__device__ __forceinline__ float ldx1(const void* p, int f32, int S, size_t slab, size_t off) {
+  float f;
+  ldx<1>(p, f32, S, slab, off, &f);
+  return f;
+}
+__device__ __forceinline__ void stx(void* p, int f32, size_t off, float v) {
+  if (f32) ((float*)p)[off] = v;
+  else ((uint16_t*)p)[off] = f2bf(v);
+}
+__device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
+// log(1 + e^x)
+__device__ __forceinline__ float softplus_x(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+__device__ __forceinline__ f32x4 mfma(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// ------------------------------------------------------------------ one token a row
+// NR: rows of S a lane holds, 8 NR >= dk; MT: most threads (32 columns a wave)
+template <int NR, int MT>
+__global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const int* __restrict__ positions) {
+  extern __shared__ float lds[];
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x, nt = blockDim.x, lane = tid & 63, wave = tid >> 6;
+  const int dk = a.dk, dv = a.dv, dvp = (dv + 3) & ~3, kh = h / (a.H / a.G);
+  float *sq = lds, *sk = sq + dk, *sa = sk + dk, *sr = sa + dk;      // q, k, decays, low-rank inputs
+  float* red = sr + a.rank;                                          // [waves]
+  const int slot = a.slots[b];
+  const int cg = lane & 7, rg = lane >> 3, c0 = wave * 32 + cg * 4;
+  const bool carry = slot >= 0 && positions[b] > 0, cok = c0 < dvp;
+  float* sp = a.state + ((size_t)max(slot, 0) * a.H + h) * dk * dvp;
+  float4 S[NR];
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const int r = i * 8 + rg;
+    S[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (carry && cok && r < dk) S[i] = *reinterpret_cast<const float4*>(sp + (size_t)r * dvp + c0);
+  }
+  const size_t xr = (size_t)b * a.ldx, zr = (size_t)b * a.ldz;
+  float v[4], g[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const bool ok = c0 + j < dv;
+    v[j] = ok ? ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.vo + h * dv + c0 + j) : 0.f;
+    g[j] = ok && rg == 0 ? ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.go + h * dv + c0 + j) : 0.f;
+  }
+  for (int i = tid; i < dk; i += nt) {
+    sq[i] = ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.qo + kh * dk + i);
+    sk[i] = ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.ko + kh * dk + i);
+  }
+  float qs = a.qs, ks = a.ks, beta = 1.f, al = 1.f;
+  if (a.kind == LIN_CHANNEL) {
+    for (int i = tid; i < a.rank; i += nt) sr[i] = ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.ao + i);
+  } else if (a.kind == LIN_FIXED) {
+    al = expf(a.w_gate[h]);
+  } else {
+    al = expf(a.w_gate[h] * softplus_x(ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.ao + h) + a.b_gate[h]));
+    beta = sigmoid_f(ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.bo + h));
+  }
+  __syncthreads();
+  if (a.kind == LIN_CHANNEL) {
+    for (int i = tid; i < dk; i += nt) {
+      const float* w = a.w_gate + ((size_t)h * dk + i) * a.rank;
+      float z = a.b_gate[h * dk + i];
+      for (int r = 0; r < a.rank; ++r) z += sr[r] * w[r];
+      sa[i] = expf(-softplus_x(-z) * a.inv_tau);
+    }
+    __syncthreads();
+  } else if (a.kind == LIN_FIXED && a.r > 0) {
+    const int r2 = a.r / 2;
+    for (int e = tid; e < a.r; e += nt) {
+      float* s = e < r2 ? sq : sk;
+      const int i = e < r2 ? e : e - r2;
+      const float c = a.cs[(size_t)b * a.r + i], si = a.cs[(size_t)b * a.r + r2 + i], x = s[i], y = s[i + r2];
+      s[i] = x * c - y * si;
+      s[i + r2] = y * c + x * si;
+    }
+    __syncthreads();
+  } else if (a.kind == LIN_DELTA) {
+    float nq = 0.f, nk = 0.f;
+    for (int i = lane; i < dk; i += 64) {
+      nq += sq[i] * sq[i];
+      nk += sk[i] * sk[i];
+    }
+    qs *= 1.f / sqrtf(wave_sum(nq) + 1e-6f);
+    ks *= 1.f / sqrtf(wave_sum(nk) + 1e-6f);
+  }
+  auto rows_sum = [](float x) {              // over the row groups of a column
+    x += __shfl_xor(x, 8, 64);
+    x += __shfl_xor(x, 16, 64);
+    x += __shfl_xor(x, 32, 64);
+    return x;
+  };
+  float p[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const int r = min(i * 8 + rg, dk - 1);   // rows past the last hold zeros
+    const float d = a.kind == LIN_CHANNEL ? sa[r] : al, k = sk[r] * ks;
+    S[i].x *= d; S[i].y *= d; S[i].z *= d; S[i].w *= d;
+    p[0] += S[i].x * k; p[1] += S[i].y * k; p[2] += S[i].z * k; p[3] += S[i].w * k;
+  }
+  if (a.kind == LIN_DELTA) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = beta * (v[j] - rows_sum(p[j]));
+  }
+  float o[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const int r = i * 8 + rg;
+    if (r < dk) {
+      const float k = sk[r] * ks, q = sq[r] * qs;
+      S[i].x += k * v[0]; S[i].y += k * v[1]; S[i].z += k * v[2]; S[i].w += k * v[3];
+      o[0] += S[i].x * q; o[1] += S[i].y * q; o[2] += S[i].z * q; o[3] += S[i].w * q;
+      if (slot >= 0 && cok) *reinterpret_cast<float4*>(sp + (size_t)r * dvp + c0) = S[i];
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    o[j] = rows_sum(o[j]);
+    if (rg == 0 && c0 + j < dv) ss += o[j] * o[j];
+  }
+  ss = wave_sum(ss);
+  if (lane == 0) red[wave] = ss;
+  __syncthreads();
+  float tot = 0.f;
+  for (int w = 0; w < (nt >> 6); ++w) tot += red[w];
+  const float inv = 1.f / sqrtf(tot / (float)dv + a.eps);
+  if (rg == 0) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (c0 + j < dv)
+        stx(a.out, a.of32, (size_t)b * a.ldo + h * dv + c0 + j, o[j] * inv * a.norm[c0 + j] * g[j] * sigmoid_f(g[j]));
+  }
+}
+
+// ------------------------------------------------------------------ prompts
+struct ScanArgs {
+  DocqaLinear a;
+  const int *cu, *ctx;
+  int nchunk;                            // most chunks of a sequence
+  float *Q, *K, *A, *G, *W, *U, *O;      // per (chunk, head): [C, dkp], [dkp, C], [C, C], [dkp], [C, dkp], [C, dvq]; O [T, H, dvq]
+};
+// chunk ids: sequence b's follow those of the sequences ahead of it, whatever their lengths
+__device__ __forceinline__ size_t chunk_id(const ScanArgs& s, int b, int ck, int C) { return (size_t)(s.cu[b] / C) + b + ck; }
+
+constexpr int NTP = 256;
+template <int C, int DKP, int KIND, int V>
+__global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
+  constexpr int PK = DKP + 4, NB = C / 16, PM = C + 4;
+  constexpr bool CH = KIND == LIN_CHANNEL, DELTA = KIND == LIN_DELTA;
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float *sQ = lds, *sK = sQ + C * PK, *sB = sK + C * PK;     // sB: [C, PK] (channel) or [C] log decays, summed
+  float* sM = sB + (CH ? C * PK : C);                        // delta: [C, PM]; channel: low-rank inputs [C, rank]
+  float* sbeta = sM + C * PM;                                // delta: [C]
+  const DocqaLinear& a = sc.a;
+  const int h = blockIdx.x, ck = blockIdx.y, b = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int q0 = sc.cu[b], L = sc.cu[b + 1] - q0, t0 = ck * C;
+  if (t0 >= L) return;
+  const int n = min(C, L - t0), dk = a.dk, dv = a.dv, kh = h / (a.H / a.G), dvq = (dv + 15) & ~15;
+  const size_t cid = chunk_id(sc, b, ck, C) * a.H + h, row0 = q0 + t0;
+
+  for (int e = tid; e < C * (DKP / V); e += NTP) {
+    const int t = e / (DKP / V), d = (e % (DKP / V)) * V;
+    float q[V], k[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) q[j] = k[j] = 0.f;
+    if (t < n && d < dk) {
+      const size_t r = (row0 + t) * a.ldx + kh * dk + d;
+      ldx<V>(a.X, a.xf32, a.Sx, a.xslab, r + a.qo, q);
+      ldx<V>(a.X, a.xf32, a.Sx, a.xslab, r + a.ko, k);
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      sQ[t * PK + d + j] = q[j];
+      sK[t * PK + d + j] = k[j];
+    }
+  }
+  if constexpr (CH) {
+    for (int e = tid; e < C * a.rank; e += NTP) {
+      const int t = e / a.rank, r = e % a.rank;
+      sM[e] = t < n ? ldx1(a.Z, a.zf32, a.Sz, a.zslab, (row0 + t) * a.ldz + a.ao + r) : 0.f;
+    }
+  } else if (wave == 0) {
+    float la = 0.f;
+    if (lane < n) {
+      la = a.w_gate[h];
+      if constexpr (DELTA) la *= softplus_x(ldx1(a.Z, a.zf32, a.Sz, a.zslab, (row0 + lane) * a.ldz + a.ao + h) + a.b_gate[h]);
+    }
+#pragma unroll
+    for (int o = 1; o < C; o <<= 1) {
+      const float u = __shfl_up(la, o, 64);
+      if (lane >= o) la += u;
+    }
+    if (lane < C) sB[lane] = la;
+  } else if (DELTA && wave == 1) {
+    if (lane < C) sbeta[lane] = lane < n ? sigmoid_f(ldx1(a.Z, a.zf32, a.Sz, a.zslab, (row0 + lane) * a.ldz + a.bo + h)) : 0.f;
+  }
+  __syncthreads();
+
+  if constexpr (KIND == LIN_FIXED) {
+    const int r2 = a.r / 2;
+    for (int e = tid; e < n * a.r; e += NTP) {
+      const int t = e / a.r, i = e % a.r, p = i % (r2 > 0 ? r2 : 1);
+      float* s = (i < r2 ? sQ : sK) + t * PK;
+      const float c = a.cs[(row0 + t) * a.r + p], si = a.cs[(row0 + t) * a.r + r2 + p], x = s[p], y = s[p + r2];
+      s[p] = x * c - y * si;
+      s[p + r2] = y * c + x * si;
+    }
+    __syncthreads();
+  }
+  // scales (and unit norms) in place
+  for (int t = wave; t < C; t += NTP / 64) {
+    float qs = a.qs, ks = a.ks;
+    if constexpr (DELTA) {
+      float nq = 0.f, nk = 0.f;
+      for (int d = lane; d < DKP; d += 64) {
+        nq += sQ[t * PK + d] * sQ[t * PK + d];
+        nk += sK[t * PK + d] * sK[t * PK + d];
+      }
+      qs *= 1.f / sqrtf(wave_sum(nq) + 1e-6f);
+      ks *= 1.f / sqrtf(wave_sum(nk) + 1e-6f);
+    }
+    for (int d = lane; d < DKP; d += 64) {
+      sQ[t * PK + d] *= qs;
+      sK[t * PK + d] *= ks;
+    }
+  }
+  if constexpr (CH) {
+    // log decays and their sums: a thread a channel and a stretch of tokens
+    constexpr int NS = NTP / DKP >= 4 ? 4 : NTP / DKP >= 2 ? 2 : 1, TS = C / NS;
+    for (int e = tid; e < DKP * NS; e += NTP) {
+      const int d = e % DKP, s = e / DKP;
+      float acc[TS];
+      const float bias = d < dk ? a.b_gate[h * dk + d] : 0.f;
+#pragma unroll
+      for (int i = 0; i < TS; ++i) acc[i] = bias;
+      if (d < dk) {
+        const float* w = a.w_gate + ((size_t)h * dk + d) * a.rank;
+        for (int r = 0; r < a.rank; ++r) {
+          const float wr = w[r];
+#pragma unroll
+          for (int i = 0; i < TS; ++i) acc[i] += wr * sM[(s * TS + i) * a.rank + r];
+        }
+      }
+      float sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < TS; ++i) {
+        if (d < dk && s * TS + i < n) sum -= softplus_x(-acc[i]) * a.inv_tau;
+        sB[(s * TS + i) * PK + d] = sum;
+      }
+    }
+    __syncthreads();
+    if constexpr (NS > 1) {
+      // every stretch's total ahead of it, then added: totals are read before any of them changes
+      static_assert(DKP * NS <= NTP, "a thread a stretch");
+      const int d = tid % DKP, st = tid / DKP;
+      float base = 0.f;
+      if (st < NS)
+        for (int p = 0; p < st; ++p) base += sB[((p + 1) * TS - 1) * PK + d];
+      __syncthreads();
+      if (st < NS)
+        for (int i = 0; i < TS; ++i) sB[(st * TS + i) * PK + d] += base;
+    }
+  }
+  __syncthreads();
+
+  // blocks of A (and M) on or below the diagonal
+  const int fr = lane & 15, g4 = lane >> 4;
+  float* gA = sc.A + cid * C * C;
+  int item = 0;
+  for (int i = 0; i < NB; ++i)
+    for (int j = 0; j <= i; ++j) {
+      if (CH && i == j) continue;
+      if ((item++ & 3) != wave) continue;
+      f32x4 qa = f32x4{0.f, 0.f, 0.f, 0.f}, ka = qa;
+      const int tr = i * 16 + fr, sr = j * 16 + fr, ref = i * 16 - 1;
+#pragma unroll 4
+      for (int k0 = 0; k0 < DKP; k0 += 16) {
+        const int k = k0 + 4 * g4;
+        float4 q = *reinterpret_cast<const float4*>(sQ + tr * PK + k);
+        float4 ks = *reinterpret_cast<const float4*>(sK + sr * PK + k);
+        if constexpr (CH) {
+          const float4 bt = *reinterpret_cast<const float4*>(sB + tr * PK + k), bs = *reinterpret_cast<const float4*>(sB + sr * PK + k);
+          const float4 br = *reinterpret_cast<const float4*>(sB + ref * PK + k);
+          q.x *= __expf(bt.x - br.x); q.y *= __expf(bt.y - br.y); q.z *= __expf(bt.z - br.z); q.w *= __expf(bt.w - br.w);
+          ks.x *= __expf(br.x - bs.x); ks.y *= __expf(br.y - bs.y); ks.z *= __expf(br.z - bs.z); ks.w *= __expf(br.w - bs.w);
+        }
+        qa = mfma(q.x, ks.x, qa); qa = mfma(q.y, ks.y, qa); qa = mfma(q.z, ks.z, qa); qa = mfma(q.w, ks.w, qa);
+        if constexpr (DELTA) {
+          const float4 kt = *reinterpret_cast<const float4*>(sK + tr * PK + k);
+          ka = mfma(kt.x, ks.x, ka); ka = mfma(kt.y, ks.y, ka); ka = mfma(kt.z, ks.z, ka); ka = mfma(kt.w, ks.w, ka);
+        }
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = i * 16 + 4 * g4 + r, s = j * 16 + fr;
+        float f = 1.f;
+        if constexpr (!CH) f = s <= t ? expf(sB[t] - sB[s]) : 0.f;
+        gA[t * C + s] = s <= t ? qa[r] * f : 0.f;
+        if constexpr (DELTA) sM[t * PM + s] = s < t ? sbeta[t] * ka[r] * f : 0.f;
+      }
+    }
+  if constexpr (CH) {
+    const int t16 = tid >> 4, s16 = tid & 15;
+    for (int i = 0; i < NB; ++i) {
+      const int t = i * 16 + t16, s = i * 16 + s16;
+      float acc = 0.f;
+      if (s <= t) {
+        for (int d = 0; d < DKP; d += 4) {
+          const float4 q = *reinterpret_cast<const float4*>(sQ + t * PK + d), k = *reinterpret_cast<const float4*>(sK + s * PK + d);
+          const float4 bt = *reinterpret_cast<const float4*>(sB + t * PK + d), bs = *reinterpret_cast<const float4*>(sB + s * PK + d);
+          acc += q.x * k.x * __expf(bt.x - bs.x) + q.y * k.y * __expf(bt.y - bs.y) + q.z * k.z * __expf(bt.z - bs.z) +
+                 q.w * k.w * __expf(bt.w - bs.w);
+        }
+      }
+      gA[t * C + s] = acc;
+    }
+  }
+  if constexpr (DELTA) __syncthreads();
+
+  // Q' and K' (transposed), the chunk's decay
+  float *gQ = sc.Q + cid * C * DKP, *gK = sc.K + cid * C * DKP;
+  for (int e = tid; e < C * (DKP / 4); e += NTP) {
+    const int t = e / (DKP / 4), d = (e % (DKP / 4)) * 4;
+    float4 q = *reinterpret_cast<const float4*>(sQ + t * PK + d);
+    float4 f;
+    if constexpr (CH) {
+      const float4 bt = *reinterpret_cast<const float4*>(sB + t * PK + d);
+      f = make_float4(__expf(bt.x), __expf(bt.y), __expf(bt.z), __expf(bt.w));
+    } else {
+      const float x = expf(sB[t]);
+      f = make_float4(x, x, x, x);
+    }
+    *reinterpret_cast<float4*>(gQ + t * DKP + d) = make_float4(q.x * f.x, q.y * f.y, q.z * f.z, q.w * f.w);
+  }
+  for (int e = tid; e < C * DKP; e += NTP) {
+    const int d = e / C, t = e % C;
+    const float f = CH ? __expf(sB[(C - 1) * PK + d] - sB[t * PK + d]) : expf(sB[C - 1] - sB[t]);
+    gK[e] = sK[t * PK + d] * f;
+  }
+  for (int d = tid; d < DKP; d += NTP) sc.G[cid * DKP + d] = CH ? expf(sB[(C - 1) * PK + d]) : expf(sB[C - 1]);
+
+  if constexpr (DELTA) {
+    // a thread a column of [beta v | beta e^b k]: x_t <- r_t - sum_{s < t} M[t, s] x_s
+    float *gW = sc.W + cid * C * DKP, *gU = sc.U + cid * C * dvq;
+    for (int c = tid; c < dvq + DKP; c += NTP) {
+      float x[C];
+      if (c < dvq) {
+#pragma unroll
+        for (int t = 0; t < C; ++t)
+          x[t] = t < n && c < dv ? ldx1(a.X, a.xf32, a.Sx, a.xslab, (row0 + min(t, n - 1)) * a.ldx + a.vo + h * dv + c) * sbeta[t] : 0.f;
+      } else {
+#pragma unroll
+        for (int t = 0; t < C; ++t) x[t] = sbeta[t] * expf(sB[t]) * sK[t * PK + c - dvq];
+      }
+#pragma unroll
+      for (int t = 1; t < C; ++t) {
+        float acc = 0.f;
+#pragma unroll
+        for (int s = 0; s < (t + 3) / 4 * 4; s += 4) {
+          const float4 m = *reinterpret_cast<const float4*>(sM + t * PM + s);      // zero from s = t on
+          acc += m.x * x[s];
+          if (s + 1 < t) acc += m.y * x[s + 1];
+          if (s + 2 < t) acc += m.z * x[s + 2];
+          if (s + 3 < t) acc += m.w * x[s + 3];
+        }
+        x[t] -= acc;
+        asm volatile("" ::: "memory");       // row by row: M is not pulled into registers ahead
+      }
+#pragma unroll
+      for (int t = 0; t < C; ++t) {
+        if (c < dvq) gU[t * dvq + c] = x[t];
+        else gW[t * DKP + c - dvq] = x[t];
+      }
+    }
+  }
+}
+
+// 4 waves; S rows in 16-row tiles dealt to the waves, token rows 16 to a wave
+template <int C, int DKP, int NT, bool DELTA>
+__global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
+  constexpr int DVT = 16 * NT, PS = DVT + 4, RT = DKP / 16, RPW = (RT + 3) / 4, NTT = C / 16;
+  __shared__ float sS[DKP * PS];
+  __shared__ float sV[C * PS];
+  const DocqaLinear& a = sc.a;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
+  const int dv = a.dv, dvp = (dv + 3) & ~3, dvq = (dv + 15) & ~15, tiles = (dvq + DVT - 1) / DVT;
+  const int u = xcd_remap(blockIdx.x, gridDim.x);              // a head's tiles share an L2
+  const int ct = u % tiles, h = u / tiles % a.H, b = u / (tiles * a.H);
+  const int q0 = sc.cu[b], L = sc.cu[b + 1] - q0, c0 = ct * DVT, slot = a.slots[b];
+  if (L <= 0) return;
+  const bool carry = sc.ctx[b] > 0 && slot >= 0;
+  float* st = a.state + ((size_t)max(slot, 0) * a.H + h) * a.dk * dvp;
+  f32x4 S[RPW][NT];
+#pragma unroll
+  for (int q = 0; q < RPW; ++q) {
+    const int rt = wave + 4 * q;
+#pragma unroll
+    for (int c = 0; c < NT; ++c)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int d = rt * 16 + 4 * g4 + r, col = c0 + c * 16 + fr;
+        S[q][c][r] = carry && rt < RT && d < a.dk && col < dv ? st[(size_t)d * dvp + col] : 0.f;
+      }
+  }
+  auto publish = [&]() {
+#pragma unroll
+    for (int q = 0; q < RPW; ++q) {
+      const int rt = wave + 4 * q;
+      if (rt < RT)
+#pragma unroll
+        for (int c = 0; c < NT; ++c)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) sS[(rt * 16 + 4 * g4 + r) * PS + c * 16 + fr] = S[q][c][r];
+    }
+  };
+  // rows of a [16, K] operand at p (row stride ld) times B [K, DVT] in LDS; k runs in steps of 16, lane
+  // group g4 taking 4 consecutive k (any order will do if both operands share it)
+  auto product = [&](const float* p, int ld, const float* B, int K, f32x4* acc) {
+    const float* pr = p + (size_t)fr * ld + 4 * g4;
+#pragma unroll 8
+    for (int k0 = 0; k0 < K; k0 += 16) {
+      const float4 x = *reinterpret_cast<const float4*>(pr + k0);
+      const float* br = B + (k0 + 4 * g4) * PS + fr;
+#pragma unroll
+      for (int c = 0; c < NT; ++c) {
+        acc[c] = mfma(x.x, br[c * 16], acc[c]);
+        acc[c] = mfma(x.y, br[PS + c * 16], acc[c]);
+        acc[c] = mfma(x.z, br[2 * PS + c * 16], acc[c]);
+        acc[c] = mfma(x.w, br[3 * PS + c * 16], acc[c]);
+      }
+    }
+  };
+  publish();
+  for (int ck = 0; ck * C < L; ++ck) {
+    const int n = min(C, L - ck * C);
+    const size_t row0 = q0 + ck * C, cid = chunk_id(sc, b, ck, C) * a.H + h;
+    __syncthreads();                                   // sS is written, sV free
+    if constexpr (DELTA) {
+      if (wave < NTT) {
+        f32x4 acc[NT];
+#pragma unroll
+        for (int c = 0; c < NT; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+        product(sc.W + cid * C * DKP + wave * 16 * DKP, DKP, sS, DKP, acc);
+#pragma unroll
+        for (int c = 0; c < NT; ++c)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int t = wave * 16 + 4 * g4 + r, col = c0 + c * 16 + fr;
+            sV[t * PS + c * 16 + fr] = col < dvq ? sc.U[(cid * C + t) * dvq + col] - acc[c][r] : 0.f;
+          }
+      }
+    } else {
+      for (int e = tid; e < C * DVT; e += 256) {
+        const int t = e / DVT, c = e % DVT;
+        sV[t * PS + c] = t < n && c0 + c < dv ? ldx1(a.X, a.xf32, a.Sx, a.xslab, (row0 + t) * a.ldx + a.vo + h * dv + c0 + c) : 0.f;
+      }
+    }
+    __syncthreads();
+    if (wave < NTT && wave * 16 < n) {
+      f32x4 acc[NT];
+#pragma unroll
+      for (int c = 0; c < NT; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+      product(sc.Q + cid * C * DKP + wave * 16 * DKP, DKP, sS, DKP, acc);
+      product(sc.A + cid * C * C + wave * 16 * C, C, sV, (wave + 1) * 16, acc);
+#pragma unroll
+      for (int c = 0; c < NT; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = wave * 16 + 4 * g4 + r, col = c0 + c * 16 + fr;
+          if (t < n && col < dvq) sc.O[((row0 + t) * a.H + h) * dvq + col] = acc[c][r];
+        }
+    }
+#pragma unroll
+    for (int q = 0; q < RPW; ++q) {
+      const int rt = wave + 4 * q;
+      if (rt < RT) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float d = sc.G[cid * DKP + rt * 16 + 4 * g4 + r];
+#pragma unroll
+          for (int c = 0; c < NT; ++c) S[q][c][r] *= d;
+        }
+        product(sc.K + (cid * DKP + rt * 16) * C, C, sV, C, S[q]);
+      }
+    }
+    __syncthreads();                                   // everyone has read sS
+    publish();
+  }
+  if (slot < 0) return;
+#pragma unroll
+  for (int q = 0; q < RPW; ++q) {
+    const int rt = wave + 4 * q;
+#pragma unroll
+    for (int c = 0; c < NT; ++c)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int d = rt * 16 + 4 * g4 + r, col = c0 + c * 16 + fr;
+        if (rt < RT && d < a.dk && col < dv) st[(size_t)d * dvp + col] = S[q][c][r];
+      }
+  }
+}
+
+// a wave a (token, head)
+__global__ __launch_bounds__(256) void linear_gate_kernel(DocqaLinear a, const float* __restrict__ O, int tokens) {
+  const int u = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int t = u / a.H, h = u % a.H, dv = a.dv, dvq = (dv + 15) & ~15;
+  if (t >= tokens) return;
+  const float* o = O + ((size_t)t * a.H + h) * dvq;
+  float x[8], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int c = lane + 64 * i;
+    x[i] = c < dv ? o[c] : 0.f;
+    ss += x[i] * x[i];
+  }
+  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)dv + a.eps);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int c = lane + 64 * i;
+    if (c < dv) {
+      const float g = ldx1(a.Z, a.zf32, a.Sz, a.zslab, (size_t)t * a.ldz + a.go + h * dv + c);
+      stx(a.out, a.of32, (size_t)t * a.ldo + h * dv + c, x[i] * inv * a.norm[c] * g * sigmoid_f(g));
+    }
+  }
+}
+
+template <int C, int DKP, int KIND>
+int launch_scan(const ScanArgs& sc, int tokens, int B, hipStream_t s) {
+  constexpr int PK = DKP + 4;
+  const DocqaLinear& a = sc.a;
+  const size_t low = KIND == LIN_CHANNEL ? (size_t)C * a.rank : (size_t)C * (C + 4) + C;
+  const size_t lds = (2 * C * PK + (KIND == LIN_CHANNEL ? C * PK : C) + low) * 4;
+  if (lds > 160 * 1024) return -1;
+  const bool vec = a.dk % 4 == 0 && a.qo % 4 == 0 && a.ko % 4 == 0 && a.ldx % 4 == 0;
+  dim3 grid(a.H, sc.nchunk, B);
+  auto prep = vec ? linear_prep_kernel<C, DKP, KIND, 4> : linear_prep_kernel<C, DKP, KIND, 1>;
+  if (lds > 64 * 1024) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(prep), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return (int)e;
+  }
+  prep<<<grid, NTP, lds, s>>>(sc);
+  DOCQA_CHECK_LAUNCH();
+  const int dvq = (a.dv + 15) & ~15;
+  const long long one = (long long)B * a.H * (dvq / 16);
+  // narrow tiles while they leave CUs without a workgroup
+  if (one <= 512 || dvq == 16) linear_chunk_kernel<C, DKP, 1, KIND == LIN_DELTA><<<(unsigned)one, 256, 0, s>>>(sc);
+  else linear_chunk_kernel<C, DKP, 2, KIND == LIN_DELTA><<<(unsigned)((long long)B * a.H * ((dvq + 31) / 32)), 256, 0, s>>>(sc);
+  DOCQA_CHECK_LAUNCH();
+  linear_gate_kernel<<<(unsigned)(((long long)tokens * a.H + 3) / 4), 256, 0, s>>>(a, sc.O, tokens);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+int dk_pad(int dk) { return dk <= 64 ? 64 : dk <= 128 ? 128 : 256; }
+
+template <int KIND>
+int dispatch_scan(const ScanArgs& sc, int tokens, int B, hipStream_t s) {
+  switch (dk_pad(sc.a.dk)) {
+    case 64: return launch_scan<64, 64, KIND>(sc, tokens, B, s);
+    case 128: return launch_scan<64, 128, KIND>(sc, tokens, B, s);
+    default: return launch_scan<32, 256, KIND>(sc, tokens, B, s);
+  }
+}
+}  // namespace
+
+int docqa_linear_step(const DocqaLinear& a, const int* positions, int B, hipStream_t s) {
+  if (B == 0) return 0;
+  if (a.dk < 1 || a.dk > 256 || a.dv < 1 || a.dv > 512 || B > 65535 || !docqa_aligned16(a.state)) return -1;
+  const int waves = (a.dv + 31) / 32;
+  const size_t lds = (size_t)(3 * a.dk + a.rank + waves) * 4;
+  dim3 grid(a.H, B);
+#define RUN(NR, MT) linear_step_kernel<NR, MT><<<grid, 64 * waves, lds, s>>>(a, positions)
+#define GO(NR)                        \
+  do {                                \
+    if (waves <= 4) RUN(NR, 256);     \
+    else if (waves <= 8) RUN(NR, 512); \
+    else RUN(NR, 1024);               \
+  } while (0)
+  if (a.dk <= 64) GO(8);
+  else if (a.dk <= 128) GO(16);
+  else GO(32);
+#undef GO
+#undef RUN
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+int docqa_linear_chunk(int dk) { return dk <= 128 ? 64 : 32; }
+
+namespace {
+struct Sizes {
+  size_t Q, A, G, W, U, O, total;
+};
+Sizes scratch_sizes(int kind, int tokens, int B, int H, int dk, int dv) {
+  const size_t C = docqa_linear_chunk(dk), dkp = dk_pad(dk), dvq = (dv + 15) & ~15;
+  const size_t n = (tokens / C + B + 1) * H;          // chunk ids are below tokens / C + B
+  const bool delta = kind == LIN_DELTA;
+  Sizes z{n * C * dkp, n * C * C, n * dkp, delta ? n * C * dkp : 0, delta ? n * C * dvq : 0, (size_t)tokens * H * dvq, 0};
+  z.total = 2 * z.Q + z.A + z.G + z.W + z.U + z.O;
+  return z;
+}
+}  // namespace
+
+size_t docqa_linear_scratch(int kind, int tokens, int B, int H, int dk, int dv) {
+  return scratch_sizes(kind, tokens, B, H, dk, dv).total;
+}
+
+int docqa_linear_scan(const DocqaLinear& a, const int* cu, const int* ctx, float* scratch, int tokens, int B, int max_len,
+                      hipStream_t s) {
+  if (B == 0 || max_len == 0) return 0;
+  if (a.dk < 1 || a.dk > 256 || a.dv < 1 || a.dv > 512 || B > 65535) return -1;
+  const int C = docqa_linear_chunk(a.dk);
+  const Sizes z = scratch_sizes(a.kind, tokens, B, a.H, a.dk, a.dv);
+  ScanArgs sc{a, cu, ctx, (max_len + C - 1) / C, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr};
+  if (sc.nchunk > 65535) return -1;
+  sc.Q = scratch; sc.K = sc.Q + z.Q; sc.A = sc.K + z.Q; sc.W = sc.A + z.A; sc.U = sc.W + z.W; sc.O = sc.U + z.U; sc.G = sc.O + z.O;
+  if (a.kind == LIN_CHANNEL) return dispatch_scan<LIN_CHANNEL>(sc, tokens, B, s);
+  if (a.kind == LIN_FIXED) return dispatch_scan<LIN_FIXED>(sc, tokens, B, s);
+  return dispatch_scan<LIN_DELTA>(sc, tokens, B, s);
+}

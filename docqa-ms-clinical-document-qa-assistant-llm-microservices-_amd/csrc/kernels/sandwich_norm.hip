@@ -6,8 +6,12 @@
 // the next projection's input in the compute dtype.  One 256-thread workgroup per row; each
 // thread keeps its elements of x in registers between the two reductions, so the residual is
 // read and written once.
+//
+// post_norm: norms after the sum, over equal parts of the row, behind a gated residual:
+//   x <- groupnorm(alpha x + sigmoid(gate + b) * y) * w
 #include "docqa_common.h"
 #include "docqa_elem.h"
+#include "docqa_hybrid.h"
 #include <type_traits>
 
 using namespace docqa;
@@ -154,7 +158,7 @@ __global__ __launch_bounds__(NT) void sandwich_rmsnorm_kernel(const PT* __restri
   }
 }
 
-// h = table[id] * scale (fp32 residual, and a second copy when ``emb``), out = rms(h) * w
+// h = table[id] * scale (fp32 residual, and a second copy when ``emb``), out = rms(h) * w (w null: h)
 template <int NV, int V, typename T>
 __global__ __launch_bounds__(256) void embed_scale_rmsnorm_kernel(const int* __restrict__ ids,
                                                                   const T* __restrict__ table, float scale,
@@ -181,13 +185,15 @@ __global__ __launch_bounds__(256) void embed_scale_rmsnorm_kernel(const int* __r
       if (emb) stv<V>(emb + row * H + c * V, x[i]);
     }
   }
-  const float ix = 1.f / sqrtf(block_sum(ss, red) / (float)H + eps);
+  const float ix = w ? 1.f / sqrtf(block_sum(ss, red) / (float)H + eps) : 1.f;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int c = tid + 256 * i;
     if (c < n) {
       float g[V], o[V];
-      ldv<V>(w + c * V, g);
+#pragma unroll
+      for (int j = 0; j < V; ++j) g[j] = 1.f;
+      if (w) ldv<V>(w + c * V, g);
 #pragma unroll
       for (int j = 0; j < V; ++j) o[j] = x[i][j] * ix * g[j];
       stv<V>(out + row * H + c * V, o);
@@ -303,7 +309,118 @@ int launch_embed(const int* ids, const T* table, float scale, const float* w, fl
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
+template <int V>
+__device__ __forceinline__ void ld_any(const void* p, int f32, int S, size_t slab, size_t off, float* f) {
+  if (f32) ld_slabs<V>((const float*)p + off, S, slab, f);
+  else ld_slabs<V>((const uint16_t*)p + off, S, slab, f);
+}
+
+// one workgroup of NT threads a row, V consecutive elements of NV pieces a thread.  A piece lies in one
+// group; where groups are whole multiples of a wave's piece (GW) the wave's sum is one LDS word, else
+// every piece's is, and a wave sums each group's.  Sums are in a fixed order either way.
+template <int NT, int NV, int V, bool GW>
+__global__ __launch_bounds__(NT) void post_norm_kernel(DocqaPostNorm a) {
+  extern __shared__ float part[];                       // GW: [NV * NT / 64], else [W / V + groups]
+  const size_t row = blockIdx.x;
+  const int tid = threadIdx.x, W = a.W, n = W / V, gn = n / a.groups;      // pieces of a row, of a group
+  const size_t pslab = (size_t)a.rows * W;
+  float x[NV][V];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = tid + NT * i;
+    float ss = 0.f;
+    if (c < n) {
+      ldv<V>(a.res + row * W + c * V, x[i]);
+#pragma unroll
+      for (int j = 0; j < V; ++j) x[i][j] *= a.alpha;
+      if (a.P) {
+        float y[V], g[V], b[V];
+        ld_any<V>(a.P, a.pf32, a.SP, pslab, row * W + c * V, y);
+        ld_any<V>(a.gate, a.gf32, a.SG, a.gslab, row * a.ldg + a.col + c * V, g);
+        ldv<V>(a.gb + c * V, b);
+        if (a.Q) {
+          float z[V];
+          ld_any<V>(a.Q, a.qf32, a.SQ, pslab, row * W + c * V, z);
+#pragma unroll
+          for (int j = 0; j < V; ++j) y[j] += z[j];
+        }
+#pragma unroll
+        for (int j = 0; j < V; ++j) x[i][j] += y[j] / (1.f + __expf(-(g[j] + b[j])));
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) ss += x[i][j] * x[i][j];
+      if constexpr (!GW) part[c] = ss;
+    }
+    if constexpr (GW) {
+      ss = wave_sum(ss);
+      if ((tid & 63) == 0) part[i * (NT / 64) + (tid >> 6)] = ss;
+    }
+  }
+  __syncthreads();
+  if constexpr (!GW) {
+    for (int g = tid >> 6; g < a.groups; g += NT / 64) {
+      float s = 0.f;
+      for (int e = tid & 63; e < gn; e += 64) s += part[g * gn + e];
+      s = wave_sum(s);
+      if ((tid & 63) == 0) part[n + g] = s;
+    }
+    __syncthreads();
+  }
+  const float rg = 1.f / ((float)gn * V);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = tid + NT * i;
+    if (c >= n) continue;
+    float s = 0.f;
+    const int g = c / gn;
+    if constexpr (GW) {
+      const int m = gn / 64;                            // waves' pieces of the group
+      for (int e = 0; e < m; ++e) s += part[g * m + e];
+    } else {
+      s = part[n + g];
+    }
+    const float inv = 1.f / sqrtf(s * rg + a.eps);
+    float w[V];
+    ldv<V>(a.w + c * V, w);
+#pragma unroll
+    for (int j = 0; j < V; ++j) x[i][j] *= inv * w[j];
+    stv<V>(a.res + row * W + c * V, x[i]);
+    if (a.out) stv<V>((uint16_t*)a.out + row * W + c * V, x[i]);
+  }
+}
+
+template <int V>
+int launch_post_norm(const DocqaPostNorm& a, hipStream_t s) {
+  const int n = a.W / V, gn = n / a.groups;
+  const bool gw = gn % 64 == 0;
+#define RUN(NT, NV, GW) \
+  post_norm_kernel<NT, NV, V, GW><<<a.rows, NT, (GW ? NV * NT / 64 : n + a.groups) * sizeof(float), s>>>(a)
+#define GO(NV)                                                                \
+  do {                                                                        \
+    if (!gw) RUN(256, NV, false);                                             \
+    else if (NV >= 4 && a.rows <= 512) RUN(1024, (NV >= 4 ? NV / 4 : 1), true); \
+    else RUN(256, NV, true);                                                  \
+  } while (0)
+  const int nv = (n + 255) / 256;
+  if (nv <= 1) GO(1);
+  else if (nv <= 2) GO(2);
+  else if (nv <= 4) GO(4);
+  else if (nv <= 8) GO(8);
+  else if (nv <= 16) GO(16);
+  else return -1;
+#undef GO
+#undef RUN
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
 }  // namespace
+
+int docqa_post_norm(const DocqaPostNorm& a, hipStream_t s) {
+  if (a.rows == 0) return 0;
+  if (a.W < 1 || a.groups < 1 || a.W % a.groups || a.SP < 1 || a.SQ < 1 || a.SG < 1 || (a.P && (!a.gate || !a.gb))) return -1;
+  const bool vec = a.W / a.groups % 4 == 0 && a.col % 4 == 0 && (!a.P || a.ldg % 4 == 0);
+  return vec ? launch_post_norm<4>(a, s) : launch_post_norm<1>(a, s);
+}
 
 int docqa_sandwich_rmsnorm(const void* P, int p_f32, int S, float* res, const float* w_post, const float* add,
                            const float* w_next, void* out, int out_f32, int rows, int H, float eps, hipStream_t s) {

@@ -114,21 +114,21 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
 
 // ------------------------------------------------------------------ convolution, decode
 // one new token a row; P [S, B, ld]: the input projection [x: C | z: C] as split-K slabs (or
-// its product).  Writes silu(conv) and, when z_out, the summed gate; advances the state.
+// its product).  Writes silu(conv) and, when z_out, the next NZ columns summed; advances the state.
 template <typename PT, typename T, int V, int K>
 __global__ __launch_bounds__(256) void conv_step_kernel(const PT* __restrict__ P, int S, size_t slab, int ld,
                                                         const float* __restrict__ w, const float* __restrict__ bias,
                                                         T* __restrict__ state, const int* __restrict__ slots,
                                                         const int* __restrict__ positions, T* __restrict__ y,
-                                                        T* __restrict__ z_out, int C, int taps, int silu) {
+                                                        T* __restrict__ z_out, int C, int NZ, int taps, int silu) {
   const int b = blockIdx.y, c0 = (blockIdx.x * 256 + threadIdx.x) * V;
   const int nt = K > 0 ? K : taps;
-  if (c0 >= (z_out ? 2 * C : C)) return;
+  if (c0 >= C + NZ) return;
   const PT* p = P + (size_t)b * ld + c0;
   float xn[V];
   ld_slabs<V>(p, S, slab, xn);
   if (c0 >= C) {
-    stv<V>(z_out + (size_t)b * C + (c0 - C), xn);
+    stv<V>(z_out + (size_t)b * NZ + (c0 - C), xn);
     return;
   }
   const int slot = slots[b];
@@ -466,10 +466,11 @@ int launch_conv(const void* x, int ldx, const float* w, const float* b, void* st
 
 template <typename PT, typename T, int V>
 int launch_conv_step(const void* P, int S, size_t slab, int ld, const float* w, const float* b, void* state,
-                     const int* slots, const int* pos, void* y, void* z, int B, int C, int taps, int silu, hipStream_t s) {
-  const int n = (z ? 2 * C : C) / V;
+                     const int* slots, const int* pos, void* y, void* z, int B, int C, int NZ, int taps, int silu,
+                     hipStream_t s) {
+  const int n = (C + NZ) / V;
   dim3 grid((n + 255) / 256, B);
-#define GO(K) conv_step_kernel<PT, T, V, K><<<grid, 256, 0, s>>>((const PT*)P, S, slab, ld, w, b, (T*)state, slots, pos, (T*)y, (T*)z, C, taps, silu)
+#define GO(K) conv_step_kernel<PT, T, V, K><<<grid, 256, 0, s>>>((const PT*)P, S, slab, ld, w, b, (T*)state, slots, pos, (T*)y, (T*)z, C, NZ, taps, silu)
   switch (taps) {
     case 2: GO(2); break;
     case 3: GO(3); break;
@@ -525,12 +526,12 @@ int docqa_causal_conv(const void* x, int ldx, const float* w, const float* b, vo
 }
 
 int docqa_conv_step(const void* P, int p_f32, int S, size_t slab, int ld, const float* w, const float* b, void* state,
-                    const int* slots, const int* positions, void* y, void* z, int f32, int B, int C, int taps,
+                    const int* slots, const int* positions, void* y, void* z, int f32, int B, int C, int NZ, int taps,
                     int silu, hipStream_t s) {
   if (B == 0) return 0;
-  if (taps < 1 || C < 1 || S < 1 || ld < (z ? 2 * C : C) || (f32 && !p_f32)) return -1;
-  const bool vec = C % 4 == 0 && ld % 4 == 0 && docqa_aligned16(P) && docqa_aligned16(state) && docqa_aligned16(y);
-#define ARGS P, S, slab, ld, w, b, state, slots, positions, y, z, B, C, taps, silu, s
+  if (taps < 1 || C < 1 || S < 1 || NZ < 0 || (NZ > 0 && !z) || ld < C + NZ || (f32 && !p_f32)) return -1;
+  const bool vec = C % 4 == 0 && NZ % 4 == 0 && ld % 4 == 0 && docqa_aligned16(P) && docqa_aligned16(state) && docqa_aligned16(y);
+#define ARGS P, S, slab, ld, w, b, state, slots, positions, y, z, B, C, NZ, taps, silu, s
   if (f32) return vec ? launch_conv_step<float, float, 4>(ARGS) : launch_conv_step<float, float, 1>(ARGS);
   if (p_f32) return vec ? launch_conv_step<float, uint16_t, 4>(ARGS) : launch_conv_step<float, uint16_t, 1>(ARGS);
   return vec ? launch_conv_step<uint16_t, uint16_t, 4>(ARGS) : launch_conv_step<uint16_t, uint16_t, 1>(ARGS);

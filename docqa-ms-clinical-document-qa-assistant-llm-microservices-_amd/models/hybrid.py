@@ -1047,8 +1047,7 @@ class HybridModel(Decoder):
         decode = all(p.decode for p in parts)
         pos = _join([p.meta.positions for p in parts])
         fw = _Forward({r: ops.rope_table(pos, f, mult) for r, (f, mult) in self.rope_freq.items()}, {})
-        x = ops.embedding(input_ids, self.embed)
-        res = x.float()
+        res, _, x = ops.embed_scale_rmsnorm(input_ids, self.embed, cfg.embed_scale, None, eps)
         for L, cache in zip(self.layers, caches):
             y, P, col = L["mixer"].run(x, parts, slot_mapping, cache, decode, fw)
             x = ops.post_norm(y, None, P, col, L["rg1_b"], res, alpha, L["norm1"], groups, eps, dt)

@@ -1196,7 +1196,7 @@ def flash_prefill_paged(qkv, cu_seqlens, max_len, Hq, Hkv, D, scale, k_cache, v_
 # projection feeding one of them is its product [M, N] or its split-K slabs [S, M, N].
 def embed_scale_rmsnorm(ids, table, scale: float, w, eps: float, keep: bool = False):
     """(h, copy of h or None, x): h = table[ids] * scale in fp32 (the residual stream),
-    x = rmsnorm(h) * w in the table's dtype."""
+    x = rmsnorm(h) * w (``w`` None: h itself) in the table's dtype."""
     if _gpu(table):
         h, e, x = _native().embed_scale_rmsnorm(ids.contiguous(), table, float(scale), w, float(eps), keep)
         return h, (e if keep else None), x

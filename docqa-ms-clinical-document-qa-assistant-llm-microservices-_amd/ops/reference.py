@@ -360,7 +360,7 @@ def sandwich_rmsnorm(P, residual, w_post, w_next, eps, add=None, out_dtype=None)
 
 def embed_scale_rmsnorm(ids, table, scale, w, eps, keep):
     h = table[ids.long()].float() * scale
-    return h, (h.clone() if keep else None), (_rms(h, eps) * w).to(table.dtype)
+    return h, (h.clone() if keep else None), (h if w is None else _rms(h, eps) * w).to(table.dtype, copy=True)
 
 
 def activation(P, act, out_dtype):
