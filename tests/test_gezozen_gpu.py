@@ -1,0 +1,131 @@
+"""Gezozen on the HIP kernels, in fp32 and bf16, against the plain oracle."""
+import sys
+from pathlib import Path
+
+import pytest
+import torch
+
+sys.path.insert(0, str(Path(__file__).parent))
+import gezozen_cases as C  # noqa: E402
+
+pytestmark = pytest.mark.gpu
+F32, BF16 = torch.float32, torch.bfloat16
+DTYPES = [F32, BF16]
+
+
+@pytest.fixture(autouse=True)
+def _native():
+    from docqa_amd import ops
+
+    assert ops.load_native(), ops.native_error()
+    torch.set_num_threads(4)
+
+
+def test_rotation():
+    C.rope_case("cuda")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("case", ["post_norm_case", "attention_case", "window_edge_case", "soft_cap_case", "batch_attention_case",
+                                  "linear_case", "decay_case", "batch_linear_case", "forgotten_state_case", "conv_case", "moe_case"])
+def test_mechanisms(case, dtype):
+    getattr(C, case)("cuda", dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", list(C.CONFIGS))
+def test_models(name, dtype):
+    C.whole_case(name, "cuda", dtype)
+    C.portions_case(name, "cuda", dtype)
+    C.batch_case(name, "cuda", dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_decoding(dtype):
+    C.long_case("edge", "cuda", dtype)
+
+
+@pytest.mark.parametrize("name", ["mixed", "odd"])
+def test_generation(name):
+    C.generate_case(name, "cuda")
+    C.generate_case(name, "cuda", use_graphs=True)
+    C.mixed_steps_case(name, "cuda")
+
+
+def test_preemption_recomputes_state():
+    C.preemption_case("mixed", "cuda")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_graph_replays_match_eager_steps(dtype):
+    """A captured decode step replayed with eager work in between: the same tokens as eager
+    steps, and capturing it leaves the states alone."""
+    js, w, m = C.make("mixed", "cuda", dtype, seed=40)
+    prompts = [C.toks(n, js["vocab"], n) for n in (9, 30, 17)]
+    sp = C.SamplingParams(max_new_tokens=25)
+    eager = C.engine(m, tokens=512, slots=4).generate(prompts, sp)
+    eng = C.engine(m, tokens=512, slots=4, use_graphs=True)
+    for _ in range(3):
+        assert eng.generate(prompts, sp) == eager
+        torch.cuda.synchronize()
+    assert any(g.graph is not None for g in eng._graphs.values())
+
+
+# widths that the GEMM kernels and the grouped tiles accept
+WIDE = C.conf(1024, 2048, [C.gla(C.left(8, 2, 128, 128, C.rot(1e4, 64), cap=30.0), 8, 128, 128, 16.0, mlp=C.moe(8, 2, 512, 512)),
+                           C.ret(C.left(8, 2, 128, 64, C.rot(1e4, 64, (8.0, 256.0, 32.0, 1.0)), window=200), 64, 128, [0.97, 0.99, 0.995, 0.999],
+                                 C.rot(1e6, 64), mlp=C.moe(4, 1, 256)),
+                           C.delta(8, 4, 128, 128, 4, C.moe(8, 2, 512, 256))], 4, 3.0)
+
+
+def wide_model(seed):
+    js = WIDE
+    w = C.O.random_weights(js, seed, rank=16)
+    C.settle_routing(w, js)
+    return C.HybridModel(C.gezozen.config_from_json(js), device="cuda", weights=w)
+
+
+@pytest.mark.parametrize("rows", [1, 3, 40, 300])
+def test_wide_layers_take_the_gemm_plans(rows):
+    """Decode rows through the slab consumers and the experts' kernels of either kind agree with the same
+    step on the reference operators."""
+    from docqa_amd import ops
+
+    m = wide_model(1)
+    eng = C.engine(m, tokens=rows * 64, bs=64, slots=rows)
+    ref = C.engine(m, tokens=rows * 64, bs=64, slots=rows)
+    seqs = [C.toks(7, 2048, r) for r in range(rows)]
+    steps = [[(str(r), s[:5]) for r, s in enumerate(seqs)], [(str(r), s[5:6]) for r, s in enumerate(seqs)],
+             [(str(r), s[6:]) for r, s in enumerate(seqs)]]
+    got = C.run_steps(eng, steps)
+    if rows > 3:                       # the reference walks sequences one by one
+        keep = [0, 1, rows - 1]
+        steps = [[s for s in st if int(s[0]) in keep] for st in steps]
+    with ops.use_reference():
+        want = C.run_steps(ref, steps)
+    for k in want:
+        C.close(got[k], want[k].cpu(), BF16, k)
+
+
+@pytest.mark.parametrize("M", [300, 2500])
+def test_long_prompt_prefill(M):
+    """A prompt long enough for the prefill GEMMs and the sorted experts: whole, cut in portions, and the
+    last tokens decoded."""
+    m = wide_model(2)
+    seq = C.toks(M, 2048, 3)
+    tail = [M - 1, M - 2, M // 2, 130, 1]
+
+    def run(sizes):
+        tr = C.TraceReplay(C.engine(m, tokens=4096, bs=64, slots=1))
+        out, t = {}, 0
+        for p in C.portions(seq, sizes):
+            w = [q - t for q in tail if t <= q < t + len(p)]
+            o = tr.step([{"id": "a", "tokens": p, "want": w}])
+            for j, q in enumerate(w):
+                out[q + t] = o[j]
+            t += len(p)
+        return torch.stack([out[q] for q in tail])
+
+    whole = run([M])
+    for sizes in ([100, 64, 2], [M - 2, 1, 1], [M // 2], [M - 66, 64, 2]):
+        C.close(run(sizes), whole.cpu(), BF16, sizes)
