@@ -557,13 +557,13 @@ Tensor selective_step(const Tensor& x, const OptT& dt, const OptT& dt_in, const 
 DocqaLinear linear_args(const Tensor& X, const Tensor& Z, at::IntArrayRef d, at::ArrayRef<double> f, const Tensor& w_gate,
                         const OptT& b_gate, const OptT& cs, const Tensor& norm, const Tensor& state, Tensor& out) {
   const Slabs x = slabs_of(X), z = slabs_of(Z);
-  CHECK_ALIGN16(X); CHECK_ALIGN16(Z); CHECK_ALIGN16(state);
+  CHECK_ALIGN16(state);
   TORCH_CHECK(d.size() == 12 && f.size() == 4, "linear attention: arguments");
   DocqaLinear a{};
-  int* di = &a.kind;
+  int* const to[12] = {&a.kind, &a.H, &a.G, &a.dk, &a.dv, &a.qo, &a.ko, &a.vo, &a.go, &a.ao, &a.bo, &a.rank};
   for (int i = 0; i < 12; ++i) {
     TORCH_CHECK(d[i] >= 0 && d[i] < (1 << 24), "linear attention: sizes");
-    di[i] = (int)d[i];
+    *to[i] = (int)d[i];
   }
   a.X = X.data_ptr(); a.Z = Z.data_ptr();
   a.xf32 = is_f32(X); a.Sx = x.S; a.ldx = x.N; a.xslab = x.slab;

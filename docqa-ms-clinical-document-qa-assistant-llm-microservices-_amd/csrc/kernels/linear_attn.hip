@@ -10,11 +10,13 @@
 // (v_mfma_f32_16x16x4_f32).
 //
 // step (one token a row): a workgroup a head; a wave holds 32 columns of S in registers (8 lanes of
-//   4 columns x 8 row groups), so the state is read and written once in 128-byte pieces.
+//   4 columns x 8 row groups; heads of more than 128 rows: 4 lanes x 16 row groups), so the state is
+//   read and written once in 128-byte pieces.
 // scan (prompts), chunks of C tokens, b_t the log decays summed inside the chunk:
 //   prep   per (chunk, head), all side by side:  Q' = q e^{b_t},  K' = k e^{b_C - b_t} (transposed),
 //          A[t, s] = q_t . k_s e^{b_t - b_s} (s <= t); delta: M[t, s] = beta_t e^{b_t - b_s} k_t . k_s
-//          (s < t) and by forward substitution U = (1 + M)^-1 beta v, W = (1 + M)^-1 beta e^{b_t} k.
+//          (s < t) and, by forward substitution over blocks of 16 tokens with the diagonal blocks
+//          inverted ahead, U = (1 + M)^-1 beta v, W = (1 + M)^-1 beta e^{b_t} k.
 //          No exponent is positive: where decays differ by channel, a 16 x 16 block of A below the
 //          diagonal takes both factors relative to the last token ahead of its rows, one on the
 //          diagonal is summed directly.
@@ -49,36 +51,37 @@ __device__ __forceinline__ float softplus_x(float x) { return fmaxf(x, 0.f) + lo
 __device__ __forceinline__ f32x4 mfma(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
 // ------------------------------------------------------------------ one token a row
-// NR: rows of S a lane holds, 8 NR >= dk; MT: most threads (32 columns a wave)
-template <int NR, int MT>
+// CG: lanes of 4 columns each; NR: rows of S a lane holds, NR 64 / CG >= dk; MT: most threads.
+// NR stays at 16: with 32 rows a lane, registers ran out and the compiler copied live row numbers
+// under a narrowed EXEC mask, which lost those of the other lanes.
+template <int CG, int NR, int MT>
 __global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const int* __restrict__ positions) {
+  constexpr int RG = 64 / CG, RP = RG * NR;
   extern __shared__ float lds[];
   const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x, nt = blockDim.x, lane = tid & 63, wave = tid >> 6;
   const int dk = a.dk, dv = a.dv, dvp = (dv + 3) & ~3, kh = h / (a.H / a.G);
-  float *sq = lds, *sk = sq + dk, *sa = sk + dk, *sr = sa + dk;      // q, k, decays, low-rank inputs
-  float* red = sr + a.rank;                                          // [waves]
+  float *sq = lds, *sk = sq + RP, *sa = sk + RP, *sv = sa + RP, *sg = sv + dvp;   // q, k, decays (zero past dk), v, gates
+  float *sr = sg + dvp, *red = sr + a.rank;                                       // low-rank inputs; [waves]
   const int slot = a.slots[b];
-  const int cg = lane & 7, rg = lane >> 3, c0 = wave * 32 + cg * 4;
+  const int cg = lane % CG, rg = lane / CG, c0 = (wave * CG + cg) * 4;
   const bool carry = slot >= 0 && positions[b] > 0, cok = c0 < dvp;
-  float* sp = a.state + ((size_t)max(slot, 0) * a.H + h) * dk * dvp;
-  float4 S[NR];
+  char* sp = reinterpret_cast<char*>(a.state + ((size_t)max(slot, 0) * a.H + h) * dk * dvp);
+  float4 S[NR];                              // rows past the last repeat it: their k and q are zero
 #pragma unroll
-  for (int i = 0; i < NR; ++i) {
-    const int r = i * 8 + rg;
-    S[i] = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (carry && cok && r < dk) S[i] = *reinterpret_cast<const float4*>(sp + (size_t)r * dvp + c0);
+  for (int i = 0; i < NR; ++i) S[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (carry && cok) {
+#pragma unroll
+    for (int i = 0; i < NR; ++i) S[i] = *reinterpret_cast<const float4*>(sp + (unsigned)(min(i * RG + rg, dk - 1) * dvp + c0) * 4u);
   }
   const size_t xr = (size_t)b * a.ldx, zr = (size_t)b * a.ldz;
-  float v[4], g[4];
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const bool ok = c0 + j < dv;
-    v[j] = ok ? ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.vo + h * dv + c0 + j) : 0.f;
-    g[j] = ok && rg == 0 ? ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.go + h * dv + c0 + j) : 0.f;
+  for (int i = tid; i < RP; i += nt) {
+    sq[i] = i < dk ? ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.qo + kh * dk + i) : 0.f;
+    sk[i] = i < dk ? ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.ko + kh * dk + i) : 0.f;
+    sa[i] = 0.f;
   }
-  for (int i = tid; i < dk; i += nt) {
-    sq[i] = ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.qo + kh * dk + i);
-    sk[i] = ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.ko + kh * dk + i);
+  for (int i = tid; i < dvp; i += nt) {
+    sv[i] = i < dv ? ldx1(a.X, a.xf32, a.Sx, a.xslab, xr + a.vo + h * dv + i) : 0.f;
+    sg[i] = i < dv ? ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.go + h * dv + i) : 0.f;
   }
   float qs = a.qs, ks = a.ks, beta = 1.f, al = 1.f;
   if (a.kind == LIN_CHANNEL) {
@@ -118,15 +121,17 @@ __global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const in
     ks *= 1.f / sqrtf(wave_sum(nk) + 1e-6f);
   }
   auto rows_sum = [](float x) {              // over the row groups of a column
-    x += __shfl_xor(x, 8, 64);
-    x += __shfl_xor(x, 16, 64);
-    x += __shfl_xor(x, 32, 64);
+#pragma unroll
+    for (int m = CG; m < 64; m <<= 1) x += __shfl_xor(x, m, 64);
     return x;
   };
+  float v[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] = cok ? sv[c0 + j] : 0.f;
   float p[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
-    const int r = min(i * 8 + rg, dk - 1);   // rows past the last hold zeros
+    const int r = i * RG + rg;
     const float d = a.kind == LIN_CHANNEL ? sa[r] : al, k = sk[r] * ks;
     S[i].x *= d; S[i].y *= d; S[i].z *= d; S[i].w *= d;
     p[0] += S[i].x * k; p[1] += S[i].y * k; p[2] += S[i].z * k; p[3] += S[i].w * k;
@@ -138,13 +143,11 @@ __global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const in
   float o[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
-    const int r = i * 8 + rg;
-    if (r < dk) {
-      const float k = sk[r] * ks, q = sq[r] * qs;
-      S[i].x += k * v[0]; S[i].y += k * v[1]; S[i].z += k * v[2]; S[i].w += k * v[3];
-      o[0] += S[i].x * q; o[1] += S[i].y * q; o[2] += S[i].z * q; o[3] += S[i].w * q;
-      if (slot >= 0 && cok) *reinterpret_cast<float4*>(sp + (size_t)r * dvp + c0) = S[i];
-    }
+    const int r = i * RG + rg;
+    const float k = sk[r] * ks, q = sq[r] * qs;
+    S[i].x += k * v[0]; S[i].y += k * v[1]; S[i].z += k * v[2]; S[i].w += k * v[3];
+    o[0] += S[i].x * q; o[1] += S[i].y * q; o[2] += S[i].z * q; o[3] += S[i].w * q;
+    if (slot >= 0 && cok && r < dk) *reinterpret_cast<float4*>(sp + (unsigned)(r * dvp + c0) * 4u) = S[i];
   }
   float ss = 0.f;
 #pragma unroll
@@ -161,8 +164,10 @@ __global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const in
   if (rg == 0) {
 #pragma unroll
     for (int j = 0; j < 4; ++j)
-      if (c0 + j < dv)
-        stx(a.out, a.of32, (size_t)b * a.ldo + h * dv + c0 + j, o[j] * inv * a.norm[c0 + j] * g[j] * sigmoid_f(g[j]));
+      if (c0 + j < dv) {
+        const float g = sg[c0 + j];
+        stx(a.out, a.of32, (size_t)b * a.ldo + h * dv + c0 + j, o[j] * inv * a.norm[c0 + j] * g * sigmoid_f(g));
+      }
   }
 }
 
@@ -176,15 +181,23 @@ struct ScanArgs {
 // chunk ids: sequence b's follow those of the sequences ahead of it, whatever their lengths
 __device__ __forceinline__ size_t chunk_id(const ScanArgs& s, int b, int ck, int C) { return (size_t)(s.cu[b] / C) + b + ck; }
 
-constexpr int NTP = 256;
+// between a wave's own writes to LDS and its reads of other lanes' parts
+__device__ __forceinline__ void wave_lds_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+
+constexpr int NTP = 256, PT = 20;
+constexpr int prep_q(int C, int DKP, bool delta) { return delta && 4 * C * PT > C * (DKP + 4) ? 4 * C * PT : C * (DKP + 4); }
 template <int C, int DKP, int KIND, int V>
 __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
   constexpr int PK = DKP + 4, NB = C / 16, PM = C + 4;
   constexpr bool CH = KIND == LIN_CHANNEL, DELTA = KIND == LIN_DELTA;
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  float *sQ = lds, *sK = sQ + C * PK, *sB = sK + C * PK;     // sB: [C, PK] (channel) or [C] log decays, summed
+  // delta: sQ's place later holds the waves' parts of the solution, [4, C, PT]
+  float *sQ = lds, *sK = sQ + prep_q(C, DKP, DELTA), *sB = sK + C * PK;   // sB: [C, PK] (channel) or [C] log decays, summed
   float* sM = sB + (CH ? C * PK : C);                        // delta: [C, PM]; channel: low-rank inputs [C, rank]
-  float* sbeta = sM + C * PM;                                // delta: [C]
+  float *sT = sM + C * PM, *sbeta = sT + C * PT;             // delta: inverses of 1 + M's diagonal blocks; [C]
   const DocqaLinear& a = sc.a;
   const int h = blockIdx.x, ck = blockIdx.y, b = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int q0 = sc.cu[b], L = sc.cu[b + 1] - q0, t0 = ck * C;
@@ -374,36 +387,53 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
   for (int d = tid; d < DKP; d += NTP) sc.G[cid * DKP + d] = CH ? expf(sB[(C - 1) * PK + d]) : expf(sB[C - 1]);
 
   if constexpr (DELTA) {
-    // a thread a column of [beta v | beta e^b k]: x_t <- r_t - sum_{s < t} M[t, s] x_s
-    float *gW = sc.W + cid * C * DKP, *gU = sc.U + cid * C * dvq;
-    for (int c = tid; c < dvq + DKP; c += NTP) {
-      float x[C];
-      if (c < dvq) {
+    if (tid < C) {                              // a thread a column of a diagonal block's inverse
+      const int i0 = tid & ~15, c = tid & 15;
+      float x[16];
 #pragma unroll
-        for (int t = 0; t < C; ++t)
-          x[t] = t < n && c < dv ? ldx1(a.X, a.xf32, a.Sx, a.xslab, (row0 + min(t, n - 1)) * a.ldx + a.vo + h * dv + c) * sbeta[t] : 0.f;
-      } else {
+      for (int t = 0; t < 16; ++t) {
+        float acc = t == c ? 1.f : 0.f;
 #pragma unroll
-        for (int t = 0; t < C; ++t) x[t] = sbeta[t] * expf(sB[t]) * sK[t * PK + c - dvq];
+        for (int s = 0; s < t; ++s) acc -= sM[(i0 + t) * PM + i0 + s] * x[s];
+        x[t] = acc;
+        sT[(i0 + t) * PT + c] = acc;
       }
+    }
+    __syncthreads();
+    // a wave 16 columns of [beta v | beta e^b k], block of tokens after block
+    float *gW = sc.W + cid * C * DKP, *gU = sc.U + cid * C * dvq, *buf = sQ + wave * C * PT;
+    for (int ct = wave; ct < (dvq + DKP) / 16; ct += NTP / 64) {
+      const bool val = ct * 16 < dvq;
+      const int c = ct * 16 - (val ? 0 : dvq) + fr;
+#pragma unroll 1
+      for (int i = 0; i < NB; ++i) {
+        f32x4 y, x = f32x4{0.f, 0.f, 0.f, 0.f}, acc = x;
 #pragma unroll
-      for (int t = 1; t < C; ++t) {
-        float acc = 0.f;
-#pragma unroll
-        for (int s = 0; s < (t + 3) / 4 * 4; s += 4) {
-          const float4 m = *reinterpret_cast<const float4*>(sM + t * PM + s);      // zero from s = t on
-          acc += m.x * x[s];
-          if (s + 1 < t) acc += m.y * x[s + 1];
-          if (s + 2 < t) acc += m.z * x[s + 2];
-          if (s + 3 < t) acc += m.w * x[s + 3];
+        for (int r = 0; r < 4; ++r) {
+          const int t = i * 16 + 4 * g4 + r;
+          if (val) y[r] = t < n && c < dv ? ldx1(a.X, a.xf32, a.Sx, a.xslab, (row0 + t) * a.ldx + a.vo + h * dv + c) * sbeta[t] : 0.f;
+          else y[r] = sbeta[t] * expf(sB[t]) * sK[t * PK + c];
         }
-        x[t] -= acc;
-        asm volatile("" ::: "memory");       // row by row: M is not pulled into registers ahead
-      }
+        for (int j = 0; j < i; ++j) {
+          const float4 m = *reinterpret_cast<const float4*>(sM + (i * 16 + fr) * PM + j * 16 + 4 * g4);
+          const float* p = buf + (j * 16 + 4 * g4) * PT + fr;
+          acc = mfma(m.x, p[0], acc); acc = mfma(m.y, p[PT], acc); acc = mfma(m.z, p[2 * PT], acc); acc = mfma(m.w, p[3 * PT], acc);
+        }
+        float* p = buf + (i * 16 + 4 * g4) * PT + fr;
 #pragma unroll
-      for (int t = 0; t < C; ++t) {
-        if (c < dvq) gU[t * dvq + c] = x[t];
-        else gW[t * DKP + c - dvq] = x[t];
+        for (int r = 0; r < 4; ++r) p[r * PT] = y[r] - acc[r];
+        wave_lds_sync();
+        const float4 m = *reinterpret_cast<const float4*>(sT + (i * 16 + fr) * PT + 4 * g4);
+        x = mfma(m.x, p[0], x); x = mfma(m.y, p[PT], x); x = mfma(m.z, p[2 * PT], x); x = mfma(m.w, p[3 * PT], x);
+        wave_lds_sync();
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = i * 16 + 4 * g4 + r;
+          p[r * PT] = x[r];
+          if (val) gU[t * dvq + c] = x[r];
+          else gW[t * DKP + c] = x[r];
+        }
+        wave_lds_sync();
       }
     }
   }
@@ -562,10 +592,10 @@ template <int C, int DKP, int KIND>
 int launch_scan(const ScanArgs& sc, int tokens, int B, hipStream_t s) {
   constexpr int PK = DKP + 4;
   const DocqaLinear& a = sc.a;
-  const size_t low = KIND == LIN_CHANNEL ? (size_t)C * a.rank : (size_t)C * (C + 4) + C;
-  const size_t lds = (2 * C * PK + (KIND == LIN_CHANNEL ? C * PK : C) + low) * 4;
+  const size_t low = KIND == LIN_CHANNEL ? (size_t)C * a.rank : KIND == LIN_DELTA ? (size_t)C * (C + 4 + PT + 1) : 0;
+  const size_t lds = (prep_q(C, DKP, KIND == LIN_DELTA) + C * PK + (KIND == LIN_CHANNEL ? C * PK : C) + low) * 4;
   if (lds > 160 * 1024) return -1;
-  const bool vec = a.dk % 4 == 0 && a.qo % 4 == 0 && a.ko % 4 == 0 && a.ldx % 4 == 0;
+  const bool vec = docqa_aligned16(a.X) && a.dk % 4 == 0 && a.qo % 4 == 0 && a.ko % 4 == 0 && a.ldx % 4 == 0;
   dim3 grid(a.H, sc.nchunk, B);
   auto prep = vec ? linear_prep_kernel<C, DKP, KIND, 4> : linear_prep_kernel<C, DKP, KIND, 1>;
   if (lds > 64 * 1024) {
@@ -600,19 +630,21 @@ int dispatch_scan(const ScanArgs& sc, int tokens, int B, hipStream_t s) {
 int docqa_linear_step(const DocqaLinear& a, const int* positions, int B, hipStream_t s) {
   if (B == 0) return 0;
   if (a.dk < 1 || a.dk > 256 || a.dv < 1 || a.dv > 512 || B > 65535 || !docqa_aligned16(a.state)) return -1;
-  const int waves = (a.dv + 31) / 32;
-  const size_t lds = (size_t)(3 * a.dk + a.rank + waves) * 4;
+  const bool tall = a.dk > 128;
+  if (tall && a.dv > 256) return -1;
+  const int waves = tall ? (a.dv + 15) / 16 : (a.dv + 31) / 32, dvp = (a.dv + 3) & ~3;
+  const size_t lds = (size_t)(3 * (tall ? 256 : a.dk <= 64 ? 64 : 128) + 2 * dvp + a.rank + waves) * 4;
   dim3 grid(a.H, B);
-#define RUN(NR, MT) linear_step_kernel<NR, MT><<<grid, 64 * waves, lds, s>>>(a, positions)
-#define GO(NR)                        \
-  do {                                \
-    if (waves <= 4) RUN(NR, 256);     \
-    else if (waves <= 8) RUN(NR, 512); \
-    else RUN(NR, 1024);               \
+#define RUN(CG, NR, MT) linear_step_kernel<CG, NR, MT><<<grid, 64 * waves, lds, s>>>(a, positions)
+#define GO(CG, NR)                        \
+  do {                                    \
+    if (waves <= 4) RUN(CG, NR, 256);     \
+    else if (waves <= 8) RUN(CG, NR, 512); \
+    else RUN(CG, NR, 1024);               \
   } while (0)
-  if (a.dk <= 64) GO(8);
-  else if (a.dk <= 128) GO(16);
-  else GO(32);
+  if (tall) GO(4, 16);
+  else if (a.dk <= 64) GO(8, 8);
+  else GO(8, 16);
 #undef GO
 #undef RUN
   DOCQA_CHECK_LAUNCH();

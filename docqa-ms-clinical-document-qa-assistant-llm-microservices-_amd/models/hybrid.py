@@ -333,7 +333,7 @@ def _check_post(sp: LayerSpec) -> None:
         if isinstance(s, AttentionSpec):
             if s.dim > 512 or s.vdim > 512 or s.window < 0 or s.softcap < 0:
                 raise ValueError(f"unsupported attention sizes {s}")
-        elif s.dim > 256 or s.vdim > 512:
+        elif s.dim > 256 or s.vdim > (512 if s.dim <= 128 else 256):
             raise ValueError(f"unsupported state sizes {s}")
         if isinstance(s, RetentionSpec) and (len(s.decay) != s.heads or not all(0 < d <= 1 for d in s.decay)):
             raise ValueError(f"one decay in (0, 1] per head expected: {s.decay}")
