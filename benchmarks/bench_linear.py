@@ -17,8 +17,8 @@ MFMA32 = 256 * 256 * 2.4e9       # dense fp32 FLOP/s: 256 CUs x 256 / clock x 2.
 
 # width, attention heads, their key / value heads, linear-attention heads, delta heads, head dim, window,
 # experts, chosen, expert width, shared width (with which a layer's active weights are the Llama's)
-SIZES = {"2b": (2048, 8, 2, 8, 16, 128, 1024, 16, 2, 1792, 2304),
-         "8b": (4096, 16, 4, 16, 32, 128, 1024, 16, 2, 3072, 3584)}
+SIZES = {"2b": (2048, 8, 2, 8, 16, 128, 1024, 16, 2, 1920, 2048),
+         "8b": (4096, 16, 4, 16, 32, 128, 1024, 16, 2, 2816, 4096)}
 RANK = 64
 
 

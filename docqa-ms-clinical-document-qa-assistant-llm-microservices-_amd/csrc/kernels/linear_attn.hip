@@ -439,7 +439,11 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
   }
 }
 
-// 4 waves; S rows in 16-row tiles dealt to the waves, token rows 16 to a wave
+// LDS reads and writes of every wave before it are done; loads from memory stay in flight
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+// 4 waves; S rows in 16-row tiles dealt to the waves, token rows 16 to a wave.  A chunk's operands are in
+// registers when its turn comes: each is loaded for the next chunk right after its use.
 template <int C, int DKP, int NT, bool DELTA>
 __global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
   constexpr int DVT = 16 * NT, PS = DVT + 4, RT = DKP / 16, RPW = (RT + 3) / 4, NTT = C / 16;
@@ -477,55 +481,108 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
           for (int r = 0; r < 4; ++r) sS[(rt * 16 + 4 * g4 + r) * PS + c * 16 + fr] = S[q][c][r];
     }
   };
-  // rows of a [16, K] operand at p (row stride ld) times B [K, DVT] in LDS; k runs in steps of 16, lane
-  // group g4 taking 4 consecutive k (any order will do if both operands share it)
-  auto product = [&](const float* p, int ld, const float* B, int K, f32x4* acc) {
-    const float* pr = p + (size_t)fr * ld + 4 * g4;
-#pragma unroll 8
-    for (int k0 = 0; k0 < K; k0 += 16) {
-      const float4 x = *reinterpret_cast<const float4*>(pr + k0);
-      const float* br = B + (k0 + 4 * g4) * PS + fr;
+  // k runs in steps of 16, lane group g4 taking 4 consecutive k (any order will do if both operands share it)
+  auto step = [&](const float4& x, const float* B, int k0, f32x4* acc) {
+    const float* br = B + (k0 + 4 * g4) * PS + fr;
 #pragma unroll
-      for (int c = 0; c < NT; ++c) {
-        acc[c] = mfma(x.x, br[c * 16], acc[c]);
-        acc[c] = mfma(x.y, br[PS + c * 16], acc[c]);
-        acc[c] = mfma(x.z, br[2 * PS + c * 16], acc[c]);
-        acc[c] = mfma(x.w, br[3 * PS + c * 16], acc[c]);
+    for (int c = 0; c < NT; ++c) {
+      acc[c] = mfma(x.x, br[c * 16], acc[c]);
+      acc[c] = mfma(x.y, br[PS + c * 16], acc[c]);
+      acc[c] = mfma(x.z, br[2 * PS + c * 16], acc[c]);
+      acc[c] = mfma(x.w, br[3 * PS + c * 16], acc[c]);
+    }
+  };
+  const int wt = min(wave, NTT - 1);                           // the wave's token tile (the last one's loads are idle copies)
+  constexpr int NV = C * DVT / 256;
+  float4 rW[DELTA ? RT : 1], rQ[RT], rA[NTT], rK[RPW][NTT], rG[RPW];
+  float rV[DELTA ? 4 * NT : NV];
+  auto row16 = [&](const float* p, int ld) { return reinterpret_cast<const float4*>(p + (size_t)fr * ld + 4 * g4); };
+  auto load_w = [&](size_t cid) {
+    if constexpr (DELTA) {
+      const float4* p = row16(sc.W + (cid * C + wt * 16) * DKP, DKP);
+#pragma unroll
+      for (int k = 0; k < RT; ++k) rW[k] = p[k * 4];
+    }
+  };
+  auto load_v = [&](size_t cid, int ck) {
+    if constexpr (DELTA) {
+#pragma unroll
+      for (int c = 0; c < NT; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          rV[c * 4 + r] = sc.U[(cid * C + wt * 16 + 4 * g4 + r) * dvq + min(c0 + c * 16 + fr, dvq - 1)];
+    } else {
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int e = tid + 256 * i, t = ck * C + e / DVT, c = c0 + e % DVT;
+        rV[i] = ldx1(a.X, a.xf32, a.Sx, a.xslab, (size_t)(q0 + min(t, L - 1)) * a.ldx + a.vo + h * dv + min(c, dv - 1));
       }
     }
   };
-  publish();
-  for (int ck = 0; ck * C < L; ++ck) {
-    const int n = min(C, L - ck * C);
-    const size_t row0 = q0 + ck * C, cid = chunk_id(sc, b, ck, C) * a.H + h;
-    __syncthreads();                                   // sS is written, sV free
-    if constexpr (DELTA) {
-      if (wave < NTT) {
-        f32x4 acc[NT];
+  auto load_qa = [&](size_t cid) {
+    const float4 *p = row16(sc.Q + (cid * C + wt * 16) * DKP, DKP), *q = row16(sc.A + (cid * C + wt * 16) * C, C);
 #pragma unroll
-        for (int c = 0; c < NT; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
-        product(sc.W + cid * C * DKP + wave * 16 * DKP, DKP, sS, DKP, acc);
+    for (int k = 0; k < RT; ++k) rQ[k] = p[k * 4];
 #pragma unroll
-        for (int c = 0; c < NT; ++c)
+    for (int k = 0; k < NTT; ++k) rA[k] = q[k * 4];
+  };
+  auto load_k = [&](size_t cid) {
 #pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const int t = wave * 16 + 4 * g4 + r, col = c0 + c * 16 + fr;
-            sV[t * PS + c * 16 + fr] = col < dvq ? sc.U[(cid * C + t) * dvq + col] - acc[c][r] : 0.f;
-          }
-      }
-    } else {
-      for (int e = tid; e < C * DVT; e += 256) {
-        const int t = e / DVT, c = e % DVT;
-        sV[t * PS + c] = t < n && c0 + c < dv ? ldx1(a.X, a.xf32, a.Sx, a.xslab, (row0 + t) * a.ldx + a.vo + h * dv + c0 + c) : 0.f;
-      }
+    for (int q = 0; q < RPW; ++q) {
+      const int rt = min(wave + 4 * q, RT - 1);
+      const float4* p = row16(sc.K + (cid * DKP + rt * 16) * C, C);
+#pragma unroll
+      for (int k = 0; k < NTT; ++k) rK[q][k] = p[k * 4];
+      rG[q] = *reinterpret_cast<const float4*>(sc.G + cid * DKP + rt * 16 + 4 * g4);
     }
-    __syncthreads();
-    if (wave < NTT && wave * 16 < n) {
+  };
+  const int chunks = (L + C - 1) / C;
+  const size_t id0 = chunk_id(sc, b, 0, C) * a.H + h;          // chunk ck's: id0 + ck H
+  load_w(id0);
+  load_v(id0, 0);
+  load_qa(id0);
+  load_k(id0);
+  publish();
+#pragma unroll 1
+  for (int ck = 0; ck < chunks; ++ck) {
+    const int n = min(C, L - ck * C), nx = min(ck + 1, chunks - 1);
+    const size_t row0 = q0 + ck * C, nid = id0 + (size_t)nx * a.H;
+    lds_barrier();                                     // sS is written, sV free
+    if constexpr (DELTA) {
       f32x4 acc[NT];
 #pragma unroll
       for (int c = 0; c < NT; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
-      product(sc.Q + cid * C * DKP + wave * 16 * DKP, DKP, sS, DKP, acc);
-      product(sc.A + cid * C * C + wave * 16 * C, C, sV, (wave + 1) * 16, acc);
+      if (wave < NTT) {
+#pragma unroll
+        for (int k = 0; k < RT; ++k) step(rW[k], sS, k * 16, acc);
+#pragma unroll
+        for (int c = 0; c < NT; ++c)
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            sV[(wave * 16 + 4 * g4 + r) * PS + c * 16 + fr] = c0 + c * 16 + fr < dvq ? rV[c * 4 + r] - acc[c][r] : 0.f;
+      }
+      load_w(nid);
+    } else {
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int e = tid + 256 * i, t = e / DVT, c = e % DVT;
+        sV[t * PS + c] = t < n && c0 + c < dv ? rV[i] : 0.f;
+      }
+    }
+    load_v(nid, nx);
+    lds_barrier();
+    f32x4 acc[NT];
+#pragma unroll
+    for (int c = 0; c < NT; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (wave < NTT && wave * 16 < n) {
+#pragma unroll
+      for (int k = 0; k < RT; ++k) step(rQ[k], sS, k * 16, acc);
+#pragma unroll
+      for (int k = 0; k < NTT; ++k)
+        if (k <= wave) step(rA[k], sV, k * 16, acc);
+    }
+    load_qa(nid);
+    if (wave < NTT) {
 #pragma unroll
       for (int c = 0; c < NT; ++c)
 #pragma unroll
@@ -536,18 +593,15 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
     }
 #pragma unroll
     for (int q = 0; q < RPW; ++q) {
-      const int rt = wave + 4 * q;
-      if (rt < RT) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const float d = sc.G[cid * DKP + rt * 16 + 4 * g4 + r];
-#pragma unroll
-          for (int c = 0; c < NT; ++c) S[q][c][r] *= d;
-        }
-        product(sc.K + (cid * DKP + rt * 16) * C, C, sV, C, S[q]);
+      for (int c = 0; c < NT; ++c) {
+        S[q][c][0] *= rG[q].x; S[q][c][1] *= rG[q].y; S[q][c][2] *= rG[q].z; S[q][c][3] *= rG[q].w;
       }
+#pragma unroll
+      for (int k = 0; k < NTT; ++k) step(rK[q][k], sV, k * 16, S[q]);
     }
-    __syncthreads();                                   // everyone has read sS
+    load_k(nid);
+    lds_barrier();                                     // everyone has read sS
     publish();
   }
   if (slot < 0) return;

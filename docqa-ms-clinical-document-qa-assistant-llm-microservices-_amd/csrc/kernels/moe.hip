@@ -6,7 +6,7 @@
 // * a (token, choice) pair p = t top + k is a row of the grouped products; gate and up rows meet in
 //   the same lane's accumulators, so the activation is the first product's epilogue.
 //   Few pairs (decode): a workgroup takes one expert and 16 (or 32) output columns, finds the expert's
-//   pairs itself, streams its weight rows once into registers, K split over 4 waves.
+//   pairs itself, streams its weight rows once into registers, K split over 4 or 8 waves.
 //   Many (prompts): pairs sorted by expert in one small launch, then 128 x 128 tiles as in gemm.hip,
 //   A rows gathered by the LDS-DMA's per-lane source addresses.
 //   fp32 and odd sizes: a wave an output element.
@@ -18,7 +18,7 @@ using namespace docqa;
 
 namespace {
 constexpr int kSkinnyPairs = 512;       // pairs up to which a launch finds its rows itself
-constexpr int BM = 128, BN = 128, BK = 64;
+constexpr int BM = 128, BK = 64, kGroup = 8;
 
 __device__ __forceinline__ float sigmoid_x(float x) { return 1.f / (1.f + expf(-x)); }
 __device__ __forceinline__ float glu_f(float g, float u, float s) {
@@ -53,38 +53,43 @@ __device__ __forceinline__ void pick(const float* sc, int E, int top, int* ids, 
   }
 }
 
-// 16 tokens a workgroup of 8 waves; x [T, K], w [N, K], K % 32 == 0
-__global__ __launch_bounds__(512) void moe_route_mfma_kernel(const uint16_t* __restrict__ x, const uint16_t* __restrict__ w,
-                                                             int* __restrict__ ids, float* __restrict__ wts,
-                                                             float* __restrict__ rest, int T, int K, int N, int E, int top) {
+// 16 tokens a workgroup of 16 waves that split K, 32 columns a pass; x [T, K], w [N, K], K % 32 == 0
+__global__ __launch_bounds__(1024) void moe_route_mfma_kernel(const uint16_t* __restrict__ x, const uint16_t* __restrict__ w,
+                                                              int* __restrict__ ids, float* __restrict__ wts,
+                                                              float* __restrict__ rest, int T, int K, int N, int E, int top) {
   extern __shared__ float sc[];              // [16][N] scores
-  __shared__ float red[8][16][17];
+  __shared__ float red[16][2][16][17];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
   const int t0 = blockIdx.x * 16;
   const uint16_t* xp = x + (size_t)min(t0 + fr, T - 1) * K + g4 * 8;
-  for (int n0 = 0; n0 < N; n0 += 16) {
-    const uint16_t* wp = w + (size_t)min(n0 + fr, N - 1) * K + g4 * 8;
-    f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int n0 = 0; n0 < N; n0 += 32) {
+    const uint16_t *w0 = w + (size_t)min(n0 + fr, N - 1) * K + g4 * 8, *w1 = w + (size_t)min(n0 + 16 + fr, N - 1) * K + g4 * 8;
+    f32x4 a0 = f32x4{0.f, 0.f, 0.f, 0.f}, a1 = a0;
 #pragma unroll 4
-    for (int k = wave * 32; k < K; k += 256)
-      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(xp + k),
-                                                    *reinterpret_cast<const bf16x8*>(wp + k), acc, 0, 0, 0);
+    for (int k = wave * 32; k < K; k += 512) {
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>(xp + k);
+      a0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, *reinterpret_cast<const bf16x8*>(w0 + k), a0, 0, 0, 0);
+      a1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, *reinterpret_cast<const bf16x8*>(w1 + k), a1, 0, 0, 0);
+    }
 #pragma unroll
-    for (int r = 0; r < 4; ++r) red[wave][g4 * 4 + r][fr] = acc[r];
+    for (int r = 0; r < 4; ++r) {
+      red[wave][0][g4 * 4 + r][fr] = a0[r];
+      red[wave][1][g4 * 4 + r][fr] = a1[r];
+    }
     __syncthreads();
-    if (tid < 256) {
-      const int t = tid >> 4, c = tid & 15;
+    if (tid < 512) {
+      const int t = tid >> 5, c = tid & 31;
       float z = 0.f;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) z += red[i][t][c];
+      for (int i = 0; i < 16; ++i) z += red[i][c >> 4][t][c & 15];
       if (n0 + c < N) sc[t * N + n0 + c] = sigmoid_x(z);
     }
     __syncthreads();
   }
-  for (int i = wave; i < 16 && t0 + i < T; i += 8) {
-    const size_t t = t0 + i;
-    pick(sc + i * N, E, top, ids + t * top, wts + t * top);
-    for (int c = E + lane; c < N; c += 64) rest[t * (N - E) + c - E] = sc[i * N + c];
+  if (t0 + wave < T) {
+    const size_t t = t0 + wave;
+    pick(sc + wave * N, E, top, ids + t * top, wts + t * top);
+    for (int c = E + lane; c < N; c += 64) rest[t * (N - E) + c - E] = sc[wave * N + c];
   }
 }
 
@@ -133,13 +138,13 @@ __global__ __launch_bounds__(256) void moe_plain_kernel(const T* __restrict__ x,
 // ------------------------------------------------------------------ few pairs
 // blockIdx.y: the expert, or (E > pairs) a pair whose expert no earlier pair has.  MT row tiles of 16 at
 // a time against two column tiles of 16: gate and up rows n0.. (UP), or rows n0.. and n0 + 16.. (down)
-template <int MT, bool UP>
-__global__ __launch_bounds__(256) void moe_skinny_kernel(const uint16_t* __restrict__ x, const int* __restrict__ ids,
+template <int MT, int NW, bool UP>
+__global__ __launch_bounds__(64 * NW) void moe_skinny_kernel(const uint16_t* __restrict__ x, const int* __restrict__ ids,
                                                          const float* __restrict__ wts, const uint16_t* __restrict__ w,
                                                          uint16_t* __restrict__ y, int Tn, int top, int E, int K, int N) {
   __shared__ int rows[kSkinnyPairs];
   __shared__ int count;
-  __shared__ float red[4][MT][2][16][17];
+  __shared__ float red[NW][MT][2][16][17];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
   const int P = Tn * top, n0 = blockIdx.x * (UP ? 16 : 32);
   int e = blockIdx.y;
@@ -151,7 +156,7 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(const uint16_t* __restr
   }
   if (tid == 0) count = 0;
   __syncthreads();
-  for (int p = tid; p < P; p += 256)
+  for (int p = tid; p < P; p += 64 * NW)
     if (ids[p] == e) rows[atomicAdd(&count, 1)] = p;
   __syncthreads();
   const int m = count;
@@ -167,7 +172,7 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(const uint16_t* __restr
       acc[i][0] = acc[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
 #pragma unroll 4
-    for (int k = wave * 32; k < K; k += 128) {
+    for (int k = wave * 32; k < K; k += 32 * NW) {
       const bf16x8 b0 = *reinterpret_cast<const bf16x8*>(w0 + k), b1 = *reinterpret_cast<const bf16x8*>(w1 + k);
 #pragma unroll
       for (int i = 0; i < MT; ++i) {
@@ -188,10 +193,14 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(const uint16_t* __restr
 #pragma unroll
     for (int i = 0; i < MT; ++i) {
       const int row = r0 + i * 16 + r;
-      if (row >= m) continue;
+      if (r >= 16 || row >= m) continue;
       const int p = rows[row];
-      const float a = (red[0][i][0][r][c] + red[1][i][0][r][c]) + (red[2][i][0][r][c] + red[3][i][0][r][c]);
-      const float b = (red[0][i][1][r][c] + red[1][i][1][r][c]) + (red[2][i][1][r][c] + red[3][i][1][r][c]);
+      float a = 0.f, b = 0.f;
+#pragma unroll
+      for (int q = 0; q < NW; ++q) {
+        a += red[q][i][0][r][c];
+        b += red[q][i][1][r][c];
+      }
       if constexpr (UP) {
         if (n0 + c < N) y[(size_t)p * N + n0 + c] = f2bf(glu_f(a, b, wts[p]));
       } else {
@@ -251,7 +260,10 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const uint16_t* __restric
   __shared__ int srow[BM];
   const int nbn = (N + (UP ? 63 : 127)) / (UP ? 64 : 128);
   const int wg = xcd_remap(blockIdx.x, gridDim.x);
-  const int bm = wg / nbn, bn = wg % nbn, P = Tn * top;
+  // row tiles in groups of kGroup, column after column: a group's tiles, mostly of one expert, share the
+  // weight rows they read at about the same time
+  const int g0 = wg / (kGroup * nbn) * kGroup, gs = min(kGroup, tiles - g0), gi = wg - g0 * nbn;
+  const int bm = g0 + gi % gs, bn = gi / gs, P = Tn * top;
   const int *te = scratch + P, *tb = te + tiles, *tn = tb + tiles;
   const int e = te[bm];
   if (e < 0) return;
@@ -369,9 +381,10 @@ template <int MT>
 int skinny(const uint16_t* x, const int* ids, const float* wts, const uint16_t* up, const uint16_t* down, uint16_t* act,
            uint16_t* out, int Tn, int top, int E, int K, int F, int W, hipStream_t s) {
   const int gy = E < Tn * top ? E : Tn * top;
-  moe_skinny_kernel<MT, true><<<dim3((F + 15) / 16, gy), 256, 0, s>>>(x, ids, wts, up, act, Tn, top, E, K, F);
+  constexpr int NW = MT == 1 ? 8 : 4;
+  moe_skinny_kernel<MT, NW, true><<<dim3((F + 15) / 16, gy), 64 * NW, 0, s>>>(x, ids, wts, up, act, Tn, top, E, K, F);
   DOCQA_CHECK_LAUNCH();
-  moe_skinny_kernel<MT, false><<<dim3((W + 31) / 32, gy), 256, 0, s>>>(act, ids, wts, down, out, Tn, top, E, F, W);
+  moe_skinny_kernel<MT, NW, false><<<dim3((W + 31) / 32, gy), 64 * NW, 0, s>>>(act, ids, wts, down, out, Tn, top, E, F, W);
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
@@ -381,8 +394,8 @@ int docqa_moe_route(const void* x, const void* w, int f32, int* ids, float* wts,
                     int top, hipStream_t s) {
   if (T == 0) return 0;
   if (E < 1 || E > 512 || N < E || N > 1024 || top < 1 || top > E || K < 1) return -1;
-  if (!f32 && K % 32 == 0 && 16 * N * 4 <= 64 * 1024 - 10 * 1024)
-    moe_route_mfma_kernel<<<(T + 15) / 16, 512, (size_t)16 * N * 4, s>>>((const uint16_t*)x, (const uint16_t*)w, ids, wts, rest, T,
+  if (!f32 && K % 32 == 0 && 16 * N * 4 <= 64 * 1024 - 36 * 1024)
+    moe_route_mfma_kernel<<<(T + 15) / 16, 1024, (size_t)16 * N * 4, s>>>((const uint16_t*)x, (const uint16_t*)w, ids, wts, rest, T,
                                                                        K, N, E, top);
   else if (f32)
     moe_route_kernel<float><<<T, 256, (size_t)N * 4, s>>>((const float*)x, (const float*)w, ids, wts, rest, K, N, E, top);
