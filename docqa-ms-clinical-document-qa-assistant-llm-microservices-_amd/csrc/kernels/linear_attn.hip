@@ -187,16 +187,18 @@ __device__ __forceinline__ void wave_lds_sync() {
   __builtin_amdgcn_wave_barrier();
 }
 
-constexpr int NTP = 256, PT = 20;
-constexpr int prep_q(int C, int DKP, bool delta) { return delta && 4 * C * PT > C * (DKP + 4) ? 4 * C * PT : C * (DKP + 4); }
+constexpr int NTP = 512, NWP = NTP / 64, PT = 20;
+constexpr int prep_q(int C, int DKP, bool delta) { return delta && NWP * C * PT > C * (DKP + 4) ? NWP * C * PT : C * (DKP + 4); }
+// pitch of the low-rank inputs: the rank in whole MFMA steps
+__host__ __device__ __forceinline__ int rank_pitch(int rank) { return ((rank + 15) & ~15) + 4; }
 template <int C, int DKP, int KIND, int V>
 __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
   constexpr int PK = DKP + 4, NB = C / 16, PM = C + 4;
   constexpr bool CH = KIND == LIN_CHANNEL, DELTA = KIND == LIN_DELTA;
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  // delta: sQ's place later holds the waves' parts of the solution, [4, C, PT]
+  // delta: sQ's place later holds the waves' parts of the solution, [NWP, C, PT]
   float *sQ = lds, *sK = sQ + prep_q(C, DKP, DELTA), *sB = sK + C * PK;   // sB: [C, PK] (channel) or [C] log decays, summed
-  float* sM = sB + (CH ? C * PK : C);                        // delta: [C, PM]; channel: low-rank inputs [C, rank]
+  float* sM = sB + (CH ? C * PK : C);                        // delta: [C, PM]; channel: low-rank inputs [C, rank_pitch]
   float *sT = sM + C * PM, *sbeta = sT + C * PT;             // delta: inverses of 1 + M's diagonal blocks; [C]
   const DocqaLinear& a = sc.a;
   const int h = blockIdx.x, ck = blockIdx.y, b = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -222,9 +224,10 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
     }
   }
   if constexpr (CH) {
-    for (int e = tid; e < C * a.rank; e += NTP) {
-      const int t = e / a.rank, r = e % a.rank;
-      sM[e] = t < n ? ldx1(a.Z, a.zf32, a.Sz, a.zslab, (row0 + t) * a.ldz + a.ao + r) : 0.f;
+    const int rp = rank_pitch(a.rank);
+    for (int e = tid; e < C * rp; e += NTP) {
+      const int t = e / rp, r = e % rp;
+      sM[e] = t < n && r < a.rank ? ldx1(a.Z, a.zf32, a.Sz, a.zslab, (row0 + t) * a.ldz + a.ao + r) : 0.f;
     }
   } else if (wave == 0) {
     float la = 0.f;
@@ -255,7 +258,7 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
     __syncthreads();
   }
   // scales (and unit norms) in place
-  for (int t = wave; t < C; t += NTP / 64) {
+  for (int t = wave; t < C; t += NWP) {
     float qs = a.qs, ks = a.ks;
     if constexpr (DELTA) {
       float nq = 0.f, nk = 0.f;
@@ -272,26 +275,37 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
     }
   }
   if constexpr (CH) {
-    // log decays and their sums: a thread a channel and a stretch of tokens
+    // log decays: z of 16 tokens x 16 channels a wave
+    const int fr = lane & 15, g4 = lane >> 4, rp = rank_pitch(a.rank);
+    for (int it = wave; it < NB * (DKP / 16); it += NWP) {
+      const int t = it % NB * 16, d = it / NB * 16 + fr;
+      const float* w = a.w_gate + ((size_t)h * dk + min(d, dk - 1)) * a.rank;
+      f32x4 z = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int k0 = 0; k0 < a.rank; k0 += 16) {
+        const int k = k0 + 4 * g4;
+        const float4 x = *reinterpret_cast<const float4*>(sM + (t + fr) * rp + k);     // zero past the rank
+        const int last = a.rank - 1;
+        z = mfma(x.x, w[min(k, last)], z);
+        z = mfma(x.y, w[min(k + 1, last)], z);
+        z = mfma(x.z, w[min(k + 2, last)], z);
+        z = mfma(x.w, w[min(k + 3, last)], z);
+      }
+      const float bias = d < dk ? a.b_gate[h * dk + d] : 0.f;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int tt = t + 4 * g4 + r;
+        sB[tt * PK + d] = d < dk && tt < n ? -softplus_x(-(z[r] + bias)) * a.inv_tau : 0.f;
+      }
+    }
+    __syncthreads();
+    // their sums: a thread a channel and a stretch of tokens
     constexpr int NS = NTP / DKP >= 4 ? 4 : NTP / DKP >= 2 ? 2 : 1, TS = C / NS;
     for (int e = tid; e < DKP * NS; e += NTP) {
       const int d = e % DKP, s = e / DKP;
-      float acc[TS];
-      const float bias = d < dk ? a.b_gate[h * dk + d] : 0.f;
-#pragma unroll
-      for (int i = 0; i < TS; ++i) acc[i] = bias;
-      if (d < dk) {
-        const float* w = a.w_gate + ((size_t)h * dk + d) * a.rank;
-        for (int r = 0; r < a.rank; ++r) {
-          const float wr = w[r];
-#pragma unroll
-          for (int i = 0; i < TS; ++i) acc[i] += wr * sM[(s * TS + i) * a.rank + r];
-        }
-      }
       float sum = 0.f;
-#pragma unroll
+#pragma unroll 8
       for (int i = 0; i < TS; ++i) {
-        if (d < dk && s * TS + i < n) sum -= softplus_x(-acc[i]) * a.inv_tau;
+        sum += sB[(s * TS + i) * PK + d];
         sB[(s * TS + i) * PK + d] = sum;
       }
     }
@@ -312,12 +326,12 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
 
   // blocks of A (and M) on or below the diagonal
   const int fr = lane & 15, g4 = lane >> 4;
-  float* gA = sc.A + cid * C * C;
+  float *gA = sc.A + cid * C * C, *gU = sc.U + cid * C * dvq;
   int item = 0;
   for (int i = 0; i < NB; ++i)
     for (int j = 0; j <= i; ++j) {
       if (CH && i == j) continue;
-      if ((item++ & 3) != wave) continue;
+      if (item++ % NWP != wave) continue;
       f32x4 qa = f32x4{0.f, 0.f, 0.f, 0.f}, ka = qa;
       const int tr = i * 16 + fr, sr = j * 16 + fr, ref = i * 16 - 1;
 #pragma unroll 4
@@ -347,8 +361,8 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
       }
     }
   if constexpr (CH) {
-    const int t16 = tid >> 4, s16 = tid & 15;
-    for (int i = 0; i < NB; ++i) {
+    const int t16 = (tid >> 4) & 15, s16 = tid & 15;
+    for (int i = tid >> 8; i < NB; i += NTP / 256) {
       const int t = i * 16 + t16, s = i * 16 + s16;
       float acc = 0.f;
       if (s <= t) {
@@ -386,6 +400,16 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
   }
   for (int d = tid; d < DKP; d += NTP) sc.G[cid * DKP + d] = CH ? expf(sB[(C - 1) * PK + d]) : expf(sB[C - 1]);
 
+  if constexpr (!DELTA) {
+    for (int e = tid; e < C * (dvq / V); e += NTP) {
+      const int t = e / (dvq / V), c = (e % (dvq / V)) * V;
+      float v[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] = 0.f;
+      if (t < n && c < dv) ldx<V>(a.X, a.xf32, a.Sx, a.xslab, (row0 + t) * a.ldx + a.vo + h * dv + c, v);
+      stv<V>(gU + t * dvq + c, v);
+    }
+  }
   if constexpr (DELTA) {
     if (tid < C) {                              // a thread a column of a diagonal block's inverse
       const int i0 = tid & ~15, c = tid & 15;
@@ -401,19 +425,38 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
     }
     __syncthreads();
     // a wave 16 columns of [beta v | beta e^b k], block of tokens after block
-    float *gW = sc.W + cid * C * DKP, *gU = sc.U + cid * C * dvq, *buf = sQ + wave * C * PT;
-    for (int ct = wave; ct < (dvq + DKP) / 16; ct += NTP / 64) {
+    float *gW = sc.W + cid * C * DKP, *buf = sQ + wave * C * PT;
+    for (int ct = wave; ct < (dvq + DKP) / 16; ct += NWP) {
       const bool val = ct * 16 < dvq;
       const int c = ct * 16 - (val ? 0 : dvq) + fr;
-#pragma unroll 1
-      for (int i = 0; i < NB; ++i) {
-        f32x4 y, x = f32x4{0.f, 0.f, 0.f, 0.f}, acc = x;
+      float y[NB][4];
+      if (val) {
+        const size_t col = (size_t)a.vo + h * dv + min(c, dv - 1);
+        if (a.Sx == 1 && !a.xf32) {             // all of them in flight together
+          const uint16_t* X = (const uint16_t*)a.X + col;
+#pragma unroll
+          for (int i = 0; i < NB; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) y[i][r] = ld1(X + (row0 + min(i * 16 + 4 * g4 + r, n - 1)) * a.ldx);
+        } else {
+#pragma unroll
+          for (int i = 0; i < NB; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+              y[i][r] = ldx1(a.X, a.xf32, a.Sx, a.xslab, (row0 + min(i * 16 + 4 * g4 + r, n - 1)) * a.ldx + col);
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < NB; ++i)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int t = i * 16 + 4 * g4 + r;
-          if (val) y[r] = t < n && c < dv ? ldx1(a.X, a.xf32, a.Sx, a.xslab, (row0 + t) * a.ldx + a.vo + h * dv + c) * sbeta[t] : 0.f;
-          else y[r] = sbeta[t] * expf(sB[t]) * sK[t * PK + c];
+          y[i][r] = sbeta[t] * (val ? (t < n && c < dv ? y[i][r] : 0.f) : expf(sB[t]) * sK[t * PK + c]);
         }
+#pragma unroll
+      for (int i = 0; i < NB; ++i) {
+        f32x4 x = f32x4{0.f, 0.f, 0.f, 0.f}, acc = x;
+#pragma unroll
         for (int j = 0; j < i; ++j) {
           const float4 m = *reinterpret_cast<const float4*>(sM + (i * 16 + fr) * PM + j * 16 + 4 * g4);
           const float* p = buf + (j * 16 + 4 * g4) * PT + fr;
@@ -421,7 +464,7 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
         }
         float* p = buf + (i * 16 + 4 * g4) * PT + fr;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) p[r * PT] = y[r] - acc[r];
+        for (int r = 0; r < 4; ++r) p[r * PT] = y[i][r] - acc[r];
         wave_lds_sync();
         const float4 m = *reinterpret_cast<const float4*>(sT + (i * 16 + fr) * PT + 4 * g4);
         x = mfma(m.x, p[0], x); x = mfma(m.y, p[PT], x); x = mfma(m.z, p[2 * PT], x); x = mfma(m.w, p[3 * PT], x);
@@ -493,9 +536,8 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
     }
   };
   const int wt = min(wave, NTT - 1);                           // the wave's token tile (the last one's loads are idle copies)
-  constexpr int NV = C * DVT / 256;
   float4 rW[DELTA ? RT : 1], rQ[RT], rA[NTT], rK[RPW][NTT], rG[RPW];
-  float rV[DELTA ? 4 * NT : NV];
+  float rV[4 * NT];
   auto row16 = [&](const float* p, int ld) { return reinterpret_cast<const float4*>(p + (size_t)fr * ld + 4 * g4); };
   auto load_w = [&](size_t cid) {
     if constexpr (DELTA) {
@@ -504,20 +546,12 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
       for (int k = 0; k < RT; ++k) rW[k] = p[k * 4];
     }
   };
-  auto load_v = [&](size_t cid, int ck) {
-    if constexpr (DELTA) {
+  auto load_v = [&](size_t cid) {
 #pragma unroll
-      for (int c = 0; c < NT; ++c)
+    for (int c = 0; c < NT; ++c)
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          rV[c * 4 + r] = sc.U[(cid * C + wt * 16 + 4 * g4 + r) * dvq + min(c0 + c * 16 + fr, dvq - 1)];
-    } else {
-#pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const int e = tid + 256 * i, t = ck * C + e / DVT, c = c0 + e % DVT;
-        rV[i] = ldx1(a.X, a.xf32, a.Sx, a.xslab, (size_t)(q0 + min(t, L - 1)) * a.ldx + a.vo + h * dv + min(c, dv - 1));
-      }
-    }
+      for (int r = 0; r < 4; ++r)
+        rV[c * 4 + r] = sc.U[(cid * C + wt * 16 + 4 * g4 + r) * dvq + min(c0 + c * 16 + fr, dvq - 1)];
   };
   auto load_qa = [&](size_t cid) {
     const float4 *p = row16(sc.Q + (cid * C + wt * 16) * DKP, DKP), *q = row16(sc.A + (cid * C + wt * 16) * C, C);
@@ -539,7 +573,7 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
   const int chunks = (L + C - 1) / C;
   const size_t id0 = chunk_id(sc, b, 0, C) * a.H + h;          // chunk ck's: id0 + ck H
   load_w(id0);
-  load_v(id0, 0);
+  load_v(id0);
   load_qa(id0);
   load_k(id0);
   publish();
@@ -548,32 +582,23 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
     const int n = min(C, L - ck * C), nx = min(ck + 1, chunks - 1);
     const size_t row0 = q0 + ck * C, nid = id0 + (size_t)nx * a.H;
     lds_barrier();                                     // sS is written, sV free
-    if constexpr (DELTA) {
-      f32x4 acc[NT];
+    f32x4 w[NT], acc[NT];
 #pragma unroll
-      for (int c = 0; c < NT; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (wave < NTT) {
+    for (int c = 0; c < NT; ++c) w[c] = acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (wave < NTT) {
+      if constexpr (DELTA) {
 #pragma unroll
-        for (int k = 0; k < RT; ++k) step(rW[k], sS, k * 16, acc);
-#pragma unroll
-        for (int c = 0; c < NT; ++c)
-#pragma unroll
-          for (int r = 0; r < 4; ++r)
-            sV[(wave * 16 + 4 * g4 + r) * PS + c * 16 + fr] = c0 + c * 16 + fr < dvq ? rV[c * 4 + r] - acc[c][r] : 0.f;
+        for (int k = 0; k < RT; ++k) step(rW[k], sS, k * 16, w);
       }
-      load_w(nid);
-    } else {
 #pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const int e = tid + 256 * i, t = e / DVT, c = e % DVT;
-        sV[t * PS + c] = t < n && c0 + c < dv ? rV[i] : 0.f;
-      }
+      for (int c = 0; c < NT; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          sV[(wave * 16 + 4 * g4 + r) * PS + c * 16 + fr] = c0 + c * 16 + fr < dvq ? rV[c * 4 + r] - w[c][r] : 0.f;
     }
-    load_v(nid, nx);
+    load_w(nid);
+    load_v(nid);
     lds_barrier();
-    f32x4 acc[NT];
-#pragma unroll
-    for (int c = 0; c < NT; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (wave < NTT && wave * 16 < n) {
 #pragma unroll
       for (int k = 0; k < RT; ++k) step(rQ[k], sS, k * 16, acc);
@@ -618,38 +643,55 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(ScanArgs sc) {
   }
 }
 
-// a wave a (token, head)
+// LR lanes a (token, head), V columns at a time each, NI times
+template <int LR, int V, int NI>
 __global__ __launch_bounds__(256) void linear_gate_kernel(DocqaLinear a, const float* __restrict__ O, int tokens) {
-  const int u = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int u = blockIdx.x * (256 / LR) + threadIdx.x / LR, lane = threadIdx.x % LR;
   const int t = u / a.H, h = u % a.H, dv = a.dv, dvq = (dv + 15) & ~15;
-  if (t >= tokens) return;
-  const float* o = O + ((size_t)t * a.H + h) * dvq;
-  float x[8], ss = 0.f;
+  const bool ok = t < tokens;
+  const float* o = O + ((size_t)(ok ? t : 0) * a.H + h) * dvq;
+  float x[NI][V], ss = 0.f;
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
-    const int c = lane + 64 * i;
-    x[i] = c < dv ? o[c] : 0.f;
-    ss += x[i] * x[i];
-  }
-  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)dv + a.eps);
+  for (int i = 0; i < NI; ++i) {
+    const int c = (lane + LR * i) * V;
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
-    const int c = lane + 64 * i;
-    if (c < dv) {
-      const float g = ldx1(a.Z, a.zf32, a.Sz, a.zslab, (size_t)t * a.ldz + a.go + h * dv + c);
-      stx(a.out, a.of32, (size_t)t * a.ldo + h * dv + c, x[i] * inv * a.norm[c] * g * sigmoid_f(g));
-    }
+    for (int j = 0; j < V; ++j) x[i][j] = 0.f;
+    if (c < dv) ldv<V>(o + c, x[i]);
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss += x[i][j] * x[i][j];
   }
+  const float inv = 1.f / sqrtf(group_sum<LR>(ss) / (float)dv + a.eps);
+  if (!ok) return;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int c = (lane + LR * i) * V;
+    if (c >= dv) continue;
+    float g[V], w[V];
+    ldx<V>(a.Z, a.zf32, a.Sz, a.zslab, (size_t)t * a.ldz + a.go + h * dv + c, g);
+    ldv<V>(a.norm + c, w);
+#pragma unroll
+    for (int j = 0; j < V; ++j) g[j] = x[i][j] * inv * w[j] * g[j] * sigmoid_f(g[j]);
+    const size_t at = (size_t)t * a.ldo + h * dv + c;
+    if (a.of32) stv<V>((float*)a.out + at, g);
+    else stv<V>((uint16_t*)a.out + at, g);
+  }
+}
+
+template <int LR, int V, int NI>
+void launch_gate(const DocqaLinear& a, const float* O, int tokens, hipStream_t s) {
+  const long long rows = (long long)tokens * a.H;
+  linear_gate_kernel<LR, V, NI><<<(unsigned)((rows + 256 / LR - 1) / (256 / LR)), 256, 0, s>>>(a, O, tokens);
 }
 
 template <int C, int DKP, int KIND>
 int launch_scan(const ScanArgs& sc, int tokens, int B, hipStream_t s) {
   constexpr int PK = DKP + 4;
   const DocqaLinear& a = sc.a;
-  const size_t low = KIND == LIN_CHANNEL ? (size_t)C * a.rank : KIND == LIN_DELTA ? (size_t)C * (C + 4 + PT + 1) : 0;
+  const size_t low = KIND == LIN_CHANNEL ? (size_t)C * rank_pitch(a.rank) : KIND == LIN_DELTA ? (size_t)C * (C + 4 + PT + 1) : 0;
   const size_t lds = (prep_q(C, DKP, KIND == LIN_DELTA) + C * PK + (KIND == LIN_CHANNEL ? C * PK : C) + low) * 4;
   if (lds > 160 * 1024) return -1;
-  const bool vec = docqa_aligned16(a.X) && a.dk % 4 == 0 && a.qo % 4 == 0 && a.ko % 4 == 0 && a.ldx % 4 == 0;
+  const bool vec = docqa_aligned16(a.X) && a.dk % 4 == 0 && a.qo % 4 == 0 && a.ko % 4 == 0 && a.ldx % 4 == 0 && a.dv % 4 == 0 &&
+                   a.vo % 4 == 0;
   dim3 grid(a.H, sc.nchunk, B);
   auto prep = vec ? linear_prep_kernel<C, DKP, KIND, 4> : linear_prep_kernel<C, DKP, KIND, 1>;
   if (lds > 64 * 1024) {
@@ -664,7 +706,12 @@ int launch_scan(const ScanArgs& sc, int tokens, int B, hipStream_t s) {
   if (one <= 512 || dvq == 16) linear_chunk_kernel<C, DKP, 1, KIND == LIN_DELTA><<<(unsigned)one, 256, 0, s>>>(sc);
   else linear_chunk_kernel<C, DKP, 2, KIND == LIN_DELTA><<<(unsigned)((long long)B * a.H * ((dvq + 31) / 32)), 256, 0, s>>>(sc);
   DOCQA_CHECK_LAUNCH();
-  linear_gate_kernel<<<(unsigned)(((long long)tokens * a.H + 3) / 4), 256, 0, s>>>(a, sc.O, tokens);
+  const bool v4 = a.dv % 4 == 0 && a.go % 4 == 0 && a.ldz % 4 == 0 && a.ldo % 4 == 0 && docqa_aligned16(a.Z) &&
+                  docqa_aligned16(a.out) && docqa_aligned16(a.norm);
+  if (!v4) launch_gate<64, 1, 8>(a, sc.O, tokens, s);
+  else if (a.dv <= 64) launch_gate<16, 4, 1>(a, sc.O, tokens, s);
+  else if (a.dv <= 128) launch_gate<32, 4, 1>(a, sc.O, tokens, s);
+  else launch_gate<64, 4, 2>(a, sc.O, tokens, s);
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
@@ -715,7 +762,7 @@ Sizes scratch_sizes(int kind, int tokens, int B, int H, int dk, int dv) {
   const size_t C = docqa_linear_chunk(dk), dkp = dk_pad(dk), dvq = (dv + 15) & ~15;
   const size_t n = (tokens / C + B + 1) * H;          // chunk ids are below tokens / C + B
   const bool delta = kind == LIN_DELTA;
-  Sizes z{n * C * dkp, n * C * C, n * dkp, delta ? n * C * dkp : 0, delta ? n * C * dvq : 0, (size_t)tokens * H * dvq, 0};
+  Sizes z{n * C * dkp, n * C * C, n * dkp, delta ? n * C * dkp : 0, n * C * dvq, (size_t)tokens * H * dvq, 0};
   z.total = 2 * z.Q + z.A + z.G + z.W + z.U + z.O;
   return z;
 }
