@@ -1,7 +1,7 @@
 // moe.hip -- routed experts: E SwiGLU feed-forwards, `top` of them a token, each reading the token
 // times its score:  y_k[t] = down_e (silu(s g) * (s u)),  g = gate_e x_t, u = up_e x_t, e = ids[t, k]
 //
-// * route: scores sigmoid(x w^T) in fp32 (bf16 operands: MFMA, K split over 8 waves), the largest
+// * route: scores sigmoid(x w^T) in fp32 (bf16 operands: MFMA, K split over 16 waves), the largest
 //   `top` of the first E, and the scores of the remaining columns.
 // * a (token, choice) pair p = t top + k is a row of the grouped products; gate and up rows meet in
 //   the same lane's accumulators, so the activation is the first product's epilogue.

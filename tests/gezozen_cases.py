@@ -359,7 +359,10 @@ LINEAR_SIZES = (("channel", 70, 3, 3, 16, 24, 0, 5), ("channel", 131, 2, 2, 64, 
                 ("channel", 40, 1, 1, 200, 33, 0, 7), ("channel", 9, 2, 2, 1, 1, 0, 1), ("channel", 66, 1, 1, 7, 300, 0, 300),
                 ("fixed", 70, 3, 3, 16, 24, 12, 0), ("fixed", 140, 4, 4, 128, 64, 128, 0), ("fixed", 67, 2, 2, 9, 5, 2, 0), ("fixed", 45, 1, 1, 256, 16, 64, 0),
                 ("delta", 70, 4, 2, 16, 24, 0, 0), ("delta", 140, 3, 1, 128, 128, 0, 0), ("delta", 129, 2, 2, 48, 72, 0, 0), ("delta", 67, 3, 3, 5, 7, 0, 0),
-                ("delta", 50, 1, 1, 256, 20, 0, 0), ("delta", 20, 2, 1, 1, 1, 0, 0))
+                ("delta", 50, 1, 1, 256, 20, 0, 0), ("delta", 20, 2, 1, 1, 1, 0, 0),
+                # tall and wide states, whose step takes 16 waves or 4 lanes a row
+                ("channel", 33, 1, 1, 160, 250, 0, 20), ("channel", 70, 1, 1, 128, 508, 0, 33), ("fixed", 33, 2, 2, 130, 100, 64, 0),
+                ("delta", 66, 2, 1, 256, 256, 0, 0), ("fixed", 20, 1, 1, 64, 510, 8, 0))
 
 
 def linear_case(device, dtype, sizes=LINEAR_SIZES):
