@@ -23,7 +23,7 @@ import torch
 
 from ..ops import reference as ref
 from .bert import BertConfig, BertEncoder, BertTokenClassifier
-from . import dolodra, gezozen, saritar
+from . import dolodra, gezozen, pifazen, saritar
 from .hybrid import HybridModel
 from .llama import LlamaConfig, LlamaModel
 
@@ -160,6 +160,11 @@ def load_gezozen(path, device="cuda", dtype=torch.bfloat16) -> HybridModel:
     return _load_hybrid(gezozen, path, device, dtype)
 
 
+def load_pifazen(path, device="cuda", dtype=torch.bfloat16) -> HybridModel:
+    """Pifazen checkpoint directory (config.json + model.safetensors) -> :class:`HybridModel`."""
+    return _load_hybrid(pifazen, path, device, dtype)
+
+
 def save_saritar(cfg, weights: Mapping, path) -> None:
     """Write a Saritar checkpoint: ``weights`` by :meth:`HybridConfig.tensor_shapes` name, in bf16."""
     _save_hybrid(saritar, cfg, weights, path)
@@ -173,6 +178,11 @@ def save_dolodra(cfg, weights: Mapping, path) -> None:
 def save_gezozen(cfg, weights: Mapping, path) -> None:
     """Write a Gezozen checkpoint: ``weights`` by :meth:`HybridConfig.tensor_shapes` name, in bf16."""
     _save_hybrid(gezozen, cfg, weights, path)
+
+
+def save_pifazen(cfg, weights: Mapping, path) -> None:
+    """Write a Pifazen checkpoint: ``weights`` by :meth:`HybridConfig.tensor_shapes` name, in bf16."""
+    _save_hybrid(pifazen, cfg, weights, path)
 
 
 def _save_hybrid(design, cfg, weights: Mapping, path) -> None:
@@ -215,6 +225,10 @@ FAMILIES = (
                   (torch.bfloat16, torch.float32)),
     DecoderFamily("gezozen", lambda js: js.get("architecture") == gezozen.ARCHITECTURE,
                   lambda n: n.startswith("gezozen"), gezozen.config_from_json, gezozen.preset, load_gezozen,
+                  lambda cfg, device, dtype, seed: HybridModel(cfg, device=device, dtype=dtype, seed=seed),
+                  (torch.bfloat16, torch.float32)),
+    DecoderFamily("pifazen", lambda js: js.get("architecture") == pifazen.ARCHITECTURE,
+                  lambda n: n.startswith("pifazen"), pifazen.config_from_json, pifazen.preset, load_pifazen,
                   lambda cfg, device, dtype, seed: HybridModel(cfg, device=device, dtype=dtype, seed=seed),
                   (torch.bfloat16, torch.float32)),
     DecoderFamily("llama", lambda js: "architecture" not in js, lambda n: True, llama_config_from_hf,
@@ -364,6 +378,7 @@ def tokenizer_json(name_or_path) -> str | None:
 
 __all__ = ["LazySafetensors", "is_checkpoint", "load_llama", "save_llama", "load_saritar", "save_saritar",
            "load_dolodra", "save_dolodra", "load_gezozen", "save_gezozen",
+           "load_pifazen", "save_pifazen",
            "DecoderFamily", "FAMILIES", "decoder_family", "resolve_decoder", "resolve_decoder_config",
            "resolve_llama", "resolve_llama_config", "load_bert_encoder", "load_bert_token_classifier", "resolve_bert",
            "resolve_bert_config", "tokenizer_json", "use_checkpoint_tokenizers", "llama_config_from_hf", "bert_config_from_hf"]

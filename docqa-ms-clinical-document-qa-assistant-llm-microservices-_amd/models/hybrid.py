@@ -2,12 +2,14 @@
 mixers, with an fp32 residual stream.
 
 A model is a list of layers (:class:`LayerSpec`: a mixer and an optional feed-forward) in one
-of three forms: a norm before and after every sublayer, one after the other; with a
+of four forms: a norm before and after every sublayer, one after the other; with a
 :class:`ParallelForm` one norm whose output both sublayers read, a convolution over time
 ahead of the mixer and a second input from the token's side embedding; with a
 :class:`PostNormForm` sublayers that read the stream itself, their gated results added to it and
-the sum normed.  Layers may run
-several passes over the same weights (``loop``).  Every RUN of a layer has its own cache or
+the sum normed; with a :class:`PreNormForm` a norm before every sublayer alone, its result scaled
+per channel ahead of the sum.  Layers may run
+several passes over the same weights (``loop``), or use another layer's (``weights_of``).  Every
+RUN of a layer has its own cache or
 state, so the engine sees as many caches as runs; a latent-attention layer may read the cache
 of an earlier one (``kv_from``) instead.
 
@@ -21,10 +23,13 @@ MI355X layout:
     conv and scan over packed sequences in prefill; in decode the conv step reads the in_proj
     slabs, and dt_proj, scan step and gate are one launch; the state is in per-request slots
     (engine/kv_cache.py StatePool);
+  * the pre-norm form's stream update (slabs or the chosen experts' outputs summed and weighted,
+    bias, layer scale) and the next norm are one launch;
   * latent attention caches one row a token for all heads and attends in one of two forms:
     with the key / value projections absorbed into the query and the output (decode, short
     portions: the cached row is key and value), or with keys and values of the visible rows
-    made once by a GEMM (prompts);
+    made once by a GEMM (prompts); queries may come through a normed latent of their own, whose
+    norm and the cache row are one launch; an output gate's rows are part of the input projection;
   * a linear-attention recurrence keeps one [key, value] matrix a head in fp32: decode is one launch
     from the projection's slabs to the gated heads, prompts run in chunks on fp32 MFMA; a mixer of
     two sides has one input projection, both sides write their part of one matrix, and one product
@@ -82,8 +87,12 @@ class SelectiveScanSpec:
 class LatentAttentionSpec:
     """Causal attention over the last ``window`` tokens whose per-head keys (``dim``) and values
     (``vdim``) are linear in one normed latent of ``kv_rank`` a token, with ``rot_dim`` more
-    query / key dimensions rotated by position (key part shared by the heads) and a learned
-    sink per head.  ``kv_from``: reads the latents of that layer's cache."""
+    query / key dimensions rotated by position (key part shared by the heads) and, unless ``sink``
+    is off, a learned sink per head.  ``window`` 0: all tokens.  ``kv_from``: reads the latents of that
+    layer's cache.  ``scaling``: as in :class:`Rotation`; ``interleaved``: rotated dimensions 2i and
+    2i + 1 are a pair (else i and i + rot_dim / 2).  ``q_rank``: the queries are linear in a normed
+    latent of their own.  ``gate``: the heads' outputs are multiplied by the sigmoid of a projection
+    of the input, one number an "element" or one a "head"."""
     heads: int
     dim: int
     rot_dim: int
@@ -93,6 +102,15 @@ class LatentAttentionSpec:
     window: int
     rope_base: float
     kv_from: int | None = None
+    scaling: tuple | None = None
+    interleaved: bool = False
+    q_rank: int = 0
+    gate: str = ""
+    sink: bool = True
+
+    @property
+    def rot(self) -> Rotation:
+        return Rotation(self.rope_base, self.rot_dim, self.scaling)
 
 
 @dataclass(frozen=True)
@@ -169,6 +187,20 @@ class GatedDeltaSpec:
 
 
 @dataclass(frozen=True)
+class ChannelDeltaSpec:
+    """Gated delta rule with a decay per head and key channel; the decay's logits and the output
+    gate's (a sigmoid) are projections through ``a_rank`` and ``g_rank`` elements (0: as the
+    checkpoint's tensors have it)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    a_rank: int = 0
+    g_rank: int = 0
+
+
+@dataclass(frozen=True)
 class TwoSidedSpec:
     """left_scale attention + right_scale linear attention of the same input."""
     left: AttentionSpec
@@ -178,13 +210,34 @@ class TwoSidedSpec:
 
 
 @dataclass(frozen=True)
+class GroupRouter:
+    """Softmax scores over the experts and ``identity`` more whose output is the input itself; chosen
+    by score + a learned correction within the ``keep`` best of ``groups`` equal groups of
+    neighbours; weights are the chosen scores over their sum, times ``scale``."""
+    identity: int = 0
+    groups: int = 1
+    keep: int = 1
+    scale: float = 1.0
+
+
+@dataclass(frozen=True)
 class MoESpec:
     """``top`` of ``experts`` SwiGLU feed-forwards of ``ff`` by sigmoid score, each reading the input
-    times its score, and one of ``shared`` (0: none) for every token times a gate."""
+    times its score, and one of ``shared`` (0: none) for every token times a gate.  With a ``router``
+    the outputs are weighted instead; ``limit`` > 0: gates clamped from above and up rows on both
+    sides, g sigmoid(1.702 g) (u + 1)."""
     experts: int
     top: int
     ff: int
     shared: int = 0
+    router: GroupRouter | None = None
+    limit: float = 0.0
+
+
+@dataclass(frozen=True)
+class PreNormForm:
+    """Layers x <- x + s1 * mixer(norm1(x)), x <- x + s2 * ff(norm2(x)), s1 and s2 a number per
+    channel."""
 
 
 @dataclass(frozen=True)
@@ -207,9 +260,10 @@ class ParallelForm:
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: WindowAttentionSpec | SelectiveScanSpec | LatentAttentionSpec | TwoSidedSpec | GatedDeltaSpec
+    mixer: WindowAttentionSpec | SelectiveScanSpec | LatentAttentionSpec | TwoSidedSpec | GatedDeltaSpec | ChannelDeltaSpec
     ff: int = 0                     # feed-forward width, 0: none
-    moe: MoESpec | None = None      # or experts (post-norm form)
+    moe: MoESpec | None = None      # or experts (pre- and post-norm forms)
+    weights_of: int | None = None   # the layer whose weights this one uses (pre-norm form)
 
 
 @dataclass
@@ -223,6 +277,8 @@ class HybridConfig:
     loop: tuple | None = None       # (start, stop, times)
     parallel: ParallelForm | None = None    # neither: norms around every sublayer
     post: PostNormForm | None = None
+    pre: PreNormForm | None = None
+    tied: bool = False              # the LM head is the embedding table
     act: str = ops.ACT_RELU2        # of the feed-forward
     norm_offset: float = 0.0        # added to the stored weights of the layers' and final norms
     logit_softcap: float | None = None
@@ -249,23 +305,35 @@ class HybridConfig:
         if self.post is not None:
             if self.loop is not None or self.parallel is not None or self.hidden % self.post.groups:
                 raise ValueError("post-norm layers: groups that divide the width, no loop")
+        if self.pre is not None and (self.loop is not None or self.parallel is not None or self.post is not None):
+            raise ValueError("pre-norm layers: no loop, no other form")
+        if self.pre is not None and self.act != ops.ACT_POLY_NORM and any(sp.ff for sp in self.layer_specs):
+            raise ValueError("pre-norm layers: dense feed-forwards with PolyNorm")
         for i, sp in enumerate(self.layer_specs):
             m = sp.mixer
-            if (self.post is not None) != isinstance(m, (TwoSidedSpec, GatedDeltaSpec)) or (sp.moe and self.post is None) or (
-                    sp.ff and self.post is not None):
-                raise ValueError("two-sided and delta mixers and experts run in post-norm layers")
+            if (self.post is not None) != isinstance(m, (TwoSidedSpec, GatedDeltaSpec)) or (
+                    sp.moe and self.post is None and self.pre is None) or (sp.ff and self.post is not None):
+                raise ValueError("two-sided and delta mixers run in post-norm layers, experts in these or pre-norm ones")
             if self.post is not None:
                 _check_post(sp)
+            if (self.pre is not None) != isinstance(m, ChannelDeltaSpec) and not (
+                    self.pre is not None and isinstance(m, LatentAttentionSpec)):
+                raise ValueError("pre-norm layers: latent attention and channel-delta mixers")
+            if self.pre is not None:
+                _check_pre(sp, i, self.layer_specs)
             if isinstance(m, LatentAttentionSpec):
-                if m.rot_dim % 2 or m.window < 1 or max(m.kv_rank, m.dim) > 2048 or min(m.heads, m.dim, m.vdim, m.kv_rank, m.rot_dim) < 1:
+                if m.rot_dim % 2 or m.window < (0 if self.pre is not None else 1) or max(m.kv_rank, m.dim) > 2048 or min(
+                        m.heads, m.dim, m.vdim, m.kv_rank, m.rot_dim) < 1:
                     raise ValueError(f"unsupported attention sizes {m}")
+                if self.pre is None and (m.q_rank or m.gate or not m.sink):
+                    raise ValueError("query latents and output gates run in pre-norm layers")
                 if m.kv_from is not None:
                     src = self.layer_specs[m.kv_from].mixer if 0 <= m.kv_from < i else None
                     if not isinstance(src, LatentAttentionSpec) or src.kv_from is not None or (
                             (src.kv_rank, src.rot_dim, src.rope_base) != (m.kv_rank, m.rot_dim, m.rope_base)):
                         raise ValueError(f"layer {i}: kv_from {m.kv_from} is no earlier layer with such latents of its own")
-                elif self.parallel is None:
-                    raise ValueError("latent attention runs in parallel layers")
+                elif self.parallel is None and self.pre is None:
+                    raise ValueError("latent attention runs in parallel and pre-norm layers")
             if isinstance(m, WindowAttentionSpec) and (m.heads % m.kv_heads or m.window < 1 or m.dim > 512):
                 raise ValueError(f"unsupported attention sizes {m}")
             if isinstance(m, SelectiveScanSpec) and (m.state > 256 or m.conv < 1):
@@ -283,6 +351,14 @@ class HybridConfig:
             for i, sp in enumerate(self.layer_specs):
                 out.update(_post_shapes(sp, W, f"l{i}."))
             out.update({"final.norm": (W,), "head": (V, W)})
+            return out
+        if self.pre is not None:
+            for i, sp in enumerate(self.layer_specs):
+                if sp.weights_of is None:
+                    out.update(_pre_shapes(sp, W, f"l{i}."))
+            out["final.norm"] = (W,)
+            if not self.tied:
+                out["head"] = (V, W)
             return out
         if par is not None:
             out["side.embed"] = (V, self.layers * par.side)
@@ -321,6 +397,35 @@ class HybridConfig:
         return sum(math.prod(s) for s in self.tensor_shapes().values())
 
 
+def _check_state(s) -> None:
+    if min(s.heads, s.dim, s.vdim) < 1 or s.heads % getattr(s, "kv_heads", 1):
+        raise ValueError(f"unsupported sizes {s}")
+    if s.dim > 256 or s.vdim > (512 if s.dim <= 128 else 256):
+        raise ValueError(f"unsupported state sizes {s}")
+    if getattr(s, "conv", 1) < 1:
+        raise ValueError(f"unsupported sizes {s}")
+
+
+def _check_pre(sp: LayerSpec, i: int, specs: list) -> None:
+    m, f = sp.mixer, sp.moe
+    if isinstance(m, ChannelDeltaSpec):
+        _check_state(m)
+    elif m.kv_from is not None or m.sink or m.gate not in ("", "head", "element") or not 0 <= m.q_rank <= 2048:
+        raise ValueError(f"unsupported attention {m}")
+    if f is not None:
+        r = f.router
+        if sp.ff or r is None or f.shared or f.limit <= 0:
+            raise ValueError(f"pre-norm layers take clamped experts behind a group router, not {f}")
+        n = f.experts + r.identity
+        if not (1 <= f.experts and r.identity >= 0 and n <= 512 and f.ff >= 1 and 1 <= r.keep <= r.groups and n % r.groups == 0
+                and 1 <= f.top <= min(16, r.keep * (n // r.groups))):
+            raise ValueError(f"unsupported experts {f}")
+    if sp.weights_of is not None:
+        j = sp.weights_of
+        if not 0 <= j < len(specs) or specs[j].weights_of is not None or replace(specs[j], weights_of=j) != sp:
+            raise ValueError(f"layer {i}: weights_of {j} is no layer of the same kind with weights of its own")
+
+
 def _check_post(sp: LayerSpec) -> None:
     m = sp.mixer
     sides = [m.left, m.right] if isinstance(m, TwoSidedSpec) else [m]
@@ -333,16 +438,14 @@ def _check_post(sp: LayerSpec) -> None:
         if isinstance(s, AttentionSpec):
             if s.dim > 512 or s.vdim > 512 or s.window < 0 or s.softcap < 0:
                 raise ValueError(f"unsupported attention sizes {s}")
-        elif s.dim > 256 or s.vdim > (512 if s.dim <= 128 else 256):
-            raise ValueError(f"unsupported state sizes {s}")
+        else:
+            _check_state(s)
         if isinstance(s, RetentionSpec) and (len(s.decay) != s.heads or not all(0 < d <= 1 for d in s.decay)):
             raise ValueError(f"one decay in (0, 1] per head expected: {s.decay}")
-        if isinstance(s, GatedDeltaSpec) and s.conv < 1:
-            raise ValueError(f"unsupported sizes {s}")
         if isinstance(s, GatedLinearSpec) and s.tau <= 0:
             raise ValueError(f"unsupported sizes {s}")
     if sp.moe is not None and not (1 <= sp.moe.top <= min(sp.moe.experts, 16) and sp.moe.ff >= 1 and sp.moe.shared >= 0
-                                   and sp.moe.experts <= 512):
+                                   and sp.moe.experts <= 512 and sp.moe.router is None and sp.moe.limit == 0):
         raise ValueError(f"unsupported experts {sp.moe}")
 
 
@@ -384,6 +487,35 @@ def _post_shapes(sp: LayerSpec, W: int, p: str) -> dict:
     return out
 
 
+def _pre_shapes(sp: LayerSpec, W: int, p: str) -> dict:
+    x, m, f = p + "mix.", sp.mixer, sp.moe
+    out = {p + "norm1": (W,), p + "ls1": (W,), x + "o": (W, m.heads * m.vdim)}
+    if isinstance(m, ChannelDeltaSpec):
+        key, val, a, g = m.kv_heads * m.dim, m.heads * m.vdim, m.a_rank, m.g_rank
+        out.update({x + "q": (key, W), x + "q.conv": (key, m.conv), x + "k": (key, W), x + "k.conv": (key, m.conv),
+                    x + "v": (val, W), x + "v.conv": (val, m.conv), x + "b": (m.heads, W), x + "A_log": (m.heads,),
+                    x + "norm": (m.vdim,), x + "a1": (a, W), x + "a2": (m.heads * m.dim, a), x + "dt_bias": (m.heads * m.dim,),
+                    x + "g1": (g, W), x + "g2": (val, g)})
+    else:
+        q = m.heads * (m.dim + m.rot_dim)
+        out.update({x + "dq": (m.q_rank, W), x + "dq.norm": (m.q_rank,), x + "uq": (q, m.q_rank)} if m.q_rank else {x + "q": (q, W)})
+        out.update({x + "dkv": (m.kv_rank + m.rot_dim, W), x + "dkv.norm": (m.kv_rank,), x + "uk": (m.heads * m.dim, m.kv_rank),
+                    x + "uv": (m.heads * m.vdim, m.kv_rank)})
+        if m.gate:
+            out[x + "g"] = (m.heads * (m.vdim if m.gate == "element" else 1), W)
+    if sp.ff or f is not None:
+        out.update({p + "norm2": (W,), p + "ls2": (W,)})
+    x = p + "mlp."
+    if sp.ff:
+        out.update({x + "up": (sp.ff, W), x + "up.b": (sp.ff,), x + "down": (W, sp.ff), x + "down.b": (W,), x + "act": (4,)})
+    elif f is not None:
+        n = f.experts + f.router.identity
+        out.update({x + "router": (n, W), x + "correction": (n,)})
+        for e in range(f.experts):
+            out.update({f"{x}e{e}.gate": (f.ff, W), f"{x}e{e}.up": (f.ff, W), f"{x}e{e}.down": (W, f.ff)})
+    return out
+
+
 # Feed-forward weights from which a captured decode step runs a parallel layer's sublayers as two
 # branches of the graph: 352 MB (width 4096, ff 21504) 1.07 -> 0.98 ms a step of 8 layers at batch 1,
 # 1.92 -> 1.69 at 64, 2.52 -> 2.47 at 256; 100 MB lose 6 % at batch 1 to 16
@@ -408,11 +540,11 @@ class _Part:
 
 
 class _Keys:
-    """The visible keys of a prompt batch under one window: every sequence's [first, end) rows,
+    """The visible keys of a prompt batch under one window (0: all): every sequence's [first, end) rows,
     packed (``cu``), and how many there are."""
 
     def __init__(self, spans: list, window: int, device):
-        lo = [max(0, a - window + 1) for a, _ in spans]
+        lo = [max(0, a - window + 1) if window else 0 for a, _ in spans]
         cu = [0]
         for k, (_, e) in zip(lo, spans):
             cu.append(cu[-1] + e - k)
@@ -422,7 +554,7 @@ class _Keys:
         self.tokens = sum(e - a for a, e in spans)
 
         def seen(n):           # (query, key) pairs of positions below n
-            k = min(n, window)
+            k = min(n, window) if window else n
             return k * (k + 1) // 2 + (n - k) * window
 
         self.pairs = sum(seen(e) - seen(a) for a, e in spans)
@@ -430,7 +562,7 @@ class _Keys:
 
 @dataclass
 class _Forward:
-    """What the layers of one forward share: rotation tables by (base, dims), the visible keys of
+    """What the layers of one forward share: tables by :class:`Rotation`, the visible keys of
     prompts by window."""
     rope: dict
     keys: dict
@@ -540,10 +672,28 @@ class LatentAttention:
         self.sp, self.eps, self.dtype = sp, eps, dtype
         H, d, vd, R = sp.heads, sp.dim, sp.vdim, sp.kv_rank
         self.d8, self.r8, self.R8, self.v8 = (_pad_up(n, 8) for n in (d, sp.rot_dim, R, vd))
-        rows = [get("q")] + ([get("dkv")] if sp.kv_from is None else [])
-        n = sum(t.shape[0] for t in rows)
-        rows.append(rows[0].new_zeros(_pad_up(n, 256 if n >= 1024 else 64) - n, rows[0].shape[1]))
-        self.w_in = torch.cat(rows).to(dtype).contiguous()          # q | latent | key part
+        self.rot = sp.rot
+        # the kernels pair rotated dimension i with i + rot_dim / 2: neighbours become that by the order
+        # of the projections' rows, the same one for queries and keys
+        order = torch.arange(sp.rot_dim)
+        if sp.interleaved:
+            order = torch.cat([order[0::2], order[1::2]])
+
+        def paired(t, keep):           # rows [.., keep | rotated]
+            t = t.view(-1, keep + sp.rot_dim, t.shape[-1])
+            return torch.cat([t[:, :keep], t[:, keep:][:, order.to(t.device)]], 1).flatten(0, 1)
+
+        # q (or its latent) | latent | key part | gate
+        rows = [get("dq") if sp.q_rank else paired(get("q"), d)] + ([paired(get("dkv"), R)] if sp.kv_from is None else [])
+        self.q_norm = self.w_uq = self.gate_at = None
+        if sp.q_rank:
+            self.q_norm = get("dq.norm").float().contiguous()
+            self.w_uq = _joint([paired(get("uq"), d)], dtype)
+        if sp.gate:
+            n = sum(t.shape[0] for t in rows)
+            self.gate_at = _pad_up(n, 8)
+            rows += [rows[0].new_zeros(self.gate_at - n, rows[0].shape[1]), get("g")]
+        self.w_in = _joint(rows, dtype)
         self.c_norm = get("dkv.norm").float().contiguous() if sp.kv_from is None else None
         uk, uv = get("uk").view(H, d, R), get("uv").view(H, vd, R)
         pad = torch.nn.functional.pad
@@ -557,9 +707,8 @@ class LatentAttention:
                             pad(uv, (0, self.R8 - R, 0, self.v8 - vd)).reshape(H * self.v8, self.R8)])
             n = kv.shape[0]
             self.w_kv = pad(kv, (0, 0, 0, _pad_up(n, 256 if n >= 1024 else 64) - n)).to(dtype).contiguous()
-        self.sink = get("sink").float().contiguous()
+        self.sink = get("sink").float().contiguous() if sp.sink else None
         self.o = get("o").to(dtype).contiguous()
-        self.rope_key = (sp.rope_base, sp.rot_dim)
 
     def cache_spec(self):
         """Its own rows, or (``kv_from``) the index of the run whose rows it reads."""
@@ -567,7 +716,8 @@ class LatentAttention:
 
     def activation_elems(self) -> int:
         H = self.sp.heads
-        return self.w_in.shape[0] + H * (self.d8 + self.r8 + self.sp.vdim) + 2 * H * (self.d8 + self.v8)
+        return (self.w_in.shape[0] + H * (self.d8 + self.r8 + self.sp.vdim) + 2 * H * (self.d8 + self.v8)
+                + (self.w_uq.shape[0] + self.sp.q_rank if self.sp.q_rank else 0))
 
     def _expanded(self, keys: _Keys | None) -> bool:
         """Whether making keys and values of the visible rows costs less than attending in the
@@ -579,9 +729,13 @@ class LatentAttention:
                 < keys.tokens * self.R8 * kv + keys.pairs * (2 * self.R8 + self.r8))
 
     def run(self, x, parts, slot_mapping, cache, decode, fw: _Forward):
-        sp = self.sp
-        q = ops.latent_store(ops.project(x, self.w_in, decode), fw.rope[self.rope_key], slot_mapping, cache, self.c_norm,
-                             sp.heads, sp.dim, sp.kv_rank, self.eps, self.dtype)
+        sp, cs = self.sp, fw.rope[self.rot]
+        P = Q = ops.project(x, self.w_in, decode)
+        c_norm = self.c_norm
+        if sp.q_rank:
+            cq = ops.latent_norm_store(P, cs, slot_mapping, cache, self.q_norm, c_norm, self.eps, self.dtype)
+            Q, c_norm = ops.project(cq, self.w_uq, decode), None
+        q = ops.latent_store(Q, cs, slot_mapping, cache, c_norm, sp.heads, sp.dim, sp.kv_rank, self.eps, self.dtype)
         out = []
         for p in parts:
             m, qp = p.meta, _split(q, p, parts)
@@ -599,7 +753,10 @@ class LatentAttention:
                 a = ops.latent_attn(qc, cache, m.block_tables, m.prefix_lens, sp.scale, self.w_cv, cu=m.cu_seqlens,
                                     max_q=m.max_len, **kw)
             out.append(a)
-        return ops.project(_join(out), self.o, decode)
+        o = _join(out)
+        if sp.gate:
+            o = ops.head_gate(o, P, self.gate_at, sp.vdim if sp.gate == "head" else 1)
+        return ops.project(o, self.o, decode)
 
 
 class MLP:
@@ -613,6 +770,26 @@ class MLP:
 
     def run(self, x, decode):
         return ops.project(ops.act_linear(x, self.up, self.act, decode), self.down, decode)
+
+
+class PolyNormMLP:
+    """down(act(up x + b)) with act the four-term PolyNorm; its own bias goes to the stream update."""
+
+    def __init__(self, get, dtype, eps: float):
+        up, down = get("up"), get("down")
+        self.n, self.eps, self.dtype = up.shape[0], eps, dtype
+        pad = _pad_up(self.n, 64) - self.n
+        self.up = _joint([up], dtype)
+        self.up_b, self.act = get("up.b").float().contiguous(), get("act").float().contiguous()
+        self.down = torch.nn.functional.pad(down, (0, pad)).to(dtype).contiguous()
+        self.down_b = get("down.b").float().contiguous()
+
+    def activation_elems(self) -> int:
+        return self.up.shape[0] + self.down.shape[1]
+
+    def run(self, x, decode):
+        a = ops.poly_norm(ops.project(x, self.up, decode), self.up_b, self.act, self.down.shape[1], self.eps, self.dtype)
+        return ops.project(a, self.down, decode), {"bias": self.down_b}
 
 
 def _joint(rows: list, dtype) -> torch.Tensor:
@@ -669,6 +846,11 @@ class LinearAttention:
             names.append("a1")
             self.w_gate, self.b_gate = get("a2").float().contiguous(), get("a2.b").float().contiguous()
             kw = dict(q_scale=sp.dim ** -0.5, inv_tau=1.0 / sp.tau, rank=self.w_gate.shape[1])
+        elif isinstance(sp, ChannelDeltaSpec):
+            # decays, gates and steps come as one matrix of their own (ops.low_rank)
+            kind, norm, names = "channel_delta", get("norm").float(), ["q", "k", "v"]
+            self.w_gate, self.b_gate = (-torch.exp(get("A_log").float())).contiguous(), get("dt_bias").float().contiguous()
+            kw = dict(q_scale=sp.dim ** -0.5, gate="sigmoid")
         elif isinstance(sp, RetentionSpec):
             kind, self.rot = "fixed", sp.rot
             self.w_gate = torch.tensor(sp.decay, dtype=torch.float64).log().float().to(norm.device)
@@ -684,7 +866,10 @@ class LinearAttention:
         for t in self.rows:
             cols.append(cols[-1] + t.shape[0])
         self.n = cols[-1] - at
-        self.mix = ops.LinearMix(kind, sp.heads, kv, sp.dim, sp.vdim, *cols[:4], a=cols[4], b=cols[5] if kind == "delta" else 0,
+        if kind == "channel_delta":
+            n = sp.heads * sp.dim
+            cols = cols[:3] + [n, 0, n + sp.heads * sp.vdim]
+        self.mix = ops.LinearMix(kind, sp.heads, kv, sp.dim, sp.vdim, *cols[:4], a=cols[4], b=cols[5] if kind.endswith("delta") else 0,
                                  eps=eps, **kw)
         self.o = get("o")
 
@@ -783,6 +968,76 @@ class DeltaMixer:
         return ops.project(out, self.o, decode), P, self.tail
 
 
+class ChannelDelta:
+    """Gated delta rule with channel decays behind short convolutions of q, k and v.  One projection
+    [q k v | decay's and gate's inner elements | steps]; a second product makes decays and gates of theirs."""
+
+    def __init__(self, sp: ChannelDeltaSpec, get, eps: float, dtype):
+        self.sp = sp
+        pad = torch.nn.functional.pad
+        self.lin = LinearAttention(sp, get, eps, dtype)
+        self.conv_w = torch.cat([get(n + ".conv") for n in "qkv"]).float().t().contiguous()      # [taps, C]
+        self.C = self.conv_w.shape[1]
+        inner = [pad(t, (0, 0, 0, _pad_up(t.shape[0], 8) - t.shape[0])) for t in (get("a1"), get("g1"))]
+        self.ranks = tuple(t.shape[0] for t in inner)
+        self.rest = sum(self.ranks) + sp.heads
+        self.w_a, self.w_g = (pad(t, (0, k - t.shape[1])).to(dtype).contiguous() for t, k in zip((get("a2"), get("g2")), self.ranks))
+        self.w_in = _joint([*self.lin.rows, *inner, get("b")], dtype)
+        self.o = self.lin.o.to(dtype).contiguous()
+        self.lin.rows = self.lin.o = None
+
+    def cache_spec(self):
+        return StateSpec(((self.sp.conv - 1, self.C), self.lin.state_shape()), (False, True))
+
+    def activation_elems(self) -> int:
+        sp = self.sp
+        return self.w_in.shape[0] + self.C + self.o.shape[1] + 2 * sp.heads * (6 * sp.dim + 5 * sp.vdim + 64)
+
+    def run(self, x, parts, slot_mapping, cache, decode, fw: _Forward):
+        conv_state, state = cache
+        one = decode and len(parts) == 1
+        P = ops.project(x, self.w_in, True) if one else ops.linear(x, self.w_in, decode)
+        out = x.new_empty(x.shape[0], self.o.shape[1])
+        for p in parts:
+            m, r = p.meta, _split(P, p, parts)
+            if p.decode:
+                y, z = ops.conv_step(r, self.conv_w, None, conv_state, m.state_slots, m.positions, rest=self.rest)
+                at = 0
+            else:
+                y, z = ops.causal_conv(r, self.conv_w, None, conv_state, m.state_slots, m.cu_seqlens, m.prefix_lens, m.max_len), r
+                at = self.C
+            self.lin.run_part(y, ops.low_rank(z, at, self.w_a, self.w_g, self.sp.heads), self.lin.mix, p, state, None,
+                              _split(out, p, parts))
+        return ops.project(out, self.o, decode)
+
+
+def _expert_weights(sp: MoESpec, get, dtype) -> tuple:
+    """([E, 2 (gate, up), F, W], [E, W, F]), F padded with zeros to 64."""
+    pad = torch.nn.functional.pad
+    F = _pad_up(sp.ff, 64)
+    up = torch.stack([torch.stack([pad(get(f"e{e}.{n}").to(dtype), (0, 0, 0, F - sp.ff)) for n in ("gate", "up")])
+                      for e in range(sp.experts)])
+    return up, torch.stack([pad(get(f"e{e}.down").to(dtype), (0, F - sp.ff)) for e in range(sp.experts)])
+
+
+class GroupExperts:
+    """Experts behind a group router, identity experts among them; the stream update weighs and sums
+    the chosen ones' outputs."""
+
+    def __init__(self, sp: MoESpec, get, dtype):
+        self.sp = sp
+        self.up, self.down = _expert_weights(sp, get, dtype)
+        self.router, self.correction = get("router").to(dtype).contiguous(), get("correction").float().contiguous()
+
+    def activation_elems(self) -> int:
+        return self.sp.top * (self.up.shape[2] + self.up.shape[3])
+
+    def run(self, x, decode):
+        sp, r = self.sp, self.sp.router
+        ids, wts = ops.moe_route_groups(x, self.router, self.correction, sp.top, r.groups, r.keep, r.scale)
+        return ops.moe_experts(x, ids, wts, self.up, self.down, sp.limit), {"mix": (ids, wts, sp.experts, x)}
+
+
 class Experts:
     """Routed experts and a shared one.  The shared expert's gate and up rows and the ``tail`` rows
     are one projection; routing is fp32."""
@@ -790,10 +1045,7 @@ class Experts:
     def __init__(self, sp: MoESpec, get, dtype, tail):
         self.sp, self.dtype = sp, dtype
         pad = torch.nn.functional.pad
-        F = _pad_up(sp.ff, 64)
-        self.up = torch.stack([torch.stack([pad(get(f"e{e}.{n}").to(dtype), (0, 0, 0, F - sp.ff)) for n in ("gate", "up")])
-                               for e in range(sp.experts)])                                     # [E, 2, F, W]
-        self.down = torch.stack([pad(get(f"e{e}.down").to(dtype), (0, F - sp.ff)) for e in range(sp.experts)])
+        self.up, self.down = _expert_weights(sp, get, dtype)
         router, rows = [get("router")], [tail]
         self.shared = None
         if sp.shared:
@@ -892,9 +1144,24 @@ class HybridModel(Decoder):
 
         par = cfg.parallel
         self.embed = get("embed").to(dt).contiguous()
-        self.lm_head = get("head").to(dt).contiguous()
+        self.lm_head = self.embed if cfg.tied else get("head").to(dt).contiguous()
         self.final_norm = norm("final.norm")
-        self.layers, self.rope_freq = [], {}
+        self.layers, self.rope_freq, self.windows = [], {}, []
+        if cfg.pre is not None:
+            own = {}
+            for i, sp in enumerate(cfg.layer_specs):
+                if sp.weights_of is not None:
+                    continue
+                p = f"l{i}."
+                L = own[i] = {"mixer": _MIXERS[type(sp.mixer)](sp.mixer, lambda n: get(p + "mix." + n), cfg.rms_eps, dt),
+                              "norm1": norm(p + "norm1"), "ls1": vec(p + "ls1"), "mlp": None}
+                if sp.ff or sp.moe is not None:
+                    tensor = lambda n: get(p + "mlp." + n)  # noqa: E731
+                    L.update(mlp=PolyNormMLP(tensor, dt, cfg.rms_eps) if sp.ff else GroupExperts(sp.moe, tensor, dt),
+                             norm2=norm(p + "norm2"), ls2=vec(p + "ls2"))
+            self.layers = [own[i if sp.weights_of is None else sp.weights_of] for i, sp in enumerate(cfg.layer_specs)]
+            self._load_rotations()
+            return
         if cfg.post is not None:
             for i, sp in enumerate(cfg.layer_specs):
                 p = f"l{i}."
@@ -924,11 +1191,15 @@ class HybridModel(Decoder):
             self.layers.append(L)
         if par is not None:
             self.side_embed = get("side.embed").to(dt).contiguous()
-            self.rope_freq = {(b, r): b ** (-torch.arange(0, r, 2, dtype=torch.float64) / r) for b, r in
-                              {L["mixer"].rope_key for L in self.layers}}
-            self.rope_freq = {k: v.to(self.device) for k, v in self.rope_freq.items()}
-            self.windows = sorted({s.mixer.window for s, L in zip(cfg.layer_specs, self.layers)
-                                   if L["mixer"].w_kv is not None})
+            self._load_rotations()
+
+    def _load_rotations(self) -> None:
+        """Of the latent-attention layers: the rotations, and the windows whose keys prompts expand."""
+        latent = [L["mixer"] for L in self.layers if isinstance(L["mixer"], LatentAttention)]
+        for rot in {m.rot for m in latent}:
+            f, mult = rot.frequencies()
+            self.rope_freq[rot] = (f.to(self.device), mult)
+        self.windows = sorted({m.sp.window for m in latent if m.w_kv is not None})
 
     # ------------------------------------------------------------------ caches
     def _run_specs(self) -> list:
@@ -946,7 +1217,7 @@ class HybridModel(Decoder):
         return [s for run in self._run_specs() for s in run if isinstance(s, StateSpec)]
 
     def bind_caches(self, kv, state) -> list:
-        """Per run its mixer's tensors; in the parallel form (latent rows, convolution inputs), in the
+        """Per run its mixer's tensors (the pre-norm form's latent rows as one); in the parallel form (latent rows, convolution inputs), in the
         post-norm form a tuple of tensors for each of its mixer's specs."""
         k, s = iter(kv.caches), iter(state.states if state is not None else [])
         out = []
@@ -955,11 +1226,14 @@ class HybridModel(Decoder):
             if self.cfg.post is not None:
                 out.append(own)
                 continue
+            if self.cfg.pre is not None:
+                out.append(own[0][0] if isinstance(run[0], KVSpec) else own[0])
+                continue
             out.append(own[0] if len(own) == 1 else (own[0][0], own[1][0]))
         return out
 
     def activation_elems(self) -> int:
-        if self.cfg.post is not None:
+        if self.cfg.post is not None or self.cfg.pre is not None:
             return 10 * self.cfg.hidden + max([max(L["mixer"].activation_elems(), L["mlp"].activation_elems() if L["mlp"] else 0)
                                                for L in self.layers] + [0])
         ff = max([s.ff for s in self.cfg.layer_specs] + [0])
@@ -989,6 +1263,8 @@ class HybridModel(Decoder):
             return self._hidden_parallel(input_ids, parts, slot_mapping, caches)
         if self.cfg.post is not None:
             return self._hidden_post(input_ids, parts, slot_mapping, caches)
+        if self.cfg.pre is not None:
+            return self._hidden_pre(input_ids, parts, slot_mapping, caches)
         cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
         decode = all(p.decode for p in parts)
         runs = cfg.runs
@@ -1010,15 +1286,34 @@ class HybridModel(Decoder):
                 self.tap.append(res - add if add is not None else res.clone())
         return x
 
-    def _hidden_parallel(self, input_ids, parts, slot_mapping, caches):
-        cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
-        decode = all(p.decode for p in parts)
-        fw = _Forward({}, {})
+    def _shared(self, parts) -> _Forward:
+        pos = _join([p.meta.positions for p in parts])
+        fw = _Forward({r: ops.rope_table(pos, f, mult) for r, (f, mult) in self.rope_freq.items()}, {})
         for p in parts:
             if not p.decode and p.meta.spans is not None:
                 fw.keys = {w: _Keys(p.meta.spans, w, self.device) for w in self.windows}
-        pos = _join([p.meta.positions for p in parts])
-        fw.rope = {k: ops.rope_table(pos, f) for k, f in self.rope_freq.items()}
+        return fw
+
+    def _hidden_pre(self, input_ids, parts, slot_mapping, caches):
+        cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
+        decode = all(p.decode for p in parts)
+        fw = self._shared(parts)
+        norms = [L["norm1"] for L in self.layers] + [self.final_norm]
+        res, _, x = ops.embed_scale_rmsnorm(input_ids, self.embed, cfg.embed_scale, norms[0], eps)
+        for L, cache, nxt in zip(self.layers, caches, norms[1:]):
+            y = L["mixer"].run(x, parts, slot_mapping, cache, decode, fw)
+            x = ops.scaled_rmsnorm(y, res, L["ls1"], nxt if L["mlp"] is None else L["norm2"], eps, out_dtype=dt)
+            if L["mlp"] is not None:
+                y, kw = L["mlp"].run(x, decode)
+                x = ops.scaled_rmsnorm(y, res, L["ls2"], nxt, eps, out_dtype=dt, **kw)
+            if self.tap is not None:
+                self.tap.append(res.clone())
+        return x
+
+    def _hidden_parallel(self, input_ids, parts, slot_mapping, caches):
+        cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
+        decode = all(p.decode for p in parts)
+        fw = self._shared(parts)
         first = self.layers[0]["norm1"] if self.layers else self.final_norm
         res, _, h = ops.embed_scale_rmsnorm(input_ids, self.embed, cfg.embed_scale, first, eps)
         hm = self.layers[0]["conv"].run(h, parts, caches[0][1]) if self.layers else h
@@ -1045,8 +1340,7 @@ class HybridModel(Decoder):
         cfg, eps, dt = self.cfg, self.cfg.rms_eps, self.dtype
         alpha, groups = cfg.post.alpha, cfg.post.groups
         decode = all(p.decode for p in parts)
-        pos = _join([p.meta.positions for p in parts])
-        fw = _Forward({r: ops.rope_table(pos, f, mult) for r, (f, mult) in self.rope_freq.items()}, {})
+        fw = self._shared(parts)
         res, _, x = ops.embed_scale_rmsnorm(input_ids, self.embed, cfg.embed_scale, None, eps)
         for L, cache in zip(self.layers, caches):
             y, P, col = L["mixer"].run(x, parts, slot_mapping, cache, decode, fw)
@@ -1089,7 +1383,7 @@ class HybridModel(Decoder):
 
 
 _MIXERS = {WindowAttentionSpec: WindowAttention, SelectiveScanSpec: SelectiveScan, LatentAttentionSpec: LatentAttention,
-           TwoSidedSpec: TwoSidedMixer, GatedDeltaSpec: DeltaMixer}
+           TwoSidedSpec: TwoSidedMixer, GatedDeltaSpec: DeltaMixer, ChannelDeltaSpec: ChannelDelta}
 
 
 class _RandomWeights:
@@ -1105,8 +1399,12 @@ class _RandomWeights:
         g.manual_seed((self.seed * 1_000_003 + zlib.crc32(name.encode())) & 0x7FFFFFFFFFFF)
         kind = name.rsplit(".", 1)[-1]
         if name.endswith("norm") or kind.startswith("norm"):
-            stored_off = self.offset if kind.startswith("norm1") or name == "final.norm" else 0.0
+            stored_off = self.offset if kind.startswith(("norm1", "norm2")) or name == "final.norm" else 0.0
             return torch.full(shape, 1.0 - stored_off, device=self.device)
+        if kind in ("ls1", "ls2", "act"):
+            return torch.full(shape, 1.0 if kind != "act" else 1 / 3, device=self.device)
+        if kind == "correction":
+            return torch.zeros(shape, device=self.device)
         if kind == "A_log" and len(shape) == 1:
             return torch.empty(shape, device=self.device).uniform_(1.0, 16.0, generator=g).log()
         if kind == "A_log":

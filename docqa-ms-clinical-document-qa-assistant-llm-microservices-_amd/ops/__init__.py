@@ -1212,7 +1212,19 @@ def sandwich_rmsnorm(P, residual, w_post, w_next, eps: float, add=None, out_dtyp
     return ref.sandwich_rmsnorm(P, residual, w_post, w_next, eps, add, out_dtype)
 
 
-ACT_RELU2, ACT_GELU_TANH = "relu2", "gelu_tanh"
+def scaled_rmsnorm(P, residual, scale, w_next, eps: float, bias=None, mix=None, out_dtype=torch.bfloat16):
+    """residual (fp32, in place) += scale (P + ``bias``), per channel; returns rmsnorm(residual) * w_next
+    in ``out_dtype``.  ``mix`` (ids [T, top], weights [T, top], experts, x): P holds the chosen experts'
+    outputs [top, T, W] of :func:`moe_experts` on x, summed by weight; ids from ``experts`` on stand for x
+    itself, and their part of P is not read."""
+    if _gpu(P):
+        ids, wts, experts, x = mix or (None, None, 0, None)
+        return _native().scaled_rmsnorm(P.contiguous(), residual, scale, bias, ids, wts, int(experts), x, w_next, float(eps),
+                                        out_dtype == torch.float32)
+    return ref.scaled_rmsnorm(P, residual, scale, w_next, eps, bias, mix, out_dtype)
+
+
+ACT_RELU2, ACT_GELU_TANH, ACT_POLY_NORM = "relu2", "gelu_tanh", "poly_norm"
 _ACT_CODE = {ACT_RELU2: 0, ACT_GELU_TANH: 1}
 
 
@@ -1221,6 +1233,14 @@ def activation(P, act: str, out_dtype=torch.bfloat16):
     if _gpu(P):
         return _native().slab_activation(P.contiguous(), _ACT_CODE[act], out_dtype == torch.float32)
     return ref.activation(P, act, out_dtype)
+
+
+def poly_norm(P, bias, act, n_out: int, eps: float, out_dtype=torch.bfloat16):
+    """PolyNorm of z = P + ``bias`` (its length n the row's): a N(z) + b N(z^2) + c N(z^3) + e, N over the
+    row's root mean square, (a, b, c, e) = ``act``; [T, n_out], zero past n."""
+    if _gpu(P):
+        return _native().poly_norm(P.contiguous(), bias, act, int(n_out), float(eps), out_dtype == torch.float32)
+    return ref.poly_norm(P, bias, act, n_out, eps, out_dtype)
 
 
 def sandwich_rmsnorm_conv(P, residual, w_post, w_next, eps: float, conv_w, state, slots, positions):
@@ -1383,6 +1403,23 @@ def latent_store(P, cs, slots, cache, c_norm, H: int, dim: int, rank: int, eps: 
     return ref.latent_store(P, cs, slots, cache, c_norm, H, dim, rank, eps, dtype)
 
 
+def latent_norm_store(P, cs, slots, cache, q_norm, c_norm, eps: float, dtype):
+    """Of a projection [query latent | latent | key part: r | ..]: the normed query latent times
+    ``q_norm`` (its length the latent's), for a projection to query heads (:func:`latent_store` with
+    ``c_norm`` None); the cache row as in :func:`latent_store`."""
+    if _gpu(P):
+        return _native().latent_norm_store(P.contiguous(), cs, slots, cache, q_norm, c_norm, float(eps))
+    return ref.latent_norm_store(P, cs, slots, cache, q_norm, c_norm, eps, dtype)
+
+
+def head_gate(x, P, col: int, per: int):
+    """x [T, n] times sigmoid of columns [col, col + n / per) of a projection, ``per`` neighbours each
+    sharing one."""
+    if _gpu(x):
+        return _native().head_gate(x.contiguous(), P.contiguous(), int(col), int(per))
+    return ref.head_gate(x, P, col, per)
+
+
 def head_project(x, w, carry: int = 0):
     """Per head: x [T, H (K + carry)] rows' first K elements times ``w`` [H, N, K]^T, followed by
     the other ``carry`` as they are: [T, H (N + carry)]."""
@@ -1502,9 +1539,10 @@ class LinearMix:
     """A linear-attention recurrence S <- decay S + k u^T, o = S^T q per head: where its operands
     stand and what is done to them.  ``kind`` "channel": decays sigmoid(a . w + b)^inv_tau per key
     channel; "fixed": a decay per head, q and k rotated; "delta": unit q and k, a decay per head
-    exp(w softplus(a + b)), u = sigmoid(beta) (v - (decay S)^T k).  Columns ``q`` ``k`` ``v`` of the
+    exp(w softplus(a + b)), u = sigmoid(beta) (v - (decay S)^T k); "channel_delta": that with a decay
+    per key channel (a: heads x dim columns, w per head, b per channel).  Columns ``q`` ``k`` ``v`` of the
     matrix X, ``g`` (the output gate), ``a`` and ``b`` of Z.  Each head's o is normed over ``vdim``
-    (``eps``), weighted, and multiplied by silu(g)."""
+    (``eps``), weighted, and multiplied by ``gate`` of g: "silu" or "sigmoid"."""
     kind: str
     heads: int
     kv_heads: int
@@ -1521,10 +1559,11 @@ class LinearMix:
     k_scale: float = 1.0
     inv_tau: float = 1.0
     eps: float = 1e-5
+    gate: str = "silu"
 
     def native(self):
-        return ([("channel", "fixed", "delta").index(self.kind), self.heads, self.kv_heads, self.dim, self.vdim, self.q, self.k,
-                 self.v, self.g, self.a, self.b, self.rank], [self.q_scale, self.k_scale, self.inv_tau, self.eps])
+        return ([("channel", "fixed", "delta", "channel_delta").index(self.kind), self.heads, self.kv_heads, self.dim, self.vdim,
+                 self.q, self.k, self.v, self.g, self.a, self.b, self.rank, ("silu", "sigmoid").index(self.gate)], [self.q_scale, self.k_scale, self.inv_tau, self.eps])
 
 
 def linear_state_shape(heads: int, dim: int, vdim: int) -> tuple:
@@ -1551,6 +1590,14 @@ def linear_scan(X, Z, m: LinearMix, w_gate, b_gate, cs, norm, state, slots, cu, 
     return ref.linear_scan(X, Z, m, w_gate, b_gate, cs, norm, state, slots, cu, ctx, out)
 
 
+def low_rank(Z, at: int, w_a, w_g, n: int):
+    """fp32 [T, Na + Ng + n] of columns [a: Ka | g: Kg | n] of Z from ``at`` on: a ``w_a`` [Na, Ka]^T,
+    g ``w_g`` [Ng, Kg]^T, and the last ``n`` as they are -- decays, gates and steps of "channel_delta"."""
+    if _gpu(Z) and Z.dtype == torch.bfloat16:
+        return _native().low_rank(Z, int(at), w_a, w_g, int(n))
+    return ref.low_rank(Z, at, w_a, w_g, n)
+
+
 def post_norm(P, Q, gate, col: int, gate_b, residual, alpha: float, w, groups: int, eps: float, out_dtype=torch.bfloat16):
     """residual (fp32, in place) <- grouped RMS norm of alpha residual + sigmoid(gate + gate_b) (P + Q)
     times ``w``; returns it in ``out_dtype``.  ``gate``: columns [col, col + W) of a projection; P, Q,
@@ -1573,6 +1620,15 @@ def moe_route(x, w, experts: int, top: int):
     return ref.moe_route(x, w, experts, top)
 
 
+def moe_route_groups(x, w, correction, top: int, groups: int, keep: int, scale: float):
+    """Router of experts in groups, in fp32: scores s = softmax(x w^T); choice scores s + ``correction``;
+    the ``top`` largest within the ``keep`` of ``groups`` equal groups whose best is largest.  (ids
+    [T, top], weights [T, top] = their s over their sum, times ``scale``)."""
+    if _gpu(x):
+        return _native().moe_route_groups(x.contiguous(), w, correction, int(top), int(groups), int(keep), float(scale))
+    return ref.moe_route_groups(x, w, correction, top, groups, keep, scale)
+
+
 def glu(P, col: int, n: int, scale=None, out_dtype=torch.bfloat16):
     """silu(gate) * up of columns [col, col + n), [col + n, col + 2 n) of a projection, rows times
     ``scale`` [T]."""
@@ -1581,12 +1637,14 @@ def glu(P, col: int, n: int, scale=None, out_dtype=torch.bfloat16):
     return ref.glu(P, col, n, scale, out_dtype)
 
 
-def moe_experts(x, ids, wts, up, down):
-    """Slabs [top, T, W]: slab k holds, for every token, expert ids[:, k]'s output for the input
-    wts[:, k] x; ``up`` [E, 2 (gate, up), F, K], ``down`` [E, W, F]."""
+def moe_experts(x, ids, wts, up, down, limit: float = 0.0):
+    """Slabs [top, T, W]: slab k holds, for every token, expert ids[:, k]'s output; ``up``
+    [E, 2 (gate, up), F, K], ``down`` [E, W, F].  The input is wts[:, k] x through SwiGLU, or with a
+    ``limit`` x through g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = up within +-limit.  Ids from
+    E on have no expert: their part is not written."""
     if _gpu(x):
-        return _native().moe_experts(x.contiguous(), ids, wts, up, down)
-    return ref.moe_experts(x, ids, wts, up, down)
+        return _native().moe_experts(x.contiguous(), ids, wts, up, down, float(limit))
+    return ref.moe_experts(x, ids, wts, up, down, limit)
 
 
 def linear(x, w, decode: bool = False):

@@ -363,6 +363,22 @@ def embed_scale_rmsnorm(ids, table, scale, w, eps, keep):
     return h, (h.clone() if keep else None), (h if w is None else _rms(h, eps) * w).to(table.dtype, copy=True)
 
 
+def scaled_rmsnorm(P, residual, scale, w_next, eps, bias, mix, out_dtype):
+    if mix is None:
+        y = _slab_sum(P)
+    else:
+        ids, wts, experts, x = mix
+        y = sum(wts[:, k, None] * torch.where(ids[:, k, None] < experts, P[k].float(), x.float()) for k in range(P.shape[0]))
+    residual.add_(scale * (y if bias is None else y + bias))
+    return (_rms(residual, eps) * w_next).to(out_dtype or residual.dtype)
+
+
+def poly_norm(P, bias, act, n_out, eps, out_dtype):
+    z = _slab_sum(P)[:, :bias.shape[0]] + bias
+    y = sum(act[i] * _rms(z.pow(i + 1), eps) for i in range(3)) + act[3]
+    return F.pad(y, (0, n_out - y.shape[1])).to(out_dtype)
+
+
 def activation(P, act, out_dtype):
     x = _slab_sum(P)
     return (F.gelu(x, approximate="tanh") if act == "gelu_tanh" else x.clamp(min=0).square()).to(out_dtype)
@@ -407,15 +423,33 @@ def latent_store(P, cs, slots, cache, c_norm, H, dim, rank, eps, dtype):
     q[..., :dim] = xq[..., :dim].to(dtype)
     q[..., d8:d8 + r] = _rotate(xq[..., dim:], cs).to(dtype)
     if c_norm is not None:
-        BS, D = cache.shape[2:]
-        xk = x[:, H * (dim + r):H * (dim + r) + rank + r]
-        row = torch.zeros(T, D, dtype=cache.dtype, device=x.device)
-        row[:, :rank] = (_rms(xk[:, :rank], eps) * c_norm).to(cache.dtype)
-        row[:, D - r8:D - r8 + r] = _rotate(xk[:, rank:], cs).to(cache.dtype)
-        sm = slots.long()
-        ok = sm >= 0
-        cache[sm[ok] // BS, 0, sm[ok] % BS] = row[ok]
+        _store_latent(x[:, H * (dim + r):], cs, slots, cache, c_norm, eps)
     return q.view(T, H * (d8 + r8))
+
+
+def _store_latent(x, cs, slots, cache, c_norm, eps):
+    """The cache row of [latent | key part | ..]."""
+    (T, r), rank = cs.shape, c_norm.shape[0]
+    BS, D = cache.shape[2:]
+    r8 = -(-r // 8) * 8
+    row = torch.zeros(T, D, dtype=cache.dtype, device=x.device)
+    row[:, :rank] = (_rms(x[:, :rank], eps) * c_norm).to(cache.dtype)
+    row[:, D - r8:D - r8 + r] = _rotate(x[:, rank:rank + r], cs).to(cache.dtype)
+    sm = slots.long()
+    ok = sm >= 0
+    cache[sm[ok] // BS, 0, sm[ok] % BS] = row[ok]
+
+
+def latent_norm_store(P, cs, slots, cache, q_norm, c_norm, eps, dtype):
+    x, n = _slab_sum(P), q_norm.shape[0]
+    _store_latent(x[:, n:], cs, slots, cache, c_norm, eps)
+    return (_rms(x[:, :n], eps) * q_norm).to(dtype)
+
+
+def head_gate(x, P, col, per):
+    T, n = x.shape
+    g = torch.sigmoid(_slab_sum(P)[:, col:col + n // per])
+    return (x.float().view(T, -1, per) * g[..., None]).view(T, n).to(x.dtype)
 
 
 def head_project(x, w, carry):
@@ -596,6 +630,10 @@ def _linear_inputs(X, Z, m, w_gate, b_gate, cs):
         q, k = (t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6) for t in (q, k))
         la = (w_gate * F.softplus(z[:, m.a:m.a + H] + b_gate))[..., None]
         beta = torch.sigmoid(z[:, m.b:m.b + H])
+    elif m.kind == "channel_delta":
+        q, k = (t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6) for t in (q, k))
+        la = w_gate[:, None] * F.softplus(z[:, m.a:m.a + H * d] + b_gate).view(T, H, d)
+        beta = torch.sigmoid(z[:, m.b:m.b + H])
     elif m.kind == "channel":
         la = (F.logsigmoid(z[:, m.a:m.a + m.rank] @ w_gate.t() + b_gate) * m.inv_tau).view(T, H, d)
     else:
@@ -609,6 +647,7 @@ def _linear_inputs(X, Z, m, w_gate, b_gate, cs):
 def linear_scan(X, Z, m, w_gate, b_gate, cs, norm, state, slots, cu, ctx, out):
     q, k, v, g, la, beta = _linear_inputs(X, Z, m, w_gate, b_gate, cs)
     H, d, vd = m.heads, m.dim, m.vdim
+    gate = torch.sigmoid if m.gate == "sigmoid" else F.silu
     for b in range(cu.numel() - 1):
         q0, q1, slot = int(cu[b]), int(cu[b + 1]), int(slots[b])
         if q1 <= q0:
@@ -620,7 +659,7 @@ def linear_scan(X, Z, m, w_gate, b_gate, cs, norm, state, slots, cu, ctx, out):
             u = v[t] if beta is None else beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
             S = S + k[t][..., None] * u[:, None]
             o = torch.einsum("hdv,hd->hv", S, q[t])
-            out[t] = (_rms(o, m.eps) * norm * F.silu(g[t])).reshape(-1).to(out.dtype)
+            out[t] = (_rms(o, m.eps) * norm * gate(g[t])).reshape(-1).to(out.dtype)
         if slot >= 0:
             state[slot, ..., :vd] = S
     return out
@@ -629,6 +668,12 @@ def linear_scan(X, Z, m, w_gate, b_gate, cs, norm, state, slots, cu, ctx, out):
 def linear_step(X, Z, m, w_gate, b_gate, cs, norm, state, slots, positions, out):
     n = X.shape[-2]
     return linear_scan(X, Z, m, w_gate, b_gate, cs, norm, state, slots, torch.arange(n + 1, dtype=torch.int32), positions, out)
+
+
+def low_rank(Z, at, w_a, w_g, n):
+    ka, kg = w_a.shape[1], w_g.shape[1]
+    z = Z[:, at:at + ka + kg + n]
+    return torch.cat([z[:, :ka].float() @ w_a.float().t(), z[:, ka:ka + kg].float() @ w_g.float().t(), z[:, ka + kg:].float()], -1)
 
 
 # ------------------------------------------------------------ norms after the sum, experts
@@ -651,20 +696,37 @@ def moe_route(x, w, experts, top):
     return best.indices.to(torch.int32), best.values, s[:, experts:].contiguous()
 
 
+def moe_route_groups(x, w, correction, top, groups, keep, scale):
+    s = torch.softmax(x.float() @ w.float().t(), -1)
+    choice = s + correction
+    T, N = s.shape
+    parts = choice.view(T, groups, N // groups)
+    best = torch.topk(parts.amax(-1), keep, -1).indices
+    alive = torch.zeros(T, groups, dtype=torch.bool, device=x.device).scatter_(1, best, True)
+    ids = torch.topk(parts.masked_fill(~alive[..., None], -math.inf).reshape(T, N), top, -1).indices
+    wts = s.gather(1, ids)
+    return ids.to(torch.int32), wts / (wts.sum(-1, keepdim=True) + 1e-20) * scale
+
+
 def glu(P, col, n, scale, out_dtype):
     x = _slab_sum(P)
     y = F.silu(x[:, col:col + n]) * x[:, col + n:col + 2 * n]
     return (y if scale is None else y * scale.view(-1, 1)).to(out_dtype)
 
 
-def moe_experts(x, ids, wts, up, down):
+def moe_experts(x, ids, wts, up, down, limit=0.0):
     T, top = ids.shape
     out = torch.zeros(top, T, down.shape[1], dtype=x.dtype, device=x.device)
     for e in range(up.shape[0]):
         t, k = (ids == e).nonzero(as_tuple=True)
         if t.numel() == 0:
             continue
-        s = wts[t, k][:, None]
-        a = (F.silu(s * (x[t].float() @ up[e, 0].float().t())) * (s * (x[t].float() @ up[e, 1].float().t()))).to(x.dtype)
+        g, u = x[t].float() @ up[e, 0].float().t(), x[t].float() @ up[e, 1].float().t()
+        if limit > 0:
+            g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+            a = (g * torch.sigmoid(1.702 * g) * (u + 1)).to(x.dtype)
+        else:
+            s = wts[t, k][:, None]
+            a = (F.silu(s * g) * (s * u)).to(x.dtype)
         out[k, t] = (a.float() @ down[e].float().t()).to(x.dtype)
     return out
