@@ -112,6 +112,65 @@ Tensor add_scaled(const Tensor& P, const OptT& Q, Tensor residual, double m, boo
   return out;
 }
 
+// residual += scale (P + bias), or scale times the weighted sum of the chosen experts' outputs P; rms(residual) w
+Tensor scaled_rmsnorm(const Tensor& P, Tensor residual, const Tensor& scale, const OptT& bias, const OptT& ids, const OptT& wts,
+                      int64_t experts, const OptT& x, const Tensor& w, double eps, bool out_f32) {
+  const Slabs p = slabs_of(P);
+  CHECK_GPU(residual); CHECK_F32(residual); CHECK_CONTIG(residual); CHECK_ALIGN16(residual); CHECK_ALIGN16(P);
+  TORCH_CHECK(residual.dim() == 2 && residual.size(0) == p.M && residual.size(1) == p.N, "residual shape mismatch");
+  check_vec(scale, p.N, "scale"); check_vec(w, p.N, "w");
+  CHECK_ALIGN16(scale); CHECK_ALIGN16(w);
+  DocqaScaledNorm a{};
+  a.P = P.data_ptr(); a.pf32 = is_f32(P); a.SP = p.S; a.rows = p.M; a.W = p.N;
+  if (bias.has_value()) {
+    check_vec(*bias, p.N, "bias");
+    CHECK_ALIGN16(*bias);
+    a.bias = bias->data_ptr<float>();
+  }
+  if (ids.has_value()) {
+    TORCH_CHECK(wts.has_value() && x.has_value() && P.dim() == 3, "scaled_rmsnorm: weights and the experts' input");
+    TORCH_CHECK(ids->dim() == 2 && ids->size(0) == p.M && ids->size(1) == p.S, "scaled_rmsnorm: ids [rows, chosen]");
+    check_i32(*ids, (int64_t)p.M * p.S, "ids");
+    check_vec(*wts, (int64_t)p.M * p.S, "wts");
+    CHECK_ACT(*x); CHECK_CONTIG(*x); CHECK_ALIGN16(*x);
+    TORCH_CHECK(x->scalar_type() == P.scalar_type() && x->dim() == 2 && x->size(0) == p.M && x->size(1) == p.N, "scaled_rmsnorm: x");
+    a.ids = ids->data_ptr<int>(); a.wts = wts->data_ptr<float>(); a.x = x->data_ptr(); a.experts = (int)experts;
+  }
+  c10::DeviceGuard g(P.device());
+  auto out = at::empty({p.M, p.N}, P.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
+  a.scale = scale.data_ptr<float>(); a.res = residual.data_ptr<float>(); a.w = w.data_ptr<float>(); a.out = out.data_ptr();
+  a.of32 = out_f32; a.eps = (float)eps;
+  CHECK_RC(docqa_scaled_rmsnorm(a, stream()), "scaled_rmsnorm");
+  return out;
+}
+
+Tensor poly_norm(const Tensor& P, const Tensor& bias, const Tensor& act, int64_t n_out, double eps, bool out_f32) {
+  const Slabs p = slabs_of(P);
+  const int n = bias.numel();
+  check_vec(bias, n, "bias"); check_vec(act, 4, "act");
+  CHECK_ALIGN16(P); CHECK_ALIGN16(bias);
+  TORCH_CHECK(n >= 1 && n <= p.N && n_out >= n && n_out <= (1 << 20), "poly_norm: columns");
+  c10::DeviceGuard g(P.device());
+  auto out = at::empty({p.M, n_out}, P.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
+  CHECK_RC(docqa_poly_norm(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, bias.data_ptr<float>(), act.data_ptr<float>(),
+                           out.data_ptr(), out_f32, p.M, n, (int)n_out, (float)eps, stream()),
+           "poly_norm");
+  return out;
+}
+
+Tensor head_gate(const Tensor& x, const Tensor& P, int64_t col, int64_t per) {
+  CHECK_ACT(x); CHECK_CONTIG(x); CHECK_ALIGN16(x); CHECK_ALIGN16(P);
+  const Slabs p = slabs_of(P);
+  TORCH_CHECK(x.dim() == 2 && x.size(0) == p.M && per >= 1 && x.size(1) % per == 0, "head_gate: shapes");
+  TORCH_CHECK(col >= 0 && col + x.size(1) / per <= p.N && (is_f32(P) || !is_f32(x)), "head_gate: columns");
+  c10::DeviceGuard g(x.device());
+  auto y = at::empty_like(x);
+  CHECK_RC(docqa_head_gate(x.data_ptr(), is_f32(x), P.data_ptr(), is_f32(P), p.S, p.slab, p.N, (int)col, (int)per, y.data_ptr(),
+                           p.M, (int)x.size(1), stream()),
+           "head_gate");
+  return y;
+}
+
 Tensor soft_cap(const Tensor& x, double cap) {
   CHECK_ACT(x); CHECK_CONTIG(x);
   TORCH_CHECK(cap > 0, "cap");
@@ -375,6 +434,28 @@ Tensor latent_store(const Tensor& P, const Tensor& cs, const Tensor& slots, Tens
   return q;
 }
 
+// P: [query latent | latent: rank | r | ..] -> the normed query latent; the cache row is stored
+Tensor latent_norm_store(const Tensor& P, const Tensor& cs, const Tensor& slots, Tensor cache, const Tensor& q_norm,
+                         const Tensor& c_norm, double eps) {
+  const Slabs p = slabs_of(P);
+  CHECK_ACT(cache); CHECK_CONTIG(cache); CHECK_ALIGN16(cache); CHECK_ALIGN16(P); CHECK_ALIGN16(cs);
+  TORCH_CHECK(cs.dim() == 2, "cs must be [tokens, r]");
+  const int64_t r = cs.size(1), Rq = q_norm.numel(), R = c_norm.numel();
+  check_vec(cs, p.M * r, "cs"); check_vec(q_norm, Rq, "q_norm"); check_vec(c_norm, R, "c_norm");
+  CHECK_ALIGN16(q_norm); CHECK_ALIGN16(c_norm);
+  check_i32(slots, p.M, "slots");
+  TORCH_CHECK(cache.dim() == 4 && cache.size(1) == 1 && cache.size(3) == (R + 7) / 8 * 8 + (r + 7) / 8 * 8,
+              "cache must be [blocks, 1, block, latent + rotated part]");
+  TORCH_CHECK(p.N >= Rq + R + r, "latent_norm_store: projection width");
+  c10::DeviceGuard g(P.device());
+  auto cq = at::empty({p.M, Rq}, cache.options());
+  CHECK_RC(docqa_latent_norm_store(P.data_ptr(), is_f32(P), p.S, p.slab, p.N, cs.data_ptr<float>(), slots.data_ptr<int>(),
+                                   q_norm.data_ptr<float>(), c_norm.data_ptr<float>(), cq.data_ptr(), cache.data_ptr(),
+                                   is_f32(cache), p.M, (int)Rq, (int)r, (int)R, (int)cache.size(2), (float)eps, stream()),
+           "latent_norm_store");
+  return cq;
+}
+
 Tensor head_project(const Tensor& x, const Tensor& w, int64_t carry) {
   CHECK_GPU(x); CHECK_BF16(x); CHECK_BF16(w); CHECK_GPU(w); CHECK_CONTIG(x); CHECK_CONTIG(w);
   TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && carry >= 0 && x.size(1) == w.size(0) * (w.size(2) + carry), "head_project: shapes");
@@ -558,10 +639,10 @@ DocqaLinear linear_args(const Tensor& X, const Tensor& Z, at::IntArrayRef d, at:
                         const OptT& b_gate, const OptT& cs, const Tensor& norm, const Tensor& state, Tensor& out) {
   const Slabs x = slabs_of(X), z = slabs_of(Z);
   CHECK_ALIGN16(state);
-  TORCH_CHECK(d.size() == 12 && f.size() == 4, "linear attention: arguments");
+  TORCH_CHECK(d.size() == 13 && f.size() == 4, "linear attention: arguments");
   DocqaLinear a{};
-  int* const to[12] = {&a.kind, &a.H, &a.G, &a.dk, &a.dv, &a.qo, &a.ko, &a.vo, &a.go, &a.ao, &a.bo, &a.rank};
-  for (int i = 0; i < 12; ++i) {
+  int* const to[13] = {&a.kind, &a.H, &a.G, &a.dk, &a.dv, &a.qo, &a.ko, &a.vo, &a.go, &a.ao, &a.bo, &a.rank, &a.sig};
+  for (int i = 0; i < 13; ++i) {
     TORCH_CHECK(d[i] >= 0 && d[i] < (1 << 24), "linear attention: sizes");
     *to[i] = (int)d[i];
   }
@@ -569,7 +650,7 @@ DocqaLinear linear_args(const Tensor& X, const Tensor& Z, at::IntArrayRef d, at:
   a.xf32 = is_f32(X); a.Sx = x.S; a.ldx = x.N; a.xslab = x.slab;
   a.zf32 = is_f32(Z); a.Sz = z.S; a.ldz = z.N; a.zslab = z.slab;
   a.qs = (float)f[0]; a.ks = (float)f[1]; a.inv_tau = (float)f[2]; a.eps = (float)f[3];
-  TORCH_CHECK(a.kind <= LIN_DELTA && a.H >= 1 && a.G >= 1 && a.H % a.G == 0 && a.dk >= 1 && a.dk <= 256 && a.dv >= 1 && a.dv <= 512,
+  TORCH_CHECK(a.kind <= LIN_CHANNEL_DELTA && a.H >= 1 && a.G >= 1 && a.H % a.G == 0 && a.dk >= 1 && a.dk <= 256 && a.dv >= 1 && a.dv <= 512,
               "linear attention: heads up to [256, 512]");
   TORCH_CHECK(a.qo + a.G * a.dk <= x.N && a.ko + a.G * a.dk <= x.N && a.vo + a.H * a.dv <= x.N && a.go + a.H * a.dv <= z.N &&
                   x.M == z.M, "linear attention: columns");
@@ -580,9 +661,10 @@ DocqaLinear linear_args(const Tensor& X, const Tensor& Z, at::IntArrayRef d, at:
     check_vec(*b_gate, n, "b_gate");
   } else {
     check_vec(w_gate, a.H, "w_gate");
-    if (a.kind == LIN_DELTA) {
-      TORCH_CHECK(a.ao + a.H <= z.N && a.bo + a.H <= z.N && b_gate.has_value(), "linear attention: decay columns");
-      check_vec(*b_gate, a.H, "b_gate");
+    if (a.kind >= LIN_DELTA) {
+      const int64_t na = a.kind == LIN_DELTA ? a.H : n;
+      TORCH_CHECK(a.ao + na <= z.N && a.bo + a.H <= z.N && b_gate.has_value(), "linear attention: decay columns");
+      check_vec(*b_gate, na, "b_gate");
     }
   }
   if (a.kind == LIN_FIXED) {
@@ -630,6 +712,21 @@ void linear_scan(const Tensor& X, const Tensor& Z, at::IntArrayRef dims, at::Arr
   CHECK_RC(docqa_linear_scan(a, cu.data_ptr<int>(), ctx.data_ptr<int>(), scratch.data_ptr<float>(), T, B, (int)max_len,
                              stream()),
            "linear_scan");
+}
+
+Tensor low_rank(const Tensor& z, int64_t at_, const Tensor& wa, const Tensor& wg, int64_t n) {
+  CHECK_GPU(z); CHECK_BF16(z); CHECK_BF16(wa); CHECK_BF16(wg); CHECK_GPU(wa); CHECK_GPU(wg); CHECK_CONTIG(wa); CHECK_CONTIG(wg);
+  CHECK_ALIGN16(wa); CHECK_ALIGN16(wg);
+  TORCH_CHECK(wa.dim() == 2 && wg.dim() == 2 && n >= 0 && at_ >= 0, "low_rank: weights [out, in]");
+  const int64_t T = z.size(0), Na = wa.size(0), Ka = wa.size(1), Ng = wg.size(0), Kg = wg.size(1);
+  check_rows(z, T, at_ + Ka + Kg + n, z, "z");
+  c10::DeviceGuard g(z.device());
+  auto y = at::empty({T, Na + Ng + n}, z.options().dtype(at::kFloat));
+  // (a row of one: its stride may be anything)
+  CHECK_RC(docqa_low_rank(z.data_ptr(), T > 1 ? (int)z.stride(0) : (int)z.size(1), (int)at_, wa.data_ptr(), (int)Na, (int)Ka,
+                          wg.data_ptr(), (int)Ng, (int)Kg, (int)n, y.data_ptr<float>(), (int)T, stream()),
+           "low_rank");
+  return y;
 }
 
 Tensor post_norm(const OptT& P, const OptT& Q, const OptT& gate, int64_t col, const OptT& gate_b, Tensor residual,
@@ -682,6 +779,23 @@ std::tuple<Tensor, Tensor, Tensor> moe_route(const Tensor& x, const Tensor& w, i
   return {ids, wts, rest};
 }
 
+std::tuple<Tensor, Tensor> moe_route_groups(const Tensor& x, const Tensor& w, const Tensor& corr, int64_t top, int64_t groups,
+                                            int64_t keep, double scale) {
+  CHECK_ACT(x); CHECK_CONTIG(x); CHECK_CONTIG(w); CHECK_GPU(w); CHECK_ALIGN16(x); CHECK_ALIGN16(w);
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.size(1) == x.size(1) && w.scalar_type() == x.scalar_type(), "moe_route_groups: shapes");
+  const int64_t T = x.size(0), N = w.size(0);
+  check_vec(corr, N, "correction");
+  TORCH_CHECK(groups >= 1 && N % groups == 0 && keep >= 1 && keep <= groups && top >= 1 && top <= keep * (N / groups),
+              "moe_route_groups: groups");
+  c10::DeviceGuard g(x.device());
+  auto ids = at::empty({T, top}, x.options().dtype(at::kInt)), wts = at::empty({T, top}, x.options().dtype(at::kFloat));
+  CHECK_RC(docqa_moe_route_groups(x.data_ptr(), w.data_ptr(), is_f32(x), corr.data_ptr<float>(), ids.data_ptr<int>(),
+                                  wts.data_ptr<float>(), (int)T, (int)x.size(1), (int)N, (int)top, (int)groups, (int)keep,
+                                  (float)scale, stream()),
+           "moe_route_groups");
+  return {ids, wts};
+}
+
 Tensor slab_glu(const Tensor& P, int64_t col, int64_t n, const OptT& scale, bool out_f32) {
   const Slabs p = slabs_of(P);
   CHECK_ALIGN16(P);
@@ -695,7 +809,7 @@ Tensor slab_glu(const Tensor& P, int64_t col, int64_t n, const OptT& scale, bool
   return out;
 }
 
-Tensor moe_experts(const Tensor& x, const Tensor& ids, const Tensor& wts, const Tensor& up, const Tensor& down) {
+Tensor moe_experts(const Tensor& x, const Tensor& ids, const Tensor& wts, const Tensor& up, const Tensor& down, double limit) {
   CHECK_ACT(x); CHECK_CONTIG(x); CHECK_CONTIG(up); CHECK_CONTIG(down); CHECK_GPU(up); CHECK_GPU(down);
   CHECK_ALIGN16(x); CHECK_ALIGN16(up); CHECK_ALIGN16(down);
   TORCH_CHECK(x.dim() == 2 && up.dim() == 4 && up.size(1) == 2 && down.dim() == 3 && ids.dim() == 2 && ids.size(0) == x.size(0),
@@ -711,7 +825,7 @@ Tensor moe_experts(const Tensor& x, const Tensor& ids, const Tensor& wts, const 
   auto scratch = at::empty({n}, ids.options());
   CHECK_RC(docqa_moe_experts(x.data_ptr(), ids.data_ptr<int>(), wts.data_ptr<float>(), up.data_ptr(), down.data_ptr(),
                              act.data_ptr(), out.data_ptr(), n ? scratch.data_ptr<int>() : nullptr, is_f32(x), (int)T,
-                             (int)top, (int)E, (int)K, (int)F, (int)W, stream()),
+                             (int)top, (int)E, (int)K, (int)F, (int)W, (float)limit, stream()),
            "moe_experts");
   return out;
 }
@@ -725,6 +839,13 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
         "-> (Tensor, Tensor, Tensor)");
   m.def("decode_act(Tensor x, Tensor w, int act) -> Tensor");
   m.def("add_scaled(Tensor P, Tensor? Q, Tensor(a!) residual, float m, bool out_f32) -> Tensor");
+  m.def("scaled_rmsnorm(Tensor P, Tensor(a!) residual, Tensor scale, Tensor? bias, Tensor? ids, Tensor? wts, int experts, "
+        "Tensor? x, Tensor w, float eps, bool out_f32) -> Tensor");
+  m.def("poly_norm(Tensor P, Tensor bias, Tensor act, int n_out, float eps, bool out_f32) -> Tensor");
+  m.def("head_gate(Tensor x, Tensor P, int col, int per) -> Tensor");
+  m.def("latent_norm_store(Tensor P, Tensor cs, Tensor slots, Tensor(a!) cache, Tensor q_norm, Tensor c_norm, float eps) -> Tensor");
+  m.def("low_rank(Tensor z, int at, Tensor wa, Tensor wg, int n) -> Tensor");
+  m.def("moe_route_groups(Tensor x, Tensor w, Tensor corr, int top, int groups, int keep, float scale) -> (Tensor, Tensor)");
   m.def("soft_cap(Tensor x, float cap) -> Tensor");
   m.def("side_gate(Tensor P, Tensor ids, Tensor table, int col, int n, bool out_f32) -> Tensor");
   m.def("side_project(Tensor P, Tensor ids, Tensor table, int col, int n, Tensor w) -> Tensor");
@@ -756,7 +877,7 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
         "int groups, float eps, bool out_f32) -> Tensor");
   m.def("moe_route(Tensor x, Tensor w, int experts, int top) -> (Tensor, Tensor, Tensor)");
   m.def("slab_glu(Tensor P, int col, int n, Tensor? scale, bool out_f32) -> Tensor");
-  m.def("moe_experts(Tensor x, Tensor ids, Tensor wts, Tensor up, Tensor down) -> Tensor");
+  m.def("moe_experts(Tensor x, Tensor ids, Tensor wts, Tensor up, Tensor down, float limit) -> Tensor");
   m.def("causal_conv(Tensor x, Tensor w, Tensor? bias, Tensor(a!) state, Tensor slots, Tensor cu, Tensor ctx, "
         "int max_len, bool silu) -> Tensor");
   m.def("conv_step(Tensor P, Tensor w, Tensor? bias, Tensor(a!) state, Tensor slots, Tensor positions, bool silu, "
@@ -772,6 +893,12 @@ TORCH_LIBRARY_IMPL(docqa, CUDA, m) {
   m.impl("embed_scale_rmsnorm", &embed_scale_rmsnorm);
   m.impl("decode_act", &decode_act);
   m.impl("add_scaled", &add_scaled);
+  m.impl("scaled_rmsnorm", &scaled_rmsnorm);
+  m.impl("poly_norm", &poly_norm);
+  m.impl("head_gate", &head_gate);
+  m.impl("latent_norm_store", &latent_norm_store);
+  m.impl("low_rank", &low_rank);
+  m.impl("moe_route_groups", &moe_route_groups);
   m.impl("soft_cap", &soft_cap);
   m.impl("side_gate", &side_gate);
   m.impl("side_project", &side_project);

@@ -18,6 +18,25 @@ int docqa_embed_scale_rmsnorm(const int* ids, const void* table, int f32, float 
 int docqa_sandwich_rmsnorm_conv(const void* P, int p_f32, int S, float* res, const float* w_post, const float* w_next,
                                 const float* cw, int taps, void* state, const int* slots, const int* positions, void* out,
                                 void* out2, int out_f32, int rows, int H, float eps, hipStream_t s);
+// res += scale (P + bias) per channel, out = rms(res) w
+struct DocqaScaledNorm {
+  const void* P;                  // [SP, rows, W]: slabs, or (ids) the SP chosen experts' outputs, of x's type
+  int pf32, SP;
+  const float *scale, *bias;      // [W]; bias null: none
+  const int* ids;                 // [rows, SP] or null; from `experts` on: x itself
+  const float* wts;               // [rows, SP]
+  const void* x;                  // [rows, W]
+  int experts;
+  float* res;
+  const float* w;
+  void* out;
+  int of32, rows, W;
+  float eps;
+};
+int docqa_scaled_rmsnorm(const DocqaScaledNorm& a, hipStream_t s);
+// z = P + bias [n]: out [T, n_out] = a N(z) + b N(z^2) + c N(z^3) + e, N over the row's RMS, zero past n
+int docqa_poly_norm(const void* P, int p_f32, int S, size_t slab, int ld, const float* bias, const float* act, void* out,
+                    int out_f32, int T, int n, int n_out, float eps, hipStream_t s);
 // res [n] += m (P + Q) (Q null: P alone), each with its own slab count; out null or bf16 [n]: a copy of res
 int docqa_add_scaled(const void* P, int p_f32, int SP, const void* Q, int q_f32, int SQ, float* res, float m, void* out,
                      size_t n, hipStream_t s);
@@ -70,6 +89,13 @@ int docqa_latent_splits(int B, int max_q, int H, int DV, int max_keys);
 int docqa_latent_attn(const void* q, const void* kc, const int* block_tables, int maxb, const int* cu, const int* ctx,
                       const float* sink, void* out, void* part, void* ml, int nsplit, int B, int max_q, int tokens, int H,
                       int D, int DV, int BS, float scale, int window, hipStream_t s);
+// P [T, ld]: [query latent Rq | latent R | key part r | ..]: the normed query latent, the cache row
+int docqa_latent_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* cs, const int* slots,
+                            const float* q_norm, const float* c_norm, void* cq, void* cache, int f32, int T, int Rq, int r,
+                            int R, int BS, float eps, hipStream_t s);
+// y [T, n] = x sigmoid(P[:, col + i / per])
+int docqa_head_gate(const void* x, int f32, const void* P, int p_f32, int S, size_t slab, int ld, int col, int per, void* y,
+                    int T, int n, hipStream_t s);
 int docqa_latent_gather(const void* cache, const int* block_tables, int maxb, const int* first, const int* cu_k, void* c,
                         void* kr, int B, int max_keys, int R8, int r8, int BS, hipStream_t s);
 
@@ -90,14 +116,16 @@ int docqa_selective_step(const void* x, const void* dt, const void* dt_in, const
                          int B, int C, int N, int Np, hipStream_t s);
 
 // ---- linear attention (linear_attn.hip)
-enum { LIN_CHANNEL = 0, LIN_FIXED = 1, LIN_DELTA = 2 };
+enum { LIN_CHANNEL = 0, LIN_FIXED = 1, LIN_DELTA = 2, LIN_CHANNEL_DELTA = 3 };
 struct DocqaLinear {
   const void *X, *Z;        // [tokens, ldx], [tokens, ldz]: products or slabs
   int xf32, Sx, ldx, zf32, Sz, ldz;
   size_t xslab, zslab;
   int kind, H, G, dk, dv, qo, ko, vo, go, ao, bo, rank, r;   // column offsets; rotated dimensions
+  int sig;                  // output gate: sigmoid(g), else silu(g)
   float qs, ks, inv_tau, eps;
-  const float *w_gate, *b_gate;   // channel: [H dk, rank], [H dk]; fixed: log decay [H], -; delta: -exp(A) [H], [H]
+  const float *w_gate, *b_gate;   // channel: [H dk, rank], [H dk]; fixed: log decay [H], -; delta: -exp(A) [H], [H];
+                                  // channel delta: -exp(A) [H], [H dk]
   const float* cs;          // [tokens, r]
   const float* norm;        // [dv]
   float* state;             // [slots, H, dk, dvp], dvp = dv rounded up to 4
@@ -111,6 +139,11 @@ int docqa_linear_chunk(int dk);
 size_t docqa_linear_scratch(int kind, int tokens, int B, int H, int dk, int dv);
 int docqa_linear_scan(const DocqaLinear& a, const int* cu, const int* ctx, float* scratch, int tokens, int B, int max_len,
                       hipStream_t s);
+
+// y fp32 [T, Na + Ng + n] of columns [Ka | Kg | n] of z [T, ldz] from `at` on: .. wa [Na, Ka]^T, .. wg [Ng, Kg]^T, as
+// they are
+int docqa_low_rank(const void* z, int ldz, int at, const void* wa, int Na, int Ka, const void* wg, int Ng, int Kg, int n,
+                   float* y, int T, hipStream_t s);
 
 // ---- norms after the sum (sandwich_norm.hip): res <- groupnorm(alpha res + sigmoid(gate[:, col:] + gb) (P + Q)) w
 struct DocqaPostNorm {
@@ -129,9 +162,13 @@ int docqa_post_norm(const DocqaPostNorm& a, hipStream_t s);
 // ---- experts (moe.hip)
 int docqa_moe_route(const void* x, const void* w, int f32, int* ids, float* wts, float* rest, int T, int K, int N, int E,
                     int top, hipStream_t s);
+// softmax scores, choice by score + corr [N] within the best `keep` of `groups`, weights over their sum times scale
+int docqa_moe_route_groups(const void* x, const void* w, int f32, const float* corr, int* ids, float* wts, int T, int K, int N,
+                           int top, int groups, int keep, float scale, hipStream_t s);
 int docqa_slab_glu(const void* P, int p_f32, int S, size_t slab, int ld, int col, int n, const float* scale, void* out,
                    int out_f32, int T, hipStream_t s);
 // int32 scratch of a sorted launch; 0: the rows are found in the launch
 int docqa_moe_scratch(int f32, int T, int top, int E, int K, int F, int W);
+// limit > 0: clamped experts on x itself (wts unused); ids from E on have no expert, nothing is written for them
 int docqa_moe_experts(const void* x, const int* ids, const float* wts, const void* up, const void* down, void* act,
-                      void* out, int* scratch, int f32, int T, int top, int E, int K, int F, int W, hipStream_t s);
+                      void* out, int* scratch, int f32, int T, int top, int E, int K, int F, int W, float limit, hipStream_t s);

@@ -348,3 +348,143 @@ int docqa_slab_glu(const void* P, int p_f32, int S, size_t slab, int ld, int col
   return out_f32 ? launch_slab_glu((const uint16_t*)P, S, slab, ld, col, n, scale, (float*)out, T, s)
                  : launch_slab_glu((const uint16_t*)P, S, slab, ld, col, n, scale, (uint16_t*)out, T, s);
 }
+
+// PolyNorm of z = P + bias over a row of n: a N(z) + b N(z^2) + c N(z^3) + e with N(v) = v / sqrt(mean(v^2) + eps),
+// (a, b, c, e) = act.  One workgroup of NT threads a row, the row in registers
+template <int NT, int NV, int V, typename PT, typename OT>
+__global__ __launch_bounds__(NT) void poly_norm_kernel(const PT* __restrict__ P, int S, size_t slab, int ld,
+                                                       const float* __restrict__ bias, const float* __restrict__ act,
+                                                       OT* __restrict__ out, int n, int n_out, float eps) {
+  __shared__ float red[3][NT / 64];
+  const size_t t = blockIdx.x;
+  const int tid = threadIdx.x;
+  float z[NV][V], s2 = 0.f, s4 = 0.f, s6 = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (tid + NT * i) * V;
+#pragma unroll
+    for (int j = 0; j < V; ++j) z[i][j] = 0.f;
+    if (c < n) {
+      float b[V];
+      docqa::ld_slabs<V>(P + t * ld + c, S, slab, z[i]);
+      docqa::ldv<V>(bias + c, b);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        z[i][j] += b[j];
+        const float q = z[i][j] * z[i][j];
+        s2 += q;
+        s4 += q * q;
+        s6 += q * q * q;
+      }
+    }
+  }
+  s2 = wave_sum(s2);
+  s4 = wave_sum(s4);
+  s6 = wave_sum(s6);
+  if ((tid & 63) == 0) {
+    red[0][tid >> 6] = s2;
+    red[1][tid >> 6] = s4;
+    red[2][tid >> 6] = s6;
+  }
+  __syncthreads();
+  s2 = s4 = s6 = 0.f;
+#pragma unroll
+  for (int w = 0; w < NT / 64; ++w) {
+    s2 += red[0][w];
+    s4 += red[1][w];
+    s6 += red[2][w];
+  }
+  const float rn = 1.f / (float)n;
+  const float a = act[0] / sqrtf(s2 * rn + eps), b = act[1] / sqrtf(s4 * rn + eps), c3 = act[2] / sqrtf(s6 * rn + eps), e = act[3];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (tid + NT * i) * V;
+    if (c >= n_out) continue;
+    float y[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) y[j] = c < n ? z[i][j] * (a + z[i][j] * (b + z[i][j] * c3)) + e : 0.f;
+    docqa::stv<V>(out + t * n_out + c, y);
+  }
+}
+
+template <int V, typename PT, typename OT>
+static int launch_poly_norm(const PT* P, int S, size_t slab, int ld, const float* bias, const float* act, OT* out, int T, int n,
+                            int n_out, float eps, hipStream_t s) {
+  const int m = n_out / V;
+#define GO(NT, NV) poly_norm_kernel<NT, NV, V, PT, OT><<<T, NT, 0, s>>>(P, S, slab, ld, bias, act, out, n, n_out, eps)
+  if (m <= 256) GO(256, 1);
+  else if (m <= 512) GO(256, 2);
+  else if (m <= 1024) GO(256, 4);
+  else if (m <= 2048) GO(1024, 2);
+  else if (m <= 4096) GO(1024, 4);
+  else if (m <= 8192) GO(1024, 8);
+  else if (V == 1 && m <= 32768) GO(1024, (V == 1 ? 32 : 8));
+  else return -1;
+#undef GO
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+template <typename PT, typename OT>
+static int poly_norm_vec(const void* P, int S, size_t slab, int ld, const float* bias, const float* act, void* out, int T, int n,
+                         int n_out, float eps, hipStream_t s) {
+  if (n % 4 == 0 && n_out % 4 == 0 && ld % 4 == 0)
+    return launch_poly_norm<4, PT, OT>((const PT*)P, S, slab, ld, bias, act, (OT*)out, T, n, n_out, eps, s);
+  return launch_poly_norm<1, PT, OT>((const PT*)P, S, slab, ld, bias, act, (OT*)out, T, n, n_out, eps, s);
+}
+
+int docqa_poly_norm(const void* P, int p_f32, int S, size_t slab, int ld, const float* bias, const float* act, void* out,
+                    int out_f32, int T, int n, int n_out, float eps, hipStream_t s) {
+  if (T == 0) return 0;
+  if (S < 1 || n < 1 || n > ld || n_out < n) return -1;
+#define ARGS P, S, slab, ld, bias, act, out, T, n, n_out, eps, s
+  if (p_f32) return out_f32 ? poly_norm_vec<float, float>(ARGS) : poly_norm_vec<float, uint16_t>(ARGS);
+  return out_f32 ? poly_norm_vec<uint16_t, float>(ARGS) : poly_norm_vec<uint16_t, uint16_t>(ARGS);
+#undef ARGS
+}
+
+// y [T, n] = x sigmoid(P[:, col + i / per]): an output gate, one number an element or (per > 1) a head
+template <int V, typename T, typename PT>
+__global__ __launch_bounds__(256) void head_gate_kernel(const T* __restrict__ x, const PT* __restrict__ P, int S, size_t slab,
+                                                        int ld, int col, int per, T* __restrict__ y, int rows, int n) {
+  const int m = n / V;
+  const size_t total = (size_t)rows * m;
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
+    const size_t t = i / m;
+    const int c = (int)(i - t * m) * V;
+    float f[V], g[V];
+    docqa::ldv<V>(x + t * n + c, f);
+    if (per == 1) {
+      docqa::ld_slabs<V>(P + t * ld + col + c, S, slab, g);
+    } else {
+      docqa::ld_slabs<1>(P + t * ld + col + c / per, S, slab, g);
+#pragma unroll
+      for (int j = 1; j < V; ++j) g[j] = g[0];
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) f[j] /= 1.f + expf(-g[j]);
+    docqa::stv<V>(y + t * n + c, f);
+  }
+}
+
+template <typename T, typename PT>
+static int launch_head_gate(const void* x, const void* P, int S, size_t slab, int ld, int col, int per, void* y, int rows, int n,
+                            hipStream_t s) {
+  const bool vec = n % 4 == 0 && (per == 1 ? ld % 4 == 0 && col % 4 == 0 : per % 4 == 0);
+  const size_t g = ((size_t)rows * (n / (vec ? 4 : 1)) + 255) / 256;
+  const int grid = (int)(g < 8192 ? g : 8192);
+  if (vec) head_gate_kernel<4, T, PT><<<grid, 256, 0, s>>>((const T*)x, (const PT*)P, S, slab, ld, col, per, (T*)y, rows, n);
+  else head_gate_kernel<1, T, PT><<<grid, 256, 0, s>>>((const T*)x, (const PT*)P, S, slab, ld, col, per, (T*)y, rows, n);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+int docqa_head_gate(const void* x, int f32, const void* P, int p_f32, int S, size_t slab, int ld, int col, int per, void* y,
+                    int T, int n, hipStream_t s) {
+  if (T == 0) return 0;
+  if (S < 1 || n < 1 || per < 1 || n % per || col < 0 || col + n / per > ld || (f32 && !p_f32)) return -1;
+#define ARGS x, P, S, slab, ld, col, per, y, T, n, s
+  if (f32) return launch_head_gate<float, float>(ARGS);
+  return p_f32 ? launch_head_gate<uint16_t, float>(ARGS) : launch_head_gate<uint16_t, uint16_t>(ARGS);
+#undef ARGS
+}

@@ -6,7 +6,8 @@
 //   * rope_table:    [cos | sin] rows of a forward's positions, angles in fp64, once for all layers;
 //   * latent_store:  consumer of the [q | latent | key part] projection: sums the split-K slabs,
 //                    rotates the query heads, normalises the latent, rotates the key part, stores
-//                    the cache row;
+//                    the cache row; with a query latent (latent_norm_store) that is normed in the same
+//                    launch, and a second one rotates the heads its projection makes;
 //   * absorbed form (decode, short portions): head_project takes the query heads into the latent
 //     space, every head attends the cached rows themselves -- key and value at once -- and
 //     head_project takes the attended latents to values (summing the key splits on the way);
@@ -58,9 +59,12 @@ struct StoreArgs {
   const float* wn;        // [R] or null: no latent in the projection
   int H, d, r, R, d8, r8, R8, D, log2BS;
   float eps;
+  const float* wq;        // [Rq] or null: a query latent ahead of the latent, H = 0
+  int Rq;
 };
 
-// grid (token, y): y < ny: 256 V-element items of the query heads; y == ny: the latent row
+// grid (token, y): y < ny: 256 V-element items of the query heads; y == ny: the latent row; y > ny: the
+// query latent, normed, to q
 template <int V, int NI, typename PT, typename T>
 __global__ __launch_bounds__(256) void latent_store_kernel(const PT* __restrict__ P, T* __restrict__ q,
                                                            T* __restrict__ cache, int ny, StoreArgs a) {
@@ -102,34 +106,41 @@ __global__ __launch_bounds__(256) void latent_store_kernel(const PT* __restrict_
     }
     return;
   }
+  auto normed = [&](const PT* x, int R, const float* wn, T* o) {
+    float f[NI][V];
+    float ss = 0.f;
+#pragma unroll
+    for (int n = 0; n < NI; ++n) {
+      const int c = (tid + 256 * n) * V;
+      if (c < R) {
+        ld_slabs<V>(x + c, a.S, a.slab, f[n]);
+#pragma unroll
+        for (int j = 0; j < V; ++j) ss += f[n][j] * f[n][j];
+      }
+    }
+    const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)R + a.eps);
+#pragma unroll
+    for (int n = 0; n < NI; ++n) {
+      const int c = (tid + 256 * n) * V;
+      if (c < R) {
+        float w[V];
+        ldv<V>(wn + c, w);
+#pragma unroll
+        for (int j = 0; j < V; ++j) f[n][j] *= inv * w[j];
+        stv<V>(o + c, f[n]);
+      }
+    }
+  };
+  if ((int)blockIdx.y > ny) {
+    normed(p, a.Rq, a.wq, q + (size_t)t * a.Rq);
+    return;
+  }
   const int slot = a.slots[t];
   if (slot < 0) return;                                  // the whole workgroup
   // one KV head: row = slot of the paged cache
   T* o = cache + (size_t)slot * a.D;
-  const PT* x = p + a.H * (a.d + a.r);
-  float f[NI][V];
-  float ss = 0.f;
-#pragma unroll
-  for (int n = 0; n < NI; ++n) {
-    const int c = (tid + 256 * n) * V;
-    if (c < a.R) {
-      ld_slabs<V>(x + c, a.S, a.slab, f[n]);
-#pragma unroll
-      for (int j = 0; j < V; ++j) ss += f[n][j] * f[n][j];
-    }
-  }
-  const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)a.R + a.eps);
-#pragma unroll
-  for (int n = 0; n < NI; ++n) {
-    const int c = (tid + 256 * n) * V;
-    if (c < a.R) {
-      float w[V];
-      ldv<V>(a.wn + c, w);
-#pragma unroll
-      for (int j = 0; j < V; ++j) f[n][j] *= inv * w[j];
-      stv<V>(o + c, f[n]);
-    }
-  }
+  const PT* x = p + a.H * (a.d + a.r) + a.Rq;
+  normed(x, a.R, a.wn, o);
   for (int i = tid; i < half / V; i += 256) rotate(x + a.R, o + a.R8, i * V);
   if (V == 1) {
     for (int i = tid; i < a.R8 - a.R; i += 256) st1(o + a.R + i, 0.f);
@@ -588,13 +599,13 @@ int dispatch_latent(const LatentArgs& a, int B, int max_q, hipStream_t s) {
 
 template <typename PT, typename T>
 int store_types(const void* P, void* q, void* cache, int T_, const StoreArgs& a, hipStream_t s) {
-  const bool v4 = a.d % 8 == 0 && a.r % 8 == 0 && a.R % 8 == 0 && a.ld % 4 == 0;
+  const bool v4 = a.d % 8 == 0 && a.r % 8 == 0 && a.R % 8 == 0 && a.Rq % 8 == 0 && a.ld % 4 == 0;
   // many tokens: 16-byte pieces of bf16 rows
   const bool v8 = v4 && T_ >= 256 && sizeof(T) == 2 && a.r % 16 == 0 && a.ld % 8 == 0;
   const int V = v8 ? 8 : v4 ? 4 : 1;
   const int per = a.d / V + a.r / 2 / V + (v4 ? 0 : a.d8 - a.d + a.r8 - a.r);
   const int ny = (a.H * per + 255) / 256;
-  dim3 grid(T_, ny + (a.wn ? 1 : 0));
+  dim3 grid(T_, ny + (a.wn ? 1 : 0) + (a.wq ? 1 : 0));
   if (v8) latent_store_kernel<8, 1, PT, T><<<grid, 256, 0, s>>>((const PT*)P, (T*)q, (T*)cache, ny, a);
   else if (v4) latent_store_kernel<4, 2, PT, T><<<grid, 256, 0, s>>>((const PT*)P, (T*)q, (T*)cache, ny, a);
   else latent_store_kernel<1, 8, PT, T><<<grid, 256, 0, s>>>((const PT*)P, (T*)q, (T*)cache, ny, a);
@@ -624,11 +635,24 @@ int docqa_latent_store(const void* P, int p_f32, int S, size_t slab, int ld, con
   if (S < 1 || H < 1 || d < 1 || r < 2 || r % 2 || R < 1 || R > 2048 || (BS & (BS - 1)) != 0) return -1;
   if (ld < H * (d + r) + (c_norm ? R + r : 0) || (f32 && !p_f32)) return -1;
   StoreArgs a{S, ld, slab, cs, slots, c_norm, H, d, r, R, (d + 7) / 8 * 8, (r + 7) / 8 * 8, (R + 7) / 8 * 8, 0,
-              log2_of(BS), eps};
+              log2_of(BS), eps, nullptr, 0};
   a.D = a.R8 + a.r8;
   if (f32) return store_types<float, float>(P, q, cache, T, a, s);
   return p_f32 ? store_types<float, uint16_t>(P, q, cache, T, a, s)
                : store_types<uint16_t, uint16_t>(P, q, cache, T, a, s);
+}
+
+int docqa_latent_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* cs, const int* slots,
+                            const float* q_norm, const float* c_norm, void* cq, void* cache, int f32, int T, int Rq, int r,
+                            int R, int BS, float eps, hipStream_t s) {
+  if (T == 0) return 0;
+  if (S < 1 || r < 2 || r % 2 || R < 1 || R > 2048 || Rq < 1 || Rq > 2048 || !q_norm || !c_norm || (BS & (BS - 1)) != 0) return -1;
+  if (ld < Rq + R + r || (f32 && !p_f32)) return -1;
+  StoreArgs a{S, ld, slab, cs, slots, c_norm, 0, 0, r, R, 0, (r + 7) / 8 * 8, (R + 7) / 8 * 8, 0, log2_of(BS), eps, q_norm, Rq};
+  a.D = a.R8 + a.r8;
+  if (f32) return store_types<float, float>(P, cq, cache, T, a, s);
+  return p_f32 ? store_types<float, uint16_t>(P, cq, cache, T, a, s)
+               : store_types<uint16_t, uint16_t>(P, cq, cache, T, a, s);
 }
 
 int docqa_head_project(const void* x, const void* part, const void* ml, int nsplit, const void* w, void* y, int T, int H,

@@ -1,8 +1,9 @@
 // linear_attn.hip -- linear-attention recurrences with one [dk, dv] matrix S a head:
-//   S_t = diag(a_t) S_{t-1} + k_t u_t^T,  o_t = S_t^T q_t,  y = rms(o) w silu(g)
+//   S_t = diag(a_t) S_{t-1} + k_t u_t^T,  o_t = S_t^T q_t,  y = rms(o) w silu(g)   (or sigmoid(g))
 //   channel: a = sigmoid(z)^(1/tau) per key channel, z = w1 . w2 + b of a low-rank projection; u = v
 //   fixed:   a constant per head; q, k rotated by position; u = v
 //   delta:   a = exp(A softplus(z + b)) per head; unit q, k; u = sigmoid(beta) (v - (a S_{t-1})^T k)
+//   channel delta: the delta rule with a per key channel, A per head
 // The state pool holds [slots, H, dk, dvp] fp32 (dvp: dv rounded up to 4, padding zero).  A sequence
 // whose first token is position 0 starts from zero whatever its slot held.
 //
@@ -17,9 +18,10 @@
 //          A[t, s] = q_t . k_s e^{b_t - b_s} (s <= t); delta: M[t, s] = beta_t e^{b_t - b_s} k_t . k_s
 //          (s < t) and, by forward substitution over blocks of 16 tokens with the diagonal blocks
 //          inverted ahead, U = (1 + M)^-1 beta v, W = (1 + M)^-1 beta e^{b_t} k.
-//          No exponent is positive: where decays differ by channel, a 16 x 16 block of A below the
-//          diagonal takes both factors relative to the last token ahead of its rows, one on the
-//          diagonal is summed directly.
+//          Where decays differ by channel, a 16 x 16 block of A (and M) below the diagonal takes both
+//          factors relative to the last token ahead of its rows, so no exponent is positive.  One on
+//          the diagonal takes them relative to its middle token while no channel decays by more than
+//          e^-kMaxDrop within the block, and is summed directly, exponent by exponent, otherwise.
 //   chunk  per (sequence, head, dv tile), chunk after chunk, S in accumulators:
 //          u = v or U - W S;  o = Q' S + A u;  S = e^{b_C} S + K'^T u
 //   gate   y = rms(o) w silu(g) per (token, head)
@@ -84,14 +86,19 @@ __global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const in
     sg[i] = i < dv ? ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.go + h * dv + i) : 0.f;
   }
   float qs = a.qs, ks = a.ks, beta = 1.f, al = 1.f;
+  const bool chan = a.kind == LIN_CHANNEL || a.kind == LIN_CHANNEL_DELTA, delta = a.kind >= LIN_DELTA;
   if (a.kind == LIN_CHANNEL) {
     for (int i = tid; i < a.rank; i += nt) sr[i] = ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.ao + i);
   } else if (a.kind == LIN_FIXED) {
     al = expf(a.w_gate[h]);
-  } else {
+  } else if (a.kind == LIN_DELTA) {
     al = expf(a.w_gate[h] * softplus_x(ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.ao + h) + a.b_gate[h]));
-    beta = sigmoid_f(ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.bo + h));
+  } else {
+    // (a thread's own i: it zeroed this element above)
+    for (int i = tid; i < dk; i += nt)
+      sa[i] = expf(a.w_gate[h] * softplus_x(ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.ao + h * dk + i) + a.b_gate[h * dk + i]));
   }
+  if (delta) beta = sigmoid_f(ldx1(a.Z, a.zf32, a.Sz, a.zslab, zr + a.bo + h));
   __syncthreads();
   if (a.kind == LIN_CHANNEL) {
     for (int i = tid; i < dk; i += nt) {
@@ -111,7 +118,7 @@ __global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const in
       s[i + r2] = y * c + x * si;
     }
     __syncthreads();
-  } else if (a.kind == LIN_DELTA) {
+  } else if (delta) {
     float nq = 0.f, nk = 0.f;
     for (int i = lane; i < dk; i += 64) {
       nq += sq[i] * sq[i];
@@ -132,11 +139,11 @@ __global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const in
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
     const int r = i * RG + rg;
-    const float d = a.kind == LIN_CHANNEL ? sa[r] : al, k = sk[r] * ks;
+    const float d = chan ? sa[r] : al, k = sk[r] * ks;
     S[i].x *= d; S[i].y *= d; S[i].z *= d; S[i].w *= d;
     p[0] += S[i].x * k; p[1] += S[i].y * k; p[2] += S[i].z * k; p[3] += S[i].w * k;
   }
-  if (a.kind == LIN_DELTA) {
+  if (delta) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) v[j] = beta * (v[j] - rows_sum(p[j]));
   }
@@ -166,7 +173,7 @@ __global__ __launch_bounds__(MT) void linear_step_kernel(DocqaLinear a, const in
     for (int j = 0; j < 4; ++j)
       if (c0 + j < dv) {
         const float g = sg[c0 + j];
-        stx(a.out, a.of32, (size_t)b * a.ldo + h * dv + c0 + j, o[j] * inv * a.norm[c0 + j] * g * sigmoid_f(g));
+        stx(a.out, a.of32, (size_t)b * a.ldo + h * dv + c0 + j, o[j] * inv * a.norm[c0 + j] * (a.sig ? 1.f : g) * sigmoid_f(g));
       }
   }
 }
@@ -187,6 +194,7 @@ __device__ __forceinline__ void wave_lds_sync() {
   __builtin_amdgcn_wave_barrier();
 }
 
+constexpr float kMaxDrop = 30.f;
 constexpr int NTP = 512, NWP = NTP / 64, PT = 20;
 constexpr int prep_q(int C, int DKP, bool delta) { return delta && NWP * C * PT > C * (DKP + 4) ? NWP * C * PT : C * (DKP + 4); }
 // pitch of the low-rank inputs: the rank in whole MFMA steps
@@ -194,7 +202,8 @@ __host__ __device__ __forceinline__ int rank_pitch(int rank) { return ((rank + 1
 template <int C, int DKP, int KIND, int V>
 __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
   constexpr int PK = DKP + 4, NB = C / 16, PM = C + 4;
-  constexpr bool CH = KIND == LIN_CHANNEL, DELTA = KIND == LIN_DELTA;
+  constexpr bool CH = KIND == LIN_CHANNEL || KIND == LIN_CHANNEL_DELTA, DELTA = KIND >= LIN_DELTA;
+  __shared__ int s_direct[NB];                               // diagonal blocks to be summed directly
   extern __shared__ __attribute__((aligned(16))) float lds[];
   // delta: sQ's place later holds the waves' parts of the solution, [NWP, C, PT]
   float *sQ = lds, *sK = sQ + prep_q(C, DKP, DELTA), *sB = sK + C * PK;   // sB: [C, PK] (channel) or [C] log decays, summed
@@ -223,7 +232,26 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
       sK[t * PK + d + j] = k[j];
     }
   }
-  if constexpr (CH) {
+  if (DELTA && wave == 1) {
+    if (lane < C) sbeta[lane] = lane < n ? sigmoid_f(ldx1(a.Z, a.zf32, a.Sz, a.zslab, (row0 + lane) * a.ldz + a.bo + h)) : 0.f;
+  }
+  if constexpr (KIND == LIN_CHANNEL_DELTA) {
+    const float A = a.w_gate[h];
+    for (int e = tid; e < C * (DKP / V); e += NTP) {
+      const int t = e / (DKP / V), d = (e % (DKP / V)) * V;
+      float z[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) z[j] = 0.f;
+      if (t < n && d < dk) {
+        float bias[V];
+        ldx<V>(a.Z, a.zf32, a.Sz, a.zslab, (row0 + t) * a.ldz + a.ao + h * dk + d, z);
+        ldv<V>(a.b_gate + h * dk + d, bias);
+#pragma unroll
+        for (int j = 0; j < V; ++j) z[j] = A * softplus_x(z[j] + bias[j]);
+      }
+      stv<V>(sB + t * PK + d, z);
+    }
+  } else if constexpr (CH) {
     const int rp = rank_pitch(a.rank);
     for (int e = tid; e < C * rp; e += NTP) {
       const int t = e / rp, r = e % rp;
@@ -241,8 +269,6 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
       if (lane >= o) la += u;
     }
     if (lane < C) sB[lane] = la;
-  } else if (DELTA && wave == 1) {
-    if (lane < C) sbeta[lane] = lane < n ? sigmoid_f(ldx1(a.Z, a.zf32, a.Sz, a.zslab, (row0 + lane) * a.ldz + a.bo + h)) : 0.f;
   }
   __syncthreads();
 
@@ -274,7 +300,7 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
       sK[t * PK + d] *= ks;
     }
   }
-  if constexpr (CH) {
+  if constexpr (KIND == LIN_CHANNEL) {
     // log decays: z of 16 tokens x 16 channels a wave
     const int fr = lane & 15, g4 = lane >> 4, rp = rank_pitch(a.rank);
     for (int it = wave; it < NB * (DKP / 16); it += NWP) {
@@ -298,6 +324,8 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
       }
     }
     __syncthreads();
+  }
+  if constexpr (CH) {
     // their sums: a thread a channel and a stretch of tokens
     constexpr int NS = NTP / DKP >= 4 ? 4 : NTP / DKP >= 2 ? 2 : 1, TS = C / NS;
     for (int e = tid; e < DKP * NS; e += NTP) {
@@ -330,24 +358,34 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
   int item = 0;
   for (int i = 0; i < NB; ++i)
     for (int j = 0; j <= i; ++j) {
-      if (CH && i == j) continue;
       if (item++ % NWP != wave) continue;
+      if (CH && i == j) {
+        float drop = 0.f;
+        for (int d = lane; d < DKP; d += 64) drop = fmaxf(drop, sB[i * 16 * PK + d] - sB[(i * 16 + 15) * PK + d]);
+        drop = wave_max(drop);
+        if (lane == 0) s_direct[i] = drop > kMaxDrop;
+        if (drop > kMaxDrop) continue;
+      }
       f32x4 qa = f32x4{0.f, 0.f, 0.f, 0.f}, ka = qa;
-      const int tr = i * 16 + fr, sr = j * 16 + fr, ref = i * 16 - 1;
+      const int tr = i * 16 + fr, sr = j * 16 + fr, ref = i == j ? i * 16 + 7 : i * 16 - 1;
 #pragma unroll 4
       for (int k0 = 0; k0 < DKP; k0 += 16) {
         const int k = k0 + 4 * g4;
         float4 q = *reinterpret_cast<const float4*>(sQ + tr * PK + k);
-        float4 ks = *reinterpret_cast<const float4*>(sK + sr * PK + k);
+        float4 ks = *reinterpret_cast<const float4*>(sK + sr * PK + k), kt;
+        if constexpr (DELTA) kt = *reinterpret_cast<const float4*>(sK + tr * PK + k);
         if constexpr (CH) {
           const float4 bt = *reinterpret_cast<const float4*>(sB + tr * PK + k), bs = *reinterpret_cast<const float4*>(sB + sr * PK + k);
           const float4 br = *reinterpret_cast<const float4*>(sB + ref * PK + k);
-          q.x *= __expf(bt.x - br.x); q.y *= __expf(bt.y - br.y); q.z *= __expf(bt.z - br.z); q.w *= __expf(bt.w - br.w);
+          const float4 f = make_float4(__expf(bt.x - br.x), __expf(bt.y - br.y), __expf(bt.z - br.z), __expf(bt.w - br.w));
+          q.x *= f.x; q.y *= f.y; q.z *= f.z; q.w *= f.w;
+          if constexpr (DELTA) {
+            kt.x *= f.x; kt.y *= f.y; kt.z *= f.z; kt.w *= f.w;
+          }
           ks.x *= __expf(br.x - bs.x); ks.y *= __expf(br.y - bs.y); ks.z *= __expf(br.z - bs.z); ks.w *= __expf(br.w - bs.w);
         }
         qa = mfma(q.x, ks.x, qa); qa = mfma(q.y, ks.y, qa); qa = mfma(q.z, ks.z, qa); qa = mfma(q.w, ks.w, qa);
         if constexpr (DELTA) {
-          const float4 kt = *reinterpret_cast<const float4*>(sK + tr * PK + k);
           ka = mfma(kt.x, ks.x, ka); ka = mfma(kt.y, ks.y, ka); ka = mfma(kt.z, ks.z, ka); ka = mfma(kt.w, ks.w, ka);
         }
       }
@@ -361,19 +399,27 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
       }
     }
   if constexpr (CH) {
+    __syncthreads();
     const int t16 = (tid >> 4) & 15, s16 = tid & 15;
     for (int i = tid >> 8; i < NB; i += NTP / 256) {
+      if (!s_direct[i]) continue;
       const int t = i * 16 + t16, s = i * 16 + s16;
-      float acc = 0.f;
+      float acc = 0.f, kk = 0.f;
       if (s <= t) {
         for (int d = 0; d < DKP; d += 4) {
-          const float4 q = *reinterpret_cast<const float4*>(sQ + t * PK + d), k = *reinterpret_cast<const float4*>(sK + s * PK + d);
+          const float4 q = *reinterpret_cast<const float4*>(sQ + t * PK + d);
+          float4 k = *reinterpret_cast<const float4*>(sK + s * PK + d);
           const float4 bt = *reinterpret_cast<const float4*>(sB + t * PK + d), bs = *reinterpret_cast<const float4*>(sB + s * PK + d);
-          acc += q.x * k.x * __expf(bt.x - bs.x) + q.y * k.y * __expf(bt.y - bs.y) + q.z * k.z * __expf(bt.z - bs.z) +
-                 q.w * k.w * __expf(bt.w - bs.w);
+          k.x *= __expf(bt.x - bs.x); k.y *= __expf(bt.y - bs.y); k.z *= __expf(bt.z - bs.z); k.w *= __expf(bt.w - bs.w);
+          acc += q.x * k.x + q.y * k.y + q.z * k.z + q.w * k.w;
+          if constexpr (DELTA) {
+            const float4 kt = *reinterpret_cast<const float4*>(sK + t * PK + d);
+            kk += kt.x * k.x + kt.y * k.y + kt.z * k.z + kt.w * k.w;
+          }
         }
       }
       gA[t * C + s] = acc;
+      if constexpr (DELTA) sM[t * PM + s] = s < t ? sbeta[t] * kk : 0.f;
     }
   }
   if constexpr (DELTA) __syncthreads();
@@ -451,7 +497,7 @@ __global__ __launch_bounds__(NTP) void linear_prep_kernel(ScanArgs sc) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int t = i * 16 + 4 * g4 + r;
-          y[i][r] = sbeta[t] * (val ? (t < n && c < dv ? y[i][r] : 0.f) : expf(sB[t]) * sK[t * PK + c]);
+          y[i][r] = sbeta[t] * (val ? (t < n && c < dv ? y[i][r] : 0.f) : expf(sB[CH ? t * PK + c : t]) * sK[t * PK + c]);
         }
 #pragma unroll
       for (int i = 0; i < NB; ++i) {
@@ -670,7 +716,7 @@ __global__ __launch_bounds__(256) void linear_gate_kernel(DocqaLinear a, const f
     ldx<V>(a.Z, a.zf32, a.Sz, a.zslab, (size_t)t * a.ldz + a.go + h * dv + c, g);
     ldv<V>(a.norm + c, w);
 #pragma unroll
-    for (int j = 0; j < V; ++j) g[j] = x[i][j] * inv * w[j] * g[j] * sigmoid_f(g[j]);
+    for (int j = 0; j < V; ++j) g[j] = x[i][j] * inv * w[j] * (a.sig ? 1.f : g[j]) * sigmoid_f(g[j]);
     const size_t at = (size_t)t * a.ldo + h * dv + c;
     if (a.of32) stv<V>((float*)a.out + at, g);
     else stv<V>((uint16_t*)a.out + at, g);
@@ -686,11 +732,13 @@ void launch_gate(const DocqaLinear& a, const float* O, int tokens, hipStream_t s
 template <int C, int DKP, int KIND>
 int launch_scan(const ScanArgs& sc, int tokens, int B, hipStream_t s) {
   constexpr int PK = DKP + 4;
+  constexpr bool CH = KIND == LIN_CHANNEL || KIND == LIN_CHANNEL_DELTA, DELTA = KIND >= LIN_DELTA;
   const DocqaLinear& a = sc.a;
-  const size_t low = KIND == LIN_CHANNEL ? (size_t)C * rank_pitch(a.rank) : KIND == LIN_DELTA ? (size_t)C * (C + 4 + PT + 1) : 0;
-  const size_t lds = (prep_q(C, DKP, KIND == LIN_DELTA) + C * PK + (KIND == LIN_CHANNEL ? C * PK : C) + low) * 4;
-  if (lds > 160 * 1024) return -1;
-  const bool vec = docqa_aligned16(a.X) && a.dk % 4 == 0 && a.qo % 4 == 0 && a.ko % 4 == 0 && a.ldx % 4 == 0 && a.dv % 4 == 0 &&
+  const size_t low = KIND == LIN_CHANNEL ? (size_t)C * rank_pitch(a.rank) : DELTA ? (size_t)C * (C + 4 + PT + 1) : 0;
+  const size_t lds = (prep_q(C, DKP, DELTA) + C * PK + (CH ? C * PK : C) + low) * 4;
+  if (lds > 160 * 1024 - 64) return -1;
+  const bool vec = (KIND != LIN_CHANNEL_DELTA || (docqa_aligned16(a.Z) && docqa_aligned16(a.b_gate) && a.ao % 4 == 0 && a.ldz % 4 == 0)) &&
+                   docqa_aligned16(a.X) && a.dk % 4 == 0 && a.qo % 4 == 0 && a.ko % 4 == 0 && a.ldx % 4 == 0 && a.dv % 4 == 0 &&
                    a.vo % 4 == 0;
   dim3 grid(a.H, sc.nchunk, B);
   auto prep = vec ? linear_prep_kernel<C, DKP, KIND, 4> : linear_prep_kernel<C, DKP, KIND, 1>;
@@ -703,8 +751,8 @@ int launch_scan(const ScanArgs& sc, int tokens, int B, hipStream_t s) {
   const int dvq = (a.dv + 15) & ~15;
   const long long one = (long long)B * a.H * (dvq / 16);
   // narrow tiles while they leave CUs without a workgroup
-  if (one <= 512 || dvq == 16) linear_chunk_kernel<C, DKP, 1, KIND == LIN_DELTA><<<(unsigned)one, 256, 0, s>>>(sc);
-  else linear_chunk_kernel<C, DKP, 2, KIND == LIN_DELTA><<<(unsigned)((long long)B * a.H * ((dvq + 31) / 32)), 256, 0, s>>>(sc);
+  if (one <= 512 || dvq == 16) linear_chunk_kernel<C, DKP, 1, DELTA><<<(unsigned)one, 256, 0, s>>>(sc);
+  else linear_chunk_kernel<C, DKP, 2, DELTA><<<(unsigned)((long long)B * a.H * ((dvq + 31) / 32)), 256, 0, s>>>(sc);
   DOCQA_CHECK_LAUNCH();
   const bool v4 = a.dv % 4 == 0 && a.go % 4 == 0 && a.ldz % 4 == 0 && a.ldo % 4 == 0 && docqa_aligned16(a.Z) &&
                   docqa_aligned16(a.out) && docqa_aligned16(a.norm);
@@ -761,7 +809,7 @@ struct Sizes {
 Sizes scratch_sizes(int kind, int tokens, int B, int H, int dk, int dv) {
   const size_t C = docqa_linear_chunk(dk), dkp = dk_pad(dk), dvq = (dv + 15) & ~15;
   const size_t n = (tokens / C + B + 1) * H;          // chunk ids are below tokens / C + B
-  const bool delta = kind == LIN_DELTA;
+  const bool delta = kind >= LIN_DELTA;
   Sizes z{n * C * dkp, n * C * C, n * dkp, delta ? n * C * dkp : 0, n * C * dvq, (size_t)tokens * H * dvq, 0};
   z.total = 2 * z.Q + z.A + z.G + z.W + z.U + z.O;
   return z;
@@ -783,5 +831,116 @@ int docqa_linear_scan(const DocqaLinear& a, const int* cu, const int* ctx, float
   sc.Q = scratch; sc.K = sc.Q + z.Q; sc.A = sc.K + z.Q; sc.W = sc.A + z.A; sc.U = sc.W + z.W; sc.O = sc.U + z.U; sc.G = sc.O + z.O;
   if (a.kind == LIN_CHANNEL) return dispatch_scan<LIN_CHANNEL>(sc, tokens, B, s);
   if (a.kind == LIN_FIXED) return dispatch_scan<LIN_FIXED>(sc, tokens, B, s);
-  return dispatch_scan<LIN_DELTA>(sc, tokens, B, s);
+  if (a.kind == LIN_DELTA) return dispatch_scan<LIN_DELTA>(sc, tokens, B, s);
+  return dispatch_scan<LIN_CHANNEL_DELTA>(sc, tokens, B, s);
+}
+
+// ------------------------------------------------------------------ projections through few elements
+namespace {
+struct LowRank {
+  const uint16_t* z;              // [T, ldz]: columns [Ka | Kg | n] from `at` on
+  int ldz, at;
+  const uint16_t *wa, *wg;        // [Na, Ka], [Ng, Kg]
+  int Na, Ka, Ng, Kg, n;
+  float* y;                       // [T, Na + Ng + n]
+  int T;
+};
+// 16 MT rows x 64 NJ outputs of one of the two products, rows staged in LDS; the first workgroup of a
+// row tile carries the other columns
+template <int MT, int NJ>
+__global__ __launch_bounds__(256) void low_rank_kernel(LowRank a) {
+  extern __shared__ __attribute__((aligned(16))) uint16_t sx[];       // [16 MT][pitch]
+  const int ta = (a.Na + 64 * NJ - 1) / (64 * NJ);
+  const bool gate = (int)blockIdx.x >= ta;
+  const int K = gate ? a.Kg : a.Ka, N = gate ? a.Ng : a.Na, off = gate ? a.Ka : 0, yo = gate ? a.Na : 0, ldy = a.Na + a.Ng + a.n;
+  const int kp = (K + 31) / 32 * 32, pitch = kp + 8, m0 = blockIdx.y * 16 * MT, tid = threadIdx.x;
+  const uint16_t *x = a.z + a.at + off, *w = gate ? a.wg : a.wa;
+  const bool vec = ((reinterpret_cast<uintptr_t>(x) | (size_t)a.ldz * 2) & 15) == 0;
+  const int per = kp / 8;
+  for (int i = tid; i < 16 * MT * per; i += 256) {
+    const int r = i / per, c = (i - r * per) * 8;
+    union {
+      uint4 v;
+      uint16_t e[8];
+    } u;
+    u.v = make_uint4(0, 0, 0, 0);
+    if (m0 + r < a.T && c < K) {
+      const uint16_t* p = x + (size_t)(m0 + r) * a.ldz + c;
+      if (vec) u.v = *reinterpret_cast<const uint4*>(p);
+      else
+#pragma unroll
+        for (int j = 0; j < 8; ++j) u.e[j] = p[j];
+    }
+    *reinterpret_cast<uint4*>(sx + r * pitch + c) = u.v;
+  }
+  if (blockIdx.x == 0)
+    for (int i = tid; i < 16 * MT * a.n; i += 256) {
+      const int r = i / a.n, c = i - r * a.n;
+      if (m0 + r < a.T) a.y[(size_t)(m0 + r) * ldy + a.Na + a.Ng + c] = bf2f(a.z[(size_t)(m0 + r) * a.ldz + a.at + a.Ka + a.Kg + c]);
+    }
+  __syncthreads();
+  const int lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
+  const int n0 = (((int)blockIdx.x - (gate ? ta : 0)) * 4 + wave) * 16 * NJ;
+  if (n0 >= N) return;
+  f32x4 acc[MT][NJ];
+#pragma unroll
+  for (int i = 0; i < MT; ++i)
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k = 0; k < kp; k += 32) {
+    const int kk = k + g4 * 8;
+    bf16x8 wf[NJ], xf[MT];
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+      const int n = n0 + 16 * j + fr;
+      uint4 v = make_uint4(0, 0, 0, 0);
+      if (n < N && kk < K) v = *reinterpret_cast<const uint4*>(w + (size_t)n * K + kk);
+      wf[j] = *reinterpret_cast<bf16x8*>(&v);
+    }
+#pragma unroll
+    for (int i = 0; i < MT; ++i) xf[i] = *reinterpret_cast<const bf16x8*>(sx + (i * 16 + fr) * pitch + kk);
+#pragma unroll
+    for (int i = 0; i < MT; ++i)
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[j], xf[i], acc[i][j], 0, 0, 0);
+  }
+  const bool v4 = ((ldy | N | yo) & 3) == 0;
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const int row = m0 + i * 16 + fr;
+    if (row >= a.T) continue;
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+      const int n = n0 + 16 * j + g4 * 4;
+      float* o = a.y + (size_t)row * ldy + yo + n;
+      const float f[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
+      if (v4) {
+        if (n < N) stv<4>(o, f);
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (n + r < N) o[r] = f[r];
+      }
+    }
+  }
+}
+}  // namespace
+
+int docqa_low_rank(const void* z, int ldz, int at, const void* wa, int Na, int Ka, const void* wg, int Ng, int Kg, int n,
+                   float* y, int T, hipStream_t s) {
+  if (T == 0) return 0;
+  if (Na < 1 || Ng < 1 || n < 0 || Ka < 8 || Ka % 8 || Kg < 8 || Kg % 8 || Ka > 1024 || Kg > 1024 || at < 0 || at + Ka + Kg + n > ldz)
+    return -1;
+  if (!docqa_aligned16(wa) || !docqa_aligned16(wg) || !docqa_aligned16(y)) return -1;
+  const LowRank a{(const uint16_t*)z, ldz, at, (const uint16_t*)wa, (const uint16_t*)wg, Na, Ka, Ng, Kg, n, y, T};
+  const int K = Ka > Kg ? Ka : Kg, pitch = (K + 31) / 32 * 32 + 8;
+#define GO(MT, NJ)                                                                                                          \
+  low_rank_kernel<MT, NJ><<<dim3((Na + 64 * NJ - 1) / (64 * NJ) + (Ng + 64 * NJ - 1) / (64 * NJ), (T + 16 * MT - 1) / (16 * MT)), \
+                            256, (size_t)16 * MT * pitch * 2, s>>>(a)
+  if (T > 64 && K <= 256) GO(4, 2);
+  else GO(1, 1);
+#undef GO
+  DOCQA_CHECK_LAUNCH();
+  return 0;
 }

@@ -1,8 +1,11 @@
 // moe.hip -- routed experts: E SwiGLU feed-forwards, `top` of them a token, each reading the token
-// times its score:  y_k[t] = down_e (silu(s g) * (s u)),  g = gate_e x_t, u = up_e x_t, e = ids[t, k]
+// times its score:  y_k[t] = down_e (silu(s g) * (s u)),  g = gate_e x_t, u = up_e x_t, e = ids[t, k];
+// or, clamped, the token itself:  down_e (g sigmoid(1.702 g) (u + 1)),  g from above, u on both sides.
+// Ids from E on have no expert: their pairs are left out.
 //
 // * route: scores sigmoid(x w^T) in fp32 (bf16 operands: MFMA, K split over 16 waves), the largest
-//   `top` of the first E, and the scores of the remaining columns.
+//   `top` of the first E, and the scores of the remaining columns.  Groups: softmax scores, the largest
+//   by score + correction within the best groups, weights normed over the chosen.
 // * a (token, choice) pair p = t top + k is a row of the grouped products; gate and up rows meet in
 //   the same lane's accumulators, so the activation is the first product's epilogue.
 //   Few pairs (decode): a workgroup takes one expert and 16 (or 32) output columns, finds the expert's
@@ -21,7 +24,12 @@ constexpr int kSkinnyPairs = 512;       // pairs up to which a launch finds its 
 constexpr int BM = 128, BK = 64, kGroup = 8;
 
 __device__ __forceinline__ float sigmoid_x(float x) { return 1.f / (1.f + expf(-x)); }
-__device__ __forceinline__ float glu_f(float g, float u, float s) {
+__device__ __forceinline__ float glu_f(float g, float u, float s, float limit) {
+  if (limit > 0.f) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.f + __expf(-1.702f * g)) * (u + 1.f);
+  }
   g *= s;
   return g / (1.f + __expf(-g)) * (u * s);
 }
@@ -53,11 +61,96 @@ __device__ __forceinline__ void pick(const float* sc, int E, int top, int* ids, 
   }
 }
 
+struct RouteArgs {
+  int* ids;
+  float *wts, *rest;       // rest: scores of columns [E, N)
+  int K, N, E, top;
+  const float* corr;       // groups: [N]
+  int groups, keep;
+  float scale;
+};
+
+// between a wave's own writes to LDS and its reads of other lanes' parts
+__device__ __forceinline__ void wave_lds_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+
+// one wave's token: logits sc[0, N) (N <= 512) -> choice; sc[N, 2 N) is scratch
+__device__ __forceinline__ void pick_groups(float* sc, const RouteArgs& a, int* ids, float* wts) {
+  const int lane = threadIdx.x & 63, N = a.N, gs = N / a.groups;
+  float s[8], c[8], m = -INFINITY, sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    s[i] = lane + 64 * i < N ? sc[lane + 64 * i] : -INFINITY;
+    m = fmaxf(m, s[i]);
+  }
+  m = wave_max(m);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    s[i] = expf(s[i] - m);
+    sum += s[i];
+  }
+  sum = 1.f / wave_sum(sum);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int n = lane + 64 * i;
+    s[i] *= sum;
+    c[i] = n < N ? s[i] + a.corr[n] : -INFINITY;
+  }
+  if (a.keep < a.groups) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      if (lane + 64 * i < N) sc[lane + 64 * i] = c[i];
+    wave_lds_sync();
+    float* best = sc + N;                     // a group's largest choice score
+    for (int g = lane; g < a.groups; g += 64) {
+      float b = sc[g * gs];
+      for (int j = 1; j < gs; ++j) b = fmaxf(b, sc[g * gs + j]);
+      best[g] = b;
+    }
+    wave_lds_sync();
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int n = lane + 64 * i;
+      if (n >= N) continue;
+      const int g = n / gs;
+      const float b = best[g];
+      int ahead = 0;
+      for (int h = 0; h < a.groups; ++h) ahead += best[h] > b || (best[h] == b && h < g);
+      if (ahead >= a.keep) c[i] = -INFINITY;
+    }
+  }
+  float own = 0.f, total = 0.f;
+  int id = 0;
+  for (int k = 0; k < a.top; ++k) {
+    float b = -INFINITY, w = 0.f;
+    int at = 1 << 30;
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      if (c[i] > b) b = c[i], at = lane + 64 * i;
+    int idx = b == wave_max(b) ? at : 1 << 30;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) idx = min(idx, __shfl_xor(idx, o, 64));
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      if (lane + 64 * i == idx) w = s[i], c[i] = -INFINITY;
+    w = wave_sum(w);
+    total += w;
+    if (lane == k) own = w, id = min(idx, N - 1);
+  }
+  if (lane < a.top) {
+    ids[lane] = id;
+    wts[lane] = own / (total + 1e-20f) * a.scale;
+  }
+}
+
 // 16 tokens a workgroup of 16 waves that split K, 32 columns a pass; x [T, K], w [N, K], K % 32 == 0
+template <bool GROUPS>
 __global__ __launch_bounds__(1024) void moe_route_mfma_kernel(const uint16_t* __restrict__ x, const uint16_t* __restrict__ w,
-                                                              int* __restrict__ ids, float* __restrict__ wts,
-                                                              float* __restrict__ rest, int T, int K, int N, int E, int top) {
-  extern __shared__ float sc[];              // [16][N] scores
+                                                              RouteArgs a, int T) {
+  extern __shared__ float sc[];              // [16][N] scores (groups: [16][2 N])
+  const int K = a.K, N = a.N, E = a.E, top = a.top, ld = GROUPS ? 2 * N : N;
   __shared__ float red[16][2][16][17];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, g4 = lane >> 4;
   const int t0 = blockIdx.x * 16;
@@ -82,44 +175,51 @@ __global__ __launch_bounds__(1024) void moe_route_mfma_kernel(const uint16_t* __
       float z = 0.f;
 #pragma unroll
       for (int i = 0; i < 16; ++i) z += red[i][c >> 4][t][c & 15];
-      if (n0 + c < N) sc[t * N + n0 + c] = sigmoid_x(z);
+      if (n0 + c < N) sc[t * ld + n0 + c] = GROUPS ? z : sigmoid_x(z);
     }
     __syncthreads();
   }
   if (t0 + wave < T) {
     const size_t t = t0 + wave;
-    pick(sc + wave * N, E, top, ids + t * top, wts + t * top);
-    for (int c = E + lane; c < N; c += 64) rest[t * (N - E) + c - E] = sc[wave * N + c];
+    if constexpr (GROUPS) {
+      pick_groups(sc + wave * ld, a, a.ids + t * top, a.wts + t * top);
+    } else {
+      pick(sc + wave * N, E, top, a.ids + t * top, a.wts + t * top);
+      for (int c = E + lane; c < N; c += 64) a.rest[t * (N - E) + c - E] = sc[wave * N + c];
+    }
   }
 }
 
 // any size and element type: a workgroup a token, a wave a score at a time
-template <typename T>
-__global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x, const T* __restrict__ w, int* __restrict__ ids,
-                                                        float* __restrict__ wts, float* __restrict__ rest, int K, int N,
-                                                        int E, int top) {
-  extern __shared__ float sc[];              // [N]
+template <typename T, bool GROUPS>
+__global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x, const T* __restrict__ w, RouteArgs a) {
+  extern __shared__ float sc[];              // [N] (groups: [2 N])
+  const int K = a.K, N = a.N, E = a.E, top = a.top;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const size_t t = blockIdx.x;
   for (int n = wave; n < N; n += 4) {
     float z = 0.f;
     for (int k = lane; k < K; k += 64) z += ld1(x + t * K + k) * ld1(w + (size_t)n * K + k);
     z = wave_sum(z);
-    if (lane == 0) sc[n] = sigmoid_x(z);
+    if (lane == 0) sc[n] = GROUPS ? z : sigmoid_x(z);
   }
   __syncthreads();
-  if (wave == 0) pick(sc, E, top, ids + t * top, wts + t * top);
-  for (int c = E + threadIdx.x; c < N; c += 256) rest[t * (N - E) + c - E] = sc[c];
+  if constexpr (GROUPS) {
+    if (wave == 0) pick_groups(sc, a, a.ids + t * top, a.wts + t * top);
+  } else {
+    if (wave == 0) pick(sc, E, top, a.ids + t * top, a.wts + t * top);
+    for (int c = E + threadIdx.x; c < N; c += 256) a.rest[t * (N - E) + c - E] = sc[c];
+  }
 }
 
 // ------------------------------------------------------------------ any size: a wave an element
 template <typename T, bool UP>
 __global__ __launch_bounds__(256) void moe_plain_kernel(const T* __restrict__ x, const int* __restrict__ ids,
                                                         const float* __restrict__ wts, const T* __restrict__ w, T* __restrict__ y,
-                                                        int Tn, int top, int K, int N) {
+                                                        int Tn, int top, int E, int K, int N, float limit) {
   const int n = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   const size_t p = blockIdx.y + (size_t)blockIdx.z * 65535;
-  if (n >= N || p >= (size_t)Tn * top) return;
+  if (n >= N || p >= (size_t)Tn * top || ids[p] >= E) return;
   const T* xp = x + (UP ? p / top : p) * K;
   const T* wp = w + ((size_t)ids[p] * (UP ? 2 : 1) * N + n) * K;
   float a = 0.f, b = 0.f;
@@ -131,7 +231,7 @@ __global__ __launch_bounds__(256) void moe_plain_kernel(const T* __restrict__ x,
   a = wave_sum(a);
   if constexpr (UP) b = wave_sum(b);
   if (lane) return;
-  if constexpr (UP) st1(y + p * N + n, glu_f(a, b, wts[p]));
+  if constexpr (UP) st1(y + p * N + n, glu_f(a, b, wts[p], limit));
   else st1(y + ((p % top) * Tn + p / top) * N + n, a);
 }
 
@@ -141,7 +241,8 @@ __global__ __launch_bounds__(256) void moe_plain_kernel(const T* __restrict__ x,
 template <int MT, int NW, bool UP>
 __global__ __launch_bounds__(64 * NW) void moe_skinny_kernel(const uint16_t* __restrict__ x, const int* __restrict__ ids,
                                                          const float* __restrict__ wts, const uint16_t* __restrict__ w,
-                                                         uint16_t* __restrict__ y, int Tn, int top, int E, int K, int N) {
+                                                         uint16_t* __restrict__ y, int Tn, int top, int E, int K, int N,
+                                                         float limit) {
   __shared__ int rows[kSkinnyPairs];
   __shared__ int count;
   __shared__ float red[NW][MT][2][16][17];
@@ -151,6 +252,7 @@ __global__ __launch_bounds__(64 * NW) void moe_skinny_kernel(const uint16_t* __r
   if (E > P) {
     const int p = e;
     e = ids[p];
+    if (e >= E) return;
     for (int i = 0; i < p; ++i)
       if (ids[i] == e) return;
   }
@@ -202,7 +304,7 @@ __global__ __launch_bounds__(64 * NW) void moe_skinny_kernel(const uint16_t* __r
         b += red[q][i][1][r][c];
       }
       if constexpr (UP) {
-        if (n0 + c < N) y[(size_t)p * N + n0 + c] = f2bf(glu_f(a, b, wts[p]));
+        if (n0 + c < N) y[(size_t)p * N + n0 + c] = f2bf(glu_f(a, b, wts[p], limit));
       } else {
         uint16_t* o = y + ((size_t)(p % top) * Tn + p / top) * N + n0;
         if (n0 + c < N) o[c] = f2bf(a);
@@ -220,7 +322,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
   const int tid = threadIdx.x;
   for (int i = tid; i < E; i += 1024) cnt[i] = 0;
   __syncthreads();
-  for (int p = tid; p < P; p += 1024) atomicAdd(&cnt[ids[p]], 1);
+  for (int p = tid; p < P; p += 1024)
+    if (ids[p] < E) atomicAdd(&cnt[ids[p]], 1);
   __syncthreads();
   int *te = scratch + P, *tb = te + tiles, *tn = tb + tiles;
   if (tid == 0) {
@@ -245,7 +348,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
   __syncthreads();
   for (int i = tid; i < E; i += 1024) cnt[i] = start[i];
   __syncthreads();
-  for (int p = tid; p < P; p += 1024) scratch[atomicAdd(&cnt[ids[p]], 1)] = p;
+  for (int p = tid; p < P; p += 1024)
+    if (ids[p] < E) scratch[atomicAdd(&cnt[ids[p]], 1)] = p;
 }
 
 __device__ __forceinline__ int sw_off(int row, int ch) { return row * BK + ((ch ^ ((row >> 1) & 7)) << 3); }
@@ -255,7 +359,8 @@ __device__ __forceinline__ int sw_off(int row, int ch) { return row * BK + ((ch 
 template <bool UP>
 __global__ __launch_bounds__(256) void moe_gemm_kernel(const uint16_t* __restrict__ x, const float* __restrict__ wts,
                                                        const uint16_t* __restrict__ w, uint16_t* __restrict__ y,
-                                                       const int* __restrict__ scratch, int Tn, int top, int K, int N, int tiles) {
+                                                       const int* __restrict__ scratch, int Tn, int top, int K, int N, int tiles,
+                                                       float limit) {
   __shared__ __attribute__((aligned(16))) uint16_t smem[4 * 64 * 65 * 2];
   __shared__ int srow[BM];
   const int nbn = (N + (UP ? 63 : 127)) / (UP ? 64 : 128);
@@ -340,7 +445,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const uint16_t* __restric
       if constexpr (UP) {
         const float s = wts[srow[wr * 64 + row]];
 #pragma unroll
-        for (int j = 0; j < 2; ++j) st[row * 65 + j * 16 + fr] = glu_f(acc[i][j][r], acc[i][2 + j][r], s);
+        for (int j = 0; j < 2; ++j) st[row * 65 + j * 16 + fr] = glu_f(acc[i][j][r], acc[i][2 + j][r], s, limit);
       } else {
 #pragma unroll
         for (int j = 0; j < 4; ++j) st[row * 65 + j * 16 + fr] = acc[i][j][r];
@@ -367,24 +472,37 @@ int tile_count(int P, int E) { return P / BM + E; }
 
 template <typename T>
 int plain(const void* x, const int* ids, const float* wts, const void* up, const void* down, void* act, void* out, int Tn, int top,
-          int K, int F, int W, hipStream_t s) {
+          int E, int K, int F, int W, float limit, hipStream_t s) {
   const long long P = (long long)Tn * top;
   const unsigned gy = (unsigned)(P < 65535 ? P : 65535), gz = (unsigned)((P + 65534) / 65535);
-  moe_plain_kernel<T, true><<<dim3((F + 3) / 4, gy, gz), 256, 0, s>>>((const T*)x, ids, wts, (const T*)up, (T*)act, Tn, top, K, F);
+  moe_plain_kernel<T, true><<<dim3((F + 3) / 4, gy, gz), 256, 0, s>>>((const T*)x, ids, wts, (const T*)up, (T*)act, Tn, top, E, K, F, limit);
   DOCQA_CHECK_LAUNCH();
-  moe_plain_kernel<T, false><<<dim3((W + 3) / 4, gy, gz), 256, 0, s>>>((const T*)act, ids, wts, (const T*)down, (T*)out, Tn, top, F, W);
+  moe_plain_kernel<T, false><<<dim3((W + 3) / 4, gy, gz), 256, 0, s>>>((const T*)act, ids, wts, (const T*)down, (T*)out, Tn, top, E, F, W, limit);
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+template <bool GROUPS>
+int route(const void* x, const void* w, int f32, const RouteArgs& a, int T, hipStream_t s) {
+  const size_t row = (size_t)a.N * (GROUPS ? 8 : 4);
+  if (!f32 && a.K % 32 == 0 && 16 * row <= 64 * 1024 - 36 * 1024)
+    moe_route_mfma_kernel<GROUPS><<<(T + 15) / 16, 1024, 16 * row, s>>>((const uint16_t*)x, (const uint16_t*)w, a, T);
+  else if (f32)
+    moe_route_kernel<float, GROUPS><<<T, 256, row, s>>>((const float*)x, (const float*)w, a);
+  else
+    moe_route_kernel<uint16_t, GROUPS><<<T, 256, row, s>>>((const uint16_t*)x, (const uint16_t*)w, a);
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
 
 template <int MT>
 int skinny(const uint16_t* x, const int* ids, const float* wts, const uint16_t* up, const uint16_t* down, uint16_t* act,
-           uint16_t* out, int Tn, int top, int E, int K, int F, int W, hipStream_t s) {
+           uint16_t* out, int Tn, int top, int E, int K, int F, int W, float limit, hipStream_t s) {
   const int gy = E < Tn * top ? E : Tn * top;
   constexpr int NW = MT == 1 ? 8 : 4;
-  moe_skinny_kernel<MT, NW, true><<<dim3((F + 15) / 16, gy), 64 * NW, 0, s>>>(x, ids, wts, up, act, Tn, top, E, K, F);
+  moe_skinny_kernel<MT, NW, true><<<dim3((F + 15) / 16, gy), 64 * NW, 0, s>>>(x, ids, wts, up, act, Tn, top, E, K, F, limit);
   DOCQA_CHECK_LAUNCH();
-  moe_skinny_kernel<MT, NW, false><<<dim3((W + 31) / 32, gy), 64 * NW, 0, s>>>(act, ids, wts, down, out, Tn, top, E, F, W);
+  moe_skinny_kernel<MT, NW, false><<<dim3((W + 31) / 32, gy), 64 * NW, 0, s>>>(act, ids, wts, down, out, Tn, top, E, F, W, limit);
   DOCQA_CHECK_LAUNCH();
   return 0;
 }
@@ -394,15 +512,16 @@ int docqa_moe_route(const void* x, const void* w, int f32, int* ids, float* wts,
                     int top, hipStream_t s) {
   if (T == 0) return 0;
   if (E < 1 || E > 512 || N < E || N > 1024 || top < 1 || top > E || K < 1) return -1;
-  if (!f32 && K % 32 == 0 && 16 * N * 4 <= 64 * 1024 - 36 * 1024)
-    moe_route_mfma_kernel<<<(T + 15) / 16, 1024, (size_t)16 * N * 4, s>>>((const uint16_t*)x, (const uint16_t*)w, ids, wts, rest, T,
-                                                                       K, N, E, top);
-  else if (f32)
-    moe_route_kernel<float><<<T, 256, (size_t)N * 4, s>>>((const float*)x, (const float*)w, ids, wts, rest, K, N, E, top);
-  else
-    moe_route_kernel<uint16_t><<<T, 256, (size_t)N * 4, s>>>((const uint16_t*)x, (const uint16_t*)w, ids, wts, rest, K, N, E, top);
-  DOCQA_CHECK_LAUNCH();
-  return 0;
+  return route<false>(x, w, f32, RouteArgs{ids, wts, rest, K, N, E, top, nullptr, 1, 1, 1.f}, T, s);
+}
+
+int docqa_moe_route_groups(const void* x, const void* w, int f32, const float* corr, int* ids, float* wts, int T, int K, int N,
+                           int top, int groups, int keep, float scale, hipStream_t s) {
+  if (T == 0) return 0;
+  if (N < 1 || N > 512 || K < 1 || !corr || groups < 1 || N % groups || keep < 1 || keep > groups || top < 1 || top > 64 ||
+      top > keep * (N / groups))
+    return -1;
+  return route<true>(x, w, f32, RouteArgs{ids, wts, nullptr, K, N, N, top, corr, groups, keep, scale}, T, s);
 }
 
 int docqa_moe_scratch(int f32, int T, int top, int E, int K, int F, int W) {
@@ -412,11 +531,11 @@ int docqa_moe_scratch(int f32, int T, int top, int E, int K, int F, int W) {
 }
 
 int docqa_moe_experts(const void* x, const int* ids, const float* wts, const void* up, const void* down, void* act, void* out,
-                      int* scratch, int f32, int T, int top, int E, int K, int F, int W, hipStream_t s) {
+                      int* scratch, int f32, int T, int top, int E, int K, int F, int W, float limit, hipStream_t s) {
   const long long P = (long long)T * top;
   if (P == 0) return 0;
   if (E < 1 || E > 512 || top < 1 || K < 1 || F < 1 || W < 1 || P >= (1ll << 30)) return -1;
-  if (f32) return plain<float>(x, ids, wts, up, down, act, out, T, top, K, F, W, s);
+  if (f32) return plain<float>(x, ids, wts, up, down, act, out, T, top, E, K, F, W, limit, s);
   const uint16_t *xp = (const uint16_t*)x, *u = (const uint16_t*)up, *d = (const uint16_t*)down;
   uint16_t *a = (uint16_t*)act, *o = (uint16_t*)out;
   if (scratch) {
@@ -424,16 +543,16 @@ int docqa_moe_experts(const void* x, const int* ids, const float* wts, const voi
     const int tiles = tile_count((int)P, E);
     moe_sort_kernel<<<1, 1024, 0, s>>>(ids, scratch, (int)P, E, tiles);
     DOCQA_CHECK_LAUNCH();
-    moe_gemm_kernel<true><<<tiles * ((F + 63) / 64), 256, 0, s>>>(xp, wts, u, a, scratch, T, top, K, F, tiles);
+    moe_gemm_kernel<true><<<tiles * ((F + 63) / 64), 256, 0, s>>>(xp, wts, u, a, scratch, T, top, K, F, tiles, limit);
     DOCQA_CHECK_LAUNCH();
-    moe_gemm_kernel<false><<<tiles * ((W + 127) / 128), 256, 0, s>>>(a, wts, d, o, scratch, T, top, F, W, tiles);
+    moe_gemm_kernel<false><<<tiles * ((W + 127) / 128), 256, 0, s>>>(a, wts, d, o, scratch, T, top, F, W, tiles, limit);
     DOCQA_CHECK_LAUNCH();
     return 0;
   }
   if (P <= kSkinnyPairs && skinny_ok(K, F) && skinny_ok(F, W)) {
-    if (P <= 16 * E || P <= 16) return skinny<1>(xp, ids, wts, u, d, a, o, T, top, E, K, F, W, s);
-    if (P <= 32 * E) return skinny<2>(xp, ids, wts, u, d, a, o, T, top, E, K, F, W, s);
-    return skinny<4>(xp, ids, wts, u, d, a, o, T, top, E, K, F, W, s);
+    if (P <= 16 * E || P <= 16) return skinny<1>(xp, ids, wts, u, d, a, o, T, top, E, K, F, W, limit, s);
+    if (P <= 32 * E) return skinny<2>(xp, ids, wts, u, d, a, o, T, top, E, K, F, W, limit, s);
+    return skinny<4>(xp, ids, wts, u, d, a, o, T, top, E, K, F, W, limit, s);
   }
-  return plain<uint16_t>(x, ids, wts, up, down, act, out, T, top, K, F, W, s);
+  return plain<uint16_t>(x, ids, wts, up, down, act, out, T, top, E, K, F, W, limit, s);
 }

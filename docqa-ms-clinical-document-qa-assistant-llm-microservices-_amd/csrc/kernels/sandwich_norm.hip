@@ -9,6 +9,9 @@
 //
 // post_norm: norms after the sum, over equal parts of the row, behind a gated residual:
 //   x <- groupnorm(alpha x + sigmoid(gate + b) * y) * w
+// scaled_rmsnorm: a norm ahead of every sublayer alone, results scaled per channel, y a product with
+// its bias or the weighted sum of the chosen experts' outputs:
+//   x <- x + scale * y;   h = rms(x) * w_next
 #include "docqa_common.h"
 #include "docqa_elem.h"
 #include "docqa_hybrid.h"
@@ -389,6 +392,108 @@ __global__ __launch_bounds__(NT) void post_norm_kernel(DocqaPostNorm a) {
   }
 }
 
+// one workgroup of NT threads a row, V consecutive elements of NV pieces a thread.  MIX: P (of type PT, as x)
+// holds the chosen experts' outputs
+template <int NT, int NV, int V, typename PT, bool MIX>
+__global__ __launch_bounds__(NT) void scaled_rmsnorm_kernel(DocqaScaledNorm a) {
+  __shared__ float red[NT / 64];
+  const size_t row = blockIdx.x, slab = (size_t)a.rows * a.W;
+  const int tid = threadIdx.x, W = a.W, n = W / V;
+  const PT *P = (const PT*)a.P + row * W, *xr = (const PT*)a.x + row * W;
+  float x[NV][V], y[NV][V];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = min(tid + NT * i, n - 1);
+    ldv<V>(a.res + row * W + c * V, x[i]);
+    if constexpr (!MIX) ld_slabs<V>(P + c * V, a.SP, slab, y[i]);
+  }
+  if constexpr (MIX) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+#pragma unroll
+      for (int j = 0; j < V; ++j) y[i][j] = 0.f;
+    for (int k0 = 0; k0 < a.SP; k0 += 4) {               // four at a time: past the last, weight 0
+      const PT* p[4];
+      float w[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int k = min(k0 + u, a.SP - 1);
+        p[u] = a.ids[row * a.SP + k] < a.experts ? P + k * slab : xr;
+        w[u] = k0 + u < a.SP ? a.wts[row * a.SP + k] : 0.f;
+      }
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = min(tid + NT * i, n - 1);
+        float f[4][V];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) ldv<V>(p[u] + c * V, f[u]);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+          for (int j = 0; j < V; ++j) y[i][j] += w[u] * f[u][j];
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = tid + NT * i;
+    if (c < n) {
+      float g[V], b[V];
+      ldv<V>(a.scale + c * V, g);
+#pragma unroll
+      for (int j = 0; j < V; ++j) b[j] = 0.f;
+      if (a.bias) ldv<V>(a.bias + c * V, b);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        x[i][j] += g[j] * (y[i][j] + b[j]);
+        ss += x[i][j] * x[i][j];
+      }
+      stv<V>(a.res + row * W + c * V, x[i]);
+    }
+  }
+  const float inv = 1.f / sqrtf(block_sum<NT>(ss, red) / (float)W + a.eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = tid + NT * i;
+    if (c < n) {
+      float g[V];
+      ldv<V>(a.w + c * V, g);
+#pragma unroll
+      for (int j = 0; j < V; ++j) g[j] *= x[i][j] * inv;
+      if (a.of32) stv<V>((float*)a.out + row * W + c * V, g);
+      else stv<V>((uint16_t*)a.out + row * W + c * V, g);
+    }
+  }
+}
+
+template <int V, typename PT, bool MIX>
+int launch_scaled(const DocqaScaledNorm& a, hipStream_t s) {
+  const int nv = (a.W / V + 255) / 256;
+#define GO(NV)                                                                                                  \
+  do {                                                                                                          \
+    if (V > 1 && NV >= 4 && a.rows <= 512)                                                                      \
+      scaled_rmsnorm_kernel<1024, (NV >= 4 ? NV / 4 : 1), V, PT, MIX><<<a.rows, 1024, 0, s>>>(a);               \
+    else                                                                                                        \
+      scaled_rmsnorm_kernel<256, NV, V, PT, MIX><<<a.rows, 256, 0, s>>>(a);                                     \
+  } while (0)
+  if (nv <= 1) GO(1);
+  else if (nv <= 2) GO(2);
+  else if (nv <= 4) GO(4);
+  else if (nv <= 8) GO(8);
+  else if (nv <= 16) GO(16);
+  else return -1;
+#undef GO
+  DOCQA_CHECK_LAUNCH();
+  return 0;
+}
+
+template <typename PT>
+int scaled_mix(const DocqaScaledNorm& a, hipStream_t s) {
+  if (a.ids) return a.W % 4 == 0 ? launch_scaled<4, PT, true>(a, s) : launch_scaled<1, PT, true>(a, s);
+  return a.W % 4 == 0 ? launch_scaled<4, PT, false>(a, s) : launch_scaled<1, PT, false>(a, s);
+}
+
 template <int V>
 int launch_post_norm(const DocqaPostNorm& a, hipStream_t s) {
   const int n = a.W / V, gn = n / a.groups;
@@ -414,6 +519,12 @@ int launch_post_norm(const DocqaPostNorm& a, hipStream_t s) {
   return 0;
 }
 }  // namespace
+
+int docqa_scaled_rmsnorm(const DocqaScaledNorm& a, hipStream_t s) {
+  if (a.rows == 0) return 0;
+  if (a.W < 1 || a.SP < 1 || !a.scale || (a.ids && (!a.wts || !a.x))) return -1;
+  return a.pf32 ? scaled_mix<float>(a, s) : scaled_mix<uint16_t>(a, s);
+}
 
 int docqa_post_norm(const DocqaPostNorm& a, hipStream_t s) {
   if (a.rows == 0) return 0;
