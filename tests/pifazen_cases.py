@@ -1,0 +1,530 @@
+"""Shared bodies of the Pifazen tests: every case takes the device (and the dtype where it
+matters), so the CPU suite runs the reference operators and the GPU suite the HIP kernels
+against the same plain oracle (tests/pifazen_oracle.py)."""
+from __future__ import annotations
+
+import torch
+
+import pifazen_oracle as O
+from docqa_amd import ops
+from docqa_amd.models import pifazen
+from docqa_amd.models.hybrid import HybridModel
+from model_cases import ModelCases
+from saritar_cases import BF16, F32, close, engine, portions, run_steps, toks
+
+F64 = torch.float64
+
+
+# ------------------------------------------------------------------ configurations
+def moe(experts, identity, top, ff, count=1, keep=1, scale=1.0, limit=2.0):
+    return {"kind": "moe", "expert": {"ff": ff, "limit": limit},
+            "router": {"experts": experts, "identity": identity, "top": top, "scale": scale, "groups": {"count": count, "keep": keep}}}
+
+
+def dense(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+def rot(base, dims, scaling=None):
+    r = {"base": base, "dims": dims}
+    if scaling:
+        r["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    return r
+
+
+def lat(heads, dim, r, vdim, rank, q_rank, scale=None, base=1e4, mlp=None):
+    return {"type": "latent_attention", "mlp": mlp, "mixer": {
+        "heads": heads, "dim": dim, "rot_dim": r, "vdim": vdim, "kv_rank": rank, "q_rank": q_rank, "scale": scale or (dim + r) ** -0.5,
+        "rot": rot(base, r)}}
+
+
+def lat2(heads, dim, r, vdim, rank, scaling, scale=None, base=1e4, mlp=None):
+    return {"type": "latent_attention_2", "mlp": mlp, "mixer": {
+        "heads": heads, "dim": dim, "rot_dim": r, "vdim": vdim, "kv_rank": rank, "scale": scale or (dim + r) ** -0.5,
+        "rot": rot(base, r, scaling)}}
+
+
+def delta(heads, kv, dim, vdim, conv, mlp=None):
+    return {"type": "channel_delta", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": conv}}
+
+
+def again(layer, i):
+    return dict(layer, weights_of=i)
+
+
+def conf(width, vocab, layers, eps=1e-5):
+    return {"architecture": "Pifazen", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
+
+
+YARN = (4.0, 64.0, 8.0, 0.5)
+_D = delta(4, 2, 16, 24, 4, moe(6, 2, 3, 24, 4, 2, 1.7))
+CONFIGS = {
+    # every mixer and feed-forward, weights used again beside their owner and ahead of it
+    "mixed": conf(64, 97, [lat(4, 16, 8, 24, 40, 32, 0.25, mlp=dense(48)), _D, lat2(3, 24, 16, 16, 32, YARN, 0.2, mlp=moe(5, 4, 2, 32, 3, 1, 2.5)),
+                           again(_D, 1), lat2(2, 16, 8, 8, 24, None, mlp=dense(40))], 1e-4),
+    # nothing a multiple of eight, layers without a feed-forward, no identity expert, one group, more key than value heads' size
+    "odd": conf(36, 50, [delta(3, 1, 10, 7, 3), lat(3, 10, 6, 7, 21, 19, 0.4, 300.0, moe(3, 0, 3, 10, scale=0.8, limit=0.7)),
+                         lat2(2, 5, 2, 9, 13, (2.0, 32.0, 4.0, 1.0), 0.5, 50.0, dense(21)), delta(2, 2, 9, 3, 2, moe(4, 5, 4, 6, 9, 5, 1.3))]),
+    # sizes of one
+    "ones": conf(40, 61, [lat(1, 1, 2, 1, 8, 8, mlp=moe(1, 1, 1, 1)), delta(1, 1, 1, 2, 1, dense(8)), lat2(1, 8, 2, 8, 16, None, mlp=moe(1, 0, 1, 8)),
+                          delta(2, 1, 2, 1, 1)]),
+    # sequences past a block and a chunk, many taps, heads that share keys, more heads than a row tile
+    "edge": conf(128, 80, [delta(6, 2, 32, 64, 7, moe(8, 4, 3, 64, 4, 2, 2.0)), lat(20, 32, 16, 32, 64, 96, base=3e5, mlp=dense(256)),
+                           lat2(8, 64, 32, 64, 128, (8.0, 48.0, 32.0, 1.0), 0.13, 1e6, moe(8, 0, 2, 64, 2, 1)), delta(4, 4, 64, 32, 4, moe(2, 14, 4, 64, 8, 4))]),
+}
+
+
+def settle_routing(w, js):
+    """The choice of experts is a step function of its input: one direction of the stream per expert is
+    the token's own, hardly touched by the sublayers, and the router reads those, so that rounding does not
+    decide.  The correction is one negative number: a group that is left out must not count as zero."""
+    sizes = [(i, L["mlp"]["router"]) for i, L in enumerate(js["layers"]) if L["mlp"] and L["mlp"]["kind"] == "moe" and "weights_of" not in L]
+    N = max([r["experts"] + r["identity"] for _, r in sizes] + [0])
+    if N == 0:
+        return
+    g = torch.Generator().manual_seed(99)
+    w["embed"][:, :N] = torch.stack([torch.randperm(N, generator=g).float() for _ in range(js["vocab"])]) * (6.0 / N) - 3.0
+    for n, t in w.items():
+        if n.endswith((".o", ".down", ".down.b")) and t.shape[0] == js["width"]:
+            t[:N] *= 0.02
+        elif n.endswith(("norm1", "norm2")):
+            t[:N] = 0.0
+        elif n.endswith("mlp.router"):
+            t *= 0.02
+            t[:, :N] += torch.eye(t.shape[0], N) * (N / 2)
+        elif n.endswith("correction"):
+            t.fill_(-0.375)
+
+
+def make(name, device, dtype=F32, seed=0, tweak=None):
+    js = CONFIGS[name] if isinstance(name, str) else name
+    w = O.random_weights(js, seed)
+    if dtype == BF16:
+        settle_routing(w, js)
+    if tweak:
+        tweak(w)
+    w = {k: v.to(BF16).float() for k, v in w.items()}
+    return js, w, HybridModel(pifazen.config_from_json(js), device=device, dtype=dtype, weights=w)
+
+
+MODELS = ModelCases(make, O.forward)
+
+
+def i32(device, *v):
+    return torch.tensor(v, dtype=torch.int32, device=device)
+
+
+def rnd(seed, *shape):
+    return torch.randn(*shape, generator=torch.Generator().manual_seed(seed))
+
+
+def slabs(x, S, seed, device, dtype):
+    """x as a product of the dtype, or as S fp32 slabs that sum to it."""
+    if S == 1:
+        return x.to(device, dtype)
+    part = rnd(seed, S - 1, *x.shape)
+    return torch.cat([part, (x - part.sum(0))[None]]).to(device)
+
+
+# ------------------------------------------------------------------ stream update
+def scaled_norm_case(device, dtype):
+    for W, rows, S, bias in ((30, 3, 1, True), (48, 2, 2, False), (64, 5, 3, True), (1024, 2, 1, False), (2050, 1, 2, True), (4096, 3, 4, True),
+                             (5120, 600, 1, False)):
+        eps = 1e-3
+        x, y, s, w = rnd(1, rows, W), rnd(2, rows, W), rnd(3, W), rnd(4, W)
+        y = y.to(dtype).float() if S == 1 else y
+        b = rnd(5, W) if bias else None
+        stream = x + s * (y if b is None else y + b)
+        res = x.clone().to(device)
+        out = ops.scaled_rmsnorm(slabs(y, S, 7, device, dtype), res, s.to(device), (1 + w).to(device), eps,
+                                 bias=None if b is None else b.to(device), out_dtype=dtype)
+        assert out.dtype == dtype
+        close(res, stream, what=W)
+        close(out, O.layer_norm(stream, w, eps), dtype, W)
+
+
+def mix_case(device, dtype):
+    """The chosen experts' outputs weighted and summed, the input itself for identity experts; what stands in
+    P for those is never read."""
+    for W, rows, top, E in ((30, 3, 1, 2), (64, 4, 3, 4), (1024, 2, 5, 6), (4096, 3, 4, 2), (48, 2, 16, 8), (2052, 520, 2, 3)):
+        g = torch.Generator().manual_seed(W)
+        x, h, P = rnd(1, rows, W), rnd(2, rows, W).to(dtype).float(), rnd(3, top, rows, W).to(dtype).float()
+        ids = torch.stack([torch.randperm(E + top, generator=g)[:top] for _ in range(rows)]).to(torch.int32)
+        wts = torch.rand(rows, top, generator=g)
+        s, w = rnd(4, W), rnd(5, W)
+        own = (ids >= E).t()[..., None]
+        y = (wts.t()[..., None] * torch.where(own, h[None], P)).sum(0)
+        stream = x + s * y
+        res = x.clone().to(device)
+        out = ops.scaled_rmsnorm(P.masked_fill(own, float("nan")).to(device, dtype), res, s.to(device), (1 + w).to(device), 1e-5,
+                                 mix=(ids.to(device), wts.to(device), E, h.to(device, dtype)), out_dtype=dtype)
+        close(res, stream, what=(W, top))
+        close(out, O.layer_norm(stream, w, 1e-5), dtype, (W, top))
+
+
+def poly_norm_case(device, dtype):
+    for n, ld, n_out, rows, S in ((1, 1, 1, 2, 1), (7, 9, 64, 3, 2), (48, 64, 64, 2, 1), (21, 64, 64, 5, 3), (1000, 1024, 1024, 2, 1), (5000, 5120, 5056, 2, 2),
+                                  (14336, 14336, 14336, 3, 1), (9001, 9216, 9024, 2, 1), (33, 40, 40, 300, 1)):
+        z = rnd(1, rows, ld).to(dtype).float() if S == 1 else rnd(1, rows, ld)
+        b, act = rnd(2, n) * 0.5, torch.tensor([0.7, -0.5, 0.4, 0.3])
+        want = O.poly_norm(z[:, :n].double() + b, act.double(), 1e-4).float()
+        got = ops.poly_norm(slabs(z, S, 3, device, dtype), b.to(device), act.to(device), n_out, 1e-4, dtype)
+        assert got.shape == (rows, n_out) and got.dtype == dtype and (got[:, n:] == 0).all()
+        close(got[:, :n], want, dtype, (n, ld))
+    # eps decides in a small row; each power has its own mean
+    z = torch.cat([rnd(1, 1, 64) * 1e-2, rnd(2, 1, 64) * 30])
+    for act in torch.eye(4):
+        close(ops.poly_norm(z.to(device), torch.zeros(64, device=device), act.to(device), 64, 1e-3, F32), O.poly_norm(z.double(), act.double(), 1e-3))
+
+
+# ------------------------------------------------------------------ latent attention
+def query_latent_case(device, dtype):
+    """One launch of the query latent's norm and the cache row; columns behind them do not matter."""
+    for Rq, R, r, T, S in ((32, 24, 8, 5, 1), (19, 21, 6, 4, 2), (1536, 512, 64, 3, 1), (1, 1, 2, 2, 1), (2048, 40, 16, 300, 1), (2047, 2045, 10, 2, 3)):
+        eps, bs = 1e-3, 16
+        x = rnd(1, T, Rq + R + r + 5)
+        x = x.to(dtype).float() if S == 1 else x
+        wq, wc = 1 + 0.3 * rnd(2, Rq), 1 + 0.3 * rnd(3, R)
+        R8, r8 = -(-R // 8) * 8, -(-r // 8) * 8
+        nb = T // bs + 2
+        cache = torch.full((nb, 1, bs, R8 + r8), 7.0, dtype=dtype, device=device)
+        slots = (torch.arange(T, dtype=torch.int32) + 3)
+        slots[T // 2] = -1                                      # a row without a place
+        cs = torch.cat([rnd(4, T, r // 2).cos(), rnd(4, T, r // 2).sin()], 1)
+        got = ops.latent_norm_store(slabs(x, S, 5, device, dtype), cs.to(device), slots.to(device), cache, wq.to(device), wc.to(device), eps, dtype)
+        assert got.shape == (T, Rq) and got.dtype == dtype
+        close(got, O.unit_rms(x[:, :Rq], eps) * wq, dtype, (Rq, R))
+        rows = cache.view(-1, R8 + r8).float().cpu()
+        c, k = O.unit_rms(x[:, Rq:Rq + R], eps) * wc, x[:, Rq + R:Rq + R + r]
+        u, v, co, si = k[:, :r // 2], k[:, r // 2:], cs[:, :r // 2], cs[:, r // 2:]
+        k = torch.cat([u * co - v * si, v * co + u * si], 1)
+        for t in range(T):
+            if slots[t] < 0:
+                assert (rows[t + 3] == 7).all()
+                continue
+            close(rows[t + 3, None, :R], c[t:t + 1], dtype, (Rq, R, t))
+            close(rows[t + 3, None, R8:R8 + r], k[t:t + 1], dtype, (Rq, R, t))
+            assert (rows[t + 3, R:R8] == 0).all() and (rows[t + 3, R8 + r:] == 0).all()
+
+
+def head_gate_case(device, dtype):
+    for T, H, vd, per_head, S, col in ((3, 4, 24, False, 1, 8), (5, 3, 7, True, 2, 3), (2, 32, 128, True, 1, 64), (70, 16, 64, False, 3, 128), (1, 1, 1, False, 1, 0),
+                                       (4, 2, 16, True, 1, 5)):
+        x, n = rnd(1, T, H * vd).to(dtype).float(), H if per_head else H * vd
+        P = rnd(2, T, col + n + 4) * 3
+        P = P.to(dtype).float() if S == 1 else P
+        want = (x.view(T, H, vd) * O.sigmoid(P[:, col:col + n]).view(T, H, -1)).view(T, -1)
+        got = ops.head_gate(x.to(device, dtype), slabs(P, S, 3, device, dtype), col, vd if per_head else 1)
+        close(got, want, dtype, (T, H, vd))
+
+
+def latent_layer_case(device, dtype):
+    """Layers of one mixer alone, through cache and portions: sizes on and off the kernels' granules, queries from
+    a latent and from the input, both gates, with and without YaRN, latents past every MFMA form."""
+    for i, L in enumerate((lat(3, 8, 8, 8, 16, 24), lat(5, 10, 6, 7, 21, 9, 0.3), lat(16, 24, 8, 40, 72, 64, base=5e3), lat(2, 96, 32, 64, 200, 136, 0.1),
+                           lat(20, 32, 64, 96, 512, 72), lat(1, 1, 2, 1, 3, 2), lat2(4, 16, 8, 24, 40, YARN), lat2(2, 5, 2, 9, 13, None, 0.6),
+                           lat2(9, 128, 64, 128, 256, (8.0, 32.0, 8.0, 1.0)), lat2(6, 40, 16, 33, 96, (16.0, 4096.0, 32.0, 1.0), 0.2, 1e5),
+                           lat2(2, 12, 70, 20, 600, (3.0, 100.0, 2.0, 2.0)))):
+        js = conf(48, 53, [L])
+        T = 75 if i % 2 else 140
+        MODELS.portions(js, device, dtype, T, ([T], [2, 1, T - 3], [T - 5, 1, 1, 1, 1, 1], [7, 1, 9, 2, 33, T - 52]))
+
+
+def far_case(device, dtype):
+    """One key far back outshines the hundreds after it: the token that makes it decides the logits of every
+    position behind it and of none ahead, at a page's border or inside, whatever the portions."""
+    for at, T in ((0, 150), (1, 90), (63, 200), (64, 140), (100, 331)):
+        for L in (lat(2, 8, 8, 16, 24, 16, 0.5), lat2(2, 8, 8, 16, 24, YARN, 0.5)):
+            js = conf(32, 40, [L])
+
+            def star(w):
+                # token 7 alone has a large first element of its embedding and of its latent; every query
+                # looks for it through a constant second element
+                w["embed"][:, 0], w["embed"][:, 1] = 0.0, 3.0
+                w["embed"][7] = 0.0
+                w["embed"][7, 0], w["embed"][7, 1] = 12.0, 3.0
+                p = "l0.mix."
+                w["l0.norm1"].zero_()
+                if p + "dq" in w:
+                    w[p + "dq"].mul_(0.1)
+                    w[p + "dq"][0] = 0.0
+                    w[p + "dq"][0, 1] = 4.0
+                    w[p + "dq.norm"].fill_(1.0)
+                q = w[p + "uq" if p + "uq" in w else p + "q"]
+                q.mul_(0.05)
+                q.view(2, 16, -1)[:, 0] = 0.0
+                q.view(2, 16, -1)[:, 0, 0 if p + "uq" in w else 1] = 4.0
+                uk = w[p + "uk"].view(2, 8, 24)
+                uk.mul_(0.1)
+                uk[:, 0] = 0.0
+                uk[:, 0, 0] = 6.0
+                w[p + "dkv"][0] = 0.0
+                w[p + "dkv"][0, 0] = 4.0
+                w[p + "dkv"][1:, 0] = 0.0
+                w[p + "dkv.norm"].fill_(1.0)
+
+            js, w, m = make(js, device, dtype, seed=8, tweak=star)
+            other = [t if t != 7 else 8 for t in toks(T, 40, 12)]
+            seq = list(other)
+            seq[at] = 7
+            wa, wb = O.forward(js, w, seq), O.forward(js, w, other)
+            gap = (wa - wb).pow(2).mean(-1).sqrt()
+            assert gap[at:].min() > 0.3 and (at == 0 or gap[:at].max() < 1e-9)
+            for sizes in ([T], [2, 50, 64, 1, 1, 1, 1], [at + 1] + [1] * (T - at - 1), [T - 3, 2, 1]):
+                for s, want in ((seq, wa), (other, wb)):
+                    close(run_steps(engine(m), [[("a", p)] for p in portions(s, sizes)])["a"], want, dtype, (L["type"], at, sizes[:4]))
+
+
+# ------------------------------------------------------------------ channel delta rule
+class ChannelDelta:
+    """One recurrence over a sequence: rows [q | k | v] and [g | a | b] drawn at random, through the operators
+    in portions, and by the oracle."""
+
+    def __init__(self, device, dtype, T, H, G, d, vd, seed=0, z_off=None, tweak=None):
+        self.device, self.dtype, self.T, self.H, self.d, self.vd, self.eps = device, dtype, T, H, d, vd, 1e-4
+        widths, at = [G * d, G * d, H * vd], [4]
+        for n in widths:
+            at.append(at[-1] + n)
+        self.X = rnd(seed, T, at[-1] + 3)
+        zat = [0, H * d, H * d + H * vd]
+        self.Z = rnd(seed + 9, T, zat[-1] + H + 2)
+        self.w_gate, self.b_gate = -torch.exp(rnd(seed + 2, H) - 1), rnd(seed + 3, H * d) - 1
+        if z_off is not None:
+            self.b_gate += z_off
+        self.at, self.zat = at, zat
+        if tweak:
+            tweak(self)
+        self.X = self.X.to(dtype).float()
+        self.norm = 1 + 0.3 * rnd(seed + 1, vd)
+        q, k, v = (self.X[:, s:s + n].double() for s, n in zip(at, widths))
+        a, g, b = (self.Z[:, s:s + n].double() for s, n in zip(zat, (H * d, H * vd, H)))
+        q, k = (O.unit(x.reshape(T, G, d)).repeat_interleave(H // G, 1) for x in (q, k))
+        dec = torch.exp(self.w_gate.double()[:, None] * O.softplus(a + self.b_gate).view(T, H, d))
+        self.o = O.delta_recurrence(q * d ** -0.5, k, v.reshape(T, H, vd), dec, O.sigmoid(b))
+        self.want = ((O.unit_rms(self.o, self.eps) * self.norm).reshape(T, -1) * O.sigmoid(g)).float()
+        self.mix = ops.LinearMix("channel_delta", H, G, d, vd, at[0], at[1], at[2], zat[1], a=zat[0], b=zat[2], q_scale=d ** -0.5, eps=self.eps,
+                                 gate="sigmoid")
+        self.shape = ops.linear_state_shape(H, d, vd)
+
+    def operands(self, lo, hi, S=1):
+        dev = self.device
+        return (slabs(self.X[lo:hi], S, hi, dev, self.dtype), self.Z[lo:hi].contiguous().to(dev), self.mix, self.w_gate.to(dev),
+                self.b_gate.to(dev), None, self.norm.to(dev))
+
+    def run(self, cuts, step=True, S=1):
+        dev, dt = self.device, self.dtype
+        state = torch.zeros(3, *self.shape, device=dev)
+        state[..., :self.vd] = 9.0                                         # a former owner's
+        out, t0, W = [], 0, self.H * self.vd
+        for n in cuts:
+            wide = torch.full((n, W + 4), 5.0, dtype=dt, device=dev)
+            a = (*self.operands(t0, t0 + n, S), state, i32(dev, 1))
+            if n == 1 and step:
+                ops.linear_step(*a, i32(dev, t0), wide[:, :W])
+            else:
+                ops.linear_scan(*a, i32(dev, 0, n), i32(dev, t0), n, wide[:, :W])
+            out.append(wide[:, :W])
+            assert (wide[:, W:] == 5).all()
+            t0 += n
+        assert t0 == self.T and (state[0, ..., :self.vd] == 9).all() and (state[2, ..., :self.vd] == 9).all()
+        return torch.cat(out)
+
+
+# T, H, G, d, vd
+DELTA_SIZES = ((70, 4, 2, 16, 24), (140, 3, 1, 128, 128), (129, 2, 2, 48, 72), (67, 3, 3, 5, 7), (50, 1, 1, 256, 20), (20, 2, 1, 1, 1), (131, 2, 2, 64, 40),
+               (66, 2, 1, 256, 256), (70, 1, 1, 128, 508), (33, 1, 1, 160, 250))
+
+
+def delta_case(device, dtype, sizes=DELTA_SIZES):
+    for T, H, G, d, vd in sizes:
+        L = ChannelDelta(device, dtype, T, H, G, d, vd, seed=T + d)
+        for k, cuts in enumerate(([T], [2] * (T // 2) + [1] * (T % 2), [1] * T, [T - 4, 1, 1, 2], [3, T - 5, 2])):
+            close(L.run(cuts, S=1 + 2 * (k == 4)), L.want, dtype, (T, H, d, vd, cuts[:4]))
+        close(L.run([1, T - 2, 1], step=False), L.want, dtype, "scan of one token")
+
+
+def delta_decay_case(device, dtype):
+    """Decays near one over many chunks, so strong that a chunk's product underflows, and of both kinds side by
+    side: channels that forget at once beside some that keep everything, tokens that forget amid others."""
+    for z_off in (-20.0, 3.0, 60.0, 400.0):
+        L = ChannelDelta(device, dtype, 200, 2, 2, 24, 16, seed=4, z_off=z_off)
+        for cuts in ([200], [70, 1, 129], [198, 1, 1]):
+            close(L.run(cuts), L.want, dtype, (z_off, cuts))
+
+    def channels(L):
+        L.b_gate[::3] = 50.0
+        L.b_gate[1::3] = -30.0
+
+    def tokens(L):
+        L.Z[20::17, :L.H * L.d] = 80.0
+        L.b_gate.fill_(-9.0)
+
+    def drop(L):                      # 16 tokens drop by just under and just over what one reference bears
+        L.w_gate = torch.tensor([-1.0, -1.0])
+        L.Z[:, :L.H * L.d] = 0.0
+        L.b_gate[:] = torch.tensor([1.8, 2.0]).repeat_interleave(L.d)
+
+    for tweak in (channels, tokens, drop):
+        for d in (24, 128, 200):
+            L = ChannelDelta(device, dtype, 150, 2, 1, d, 16, seed=5, tweak=tweak)
+            for cuts in ([150], [70, 1, 79], [148, 1, 1]):
+                close(L.run(cuts), L.want, dtype, (tweak.__name__, d, cuts))
+
+
+def delta_batch_case(device, dtype):
+    """Packed sequences of unequal length -- empty ones among them --, new and carried, rows without a
+    slot, against each alone."""
+    L = ChannelDelta(device, dtype, 210, 3, 1, 16, 20, seed=9)
+    lens, ctx0, sl = [1, 64, 0, 130, 2, 13], [7, 0, 0, 70, 3, 0], [4, 2, 0, -1, 1, 5]
+    cu = [0]
+    for n in lens:
+        cu.append(cu[-1] + n)
+    assert cu[-1] == 210
+    st0 = torch.zeros(6, *L.shape)
+    st0[..., :20] = rnd(10, 6, *L.shape[:2], 20)
+
+    def scan(lo, hi, state, slots, cu_, ctx, most):
+        out = torch.empty(hi - lo, 60, dtype=dtype, device=device)
+        return ops.linear_scan(*L.operands(lo, hi), state, i32(device, *slots), i32(device, *cu_), i32(device, *ctx), most, out)
+
+    state = st0.clone().to(device)
+    both = scan(0, 210, state, sl, cu, ctx0, max(lens))
+    assert torch.equal(state[0].cpu(), st0[0]) and torch.equal(state[3].cpu(), st0[3])       # an empty sequence's, nobody's
+    for b, n in enumerate(lens):
+        if n == 0:
+            continue
+        s1 = st0.clone().to(device)
+        one = scan(cu[b], cu[b + 1], s1, [sl[b]], [0, n], [ctx0[b]], n)
+        close(both[cu[b]:cu[b + 1]], one.cpu(), dtype, b)
+        if sl[b] >= 0:
+            close(state[sl[b]].reshape(3, -1), s1[sl[b]].cpu().reshape(3, -1), what=b)
+    # one token a row, rows without a slot among them
+    state = st0.clone().to(device)
+    out = torch.empty(4, 60, dtype=dtype, device=device)
+    ops.linear_step(*L.operands(0, 4), state, i32(device, 3, -1, 0, 5), i32(device, 9, 4, 0, 1), out)
+    for b, (slot, pos) in enumerate(((3, 9), (-1, 4), (0, 0), (5, 1))):
+        s1 = st0.clone().to(device)
+        close(out[b:b + 1], scan(b, b + 1, s1, [slot], [0, 1], [pos], 1).cpu(), dtype, ("step", b))
+        if slot >= 0:
+            close(state[slot].reshape(3, -1), s1[slot].cpu().reshape(3, -1), what=("step", b))
+    assert torch.equal(state[1].cpu(), st0[1])
+
+
+def forgotten_state_case(device, dtype):
+    """A token's write is read back many chunks later through a decay of nearly one in its channel: a state lost
+    between portions would leave nothing of it."""
+    def tweak(L):
+        q, k = L.X[:, L.at[0]:L.at[1]], L.X[:, L.at[1]:L.at[2]]
+        k *= 0.01
+        q.zero_()
+        q[:, 0] = 2.0
+        k[:, 0] = 0.0
+        k[5, 0] = 8.0
+        L.b_gate.fill_(20.0)                  # every other channel forgets
+        L.b_gate[0] = -40.0
+
+    T = 230
+    L = ChannelDelta(device, dtype, T, 1, 1, 32, 8, seed=6, tweak=tweak)
+    assert L.o[-1].abs().max() > 0.05                       # still there
+    # (ahead of the write there is nothing to read but rounding)
+    for cuts in ([T], [6, 64, 64, T - 134], [7] + [1] * (T - 7), [40, 2, 2, 1, T - 45]):
+        close(L.run(cuts)[5:], L.want[5:], dtype, cuts[:4])
+
+
+def low_rank_case(device, dtype):
+    """Two products through few elements and the columns behind them, from any column of a wider matrix."""
+    for T, at, Ka, Kg, Na, Ng, n in ((1, 0, 8, 16, 20, 12, 3), (5, 13, 24, 8, 7, 130, 1), (33, 8, 128, 64, 256, 300, 16), (70, 5, 16, 40, 64, 65, 4),
+                                     (100, 16, 256, 128, 96, 128, 32), (9, 0, 1024, 8, 64, 64, 0), (200, 24, 520, 32, 40, 72, 8)):
+        z = rnd(1, T, at + Ka + Kg + n + 3).to(dtype)
+        wa, wg = ((rnd(s, *sh) * sh[1] ** -0.5).to(dtype) for s, sh in ((2, (Na, Ka)), (3, (Ng, Kg))))
+        zf = z.double()
+        want = torch.cat([zf[:, at:at + Ka] @ wa.double().T, zf[:, at + Ka:at + Ka + Kg] @ wg.double().T,
+                          zf[:, at + Ka + Kg:at + Ka + Kg + n]], 1)
+        got = ops.low_rank(z.to(device), at, wa.to(device), wg.to(device), n)
+        assert got.dtype == F32 and got.shape == (T, Na + Ng + n)
+        close(got, want, what=(T, at, Ka))
+        wide = torch.zeros(T + 2, z.shape[1] + 5, dtype=dtype, device=device)        # rows of a part of a batch
+        wide[1:T + 1, :z.shape[1]] = z.to(device)
+        close(ops.low_rank(wide[1:T + 1], at, wa.to(device), wg.to(device), n), want, what=("rows", T))
+
+
+def delta_layer_case(device, dtype):
+    for i, L in enumerate((delta(3, 3, 16, 24, 1), delta(4, 2, 9, 5, 3), delta(2, 1, 64, 32, 4), delta(2, 2, 128, 64, 7), delta(1, 1, 1, 1, 2), delta(2, 1, 160, 16, 4))):
+        if L["mixer"]["dim"] == 1 and dtype == BF16:
+            continue                    # (a unit vector of one element is its sign)
+        js = conf(48, 53, [L])
+        T = 75 if i % 2 else 140
+        w = O.random_weights(js, 2, rank=((5, 7), (8, 16), (1, 1))[i % 3])
+        m = HybridModel(pifazen.config_from_json(js), device=device, dtype=dtype, weights=w)
+        seq = toks(T, 53, 3)
+        want = O.forward(js, w, seq)
+        for sizes in ([T], [2, 1, T - 3], [T - 5, 1, 1, 1, 1, 1], [7, 1, 9, 2, 33, T - 52], [1] * T):
+            close(run_steps(engine(m), [[("a", p)] for p in portions(seq, sizes)])["a"], want, dtype, (L["mixer"], sizes[:4]))
+
+
+# ------------------------------------------------------------------ experts
+# T, K, experts, identity, top, ff, groups, keep
+MOE_SIZES = ((1, 64, 4, 2, 2, 64, 3, 2), (3, 64, 8, 0, 2, 64, 1, 1), (40, 96, 6, 3, 3, 32, 3, 1), (130, 128, 4, 4, 2, 96, 4, 3), (7, 36, 3, 1, 3, 10, 2, 2),
+             (5, 40, 1, 1, 1, 8, 2, 1), (300, 128, 8, 8, 2, 128, 4, 2), (700, 192, 5, 1, 1, 64, 3, 2), (60, 64, 300, 20, 4, 64, 80, 10),
+             (260, 64, 70, 2, 16, 64, 6, 2), (20, 64, 2, 30, 6, 32, 8, 4), (400, 128, 3, 13, 4, 64, 16, 8), (9, 32, 500, 12, 5, 8, 128, 3))
+
+
+def moe_case(device, dtype, sizes=MOE_SIZES):
+    """Routing in groups and the experts, identity ones among them, against the oracle.  The router's operands are
+    exact in both, so the choice is the same."""
+    for T, K, E, ident, top, F, count, keep in sizes:
+        N = E + ident
+        x = rnd(T, T, K).to(dtype).float()
+        wr = (rnd(T + 1, N, K) * 2 * K ** -0.5).to(dtype).float()
+        t = {"router": wr, "correction": rnd(T + 2, N) * 0.3 - 0.5}          # (scores below zero)
+        up, down = (rnd(T + 3, E, 2, F, K) * 2 * K ** -0.5).to(dtype).float(), (rnd(T + 4, E, K, F) * F ** -0.5).to(dtype).float()
+        for e in range(E):
+            t.update({f"e{e}.gate": up[e, 0], f"e{e}.up": up[e, 1], f"e{e}.down": down[e]})
+        m = moe(E, ident, top, F, count, keep, 1.8, 1.1)
+        best, w = O.route(x.double(), m["router"], {k: v.double() for k, v in t.items() if k in ("router", "correction")})
+        xd = x.to(device, dtype)
+        ids, wts = ops.moe_route_groups(xd, wr.to(device, dtype), t["correction"].to(device), top, count, keep, 1.8)
+        assert ids.dtype == torch.int32 and ids.shape == wts.shape == (T, top)
+        a, b = (i.cpu().long().sort(-1) for i in (ids, best))
+        assert torch.equal(a.values, b.values), (T, E, ident, top)
+        close(wts.cpu().gather(1, a.indices), w.gather(1, b.indices), what=(T, E, top))
+        y = ops.moe_experts(xd, ids, wts, up.to(device, dtype), down.to(device, dtype), 1.1)
+        assert y.shape == (top, T, K)
+        res = torch.zeros(T, K, device=device)
+        one = torch.ones(K, device=device)
+        ops.scaled_rmsnorm(y, res, one, one, 1e-5, mix=(ids, wts, E, xd), out_dtype=dtype)
+        close(res, O.experts(x, m, t), dtype, (T, K, E, ident, top, F))
+
+
+def group_case(device, dtype):
+    """A group counts by its best expert alone, is left out even where its scores are the higher ones of the rest,
+    and never comes back as zero; the correction decides the choice and not the weights."""
+    K, eye = 64, torch.eye(12, 64)
+    x = torch.zeros(3, K)
+    x[:, :12] = torch.randperm(12, generator=torch.Generator().manual_seed(1)).float() * -0.03125      # no two alike
+    x[0, [0, 4, 5, 8]] = torch.tensor([3.0, 2.5, 2.375, 1.0])      # groups of four: 0 has one high score, 1 two, 2 a low one
+    x[1, [3, 9, 10, 11]] = torch.tensor([1.0, 3.0, 2.0, 1.5])
+    x[2, :12] = torch.arange(12.0) * 0.125
+    for corr in (torch.zeros(12), torch.full((12,), -5.0), torch.arange(12.0) * -0.3, torch.arange(12.0) * 0.5):
+        for keep, top in ((1, 3), (2, 3), (2, 8), (3, 12)):
+            r = {"groups": {"count": 3, "keep": keep}, "top": top, "scale": 2.0}
+            best, w = O.route(x.double(), r, {"router": eye.double() * 2, "correction": corr.double()})
+            ids, wts = ops.moe_route_groups(x.to(device, dtype), (eye * 2).to(device, dtype), corr.to(device), top, 3, keep, 2.0)
+            a, b = (i.cpu().long().sort(-1) for i in (ids, best))
+            assert torch.equal(a.values, b.values), (corr[1], keep, top)
+            close(wts.cpu().gather(1, a.indices), w.gather(1, b.indices))
+            assert torch.allclose(wts.sum(-1).cpu(), torch.full((3,), 2.0))
+
+
+def clamp_case(device, dtype):
+    """Gates far past the limit on either side, up rows on both: what is cut and what is not."""
+    K, F = 64, 32
+    x = torch.ones(6, K) * torch.tensor([-8.0, -1.0, -0.1, 0.1, 1.0, 8.0])[:, None]
+    up = torch.ones(1, 2, F, K) * 0.125
+    up[0, 1] *= torch.where(torch.arange(F) % 2 == 0, 1.0, -1.0)[:, None]
+    down = rnd(1, 1, K, F).to(BF16).float()
+    ids, wts = torch.zeros(6, 1, dtype=torch.int32), torch.ones(6, 1)
+    for limit in (0.5, 7.0, 100.0):
+        want = O.expert(x.to(dtype).float(), {"gate": up[0, 0], "up": up[0, 1], "down": down[0]}, limit)
+        got = ops.moe_experts(x.to(device, dtype), ids.to(device), wts.to(device), up.to(device, dtype), down.to(device, dtype), limit)[0]
+        close(got, want, dtype, limit)
