@@ -76,17 +76,18 @@ def main() -> None:
                          "flat search over the whole corpus (exit 3 on a mismatch); untimed.  Default: on "
                          "whenever WORLD_SIZE > 1 (the sharded index), off on one GPU")
     ap.add_argument("--no-check-retrieval", dest="check_retrieval", action="store_false")
-    ap.add_argument("--arch", choices=("rag", "saritar", "dolodra", "gezozen"), default="rag",
-                    help="rag: the headline workload; saritar, dolodra, gezozen: prefill / decode throughput and kernel times "
-                         "of that decoder's layers beside a Llama of equal size (benchmarks/bench_hybrid.py, bench_latent.py, "
-                         "bench_linear.py)")
-    ap.add_argument("--arch-sizes", default="2b,8b", help="--arch saritar, dolodra, gezozen: layer sizes, comma-separated")
+    ap.add_argument("--arch", choices=("rag", "saritar", "dolodra", "gezozen", "pifazen"), default="rag",
+                    help="rag: the headline workload; saritar, dolodra, gezozen, pifazen: prefill / decode throughput and kernel "
+                         "times of that decoder's layers beside a Llama of equal size (benchmarks/bench_hybrid.py, "
+                         "bench_latent.py, bench_linear.py, bench_channel_delta.py)")
+    ap.add_argument("--arch-sizes", default="2b,8b", help="--arch saritar, dolodra, gezozen, pifazen: layer sizes, comma-separated")
     ap.add_argument("--arch-part", choices=("all", "models", "kernels"), default="all")
     a = ap.parse_args()
     if a.arch != "rag":
-        from benchmarks import bench_hybrid, bench_latent, bench_linear
+        from benchmarks import bench_channel_delta, bench_hybrid, bench_latent, bench_linear
 
-        {"saritar": bench_hybrid, "dolodra": bench_latent, "gezozen": bench_linear}[a.arch].main(a)
+        {"saritar": bench_hybrid, "dolodra": bench_latent, "gezozen": bench_linear,
+         "pifazen": bench_channel_delta}[a.arch].main(a)
         return
     os.environ["QA_TEMPLATE"] = a.template or os.environ.get("QA_TEMPLATE", "cache_friendly")
 

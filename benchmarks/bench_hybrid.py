@@ -274,8 +274,8 @@ def beside_like(out: list[dict]) -> list[dict]:
     return out
 
 
-def main(args, name: str = "saritar", build=build_model, kernels=bench_kernels) -> None:
-    """Every row of design ``name`` and of the Llama beside it, as JSON lines."""
+def main(args, name: str = "saritar", build=build_model, kernels=bench_kernels, beside: tuple = ("llama",)) -> None:
+    """Every row of design ``name`` and of the models ``beside`` it, as JSON lines."""
     from docqa_amd import ops
 
     assert ops.load_native(), ops.native_error()
@@ -283,15 +283,16 @@ def main(args, name: str = "saritar", build=build_model, kernels=bench_kernels) 
     t0 = time.time()
     for size in args.arch_sizes.split(","):
         if args.arch_part in ("all", "models"):
-            rows = []
-            for kind in (name, "llama"):
+            rows = {}
+            for kind in (name, *beside):
+                rows[kind] = []
                 for r in bench_model(kind, size, args.warmup, args.steps, build):
-                    rows.append(r)
+                    rows[kind].append(r)
                     print(json.dumps(r), flush=True)
-            half = len(rows) // 2
-            for a, b in zip(rows[:half], rows[half:]):
-                print(json.dumps({"size": size, "phase": a["phase"], "batch": a["batch"], "tokens": a.get("tokens", a["batch"]),
-                                  f"{name}_over_llama": round(a["tokens_per_s"] / b["tokens_per_s"], 2)}), flush=True)
+            for kind in beside:
+                for a, b in zip(rows[name], rows[kind]):
+                    print(json.dumps({"size": size, "phase": a["phase"], "batch": a["batch"], "tokens": a.get("tokens", a["batch"]),
+                                      f"{name}_over_{kind}": round(a["tokens_per_s"] / b["tokens_per_s"], 2)}), flush=True)
         if args.arch_part in ("all", "kernels"):
             for r in kernels(size):
                 print(json.dumps(r), flush=True)
