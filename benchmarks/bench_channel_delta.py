@@ -18,7 +18,7 @@ from .bench_linear import MFMA32
 
 # width, heads of both mixers, head dim, rotated dim, latent, query latent, inner size of decay and gate, experts,
 # identity experts, chosen, groups, kept, expert width, dense width (with which a layer's active weights are the Llama's)
-SIZES = {"2b": (2048, 16, 128, 64, 512, 768, 128, 16, 2, 4, 3, 2, 1792, 10752),
+SIZES = {"2b": (2048, 16, 128, 64, 512, 768, 128, 16, 2, 4, 3, 2, 1792, 10240),
          "8b": (4096, 32, 128, 64, 512, 1536, 128, 16, 2, 4, 3, 2, 3072, 18432)}
 YARN = (8.0, 4096.0, 32.0, 1.0)
 
@@ -142,8 +142,8 @@ def bench_kernels(size: str) -> list[dict]:
                 M * (nq + 3 * H * d + r) * 2, 2.0 * H * (2 * d + r) * pairs, like=like)
         o, P = [rnd(M, H * d) for _ in range(copies(M * H * d * 4))], rnd(M, pad(n_lat))
         g2, sc = [rnd(M, 2 * H * d) for _ in range(copies(M * H * d * 4))], torch.ones(M, device=dev)
-        row("head_gate (element)", ph, M, lambda i: ops.head_gate(o[i % len(o)], P, Q + D, 1), M * H * d * 6, like="glu")
-        row("head_gate (head)", ph, M, lambda i: ops.head_gate(o[i % len(o)], P, Q + D, d), M * H * d * 4, like="glu")
+        row("head_gate (element)", ph, M, lambda i: ops.head_gate(o[i % len(o)], (P, Q + D, 1, 0)), M * H * d * 6, like="glu")
+        row("head_gate (head)", ph, M, lambda i: ops.head_gate(o[i % len(o)], (P, Q + D, d, 0)), M * H * d * 4, like="glu")
         row("glu", ph, M, lambda i: ops.glu(g2[i % len(g2)], 0, H * d, sc), M * H * d * 6)
         del o, g2
         P = [rnd(M, FD) for _ in range(copies(M * FD * 4))]
@@ -192,8 +192,8 @@ def bench_kernels(size: str) -> list[dict]:
         row("latent_norm_store", ph, B, lambda i: ops.latent_norm_store(P, cs, slots, cache, qn, norm, eps, bf), B * (Q + D) * (S * eb + 2),
             like="latent_store")
         o = rnd(B, H * d)
-        row("head_gate (element)", ph, B, lambda i: ops.head_gate(o, P, Q + D, 1), B * H * d * (S * eb + 4), like="glu")
-        row("head_gate (head)", ph, B, lambda i: ops.head_gate(o, P, Q + D, d), B * H * (S * eb + d * 4), like="glu")
+        row("head_gate (element)", ph, B, lambda i: ops.head_gate(o, (P, Q + D, 1, 0)), B * H * d * (S * eb + 4), like="glu")
+        row("head_gate (head)", ph, B, lambda i: ops.head_gate(o, (P, Q + D, d, 0)), B * H * (S * eb + d * 4), like="glu")
         P, sc = ops.project(rnd(B, W), rnd(2 * H * d, W), True), torch.ones(B, device=dev)
         S, eb = (P.shape[0] if P.dim() == 3 else 1), P.element_size()
         row("glu", ph, B, lambda i: ops.glu(P, 0, H * d, sc), B * H * d * (2 * S * eb + 2))

@@ -46,6 +46,16 @@ void check_rows(const Tensor& t, int64_t rows, int64_t cols, const Tensor& like,
               name, ": rows [", rows, ", >= ", cols, "] of the activations' dtype expected");
 }
 
+// gates of `rows` rows of `n` head elements: columns [col, col + n / per) of P from row row0 on
+DocqaGate gate_args(const OptT& P, int64_t col, int64_t per, int64_t row0, int64_t rows, int64_t n) {
+  DocqaGate g{};
+  if (!P.has_value()) return g;
+  const Slabs p = slabs_of(*P);
+  TORCH_CHECK(per >= 1 && n % per == 0 && col >= 0 && col + n / per <= p.N && row0 >= 0 && row0 + rows <= p.M, "output gate: columns");
+  g.P = P->data_ptr(); g.f32 = is_f32(*P); g.S = p.S; g.slab = p.slab; g.ld = p.N; g.col = (int)col; g.per = (int)per; g.row0 = (int)row0;
+  return g;
+}
+
 Tensor sandwich_rmsnorm(const Tensor& P, Tensor residual, const Tensor& w_post, const OptT& add, const Tensor& w_next,
                         double eps, bool out_f32) {
   const Slabs p = slabs_of(P);
@@ -158,16 +168,13 @@ Tensor poly_norm(const Tensor& P, const Tensor& bias, const Tensor& act, int64_t
   return out;
 }
 
-Tensor head_gate(const Tensor& x, const Tensor& P, int64_t col, int64_t per) {
-  CHECK_ACT(x); CHECK_CONTIG(x); CHECK_ALIGN16(x); CHECK_ALIGN16(P);
-  const Slabs p = slabs_of(P);
-  TORCH_CHECK(x.dim() == 2 && x.size(0) == p.M && per >= 1 && x.size(1) % per == 0, "head_gate: shapes");
-  TORCH_CHECK(col >= 0 && col + x.size(1) / per <= p.N && (is_f32(P) || !is_f32(x)), "head_gate: columns");
+Tensor head_gate(const Tensor& x, const Tensor& P, int64_t col, int64_t per, int64_t row0) {
+  CHECK_ACT(x); CHECK_CONTIG(x); CHECK_ALIGN16(x);
+  TORCH_CHECK(x.dim() == 2, "head_gate: x must be [rows, heads * dim]");
+  const DocqaGate gate = gate_args(P, col, per, row0, x.size(0), x.size(1));
   c10::DeviceGuard g(x.device());
   auto y = at::empty_like(x);
-  CHECK_RC(docqa_head_gate(x.data_ptr(), is_f32(x), P.data_ptr(), is_f32(P), p.S, p.slab, p.N, (int)col, (int)per, y.data_ptr(),
-                           p.M, (int)x.size(1), stream()),
-           "head_gate");
+  CHECK_RC(docqa_head_gate(x.data_ptr(), is_f32(x), gate, y.data_ptr(), (int)x.size(0), (int)x.size(1), stream()), "head_gate");
   return y;
 }
 
@@ -341,7 +348,8 @@ Tensor qkv_rope_store(const Tensor& P, const OptT& bias, const OptT& qw, const O
 // window_attn in the latent space (one KV head, values = the first K elements of a cached row, K =
 // w.size(2)) followed by head_project with w [H, N, K]; bf16, sizes by docqa_latent_attn_ok
 Tensor latent_attn(const Tensor& q, const Tensor& cache, const Tensor& block_tables, const OptT& cu, const Tensor& ctx,
-                   int64_t max_q, double scale, int64_t window, const OptT& sink, const Tensor& w) {
+                   int64_t max_q, double scale, int64_t window, const OptT& sink, const Tensor& w, const OptT& gp, int64_t gcol,
+                   int64_t gper, int64_t grow) {
   CHECK_GPU(q); CHECK_BF16(q); CHECK_CONTIG(q); CHECK_GPU(cache); CHECK_BF16(cache); CHECK_CONTIG(cache);
   CHECK_GPU(w); CHECK_BF16(w); CHECK_CONTIG(w);
   TORCH_CHECK(cache.dim() == 4 && cache.size(1) == 1 && w.dim() == 3, "latent_attn: cache [blocks, 1, block, D], w [H, N, K]");
@@ -371,14 +379,15 @@ Tensor latent_attn(const Tensor& q, const Tensor& cache, const Tensor& block_tab
                              (int)max_q, T, H, D, DV, BS, (float)scale, (int)window, stream()),
            "latent_attn");
   auto y = at::empty({T, (int64_t)H * N}, q.options());
-  CHECK_RC(docqa_head_project(x.data_ptr(), pp, mp, ns, w.data_ptr(), y.data_ptr(), T, H, DV, N, 0, stream()),
+  const DocqaGate gate = gate_args(gp, gcol, gper, grow, T, (int64_t)H * N);
+  CHECK_RC(docqa_head_project(x.data_ptr(), pp, mp, ns, w.data_ptr(), y.data_ptr(), T, H, DV, N, 0, gate, stream()),
            "latent_attn values");
   return y;
 }
 
 Tensor packed_window_attn(const Tensor& q, const Tensor& kv, const Tensor& kr, int64_t H, int64_t dim, int64_t vdim,
                           const Tensor& cu, const Tensor& cu_k, int64_t max_q, double scale, int64_t window,
-                          const OptT& sink) {
+                          const OptT& sink, const OptT& gp, int64_t gcol, int64_t gper, int64_t grow) {
   CHECK_GPU(q); CHECK_BF16(q); CHECK_BF16(kv); CHECK_BF16(kr); CHECK_CONTIG(q); CHECK_CONTIG(kv); CHECK_CONTIG(kr);
   CHECK_GPU(kv); CHECK_GPU(kr);
   TORCH_CHECK(q.dim() == 2 && kv.dim() == 2 && kr.dim() == 2 && kr.size(0) == kv.size(0) && H >= 1, "packed_window_attn: shapes");
@@ -392,7 +401,7 @@ Tensor packed_window_attn(const Tensor& q, const Tensor& kv, const Tensor& kr, i
   CHECK_RC(docqa_packed_window_attn(q.data_ptr(), kv.data_ptr(), kr.data_ptr(), cu.data_ptr<int>(), cu_k.data_ptr<int>(),
                                     sink.has_value() ? sink->data_ptr<float>() : nullptr, out.data_ptr(), B, (int)max_q,
                                     (int)H, (int)d8, (int)r8, (int)vdim, (int)kv.size(1), (float)scale, (int)window,
-                                    stream()),
+                                    gate_args(gp, gcol, gper, grow, q.size(0), H * vdim), stream()),
            "packed_window_attn");
   return out;
 }
@@ -462,7 +471,7 @@ Tensor head_project(const Tensor& x, const Tensor& w, int64_t carry) {
   c10::DeviceGuard g(x.device());
   auto y = at::empty({x.size(0), w.size(0) * (w.size(1) + carry)}, x.options());
   CHECK_RC(docqa_head_project(x.data_ptr(), nullptr, nullptr, 1, w.data_ptr(), y.data_ptr(), (int)x.size(0), (int)w.size(0), (int)w.size(2),
-                              (int)w.size(1), (int)carry, stream()),
+                              (int)w.size(1), (int)carry, DocqaGate{}, stream()),
            "head_project");
   return y;
 }
@@ -842,7 +851,7 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
   m.def("scaled_rmsnorm(Tensor P, Tensor(a!) residual, Tensor scale, Tensor? bias, Tensor? ids, Tensor? wts, int experts, "
         "Tensor? x, Tensor w, float eps, bool out_f32) -> Tensor");
   m.def("poly_norm(Tensor P, Tensor bias, Tensor act, int n_out, float eps, bool out_f32) -> Tensor");
-  m.def("head_gate(Tensor x, Tensor P, int col, int per) -> Tensor");
+  m.def("head_gate(Tensor x, Tensor P, int col, int per, int row0) -> Tensor");
   m.def("latent_norm_store(Tensor P, Tensor cs, Tensor slots, Tensor(a!) cache, Tensor q_norm, Tensor c_norm, float eps) -> Tensor");
   m.def("low_rank(Tensor z, int at, Tensor wa, Tensor wg, int n) -> Tensor");
   m.def("moe_route_groups(Tensor x, Tensor w, Tensor corr, int top, int groups, int keep, float scale) -> (Tensor, Tensor)");
@@ -850,11 +859,11 @@ TORCH_LIBRARY_FRAGMENT(docqa, m) {
   m.def("side_gate(Tensor P, Tensor ids, Tensor table, int col, int n, bool out_f32) -> Tensor");
   m.def("side_project(Tensor P, Tensor ids, Tensor table, int col, int n, Tensor w) -> Tensor");
   m.def("latent_attn(Tensor q, Tensor cache, Tensor block_tables, Tensor? cu, Tensor ctx, int max_q, float scale, "
-        "int window, Tensor? sink, Tensor w) -> Tensor");
+        "int window, Tensor? sink, Tensor w, Tensor? gp, int gcol, int gper, int grow) -> Tensor");
   m.def("sandwich_rmsnorm_conv(Tensor P, Tensor(a!) residual, Tensor w_post, Tensor w_next, Tensor cw, "
         "Tensor(b!) state, Tensor slots, Tensor positions, float eps) -> (Tensor, Tensor)");
   m.def("packed_window_attn(Tensor q, Tensor kv, Tensor kr, int H, int dim, int vdim, Tensor cu, Tensor cu_k, int max_q, "
-        "float scale, int window, Tensor? sink) -> Tensor");
+        "float scale, int window, Tensor? sink, Tensor? gp, int gcol, int gper, int grow) -> Tensor");
   m.def("rope_table(Tensor positions, Tensor freq, float mult) -> Tensor");
   m.def("latent_store(Tensor P, Tensor cs, Tensor slots, Tensor(a!) cache, Tensor? c_norm, int H, int dim, int rank, "
         "float eps) -> Tensor");

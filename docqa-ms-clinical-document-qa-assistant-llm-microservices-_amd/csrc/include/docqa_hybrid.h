@@ -68,10 +68,17 @@ int docqa_window_attn(const void* q, const void* kc, const void* vc, const float
 int docqa_qkv_rope_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* bias, const float* qw,
                          const float* kw, const float* cs, int r, const int* slots, void* q, void* kc, void* vc, int f32,
                          int tokens, int H, int G, int D, int DV, int BS, float eps, hipStream_t s);
+// an output gate: row t's head elements i times sigmoid(P[row0 + t, col + i / per])
+struct DocqaGate {
+  const void* P;            // product or slabs; null: no gate
+  int f32, S;
+  size_t slab;
+  int ld, col, per, row0;
+};
 // kv [keys, ld] rows [H x d8 keys | H x v8 values], kr [keys, r8]; bf16
 int docqa_packed_window_attn(const void* q, const void* kv, const void* kr, const int* cu, const int* cu_k,
                              const float* sink, void* out, int B, int max_q, int H, int d8, int r8, int vdim, int ld,
-                             float scale, int window, hipStream_t s);
+                             float scale, int window, const DocqaGate& gate, hipStream_t s);
 
 int docqa_rope_table(const int* positions, const double* freq, float* out, int T, int half, double mult, hipStream_t s);
 // c_norm null: the projection holds query heads only
@@ -80,7 +87,7 @@ int docqa_latent_store(const void* P, int p_f32, int S, size_t slab, int ld, con
                        float eps, hipStream_t s);
 // part null: rows x; else the rows are docqa_latent_attn's nsplit partials (E = 0)
 int docqa_head_project(const void* x, const void* part, const void* ml, int nsplit, const void* w, void* y, int T, int H,
-                       int K, int N, int E, hipStream_t s);
+                       int K, int N, int E, const DocqaGate& gate, hipStream_t s);
 // attention in the latent space, bf16, one KV head, values = the first DV elements of a row (sizes:
 // latent_attn_ok).  nsplit > 1 (latent_splits): partials for docqa_head_project instead of out -- part
 // bf16 [nsplit, tokens H, DV] each split's output, ml float2 [nsplit, tokens H] (maximum, sum)
@@ -93,9 +100,7 @@ int docqa_latent_attn(const void* q, const void* kc, const int* block_tables, in
 int docqa_latent_norm_store(const void* P, int p_f32, int S, size_t slab, int ld, const float* cs, const int* slots,
                             const float* q_norm, const float* c_norm, void* cq, void* cache, int f32, int T, int Rq, int r,
                             int R, int BS, float eps, hipStream_t s);
-// y [T, n] = x sigmoid(P[:, col + i / per])
-int docqa_head_gate(const void* x, int f32, const void* P, int p_f32, int S, size_t slab, int ld, int col, int per, void* y,
-                    int T, int n, hipStream_t s);
+int docqa_head_gate(const void* x, int f32, const DocqaGate& gate, void* y, int T, int n, hipStream_t s);   // [T, n]
 int docqa_latent_gather(const void* cache, const int* block_tables, int maxb, const int* first, const int* cu_k, void* c,
                         void* kr, int B, int max_keys, int R8, int r8, int BS, hipStream_t s);
 

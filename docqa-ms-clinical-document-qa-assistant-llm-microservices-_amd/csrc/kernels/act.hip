@@ -9,6 +9,7 @@
 // Guideline 11 grid sizing: <= 2048 blocks, grid-stride the rest).
 #include "docqa_common.h"
 #include "docqa_elem.h"
+#include "docqa_gate.h"
 
 using namespace docqa;
 
@@ -407,19 +408,27 @@ __global__ __launch_bounds__(NT) void poly_norm_kernel(const PT* __restrict__ P,
   }
 }
 
-template <int V, typename PT, typename OT>
+template <int NT, int V, typename PT, typename OT>
 static int launch_poly_norm(const PT* P, int S, size_t slab, int ld, const float* bias, const float* act, OT* out, int T, int n,
                             int n_out, float eps, hipStream_t s) {
-  const int m = n_out / V;
-#define GO(NT, NV) poly_norm_kernel<NT, NV, V, PT, OT><<<T, NT, 0, s>>>(P, S, slab, ld, bias, act, out, n, n_out, eps)
-  if (m <= 256) GO(256, 1);
-  else if (m <= 512) GO(256, 2);
-  else if (m <= 1024) GO(256, 4);
-  else if (m <= 2048) GO(1024, 2);
-  else if (m <= 4096) GO(1024, 4);
-  else if (m <= 8192) GO(1024, 8);
-  else if (V == 1 && m <= 32768) GO(1024, (V == 1 ? 32 : 8));
-  else return -1;
+  constexpr int MAX = V == 1 ? 32 : 64 / V;      // most pieces a thread
+  const int nv = (n_out / V + NT - 1) / NT;
+#define GO(NV)                                                                                                          \
+  do {                                                                                                                  \
+    constexpr int M = NV < MAX ? NV : MAX;                                                                              \
+    poly_norm_kernel<NT, M, V, PT, OT><<<T, NT, 0, s>>>(P, S, slab, ld, bias, act, out, n, n_out, eps);                 \
+  } while (0)
+  if (nv > MAX) return -1;
+  switch (nv) {
+    case 1: GO(1); break;
+    case 2: GO(2); break;
+    case 3: GO(3); break;
+    case 4: GO(4); break;
+    case 5: GO(5); break;
+    case 6: GO(6); break;
+    case 7: case 8: GO(8); break;
+    default: GO(32);                             // (MAX pieces)
+  }
 #undef GO
   DOCQA_CHECK_LAUNCH();
   return 0;
@@ -428,9 +437,18 @@ static int launch_poly_norm(const PT* P, int S, size_t slab, int ld, const float
 template <typename PT, typename OT>
 static int poly_norm_vec(const void* P, int S, size_t slab, int ld, const float* bias, const float* act, void* out, int T, int n,
                          int n_out, float eps, hipStream_t s) {
-  if (n % 4 == 0 && n_out % 4 == 0 && ld % 4 == 0)
-    return launch_poly_norm<4, PT, OT>((const PT*)P, S, slab, ld, bias, act, (OT*)out, T, n, n_out, eps, s);
-  return launch_poly_norm<1, PT, OT>((const PT*)P, S, slab, ld, bias, act, (OT*)out, T, n, n_out, eps, s);
+#define GO(NT, V) return launch_poly_norm<NT, V, PT, OT>((const PT*)P, S, slab, ld, bias, act, (OT*)out, T, n, n_out, eps, s)
+  if (n % 4 || n_out % 4 || ld % 4) {
+    if (n_out <= 8192) GO(256, 1);
+    GO(1024, 1);
+  }
+  if (n_out <= 4096) GO(256, 4);
+  if (n % 8 == 0 && n_out % 8 == 0 && ld % 8 == 0) {
+    if (T <= 512 || n_out > 32768) GO(1024, 8);
+    GO(512, 8);
+  }
+  GO(1024, 4);
+#undef GO
 }
 
 int docqa_poly_norm(const void* P, int p_f32, int S, size_t slab, int ld, const float* bias, const float* act, void* out,
@@ -443,48 +461,34 @@ int docqa_poly_norm(const void* P, int p_f32, int S, size_t slab, int ld, const 
 #undef ARGS
 }
 
-// y [T, n] = x sigmoid(P[:, col + i / per]): an output gate, one number an element or (per > 1) a head
-template <int V, typename T, typename PT>
-__global__ __launch_bounds__(256) void head_gate_kernel(const T* __restrict__ x, const PT* __restrict__ P, int S, size_t slab,
-                                                        int ld, int col, int per, T* __restrict__ y, int rows, int n) {
+// heads times their output gate, where no kernel that writes them takes it (docqa_gate.h)
+template <int V, typename T>
+__global__ __launch_bounds__(256) void head_gate_kernel(const T* __restrict__ x, DocqaGate gate, T* __restrict__ y, int rows, int n) {
   const int m = n / V;
   const size_t total = (size_t)rows * m;
   for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
     const size_t t = i / m;
     const int c = (int)(i - t * m) * V;
-    float f[V], g[V];
+    float f[V];
     docqa::ldv<V>(x + t * n + c, f);
-    if (per == 1) {
-      docqa::ld_slabs<V>(P + t * ld + col + c, S, slab, g);
-    } else {
-      docqa::ld_slabs<1>(P + t * ld + col + c / per, S, slab, g);
-#pragma unroll
-      for (int j = 1; j < V; ++j) g[j] = g[0];
-    }
-#pragma unroll
-    for (int j = 0; j < V; ++j) f[j] /= 1.f + expf(-g[j]);
+    docqa::apply_gate<V>(gate, t, c, f);
     docqa::stv<V>(y + t * n + c, f);
   }
 }
 
-template <typename T, typename PT>
-static int launch_head_gate(const void* x, const void* P, int S, size_t slab, int ld, int col, int per, void* y, int rows, int n,
-                            hipStream_t s) {
-  const bool vec = n % 4 == 0 && (per == 1 ? ld % 4 == 0 && col % 4 == 0 : per % 4 == 0);
-  const size_t g = ((size_t)rows * (n / (vec ? 4 : 1)) + 255) / 256;
+int docqa_head_gate(const void* x, int f32, const DocqaGate& gate, void* y, int T, int n, hipStream_t s) {
+  if (T == 0) return 0;
+  if (!gate.P || gate.S < 1 || n < 1 || gate.per < 1 || n % gate.per || gate.col < 0 || gate.col + n / gate.per > gate.ld) return -1;
+  const bool vec = n % 4 == 0 && docqa_gate_vec(gate, 4);
+  const size_t g = ((size_t)T * (n / (vec ? 4 : 1)) + 255) / 256;
   const int grid = (int)(g < 8192 ? g : 8192);
-  if (vec) head_gate_kernel<4, T, PT><<<grid, 256, 0, s>>>((const T*)x, (const PT*)P, S, slab, ld, col, per, (T*)y, rows, n);
-  else head_gate_kernel<1, T, PT><<<grid, 256, 0, s>>>((const T*)x, (const PT*)P, S, slab, ld, col, per, (T*)y, rows, n);
+  if (f32) {
+    if (vec) head_gate_kernel<4, float><<<grid, 256, 0, s>>>((const float*)x, gate, (float*)y, T, n);
+    else head_gate_kernel<1, float><<<grid, 256, 0, s>>>((const float*)x, gate, (float*)y, T, n);
+  } else {
+    if (vec) head_gate_kernel<4, uint16_t><<<grid, 256, 0, s>>>((const uint16_t*)x, gate, (uint16_t*)y, T, n);
+    else head_gate_kernel<1, uint16_t><<<grid, 256, 0, s>>>((const uint16_t*)x, gate, (uint16_t*)y, T, n);
+  }
   DOCQA_CHECK_LAUNCH();
   return 0;
-}
-
-int docqa_head_gate(const void* x, int f32, const void* P, int p_f32, int S, size_t slab, int ld, int col, int per, void* y,
-                    int T, int n, hipStream_t s) {
-  if (T == 0) return 0;
-  if (S < 1 || n < 1 || per < 1 || n % per || col < 0 || col + n / per > ld || (f32 && !p_f32)) return -1;
-#define ARGS x, P, S, slab, ld, col, per, y, T, n, s
-  if (f32) return launch_head_gate<float, float>(ARGS);
-  return p_f32 ? launch_head_gate<uint16_t, float>(ARGS) : launch_head_gate<uint16_t, uint16_t>(ARGS);
-#undef ARGS
 }

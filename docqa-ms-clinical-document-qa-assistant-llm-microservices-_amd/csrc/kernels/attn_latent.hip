@@ -10,7 +10,8 @@
 //                    launch, and a second one rotates the heads its projection makes;
 //   * absorbed form (decode, short portions): head_project takes the query heads into the latent
 //     space, every head attends the cached rows themselves -- key and value at once -- and
-//     head_project takes the attended latents to values (summing the key splits on the way);
+//     head_project takes the attended latents to values (summing the key splits on the way, an
+//     output gate in its epilogue);
 //   * expanded form (prompts): latent_gather packs the visible rows, a GEMM makes every head's
 //     keys and values of them, attn_window.hip's packed form attends.
 //
@@ -22,6 +23,7 @@
 // sequences: the keys are split over workgroups; the value projection sums the splits' outputs.
 #include "docqa_common.h"
 #include "docqa_elem.h"
+#include "docqa_gate.h"
 #include "docqa_hybrid.h"
 
 using namespace docqa;
@@ -154,12 +156,12 @@ __global__ __launch_bounds__(256) void latent_store_kernel(const PT* __restrict_
 // rows are attended latents as key splits' outputs, x = sum_s w_s part_s, w_s = e^(m_s - m) l_s / sum.
 constexpr int kMaxSplit = 32;
 
-template <int MT, int NJ, bool MERGE>
+template <int MT, int NJ, bool MERGE, bool GATE>
 __global__ __launch_bounds__(256) void head_project_kernel(const uint16_t* __restrict__ x,
                                                            const uint16_t* __restrict__ part,
                                                            const float2* __restrict__ ml, int nsplit,
                                                            const uint16_t* __restrict__ w, uint16_t* __restrict__ y,
-                                                           int T, int H, int K, int N, int E) {
+                                                           int T, int H, int K, int N, int E, DocqaGate gate) {
   extern __shared__ __attribute__((aligned(16))) uint16_t sx[];       // [16 MT][pitch]
   __shared__ float sw[MERGE ? 16 * MT : 1][kMaxSplit];                // a row's weight of each split
   const int kp = (K + 31) / 32 * 32, pitch = kp + 8;
@@ -255,13 +257,18 @@ __global__ __launch_bounds__(256) void head_project_kernel(const uint16_t* __res
       uint16_t* op = yh + (size_t)row * ldy + n;
       if (N % 4 == 0) {
         if (n < N) {
-          const float f[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
+          float f[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
+          if constexpr (GATE) apply_gate<4>(gate, row, h * N + n, f);
           stv<4>(op, f);
         }
       } else {
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          if (n + r < N) op[r] = f2bf(acc[i][j][r]);
+          if (n + r < N) {
+            float f = acc[i][j][r];
+            if constexpr (GATE) apply_gate<1>(gate, row, h * N + n + r, &f);
+            op[r] = f2bf(f);
+          }
       }
     }
   }
@@ -656,28 +663,31 @@ int docqa_latent_norm_store(const void* P, int p_f32, int S, size_t slab, int ld
 }
 
 int docqa_head_project(const void* x, const void* part, const void* ml, int nsplit, const void* w, void* y, int T, int H,
-                       int K, int N, int E, hipStream_t s) {
+                       int K, int N, int E, const DocqaGate& gate, hipStream_t s) {
   if (T == 0) return 0;
+  if (gate.P && (E > 0 || (N % 4 == 0 && !docqa_gate_vec(gate, 4)))) return -1;
   if (H < 1 || K < 8 || K % 8 || K > 2048 || N < 1 || E < 0 || E % 8 || (E > 0 && N % 8)) return -1;
   if (!docqa_aligned16(w) || !docqa_aligned16(y) || !docqa_aligned16(part ? part : x)) return -1;
   if (part && (!ml || nsplit < 1 || nsplit > kMaxSplit || E > 0)) return -1;
   const int pitch = (K + 31) / 32 * 32 + 8;
-#define LAUNCH(MT, NJ, MERGE)                                                                                         \
+#define LAUNCH(MT, NJ, MERGE, GATE)                                                                                         \
   do {                                                                                                                \
     const size_t lds = (size_t)16 * MT * pitch * 2;                                                                   \
-    auto kern = head_project_kernel<MT, NJ, MERGE>;                                                                   \
+    auto kern = head_project_kernel<MT, NJ, MERGE, GATE>;                                                                   \
     if (lds > 56 * 1024) {                                                                                            \
       static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern),                            \
                                                       hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 1024);         \
       if (e != hipSuccess) return (int)e;                                                                             \
     }                                                                                                                 \
     kern<<<dim3(H, (T + 16 * MT - 1) / (16 * MT), (N + 64 * NJ - 1) / (64 * NJ)), 256, lds, s>>>(                     \
-        (const uint16_t*)x, (const uint16_t*)part, (const float2*)ml, nsplit, (const uint16_t*)w, (uint16_t*)y, T, H, K, N, E);        \
+        (const uint16_t*)x, (const uint16_t*)part, (const float2*)ml, nsplit, (const uint16_t*)w, (uint16_t*)y, T, H, K, N, E, gate);  \
   } while (0)
 #define GO(MT, NJ)                       \
   do {                                   \
-    if (part) LAUNCH(MT, NJ, true);      \
-    else LAUNCH(MT, NJ, false);          \
+    if (part && gate.P) LAUNCH(MT, NJ, true, true);  \
+    else if (part) LAUNCH(MT, NJ, true, false);      \
+    else if (gate.P) LAUNCH(MT, NJ, false, true);    \
+    else LAUNCH(MT, NJ, false, false);               \
   } while (0)
   if (T > 64 && K <= 256) GO(4, 2);
   else if (T > 64 && K <= 1024) GO(2, 2);

@@ -18,6 +18,7 @@
 //   up to 256 elements run on MFMA, fp32 and odd head sizes on a wave-per-row kernel.
 #include "docqa_common.h"
 #include "docqa_elem.h"
+#include "docqa_gate.h"
 #include <float.h>
 #include <type_traits>
 
@@ -102,6 +103,7 @@ struct WindowArgs {
   const int* cu_k;
   const uint16_t* kr;
   int ld, kd, vd;
+  DocqaGate gate;         // packed form
 };
 
 // LDS written by some lanes of a wave and read by others: in order in hardware, so only the
@@ -499,10 +501,11 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void window_attn_mfma_ker
       for (int i = 0; i < NDT; ++i) {
         const int c = i * 16 + g4 * 4;
         if (c < DV) {
-          uint2 v;
-          v.x = pack2(o[t][i][0] * inv, o[t][i][1] * inv);
-          v.y = pack2(o[t][i][2] * inv, o[t][i][3] * inv);
-          *reinterpret_cast<uint2*>(op + c) = v;
+          float f[4] = {o[t][i][0] * inv, o[t][i][1] * inv, o[t][i][2] * inv, o[t][i][3] * inv};
+          if constexpr (PACKED) {
+            if (a.gate.P) apply_gate<4>(a.gate, q0 + r, kvh * DV + c, f);
+          }
+          stv<4>(op + c, f);
         }
       }
     }
@@ -799,7 +802,7 @@ int docqa_window_attn(const void* q, const void* kc, const void* vc, const float
   int log2BS = 0;
   while ((1 << log2BS) < BS) ++log2BS;
   const WindowArgs a{block_tables, maxb, cu, ctx, k_scale, sink, H, G, D, BS, log2BS, scale, window, DV,
-                     shared ? D : DV, cap, out_scale, ldo, nullptr, nullptr, 0, 0, 0};
+                     shared ? D : DV, cap, out_scale, ldo, nullptr, nullptr, 0, 0, 0, {}};
   // rows are stored 8 bytes at a time
   const bool stores = ldo % 4 == 0 && DV % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & 7) == 0;
   if (!f32 && D % 8 == 0 && DV % 8 == 0 && D <= 256 && DV <= 256 && (!shared || DV == D) && docqa_aligned16(q) && stores)
@@ -826,14 +829,15 @@ int docqa_window_attn(const void* q, const void* kc, const void* vc, const float
 
 int docqa_packed_window_attn(const void* q, const void* kv, const void* kr, const int* cu, const int* cu_k,
                              const float* sink, void* out, int B, int max_q, int H, int d8, int r8, int vdim, int ld,
-                             float scale, int window, hipStream_t s) {
+                             float scale, int window, const DocqaGate& gate, hipStream_t s) {
   if (B == 0 || max_q == 0) return 0;
+  if (gate.P && !docqa_gate_vec(gate, 4)) return -1;
   const int D = d8 + r8, v8 = (vdim + 7) / 8 * 8;
   if (H < 1 || d8 < 8 || d8 % 8 || r8 < 0 || r8 % 8 || D > 256 || vdim < 4 || vdim % 4 || vdim > 256) return -1;
   if (ld % 8 || ld < H * (d8 + v8) || B > 65535) return -1;
   if (!docqa_aligned16(q) || !docqa_aligned16(kv) || !docqa_aligned16(kr) || !docqa_aligned16(out)) return -1;
   const WindowArgs a{nullptr, 0, cu, nullptr, nullptr, sink, H, H, D, 64, 6, scale, window, vdim, 0, 0.f, 1.f, H * vdim,
-                     cu_k, (const uint16_t*)kr, ld, d8, v8};
+                     cu_k, (const uint16_t*)kr, ld, d8, v8, gate};
   const uint16_t* v = (const uint16_t*)kv + (size_t)H * d8;
   // 128 query rows a workgroup, 64 where that leaves CUs without one
   const bool few = (long long)B * H * ((max_q + 127) / 128) < 384;

@@ -740,23 +740,21 @@ class LatentAttention:
         for p in parts:
             m, qp = p.meta, _split(q, p, parts)
             keys = None if p.decode else fw.keys.get(sp.window)
+            kw = dict(window=sp.window, sink=self.sink,
+                      gate=(P, self.gate_at, sp.vdim if sp.gate == "head" else 1, p.lo) if sp.gate else None)
             if self._expanded(keys):
                 c, kr = ops.latent_gather(cache, m.block_tables, keys.first, keys.cu, keys.total, self.R8)
                 out.append(ops.packed_window_attn(qp, ops.linear(c, self.w_kv), kr, sp.heads, sp.dim, sp.vdim, m.cu_seqlens,
-                                                  keys.cu, m.max_len, sp.scale, window=sp.window, sink=self.sink))
+                                                  keys.cu, m.max_len, sp.scale, **kw))
                 continue
             qc = ops.head_project(qp, self.w_qc, self.r8)
-            kw = dict(window=sp.window, sink=self.sink)
             if p.decode:
                 a = ops.latent_attn(qc, cache, m.block_tables, m.context_lens, sp.scale, self.w_cv, **kw)
             else:
                 a = ops.latent_attn(qc, cache, m.block_tables, m.prefix_lens, sp.scale, self.w_cv, cu=m.cu_seqlens,
                                     max_q=m.max_len, **kw)
             out.append(a)
-        o = _join(out)
-        if sp.gate:
-            o = ops.head_gate(o, P, self.gate_at, sp.vdim if sp.gate == "head" else 1)
-        return ops.project(o, self.o, decode)
+        return ops.project(_join(out), self.o, decode)
 
 
 class MLP:

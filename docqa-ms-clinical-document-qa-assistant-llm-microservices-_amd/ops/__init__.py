@@ -1412,12 +1412,17 @@ def latent_norm_store(P, cs, slots, cache, q_norm, c_norm, eps: float, dtype):
     return ref.latent_norm_store(P, cs, slots, cache, q_norm, c_norm, eps, dtype)
 
 
-def head_gate(x, P, col: int, per: int):
-    """x [T, n] times sigmoid of columns [col, col + n / per) of a projection, ``per`` neighbours each
-    sharing one."""
+def head_gate(x, gate):
+    """x [T, n] times an output gate (P, col, per, row): sigmoid of columns [col, col + n / per) of the
+    projection's rows from ``row`` on, ``per`` neighbours each sharing one."""
+    P, col, per, row = gate
     if _gpu(x):
-        return _native().head_gate(x.contiguous(), P.contiguous(), int(col), int(per))
-    return ref.head_gate(x, P, col, per)
+        return _native().head_gate(x.contiguous(), P.contiguous(), int(col), int(per), int(row))
+    return ref.head_gate(x, P, col, per, row)
+
+
+def _gate_args(gate) -> tuple:
+    return (None, 0, 1, 0) if gate is None else (gate[0].contiguous(), *map(int, gate[1:]))
 
 
 def head_project(x, w, carry: int = 0):
@@ -1431,17 +1436,17 @@ def head_project(x, w, carry: int = 0):
 _LATENT_ROW = {64: 128, 128: 192, 256: 320, 512: 576}      # latent columns -> row elements, attn_latent.hip
 
 
-def latent_attn(q, cache, block_tables, ctx, scale: float, w, window: int = 0, sink=None, cu=None, max_q: int = 1):
+def latent_attn(q, cache, block_tables, ctx, scale: float, w, window: int = 0, sink=None, cu=None, max_q: int = 1, gate=None):
     """Attention in the latent space and the projection of what it attends: :func:`window_attn` of
     queries [T, H (R8 + r8)] over the cached rows, whose first R8 elements are the values, then
-    :func:`head_project` with ``w`` [H, vdim, R8].  bf16 rows run on MFMA, the keys split over
-    workgroups where sequences are few and summed by the projection."""
+    :func:`head_project` with ``w`` [H, vdim, R8] and :func:`head_gate` of a ``gate``.  bf16 rows run on
+    MFMA, the keys split over workgroups where sequences are few and summed by the projection."""
     K, D = w.shape[2], cache.shape[3]
     if _gpu(q) and q.dtype == torch.bfloat16 and D <= next((_LATENT_ROW[n] for n in _LATENT_ROW if K <= n), 0):
         return _native().latent_attn(q.contiguous(), cache, block_tables, cu, ctx, int(max_q), float(scale), int(window),
-                                     sink, w)
-    return head_project(window_attn(q, cache, block_tables, ctx, scale, window=window, sink=sink, cu=cu, max_q=max_q,
-                                    v_dim=K), w)
+                                     sink, w, *_gate_args(gate))
+    y = head_project(window_attn(q, cache, block_tables, ctx, scale, window=window, sink=sink, cu=cu, max_q=max_q, v_dim=K), w)
+    return y if gate is None else head_gate(y, gate)
 
 
 def latent_gather(cache, block_tables, first, cu_k, total: int, rank: int):
@@ -1453,14 +1458,16 @@ def latent_gather(cache, block_tables, first, cu_k, total: int, rank: int):
 
 
 def packed_window_attn(q, kv, kr, H: int, dim: int, vdim: int, cu, cu_k, max_q: int, scale: float, window: int = 0,
-                       sink=None):
+                       sink=None, gate=None):
     """Causal attention of packed queries [T, H (d8 + r8)] over packed keys and values: ``kv``
     [keys, >= H d8 + H v8] per-head keys then values, ``kr`` [keys, r8] the key part all heads
-    share.  Sequence b's keys end at its last query token.  [T, H vdim]."""
+    share.  Sequence b's keys end at its last query token.  [T, H vdim], through :func:`head_gate` of a
+    ``gate``."""
     if _gpu(q):
         return _native().packed_window_attn(q.contiguous(), kv, kr, int(H), int(dim), int(vdim), cu, cu_k, int(max_q),
-                                            float(scale), int(window), sink)
-    return ref.packed_window_attn(q, kv, kr, H, dim, vdim, cu, cu_k, scale, window, sink)
+                                            float(scale), int(window), sink, *_gate_args(gate))
+    y = ref.packed_window_attn(q, kv, kr, H, dim, vdim, cu, cu_k, scale, window, sink)
+    return y if gate is None else head_gate(y, gate)
 
 
 def packed_attn_ok(dtype, dim: int, rot: int, vdim: int) -> bool:

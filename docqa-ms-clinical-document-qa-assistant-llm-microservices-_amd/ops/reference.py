@@ -446,9 +446,9 @@ def latent_norm_store(P, cs, slots, cache, q_norm, c_norm, eps, dtype):
     return (_rms(x[:, :n], eps) * q_norm).to(dtype)
 
 
-def head_gate(x, P, col, per):
+def head_gate(x, P, col, per, row):
     T, n = x.shape
-    g = torch.sigmoid(_slab_sum(P)[:, col:col + n // per])
+    g = torch.sigmoid(_slab_sum(P)[row:row + T, col:col + n // per])
     return (x.float().view(T, -1, per) * g[..., None]).view(T, n).to(x.dtype)
 
 
