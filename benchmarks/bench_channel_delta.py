@@ -136,16 +136,16 @@ def bench_kernels(size: str) -> list[dict]:
         row("latent_store", ph, M, lambda i: ops.latent_store(P[i % len(P)], cs, slots, cache, norm, H, d, R, eps, bf), M * ((nq + D) * 4 + r * 4))
         del P
         q, kv, kr, sink = rnd(M, nq), rnd(M, 2 * H * d), rnd(M, r), torch.zeros(H, device=dev)
-        for name, win, s, like in (("packed_attn", 0, None, "packed_window_attn"), ("packed_window_attn", 1024, sink, "")):
-            pairs = sum(min(p + 1, win or M) for p in range(M))
-            row(name, ph, M, lambda i: ops.packed_window_attn(q, kv, kr, H, d, d, cu, cu, M, (d + r) ** -0.5, win, s),
-                M * (nq + 3 * H * d + r) * 2, 2.0 * H * (2 * d + r) * pairs, like=like)
-        o, P = [rnd(M, H * d) for _ in range(copies(M * H * d * 4))], rnd(M, pad(n_lat))
+        P = rnd(M, pad(n_lat))
+        for name, win, s, gate, like in (("packed_attn (gate an element)", 0, None, (P, Q + D, 1, 0), "packed_window_attn"),
+                                         ("packed_attn (gate a head)", 0, None, (P, Q + D, d, 0), "packed_window_attn"),
+                                         ("packed_window_attn", 1024, sink, None, "")):
+            pairs, ng = sum(min(p + 1, win or M) for p in range(M)), 0 if gate is None else H * d // gate[2]
+            row(name, ph, M, lambda i: ops.packed_window_attn(q, kv, kr, H, d, d, cu, cu, M, (d + r) ** -0.5, win, s, gate),
+                M * (nq + 3 * H * d + r + ng) * 2, 2.0 * H * (2 * d + r) * pairs, like=like)
         g2, sc = [rnd(M, 2 * H * d) for _ in range(copies(M * H * d * 4))], torch.ones(M, device=dev)
-        row("head_gate (element)", ph, M, lambda i: ops.head_gate(o[i % len(o)], (P, Q + D, 1, 0)), M * H * d * 6, like="glu")
-        row("head_gate (head)", ph, M, lambda i: ops.head_gate(o[i % len(o)], (P, Q + D, d, 0)), M * H * d * 4, like="glu")
         row("glu", ph, M, lambda i: ops.glu(g2[i % len(g2)], 0, H * d, sc), M * H * d * 6)
-        del o, g2
+        del g2
         P = [rnd(M, FD) for _ in range(copies(M * FD * 4))]
         row("poly_norm", ph, M, lambda i: ops.poly_norm(P[i % len(P)], fb, act, FD, eps), M * FD * 4, like="activation")
         row("activation", ph, M, lambda i: ops.activation(P[i % len(P)], "gelu_tanh"), M * FD * 4)
@@ -191,9 +191,7 @@ def bench_kernels(size: str) -> list[dict]:
         S, eb = (P.shape[0] if P.dim() == 3 else 1), P.element_size()
         row("latent_norm_store", ph, B, lambda i: ops.latent_norm_store(P, cs, slots, cache, qn, norm, eps, bf), B * (Q + D) * (S * eb + 2),
             like="latent_store")
-        o = rnd(B, H * d)
-        row("head_gate (element)", ph, B, lambda i: ops.head_gate(o, (P, Q + D, 1, 0)), B * H * d * (S * eb + 4), like="glu")
-        row("head_gate (head)", ph, B, lambda i: ops.head_gate(o, (P, Q + D, d, 0)), B * H * (S * eb + d * 4), like="glu")
+        gp, ge = P, S * eb
         P, sc = ops.project(rnd(B, W), rnd(2 * H * d, W), True), torch.ones(B, device=dev)
         S, eb = (P.shape[0] if P.dim() == 3 else 1), P.element_size()
         row("glu", ph, B, lambda i: ops.glu(P, 0, H * d, sc), B * H * d * (2 * S * eb + 2))
@@ -207,10 +205,12 @@ def bench_kernels(size: str) -> list[dict]:
         bt = i32(torch.arange(B * nbs).view(B, nbs))
         caches = [rnd(B * nbs, 1, BS, D) for _ in range(copies(B * nbs * BS * D * 2))]
         qc, sink, wv = rnd(B, H * D), torch.zeros(H, device=dev), [rnd(H, d, R) for _ in range(8)]
-        for name, win, s, like in (("latent_attn", 0, None, "latent_attn (window)"), ("latent_attn (window)", 1024, sink, "")):
-            n = win or 1025
-            row(name, ph, B, lambda i: ops.latent_attn(qc, caches[i % len(caches)], bt, ctx, (d + r) ** -0.5, wv[i % 8], window=win, sink=s),
-                (B * (n * D + H * (D + d)) + H * d * R) * 2.0, 2.0 * B * H * (n * (D + R) + d * R), like=like)
+        for name, win, s, gate, like in (("latent_attn (gate an element)", 0, None, (gp, Q + D, 1, 0), "latent_attn (window)"),
+                                         ("latent_attn (gate a head)", 0, None, (gp, Q + D, d, 0), "latent_attn (window)"),
+                                         ("latent_attn (window)", 1024, sink, None, "")):
+            n, ng = win or 1025, 0 if gate is None else H * d // gate[2]
+            row(name, ph, B, lambda i: ops.latent_attn(qc, caches[i % len(caches)], bt, ctx, (d + r) ** -0.5, wv[i % 8], window=win, sink=s, gate=gate),
+                (B * (n * D + H * (D + d)) + H * d * R) * 2.0 + B * ng * ge, 2.0 * B * H * (n * (D + R) + d * R), like=like)
         del caches
         ws, x = [rnd(H, R, d) for _ in range(copies(H * R * d * 2))], rnd(B, nq)
         row("absorb_q", ph, B, lambda i: ops.head_project(x, ws[i % len(ws)], r), (H * R * d + B * H * (R + d + 2 * r)) * 2.0, 2.0 * B * H * R * d, like="o_proj")

@@ -839,8 +839,9 @@ int docqa_packed_window_attn(const void* q, const void* kv, const void* kr, cons
   const WindowArgs a{nullptr, 0, cu, nullptr, nullptr, sink, H, H, D, 64, 6, scale, window, vdim, 0, 0.f, 1.f, H * vdim,
                      cu_k, (const uint16_t*)kr, ld, d8, v8, gate};
   const uint16_t* v = (const uint16_t*)kv + (size_t)H * d8;
-  // 128 query rows a workgroup, 64 where that leaves CUs without one
-  const bool few = (long long)B * H * ((max_q + 127) / 128) < 384;
+  // 128 query rows a workgroup, 64 where that leaves CUs without one, or (no window: the last rows see
+  // all keys, the first few) without a second one to even out their work
+  const bool few = (long long)B * H * ((max_q + 127) / 128) < (window > 0 ? 384 : 640);
 #define RUN(DP, DPV, QT, KB) return launch_mfma<DP, DPV, QT, KB, 4, false, false, true>(q, kv, v, out, a, B, max_q, s)
 #define GO(DP, DPV, KB)               \
   do {                                \
